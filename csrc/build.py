@@ -65,7 +65,10 @@ def torch_paths():
 def write_ninja(path: str, out: str = OUT, build_dir: str = BUILD, debug: bool = False) -> dict:
     inc, tlib, abi = torch_paths()
     hipcc = os.path.join(ROCM, "bin", "hipcc")
-    kflags = f"--offload-arch={ARCH} -O3 -std=c++17 -fPIC -ffp-contract=fast -Wno-unused-result -I{CSRC}"
+    # packed fp32 (v_pk_add / mul / fma_f32) stays off: some of the forms the compiler picks have been seen to give
+    # wrong results on gfx950, without an error
+    kflags = (f"--offload-arch={ARCH} -O3 -std=c++17 -fPIC -ffp-contract=fast -Wno-unused-result "
+              f"-Xclang -target-feature -Xclang -packed-fp32-ops -I{CSRC}")
     if debug:
         kflags += " -DSHAI_KERNEL_DEBUG"
     incs = " ".join(f"-isystem {p}" for p in inc)
