@@ -6,6 +6,7 @@ box with the repo snapshot):
 
   * ``<pkg>/_native/libshai_kernels.so`` -- HIP kernels (hipcc --offload-arch=gfx950)
     plus the torch operator registrations (``torch.ops.shai.*``).
+  * ``<pkg>/_native/libshai_lm.so`` -- the decoder-block kernels (csrc/lm) and the sampler, registered the same way.
   * ``<pkg>/_native/libshai_runtime.so`` -- host C++ runtime (paged-KV block
     manager, batching scheduler helpers) exposed through a C ABI (ctypes).
   * ``<pkg>/_native/libshai_comm.so`` -- xGMI peer-to-peer all-reduce (HIP IPC).
@@ -38,7 +39,7 @@ ARCH = os.environ.get("PYTORCH_ROCM_ARCH", "gfx950")
 ROCM = os.environ.get("ROCM_PATH", "/opt/rocm")
 
 KERNEL_SRCS = ["kernels/norm.hip", "kernels/gemm.hip", "kernels/gemm_lds.hip", "kernels/gemm_8ph.hip", "kernels/gemm_w4.hip", "kernels/gemm_ws.hip", "kernels/conv_halo.hip", "kernels/attention.hip", "kernels/attention2.hip", "kernels/attention3.hip", "kernels/elementwise.hip", "kernels/dit.hip",
-               "kernels/sampling.hip", "kernels/gemv.hip", "kernels/gemv2.hip",
+               "kernels/gemv.hip", "kernels/gemv2.hip",
                "kernels/gemm_f8.hip"]
 # per-source extra hipcc flags: gemm_w4's epilogue (256 accumulators x an activation) is larger than LLVM's
 # default pragma-unroll budget; partially unrolled it would index the accumulators at run time (scratch)
@@ -49,6 +50,10 @@ EXTRA_KFLAGS = {"kernels/attention3.hip": "-mllvm -amdgpu-mfma-vgpr-form -fno-sl
                 "kernels/gemm_ws.hip": "-mllvm -pragma-unroll-threshold=100000 -fno-slp-vectorize",
                 "kernels/conv_halo.hip": "-mllvm -pragma-unroll-threshold=100000 -fno-slp-vectorize"}
 BINDING_SRCS = ["bindings.cpp"]
+# the decoder-block kernels and the token-level ops of every language model's step (their own library: a model that
+# runs on them alone needs nothing else compiled)
+LM_SRCS = ["lm/norm.hip", "lm/gemm.hip", "lm/gemm_tile.hip", "lm/moe.hip", "lm/attn.hip", "kernels/sampling.hip"]
+LM_BINDING_SRCS = ["lm/bindings.cpp"]
 RUNTIME_SRCS = ["runtime/block_manager.cpp", "runtime/scheduler.cpp"]
 COMM_SRCS = ["comm/p2p_allreduce.hip"]
 
@@ -126,6 +131,9 @@ def write_ninja(path: str, out: str = OUT, build_dir: str = BUILD, debug: bool =
     k = objs(KERNEL_SRCS, "hip") + objs(BINDING_SRCS, "cxx")
     targets["kernels"] = os.path.join(out, "libshai_kernels.so")
     lines.append(f"build {targets['kernels']}: link_kernels {' '.join(k)}")
+    m = objs(LM_SRCS, "hip") + objs(LM_BINDING_SRCS, "cxx")
+    targets["lm"] = os.path.join(out, "libshai_lm.so")
+    lines.append(f"build {targets['lm']}: link_kernels {' '.join(m)}")
     r = objs(RUNTIME_SRCS, "rcxx")
     if r:
         targets["runtime"] = os.path.join(out, "libshai_runtime.so")
@@ -143,7 +151,9 @@ def write_ninja(path: str, out: str = OUT, build_dir: str = BUILD, debug: bool =
 LAST_BUILD: dict = {}
 
 
-def build(clean: bool = False, jobs: int | None = None, verbose: bool = False, debug: bool = False) -> dict:
+def build(clean: bool = False, jobs: int | None = None, verbose: bool = False, debug: bool = False,
+          only: tuple = ()) -> dict:
+    """Compile every library, or those named in ``only`` ("kernels", "lm", "runtime", "comm")."""
     out, bdir = (OUT_DEBUG, BUILD_DEBUG) if debug else (OUT, BUILD)
     if clean and os.path.isdir(bdir):
         shutil.rmtree(bdir)
@@ -160,6 +170,7 @@ def build(clean: bool = False, jobs: int | None = None, verbose: bool = False, d
         cmd += ["-j", str(jobs)]
     if verbose:
         cmd.append("-v")
+    cmd += [targets[t] for t in only]
     r = subprocess.run(cmd, cwd=bdir, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
     sys.stdout.write(r.stdout)
     if r.returncode != 0:
@@ -170,7 +181,7 @@ def build(clean: bool = False, jobs: int | None = None, verbose: bool = False, d
     LAST_BUILD.clear()
     LAST_BUILD.update(compiled=compiled, linked=sum("] LINK " in ln for ln in r.stdout.splitlines()),
                       up_to_date="no work to do" in r.stdout)
-    return targets
+    return {t: p for t, p in targets.items() if not only or t in only}
 
 
 def summary() -> str:

@@ -1,0 +1,522 @@
+// Attention inside fixed-size chunks of the sequence, over a paged cache ([blocks, G, 64, dk | dv]).
+//
+// Position i sees the keys lo .. i with lo = i - i % chunk; scores are (q . k) * scale, softmaxed in fp32, and every
+// head's output is multiplied by sigmoid(its gate logit).  The rows of a step are [q | k | v | gate] (one GEMM).
+//
+// kv_store      the step's k / v rows into the cache.
+// prefill       bf16: flash attention, 4 waves x 32 queries, scores swapped (S^T = K Q^T) so that a lane holds one
+//               query's scores, P feeds O^T = V^T P^T from registers; only the 64-key blocks of the chunks that the
+//               workgroup's queries lie in are visited.  fp32: attn_rows.
+// decode        bf16: one workgroup per (sequence, kv head, split); each wave takes whole 64-key blocks, K straight from
+//               memory into the matrix cores (the group's query heads are the 16 columns), fp32 P against V on the
+//               VALU; the new token's k / v are written to the cache by the workgroup that reads them.
+// attn_rows     fp32 (any sizes): one wave per (row, head), plain online softmax.
+#include "lm_device.h"
+
+namespace shai_lm {
+
+typedef short s4v __attribute__((ext_vector_type(4)));
+constexpr float kLog2e = 1.4426950408889634f;
+
+template <typename T>
+__global__ void __launch_bounds__(256) kv_store_kernel(const AttnArgs p) {
+  constexpr int V = 16 / sizeof(T);
+  const long t = blockIdx.x;
+  const int slot = p.slots[t];
+  if (slot < 0) return;
+  const T* row = static_cast<const T*>(p.qkvg) + t * p.ld + (long)p.H * p.dk;
+  const int blk = slot >> 6, in = slot & 63;
+  const int nk = p.G * p.dk / V, nv = p.G * p.dv / V;
+  for (int i = threadIdx.x; i < nk + nv; i += 256) {
+    const bool isv = i >= nk;
+    const int e = (isv ? i - nk : i) * V, d = isv ? p.dv : p.dk, g = e / d;
+    T* dst = static_cast<T*>(isv ? p.vc : p.kc) + (((long)blk * p.G + g) * 64 + in) * d + (e - g * d);
+    *reinterpret_cast<uint4_*>(dst) = *reinterpret_cast<const uint4_*>(row + (isv ? (long)p.G * p.dk : 0L) + e);
+  }
+}
+
+void launch_kv_store(const AttnArgs& a, bool f32, hipStream_t s) {
+  if (f32) kv_store_kernel<float><<<a.T, 256, 0, s>>>(a);
+  else kv_store_kernel<bf16_t><<<a.T, 256, 0, s>>>(a);
+  SHAI_CHECK_LAUNCH();
+}
+
+// ------------------------------------------------------------------------------------------------ any-size rows
+template <typename T>
+__global__ void __launch_bounds__(256) attn_rows_kernel(const AttnArgs p) {
+  __shared__ float sq[4][256];
+  __shared__ float sp[4][64];
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const int b = blockIdx.z, i = blockIdx.x, h = blockIdx.y * 4 + w;
+  const int q_len = p.q_lens ? p.q_lens[b] : 1;
+  if (i >= q_len || h >= p.H) return;            // whole waves: no barrier below, only wave-local LDS
+  const long t = (p.q_lens ? p.q_start[b] : b) + i;
+  const int pos = p.ctx[b] - q_len + i, lo = pos - pos % p.chunk;
+  const int g = h / (p.H / p.G);
+  const T* row = static_cast<const T*>(p.qkvg) + t * p.ld;
+  for (int d = lane; d < p.dk; d += 64) sq[w][d] = load1(row + (long)h * p.dk + d);
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  float o[4] = {0.f, 0.f, 0.f, 0.f}, m = -INFINITY, l = 0.f;
+  for (int kb = lo >> 6; kb <= pos >> 6; ++kb) {
+    const long cell = ((long)p.bt[(long)b * p.max_blocks + kb] * p.G + g) * 64;
+    const int key = kb * 64 + lane;
+    float s = -INFINITY;
+    if (key >= lo && key <= pos) {
+      const T* kr = static_cast<const T*>(p.kc) + (cell + lane) * p.dk;
+      float acc = 0.f;
+      for (int d = 0; d < p.dk; d += 4) {
+        const float4_ k4 = load4(kr + d), q4 = load4(&sq[w][d]);
+        acc += k4[0] * q4[0] + k4[1] * q4[1] + k4[2] * q4[2] + k4[3] * q4[3];
+      }
+      s = acc * p.scale;
+    }
+    const float mn = fmaxf(m, wave_max(s));      // finite: the first block holds lo, every later one a visible key
+    const float alpha = expf(m - mn), e = expf(s - mn);
+    m = mn;
+    l = l * alpha + wave_sum(e);
+    sp[w][lane] = e;
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    const T* vr = static_cast<const T*>(p.vc) + cell * p.dv;
+    const int j0 = max(0, lo - kb * 64), j1 = min(63, pos - kb * 64);
+#pragma unroll
+    for (int c = 0; c < 4; ++c) {
+      const int col = lane + 64 * c;
+      if (col < p.dv) {
+        float acc = o[c] * alpha;
+        for (int j = j0; j <= j1; ++j) acc += sp[w][j] * load1(vr + (long)j * p.dv + col);
+        o[c] = acc;
+      }
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  }
+  const float gate = sigmoid_f(load1(row + (long)p.H * p.dk + (long)p.G * (p.dk + p.dv) + h)) / l;
+  T* out = static_cast<T*>(p.o) + t * (long)p.H * p.dv + (long)h * p.dv;
+#pragma unroll
+  for (int c = 0; c < 4; ++c)
+    if (lane + 64 * c < p.dv) store1(out + lane + 64 * c, o[c] * gate);
+}
+
+// ------------------------------------------------------------------------------------------------ prefill (bf16)
+template <int D>
+__device__ __forceinline__ int k_swz(int row, int ch) {
+  if constexpr (D >= 128) return row * D + ((ch ^ (row & 15)) << 3);
+  else return row * D + ((ch ^ ((row >> 1) & 7)) << 3);
+}
+template <int D>
+__device__ __forceinline__ int v_swz(int row, int ch) {
+  if constexpr (D >= 128) return row * D + ((ch ^ ((row & 3) << 2)) << 3);
+  else return row * D + ((ch ^ (((row >> 1) & 1) << 2)) << 3);
+}
+
+template <int DK, int DV>
+__global__ void __launch_bounds__(256, DK + DV > 256 ? 1 : 2) attn_prefill_kernel(const AttnArgs p) {
+  constexpr int KT = 64, CK = DK / 8, CV = DV / 8, NK = KT * CK / 256, NV = KT * CV / 256;
+  constexpr int NS = DK / 16, ND = DV / 32;
+  extern __shared__ __attribute__((aligned(16))) bf16_t smem[];
+  bf16_t* sK = smem;
+  bf16_t* sV = smem + 2 * KT * DK;
+  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+  const int fr = lane & 31, fh = lane >> 5;
+  const int b = blockIdx.z, h = blockIdx.y;
+  const int hk = h / (p.H / p.G);
+  const int q_len = p.q_lens[b], q0 = blockIdx.x * 128;
+  if (q0 >= q_len) return;
+  const int ctx = p.ctx[b], c_off = ctx - q_len;
+  const int qi = q0 + wid * 32 + fr, pos = qi + c_off, lo = pos - pos % p.chunk;
+  const long row0 = p.q_start[b];
+  const bf16_t* rows = static_cast<const bf16_t*>(p.qkvg) + row0 * p.ld;
+
+  bf16x8 qf[NS];
+  {
+    const bf16_t* qp = rows + (long)min(qi, q_len - 1) * p.ld + (long)h * DK;
+#pragma unroll
+    for (int s = 0; s < NS; ++s)
+      qf[s] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4_*>(qp + 16 * s + 8 * fh));
+  }
+  // blocks from the first query's chunk to the last query's position
+  const int p_first = q0 + c_off, p_last = min(q0 + 127, q_len - 1) + c_off;
+  const int t0 = (p_first - p_first % p.chunk) >> 6, t1 = (p_last >> 6) + 1;
+  const int lo_last = p_last - p_last % p.chunk;
+
+  uint4_ rk[NK], rv[NV];
+  auto load_tile = [&](int t) {
+    const long cell = ((long)p.bt[(long)b * p.max_blocks + t] * p.G + hk) * 64;
+    const bf16_t* kb = static_cast<const bf16_t*>(p.kc) + cell * DK;
+    const bf16_t* vb = static_cast<const bf16_t*>(p.vc) + cell * DV;
+    const int left = ctx - t * KT;               // rows of this block that hold keys of the sequence
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const int id = tid + 256 * i;
+      rk[i] = id / CK < left ? *reinterpret_cast<const uint4_*>(kb + (long)id * 8) : uint4_{0u, 0u, 0u, 0u};
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int id = tid + 256 * i;
+      rv[i] = id / CV < left ? *reinterpret_cast<const uint4_*>(vb + (long)id * 8) : uint4_{0u, 0u, 0u, 0u};
+    }
+  };
+  auto store_tile = [&](int st) {
+#pragma unroll
+    for (int i = 0; i < NK; ++i) {
+      const int id = tid + 256 * i;
+      *reinterpret_cast<uint4_*>(sK + st * KT * DK + k_swz<DK>(id / CK, id % CK)) = rk[i];
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int id = tid + 256 * i;
+      *reinterpret_cast<uint4_*>(sV + st * KT * DV + v_swz<DV>(id / CV, id % CV)) = rv[i];
+    }
+  };
+
+  float16_ o[ND];
+#pragma unroll
+  for (int d = 0; d < ND; ++d)
+#pragma unroll
+    for (int r = 0; r < 16; ++r) o[d][r] = 0.f;
+  float m_run = -INFINITY, l_run = 0.f;
+  const float sl2 = p.scale * kLog2e;
+  const int g16 = lane >> 4, i16 = lane & 15, tq = i16 >> 2, tp = i16 & 3;
+
+  load_tile(t0);
+  store_tile(0);
+  __syncthreads();
+  for (int t = t0; t < t1; ++t) {
+    const int cur = (t - t0) & 1;
+    if (t + 1 < t1) load_tile(t + 1);
+    const bf16_t* ks = sK + cur * KT * DK;
+    const bf16_t* vs = sV + cur * KT * DV;
+    float16_ sacc[2];
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb) {
+#pragma unroll
+      for (int r = 0; r < 16; ++r) sacc[kb][r] = 0.f;
+#pragma unroll
+      for (int s = 0; s < NS; ++s) {
+        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(ks + k_swz<DK>(kb * 32 + fr, 2 * s + fh));
+        sacc[kb] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, qf[s], sacc[kb], 0, 0, 0);
+      }
+    }
+    const int key0 = t * KT;
+    // scale first (it may be negative or zero), then mask
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) sacc[kb][r] *= sl2;
+    if (key0 + KT - 1 > p_first || key0 < lo_last) {
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+          const int key = key0 + kb * 32 + (r & 3) + 8 * (r >> 2) + 4 * fh;
+          sacc[kb][r] = key > pos || key < lo ? -INFINITY : sacc[kb][r];
+        }
+    }
+    float m4[4] = {-INFINITY, -INFINITY, -INFINITY, -INFINITY};
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) m4[r & 3] = fmaxf(m4[r & 3], sacc[kb][r]);
+    float mloc = fmaxf(fmaxf(m4[0], m4[1]), fmaxf(m4[2], m4[3]));
+    mloc = fmaxf(mloc, __shfl_xor(mloc, 32, 64));
+    const float m_new = fmaxf(m_run, mloc);
+    const bool grew = __any(m_new > m_run);
+    const float m_use = m_new == -INFINITY ? 0.f : m_new;
+    const float alpha = __builtin_amdgcn_exp2f(m_run - m_use);
+    m_run = m_new;
+    float ls4[4] = {0.f, 0.f, 0.f, 0.f};
+    bf16x8 pf[2][2];
+#pragma unroll
+    for (int kb = 0; kb < 2; ++kb) {
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        const float e = __builtin_amdgcn_exp2f(sacc[kb][r] - m_use);
+        sacc[kb][r] = e;
+        ls4[r & 3] += e;
+      }
+#pragma unroll
+      for (int s = 0; s < 2; ++s) {
+        bf16x8 v;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[j] = (__bf16)sacc[kb][8 * s + j];
+        pf[kb][s] = v;
+      }
+    }
+    l_run = l_run * alpha + ((ls4[0] + ls4[1]) + (ls4[2] + ls4[3]));
+    if (grew) {
+#pragma unroll
+      for (int d = 0; d < ND; ++d)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) o[d][r] *= alpha;
+    }
+#pragma unroll
+    for (int d = 0; d < ND; ++d) {
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb) {
+#pragma unroll
+        for (int s = 0; s < 2; ++s) {
+          const int r0 = kb * 32 + 16 * s + 4 * fh + tq;
+          const int col = d * 32 + 16 * (g16 & 1) + 4 * tp;
+          const int ch = col >> 3, half = (col >> 2) & 1;
+          const bf16_t* a0 = vs + v_swz<DV>(r0, ch) + 4 * half;
+          const bf16_t* a1 = vs + v_swz<DV>(r0 + 8, ch) + 4 * half;
+          const s4v u0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s4v*)(a0));
+          const s4v u1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s4v*)(a1));
+          short8 vv;
+#pragma unroll
+          for (int j = 0; j < 4; ++j) { vv[j] = u0[j]; vv[4 + j] = u1[j]; }
+          o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, vv), pf[kb][s], o[d], 0, 0, 0);
+        }
+      }
+    }
+    if (t + 1 < t1) store_tile(cur ^ 1);
+    __syncthreads();
+  }
+  const float l_tot = l_run + __shfl_xor(l_run, 32, 64);
+  if (qi < q_len) {
+    const float gate = bf2f(rows[(long)qi * p.ld + (long)p.H * DK + (long)p.G * (DK + DV) + h]);
+    const float inv = sigmoid_f(gate) / l_tot;
+    bf16_t* op = static_cast<bf16_t*>(p.o) + (row0 + qi) * (long)p.H * DV + (long)h * DV;
+#pragma unroll
+    for (int d = 0; d < ND; ++d)
+#pragma unroll
+      for (int g = 0; g < 4; ++g)
+        store4(op + d * 32 + 8 * g + 4 * fh, float4_{o[d][4 * g], o[d][4 * g + 1], o[d][4 * g + 2], o[d][4 * g + 3]} * inv);
+  }
+}
+
+template <int DK, int DV>
+static void prefill(const AttnArgs& a, hipStream_t s) {
+  constexpr int lds = 2 * 64 * (DK + DV) * 2;
+  (void)hipFuncSetAttribute(reinterpret_cast<const void*>(attn_prefill_kernel<DK, DV>),
+                            hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+  attn_prefill_kernel<DK, DV><<<dim3((a.max_q + 127) / 128, a.H, a.B), 256, lds, s>>>(a);
+}
+
+#define SHAI_LM_HEADS(FN, ...)                                      \
+  do {                                                              \
+    if (a.dk == 64 && a.dv == 64) FN<64, 64>(__VA_ARGS__);          \
+    else if (a.dk == 64 && a.dv == 128) FN<64, 128>(__VA_ARGS__);   \
+    else if (a.dk == 128 && a.dv == 64) FN<128, 64>(__VA_ARGS__);   \
+    else if (a.dk == 128 && a.dv == 128) FN<128, 128>(__VA_ARGS__); \
+    else FN<256, 256>(__VA_ARGS__);                                 \
+  } while (0)
+
+void launch_attn_prefill(const AttnArgs& a, bool f32, hipStream_t s) {
+  if (f32) attn_rows_kernel<float><<<dim3(a.max_q, (a.H + 3) / 4, a.B), 256, 0, s>>>(a);
+  else SHAI_LM_HEADS(prefill, a, s);
+  SHAI_CHECK_LAUNCH();
+}
+
+// ------------------------------------------------------------------------------------------------ decode (bf16)
+// One workgroup: kv head g's query heads h0 .. h0 + R - 1 (R <= 16, RH = R rounded up) of sequence b, one split of the
+// visible 64-key blocks.  Wave w takes blocks w, w + 4, ... of the split.
+template <int DK, int DV, int RH>
+__global__ void __launch_bounds__(256) attn_decode_kernel(const AttnArgs p, int per_group, int store) {
+  constexpr int LPK = DV / 8, KP = 64 / LPK, IT = 64 / KP;   // V: LPK lanes per key, KP keys at a time
+  constexpr int VB = IT > 16 ? 16 : IT;                      // V loads in flight
+  __shared__ float sp[4][64][RH];
+  __shared__ float so[4][RH][DV];
+  __shared__ float sm[4][16], sl[4][16];
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+  const int c = lane & 15, q4 = lane >> 4;
+  const int group = p.H / p.G, parts = (group + per_group - 1) / per_group;
+  const int g = blockIdx.x / parts, part = blockIdx.x % parts;
+  const int b = blockIdx.y, split = blockIdx.z;
+  const int h0 = g * group + part * per_group, R = min(per_group, group - part * per_group);
+  const int pos = p.ctx[b] - 1, lo = pos - pos % p.chunk;
+  const int b0 = lo >> 6, b1 = (pos >> 6) + 1;
+  const int per = (b1 - b0 + p.splits - 1) / p.splits;
+  const int s0 = b0 + split * per, s1 = min(b1, s0 + per);
+  const bf16_t* row = static_cast<const bf16_t*>(p.qkvg) + (long)b * p.ld;
+  bf16_t* kc = static_cast<bf16_t*>(p.kc);
+  bf16_t* vc = static_cast<bf16_t*>(p.vc);
+
+  // this step's k / v: stored by the only workgroup that reads them (the one with the last block)
+  const int slot = p.slots[b];
+  if (store && slot >= 0 && s1 == b1 && s0 < s1) {
+    const long cell = ((long)(slot >> 6) * p.G + g) * 64 + (slot & 63);
+    const bf16_t* kn = row + (long)p.H * DK + (long)g * DK;
+    const bf16_t* vn = row + (long)p.H * DK + (long)p.G * DK + (long)g * DV;
+    if (tid < DK / 8) reinterpret_cast<uint4_*>(kc + cell * DK)[tid] = reinterpret_cast<const uint4_*>(kn)[tid];
+    else if (tid >= 64 && tid - 64 < DV / 8)
+      reinterpret_cast<uint4_*>(vc + cell * DV)[tid - 64] = reinterpret_cast<const uint4_*>(vn)[tid - 64];
+  }
+  __syncthreads();
+
+  uint4_ qf[DK / 64][2];
+#pragma unroll
+  for (int s = 0; s < DK / 64; ++s)
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+      qf[s][u] = c < R ? *reinterpret_cast<const uint4_*>(row + (long)(h0 + c) * DK + 64 * s + 16 * q4 + 8 * u)
+                       : uint4_{0u, 0u, 0u, 0u};
+  float o[RH][8];
+#pragma unroll
+  for (int r = 0; r < RH; ++r)
+#pragma unroll
+    for (int j = 0; j < 8; ++j) o[r][j] = 0.f;
+  float m = -INFINITY, l = 0.f;                  // of head c (replicated over q4)
+  const float sl2 = p.scale * kLog2e;
+  const int vk = lane / LPK, vcol = (lane % LPK) * 8;
+
+  for (int kb = s0 + w; kb < s1; kb += 4) {
+    const long cell = ((long)p.bt[(long)b * p.max_blocks + kb] * p.G + g) * 64;
+    const bf16_t* kp = kc + (cell + c) * DK + 16 * q4;
+    const bf16_t* vp = vc + (cell + vk) * DV + vcol;
+    float4_ s[4];
+#pragma unroll
+    for (int t = 0; t < 4; ++t) {
+      s[t] = float4_{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int d = 0; d < DK / 64; ++d)
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+          const uint4_ kf = *reinterpret_cast<const uint4_*>(kp + (long)16 * t * DK + 64 * d + 8 * u);
+          s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, kf),
+                                                         __builtin_bit_cast(bf16x8, qf[d][u]), s[t], 0, 0, 0);
+        }
+    }
+    uint4_ v[VB];
+#pragma unroll
+    for (int i = 0; i < VB; ++i) v[i] = *reinterpret_cast<const uint4_*>(vp + (long)i * KP * DV);
+    float mx = -INFINITY;
+#pragma unroll
+    for (int t = 0; t < 4; ++t)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int key = kb * 64 + 16 * t + 4 * q4 + i;
+        s[t][i] = key < lo || key > pos ? -INFINITY : s[t][i] * sl2;
+        mx = fmaxf(mx, s[t][i]);
+      }
+    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    const float mn = fmaxf(m, mx);               // finite: every visited block holds a visible key
+    const float alpha = __builtin_amdgcn_exp2f(m - mn);
+    m = mn;
+    float sum = 0.f;
+#pragma unroll
+    for (int t = 0; t < 4; ++t)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float e = __builtin_amdgcn_exp2f(s[t][i] - mn);
+        sum += e;
+        if (c < RH) sp[w][16 * t + 4 * q4 + i][c] = e;
+      }
+    sum += __shfl_xor(sum, 16, 64);
+    sum += __shfl_xor(sum, 32, 64);
+    l = l * alpha + sum;
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+#pragma unroll
+    for (int r = 0; r < RH; ++r) {
+      const float ar = __shfl(alpha, r, 64);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) o[r][j] *= ar;
+    }
+#pragma unroll
+    for (int i0 = 0; i0 < IT; i0 += VB) {
+      if (i0 > 0) {
+#pragma unroll
+        for (int i = 0; i < VB; ++i) v[i] = *reinterpret_cast<const uint4_*>(vp + (long)(i0 + i) * KP * DV);
+      }
+#pragma unroll
+      for (int i = 0; i < VB; ++i) {
+        float f[8];
+        unpack8(v[i], f);
+        const float* pr = &sp[w][(i0 + i) * KP + vk][0];
+#pragma unroll
+        for (int r = 0; r < RH; ++r) {
+          const float pv = pr[r];
+#pragma unroll
+          for (int j = 0; j < 8; ++j) o[r][j] = fmaf(pv, f[j], o[r][j]);
+        }
+      }
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  }
+  // fold the key lanes of the wave, then the waves
+#pragma unroll
+  for (int r = 0; r < RH; ++r)
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      float x = o[r][j];
+#pragma unroll
+      for (int d = LPK; d < 64; d <<= 1) x += __shfl_xor(x, d, 64);
+      if (vk == 0) so[w][r][vcol + j] = x;
+    }
+  if (lane < 16) {
+    sm[w][lane] = m;
+    sl[w][lane] = l;
+  }
+  __syncthreads();
+  for (int i = tid; i < R * DV; i += 256) {
+    const int r = i / DV, d = i - r * DV, h = h0 + r;
+    const float M = fmaxf(fmaxf(sm[0][r], sm[1][r]), fmaxf(sm[2][r], sm[3][r]));
+    float L = 0.f, x = 0.f;
+    if (M > -INFINITY) {
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        const float e = __builtin_amdgcn_exp2f(sm[k][r] - M);
+        L += sl[k][r] * e;
+        x += so[k][r][d] * e;
+      }
+    }
+    if (p.splits == 1) {
+      const float gate = bf2f(row[(long)p.H * DK + (long)p.G * (DK + DV) + h]);
+      static_cast<bf16_t*>(p.o)[((long)b * p.H + h) * DV + d] = f2bf(x / L * sigmoid_f(gate));
+    } else {
+      float* ws = p.ws + (((long)b * p.H + h) * p.splits + split) * (DV + 2);
+      ws[d] = x;
+      if (d == 0) {
+        ws[DV] = M;
+        ws[DV + 1] = L;
+      }
+    }
+  }
+}
+
+__global__ void __launch_bounds__(256) attn_decode_fold_kernel(const AttnArgs p) {
+  const int h = blockIdx.x, b = blockIdx.y, d = threadIdx.x;
+  if (d >= p.dv) return;
+  const float* ws = p.ws + ((long)b * p.H + h) * p.splits * (p.dv + 2);
+  float M = -INFINITY;
+  for (int s = 0; s < p.splits; ++s) M = fmaxf(M, ws[(long)s * (p.dv + 2) + p.dv]);
+  float L = 0.f, x = 0.f;
+  for (int s = 0; s < p.splits; ++s) {
+    const float* q = ws + (long)s * (p.dv + 2);
+    const float e = __builtin_amdgcn_exp2f(q[p.dv] - M);
+    L += q[p.dv + 1] * e;
+    x += q[d] * e;
+  }
+  const float gate = bf2f(static_cast<const bf16_t*>(p.qkvg)[(long)b * p.ld + (long)p.H * p.dk +
+                                                             (long)p.G * (p.dk + p.dv) + h]);
+  static_cast<bf16_t*>(p.o)[((long)b * p.H + h) * p.dv + d] = f2bf(x / L * sigmoid_f(gate));
+}
+
+template <int DK, int DV>
+static void decode(const AttnArgs& a, hipStream_t s) {
+  const int group = a.H / a.G;
+  // heads per workgroup: 16 columns, 8 at the largest head size (LDS); more heads take several workgroups, and the
+  // cache write is then a launch of its own (no single workgroup reads the new row)
+  constexpr int MAXR = DV > 128 ? 8 : 16;
+  const int per = group < MAXR ? group : MAXR, parts = (group + per - 1) / per;
+  if (parts > 1) launch_kv_store(a, false, s);
+  const dim3 grid(a.G * parts, a.B, a.splits);
+  const int store = parts == 1;
+  if (per == 1) attn_decode_kernel<DK, DV, 1><<<grid, 256, 0, s>>>(a, per, store);
+  else if (per <= 4) attn_decode_kernel<DK, DV, 4><<<grid, 256, 0, s>>>(a, per, store);
+  else if (per <= 8) attn_decode_kernel<DK, DV, 8><<<grid, 256, 0, s>>>(a, per, store);
+  else if constexpr (DV <= 128) attn_decode_kernel<DK, DV, 16><<<grid, 256, 0, s>>>(a, per, store);
+  if (a.splits > 1) attn_decode_fold_kernel<<<dim3(a.H, a.B), 256, 0, s>>>(a);
+}
+
+void launch_attn_decode(const AttnArgs& a, bool f32, hipStream_t s) {
+  if (f32) {
+    launch_kv_store(a, true, s);
+    attn_rows_kernel<float><<<dim3(1, (a.H + 3) / 4, a.B), 256, 0, s>>>(a);
+  } else {
+    SHAI_LM_HEADS(decode, a, s);
+  }
+  SHAI_CHECK_LAUNCH();
+}
+
+}  // namespace shai_lm

@@ -1,0 +1,145 @@
+// C = epi(A W^T), streaming form: a workgroup owns NT x 16 rows of W and up to MT x 16 rows of A, its waves split K and
+// fold their fp32 partials through LDS.  W goes straight from memory to the matrix cores (no LDS round trip), so the
+// kernel runs at the speed the weights arrive: decode steps, routers, and expert products with few rows per expert.
+// bf16: v_mfma_f32_16x16x32_bf16; fp32: v_mfma_f32_16x16x4_f32 (full fp32 products).
+//
+// Operands are swapped (C^T = W A^T): a lane ends up with 4 consecutive output columns of one row, so a (gate, up) row
+// pair of W is folded in registers.  A k-step covers 64 values; lane group g = lane / 16 takes values 16 g .. 16 g + 15
+// of it in both operands (the order of k inside a dot product is free), i.e. every W row is read 128 bytes at a time.
+//
+// Dense: row tiles of A are blockIdx.y.  Grouped (experts): blockIdx.y is an entry of the tile list and blockIdx.z a
+// 16 MT-row part of it; rows past the expert's last slot are computed on a clamped row and not stored.
+#include "lm_device.h"
+#include "lm.h"
+
+namespace shai_lm {
+
+template <typename T>
+struct Frag;
+template <>
+struct Frag<bf16_t> {
+  uint4_ v[2];
+  __device__ __forceinline__ void load(const bf16_t* p) {
+    v[0] = *reinterpret_cast<const uint4_*>(p);
+    v[1] = *reinterpret_cast<const uint4_*>(p + 8);
+  }
+  static __device__ __forceinline__ float4_ mac(const Frag& w, const Frag& a, float4_ c) {
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+      c = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, w.v[i]),
+                                                  __builtin_bit_cast(bf16x8, a.v[i]), c, 0, 0, 0);
+    return c;
+  }
+};
+template <>
+struct Frag<float> {
+  float4_ v[4];
+  __device__ __forceinline__ void load(const float* p) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = *reinterpret_cast<const float4_*>(p + 4 * i);
+  }
+  static __device__ __forceinline__ float4_ mac(const Frag& w, const Frag& a, float4_ c) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) c = __builtin_amdgcn_mfma_f32_16x16x4f32(w.v[i][j], a.v[i][j], c, 0, 0, 0);
+    return c;
+  }
+};
+
+template <typename T, typename O, int MT, int NT, int NW>
+__global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) {
+  constexpr int U = sizeof(T) == 2 ? (NT == 1 ? 4 : 2) : 1;   // k-steps of W in flight per wave
+  __shared__ float4_ red[NW][NT * MT][64];
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int r = lane & 15, g = lane >> 4;
+  const int n0 = blockIdx.x * 16 * NT;
+  int row0 = blockIdx.y * 16 * MT, rows_end = p.M, expert = 0;
+  if (p.tiles) {
+    expert = p.tiles[2 * blockIdx.y];
+    if (expert < 0) return;
+    row0 = p.tiles[2 * blockIdx.y + 1];
+    rows_end = min(p.offsets[expert + 1], row0 + p.bm);
+    row0 += blockIdx.z * 16 * MT;
+  }
+  if (row0 >= rows_end) return;
+  const T* W = static_cast<const T*>(p.W) + (long)expert * p.N * p.K;
+  const T* A = static_cast<const T*>(p.A);
+  const T* wp[NT];
+  const T* ap[MT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i) wp[i] = W + (long)min(n0 + 16 * i + r, p.N - 1) * p.K + g * 16;
+#pragma unroll
+  for (int j = 0; j < MT; ++j) {
+    int m = min(row0 + 16 * j + r, rows_end - 1);
+    if (p.gather) m = p.gather[m];
+    ap[j] = A + (long)m * p.K + g * 16;
+  }
+  float4_ acc[NT][MT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i)
+#pragma unroll
+    for (int j = 0; j < MT; ++j) acc[i][j] = float4_{0.f, 0.f, 0.f, 0.f};
+  const int steps = p.K / 64;
+  for (int s0 = wid; s0 < steps; s0 += NW * U) {
+    Frag<T> w[U][NT];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const long k = (long)min(s0 + u * NW, steps - 1) * 64;
+#pragma unroll
+      for (int i = 0; i < NT; ++i) w[u][i].load(wp[i] + k);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      if (s0 + u * NW < steps) {
+        const long k = (long)(s0 + u * NW) * 64;
+#pragma unroll
+        for (int j = 0; j < MT; ++j) {
+          Frag<T> a;
+          a.load(ap[j] + k);
+#pragma unroll
+          for (int i = 0; i < NT; ++i) acc[i][j] = Frag<T>::mac(w[u][i], a, acc[i][j]);
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < NT; ++i)
+#pragma unroll
+    for (int j = 0; j < MT; ++j) red[wid][i * MT + j][lane] = acc[i][j];
+  __syncthreads();
+  for (int t = wid; t < NT * MT; t += NW) {
+    float4_ c = red[0][t][lane];
+#pragma unroll
+    for (int w = 1; w < NW; ++w) c += red[w][t][lane];
+    const int m = row0 + 16 * (t % MT) + r;
+    if (m < rows_end) store_cols<O>(p, m, n0 + 16 * (t / MT) + 4 * g, c);
+  }
+}
+
+template <typename T, typename O>
+static void stream(const GemmArgs& a, hipStream_t s) {
+  const int rows = a.tiles ? a.bm : a.M;
+  const int mt = rows <= 16 ? 1 : rows <= 32 ? 2 : 4, nt = mt == 1 ? 1 : 2;
+  const dim3 grid((a.N + 16 * nt - 1) / (16 * nt), a.tiles ? a.n_tiles : (a.M + 16 * mt - 1) / (16 * mt),
+                  a.tiles ? (a.bm + 16 * mt - 1) / (16 * mt) : 1);
+  const bool deep = (long)grid.x * grid.y * grid.z < 1024 && a.K >= 1024;
+#define GO(MT_, NT_)                                                               \
+  do {                                                                             \
+    if (deep) gemm_stream_kernel<T, O, MT_, NT_, 8><<<grid, 512, 0, s>>>(a);       \
+    else gemm_stream_kernel<T, O, MT_, NT_, 4><<<grid, 256, 0, s>>>(a);            \
+  } while (0)
+  if (mt == 1) GO(1, 1);
+  else if (mt == 2) GO(2, 2);
+  else GO(4, 2);
+#undef GO
+  SHAI_CHECK_LAUNCH();
+}
+
+void launch_gemm(const GemmArgs& a, bool f32, hipStream_t s) {
+  if (f32) stream<float, float>(a, s);
+  else if (a.out_f32) stream<bf16_t, float>(a, s);
+  else stream<bf16_t, bf16_t>(a, s);
+}
+
+}  // namespace shai_lm

@@ -1,0 +1,144 @@
+// C = epi(A W^T), LDS-tiled bf16 form for many rows (prefill): 128 x 128 tiles of 4 waves, 64-wide k-tiles moved global
+// -> LDS by DMA (buffer_load ... lds, 16 bytes per lane) into two stages; the load of k-tile t + 1 is issued before the
+// MFMAs of t.  The bank swizzle is applied to the per-lane source chunk.  Buffer range checks zero-fill rows past the
+// ends.  Dense or grouped by expert: the row tiles of a grouped product come from the tile list, each with its own W and
+// with A rows gathered per lane.  Tiles are walked XCD by XCD in groups of 8 row tiles that share their W columns.
+#include "lm_device.h"
+#include "lm.h"
+
+namespace shai_lm {
+
+typedef __attribute__((address_space(3))) void lds_void;
+constexpr uint32_t kOob = 0x80000000u;
+
+__device__ __forceinline__ int swz(int row, int ch) { return row * 64 + ((ch ^ ((row >> 1) & 7)) << 3); }
+
+__device__ __forceinline__ __amdgpu_buffer_rsrc_t rsrc(const void* b, long bytes) {
+  return __builtin_amdgcn_make_buffer_rsrc(const_cast<void*>(b), (short)0, (int)bytes, 0x00020000);
+}
+
+__device__ __forceinline__ void dma16(__amdgpu_buffer_rsrc_t r, bf16_t* lds_wave_base, uint32_t voff) {
+  __builtin_amdgcn_raw_ptr_buffer_load_lds(r, (lds_void*)lds_wave_base, 16, voff, 0, 0, 0);
+}
+
+template <typename O, int BM, int BN, int WM, int WN>
+__global__ void __launch_bounds__(WM * WN * 64, 2) gemm_tile_kernel(const GemmArgs p) {
+  constexpr int NW = WM * WN, TM = BM / WM, TN = BN / WN, IM = TM / 32, JN = TN / 32;
+  constexpr int JA = BM / 8 / NW, JB = BN / 8 / NW, STAGE = (BM + BN) * 64;
+  extern __shared__ __attribute__((aligned(16))) bf16_t smem[];
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int wm = wid / WN, wn = wid % WN;
+
+  const int tiles_m = p.tiles ? p.n_tiles : (p.M + BM - 1) / BM, tiles_n = (p.N + BN - 1) / BN;
+  const int total = tiles_m * tiles_n;
+  int bid = blockIdx.x;
+  {
+    const int xcd = bid & 7, q = total >> 3, r = total & 7;
+    bid = (xcd < r ? xcd * (q + 1) : r * (q + 1) + (xcd - r) * q) + (bid >> 3);
+  }
+  constexpr int GROUP = 8;
+  const int group = bid / (GROUP * tiles_n), first_m = group * GROUP;
+  const int gsize = min(tiles_m - first_m, GROUP);
+  const int in_group = bid - group * GROUP * tiles_n;
+  const int mt = first_m + in_group % gsize, n0 = (in_group / gsize) * BN;
+  int m0 = mt * BM, m_end = p.M, expert = 0;
+  if (p.tiles) {
+    expert = p.tiles[2 * mt];
+    if (expert < 0) return;
+    m0 = p.tiles[2 * mt + 1];
+    m_end = min(p.offsets[expert + 1], m0 + BM);
+  }
+  const bf16_t* Wt = static_cast<const bf16_t*>(p.W) + (long)expert * p.N * p.K;
+  const __amdgpu_buffer_rsrc_t rW = rsrc(Wt, (long)p.N * p.K * 2), rA = rsrc(p.A, (long)p.a_rows * p.K * 2);
+
+  // byte offset of this lane's 16-byte chunk of every staged row at k = 0 (kOob: the row does not exist)
+  const int lrow = lane >> 3, lpos = lane & 7;
+  uint32_t offA[JA], offW[JB];
+#pragma unroll
+  for (int j = 0; j < JA; ++j) {
+    const int r = (wid * JA + j) * 8 + lrow, m = m0 + r;
+    const long src = m < m_end ? (p.gather ? p.gather[m] : m) : -1;
+    offA[j] = src < 0 ? kOob : (uint32_t)((src * p.K + (lpos ^ ((r >> 1) & 7)) * 8) * 2);
+  }
+#pragma unroll
+  for (int j = 0; j < JB; ++j) {
+    const int r = (wid * JB + j) * 8 + lrow, n = n0 + r;
+    offW[j] = n < p.N ? (uint32_t)(((long)n * p.K + (lpos ^ ((r >> 1) & 7)) * 8) * 2) : kOob;
+  }
+  auto stage = [&](int buf, int kt) {
+    bf16_t* sa = smem + buf * STAGE;
+    bf16_t* sw = sa + BM * 64;
+    const uint32_t kb = (uint32_t)kt * 128u;
+#pragma unroll
+    for (int j = 0; j < JB; ++j)
+      dma16(rW, sw + (wid * JB + j) * 512, offW[j] == kOob ? kOob : offW[j] + kb);
+#pragma unroll
+    for (int j = 0; j < JA; ++j)
+      dma16(rA, sa + (wid * JA + j) * 512, offA[j] == kOob ? kOob : offA[j] + kb);
+  };
+
+  float16_ acc[IM][JN];
+#pragma unroll
+  for (int i = 0; i < IM; ++i)
+#pragma unroll
+    for (int j = 0; j < JN; ++j)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) acc[i][j][r] = 0.f;
+
+  const int nk = p.K / 64;
+  const int fr = lane & 31, fh = lane >> 5;
+  stage(0, 0);
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  __syncthreads();
+  for (int kt = 0; kt < nk; ++kt) {
+    const int cur = kt & 1;
+    if (kt + 1 < nk) stage(cur ^ 1, kt + 1);
+    const bf16_t* sa = smem + cur * STAGE;
+    const bf16_t* sw = sa + BM * 64;
+#pragma unroll
+    for (int s = 0; s < 4; ++s) {
+      bf16x8 af[IM], wf[JN];
+#pragma unroll
+      for (int i = 0; i < IM; ++i)
+        af[i] = *reinterpret_cast<const bf16x8*>(sa + swz(wm * TM + i * 32 + fr, 2 * s + fh));
+#pragma unroll
+      for (int j = 0; j < JN; ++j)
+        wf[j] = *reinterpret_cast<const bf16x8*>(sw + swz(wn * TN + j * 32 + fr, 2 * s + fh));
+#pragma unroll
+      for (int i = 0; i < IM; ++i)
+#pragma unroll
+        for (int j = 0; j < JN; ++j)
+          acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wf[j], af[i], acc[i][j], 0, 0, 0);
+    }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+  }
+#pragma unroll
+  for (int i = 0; i < IM; ++i) {
+    const int m = m0 + wm * TM + i * 32 + fr;
+    if (m >= m_end) continue;
+#pragma unroll
+    for (int j = 0; j < JN; ++j)
+#pragma unroll
+      for (int g = 0; g < 4; ++g)
+        store_cols<O>(p, m, n0 + wn * TN + j * 32 + 8 * g + 4 * fh,
+                      float4_{acc[i][j][4 * g], acc[i][j][4 * g + 1], acc[i][j][4 * g + 2], acc[i][j][4 * g + 3]});
+  }
+}
+
+void launch_gemm_tile(const GemmArgs& a, hipStream_t s) {
+  constexpr int BM = 128, BN = 128;
+  const int tiles_m = a.tiles ? a.n_tiles : (a.M + BM - 1) / BM;
+  const int grid = tiles_m * ((a.N + BN - 1) / BN);
+  constexpr int lds = 2 * (BM + BN) * 64 * 2;
+  auto go = [&](auto k) {
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    k<<<grid, 256, lds, s>>>(a);
+  };
+  if (a.out_f32) go(gemm_tile_kernel<float, BM, BN, 2, 2>);
+  else go(gemm_tile_kernel<bf16_t, BM, BN, 2, 2>);
+  SHAI_CHECK_LAUNCH();
+}
+
+}  // namespace shai_lm

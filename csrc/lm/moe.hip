@@ -1,0 +1,158 @@
+// Mixture-of-experts routing: group-limited top-k of softmax scores, and the sort of (token, k) pairs by expert.
+#include "lm_device.h"
+#include "lm.h"
+
+namespace shai_lm {
+
+// One wave per token; lane l holds experts l, l + 64, ...  All comparisons break ties by the lower expert index, and
+// picks are by a strictly decreasing (score, index) order, so every pick is a distinct expert whatever the scores are.
+template <int NE>
+__global__ void __launch_bounds__(256) route_kernel(const RouteArgs p) {
+  extern __shared__ float sh[];                 // [4][E] scores, [4][groups] group scores
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int t = blockIdx.x * 4 + wid;
+  float* sc = sh + wid * (p.E + p.groups);
+  float* gs = sc + p.E;
+  const bool live = t < p.T;
+  float z[NE];
+  float m = -INFINITY;
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int e = lane + 64 * i;
+    z[i] = live && e < p.E ? p.logits[(long)t * p.E + e] : -INFINITY;
+    if (!(z[i] == z[i])) z[i] = -INFINITY;      // a padding row may carry NaN: it still needs valid picks
+    m = fmaxf(m, z[i]);
+  }
+  m = wave_max(m);
+  if (m == -INFINITY) m = 0.f;
+  float sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    z[i] = expf(z[i] - m);
+    sum += lane + 64 * i < p.E ? z[i] : 0.f;
+  }
+  sum = wave_sum(sum);
+  const float inv = sum > 0.f ? 1.f / sum : 0.f;
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int e = lane + 64 * i;
+    z[i] *= inv;
+    if (e < p.E) sc[e] = z[i];
+  }
+  __syncthreads();
+  const int per = p.E / p.groups;
+  for (int g = lane; g < p.groups; g += 64) {
+    float b = -1.f;
+    for (int j = 0; j < per; ++j) b = fmaxf(b, sc[g * per + j]);
+    gs[g] = b;
+  }
+  __syncthreads();
+  // a group is kept when fewer than `keep` groups beat it
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const int e = lane + 64 * i;
+    if (e < p.E && p.keep < p.groups) {
+      const int g = e / per;
+      const float mine = gs[g];
+      int better = 0;
+      for (int j = 0; j < p.groups; ++j) better += gs[j] > mine || (gs[j] == mine && j < g);
+      if (better >= p.keep) z[i] = -1.f;
+    }
+    if (e >= p.E) z[i] = -2.f;
+  }
+  for (int k = 0; k < p.top; ++k) {
+    float bv = -3.f;
+    int bi = 0x7fffffff;
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      const int e = lane + 64 * i;
+      if (z[i] > bv) { bv = z[i]; bi = e; }     // ascending e: the first of equal scores stays
+    }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ov = __shfl_xor(bv, o, 64);
+      const int oi = __shfl_xor(bi, o, 64);
+      if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+    }
+#pragma unroll
+    for (int i = 0; i < NE; ++i)
+      if (lane + 64 * i == bi) z[i] = -4.f;
+    if (live && lane == 0) {
+      p.ids[(long)t * p.top + k] = bi;
+      p.wts[(long)t * p.top + k] = bv;
+    }
+  }
+}
+
+void launch_route(const RouteArgs& a, hipStream_t s) {
+  const int grid = (a.T + 3) / 4;
+  const size_t lds = sizeof(float) * 4 * (a.E + a.groups);
+  if (a.E <= 64) route_kernel<1><<<grid, 256, lds, s>>>(a);
+  else if (a.E <= 128) route_kernel<2><<<grid, 256, lds, s>>>(a);
+  else if (a.E <= 256) route_kernel<4><<<grid, 256, lds, s>>>(a);
+  else route_kernel<16><<<grid, 256, lds, s>>>(a);
+  SHAI_CHECK_LAUNCH();
+}
+
+// One workgroup: LDS histogram, scan, tile list, scatter.  The order of rows inside an expert is arbitrary (each row is
+// computed alone, and the combine reads a token's slots in k order), so LDS atomics are enough.
+__global__ void __launch_bounds__(1024) plan_kernel(const PlanArgs p) {
+  __shared__ int cnt[1024], start[1025], tile0[1025];
+  const int tid = threadIdx.x;
+  for (int e = tid; e < p.E; e += 1024) cnt[e] = 0;
+  __syncthreads();
+  for (int i = tid; i < p.P; i += 1024) atomicAdd(&cnt[p.ids[i]], 1);
+  __syncthreads();
+  if (tid < 64) {                                // wave 0: exclusive scans of the counts and of the tile counts
+    int base = 0, tbase = 0;
+    for (int e0 = 0; e0 < p.E; e0 += 64) {
+      const int e = e0 + tid;
+      const int c = e < p.E ? cnt[e] : 0;
+      const int n = (c + p.bm - 1) / p.bm;
+      int a = c, b = n;
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const int ua = __shfl_up(a, o, 64), ub = __shfl_up(b, o, 64);
+        if (tid >= o) { a += ua; b += ub; }
+      }
+      if (e < p.E) {
+        start[e] = base + a - c;
+        tile0[e] = tbase + b - n;
+      }
+      base += __shfl(a, 63, 64);
+      tbase += __shfl(b, 63, 64);
+    }
+    if (tid == 0) {
+      start[p.E] = base;
+      tile0[p.E] = tbase;
+    }
+  }
+  __syncthreads();
+  for (int e = tid; e <= p.E; e += 1024) p.offsets[e] = start[e];
+  for (int e = tid; e < p.E; e += 1024) {
+    const int n = tile0[e + 1] - tile0[e];
+    for (int j = 0; j < n; ++j) {
+      p.tiles[2 * (tile0[e] + j)] = e;
+      p.tiles[2 * (tile0[e] + j) + 1] = start[e] + j * p.bm;
+    }
+  }
+  for (int i = tile0[p.E] + tid; i < p.n_tiles; i += 1024) {
+    p.tiles[2 * i] = -1;
+    p.tiles[2 * i + 1] = 0;
+  }
+  __syncthreads();
+  for (int e = tid; e < p.E; e += 1024) cnt[e] = start[e];
+  __syncthreads();
+  for (int i = tid; i < p.P; i += 1024) {
+    const int s = atomicAdd(&cnt[p.ids[i]], 1);
+    p.token_of[s] = i / p.top;
+    p.slot_of[i] = s;
+  }
+}
+
+void launch_plan(const PlanArgs& a, hipStream_t s) {
+  plan_kernel<<<1, 1024, 0, s>>>(a);
+  SHAI_CHECK_LAUNCH();
+}
+
+}  // namespace shai_lm

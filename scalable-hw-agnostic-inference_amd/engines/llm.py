@@ -44,7 +44,8 @@ import torch
 from ..utils import profiling as prof
 from .. import ops
 from . import new_graph
-from ..models.llama import (KV_BLOCK, Batch, LlamaConfig, LlamaForCausalLM, allocate_kv_cache, kv_bytes_per_block)
+from ..models.llama import KV_BLOCK, Batch, LlamaConfig
+from ..models.registry import config_from_path, model_class
 from ..parallel.state import tp
 from ..weights import materialize
 
@@ -184,7 +185,7 @@ class _DecodeGraph:
     previous decode step's output (``engine.last_tokens``) instead of the host id.  This is what lets the
     engine enqueue step t+1 before it has read step t's tokens back (``LLMEngine.async_decode``)."""
 
-    NF = 9  # per-row int32 fields before the block table
+    NF = 10  # per-row int32 fields before the block table
 
     def __init__(self, engine: "LLMEngine", Bc: int, cross: bool = False, greedy: bool = False,
                  splits: Optional[int] = None, full_vocab: bool = False):
@@ -201,11 +202,12 @@ class _DecodeGraph:
         f = lambda i: self.dbuf[i * Bc:(i + 1) * Bc]
         self.ids, self.pos, self.slots, self.lens, self.topk = f(0), f(1), f(2), f(3), f(4)
         self.temps, self.topp, self.u = f(5).view(torch.float32), f(6).view(torch.float32), f(7).view(torch.float32)
-        self.rowmap = f(8)
+        self.rowmap, self.prev = f(8), f(9)
         self.bt = self.dbuf[self.NF * Bc:].view(Bc, mb)
         self.slots.fill_(-1)
         self.lens.fill_(1)
         self.rowmap.fill_(-1)
+        self.prev.fill_(-1)
         self.toks = torch.zeros(Bc, dtype=torch.int32, device=dev)
         pin = dev.type == "cuda"
         self.host = [torch.zeros(self.words, dtype=torch.int32, pin_memory=pin) for _ in range(2)]
@@ -213,7 +215,8 @@ class _DecodeGraph:
         self.host_ev = [None, None]
         self.flip = 0
         self.splits = splits if splits is not None else engine.decode_splits(Bc, 0)
-        self.batch = Batch(self.ids, self.pos, self.slots, self.bt, self.lens, None, Bc, 1, False, self.splits)
+        self.batch = Batch(self.ids, self.pos, self.slots, self.bt, self.lens, None, Bc, 1, False, self.splits,
+                           prev_ids=self.prev)
         self.cross = cross
         self.greedy = greedy
         if cross:  # static image-K/V inputs of the cross-attention layers
@@ -254,8 +257,9 @@ class _DecodeGraph:
             self.toks.copy_(sample(logits, self.temps, self.topk, self.topp, uniforms=self.u))
         eng.last_tokens[:self.Bc].copy_(self.toks)
 
-    def launch(self, seqs, pos, slots, lens, bt, ids, rowmap, uniforms, cross=None):
-        """Enqueue one decode step; returns (host int32 token view, completion event or None)."""
+    def launch(self, seqs, pos, slots, lens, bt, ids, rowmap, uniforms, cross=None, prev=None, sampled=True):
+        """Enqueue one decode step; returns (host int32 token view, completion event or None).  ``sampled=False``
+        (a ``full_vocab`` program): the step ends at its logits (``self.logits``) and no token is drawn."""
         B, Bc = len(seqs), self.Bc
         i = self.flip
         self.flip ^= 1
@@ -272,6 +276,7 @@ class _DecodeGraph:
         v(6).view(np.float32)[:B] = [s.params.top_p for s in seqs]
         v(7).view(np.float32)[:B] = uniforms
         v(8)[:B] = rowmap
+        v(9)[:B] = -1 if prev is None else prev
         btv = h[self.NF * Bc:].reshape(Bc, -1)
         btv[:B] = bt
         if B < Bc:  # padding rows: no KV write, one-token context, greedy, no feedback
@@ -284,6 +289,7 @@ class _DecodeGraph:
             v(6).view(np.float32)[B:] = 1.0
             v(7).view(np.float32)[B:] = 0.0
             v(8)[B:] = -1
+            v(9)[B:] = -1
             btv[B:] = 0
         self.dbuf.copy_(self.host[i], non_blocking=True)
         if self.cross:
@@ -308,6 +314,8 @@ class _DecodeGraph:
         else:
             self._program()
         eng = self.engine
+        if not sampled:
+            return None, None
         if self.full_vocab:   # exact full-vocabulary top-k / top-p at the same uniforms, outside the graph
             self.toks.copy_(sample(self.logits, self.temps, self.topk, self.topp, uniforms=self.u, full_vocab=True))
             eng.last_tokens[:self.Bc].copy_(self.toks)
@@ -330,22 +338,26 @@ class _Inflight:
 
 
 class LLMEngine:
-    def __init__(self, cfg: LlamaConfig, device="cuda", model_path: Optional[str] = None, seed: int = 0,
+    """``cfg``: a config of :mod:`shai_amd.models.registry` (Llama family, mllama, Golulix)."""
+
+    def __init__(self, cfg, device="cuda", model_path: Optional[str] = None, seed: int = 0,
                  max_num_seqs: int = 64, max_model_len: int = 4096, num_kv_blocks: Optional[int] = None,
                  gpu_memory_utilization: float = 0.85, prefill_token_budget: int = 8192, use_graphs: bool = True,
                  enable_prefix_caching: bool = True, prefill_chunk: Optional[int] = None,
                  quantization: Optional[str] = None, async_decode: Optional[bool] = None,
-                 packed_prefill: bool = True, mixed_steps: bool = True):
-        from ..models.mllama import MllamaConfig, MllamaForConditionalGeneration
+                 packed_prefill: bool = True, mixed_steps: bool = True, dtype: torch.dtype = torch.bfloat16):
+        from ..models.mllama import MllamaConfig
         from ..runtime import BlockManager
         self.mcfg = cfg if isinstance(cfg, MllamaConfig) else None
+        cls = model_class(cfg)
+        if dtype not in cls.dtypes:
+            raise ValueError(f"{cls.__name__} runs in {cls.dtypes}, not {dtype}")
+        self.device = torch.device(device)
+        with torch.device(self.device):
+            self.model = cls(cfg, dtype=dtype) if len(cls.dtypes) > 1 else cls(cfg)
         if self.mcfg is not None:
             cfg = self.mcfg.text
         self.cfg = cfg
-        self.device = torch.device(device)
-        with torch.device(self.device):
-            self.model = (MllamaForConditionalGeneration(self.mcfg) if self.mcfg is not None
-                          else LlamaForCausalLM(cfg))
         materialize(self.model, self.device, model_path, None, seed)
         self.model.fold_norms()  # before any graph capture (re-folded lazily after a later load)
         self.weights = self.model._shai_weights
@@ -353,6 +365,8 @@ class LLMEngine:
         # (after the norm fold, which rescales weight columns); decode GEMMs stream half the bytes
         self.quantization = (quantization or "").lower() or None
         if self.quantization == "fp8":
+            if len(cls.dtypes) > 1:
+                raise ValueError(f"{cls.__name__} has no fp8 weights")
             from ..parallel.layers import quantize_fp8_
             quantize_fp8_(self.model)
         elif self.quantization not in (None, "none", "bf16"):
@@ -362,25 +376,25 @@ class LLMEngine:
         self.max_blocks = (self.max_model_len + KV_BLOCK - 1) // KV_BLOCK
         self.cross_tokens = self.model.tokens_per_image if self.mcfg is not None else 0
         self.max_cross_blocks = (self.cross_tokens + KV_BLOCK - 1) // KV_BLOCK
-        hk = self.model.kv_heads_local
         per_seq = self.max_blocks + self.max_cross_blocks
         if num_kv_blocks is None:
             if self.device.type == "cuda":
                 free, total = torch.cuda.mem_get_info(self.device)
                 budget = free - (1 - gpu_memory_utilization) * total
-                num_kv_blocks = int(max(budget, 0) // kv_bytes_per_block(cfg, hk))
+                num_kv_blocks = int(max(budget, 0) // self.model.cache_bytes_per_block())
                 num_kv_blocks = max(16, min(num_kv_blocks, max_num_seqs * per_seq + 64))
             else:
                 num_kv_blocks = max_num_seqs * per_seq + 8
         self.num_kv_blocks = num_kv_blocks
-        self.kv_buf, self.kv = allocate_kv_cache(cfg, hk, num_kv_blocks, self.device)
+        self.kv_buf, self.kv = self.model.allocate_cache(num_kv_blocks, self.device)
         self.bm = BlockManager(num_kv_blocks)
         self.prefill_token_budget = prefill_token_budget
         # longest prompt slice one prefill step processes (chunked prefill; SURVEY 5.7: <= 8k tokens)
         self.prefill_chunk = max(KV_BLOCK, prefill_chunk or prefill_token_budget)
         self._last_step = "decode"
         # packed varlen prefill (no [B, S_max] padding) with decode rows mixed into prefill steps (text models)
-        self.packed_prefill = packed_prefill and os.environ.get("SHAI_PADDED_PREFILL", "0") != "1"
+        self.packed_prefill = ((packed_prefill and os.environ.get("SHAI_PADDED_PREFILL", "0") != "1")
+                               or self.model.needs_prev_token)   # those models have the packed layout only
         self.mixed_steps = mixed_steps
         self.prefix_caching = enable_prefix_caching
         self.use_graphs = use_graphs and self.device.type == "cuda"
@@ -402,7 +416,8 @@ class LLMEngine:
         self.tok_host = [torch.zeros(bmax, dtype=torch.int32, pin_memory=pin) for _ in range(2)]
         self.tok_flip = 0
         self.stats = {"prefill_tokens": 0, "decode_tokens": 0, "steps": 0, "prefix_hit_tokens": 0}
-        self.eos = {cfg.eos_token_id}
+        self.eos = {cfg.eos_token_id} - {None}
+        self.driven: List[Sequence_] = []   # requests fed from outside (open_request / extend / close_request)
 
     def decode_splits(self, Bc: int, max_ctx: int) -> int:
         """Split-K factor of the decode attention for a batch whose longest context is ``max_ctx`` tokens:
@@ -410,7 +425,9 @@ class LLMEngine:
         head) workgroup walks more than ``SHAI_DECODE_SPLIT_TOKENS`` (1024) tokens when a long-context
         sequence is in the batch (one 16k-token sequence among short ones would otherwise stream its whole
         cache through 1-2 workgroups per head).  Powers of two: each value is one captured graph."""
-        base = ops.decode_splits(Bc, self.model.kv_heads_local, self.max_model_len)
+        span = self.model.attn_span or self.max_model_len
+        max_ctx = min(max_ctx, span)
+        base = ops.decode_splits(Bc, self.model.kv_heads_local, min(self.max_model_len, span))
         per = int(os.environ.get("SHAI_DECODE_SPLIT_TOKENS", "1024"))
         need = 1
         while need < 64 and need * per < max_ctx:
@@ -561,14 +578,7 @@ class LLMEngine:
         d = self.device
         t = lambda a: torch.from_numpy(a).to(d, non_blocking=True)
         if packed:
-            from ..runtime import build_prefill_packed
-            pos, slots, lens, qlens, qstart, bt, last = build_prefill_packed([s.n_cached for s in rows], news,
-                                                                             [s.blocks for s in rows],
-                                                                             self.max_blocks)
-            ids = np.concatenate([np.asarray((s.prompt if not s.output else s.tokens)[s.n_cached:s.n_cached + n],
-                                             dtype=np.int32) for s, n in zip(rows, news)])
-            batch = Batch(t(ids), t(pos), t(slots), t(bt), t(lens), t(qlens), len(rows), S, True, 1,
-                          t(last).long(), q_start=t(qstart))
+            batch = self._packed_batch(rows, news)
         else:
             from ..runtime import build_prefill
             pos, slots, lens, qlens, bt, last = build_prefill([s.n_cached for s in seqs], news,
@@ -602,6 +612,73 @@ class LLMEngine:
         if done:
             sel = logits if len(done) == len(rows) else logits.index_select(0, torch.tensor(done, device=d))
             self._sample_and_append([rows[i] for i in done], sel)
+
+    def _packed_batch(self, rows: Sequence[Sequence_], news: Sequence[int], want: Optional[np.ndarray] = None) -> Batch:
+        """The varlen batch of the next ``news[i]`` tokens of every sequence (prompt chunks and single decode tokens
+        alike).  ``want``: flat rows whose logits the step returns (default: each sequence's last)."""
+        from ..runtime import build_prefill_packed
+        t = lambda a: torch.from_numpy(a).to(self.device, non_blocking=True)
+        pos, slots, lens, qlens, qstart, bt, last = build_prefill_packed([s.n_cached for s in rows], news,
+                                                                         [s.blocks for s in rows], self.max_blocks)
+        ids = np.empty(len(pos), dtype=np.int32)
+        prev = np.full(len(pos), -1, dtype=np.int32)
+        for s, n, at in zip(rows, news, qstart.tolist()):
+            toks = s.prompt if not s.output else s.tokens
+            ids[at:at + n] = toks[s.n_cached:s.n_cached + n]
+            prev[at + 1:at + n] = ids[at:at + n - 1]
+            if s.n_cached:
+                prev[at] = toks[s.n_cached - 1]
+        return Batch(t(ids), t(pos), t(slots), t(bt), t(lens), t(qlens), len(rows), max(news), True, 1,
+                     t(last if want is None else want).long(), q_start=t(qstart),
+                     prev_ids=t(prev) if self.model.needs_prev_token else None)
+
+    # ------------------------------------------------------------------ externally driven requests
+    def open_request(self) -> Sequence_:
+        """A request whose tokens are supplied by :meth:`extend` instead of being sampled (trace replay, scoring).
+        It takes a sequence slot and KV blocks like a generated one; :meth:`close_request` gives them back."""
+        if len(self.driven) + len(self.running) >= self.max_num_seqs:
+            raise MemoryError(f"all {self.max_num_seqs} sequence slots are in use")
+        s = Sequence_(next(self._ids), [], SamplingParams())
+        self.driven.append(s)
+        return s
+
+    def close_request(self, s: Sequence_) -> None:
+        self._free(s)
+        s.finished = True
+        self.driven.remove(s)
+
+    @torch.inference_mode()
+    def extend(self, entries: Sequence[tuple]) -> Optional[torch.Tensor]:
+        """Run one step on ``entries`` = [(request, its next tokens, places among them whose logits are wanted)] as
+        one batch, from the cache earlier steps left: single tokens through the decode program (HIP graph), anything
+        else as a packed prefill step.  Returns the wanted logits [n, vocab] in entry order (None: nothing wanted)."""
+        if any(not toks for _, toks, _ in entries):
+            raise ValueError("an entry needs at least one token")
+        vocab = self.cfg.vocab_size
+        if any(not 0 <= t < vocab for _, toks, _ in entries for t in toks):
+            raise ValueError(f"token ids must lie in 0 .. {vocab - 1}")
+        for s, toks, _ in entries:
+            if s.length + len(toks) > self.max_blocks * KV_BLOCK:
+                raise ValueError(f"request longer than max_model_len {self.max_model_len}")
+            if not self._ensure_blocks(s, s.length + len(toks)):
+                raise MemoryError("KV block pool exhausted")
+        rows = [s for s, _, _ in entries]
+        news = [len(toks) for _, toks, _ in entries]
+        for s, toks, _ in entries:
+            s.prompt += list(toks)
+        first = np.concatenate([[0], np.cumsum(news)])[:-1]
+        want = np.asarray([int(at) + w for at, (_, _, ws) in zip(first, entries) for w in ws], dtype=np.int32)
+        if max(news) == 1:
+            g = self._decode_program(rows, [s.n_cached for s in rows], logits=True)[0]
+            self._enqueue(g, rows, [s.n_cached for s in rows], [s.prompt[-1] for s in rows], [-1] * len(rows),
+                          [s.prompt[-2] if s.n_cached else -1 for s in rows], sampled=False)
+            out = g.logits.index_select(0, torch.from_numpy(want).to(self.device).long()) if len(want) else None
+        else:
+            out = self.model(self._packed_batch(rows, news, want if len(want) else None), self.kv)
+            out = out if len(want) else None
+        for s, n in zip(rows, news):
+            s.n_cached += n
+        return out
 
     # ------------------------------------------------------------------ images (multimodal models)
     def _encode_images(self, seqs: List[Sequence_]):
@@ -661,27 +738,40 @@ class LLMEngine:
         seqs = [s for s in seqs if id(s) in running]
         if not seqs:
             return None
-        return self._launch(seqs, [s.length - 1 for s in seqs], [s.last_token for s in seqs], [-1] * len(seqs))
+        prev = ([s.output[-2] if len(s.output) > 1 else s.tokens[-2] if s.length > 1 else -1 for s in seqs]
+                if self.model.needs_prev_token else None)
+        return self._launch(seqs, [s.length - 1 for s in seqs], [s.last_token for s in seqs], [-1] * len(seqs), prev)
 
-    def _launch(self, seqs, ctx_before, ids, rowmap) -> _Inflight:
-        from ..runtime import build_decode
+    def _decode_program(self, seqs, ctx_before, logits: bool = False):
+        """The decode program (captured on first use) for this batch, and whether it is all-greedy.  ``logits``: one
+        that publishes its logits instead of sampling inside."""
         B = len(seqs)
-        pos, slots, lens, bt = build_decode(ctx_before, [s.blocks for s in seqs], self.max_blocks)
         Bc = 1 << max(0, math.ceil(math.log2(B)))
         cross = self._cross_tables(seqs) if any(s.cross_blocks for s in seqs) else None
-        greedy = all(s.params.temperature <= 0 for s in seqs)
-        splits = self.decode_splits(Bc, int(lens.max()) if B else 0)
-        full = (not greedy) and any(s.params.temperature > 0 and not 0 < s.params.top_k <= ops.SAMPLER_MAX_K
+        greedy = not logits and all(s.params.temperature <= 0 for s in seqs)
+        splits = self.decode_splits(Bc, max(ctx_before) + 1 if B else 0)
+        full = logits or (not greedy) and any(s.params.temperature > 0 and not 0 < s.params.top_k <= ops.SAMPLER_MAX_K
                                     for s in seqs)
         key = (Bc, cross is not None, greedy, splits) + ((True,) if full else ())
         g = self._graphs.get(key)
         if g is None:
             g = self._graphs[key] = _DecodeGraph(self, Bc, cross=cross is not None, greedy=greedy, splits=splits,
                                                  full_vocab=full)
+        return g, cross, greedy
+
+    def _enqueue(self, g, seqs, ctx_before, ids, rowmap, prev, cross=None, uniforms=None, sampled=True):
+        from ..runtime import build_decode
+        pos, slots, lens, bt = build_decode(ctx_before, [s.blocks for s in seqs], self.max_blocks)
+        u = uniforms if uniforms is not None else np.zeros(len(seqs), np.float32)
+        return g.launch(seqs, pos, slots, lens, bt, ids, rowmap, u, cross, prev, sampled)
+
+    def _launch(self, seqs, ctx_before, ids, rowmap, prev=None) -> _Inflight:
+        B = len(seqs)
+        g, cross, greedy = self._decode_program(seqs, ctx_before)
         # noise for the token each row samples, at absolute position ctx_before + 1
         u = (seq_uniforms([s.rng_key for s in seqs], [c + 1 for c in ctx_before]) if not greedy
-             else np.zeros(B, np.float32))
-        toks, ev = g.launch(seqs, pos, slots, lens, bt, ids, rowmap, u, cross)
+             else None)
+        toks, ev = self._enqueue(g, seqs, ctx_before, ids, rowmap, prev, cross, u)
         self.stats["decode_tokens"] += B
         return _Inflight(seqs, toks, ev, cross is not None)
 
@@ -722,7 +812,8 @@ class LLMEngine:
         for s in nxt:  # blocks for the token fed at position s.length (prev's output)
             if not self._ensure_blocks(s, s.length + 1):
                 return None
-        return self._launch(nxt, [s.length for s in nxt], [0] * len(nxt), rows)
+        # the token fed follows prev's input token, which the host already knows
+        return self._launch(nxt, [s.length for s in nxt], [0] * len(nxt), rows, [s.last_token for s in nxt])
 
     def _sample_and_append(self, seqs, logits):
         d = self.device
@@ -978,17 +1069,18 @@ class LLMService:
         return text, time.time() - t0, s
 
 
-def llama_config_for(model_id: str, model_path: Optional[str] = None, size: str = "") -> LlamaConfig:
-    import json
+def llama_config_for(model_id: str, model_path: Optional[str] = None, size: str = ""):
+    """The config of a checkpoint folder (its config.json), else the one a model id names."""
+    from ..models.golulix import GolulixConfig
     from ..models.mllama import MllamaConfig
-    if model_path and os.path.exists(os.path.join(model_path, "config.json")):
-        with open(os.path.join(model_path, "config.json")) as f:
-            d = json.load(f)
-        if "vision_config" in d and "text_config" in d:
-            return MllamaConfig.from_hf(d)
-        d = d.get("text_config", d)
-        return LlamaConfig.from_hf(d)
+    cfg = config_from_path(model_path)
+    if cfg is not None:
+        return cfg
     m = (model_id or "").lower()
+    if "golulix" in m:
+        if size != "tiny":
+            raise ValueError("Golulix has no published size: give the folder of a checkpoint (config.json)")
+        return GolulixConfig.tiny()
     vision = "vision" in m or "mllama" in m
     if size == "tiny":
         return MllamaConfig.tiny() if vision else LlamaConfig.tiny()

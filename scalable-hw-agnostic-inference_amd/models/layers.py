@@ -239,6 +239,10 @@ def init_random_(module: nn.Module, seed: int = 0, std_scale: float = 1.0) -> nn
             continue
         g = torch.Generator(device=own[0].device)
         g.manual_seed(seed * 1000003 + i)
+        if hasattr(m, "init_random_"):   # blocks with padded / packed weights fill their own
+            m.init_random_(g)
+            covered.update(id(p) for p in own)
+            continue
         if hasattr(m, "full_shape") and hasattr(m, "_shard"):
             # tensor-parallel layer: draw the FULL (unsharded) tensor from the shared seed and keep this rank's
             # shard, so a TP=n replica holds exactly the TP=1 model's weights (random-init serving at any TP)

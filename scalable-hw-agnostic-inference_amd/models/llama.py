@@ -158,6 +158,8 @@ class Batch:
     # packed varlen prefill: T = sum(q_lens) rows, sequence b's rows start at q_start[b] (no padding rows);
     # S is then max(q_lens).  None = the padded [B, S] layout.
     q_start: Optional[torch.Tensor] = None
+    # each row's preceding token (-1: the row is its sequence's first), for models with ``needs_prev_token``
+    prev_ids: Optional[torch.Tensor] = None
 
 
 class LlamaAttention(nn.Module):
@@ -231,6 +233,10 @@ class LlamaDecoderLayer(nn.Module):
 
 
 class LlamaForCausalLM(nn.Module):
+    dtypes = (torch.bfloat16,)
+    needs_prev_token = False
+    attn_span: Optional[int] = None   # full causal attention
+
     def __init__(self, cfg: LlamaConfig):
         super().__init__()
         self.cfg = cfg
@@ -267,6 +273,12 @@ class LlamaForCausalLM(nn.Module):
     @property
     def kv_heads_local(self) -> int:
         return self.layers[0].self_attn.hk
+
+    def cache_bytes_per_block(self) -> int:
+        return kv_bytes_per_block(self.cfg, self.kv_heads_local)
+
+    def allocate_cache(self, blocks: int, device):
+        return allocate_kv_cache(self.cfg, self.kv_heads_local, blocks, device)
 
     def rope(self, device):
         if self._rope is None or self._rope[0].device != torch.device(device):

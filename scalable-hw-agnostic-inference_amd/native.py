@@ -18,18 +18,37 @@ import torch
 DEBUG = os.environ.get("SHAI_KERNEL_DEBUG", "0") == "1"
 _DIR = os.path.join(os.path.dirname(os.path.abspath(__file__)), "_native_debug" if DEBUG else "_native")
 KERNELS_LIB = os.path.join(_DIR, "libshai_kernels.so")
+LM_LIB = os.path.join(_DIR, "libshai_lm.so")
 RUNTIME_LIB = os.path.join(_DIR, "libshai_runtime.so")
 COMM_LIB = os.path.join(_DIR, "libshai_comm.so")
 
 _lock = threading.Lock()
 _kernels_loaded = False
 _kernels_error: Exception | None = None
+_lm_loaded = False
 _runtime = None
 _comm = None
 
 
 class NativeUnavailable(RuntimeError):
     pass
+
+
+def _load_lm() -> None:
+    global _lm_loaded
+    if not _lm_loaded:
+        if not os.path.exists(LM_LIB):
+            raise NativeUnavailable(f"{LM_LIB} not found; run `python csrc/build.py`")
+        torch.ops.load_library(LM_LIB)
+        _lm_loaded = True
+
+
+def lm_ops():
+    """``torch.ops.shai`` with the decoder-block and token-level ops (``libshai_lm.so``) loaded; raises if missing."""
+    if not _lm_loaded:
+        with _lock:
+            _load_lm()
+    return torch.ops.shai
 
 
 def _load_kernels() -> None:
@@ -41,6 +60,7 @@ def _load_kernels() -> None:
             if not os.path.exists(KERNELS_LIB):
                 raise NativeUnavailable(f"{KERNELS_LIB} not found; run `python csrc/build.py`")
             torch.ops.load_library(KERNELS_LIB)
+            _load_lm()
             _kernels_loaded = True
             _autoload_tuning()
         except Exception as e:  # pragma: no cover - depends on build state

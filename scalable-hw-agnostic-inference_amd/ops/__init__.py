@@ -686,7 +686,7 @@ def rope_qkv_cache(qkv, positions, cos, sin, k_cache, v_cache, slots, heads: int
 
 def sample(logits, temps, top_k, top_p, uniforms, out):
     """Fused temperature / top-k / top-p sampling (GPU only; one workgroup per row)."""
-    _K().sample(logits, temps, top_k, top_p, uniforms, out)
+    native.lm_ops().sample(logits, temps, top_k, top_p, uniforms, out)
     return out
 
 
@@ -751,7 +751,7 @@ def token_feedback(ids, rowmap, prev):
         prev_rows = prev.index_select(0, rowmap.clamp(min=0).long())
         ids.copy_(torch.where(rowmap >= 0, prev_rows, ids))
         return ids
-    _K().token_feedback(ids, rowmap, prev)
+    native.lm_ops().token_feedback(ids, rowmap, prev)
     return ids
 
 

@@ -10,7 +10,7 @@ from setuptools.command.build_py import build_py
 
 ROOT = os.path.dirname(os.path.abspath(__file__))
 PKG_DIR = "scalable-hw-agnostic-inference_amd"
-LIBS = ["libshai_kernels.so", "libshai_runtime.so", "libshai_comm.so"]
+LIBS = ["libshai_kernels.so", "libshai_lm.so", "libshai_runtime.so", "libshai_comm.so"]
 
 
 class BuildWithNative(build_py):

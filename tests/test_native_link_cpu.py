@@ -8,7 +8,7 @@ import pytest
 from shai_amd import native
 
 
-@pytest.mark.parametrize("lib", [native.KERNELS_LIB, native.RUNTIME_LIB, native.COMM_LIB])
+@pytest.mark.parametrize("lib", [native.KERNELS_LIB, native.LM_LIB, native.RUNTIME_LIB, native.COMM_LIB])
 def test_native_library_links(lib):
     if not os.path.exists(lib):
         pytest.skip(f"{lib} not built (python csrc/build.py)")
