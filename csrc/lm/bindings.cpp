@@ -4,6 +4,7 @@
 #include <ATen/ATen.h>
 #include <c10/hip/HIPStream.h>
 #include <torch/library.h>
+#include <algorithm>
 
 #include "kernels/launchers.h"
 #include "lm/lm.h"
@@ -155,7 +156,7 @@ void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<T
     SHAI_CHECK(offsets.has_value() && W.dim() == 3, "grouped lm_gemm: W [E, N, K], tiles and offsets");
     check_i32(*tiles, "tiles");
     check_i32(*offsets, "offsets");
-    SHAI_CHECK(offsets->numel() == W.size(0) + 1 && (bm == 16 || bm == 128), "grouped lm_gemm: offsets [E + 1], bm");
+    SHAI_CHECK(offsets->numel() == W.size(0) + 1 && (bm == 16 || bm == 128 || bm == 256), "grouped lm_gemm: offsets [E + 1], bm");
     g.tiles = tiles->data_ptr<int>();
     g.offsets = offsets->data_ptr<int>();
     g.n_tiles = tiles->size(0);
@@ -172,7 +173,7 @@ void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<T
   }
   if (g.M == 0) return;
   const long lim = 0x7fffffffL;
-  const bool tile = !f32 && (g.tiles ? bm == 128 : g.M > 64) && (long)g.a_rows * g.K * 2 < lim &&
+  const bool tile = !f32 && (g.tiles ? bm >= 128 : g.M > 64) && (long)g.a_rows * g.K * 2 < lim &&
                     (long)g.N * g.K * 2 < lim;
   if (tile) shai_lm::launch_gemm_tile(g, stream());
   else shai_lm::launch_gemm(g, f32, stream());
@@ -207,7 +208,7 @@ void moe_plan(const Tensor& ids, int64_t bm, const Tensor& offsets, const Tensor
   a.E = offsets.numel() - 1;
   a.bm = bm;
   a.n_tiles = tiles.size(0);
-  SHAI_CHECK(a.E >= 1 && a.E <= 1024 && (bm == 16 || bm == 128), "moe_plan: up to 1024 experts, bm 16 or 128");
+  SHAI_CHECK(a.E >= 1 && a.E <= 1024 && (bm == 16 || bm == 128 || bm == 256), "moe_plan: up to 1024 experts, bm 16 / 128 / 256");
   SHAI_CHECK(token_of.numel() == a.P && slot_of.numel() == a.P && tiles.size(1) == 2 &&
                  a.n_tiles >= std::min<long>(a.P, a.E + a.P / bm), "moe_plan outputs");
   a.ids = ids.data_ptr<int>();

@@ -49,8 +49,9 @@ struct Frag<float> {
 
 template <typename T, typename O, int MT, int NT, int NW>
 __global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) {
-  constexpr int U = sizeof(T) == 2 ? (NT == 1 ? 4 : 2) : 1;   // k-steps of W in flight per wave
-  __shared__ float4_ red[NW][NT * MT][64];
+  // k-steps of W in flight per wave
+  constexpr int U = sizeof(T) == 2 ? (MT * NT == 1 ? 8 : NT == 1 ? 4 : NT == 2 ? 2 : 1) : 1;
+  __shared__ float4_ red[NW][MT][64];
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int r = lane & 15, g = lane >> 4;
   const int n0 = blockIdx.x * 16 * NT;
@@ -104,34 +105,48 @@ __global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) 
     }
   }
 #pragma unroll
-  for (int i = 0; i < NT; ++i)
+  for (int i = 0; i < NT; ++i) {
+    if (i > 0) __syncthreads();
 #pragma unroll
-    for (int j = 0; j < MT; ++j) red[wid][i * MT + j][lane] = acc[i][j];
-  __syncthreads();
-  for (int t = wid; t < NT * MT; t += NW) {
-    float4_ c = red[0][t][lane];
+    for (int j = 0; j < MT; ++j) red[wid][j][lane] = acc[i][j];
+    __syncthreads();
+    for (int t = wid; t < MT; t += NW) {
+      float4_ c = red[0][t][lane];
 #pragma unroll
-    for (int w = 1; w < NW; ++w) c += red[w][t][lane];
-    const int m = row0 + 16 * (t % MT) + r;
-    if (m < rows_end) store_cols<O>(p, m, n0 + 16 * (t / MT) + 4 * g, c);
+      for (int w = 1; w < NW; ++w) c += red[w][t][lane];
+      const int m = row0 + 16 * t + r;
+      if (m < rows_end) store_cols<O>(p, m, n0 + 16 * i + 4 * g, c);
+    }
   }
 }
 
+// Workgroup shapes (16 MT rows of A x 16 NT rows of W, NW waves along K), from a sweep at decode sizes: enough
+// workgroups to fill the chip come first, then fewer passes over W (MT), then fewer re-reads of A (NT).
 template <typename T, typename O>
 static void stream(const GemmArgs& a, hipStream_t s) {
+  auto go = [&](auto kernel, int mt, int nt, int nw) {
+    const dim3 grid((a.N + 16 * nt - 1) / (16 * nt), a.tiles ? a.n_tiles : (a.M + 16 * mt - 1) / (16 * mt),
+                    a.tiles ? (a.bm + 16 * mt - 1) / (16 * mt) : 1);
+    kernel<<<grid, 64 * nw, 0, s>>>(a);
+  };
+#define GO(MT_, NT_, NW_) go(gemm_stream_kernel<T, O, MT_, NT_, NW_>, MT_, NT_, NW_)
   const int rows = a.tiles ? a.bm : a.M;
-  const int mt = rows <= 16 ? 1 : rows <= 32 ? 2 : 4, nt = mt == 1 ? 1 : 2;
-  const dim3 grid((a.N + 16 * nt - 1) / (16 * nt), a.tiles ? a.n_tiles : (a.M + 16 * mt - 1) / (16 * mt),
-                  a.tiles ? (a.bm + 16 * mt - 1) / (16 * mt) : 1);
-  const bool deep = (long)grid.x * grid.y * grid.z < 1024 && a.K >= 1024;
-#define GO(MT_, NT_)                                                               \
-  do {                                                                             \
-    if (deep) gemm_stream_kernel<T, O, MT_, NT_, 8><<<grid, 512, 0, s>>>(a);       \
-    else gemm_stream_kernel<T, O, MT_, NT_, 4><<<grid, 256, 0, s>>>(a);            \
-  } while (0)
-  if (mt == 1) GO(1, 1);
-  else if (mt == 2) GO(2, 2);
-  else GO(4, 2);
+  if (rows <= 16) {
+    if (a.tiles && a.K < 2048) GO(1, 4, 4);
+    else GO(1, 1, 4);
+  } else if (a.tiles) {
+    GO(4, 2, 4);
+  } else if (a.N < 512) {
+    GO(1, 1, 4);
+  } else if (a.N < 3072) {
+    GO(2, 1, 8);
+  } else if (a.N < 5120) {
+    GO(2, 2, 8);
+  } else if (a.N < 16384 || rows <= 32) {
+    GO(2, 4, 8);
+  } else {
+    GO(4, 4, 4);
+  }
 #undef GO
   SHAI_CHECK_LAUNCH();
 }

@@ -1,5 +1,5 @@
-// C = epi(A W^T), LDS-tiled bf16 form for many rows (prefill): 128 x 128 tiles of 4 waves, 64-wide k-tiles moved global
-// -> LDS by DMA (buffer_load ... lds, 16 bytes per lane) into two stages; the load of k-tile t + 1 is issued before the
+// C = epi(A W^T), LDS-tiled bf16 form for many rows (prefill): 128 x 128 tiles of 4 waves or 256 x 256 tiles of 8, 64-wide
+// k-tiles moved global -> LDS by DMA (buffer_load ... lds, 16 bytes per lane) into two stages; the load of k-tile t + 1 is issued before the
 // MFMAs of t.  The bank swizzle is applied to the per-lane source chunk.  Buffer range checks zero-fill rows past the
 // ends.  Dense or grouped by expert: the row tiles of a grouped product come from the tile list, each with its own W and
 // with A rows gathered per lane.  Tiles are walked XCD by XCD in groups of 8 row tiles that share their W columns.
@@ -22,7 +22,7 @@ __device__ __forceinline__ void dma16(__amdgpu_buffer_rsrc_t r, bf16_t* lds_wave
 }
 
 template <typename O, int BM, int BN, int WM, int WN>
-__global__ void __launch_bounds__(WM * WN * 64, 2) gemm_tile_kernel(const GemmArgs p) {
+__global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_kernel(const GemmArgs p) {
   constexpr int NW = WM * WN, TM = BM / WM, TN = BN / WN, IM = TM / 32, JN = TN / 32;
   constexpr int JA = BM / 8 / NW, JB = BN / 8 / NW, STAGE = (BM + BN) * 64;
   extern __shared__ __attribute__((aligned(16))) bf16_t smem[];
@@ -127,18 +127,25 @@ __global__ void __launch_bounds__(WM * WN * 64, 2) gemm_tile_kernel(const GemmAr
   }
 }
 
-void launch_gemm_tile(const GemmArgs& a, hipStream_t s) {
-  constexpr int BM = 128, BN = 128;
+template <int BM, int BN, int WM, int WN>
+static void tile(const GemmArgs& a, hipStream_t s) {
   const int tiles_m = a.tiles ? a.n_tiles : (a.M + BM - 1) / BM;
   const int grid = tiles_m * ((a.N + BN - 1) / BN);
   constexpr int lds = 2 * (BM + BN) * 64 * 2;
   auto go = [&](auto k) {
     (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-    k<<<grid, 256, lds, s>>>(a);
+    k<<<grid, WM * WN * 64, lds, s>>>(a);
   };
-  if (a.out_f32) go(gemm_tile_kernel<float, BM, BN, 2, 2>);
-  else go(gemm_tile_kernel<bf16_t, BM, BN, 2, 2>);
+  if (a.out_f32) go(gemm_tile_kernel<float, BM, BN, WM, WN>);
+  else go(gemm_tile_kernel<bf16_t, BM, BN, WM, WN>);
   SHAI_CHECK_LAUNCH();
+}
+
+void launch_gemm_tile(const GemmArgs& a, hipStream_t s) {
+  // 256 x 256 tiles (8 waves) once they fill the chip, 128 x 128 (4 waves, two workgroups per CU) below
+  const bool big = a.tiles ? a.bm == 256 : (long)((a.M + 255) / 256) * ((a.N + 255) / 256) >= 192;
+  if (big) tile<256, 256, 2, 4>(a, s);
+  else tile<128, 128, 2, 2>(a, s);
 }
 
 }  // namespace shai_lm

@@ -48,7 +48,7 @@ struct GemmArgs {
   int M, N, K;
   int n_tiles;
   int a_rows;              // rows of A
-  int bm;                  // grouped row tile (16 or 128)
+  int bm;                  // grouped row tile (16, 128 or 256)
   int epi;
   float param;
   bool out_f32;

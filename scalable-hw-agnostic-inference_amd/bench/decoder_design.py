@@ -1,0 +1,104 @@
+"""Prefill and decode throughput of the Golulix design beside a Llama-family model of equal size.
+
+Both run through :class:`LLMEngine` (scheduler, paged cache, HIP-graph decode) with random weights.  A pair has the same
+width, layers, heads, head size and vocabulary, and the Llama MLP is as wide as the feed-forward work one Golulix token
+does (top x expert + shared expert), so the two do the same matrix work per token.
+
+    python bench.py --workload golulix [--golulix-size small|large|both]
+    python -m shai_amd.bench.decoder_design --model golulix --size small --phase decode --batch 64   # profiling
+"""
+from __future__ import annotations
+
+import argparse
+import time
+
+# width, layers, heads, kv heads, head size, chunk, experts, top, expert ff, shared ff, vocab, expert groups, kept
+SIZES = {"small": (2048, 8, 16, 4, 128, 2048, 64, 6, 1408, 2816, 32768, 8, 4),
+         "large": (4096, 6, 32, 8, 128, 8192, 64, 4, 2048, 4096, 65536, 4, 2)}
+
+
+def configs(size: str):
+    from ..models.golulix import GolulixConfig
+    from ..models.llama import LlamaConfig
+    D, L, H, G, d, chunk, E, top, ff, sff, V, groups, keep = SIZES[size]
+    gol = GolulixConfig.uniform(layers=L, width=D, heads=H, kv_heads=G, dim=d, chunk=chunk, experts=E, top=top, ff=ff,
+                                shared_ff=sff, vocab=V, groups=groups, keep=keep)
+    ll = LlamaConfig(vocab_size=V, hidden_size=D, intermediate_size=top * ff + sff, num_hidden_layers=L,
+                     num_attention_heads=H, num_key_value_heads=G, head_dim=d, max_position_embeddings=32768)
+    return {"golulix": gol, "llama": ll}
+
+
+def measure(cfg, batch: int, prompt: int, gen: int, repeats: int = 3, device: str = "cuda:0") -> dict:
+    """Median prefill and decode tokens/s of ``batch`` prompts of ``prompt`` tokens, ``gen`` sampled tokens each."""
+    import numpy as np
+    import torch
+    from ..engines.llm import LLMEngine, SamplingParams
+    eng = LLMEngine(cfg, device=device, max_num_seqs=batch, max_model_len=prompt + gen + 64, enable_prefix_caching=False,
+                    prefill_token_budget=batch * prompt)
+    rng = np.random.default_rng(0)
+    params = SamplingParams(temperature=0.7, top_k=50, top_p=0.9, max_tokens=gen, ignore_eos=True)
+    sync = torch.cuda.synchronize if eng.device.type == "cuda" else (lambda: None)
+    pre, dec = [], []
+    with torch.inference_mode():
+        for r in range(repeats + 1):            # the first pass captures graphs and tunes GEMMs: not counted
+            seqs = [eng.add_request(rng.integers(0, cfg.vocab_size, prompt).tolist(), params) for _ in range(batch)]
+            sync()
+            t0 = time.perf_counter()
+            while any(not s.output for s in seqs):
+                eng.step()
+            sync()
+            t1 = time.perf_counter()
+            while eng.has_work():
+                eng.step()
+            sync()
+            t2 = time.perf_counter()
+            if r:
+                pre.append(batch * prompt / (t1 - t0))
+                dec.append(batch * (gen - 1) / (t2 - t1) if gen > 1 else 0.0)
+    del eng
+    if device != "cpu":
+        torch.cuda.empty_cache()
+    return {"prefill_tok_s": round(sorted(pre)[len(pre) // 2], 1), "decode_tok_s": round(sorted(dec)[len(dec) // 2], 1)}
+
+
+def bench(args, rank: int, world: int) -> dict:
+    """The bench.py line: every (size, batch) pair of both models; ``value`` is Golulix decode at the largest batch."""
+    import torch
+    if world != 1:
+        raise SystemExit("--workload golulix runs on one GPU")
+    sizes = list(SIZES) if args.golulix_size == "both" else [args.golulix_size]
+    rows, P, G, t0 = [], 1024, 64, time.perf_counter()
+    steps = max(1, args.steps)
+    for size in sizes:
+        cfgs = configs(size)
+        for batch in (1, 8, args.batch):
+            row = {"size": size, "batch": batch, "prompt_len": P, "gen_len": G}
+            for name, cfg in cfgs.items():
+                row[name] = measure(cfg, batch, P, G, steps, f"cuda:{torch.cuda.current_device()}")
+            rows.append(row)
+    last = rows[-1]
+    return {"metric": "Golulix decode tokens/s (random weights, beside a Llama model of equal size)",
+            "value": last["golulix"]["decode_tok_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": 1,
+            "ms_per_step": round(1000 * (time.perf_counter() - t0) / (len(rows) * 2 * (steps + 1)), 2),
+            "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16",
+            "data": "synthetic prompts, random-init weights",
+            "config": {"model": f"Golulix {last['size']}: (width, layers, heads, kv heads, head size, chunk, experts, "
+                                f"top, expert ff, shared ff, vocab, groups, kept) = {SIZES[last['size']]}",
+                       "global_batch": last["batch"], "seq_len": P + G, "parallelism": "dp1"},
+            "pairs": rows}
+
+
+def main(argv=None):
+    ap = argparse.ArgumentParser()
+    ap.add_argument("--model", choices=["golulix", "llama"], default="golulix")
+    ap.add_argument("--size", choices=sorted(SIZES), default="small")
+    ap.add_argument("--batch", type=int, default=64)
+    ap.add_argument("--prompt", type=int, default=1024)
+    ap.add_argument("--gen", type=int, default=64)
+    ap.add_argument("--repeats", type=int, default=2)
+    a = ap.parse_args(argv)
+    print(measure(configs(a.size)[a.model], a.batch, a.prompt, a.gen, a.repeats), flush=True)
+
+
+if __name__ == "__main__":
+    main()

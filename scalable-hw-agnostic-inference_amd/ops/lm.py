@@ -112,9 +112,9 @@ def matmul(a, w, out_dtype=None, epi: int = EPI_NONE, param: float = 0.0, plan: 
 
 
 def grouped_bm(rows: int, experts: int) -> int:
-    """Row tile of a grouped product over ``rows`` slots: 16-row streaming tiles while an expert sees few rows, 128-row
-    LDS tiles once it sees enough of them to be compute-bound."""
-    return 16 if rows < 48 * experts else 128
+    """Row tile of a grouped product over ``rows`` slots: 16-row streaming tiles while an expert sees few rows, LDS
+    tiles of 128 rows once it sees enough of them to be compute-bound, of 256 when those fill up."""
+    return 16 if rows < 48 * experts else 128 if rows < 512 * experts else 256
 
 
 def route(logits, top: int, groups: int, keep: int):

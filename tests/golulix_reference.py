@@ -32,6 +32,19 @@ def chunk_visible(n, size):
     return (i[None, :] <= i[:, None]) & (i[None, :] // size == i[:, None] // size)
 
 
+def attend(q, k, v, gate, chunk, scale):
+    """q [n, H, dk], k [n, G, dk], v [n, G, dv], gate logits [n, H] -> [n, H * dv]."""
+    n, H, G = q.shape[0], q.shape[1], k.shape[1]
+    see = chunk_visible(n, chunk)
+    outs = []
+    for hd in range(H):
+        g = hd // (H // G)
+        s = (q[:, hd] @ k[:, g].T) * scale
+        p = torch.softmax(s.masked_fill(~see, float("-inf")), -1)
+        outs.append((p @ v[:, g]) * torch.sigmoid(gate[:, hd:hd + 1]))
+    return torch.cat(outs, -1)
+
+
 def attention(h, mc, get):
     """h [n, width] -> [n, width]; ``get(name)`` returns the mixer's tensor."""
     n = h.shape[0]
@@ -39,15 +52,7 @@ def attention(h, mc, get):
     q = (h @ get("q").T).view(n, H, dk)
     k = (h @ get("k").T).view(n, G, dk)
     v = (h @ get("v").T).view(n, G, dv)
-    gate = torch.sigmoid(h @ get("g").T)
-    see = chunk_visible(n, mc["mask"]["size"])
-    outs = []
-    for hd in range(H):
-        g = hd // (H // G)
-        s = (q[:, hd] @ k[:, g].T) * mc["scale"]
-        p = torch.softmax(s.masked_fill(~see, float("-inf")), -1)
-        outs.append((p @ v[:, g]) * gate[:, hd:hd + 1])
-    return torch.cat(outs, -1) @ get("o").T
+    return attend(q, k, v, h @ get("g").T, mc["mask"]["size"], mc["scale"]) @ get("o").T
 
 
 def expert(h, gate, up, down, limit):
@@ -116,7 +121,7 @@ def forward(tokens, cfg, w, dtype=torch.float64):
 
 
 def random_config(vocab=96, width=48, layers=3, heads=4, kv_heads=2, dim=16, vdim=24, chunk=20, scale=0.3, ff=24,
-                  limit=1.5, experts=8, top=2, groups=4, keep=2, shared_ff=40, shared_limit=0.75, eps=1e-5, cap=9.0,
+                  limit=1.5, experts=12, top=2, groups=3, keep=1, shared_ff=40, shared_limit=0.75, eps=1e-5, cap=9.0,
                   loop=(1, 2, 3), bigram=(61, 29, 5), no_mlp=()):
     layer = lambda i: {
         "type": "attention",
