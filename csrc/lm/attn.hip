@@ -5,7 +5,7 @@
 //
 // kv_store      the step's k / v rows into the cache.
 // prefill       bf16: flash attention, 4 waves x 32 queries, scores swapped (S^T = K Q^T) so that a lane holds one
-//               query's scores, P feeds O^T = V^T P^T from registers; only the 64-key blocks of the chunks that the
+//               query's scores, P feeds O^T = V^T P^T from registers as a bf16 pair (value + remainder); only the 64-key blocks of the chunks that the
 //               workgroup's queries lie in are visited.  fp32: attn_rows.
 // decode        bf16: one workgroup per (sequence, kv head, split); each wave takes whole 64-key blocks, K straight from
 //               memory into the matrix cores (the group's query heads are the 16 columns), fp32 P against V on the
@@ -224,7 +224,7 @@ __global__ void __launch_bounds__(256, DK + DV > 256 ? 1 : 2) attn_prefill_kerne
     const float alpha = __builtin_amdgcn_exp2f(m_run - m_use);
     m_run = m_new;
     float ls4[4] = {0.f, 0.f, 0.f, 0.f};
-    bf16x8 pf[2][2];
+    bf16x8 pf[2][2], pl[2][2];                   // P as bf16 plus its bf16 remainder: 16 significant bits
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb) {
 #pragma unroll
@@ -235,10 +235,14 @@ __global__ void __launch_bounds__(256, DK + DV > 256 ? 1 : 2) attn_prefill_kerne
       }
 #pragma unroll
       for (int s = 0; s < 2; ++s) {
-        bf16x8 v;
+        bf16x8 v, u;
 #pragma unroll
-        for (int j = 0; j < 8; ++j) v[j] = (__bf16)sacc[kb][8 * s + j];
+        for (int j = 0; j < 8; ++j) {
+          v[j] = (__bf16)sacc[kb][8 * s + j];
+          u[j] = (__bf16)(sacc[kb][8 * s + j] - (float)v[j]);
+        }
         pf[kb][s] = v;
+        pl[kb][s] = u;
       }
     }
     l_run = l_run * alpha + ((ls4[0] + ls4[1]) + (ls4[2] + ls4[3]));
@@ -265,6 +269,7 @@ __global__ void __launch_bounds__(256, DK + DV > 256 ? 1 : 2) attn_prefill_kerne
 #pragma unroll
           for (int j = 0; j < 4; ++j) { vv[j] = u0[j]; vv[4 + j] = u1[j]; }
           o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, vv), pf[kb][s], o[d], 0, 0, 0);
+          o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, vv), pl[kb][s], o[d], 0, 0, 0);
         }
       }
     }
@@ -475,18 +480,24 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(const AttnArgs p, int 
 }
 
 __global__ void __launch_bounds__(256) attn_decode_fold_kernel(const AttnArgs p) {
+  __shared__ float se[64];
+  __shared__ float total;
   const int h = blockIdx.x, b = blockIdx.y, d = threadIdx.x;
-  if (d >= p.dv) return;
   const float* ws = p.ws + ((long)b * p.H + h) * p.splits * (p.dv + 2);
-  float M = -INFINITY;
-  for (int s = 0; s < p.splits; ++s) M = fmaxf(M, ws[(long)s * (p.dv + 2) + p.dv]);
-  float L = 0.f, x = 0.f;
-  for (int s = 0; s < p.splits; ++s) {
-    const float* q = ws + (long)s * (p.dv + 2);
-    const float e = __builtin_amdgcn_exp2f(q[p.dv] - M);
-    L += q[p.dv + 1] * e;
-    x += q[d] * e;
+  if (d < 64) {                                  // one lane per split (at most 64)
+    const float* q = ws + (long)min(d, p.splits - 1) * (p.dv + 2) + p.dv;
+    const float m = d < p.splits ? q[0] : -INFINITY, l = q[1];
+    const float e = d < p.splits ? __builtin_amdgcn_exp2f(m - wave_max(m)) : 0.f;
+    se[d] = e;
+    const float L = wave_sum(l * e);
+    if (d == 0) total = L;
   }
+  __syncthreads();
+  if (d >= p.dv) return;
+  float x = 0.f;
+#pragma unroll 8
+  for (int s = 0; s < p.splits; ++s) x += ws[(long)s * (p.dv + 2) + d] * se[s];
+  const float L = total;
   const float gate = bf2f(static_cast<const bf16_t*>(p.qkvg)[(long)b * p.ld + (long)p.H * p.dk +
                                                              (long)p.G * (p.dk + p.dv) + h]);
   static_cast<bf16_t*>(p.o)[((long)b * p.H + h) * p.dv + d] = f2bf(x / L * sigmoid_f(gate));

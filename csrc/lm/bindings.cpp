@@ -132,7 +132,8 @@ void add_norm(const Tensor& x, const optional<Tensor>& dense, const optional<Ten
 }
 
 void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<Tensor>& tiles,
-             const optional<Tensor>& offsets, const optional<Tensor>& gather, int64_t bm, int64_t epi, double param) {
+             const optional<Tensor>& offsets, const optional<Tensor>& gather, int64_t bm, int64_t epi, double param,
+             const optional<Tensor>& side) {
   const bool f32 = is_f32(A);
   check(A, A.scalar_type(), "A");
   check(W, A.scalar_type(), "W");
@@ -147,8 +148,18 @@ void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<T
   g.param = param;
   g.out_f32 = C.scalar_type() == at::kFloat;
   SHAI_CHECK(A.size(1) == g.K && g.K % 64 == 0 && g.N >= 1, "lm_gemm: K must match and be a multiple of 64");
-  SHAI_CHECK(epi >= 0 && epi <= 2 && (epi != shai_lm::EPI_CLAMP_GLU || g.N % 2 == 0), "lm_gemm epilogue");
-  SHAI_CHECK(C.size(1) == (epi == shai_lm::EPI_CLAMP_GLU ? g.N / 2 : g.N), "lm_gemm output columns");
+  SHAI_CHECK(epi >= 0 && epi <= 2, "lm_gemm epilogue");
+  g.n_main = g.N;
+  if (side) {  // the last rows of W are a plain product, stored in fp32
+    check(*side, at::kFloat, "side");
+    SHAI_CHECK(!tiles && epi == shai_lm::EPI_CLAMP_GLU && side->dim() == 2 && side->size(0) == g.M && side->size(1) >= 1 &&
+                   side->size(1) < g.N, "side output: dense GLU products, [M, last rows of W]");
+    g.n_main = g.N - side->size(1);
+    SHAI_CHECK(g.n_main % 4 == 0, "side output: the GLU rows of W must be a multiple of 4");
+    g.side = side->data_ptr<float>();
+  }
+  SHAI_CHECK(epi != shai_lm::EPI_CLAMP_GLU || g.n_main % 2 == 0, "GLU products need (gate, up) row pairs");
+  SHAI_CHECK(C.size(1) == (epi == shai_lm::EPI_CLAMP_GLU ? g.n_main / 2 : g.N), "lm_gemm output columns");
   g.A = A.data_ptr();
   g.W = W.data_ptr();
   g.C = C.data_ptr();
@@ -198,6 +209,42 @@ void moe_route(const Tensor& logits, int64_t groups, int64_t keep, const Tensor&
   if (a.T > 0) shai_lm::launch_route(a, stream());
 }
 
+// logits -> picks -> slots for up to 16 tokens in one launch (moe_route + moe_plan with 16-row tiles)
+void moe_route_plan(const Tensor& logits, int64_t groups, int64_t keep, const Tensor& ids, const Tensor& wts,
+                    const Tensor& offsets, const Tensor& token_of, const Tensor& slot_of, const Tensor& tiles) {
+  check(logits, at::kFloat, "logits");
+  check(wts, at::kFloat, "wts");
+  for (auto* t : {&ids, &offsets, &token_of, &slot_of, &tiles}) check_i32(*t, "moe_route_plan tensor");
+  shai_lm::RouteArgs r{};
+  r.T = logits.size(0);
+  r.E = logits.size(1);
+  r.top = ids.size(1);
+  r.groups = groups;
+  r.keep = keep;
+  SHAI_CHECK(r.T >= 1 && r.T <= 16 && r.E <= 256, "moe_route_plan: up to 16 tokens and 256 experts");
+  SHAI_CHECK(ids.size(0) == r.T && wts.sizes() == ids.sizes(), "route outputs must be [T, top]");
+  SHAI_CHECK(reinterpret_cast<uintptr_t>(ids.data_ptr()) % 16 == 0, "moe_route_plan: ids must be 16-byte aligned");
+  SHAI_CHECK(groups >= 1 && r.E % groups == 0 && keep >= 1 && keep <= groups && r.top >= 1 &&
+                 r.top <= keep * (r.E / groups), "route: experts in equal groups, top within the kept ones");
+  r.logits = logits.data_ptr<float>();
+  r.ids = ids.data_ptr<int>();
+  r.wts = wts.data_ptr<float>();
+  shai_lm::PlanArgs a{};
+  a.P = ids.numel();
+  a.top = r.top;
+  a.E = r.E;
+  a.bm = 16;
+  a.n_tiles = tiles.size(0);
+  SHAI_CHECK(offsets.numel() == a.E + 1 && token_of.numel() == a.P && slot_of.numel() == a.P && tiles.size(1) == 2 &&
+                 a.n_tiles >= std::min<long>(a.P, a.E + a.P / 16), "moe_route_plan outputs");
+  a.ids = r.ids;
+  a.offsets = offsets.data_ptr<int>();
+  a.token_of = token_of.data_ptr<int>();
+  a.slot_of = slot_of.data_ptr<int>();
+  a.tiles = tiles.data_ptr<int>();
+  shai_lm::launch_route_plan(r, a, stream());
+}
+
 // `ids` comes from moe_route (every entry in 0 .. E - 1)
 void moe_plan(const Tensor& ids, int64_t bm, const Tensor& offsets, const Tensor& token_of, const Tensor& slot_of,
               const Tensor& tiles) {
@@ -208,6 +255,7 @@ void moe_plan(const Tensor& ids, int64_t bm, const Tensor& offsets, const Tensor
   a.E = offsets.numel() - 1;
   a.bm = bm;
   a.n_tiles = tiles.size(0);
+  SHAI_CHECK(reinterpret_cast<uintptr_t>(ids.data_ptr()) % 16 == 0, "moe_plan: ids must be 16-byte aligned");
   SHAI_CHECK(a.E >= 1 && a.E <= 1024 && (bm == 16 || bm == 128 || bm == 256), "moe_plan: up to 1024 experts, bm 16 / 128 / 256");
   SHAI_CHECK(token_of.numel() == a.P && slot_of.numel() == a.P && tiles.size(1) == 2 &&
                  a.n_tiles >= std::min<long>(a.P, a.E + a.P / bm), "moe_plan outputs");
@@ -285,7 +333,7 @@ void chunk_attn_decode(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, c
   a.max_blocks = bt.size(1);
   SHAI_CHECK(a.B == a.T && ctx.numel() >= a.B && slots.numel() >= a.B && chunk >= 1 && a.B <= 65535,
              "decode: one row per sequence");
-  SHAI_CHECK(splits >= 1 && splits <= 65535 &&
+  SHAI_CHECK(splits >= 1 && splits <= 64 &&
                  (splits == 1 || (ws.scalar_type() == at::kFloat && ws.is_contiguous() &&
                                   ws.numel() >= (long)a.B * a.H * splits * (a.dv + 2))), "decode split workspace");
   a.bt = bt.data_ptr<int>();
@@ -331,8 +379,9 @@ void token_feedback(const Tensor& ids, const Tensor& rowmap, const Tensor& prev)
 TORCH_LIBRARY_FRAGMENT(shai, m) {
   m.def("embed_norm(Tensor ids, Tensor? prev, Tensor table, Tensor? bigram, int mul_prev, int mul_cur, Tensor w, float eps, int width, Tensor(a!) x, Tensor(b!) h) -> ()");
   m.def("add_norm(Tensor(a!) x, Tensor? dense, Tensor? ye, Tensor? slot_of, Tensor? wts, Tensor? inject, Tensor? rows, Tensor? w, float eps, int width, Tensor(b!)? h) -> ()");
-  m.def("lm_gemm(Tensor a, Tensor w, Tensor(a!) c, Tensor? tiles, Tensor? offsets, Tensor? gather, int bm, int epi, float param) -> ()");
+  m.def("lm_gemm(Tensor a, Tensor w, Tensor(a!) c, Tensor? tiles, Tensor? offsets, Tensor? gather, int bm, int epi, float param, Tensor(b!)? side=None) -> ()");
   m.def("moe_route(Tensor logits, int groups, int keep, Tensor(a!) ids, Tensor(b!) wts) -> ()");
+  m.def("moe_route_plan(Tensor logits, int groups, int keep, Tensor(a!) ids, Tensor(b!) wts, Tensor(c!) offsets, Tensor(d!) token_of, Tensor(e!) slot_of, Tensor(f!) tiles) -> ()");
   m.def("moe_plan(Tensor ids, int bm, Tensor(a!) offsets, Tensor(b!) token_of, Tensor(c!) slot_of, Tensor(d!) tiles) -> ()");
   m.def("kv_store(Tensor qkvg, Tensor(a!) k_cache, Tensor(b!) v_cache, Tensor slots, int heads) -> ()");
   m.def("chunk_attn_prefill(Tensor qkvg, Tensor k_cache, Tensor v_cache, Tensor(a!) o, Tensor block_table, Tensor ctx_lens, Tensor q_lens, Tensor q_start, int max_q, int heads, int chunk, float scale) -> ()");
@@ -346,6 +395,7 @@ TORCH_LIBRARY_IMPL(shai, CUDA, m) {
   m.impl("add_norm", &add_norm);
   m.impl("lm_gemm", &lm_gemm);
   m.impl("moe_route", &moe_route);
+  m.impl("moe_route_plan", &moe_route_plan);
   m.impl("moe_plan", &moe_plan);
   m.impl("kv_store", &kv_store);
   m.impl("chunk_attn_prefill", &chunk_attn_prefill);

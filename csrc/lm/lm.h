@@ -51,6 +51,8 @@ struct GemmArgs {
   int bm;                  // grouped row tile (16, 128 or 256)
   int epi;
   float param;
+  int n_main;              // columns n_main .. N - 1 are a plain fp32 product, stored in side [M, N - n_main]
+  float* side;
   bool out_f32;
 };
 void launch_gemm(const GemmArgs& a, bool f32, hipStream_t s);          // streaming kernel, any M
@@ -73,6 +75,7 @@ struct PlanArgs {
   int* tiles;              // [n_tiles][2]
 };
 void launch_plan(const PlanArgs& a, hipStream_t s);
+void launch_route_plan(const RouteArgs& r, const PlanArgs& a, hipStream_t s);   // T <= 16, E <= 256
 
 struct AttnArgs {
   const void* qkvg;        // [T, ld]: q (H dk), k (G dk), v (G dv), gate logits (H)

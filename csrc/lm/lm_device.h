@@ -42,8 +42,14 @@ __device__ __forceinline__ float block_sum256(float v, float* red) {
 template <typename O>
 __device__ __forceinline__ void store_cols(const GemmArgs& p, long m, int n, float4_ c) {
   O* out = static_cast<O*>(p.C);
+  if (n >= p.n_main) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (n + i < p.N) p.side[m * (p.N - p.n_main) + n + i - p.n_main] = c[i];
+    return;
+  }
   if (p.epi == EPI_CLAMP_GLU) {
-    const int ld = p.N >> 1, j = n >> 1;
+    const int ld = p.n_main >> 1, j = n >> 1;
     if (n < p.N) store1(out + m * ld + j, clamp_glu(c[0], c[1], p.param));
     if (n + 2 < p.N) store1(out + m * ld + j + 1, clamp_glu(c[2], c[3], p.param));
     return;

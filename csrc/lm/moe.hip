@@ -6,12 +6,10 @@ namespace shai_lm {
 
 // One wave per token; lane l holds experts l, l + 64, ...  All comparisons break ties by the lower expert index, and
 // picks are by a strictly decreasing (score, index) order, so every pick is a distinct expert whatever the scores are.
+// `sc` is the wave's LDS scratch, [E + groups] floats.  Every wave of the workgroup calls it (barriers inside).
 template <int NE>
-__global__ void __launch_bounds__(256) route_kernel(const RouteArgs p) {
-  extern __shared__ float sh[];                 // [4][E] scores, [4][groups] group scores
-  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
-  const int t = blockIdx.x * 4 + wid;
-  float* sc = sh + wid * (p.E + p.groups);
+__device__ __forceinline__ void route_token(const RouteArgs& p, int t, float* sc) {
+  const int lane = threadIdx.x & 63;
   float* gs = sc + p.E;
   const bool live = t < p.T;
   float z[NE];
@@ -84,6 +82,13 @@ __global__ void __launch_bounds__(256) route_kernel(const RouteArgs p) {
   }
 }
 
+template <int NE>
+__global__ void __launch_bounds__(256) route_kernel(const RouteArgs p) {
+  extern __shared__ float sh[];
+  const int wid = threadIdx.x >> 6;
+  route_token<NE>(p, blockIdx.x * 4 + wid, sh + wid * (p.E + p.groups));
+}
+
 void launch_route(const RouteArgs& a, hipStream_t s) {
   const int grid = (a.T + 3) / 4;
   const size_t lds = sizeof(float) * 4 * (a.E + a.groups);
@@ -96,12 +101,21 @@ void launch_route(const RouteArgs& a, hipStream_t s) {
 
 // One workgroup: LDS histogram, scan, tile list, scatter.  The order of rows inside an expert is arbitrary (each row is
 // computed alone, and the combine reads a token's slots in k order), so LDS atomics are enough.
-__global__ void __launch_bounds__(1024) plan_kernel(const PlanArgs p) {
-  __shared__ int cnt[1024], start[1025], tile0[1025];
+__device__ __forceinline__ void plan_body(const PlanArgs& p, int* cnt, int* start, int* tile0) {
   const int tid = threadIdx.x;
+  const int4* ids4 = reinterpret_cast<const int4*>(p.ids);
+  const int n4 = p.P / 4;
   for (int e = tid; e < p.E; e += 1024) cnt[e] = 0;
   __syncthreads();
-  for (int i = tid; i < p.P; i += 1024) atomicAdd(&cnt[p.ids[i]], 1);
+#pragma unroll 4
+  for (int i = tid; i < n4; i += 1024) {
+    const int4 v = ids4[i];
+    atomicAdd(&cnt[v.x], 1);
+    atomicAdd(&cnt[v.y], 1);
+    atomicAdd(&cnt[v.z], 1);
+    atomicAdd(&cnt[v.w], 1);
+  }
+  for (int i = 4 * n4 + tid; i < p.P; i += 1024) atomicAdd(&cnt[p.ids[i]], 1);
   __syncthreads();
   if (tid < 64) {                                // wave 0: exclusive scans of the counts and of the tile counts
     int base = 0, tbase = 0;
@@ -143,15 +157,49 @@ __global__ void __launch_bounds__(1024) plan_kernel(const PlanArgs p) {
   __syncthreads();
   for (int e = tid; e < p.E; e += 1024) cnt[e] = start[e];
   __syncthreads();
-  for (int i = tid; i < p.P; i += 1024) {
-    const int s = atomicAdd(&cnt[p.ids[i]], 1);
+  auto place = [&](int i, int e) {
+    const int s = atomicAdd(&cnt[e], 1);
     p.token_of[s] = i / p.top;
     p.slot_of[i] = s;
+  };
+#pragma unroll 4
+  for (int i = tid; i < n4; i += 1024) {
+    const int4 v = ids4[i];
+    place(4 * i, v.x);
+    place(4 * i + 1, v.y);
+    place(4 * i + 2, v.z);
+    place(4 * i + 3, v.w);
   }
+  for (int i = 4 * n4 + tid; i < p.P; i += 1024) place(i, p.ids[i]);
+}
+
+__global__ void __launch_bounds__(1024) plan_kernel(const PlanArgs p) {
+  __shared__ int cnt[1024], start[1025], tile0[1025];
+  plan_body(p, cnt, start, tile0);
 }
 
 void launch_plan(const PlanArgs& a, hipStream_t s) {
   plan_kernel<<<1, 1024, 0, s>>>(a);
+  SHAI_CHECK_LAUNCH();
+}
+
+// A decode step's few tokens: one wave routes each, then the same workgroup sorts the picks (they pass through global
+// memory inside the workgroup: written before the barrier, read after it).
+template <int NE>
+__global__ void __launch_bounds__(1024) route_plan_kernel(const RouteArgs r, const PlanArgs p) {
+  __shared__ int cnt[256], start[257], tile0[257];
+  extern __shared__ float sh[];
+  const int wid = threadIdx.x >> 6;
+  route_token<NE>(r, wid, sh + wid * (r.E + r.groups));
+  __syncthreads();
+  plan_body(p, cnt, start, tile0);
+}
+
+void launch_route_plan(const RouteArgs& r, const PlanArgs& a, hipStream_t s) {
+  const size_t lds = sizeof(float) * 16 * (r.E + r.groups);
+  if (r.E <= 64) route_plan_kernel<1><<<1, 1024, lds, s>>>(r, a);
+  else if (r.E <= 128) route_plan_kernel<2><<<1, 1024, lds, s>>>(r, a);
+  else route_plan_kernel<4><<<1, 1024, lds, s>>>(r, a);
   SHAI_CHECK_LAUNCH();
 }
 

@@ -157,12 +157,12 @@ class MoE(nn.Module):
         super().__init__()
         self.c, self.width = c, width
         W, F = lm.pad64(width), lm.pad64(c.expert.ff)
-        self.router = _param(c.experts, W, dtype=dtype)
+        # the shared expert's gate / up rows and the router's rows: one product
+        S = lm.pad64(c.shared.ff) if c.shared is not None else 0
+        self.front = _param(2 * S + c.experts, W, dtype=dtype)
         self.gate_up = _param(c.experts, 2 * F, W, dtype=dtype)
         self.down = _param(c.experts, W, F, dtype=dtype)
         if c.shared is not None:
-            S = lm.pad64(c.shared.ff)
-            self.shared_gate_up = _param(2 * S, W, dtype=dtype)
             self.shared_down = _param(W, S, dtype=dtype)
 
     def shapes(self) -> Dict[str, tuple]:
@@ -174,27 +174,27 @@ class MoE(nn.Module):
         return s
 
     def pack(self, get: Callable[[str], torch.Tensor]) -> Dict[str, torch.Tensor]:
-        c, W, F = self.c, self.router.shape[1], self.down.shape[2]
-        out = {"router": _padded(get("router"), c.experts, W),
+        c, W, F = self.c, self.front.shape[1], self.down.shape[2]
+        out = {"front": _padded(get("router"), c.experts, W),
                "gate_up": torch.stack([_interleave(get(f"e{i}.gate"), get(f"e{i}.up"), F, W)
                                        for i in range(c.experts)]),
                "down": torch.stack([_padded(get(f"e{i}.down"), W, F) for i in range(c.experts)])}
         if c.shared is not None:
             S = self.shared_down.shape[1]
-            out["shared_gate_up"] = _interleave(get("shared.gate"), get("shared.up"), S, W)
+            out["front"] = torch.cat([_interleave(get("shared.gate"), get("shared.up"), S, W), out["front"]])
             out["shared_down"] = _padded(get("shared.down"), W, S)
         return out
 
     def forward(self, h) -> lm.Experts:
         c = self.c
-        ids, wts = lm.route(lm.matmul(h, self.router, torch.float32), c.top, c.groups, c.keep)
-        plan = lm.plan_experts(ids, c.experts)
+        if c.shared is not None:
+            s, z = lm.glu_with_side(h, self.front, c.experts, c.shared.limit)
+        else:
+            z = lm.matmul(h, self.front, torch.float32)
+        wts, plan = lm.route_experts(z, c.top, c.groups, c.keep)
         a = lm.matmul(h, self.gate_up, epi=lm.EPI_CLAMP_GLU, param=c.expert.limit, plan=plan, gather=True)
         y = lm.matmul(a, self.down, plan=plan)
-        dense = None
-        if c.shared is not None:
-            s = lm.matmul(h, self.shared_gate_up, epi=lm.EPI_CLAMP_GLU, param=c.shared.limit)
-            dense = lm.matmul(s, self.shared_down)
+        dense = lm.matmul(s, self.shared_down) if c.shared is not None else None
         return lm.Experts(y, plan.slot_of, wts, dense)
 
     def init_random_(self, gen):

@@ -111,6 +111,18 @@ def matmul(a, w, out_dtype=None, epi: int = EPI_NONE, param: float = 0.0, plan: 
     return c
 
 
+def glu_with_side(a, w, side: int, param: float):
+    """One product for two consumers of ``a``: the rows of w but the last ``side`` are (gate, up) pairs of a clamped GLU
+    (:func:`matmul` EPI_CLAMP_GLU), the last ``side`` rows a plain product in fp32.  Returns (glu, side product)."""
+    if not a.is_cuda:
+        return ref.matmul(a, w[:-side], a.dtype, EPI_CLAMP_GLU, param), ref.matmul(a, w[-side:], torch.float32, 0, 0.0)
+    M, N = a.shape[0], w.shape[0]
+    c = torch.empty(M, (N - side) // 2, dtype=a.dtype, device=a.device)
+    s = torch.empty(M, side, dtype=torch.float32, device=a.device)
+    _K().lm_gemm(a, w, c, None, None, None, 0, EPI_CLAMP_GLU, float(param), s)
+    return c, s
+
+
 def grouped_bm(rows: int, experts: int) -> int:
     """Row tile of a grouped product over ``rows`` slots: 16-row streaming tiles while an expert sees few rows, LDS
     tiles of 128 rows once it sees enough of them to be compute-bound, of 256 when those fill up."""
@@ -142,6 +154,20 @@ def plan_experts(ids, experts: int) -> Plan:
     return plan
 
 
+def route_experts(logits, top: int, groups: int, keep: int):
+    """:func:`route` and :func:`plan_experts` -> (combine weights [T, top], plan); one launch for a few tokens."""
+    T, E = logits.shape
+    if not logits.is_cuda or T > 16 or E > 256 or grouped_bm(T * top, E) != 16:
+        ids, wts = route(logits, top, groups, keep)
+        return wts, plan_experts(ids, E)
+    P = T * top
+    i32 = lambda *s: torch.empty(*s, dtype=torch.int32, device=logits.device)
+    ids, wts = i32(T, top), torch.empty(T, top, dtype=torch.float32, device=logits.device)
+    plan = Plan(i32(E + 1), i32(P), i32(T, top), i32(min(P, E + P // 16), 2), 16)
+    _K().moe_route_plan(logits, int(groups), int(keep), ids, wts, plan.offsets, plan.token_of, plan.slot_of, plan.tiles)
+    return wts, plan
+
+
 def chunk_attention(qkvg, k_cache, v_cache, batch, heads: int, chunk: int, scale: float):
     """Attention of one step over a paged cache: softmax over the keys j <= i of position i's own chunk (positions
     chunk * n .. chunk * (n + 1) - 1), each head's output times sigmoid(its gate).
@@ -158,7 +184,7 @@ def chunk_attention(qkvg, k_cache, v_cache, batch, heads: int, chunk: int, scale
         _K().chunk_attn_prefill(qkvg, k_cache, v_cache, o, batch.block_table, batch.ctx_lens, batch.q_lens,
                                 batch.q_start, int(batch.S), int(heads), int(chunk), float(scale))
         return o
-    ns = max(1, min(int(batch.num_splits or 1), (chunk + 63) // 64))
+    ns = max(1, min(int(batch.num_splits or 1), (chunk + 63) // 64, 64))
     ws = torch.empty(T * heads * ns * (dv + 2) if ns > 1 else 0, dtype=torch.float32, device=qkvg.device)
     _K().chunk_attn_decode(qkvg, k_cache, v_cache, o, batch.block_table, batch.ctx_lens, batch.slots, ws, int(heads),
                            ns, int(chunk), float(scale))

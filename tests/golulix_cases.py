@@ -102,6 +102,12 @@ def check_matmul(device, dtype):
         assert torch.allclose(y.cpu().double(), 1.5 * torch.tanh(ref / 1.5), atol=2e-4)
         y = lm.matmul(a.to(device), w.to(device), epi=lm.EPI_CLAMP_GLU, param=0.8)
         eye = torch.eye(n // 2).double()
+        if n > 8:                                   # the same with a plain fp32 product of the last rows beside it
+            main = n // 8 * 4
+            y2, side = lm.glu_with_side(a.to(device), w.to(device), n - main, 0.8)
+            want = R.expert(a.double(), w[0:main:2].double(), w[1:main:2].double(), eye[:main // 2, :main // 2], 0.8)
+            assert torch.allclose(y2.cpu().double(), want, atol=2e-4 if dtype == torch.float32 else 0.02)
+            assert torch.allclose(side.cpu().double(), ref[:, main:], atol=2e-4)
         want = R.expert(a.double(), w[0::2].double(), w[1::2].double(), eye, 0.8)
         assert torch.allclose(y.cpu().double(), want, atol=2e-4 if dtype == torch.float32 else 0.02)
 
@@ -115,6 +121,14 @@ def check_route(device, dtype):
         for t in range(T):
             assert ids[t].tolist() == [e for e, _ in picks[t]]
             assert np.allclose(wts[t].cpu().numpy(), [s for _, s in picks[t]], rtol=1e-5)
+        wts2, plan = lm.route_experts(z.to(device), top, n, keep)
+        assert torch.equal(wts2, wts)
+        off, slots, tok = plan.offsets.tolist(), plan.slot_of.tolist(), plan.token_of.tolist()
+        assert sorted(s for row in slots for s in row) == list(range(T * top))
+        for t in range(T):
+            for k in range(top):
+                e = ids[t, k].item()
+                assert off[e] <= slots[t][k] < off[e + 1] and tok[slots[t][k]] == t
 
 
 def check_moe(device, dtype):
