@@ -487,7 +487,8 @@ __global__ void __launch_bounds__(256) attn_decode_fold_kernel(const AttnArgs p)
   if (d < 64) {                                  // one lane per split (at most 64)
     const float* q = ws + (long)min(d, p.splits - 1) * (p.dv + 2) + p.dv;
     const float m = d < p.splits ? q[0] : -INFINITY, l = q[1];
-    const float e = d < p.splits ? __builtin_amdgcn_exp2f(m - wave_max(m)) : 0.f;
+    const float M = wave_max(m);                 // whole wave: every lane takes part in the shuffles
+    const float e = d < p.splits ? __builtin_amdgcn_exp2f(m - M) : 0.f;
     se[d] = e;
     const float L = wave_sum(l * e);
     if (d == 0) total = L;

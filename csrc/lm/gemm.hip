@@ -47,12 +47,11 @@ struct Frag<float> {
   }
 };
 
-template <typename T, typename O, int MT, int NT, int NW>
+template <typename T, typename O, int MT, int NT, int NW, int D>
 __global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) {
-  // k-steps of W in flight per wave
-  constexpr int U = sizeof(T) == 2 ? (MT * NT == 1 ? 8 : NT == 1 ? 4 : NT == 2 ? 2 : 1) : 1;
   __shared__ float4_ red[NW][MT][64];
-  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int lane = threadIdx.x & 63;
+  const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int r = lane & 15, g = lane >> 4;
   const int n0 = blockIdx.x * 16 * NT;
   int row0 = blockIdx.y * 16 * MT, rows_end = p.M, expert = 0;
@@ -81,26 +80,29 @@ __global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) 
   for (int i = 0; i < NT; ++i)
 #pragma unroll
     for (int j = 0; j < MT; ++j) acc[i][j] = float4_{0.f, 0.f, 0.f, 0.f};
+  // this wave's k-steps are wid, wid + NW, ...; D of them are in flight
   const int steps = p.K / 64;
-  for (int s0 = wid; s0 < steps; s0 += NW * U) {
-    Frag<T> w[U][NT];
-#pragma unroll
-    for (int u = 0; u < U; ++u) {
-      const long k = (long)min(s0 + u * NW, steps - 1) * 64;
+  Frag<T> w[D][NT], x[D][MT];
+  auto fetch = [&](int u, int s) {
+    if (s < steps) {
+      const long k = (long)s * 64;
 #pragma unroll
       for (int i = 0; i < NT; ++i) w[u][i].load(wp[i] + k);
+#pragma unroll
+      for (int j = 0; j < MT; ++j) x[u][j].load(ap[j] + k);
     }
+  };
 #pragma unroll
-    for (int u = 0; u < U; ++u) {
+  for (int u = 0; u < D; ++u) fetch(u, wid + u * NW);
+  for (int s0 = wid; s0 < steps; s0 += NW * D) {
+#pragma unroll
+    for (int u = 0; u < D; ++u) {
       if (s0 + u * NW < steps) {
-        const long k = (long)(s0 + u * NW) * 64;
 #pragma unroll
-        for (int j = 0; j < MT; ++j) {
-          Frag<T> a;
-          a.load(ap[j] + k);
+        for (int j = 0; j < MT; ++j)
 #pragma unroll
-          for (int i = 0; i < NT; ++i) acc[i][j] = Frag<T>::mac(w[u][i], a, acc[i][j]);
-        }
+          for (int i = 0; i < NT; ++i) acc[i][j] = Frag<T>::mac(w[u][i], x[u][j], acc[i][j]);
+        fetch(u, s0 + (u + D) * NW);
       }
     }
   }
@@ -120,7 +122,7 @@ __global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) 
   }
 }
 
-// Workgroup shapes (16 MT rows of A x 16 NT rows of W, NW waves along K), from a sweep at decode sizes: enough
+// Workgroup shapes (16 MT rows of A x 16 NT rows of W, NW waves along K, D k-steps in flight), from a sweep at decode sizes: enough
 // workgroups to fill the chip come first, then fewer passes over W (MT), then fewer re-reads of A (NT).
 template <typename T, typename O>
 static void stream(const GemmArgs& a, hipStream_t s) {
@@ -129,24 +131,16 @@ static void stream(const GemmArgs& a, hipStream_t s) {
                     a.tiles ? (a.bm + 16 * mt - 1) / (16 * mt) : 1);
     kernel<<<grid, 64 * nw, 0, s>>>(a);
   };
-#define GO(MT_, NT_, NW_) go(gemm_stream_kernel<T, O, MT_, NT_, NW_>, MT_, NT_, NW_)
+  constexpr bool H = sizeof(T) == 2;              // fp32 fragments are twice the registers
+#define GO(MT_, NT_, NW_, D_) go(gemm_stream_kernel<T, O, MT_, NT_, NW_, H ? D_ : 1>, MT_, NT_, NW_)
   const int rows = a.tiles ? a.bm : a.M;
-  if (rows <= 16) {
-    if (a.tiles && a.K < 2048) GO(1, 4, 4);
-    else GO(1, 1, 4);
-  } else if (a.tiles) {
-    GO(4, 2, 4);
-  } else if (a.N < 512) {
-    GO(1, 1, 4);
-  } else if (a.N < 3072) {
-    GO(2, 1, 8);
-  } else if (a.N < 5120) {
-    GO(2, 2, 8);
-  } else if (a.N < 16384 || rows <= 32) {
-    GO(2, 4, 8);
-  } else {
-    GO(4, 4, 4);
-  }
+  if (rows <= 16 || a.N < 512) GO(1, 1, 8, 4);
+  else if (a.tiles) GO(4, 2, 4, 2);
+  else if (a.N < 3072 || (rows <= 32 && a.N < 5120)) GO(2, 1, 8, 4);
+  else if (a.N < 5120) GO(2, 2, 8, 2);
+  else if (rows <= 32) GO(2, 4, 4, 3);
+  else if (a.N < 8192) GO(4, 2, 4, 2);
+  else GO(4, 4, 4, 2);
 #undef GO
   SHAI_CHECK_LAUNCH();
 }

@@ -4,6 +4,23 @@
 
 namespace shai_lm {
 
+// max over the wave by lane shifts inside the register file (rows of 16, then the two row broadcasts)
+template <int CTRL>
+__device__ __forceinline__ float dpp_max(float v) {
+  const int neg_inf = 0xff800000;
+  const int o = __builtin_amdgcn_update_dpp(neg_inf, __float_as_int(v), CTRL, 0xf, 0xf, false);
+  return fmaxf(v, __int_as_float(o));
+}
+__device__ __forceinline__ float wave_max_dpp(float v) {
+  v = dpp_max<0x111>(v);   // row_shr 1, 2, 4, 8
+  v = dpp_max<0x112>(v);
+  v = dpp_max<0x114>(v);
+  v = dpp_max<0x118>(v);
+  v = dpp_max<0x142>(v);   // row_bcast 15, 31
+  v = dpp_max<0x143>(v);
+  return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), 63));
+}
+
 // One wave per token; lane l holds experts l, l + 64, ...  All comparisons break ties by the lower expert index, and
 // picks are by a strictly decreasing (score, index) order, so every pick is a distinct expert whatever the scores are.
 // `sc` is the wave's LDS scratch, [E + groups] floats.  Every wave of the workgroup calls it (barriers inside).
@@ -21,7 +38,7 @@ __device__ __forceinline__ void route_token(const RouteArgs& p, int t, float* sc
     if (!(z[i] == z[i])) z[i] = -INFINITY;      // a padding row may carry NaN: it still needs valid picks
     m = fmaxf(m, z[i]);
   }
-  m = wave_max(m);
+  m = wave_max_dpp(m);
   if (m == -INFINITY) m = 0.f;
   float sum = 0.f;
 #pragma unroll
@@ -59,18 +76,21 @@ __device__ __forceinline__ void route_token(const RouteArgs& p, int t, float* sc
     if (e >= p.E) z[i] = -2.f;
   }
   for (int k = 0; k < p.top; ++k) {
-    float bv = -3.f;
+    float best = -3.f;
     int bi = 0x7fffffff;
 #pragma unroll
     for (int i = 0; i < NE; ++i) {
       const int e = lane + 64 * i;
-      if (z[i] > bv) { bv = z[i]; bi = e; }     // ascending e: the first of equal scores stays
+      if (z[i] > best) { best = z[i]; bi = e; } // ascending e: the first of equal scores stays
     }
+    const float bv = wave_max_dpp(best);
+    const unsigned long long who = __ballot(best == bv);
+    if (__popcll(who) == 1) {
+      bi = __builtin_amdgcn_readlane(bi, __ffsll(who) - 1);
+    } else {                                      // equal scores in several lanes: the lowest expert
+      if (best != bv) bi = 0x7fffffff;
 #pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float ov = __shfl_xor(bv, o, 64);
-      const int oi = __shfl_xor(bi, o, 64);
-      if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+      for (int o = 32; o > 0; o >>= 1) bi = min(bi, __shfl_xor(bi, o, 64));
     }
 #pragma unroll
     for (int i = 0; i < NE; ++i)

@@ -53,6 +53,7 @@ __global__ void __launch_bounds__(256) add_norm_kernel(const AddNormArgs p) {
     v[i] = c < p.Dp ? load4(x + c) : float4_{0.f, 0.f, 0.f, 0.f};
   }
   if (p.ye) {
+#pragma unroll 4
     for (int k = 0; k < p.top; ++k) {
       const float wk = p.wts[row * p.top + k];
       const T* y = static_cast<const T*>(p.ye) + (long)p.slot_of[row * p.top + k] * p.Dp;

@@ -894,8 +894,8 @@ class LLMEngine:
 
 
 # ---------------------------------------------------------------------- helpers
-def smoke_llm(device="cuda:0"):
-    eng = LLMEngine(LlamaConfig.tiny(), device=device, max_num_seqs=4, max_model_len=256)
+def smoke_llm(device="cuda:0", cfg=None):
+    eng = LLMEngine(cfg or LlamaConfig.tiny(), device=device, max_num_seqs=4, max_model_len=256)
     out = eng.generate([[1, 5, 9, 200], list(range(3, 90))], SamplingParams(max_tokens=4, temperature=0.0,
                                                                             ignore_eos=True))
     assert all(len(s.output) == 4 for s in out)

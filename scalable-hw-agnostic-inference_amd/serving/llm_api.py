@@ -13,7 +13,7 @@ greedy).  Unlike vllm_model_api.py:38-43, ``max_new_tokens`` is honoured (the _m
 variant's behaviour).  Engine kwargs come from a /vllm_config.yaml-style file
 (``VLLM_CONFIG``): tensor_parallel_size, max_num_seqs, max_model_len, block_size
 (rounded to 64-token KV blocks), quantization (``fp8``: e4m3 weights + per-row
-scales, bf16 activations).
+scales, bf16 activations), dtype (bfloat16; float32 for models that run in it).
 
 Tensor parallelism (``tensor_parallel_size: N``, app/vllm_model_api.py:127-129 with
 cova/mllama-32-11b-vllm-trn1-config.yaml:9): the worker runs as N processes, one
@@ -61,11 +61,12 @@ def build_engine(env: ServerEnv, vc: Optional[dict] = None):
     vc = _vllm_config() if vc is None else vc
     cfg = llama_config_for(env.model_id, env.model_path, env.config)
     text = getattr(cfg, "text", cfg)   # MllamaConfig (vision) or LlamaConfig
-    eng = LLMEngine(cfg, device=env.torch_device, model_path=env.model_path,
+    import torch
+    dtype = {"float32": torch.float32, "float": torch.float32}.get(str(vc.get("dtype", "")), torch.bfloat16)
+    eng = LLMEngine(cfg, device=env.torch_device, model_path=env.model_path, dtype=dtype,
                     max_num_seqs=int(vc.get("max_num_seqs", 64)),
                     max_model_len=int(vc.get("max_model_len", min(8192, text.max_position_embeddings))),
                     enable_prefix_caching=True, quantization=vc.get("quantization"))
-    import torch
     with torch.inference_mode():
         # every decode batch bucket (sampled and all-greedy) captured before the first request
         eng.warmup_graphs(greedy_too=True)

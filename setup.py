@@ -35,6 +35,7 @@ SCRIPTS = {
     "shai-load-client": "shai_amd.bench.client:main",
     "shai-loadshape": "shai_amd.bench.loadshape:main",
     "shai-llm-offline": "shai_amd.bench.llm_offline:main",
+    "shai-trace-run": "shai_amd.engines.trace:main",
     "shai-long-context": "shai_amd.bench.long_context:main",
 }
 

@@ -212,6 +212,22 @@ def check_attention(device, dtype):
             assert (got - want).abs().max() < (2e-5 if dtype == torch.float32 else 0.03), (n, cuts)
 
 
+def check_low_scores(device, dtype):
+    """Every score far below zero (softmax does not care, a running maximum that starts at 0 would), in one to many
+    splits of a decode step, some of them empty."""
+    n, H, G, dk, dv, chunk = 450, 4, 2, 32, 32, 1000
+    g = torch.Generator().manual_seed(17)
+    r = lambda *s: torch.randn(*s, generator=g).bfloat16().float()
+    q, k, v, gate = r(n, H, dk), r(n, G, dk), r(n, G, dv), r(n, H)
+    q[..., 0], k[..., 0] = 8.0, -8.0
+    k[:, 0, 1] -= torch.arange(n) * 0.02                # the splits' maxima differ
+    k = k.bfloat16().float()
+    want = R.attend(*(t.double() for t in (q, k, v, gate)), chunk, 1.0)
+    for splits in (1, 2, 3, 5, 7, 16):
+        got = attention_step(q, k, v, gate, chunk, 1.0, (430, 1, 3, 1), device, dtype, splits).cpu().double()
+        assert (got - want).abs().max() < (1e-4 if dtype == torch.float32 else 0.04), splits
+
+
 def check_needle(device, dtype):
     """One key whose score stands out, at chunk edges, page borders and far away: a query of its chunk copies its value,
     any other query is unmoved."""
@@ -233,7 +249,8 @@ def check_needle(device, dtype):
             assert (got - want).abs().max() < (1e-4 if dtype == torch.float32 else 0.04), (chunk, at)
 
 
-MECHANISMS = [check_embed_norm, check_matmul, check_route, check_moe, check_add_norm, check_attention, check_needle]
+MECHANISMS = [check_embed_norm, check_matmul, check_route, check_moe, check_add_norm, check_attention, check_low_scores,
+              check_needle]
 
 # ---------------------------------------------------------------------------------------------- whole models
 SHAPES = {
