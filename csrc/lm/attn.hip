@@ -5,8 +5,9 @@
 //
 // kv_store      the step's k / v rows into the cache.
 // prefill       bf16: flash attention, 4 waves x 32 queries, scores swapped (S^T = K Q^T) so that a lane holds one
-//               query's scores, P feeds O^T = V^T P^T from registers as a bf16 pair (value + remainder); only the 64-key blocks of the chunks that the
-//               workgroup's queries lie in are visited.  fp32: attn_rows.
+//               query's scores; P feeds O^T = V^T P^T from registers as a bf16 pair (value + remainder, 16 significant
+//               bits).  Only the 64-key blocks of the chunks that the workgroup's queries lie in are visited.
+//               fp32: attn_rows.
 // decode        bf16: one workgroup per (sequence, kv head, split); each wave takes whole 64-key blocks, K straight from
 //               memory into the matrix cores (the group's query heads are the 16 columns), fp32 P against V on the
 //               VALU; the new token's k / v are written to the cache by the workgroup that reads them.

@@ -1,8 +1,9 @@
 // C = epi(A W^T), LDS-tiled bf16 form for many rows (prefill): 128 x 128 tiles of 4 waves or 256 x 256 tiles of 8, 64-wide
-// k-tiles moved global -> LDS by DMA (buffer_load ... lds, 16 bytes per lane) into two stages; the load of k-tile t + 1 is issued before the
-// MFMAs of t.  The bank swizzle is applied to the per-lane source chunk.  Buffer range checks zero-fill rows past the
-// ends.  Dense or grouped by expert: the row tiles of a grouped product come from the tile list, each with its own W and
-// with A rows gathered per lane.  Tiles are walked XCD by XCD in groups of 8 row tiles that share their W columns.
+// k-tiles moved global -> LDS by DMA (buffer_load ... lds, 16 bytes per lane) into two stages; the load of k-tile t + 1 is
+// issued before the MFMAs of t.  The bank swizzle is applied to the per-lane source chunk.  Buffer range checks zero-fill
+// rows past the ends.  Dense or grouped by expert: the row tiles of a grouped product come from the tile list, each with
+// its own W and with A rows gathered per lane.  Tiles are walked XCD by XCD in groups of 8 row tiles that share their W
+// columns.
 #include "lm_device.h"
 #include "lm.h"
 

@@ -5,9 +5,9 @@ several times with the same weights, and a logit softcap.
 The model runs on the engine's paged KV cache like the Llama family: :class:`shai_amd.engines.llm.LLMEngine` owns
 blocks, scheduling, prefix reuse and sampling.  Every layer RUN (a looped layer counts once per pass) has its own K/V
 pools, indexed by the same block table.  The residual stream is fp32; every add is fused with the norm that follows it
-(and, after an MoE layer, with the weighted sum of the expert outputs), so a layer is 10 launches in a decode step:
-norm, q/k/v/gate GEMM, attention (cache write and gate inside), output GEMM, norm, router GEMM, route + plan, expert
-GEMMs and the shared expert's.
+(and, after an MoE layer, with the weighted sum of the expert outputs).  A layer of a decode step is 10 launches: norm,
+q/k/v/gate GEMM, attention (cache write and gate inside; one more to fold its splits), output GEMM, norm, router + shared
+gate/up GEMM, routing and sort (two above 16 rows), expert gate/up, expert down, shared down.
 """
 from __future__ import annotations
 
