@@ -7,7 +7,8 @@
 // prefill       bf16: flash attention, 4 waves x 32 queries, scores swapped (S^T = K Q^T) so that a lane holds one
 //               query's scores; P feeds O^T = V^T P^T from registers as a bf16 pair (value + remainder, 16 significant
 //               bits).  Only the 64-key blocks of the chunks that the workgroup's queries lie in are visited.
-//               fp32: attn_rows.
+//               fp32: attn_rows.  The latent form (LAT) is the same kernel on keys and values expanded per head from
+//               cached latents: plain causal, no gate, a sink per head in the denominator.
 // decode        bf16: one workgroup per (sequence, kv head, split); each wave takes whole 64-key blocks, K straight from
 //               memory into the matrix cores (the group's query heads are the 16 columns), fp32 P against V on the
 //               VALU; the new token's k / v are written to the cache by the workgroup that reads them.
@@ -100,7 +101,7 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(const AttnArgs p) {
 // ------------------------------------------------------------------------------------------------ prefill (bf16)
 template <int D>
 __device__ __forceinline__ int k_swz(int row, int ch) {
-  if constexpr (D >= 128) return row * D + ((ch ^ (row & 15)) << 3);
+  if constexpr (D % 128 == 0) return row * D + ((ch ^ (row & 15)) << 3);
   else return row * D + ((ch ^ ((row >> 1) & 7)) << 3);
 }
 template <int D>
@@ -109,7 +110,7 @@ __device__ __forceinline__ int v_swz(int row, int ch) {
   else return row * D + ((ch ^ (((row >> 1) & 1) << 2)) << 3);
 }
 
-template <int DK, int DV>
+template <int DK, int DV, bool LAT>
 __global__ void __launch_bounds__(256, DK + DV > 256 ? 1 : 2) attn_prefill_kernel(const AttnArgs p) {
   constexpr int KT = 64, CK = DK / 8, CV = DV / 8, NK = KT * CK / 256, NV = KT * CV / 256;
   constexpr int NS = DK / 16, ND = DV / 32;
@@ -123,7 +124,7 @@ __global__ void __launch_bounds__(256, DK + DV > 256 ? 1 : 2) attn_prefill_kerne
   const int q_len = p.q_lens[b], q0 = blockIdx.x * 128;
   if (q0 >= q_len) return;
   const int ctx = p.ctx[b], c_off = ctx - q_len;
-  const int qi = q0 + wid * 32 + fr, pos = qi + c_off, lo = pos - pos % p.chunk;
+  const int qi = q0 + wid * 32 + fr, pos = qi + c_off, lo = LAT ? 0 : pos - pos % p.chunk;
   const long row0 = p.q_start[b];
   const bf16_t* rows = static_cast<const bf16_t*>(p.qkvg) + row0 * p.ld;
 
@@ -136,11 +137,32 @@ __global__ void __launch_bounds__(256, DK + DV > 256 ? 1 : 2) attn_prefill_kerne
   }
   // blocks from the first query's chunk to the last query's position
   const int p_first = q0 + c_off, p_last = min(q0 + 127, q_len - 1) + c_off;
-  const int t0 = (p_first - p_first % p.chunk) >> 6, t1 = (p_last >> 6) + 1;
-  const int lo_last = p_last - p_last % p.chunk;
+  const int t0 = LAT ? 0 : (p_first - p_first % p.chunk) >> 6, t1 = (p_last >> 6) + 1;
+  const int lo_last = LAT ? 0 : p_last - p_last % p.chunk;
 
   uint4_ rk[NK], rv[NV];
   auto load_tile = [&](int t) {
+    if constexpr (LAT) {
+      const int left = ctx - t * KT, ld = p.np + DV;
+      const long key = p.kv_start[b] + t * KT;
+      const bf16_t* kv = static_cast<const bf16_t*>(p.kv) + (key * p.H + h) * ld;
+      const bf16_t* lat = static_cast<const bf16_t*>(p.lat) + key * p.lat_ld + p.rank;
+#pragma unroll
+      for (int i = 0; i < NK; ++i) {
+        const int id = tid + 256 * i, r = id / CK, col = (id % CK) * 8;
+        rk[i] = uint4_{0u, 0u, 0u, 0u};
+        if (r < left && col < p.np + p.rot)
+          rk[i] = *reinterpret_cast<const uint4_*>(col < p.np ? kv + (long)r * p.H * ld + col
+                                                              : lat + (long)r * p.lat_ld + col - p.np);
+      }
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int id = tid + 256 * i, r = id / CV;
+        rv[i] = r < left ? *reinterpret_cast<const uint4_*>(kv + (long)r * p.H * ld + p.np + (id % CV) * 8)
+                         : uint4_{0u, 0u, 0u, 0u};
+      }
+      return;
+    }
     const long cell = ((long)p.bt[(long)b * p.max_blocks + t] * p.G + hk) * 64;
     const bf16_t* kb = static_cast<const bf16_t*>(p.kc) + cell * DK;
     const bf16_t* vb = static_cast<const bf16_t*>(p.vc) + cell * DV;
@@ -279,8 +301,13 @@ __global__ void __launch_bounds__(256, DK + DV > 256 ? 1 : 2) attn_prefill_kerne
   }
   const float l_tot = l_run + __shfl_xor(l_run, 32, 64);
   if (qi < q_len) {
-    const float gate = bf2f(rows[(long)qi * p.ld + (long)p.H * DK + (long)p.G * (DK + DV) + h]);
-    const float inv = sigmoid_f(gate) / l_tot;
+    float inv;
+    if constexpr (LAT) {
+      const float sk = p.sink[h] * kLog2e, top = fmaxf(m_run, sk), a = __builtin_amdgcn_exp2f(m_run - top);
+      inv = a / (l_tot * a + __builtin_amdgcn_exp2f(sk - top));
+    } else {
+      inv = sigmoid_f(bf2f(rows[(long)qi * p.ld + (long)p.H * DK + (long)p.G * (DK + DV) + h])) / l_tot;
+    }
     bf16_t* op = static_cast<bf16_t*>(p.o) + (row0 + qi) * (long)p.H * DV + (long)h * DV;
 #pragma unroll
     for (int d = 0; d < ND; ++d)
@@ -290,12 +317,21 @@ __global__ void __launch_bounds__(256, DK + DV > 256 ? 1 : 2) attn_prefill_kerne
   }
 }
 
-template <int DK, int DV>
+template <int DK, int DV, bool LAT = false>
 static void prefill(const AttnArgs& a, hipStream_t s) {
   constexpr int lds = 2 * 64 * (DK + DV) * 2;
-  (void)hipFuncSetAttribute(reinterpret_cast<const void*>(attn_prefill_kernel<DK, DV>),
+  (void)hipFuncSetAttribute(reinterpret_cast<const void*>(attn_prefill_kernel<DK, DV, LAT>),
                             hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-  attn_prefill_kernel<DK, DV><<<dim3((a.max_q + 127) / 128, a.H, a.B), 256, lds, s>>>(a);
+  attn_prefill_kernel<DK, DV, LAT><<<dim3((a.max_q + 127) / 128, a.H, a.B), 256, lds, s>>>(a);
+}
+
+void launch_latent_prefill(const AttnArgs& a, hipStream_t s) {
+  if (a.dk == 64 && a.dv == 64) prefill<64, 64, true>(a, s);
+  else if (a.dk == 128 && a.dv == 64) prefill<128, 64, true>(a, s);
+  else if (a.dk == 128 && a.dv == 128) prefill<128, 128, true>(a, s);
+  else if (a.dk == 192 && a.dv == 128) prefill<192, 128, true>(a, s);
+  else prefill<256, 256, true>(a, s);
+  SHAI_CHECK_LAUNCH();
 }
 
 #define SHAI_LM_HEADS(FN, ...)                                      \

@@ -133,9 +133,11 @@ void add_norm(const Tensor& x, const optional<Tensor>& dense, const optional<Ten
 
 void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<Tensor>& tiles,
              const optional<Tensor>& offsets, const optional<Tensor>& gather, int64_t bm, int64_t epi, double param,
-             const optional<Tensor>& side) {
+             const optional<Tensor>& side, const optional<Tensor>& vec, const optional<Tensor>& rope, int64_t head,
+             int64_t rot0) {
   const bool f32 = is_f32(A);
-  check(A, A.scalar_type(), "A");
+  SHAI_CHECK(A.is_cuda() && A.dim() == 2 && A.stride(1) == 1 && A.stride(0) % 8 == 0 && A.stride(0) >= A.size(1) &&
+                 reinterpret_cast<uintptr_t>(A.data_ptr()) % 16 == 0, "A rows must be contiguous and 16-byte aligned");
   check(W, A.scalar_type(), "W");
   check(C, f32 || C.scalar_type() == at::kFloat ? at::kFloat : at::kBFloat16, "C");
   shai_lm::GemmArgs g{};
@@ -148,18 +150,37 @@ void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<T
   g.param = param;
   g.out_f32 = C.scalar_type() == at::kFloat;
   SHAI_CHECK(A.size(1) == g.K && g.K % 64 == 0 && g.N >= 1, "lm_gemm: K must match and be a multiple of 64");
-  SHAI_CHECK(epi >= 0 && epi <= 2, "lm_gemm epilogue");
+  SHAI_CHECK(epi >= 0 && epi <= 4, "lm_gemm epilogue");
   g.n_main = g.N;
+  g.lda = A.stride(0);
+  g.batch = 1;
   if (side) {  // the last rows of W are a plain product, stored in fp32
     check(*side, at::kFloat, "side");
-    SHAI_CHECK(!tiles && epi == shai_lm::EPI_CLAMP_GLU && side->dim() == 2 && side->size(0) == g.M && side->size(1) >= 1 &&
-                   side->size(1) < g.N, "side output: dense GLU products, [M, last rows of W]");
+    SHAI_CHECK(!tiles && (epi == shai_lm::EPI_CLAMP_GLU || epi == shai_lm::EPI_NONE) && side->dim() == 2 &&
+                   side->size(0) == g.M && side->size(1) >= 1 && side->size(1) < g.N,
+               "side output: dense plain or GLU products, [M, last rows of W]");
     g.n_main = g.N - side->size(1);
-    SHAI_CHECK(g.n_main % 4 == 0, "side output: the GLU rows of W must be a multiple of 4");
+    SHAI_CHECK(g.n_main % 4 == 0, "side output: the other rows of W must be a multiple of 4");
     g.side = side->data_ptr<float>();
   }
   SHAI_CHECK(epi != shai_lm::EPI_CLAMP_GLU || g.n_main % 2 == 0, "GLU products need (gate, up) row pairs");
-  SHAI_CHECK(C.size(1) == (epi == shai_lm::EPI_CLAMP_GLU ? g.n_main / 2 : g.N), "lm_gemm output columns");
+  g.ldc = epi == shai_lm::EPI_CLAMP_GLU ? g.n_main / 2 : g.n_main;
+  SHAI_CHECK(C.size(1) == g.ldc, "lm_gemm output columns");
+  if (epi == shai_lm::EPI_XIELU) {
+    SHAI_CHECK(vec.has_value() && vec->numel() == 2, "the xIELU epilogue needs its two coefficients");
+    check_f32(*vec, "vec");
+    g.vec = vec->data_ptr<float>();
+  }
+  if (epi == shai_lm::EPI_ROTARY) {
+    SHAI_CHECK(rope.has_value() && rope->dim() == 2 && rope->size(0) == g.M && !tiles, "rotary epilogue: rope [M, dims]");
+    check_f32(*rope, "rope");
+    g.rope = rope->data_ptr<float>();
+    g.rot = rope->size(1);
+    g.head = head;
+    g.rot0 = rot0;
+    SHAI_CHECK(g.rot % 2 == 0 && rot0 % 4 == 0 && rot0 >= 0 && head % 4 == 0 && rot0 + g.rot <= head && g.N % head == 0,
+               "rotary epilogue: heads of ", head, " columns, the rotated ones from a multiple of 4");
+  }
   g.A = A.data_ptr();
   g.W = W.data_ptr();
   g.C = C.data_ptr();
@@ -184,10 +205,369 @@ void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<T
   }
   if (g.M == 0) return;
   const long lim = 0x7fffffffL;
-  const bool tile = !f32 && (g.tiles ? bm >= 128 : g.M > 64) && (long)g.a_rows * g.K * 2 < lim &&
+  const bool tile = !f32 && (g.tiles ? bm >= 128 : g.M > 64) && (long)g.a_rows * g.lda * 2 < lim &&
                     (long)g.N * g.K * 2 < lim;
   if (tile) shai_lm::launch_gemm_tile(g, stream());
   else shai_lm::launch_gemm(g, f32, stream());
+}
+
+// c[t, h] = a[t, h] w[h]^T for every head h: a [T, H, K], w [H, N, K], c [T, H, N], any strides between rows and heads
+void lm_gemm_heads(const Tensor& A, const Tensor& W, const Tensor& C) {
+  const bool f32 = is_f32(A);
+  SHAI_CHECK(A.dim() == 3 && W.dim() == 3 && C.dim() == 3 && W.scalar_type() == A.scalar_type() &&
+                 C.scalar_type() == A.scalar_type(), "lm_gemm_heads: three [.., .., ..] tensors of one type");
+  for (auto* t : {&A, &W, &C})
+    SHAI_CHECK(t->is_cuda() && t->stride(2) == 1 && t->stride(0) % 8 == 0 && t->stride(1) % 8 == 0 && t->stride(0) >= 0 &&
+                   t->stride(1) >= 0 && reinterpret_cast<uintptr_t>(t->data_ptr()) % 16 == 0,
+               "lm_gemm_heads: rows must be contiguous and 16-byte aligned");
+  shai_lm::GemmArgs g{};
+  g.M = g.a_rows = A.size(0);
+  g.batch = A.size(1);
+  g.K = A.size(2);
+  g.N = g.n_main = W.size(1);
+  SHAI_CHECK(W.size(0) == g.batch && W.size(2) == g.K && W.stride(1) == g.K && g.K % 64 == 0 && g.N % 4 == 0 &&
+                 C.size(0) == g.M && C.size(1) == g.batch && C.size(2) == g.N && g.batch <= 65535, "lm_gemm_heads shapes");
+  g.A = A.data_ptr();
+  g.W = W.data_ptr();
+  g.C = C.data_ptr();
+  g.lda = A.stride(0);
+  g.a_batch = A.stride(1);
+  g.w_batch = W.stride(0);
+  g.ldc = C.stride(0);
+  g.c_batch = C.stride(1);
+  g.out_f32 = f32;
+  if (g.M > 0) shai_lm::launch_gemm(g, f32, stream());
+}
+
+void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const optional<Tensor>& table, double scale,
+                   const optional<Tensor>& delta, const optional<Tensor>& wb, double mult, const optional<Tensor>& step,
+                   const optional<Tensor>& x_out, const optional<Tensor>& rows, const optional<Tensor>& w, double eps,
+                   int64_t width, const optional<Tensor>& h, const optional<Tensor>& cw, const optional<Tensor>& state,
+                   const optional<Tensor>& tail, const optional<Tensor>& row_seq, const optional<Tensor>& q_start,
+                   const optional<Tensor>& q_lens, const optional<Tensor>& pos, const optional<Tensor>& slots) {
+  shai_lm::ResidualNormArgs a{};
+  a.width = width;
+  a.eps = eps;
+  long R;
+  at::ScalarType dt = h ? h->scalar_type() : delta ? delta->scalar_type() : table ? table->scalar_type() : at::kFloat;
+  SHAI_CHECK(dt == at::kFloat || dt == at::kBFloat16, "bf16 or fp32");
+  SHAI_CHECK(x.has_value() != ids.has_value(), "residual_norm: a residual or token ids");
+  if (x) {
+    check(*x, at::kFloat, "x");
+    R = x->size(0);
+    a.Dp = x->size(1);
+    a.x = x->data_ptr<float>();
+  } else {
+    check_i32(*ids, "ids");
+    SHAI_CHECK(table.has_value(), "token ids need a table");
+    check(*table, dt, "table");
+    R = ids->numel();
+    a.V = table->size(0);
+    a.Dp = table->size(1);
+    a.ids = ids->data_ptr<int>();
+    a.table = table->data_ptr();
+    a.scale = scale;
+  }
+  a.T = R;
+  check_width(a.Dp, width);
+  auto row_vec = [&](const optional<Tensor>& t, const char* name) -> const float* {
+    if (!t) return nullptr;
+    check(*t, at::kFloat, name);
+    SHAI_CHECK(t->numel() == a.Dp, name, " must be [D]");
+    return t->data_ptr<float>();
+  };
+  if (delta) {
+    check(*delta, dt, "delta");
+    SHAI_CHECK(delta->dim() == 2 && delta->size(0) == R && delta->size(1) == a.Dp && wb.has_value(),
+               "delta must be [rows, D], with its norm's gain");
+    a.delta = delta->data_ptr();
+  }
+  a.wb = row_vec(wb, "wb");
+  a.mult = mult;
+  a.step = row_vec(step, "step");
+  a.w = row_vec(w, "w");
+  if (x_out) {
+    check(*x_out, at::kFloat, "x_out");
+    SHAI_CHECK(x_out->size(0) == R && x_out->size(1) == a.Dp, "x_out must be [rows, D]");
+    a.x_out = x_out->data_ptr<float>();
+  }
+  if (rows) {
+    check_i32(*rows, "rows");
+    SHAI_CHECK(!cw && w.has_value(), "rows selects rows to normalise");
+    a.rows = rows->data_ptr<int>();
+    a.T = rows->numel();
+  }
+  if (w) {
+    SHAI_CHECK(h.has_value(), "a norm needs an output h");
+    check(*h, dt, "h");
+    SHAI_CHECK(h->numel() == (long)a.T * a.Dp, "h must be [rows, D]");
+    a.h = h->data_ptr();
+  }
+  if (cw) {
+    check(*cw, at::kFloat, "cw");
+    SHAI_CHECK(cw->dim() == 2 && cw->size(1) == a.Dp && cw->size(0) >= 1 && cw->size(0) <= 16, "convolution: 1 to 16 taps");
+    a.taps = cw->size(0);
+    SHAI_CHECK(w.has_value() && x_out.has_value() && (!x || x->data_ptr() != x_out->data_ptr()),
+               "convolution: needs the norm, and x_out apart from x");
+    SHAI_CHECK(state.has_value() && pos.has_value() && slots.has_value() && pos->numel() >= R, "convolution: state, pos, slots");
+    check(*state, at::kFloat, "state");
+    check_i32(*pos, "pos");
+    check_i32(*slots, "slots");
+    SHAI_CHECK(state->dim() == 3 && state->size(1) == a.taps - 1 && state->size(2) == a.Dp, "state must be [slots, taps - 1, D]");
+    a.cw = cw->data_ptr<float>();
+    a.state = state->data_ptr<float>();
+    a.pos = pos->data_ptr<int>();
+    a.slots = slots->data_ptr<int>();
+    a.B = R;
+    a.run = 1;
+    if (tail) {
+      SHAI_CHECK(row_seq.has_value() && q_start.has_value() && q_lens.has_value(), "prefill convolution: row_seq, q_start, q_lens");
+      check(*tail, at::kFloat, "tail");
+      check_i32(*row_seq, "row_seq");
+      check_i32(*q_start, "q_start");
+      check_i32(*q_lens, "q_lens");
+      a.B = q_lens->numel();
+      SHAI_CHECK(tail->dim() == 3 && tail->size(0) == a.B && tail->size(1) == a.taps - 1 && tail->size(2) == a.Dp &&
+                     row_seq->numel() == R && q_start->numel() == a.B, "tail must be [B, taps - 1, D]");
+      a.tail = tail->data_ptr<float>();
+      a.row_seq = row_seq->data_ptr<int>();
+      a.q_start = q_start->data_ptr<int>();
+      a.q_lens = q_lens->data_ptr<int>();
+      a.run = R >= 16384 ? 16 : R >= 4096 ? 8 : 4;
+    }
+    SHAI_CHECK(slots->numel() >= a.B, "one state slot per sequence");
+  }
+  if (a.T > 0) shai_lm::launch_residual_norm(a, dt == at::kFloat, stream());
+}
+
+void conv_commit(const Tensor& state, const Tensor& tail, const Tensor& q_lens, const Tensor& slots) {
+  check(state, at::kFloat, "state");
+  check(tail, at::kFloat, "tail");
+  check_i32(q_lens, "q_lens");
+  check_i32(slots, "slots");
+  SHAI_CHECK(state.dim() == 4 && tail.dim() == 4 && state.size(0) == tail.size(0) && state.size(2) == tail.size(2) &&
+                 state.size(3) == tail.size(3) && state.size(3) % 4 == 0, "state [runs, slots, taps - 1, D], tail [runs, B, taps - 1, D]");
+  shai_lm::ConvCommitArgs a{};
+  a.runs = state.size(0);
+  a.n_slots = state.size(1);
+  a.B = tail.size(1);
+  a.taps = state.size(2) + 1;
+  a.Dp = state.size(3);
+  SHAI_CHECK(q_lens.numel() == a.B && slots.numel() == a.B && a.B <= 65535 && a.runs <= 65535, "one length and slot per sequence");
+  a.state = state.data_ptr<float>();
+  a.tail = tail.data_ptr<float>();
+  a.q_lens = q_lens.data_ptr<int>();
+  a.slots = slots.data_ptr<int>();
+  if (tail.numel() > 0) shai_lm::launch_conv_commit(a, stream());
+}
+
+void rope_rows(const Tensor& pos, const Tensor& freq, const Tensor& out) {
+  check_i32(pos, "pos");
+  check_f32(freq, "freq");
+  check_f32(out, "out");
+  SHAI_CHECK(freq.dim() == 2 && freq.size(1) == 2 && out.dim() == 2 && out.size(0) <= pos.numel() &&
+                 out.size(1) == 2 * freq.size(0), "rope_rows: freq [n, 2], out [T, 2 n]");
+  shai_lm::RopeRowsArgs a{pos.data_ptr<int>(), freq.data_ptr<float>(), (int)out.size(0), (int)freq.size(0),
+                          out.data_ptr<float>()};
+  if (out.numel() > 0) shai_lm::launch_rope_rows(a, stream());
+}
+
+void latent_prep(const Tensor& d, const Tensor& wq, const Tensor& wkv, const Tensor& rope, const Tensor& slots,
+                 const Tensor& cache, const Tensor& cq, double eps, int64_t q_rank, int64_t kv_rank) {
+  const auto dt = cq.scalar_type();
+  const bool f32 = is_f32(cq);
+  check(d, at::kFloat, "d");
+  check(wq, at::kFloat, "wq");
+  check(wkv, at::kFloat, "wkv");
+  check(rope, at::kFloat, "rope");
+  check_i32(slots, "slots");
+  check(cache, dt, "cache");
+  check(cq, dt, "cq");
+  shai_lm::LatentPrepArgs a{};
+  SHAI_CHECK(d.dim() == 2 && cq.dim() == 2 && cache.dim() == 3 && cache.size(1) == 64 && rope.dim() == 2, "latent_prep ranks");
+  a.T = d.size(0);
+  a.qp = cq.size(1);
+  a.rp = wkv.numel();
+  a.op = cache.size(2) - a.rp;
+  a.rot = rope.size(1);
+  a.q_rank = q_rank;
+  a.kv_rank = kv_rank;
+  a.eps = eps;
+  SHAI_CHECK(a.qp % 64 == 0 && a.rp % 64 == 0 && a.op % 2 == 0 && a.op >= a.rot && a.rot % 2 == 0 && wq.numel() == a.qp &&
+                 d.size(1) == a.qp + a.rp + a.op && cq.size(0) == a.T && rope.size(0) == a.T && slots.numel() >= a.T &&
+                 q_rank >= 1 && q_rank <= a.qp && kv_rank >= 1 && kv_rank <= a.rp, "latent_prep shapes");
+  a.d = d.data_ptr<float>();
+  a.wq = wq.data_ptr<float>();
+  a.wkv = wkv.data_ptr<float>();
+  a.rope = rope.data_ptr<float>();
+  a.slots = slots.data_ptr<int>();
+  a.cache = cache.data_ptr();
+  a.cq = cq.data_ptr();
+  if (a.T > 0) shai_lm::launch_latent_prep(a, f32, stream());
+}
+
+// start: first output row of every listed sequence; the caller sized `out` for all of them
+void latent_gather(const Tensor& cache, const Tensor& bt, const Tensor& seqs, const Tensor& ctx, const Tensor& start,
+                   int64_t max_ctx, const Tensor& out) {
+  check(cache, out.scalar_type(), "cache");
+  check(out, out.scalar_type(), "out");
+  for (auto* t : {&bt, &seqs, &ctx, &start}) check_i32(*t, "latent_gather tensor");
+  shai_lm::LatentGatherArgs a{};
+  a.n = seqs.numel();
+  a.max_ctx = max_ctx;
+  a.max_blocks = bt.size(1);
+  a.ld_bytes = cache.size(2) * cache.element_size();
+  SHAI_CHECK(cache.dim() == 3 && cache.size(1) == 64 && out.dim() == 2 && out.size(1) == cache.size(2) && a.ld_bytes % 16 == 0 &&
+                 ctx.numel() == a.n && start.numel() == a.n && a.n <= 65535 && max_ctx <= (int64_t)a.max_blocks * 64,
+             "latent_gather shapes");
+  a.cache = cache.data_ptr();
+  a.out = out.data_ptr();
+  a.bt = bt.data_ptr<int>();
+  a.seqs = seqs.data_ptr<int>();
+  a.ctx = ctx.data_ptr<int>();
+  a.start = start.data_ptr<int>();
+  if (a.n > 0 && max_ctx > 0) shai_lm::launch_latent_gather(a, stream());
+}
+
+void latent_attn_prefill(const Tensor& q, const Tensor& kv, const Tensor& lat, const Tensor& o, const Tensor& ctx,
+                         const Tensor& q_lens, const Tensor& q_start, const Tensor& kv_start, const Tensor& sink,
+                         int64_t max_q, int64_t heads, int64_t np, int64_t rot, int64_t rank, double scale) {
+  for (auto* t : {&q, &kv, &lat, &o}) check(*t, at::kBFloat16, "latent prefill tensor");
+  for (auto* t : {&ctx, &q_lens, &q_start, &kv_start}) check_i32(*t, "batch tensor");
+  check_f32(sink, "sink");
+  shai_lm::AttnArgs a{};
+  a.B = ctx.numel();
+  a.H = a.G = heads;
+  SHAI_CHECK(heads >= 1 && q.dim() == 2 && o.dim() == 2 && kv.dim() == 2 && lat.dim() == 2 && q.size(1) % heads == 0 &&
+                 o.size(1) % heads == 0 && q.size(0) == o.size(0), "latent prefill: q [T, H dk], o [T, H dv]");
+  a.T = q.size(0);
+  a.ld = q.size(1);
+  a.dk = q.size(1) / heads;
+  a.dv = o.size(1) / heads;
+  SHAI_CHECK((a.dk == 64 && a.dv == 64) || (a.dk == 128 && (a.dv == 64 || a.dv == 128)) || (a.dk == 192 && a.dv == 128) ||
+                 (a.dk == 256 && a.dv == 256), "latent prefill head sizes: 64/64, 128/64, 128/128, 192/128 or 256/256");
+  a.np = np;
+  a.rot = (rot + 7) / 8 * 8;
+  a.rank = rank;
+  a.lat_ld = lat.size(1);
+  SHAI_CHECK(np >= 0 && np % 8 == 0 && np + a.rot <= a.dk && rank % 8 == 0 && rank + a.rot <= a.lat_ld && a.lat_ld % 8 == 0 &&
+                 kv.size(1) == heads * (np + a.dv) && kv.size(0) == lat.size(0), "latent prefill: kv [rows, H (np + dv)]");
+  SHAI_CHECK(q_lens.numel() == a.B && q_start.numel() == a.B && kv_start.numel() == a.B && sink.numel() == heads && max_q >= 1 &&
+                 a.B <= 65535 && a.H <= 65535, "per-sequence [B] tensors");
+  a.qkvg = q.data_ptr();
+  a.kv = kv.data_ptr();
+  a.lat = lat.data_ptr();
+  a.o = o.data_ptr();
+  a.ctx = ctx.data_ptr<int>();
+  a.q_lens = q_lens.data_ptr<int>();
+  a.q_start = q_start.data_ptr<int>();
+  a.kv_start = kv_start.data_ptr<int>();
+  a.sink = sink.data_ptr<float>();
+  a.max_q = max_q;
+  a.chunk = 1;
+  a.scale = scale;
+  if (a.T > 0 && a.B > 0) shai_lm::launch_latent_prefill(a, stream());
+}
+
+void latent_attn_rows(const Tensor& ql, const Tensor& q, const Tensor& cache, const Tensor& o, const Tensor& bt,
+                      const optional<Tensor>& seqs, const Tensor& ctx, const Tensor& sink, const Tensor& ws, int64_t splits,
+                      int64_t np, int64_t rot, double scale) {
+  const auto dt = q.scalar_type();
+  const bool f32 = is_f32(q);
+  check(ql, dt, "ql");
+  check(q, dt, "q");
+  check(cache, dt, "cache");
+  check(o, dt, "o");
+  check_i32(bt, "block table");
+  check_i32(ctx, "ctx");
+  check_f32(sink, "sink");
+  shai_lm::LatentArgs a{};
+  SHAI_CHECK(ql.dim() == 3 && q.dim() == 2 && cache.dim() == 3 && cache.size(1) == 64 && bt.dim() == 2, "latent_attn_rows ranks");
+  a.n = ql.size(0);
+  a.H = ql.size(1);
+  a.rp = ql.size(2);
+  a.op = cache.size(2) - a.rp;
+  a.ldq = q.size(1);
+  a.head = q.size(1) / a.H;
+  a.np = np;
+  a.rot = rot;
+  a.max_blocks = bt.size(1);
+  a.splits = splits;
+  a.scale = scale;
+  SHAI_CHECK(q.size(0) == a.n && q.size(1) % a.H == 0 && a.rp % 64 == 0 && a.rp <= 1024 && a.op >= (rot + 7) / 8 * 8 &&
+                 a.op % 4 == 0 && np % 8 == 0 && np + (rot + 7) / 8 * 8 <= a.head && o.sizes() == ql.sizes() &&
+                 ctx.numel() >= a.n && sink.numel() == a.H && a.n <= 65535, "latent_attn_rows shapes");
+  if (seqs) {
+    check_i32(*seqs, "seqs");
+    SHAI_CHECK(seqs->numel() == a.n, "seqs: one per row");
+    a.seqs = seqs->data_ptr<int>();
+  } else {
+    SHAI_CHECK(bt.size(0) >= a.n, "one block table row per entry");
+  }
+  a.ql = ql.data_ptr();
+  a.q = q.data_ptr();
+  a.cache = cache.data_ptr();
+  a.o = o.data_ptr();
+  a.bt = bt.data_ptr<int>();
+  a.ctx = ctx.data_ptr<int>();
+  a.sink = sink.data_ptr<float>();
+  if (a.n == 0) return;
+  if (f32 || !shai_lm::latent_decode_fits(a.rp, a.op)) {
+    SHAI_CHECK((a.rp + a.op + 64) * 16 <= 65536, "latent rows of up to 4032 values");
+    shai_lm::launch_latent_rows(a, f32, stream());
+    return;
+  }
+  SHAI_CHECK(splits >= 1 && splits <= 64 &&
+                 (splits == 1 || (ws.scalar_type() == at::kFloat && ws.is_contiguous() &&
+                                  ws.numel() >= (long)a.n * a.H * splits * (a.rp + 4))), "split workspace");
+  a.ws = splits > 1 ? ws.data_ptr<float>() : nullptr;
+  shai_lm::launch_latent_decode(a, stream());
+}
+
+void mingru_scan(const Tensor& zx, const Tensor& g, const Tensor& bias, const Tensor& state, const Tensor& out,
+                 const Tensor& pos, const optional<Tensor>& q_start, const optional<Tensor>& q_lens, const Tensor& slots,
+                 const Tensor& ws, int64_t max_q, int64_t len) {
+  const bool f32 = is_f32(g);
+  check(zx, at::kFloat, "zx");
+  check(g, g.scalar_type(), "g");
+  check(bias, at::kFloat, "bias");
+  check(state, at::kFloat, "state");
+  check(out, g.scalar_type(), "out");
+  check_i32(pos, "pos");
+  check_i32(slots, "slots");
+  shai_lm::ScanArgs a{};
+  SHAI_CHECK(g.dim() == 2 && zx.dim() == 2 && state.dim() == 2 && len >= 1 && max_q >= 1, "mingru_scan ranks");
+  a.T = g.size(0);
+  a.W = g.size(1);
+  SHAI_CHECK(zx.size(0) == a.T && zx.size(1) == 2 * a.W && bias.numel() == 2 * a.W && state.size(1) == a.W &&
+                 out.sizes() == g.sizes() && pos.numel() >= a.T, "mingru_scan shapes");
+  a.B = a.T;
+  a.len = len;
+  a.max_q = max_q;
+  a.chunks = (max_q + len - 1) / len;
+  if (q_lens) {
+    SHAI_CHECK(q_start.has_value(), "prefill scan: q_start");
+    check_i32(*q_lens, "q_lens");
+    check_i32(*q_start, "q_start");
+    a.B = q_lens->numel();
+    SHAI_CHECK(q_start->numel() == a.B, "one start per sequence");
+    a.q_lens = q_lens->data_ptr<int>();
+    a.q_start = q_start->data_ptr<int>();
+  } else {
+    SHAI_CHECK(a.chunks == 1, "decode scan: one row per sequence");
+  }
+  SHAI_CHECK(slots.numel() >= a.B && a.B <= 65535 && a.chunks <= 65535, "one state slot per sequence");
+  SHAI_CHECK(a.chunks == 1 || (ws.scalar_type() == at::kFloat && ws.is_contiguous() &&
+                               ws.numel() >= (long)a.B * a.chunks * 2 * a.W), "scan workspace");
+  a.zx = zx.data_ptr<float>();
+  a.g = g.data_ptr();
+  a.bias = bias.data_ptr<float>();
+  a.state = state.data_ptr<float>();
+  a.out = out.data_ptr();
+  a.pos = pos.data_ptr<int>();
+  a.slots = slots.data_ptr<int>();
+  a.ws = a.chunks > 1 ? ws.data_ptr<float>() : nullptr;
+  if (a.T > 0) shai_lm::launch_mingru_scan(a, f32, stream());
 }
 
 void moe_route(const Tensor& logits, int64_t groups, int64_t keep, const Tensor& ids, const Tensor& wts) {
@@ -379,7 +759,16 @@ void token_feedback(const Tensor& ids, const Tensor& rowmap, const Tensor& prev)
 TORCH_LIBRARY_FRAGMENT(shai, m) {
   m.def("embed_norm(Tensor ids, Tensor? prev, Tensor table, Tensor? bigram, int mul_prev, int mul_cur, Tensor w, float eps, int width, Tensor(a!) x, Tensor(b!) h) -> ()");
   m.def("add_norm(Tensor(a!) x, Tensor? dense, Tensor? ye, Tensor? slot_of, Tensor? wts, Tensor? inject, Tensor? rows, Tensor? w, float eps, int width, Tensor(b!)? h) -> ()");
-  m.def("lm_gemm(Tensor a, Tensor w, Tensor(a!) c, Tensor? tiles, Tensor? offsets, Tensor? gather, int bm, int epi, float param, Tensor(b!)? side=None) -> ()");
+  m.def("lm_gemm(Tensor a, Tensor w, Tensor(a!) c, Tensor? tiles, Tensor? offsets, Tensor? gather, int bm, int epi, float param, Tensor(b!)? side=None, Tensor? vec=None, Tensor? rope=None, int head=0, int rot0=0) -> ()");
+  m.def("lm_gemm_heads(Tensor a, Tensor w, Tensor(a!) c) -> ()");
+  m.def("residual_norm(Tensor? x, Tensor? ids, Tensor? table, float scale, Tensor? delta, Tensor? wb, float mult, Tensor? step, Tensor(a!)? x_out, Tensor? rows, Tensor? w, float eps, int width, Tensor(b!)? h, Tensor? cw=None, Tensor(c!)? state=None, Tensor(d!)? tail=None, Tensor? row_seq=None, Tensor? q_start=None, Tensor? q_lens=None, Tensor? pos=None, Tensor? slots=None) -> ()");
+  m.def("conv_commit(Tensor(a!) state, Tensor tail, Tensor q_lens, Tensor slots) -> ()");
+  m.def("rope_rows(Tensor pos, Tensor freq, Tensor(a!) out) -> ()");
+  m.def("latent_prep(Tensor d, Tensor wq, Tensor wkv, Tensor rope, Tensor slots, Tensor(a!) cache, Tensor(b!) cq, float eps, int q_rank, int kv_rank) -> ()");
+  m.def("latent_gather(Tensor cache, Tensor block_table, Tensor seqs, Tensor ctx, Tensor start, int max_ctx, Tensor(a!) out) -> ()");
+  m.def("latent_attn_prefill(Tensor q, Tensor kv, Tensor lat, Tensor(a!) o, Tensor ctx, Tensor q_lens, Tensor q_start, Tensor kv_start, Tensor sink, int max_q, int heads, int np, int rot, int rank, float scale) -> ()");
+  m.def("latent_attn_rows(Tensor ql, Tensor q, Tensor cache, Tensor(a!) o, Tensor block_table, Tensor? seqs, Tensor ctx, Tensor sink, Tensor(b!) ws, int splits, int np, int rot, float scale) -> ()");
+  m.def("mingru_scan(Tensor zx, Tensor g, Tensor bias, Tensor(a!) state, Tensor(b!) out, Tensor pos, Tensor? q_start, Tensor? q_lens, Tensor slots, Tensor(c!) ws, int max_q, int len) -> ()");
   m.def("moe_route(Tensor logits, int groups, int keep, Tensor(a!) ids, Tensor(b!) wts) -> ()");
   m.def("moe_route_plan(Tensor logits, int groups, int keep, Tensor(a!) ids, Tensor(b!) wts, Tensor(c!) offsets, Tensor(d!) token_of, Tensor(e!) slot_of, Tensor(f!) tiles) -> ()");
   m.def("moe_plan(Tensor ids, int bm, Tensor(a!) offsets, Tensor(b!) token_of, Tensor(c!) slot_of, Tensor(d!) tiles) -> ()");
@@ -394,6 +783,15 @@ TORCH_LIBRARY_IMPL(shai, CUDA, m) {
   m.impl("embed_norm", &embed_norm);
   m.impl("add_norm", &add_norm);
   m.impl("lm_gemm", &lm_gemm);
+  m.impl("lm_gemm_heads", &lm_gemm_heads);
+  m.impl("residual_norm", &residual_norm);
+  m.impl("conv_commit", &conv_commit);
+  m.impl("rope_rows", &rope_rows);
+  m.impl("latent_prep", &latent_prep);
+  m.impl("latent_gather", &latent_gather);
+  m.impl("latent_attn_prefill", &latent_attn_prefill);
+  m.impl("latent_attn_rows", &latent_attn_rows);
+  m.impl("mingru_scan", &mingru_scan);
   m.impl("moe_route", &moe_route);
   m.impl("moe_route_plan", &moe_route_plan);
   m.impl("moe_plan", &moe_plan);

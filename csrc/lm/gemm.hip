@@ -7,7 +7,7 @@
 // pair of W is folded in registers.  A k-step covers 64 values; lane group g = lane / 16 takes values 16 g .. 16 g + 15
 // of it in both operands (the order of k inside a dot product is free), i.e. every W row is read 128 bytes at a time.
 //
-// Dense: row tiles of A are blockIdx.y.  Grouped (experts): blockIdx.y is an entry of the tile list and blockIdx.z a
+// Dense: row tiles of A are blockIdx.y, products of a batch (one per attention head, say) blockIdx.z.  Grouped (experts): blockIdx.y is an entry of the tile list and blockIdx.z a
 // 16 MT-row part of it; rows past the expert's last slot are computed on a clamped row and not stored.
 #include "lm_device.h"
 #include "lm.h"
@@ -65,6 +65,12 @@ __global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) 
   if (row0 >= rows_end) return;
   const T* W = static_cast<const T*>(p.W) + (long)expert * p.N * p.K;
   const T* A = static_cast<const T*>(p.A);
+  O* C = static_cast<O*>(p.C);
+  if (p.batch > 1) {
+    W += blockIdx.z * p.w_batch;
+    A += blockIdx.z * p.a_batch;
+    C += blockIdx.z * p.c_batch;
+  }
   const T* wp[NT];
   const T* ap[MT];
 #pragma unroll
@@ -73,7 +79,7 @@ __global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) 
   for (int j = 0; j < MT; ++j) {
     int m = min(row0 + 16 * j + r, rows_end - 1);
     if (p.gather) m = p.gather[m];
-    ap[j] = A + (long)m * p.K + g * 16;
+    ap[j] = A + m * p.lda + g * 16;
   }
   float4_ acc[NT][MT];
 #pragma unroll
@@ -117,7 +123,7 @@ __global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) 
 #pragma unroll
       for (int w = 1; w < NW; ++w) c += red[w][t][lane];
       const int m = row0 + 16 * t + r;
-      if (m < rows_end) store_cols<O>(p, m, n0 + 16 * i + 4 * g, c);
+      if (m < rows_end) store_cols<O>(p, C, m, n0 + 16 * i + 4 * g, c);
     }
   }
 }
@@ -128,7 +134,7 @@ template <typename T, typename O>
 static void stream(const GemmArgs& a, hipStream_t s) {
   auto go = [&](auto kernel, int mt, int nt, int nw) {
     const dim3 grid((a.N + 16 * nt - 1) / (16 * nt), a.tiles ? a.n_tiles : (a.M + 16 * mt - 1) / (16 * mt),
-                    a.tiles ? (a.bm + 16 * mt - 1) / (16 * mt) : 1);
+                    a.tiles ? (a.bm + 16 * mt - 1) / (16 * mt) : a.batch);
     kernel<<<grid, 64 * nw, 0, s>>>(a);
   };
   constexpr bool H = sizeof(T) == 2;              // fp32 fragments are twice the registers

@@ -51,7 +51,7 @@ __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_
     m_end = min(p.offsets[expert + 1], m0 + BM);
   }
   const bf16_t* Wt = static_cast<const bf16_t*>(p.W) + (long)expert * p.N * p.K;
-  const __amdgpu_buffer_rsrc_t rW = rsrc(Wt, (long)p.N * p.K * 2), rA = rsrc(p.A, (long)p.a_rows * p.K * 2);
+  const __amdgpu_buffer_rsrc_t rW = rsrc(Wt, (long)p.N * p.K * 2), rA = rsrc(p.A, ((long)(p.a_rows - 1) * p.lda + p.K) * 2);
 
   // byte offset of this lane's 16-byte chunk of every staged row at k = 0 (kOob: the row does not exist)
   const int lrow = lane >> 3, lpos = lane & 7;
@@ -60,7 +60,7 @@ __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_
   for (int j = 0; j < JA; ++j) {
     const int r = (wid * JA + j) * 8 + lrow, m = m0 + r;
     const long src = m < m_end ? (p.gather ? p.gather[m] : m) : -1;
-    offA[j] = src < 0 ? kOob : (uint32_t)((src * p.K + (lpos ^ ((r >> 1) & 7)) * 8) * 2);
+    offA[j] = src < 0 ? kOob : (uint32_t)((src * p.lda + (lpos ^ ((r >> 1) & 7)) * 8) * 2);
   }
 #pragma unroll
   for (int j = 0; j < JB; ++j) {
@@ -123,7 +123,7 @@ __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_
     for (int j = 0; j < JN; ++j)
 #pragma unroll
       for (int g = 0; g < 4; ++g)
-        store_cols<O>(p, m, n0 + wn * TN + j * 32 + 8 * g + 4 * fh,
+        store_cols<O>(p, static_cast<O*>(p.C), m, n0 + wn * TN + j * 32 + 8 * g + 4 * fh,
                       float4_{acc[i][j][4 * g], acc[i][j][4 * g + 1], acc[i][j][4 * g + 2], acc[i][j][4 * g + 3]});
   }
 }

@@ -1,5 +1,5 @@
 // Launchers of the decoder-block kernels (libshai_lm.so): decoders with an fp32 residual stream, mixture-of-experts
-// layers and chunked attention.  Every kernel takes bf16 or fp32 weights / activations (`f32`); norms, routing, scores
+// layers, chunked and latent attention, and gated recurrences.  Every kernel takes bf16 or fp32 weights / activations (`f32`); norms, routing, scores
 // and the residual are fp32 in both.  The model width is padded to a multiple of 64 by the caller.
 #pragma once
 #include <hip/hip_runtime.h>
@@ -37,7 +37,57 @@ struct AddNormArgs {
 };
 void launch_add_norm(const AddNormArgs& a, bool f32, hipStream_t s);
 
-enum Epi : int { EPI_NONE = 0, EPI_CLAMP_GLU = 1, EPI_SOFTCAP = 2 };
+// Residual add with a norm of its own, the next sublayer's norm, and its input convolution:
+//   x' = x + mult * RMSNorm(delta) wb (+ step),   h = RMSNorm(x') w,   h += causal convolution of h over time
+// Every part but the source of x may be absent.
+struct ResidualNormArgs {
+  const float* x;          // [*, Dp], or null: x = table[ids] * scale
+  const int* ids;
+  const void* table;       // [V, Dp]
+  float scale;
+  int V;
+  const void* delta;       // [*, Dp] sublayer output, or null
+  const float* wb;         // its norm's gain
+  float mult;
+  const float* step;       // [Dp] added to every row, or null
+  float* x_out;            // [*, Dp], or null
+  const int* rows;         // optional: only these rows (no convolution)
+  const float* w;          // gain, or null: no norm output
+  float eps;
+  int T, Dp, width;
+  void* h;                 // [T, Dp]
+  // convolution (cw null: none)
+  const float* cw;         // [taps, Dp], oldest tap first
+  int taps;
+  float* state;            // [slots, taps - 1, Dp]: the last inputs of every sequence, oldest first
+  float* tail;             // [B, taps - 1, Dp]: this step's last inputs (prefill); null: decode, state updated in place
+  const int* row_seq;      // prefill: sequence of every row
+  const int* q_start;      // prefill: [B] first row
+  const int* q_lens;       // prefill: [B]
+  const int* pos;          // [T]
+  const int* slots;        // [B] state slot, -1: none
+  int B, run;              // rows per workgroup
+};
+void launch_residual_norm(const ResidualNormArgs& a, bool f32, hipStream_t s);
+
+struct ConvCommitArgs {    // the tails of a prefill step into the state of every layer run
+  float* state;            // [runs, slots, taps - 1, Dp]
+  const float* tail;       // [runs, B, taps - 1, Dp]
+  const int* q_lens;
+  const int* slots;
+  int runs, n_slots, B, taps, Dp;
+};
+void launch_conv_commit(const ConvCommitArgs& a, hipStream_t s);
+
+struct RopeRowsArgs {      // cos / sin of pos * freq, every row of a step
+  const int* pos;
+  const float* freq;       // [n][2]: frequency as a float and its remainder
+  int T, n;
+  float* out;              // [T, n, 2]
+};
+void launch_rope_rows(const RopeRowsArgs& a, hipStream_t s);
+
+enum Epi : int { EPI_NONE = 0, EPI_CLAMP_GLU = 1, EPI_SOFTCAP = 2, EPI_XIELU = 3, EPI_ROTARY = 4 };
 struct GemmArgs {
   const void* A;           // [rows, K]
   const void* W;           // [N, K] or [E, N, K]
@@ -54,6 +104,12 @@ struct GemmArgs {
   int n_main;              // columns n_main .. N - 1 are a plain fp32 product, stored in side [M, N - n_main]
   float* side;
   bool out_f32;
+  long lda, ldc;           // row strides of A and C
+  int batch;               // dense: products batched over blockIdx.z (streaming kernel only)
+  long a_batch, w_batch, c_batch;
+  const float* vec;        // EPI_XIELU: (alpha_p, alpha_n)
+  const float* rope;       // EPI_ROTARY: [M, rot] cos / sin pairs; columns rot0 .. rot0 + rot - 1 of every `head` columns
+  int head, rot0, rot;
 };
 void launch_gemm(const GemmArgs& a, bool f32, hipStream_t s);          // streaming kernel, any M
 void launch_gemm_tile(const GemmArgs& a, hipStream_t s);               // LDS-tiled bf16 kernel (gemm_tile.hip)
@@ -91,9 +147,74 @@ struct AttnArgs {
   float* ws;               // decode split partials
   int B, T, max_q, H, G, dk, dv, max_blocks, splits, chunk;
   float scale;
+  // latent form of the prefill kernel: q rows at `qkvg`; keys of sequence b are rows kv_start[b] ..; a key is
+  // [kv[0 .. np) | lat[rank .. rank + rot)], its value kv[np .. np + dv)
+  const void* kv;          // [rows, H, np + dv]
+  const void* lat;         // [rows, lat_ld]
+  const int* kv_start;
+  const float* sink;       // [H]
+  int np, rot, rank, lat_ld;
 };
 void launch_kv_store(const AttnArgs& a, bool f32, hipStream_t s);
 void launch_attn_prefill(const AttnArgs& a, bool f32, hipStream_t s);
 void launch_attn_decode(const AttnArgs& a, bool f32, hipStream_t s);
+void launch_latent_prefill(const AttnArgs& a, hipStream_t s);          // bf16
+
+struct LatentPrepArgs {
+  const float* d;          // [T, qp + rp + op]: query latent, key/value latent, rotated key part
+  const float* wq;         // [qp] gains (zero in the pads)
+  const float* wkv;        // [rp]
+  const float* rope;       // [T, rot]
+  const int* slots;        // [T] cache slot, -1: none
+  void* cache;             // [blocks, 64, rp + op]
+  void* cq;                // [T, qp]
+  float eps;
+  int T, q_rank, kv_rank, rot, qp, rp, op;
+};
+void launch_latent_prep(const LatentPrepArgs& a, bool f32, hipStream_t s);
+
+struct LatentGatherArgs {  // cached rows of the listed sequences, back to back
+  const void* cache;       // [blocks, 64, ld]
+  void* out;               // [rows, ld]
+  const int* bt;           // [B, max_blocks]
+  const int* seqs;         // [n]
+  const int* ctx;          // [n]
+  const int* start;        // [n] first output row
+  int n, max_ctx, max_blocks, ld_bytes;
+};
+void launch_latent_gather(const LatentGatherArgs& a, hipStream_t s);
+
+struct LatentArgs {        // attention of single rows over the cached latents
+  const void* ql;          // [n, H, rp] queries in latent space
+  const void* q;           // [n, ldq]: the rotated part of head h at h * head + np
+  const void* cache;       // [blocks, 64, rp + op]
+  void* o;                 // [n, H, rp]
+  const int* bt;           // [B, max_blocks]
+  const int* seqs;         // [n] block table row of every entry, or null: entry i
+  const int* ctx;          // [n] keys that an entry sees
+  const float* sink;       // [H]
+  float* ws;               // [n, H, splits, rp + 4]: partial output, maximum, denominator
+  float scale;
+  long ldq;
+  int n, H, head, np, rot, rp, op, max_blocks, splits;
+};
+bool latent_decode_fits(int rp, int op);
+void launch_latent_decode(const LatentArgs& a, hipStream_t s);         // bf16, sizes that fit
+void launch_latent_rows(const LatentArgs& a, bool f32, hipStream_t s); // any size
+
+struct ScanArgs {          // minGRU: S = (1 - z) S + z c, out = S silu(g)
+  const float* zx;         // [T, 2 W]: z and u before their biases
+  const void* g;           // [T, W]
+  const float* bias;       // [2 W]
+  float* state;            // [slots, W]
+  void* out;               // [T, W]
+  const int* pos;          // [T]
+  const int* q_start;      // [B], null: one row per sequence (decode)
+  const int* q_lens;
+  const int* slots;        // [B], -1: none
+  float* ws;               // [B, chunks, 2, W] when a sequence has several chunks
+  int T, B, W, max_q, len, chunks;
+};
+void launch_mingru_scan(const ScanArgs& a, bool f32, hipStream_t s);
 
 }  // namespace shai_lm

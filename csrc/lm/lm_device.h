@@ -37,29 +37,65 @@ __device__ __forceinline__ float block_sum256(float v, float* red) {
   __syncthreads();
   return (red[0] + red[1]) + (red[2] + red[3]);
 }
+// the same with `red` changing between two buffers (`turn`), so that calls may follow each other with one barrier each
+__device__ __forceinline__ float block_sum256(float v, float (*red)[4], int& turn) {
+  v = wave_sum(v);
+  float* r = red[turn];
+  turn ^= 1;
+  if ((threadIdx.x & 63) == 0) r[threadIdx.x >> 6] = v;
+  __syncthreads();
+  return (r[0] + r[1]) + (r[2] + r[3]);
+}
 
-// Store 4 consecutive columns n .. n + 3 of row m after the epilogue.
+// xIELU: ap z^2 + z / 2 above zero, an (exp(z) - 1 - z) + z / 2 below
+__device__ __forceinline__ float xielu(float z, float ap, float an) {
+  return (z > 0.f ? ap * z * z : an * (expm1f(z) - z)) + 0.5f * z;
+}
+
+// Store 4 consecutive columns n .. n + 3 of row m after the epilogue.  `out`: C of this product.
 template <typename O>
-__device__ __forceinline__ void store_cols(const GemmArgs& p, long m, int n, float4_ c) {
-  O* out = static_cast<O*>(p.C);
+__device__ __forceinline__ void store_cols(const GemmArgs& p, O* out, long m, int n, float4_ c) {
   if (n >= p.n_main) {
+    const int ld = p.N - p.n_main, j = n - p.n_main;
+    float* o = p.side + m * ld + j;
+    if ((ld & 3) == 0) {
+      if (n < p.N) store4(o, c);
+      return;
+    }
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-      if (n + i < p.N) p.side[m * (p.N - p.n_main) + n + i - p.n_main] = c[i];
+      if (n + i < p.N) o[i] = c[i];
     return;
   }
   if (p.epi == EPI_CLAMP_GLU) {
-    const int ld = p.n_main >> 1, j = n >> 1;
-    if (n < p.N) store1(out + m * ld + j, clamp_glu(c[0], c[1], p.param));
-    if (n + 2 < p.N) store1(out + m * ld + j + 1, clamp_glu(c[2], c[3], p.param));
+    const int j = n >> 1;
+    if (n < p.N) store1(out + m * p.ldc + j, clamp_glu(c[0], c[1], p.param));
+    if (n + 2 < p.N) store1(out + m * p.ldc + j + 1, clamp_glu(c[2], c[3], p.param));
     return;
   }
   if (p.epi == EPI_SOFTCAP) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) c[i] = p.param * tanhf(c[i] / p.param);
+  } else if (p.epi == EPI_XIELU) {
+    const float ap = p.vec[0], an = p.vec[1];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) c[i] = xielu(c[i], ap, an);
+  } else if (p.epi == EPI_ROTARY) {
+    const int d = n % p.head - p.rot0;
+    if (d >= 0 && d < p.rot && n < p.N) {
+      const float* t = p.rope + m * p.rot + d;
+      const float u = c[0], v = c[1];
+      c[0] = u * t[0] - v * t[1];
+      c[1] = v * t[0] + u * t[1];
+      if (d + 2 < p.rot) {
+        const float u2 = c[2], v2 = c[3];
+        c[2] = u2 * t[2] - v2 * t[3];
+        c[3] = v2 * t[2] + u2 * t[3];
+      }
+    }
   }
-  O* o = out + m * p.N + n;
-  if ((p.N & 3) == 0) {
+  O* o = out + m * p.ldc + n;
+  if (((p.N | p.ldc) & 3) == 0) {
     if (n < p.N) store4(o, c);
   } else {
 #pragma unroll

@@ -1,4 +1,5 @@
-// Embedding + first norm, and residual add (+ expert combine) + norm, on the fp32 residual stream.
+// Embedding + first norm, residual add (+ expert combine) + norm, and normed residual add + norm + input convolution,
+// on the fp32 residual stream.
 // One 256-thread workgroup per row; the row stays in registers between the add and the norm (width <= 16384).
 #include "lm_device.h"
 #include "lm.h"
@@ -86,6 +87,170 @@ __global__ void __launch_bounds__(256) add_norm_kernel(const AddNormArgs p) {
   }
 }
 
+// The row stays in registers through both norms.  With a convolution a workgroup walks `run` consecutive rows and keeps
+// the last taps - 1 inputs in registers; the ones before its first row are recomputed from their residual rows (which is
+// why x_out is not x then) or, before the step's first row of a sequence, come from the sequence's state.
+template <typename T, int NV, int TAPS>
+__global__ void __launch_bounds__(256) residual_norm_kernel(const ResidualNormArgs p) {
+  __shared__ float red[2][4];
+  int turn = 0;
+  const int c0 = threadIdx.x * 4;
+  const float inv_w = 1.f / (float)p.width;
+  auto load = [&](long row, float4_(&v)[NV]) {
+    const float* x = p.x ? p.x + row * p.Dp : nullptr;
+    const T* e = x ? nullptr : static_cast<const T*>(p.table) + (long)min(max(p.ids[row], 0), p.V - 1) * p.Dp;
+    float4_ d[NV];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = i * 1024 + c0;
+      v[i] = float4_{0.f, 0.f, 0.f, 0.f};
+      d[i] = v[i];
+      if (c < p.Dp) {
+        v[i] = x ? load4(x + c) : load4(e + c) * p.scale;
+        if (p.delta) d[i] = load4(static_cast<const T*>(p.delta) + row * p.Dp + c);
+        ss += d[i][0] * d[i][0] + d[i][1] * d[i][1] + d[i][2] * d[i][2] + d[i][3] * d[i][3];
+      }
+    }
+    if (p.delta) {
+      ss = block_sum256(ss, red, turn);
+      const float r = p.mult / sqrtf(ss * inv_w + p.eps);
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = i * 1024 + c0;
+        if (c < p.Dp) v[i] += d[i] * r * load4(p.wb + c);
+      }
+    }
+    if (p.step) {
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = i * 1024 + c0;
+        if (c < p.Dp) v[i] += load4(p.step + c);
+      }
+    }
+  };
+  auto norm = [&](float4_(&v)[NV]) {
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) ss += v[i][0] * v[i][0] + v[i][1] * v[i][1] + v[i][2] * v[i][2] + v[i][3] * v[i][3];
+    ss = block_sum256(ss, red, turn);
+    const float r = 1.f / sqrtf(ss * inv_w + p.eps);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = i * 1024 + c0;
+      if (c < p.Dp) v[i] = v[i] * r * load4(p.w + c);
+    }
+  };
+  auto put = [&](auto* dst, const float4_(&v)[NV]) {
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+      if (i * 1024 + c0 < p.Dp) store4(dst + i * 1024 + c0, v[i]);
+  };
+
+  float4_ v[NV];
+  if constexpr (TAPS == 0) {
+    const long row = p.rows ? p.rows[blockIdx.x] : blockIdx.x;
+    load(row, v);
+    if (p.x_out) put(p.x_out + row * p.Dp, v);
+    if (!p.w) return;
+    norm(v);
+    put(static_cast<T*>(p.h) + (long)blockIdx.x * p.Dp, v);
+  } else {
+    float4_ hist[TAPS - 1][NV];                  // hist[j]: input of the row j + 1 before
+    const int row0 = blockIdx.x * p.run, row1 = min(row0 + p.run, p.T);
+    int seq = -1;
+    for (int t = row0; t < row1; ++t) {
+      const int b = p.row_seq ? p.row_seq[t] : t;
+      const int at = p.row_seq ? t - p.q_start[b] : 0, pos = p.pos[t], slot = p.slots[b];
+      float* st = p.state + (long)max(slot, 0) * (p.taps - 1) * p.Dp;
+      if (b != seq) {
+        seq = b;
+#pragma unroll
+        for (int j = 0; j < TAPS - 1; ++j) {
+#pragma unroll
+          for (int i = 0; i < NV; ++i) hist[j][i] = float4_{0.f, 0.f, 0.f, 0.f};
+          const int back = j + 1;
+          if (back >= p.taps || back > pos) continue;
+          if (back <= at) {                      // a row of this step
+            load(t - back, hist[j]);
+            norm(hist[j]);
+          } else if (slot >= 0) {
+            const float* s = st + (long)(p.taps - 1 - (back - at)) * p.Dp;
+#pragma unroll
+            for (int i = 0; i < NV; ++i)
+              if (i * 1024 + c0 < p.Dp) hist[j][i] = load4(s + i * 1024 + c0);
+          }
+        }
+      }
+      load(t, v);
+      put(p.x_out + (long)t * p.Dp, v);
+      norm(v);
+      float4_ y[NV];
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = i * 1024 + c0;
+        y[i] = v[i];
+        if (c < p.Dp) {
+          y[i] += load4(p.cw + (long)(p.taps - 1) * p.Dp + c) * v[i];
+#pragma unroll
+          for (int j = 0; j < TAPS - 1; ++j)
+            if (j + 1 < p.taps) y[i] += load4(p.cw + (long)(p.taps - 2 - j) * p.Dp + c) * hist[j][i];
+        }
+      }
+      put(static_cast<T*>(p.h) + (long)t * p.Dp, y);
+      if (p.row_seq) {
+        const int left = p.q_lens[b] - 1 - at;   // rows of the sequence after this one
+        if (left < p.taps - 1) put(p.tail + ((long)b * (p.taps - 1) + p.taps - 2 - left) * p.Dp, v);
+      } else if (slot >= 0 && p.taps > 1) {      // the only workgroup that reads this state
+        put(st + (long)(p.taps - 2) * p.Dp, v);
+#pragma unroll
+        for (int j = 0; j < TAPS - 1; ++j)
+          if (j + 2 < p.taps) put(st + (long)(p.taps - 3 - j) * p.Dp, hist[j]);
+      }
+#pragma unroll
+      for (int j = TAPS - 2; j > 0; --j)
+#pragma unroll
+        for (int i = 0; i < NV; ++i) hist[j][i] = hist[j - 1][i];
+#pragma unroll
+      for (int i = 0; i < NV; ++i) hist[0][i] = v[i];
+    }
+  }
+}
+
+// Newest inputs first come from the step's tail, older ones move down inside the state (a portion shorter than the window).
+__global__ void __launch_bounds__(256) conv_commit_kernel(const ConvCommitArgs p) {
+  const int b = blockIdx.y, run = blockIdx.z, c = (blockIdx.x * 256 + threadIdx.x) * 4;
+  const int slot = p.slots[b], n = p.q_lens[b], k = p.taps - 1;
+  if (c >= p.Dp || slot < 0 || slot >= p.n_slots) return;
+  float* st = p.state + ((long)run * p.n_slots + slot) * k * p.Dp + c;
+  const float* tail = p.tail + ((long)run * p.B + b) * k * p.Dp + c;
+  for (int j = 0; j < k; ++j)
+    store4(st + (long)j * p.Dp, k - 1 - j < n ? load4(tail + (long)j * p.Dp) : load4(st + (long)(j + n) * p.Dp));
+}
+
+void launch_conv_commit(const ConvCommitArgs& a, hipStream_t s) {
+  conv_commit_kernel<<<dim3((a.Dp + 1023) / 1024, a.B, a.runs), 256, 0, s>>>(a);
+  SHAI_CHECK_LAUNCH();
+}
+
+// The angle is a float pair: position * frequency and its rounding error plus the frequency's remainder.
+__global__ void __launch_bounds__(256) rope_rows_kernel(const RopeRowsArgs p) {
+  const long id = (long)blockIdx.x * 256 + threadIdx.x;
+  if (id >= (long)p.T * p.n) return;
+  const int t = id / p.n, i = id % p.n;
+  const float x = (float)p.pos[t], f = p.freq[2 * i], a = x * f;
+  const float e = fmaf(x, f, -a) + x * p.freq[2 * i + 1];
+  float s, c;
+  sincosf(a, &s, &c);
+  p.out[2 * id] = c - s * e;
+  p.out[2 * id + 1] = s + c * e;
+}
+
+void launch_rope_rows(const RopeRowsArgs& a, hipStream_t s) {
+  rope_rows_kernel<<<((long)a.T * a.n + 255) / 256, 256, 0, s>>>(a);
+  SHAI_CHECK_LAUNCH();
+}
+
 #define SHAI_LM_ROWS(KERNEL, a, f32, s)                                                            \
   do {                                                                                             \
     const int nv = ((a).Dp + 1023) / 1024;                                                         \
@@ -104,5 +269,31 @@ __global__ void __launch_bounds__(256) add_norm_kernel(const AddNormArgs p) {
 
 void launch_embed_norm(const EmbedNormArgs& a, bool f32, hipStream_t s) { SHAI_LM_ROWS(embed_norm_kernel, a, f32, s); }
 void launch_add_norm(const AddNormArgs& a, bool f32, hipStream_t s) { SHAI_LM_ROWS(add_norm_kernel, a, f32, s); }
+
+template <typename T, int NV>
+static void residual_norm(const ResidualNormArgs& a, hipStream_t s) {
+  if (!a.cw) {
+    residual_norm_kernel<T, NV, 0><<<a.T, 256, 0, s>>>(a);
+    return;
+  }
+  const int grid = (a.T + a.run - 1) / a.run;
+  if (NV <= 8 && a.taps <= 4) residual_norm_kernel<T, NV, NV <= 8 ? 4 : 16><<<grid, 256, 0, s>>>(a);
+  else residual_norm_kernel<T, NV, 16><<<grid, 256, 0, s>>>(a);
+}
+
+void launch_residual_norm(const ResidualNormArgs& a, bool f32, hipStream_t s) {
+  const int nv = (a.Dp + 1023) / 1024;
+  auto go = [&](auto tag) {
+    using T = decltype(tag);
+    if (nv <= 1) residual_norm<T, 1>(a, s);
+    else if (nv <= 2) residual_norm<T, 2>(a, s);
+    else if (nv <= 4) residual_norm<T, 4>(a, s);
+    else if (nv <= 8) residual_norm<T, 8>(a, s);
+    else residual_norm<T, 16>(a, s);
+  };
+  if (f32) go(float{});
+  else go(bf16_t{});
+  SHAI_CHECK_LAUNCH();
+}
 
 }  // namespace shai_lm

@@ -68,6 +68,7 @@ class Sequence_:
     params: SamplingParams
     output: List[int] = field(default_factory=list)
     blocks: List[int] = field(default_factory=list)
+    state_slot: int = -1     # models with per-sequence state
     n_cached: int = 0        # tokens whose K/V are in the cache
     image: Optional[dict] = None                                 # preprocessed image (multimodal models)
     img_pos: int = -1                                            # index of <|image|> in the prompt
@@ -185,7 +186,7 @@ class _DecodeGraph:
     previous decode step's output (``engine.last_tokens``) instead of the host id.  This is what lets the
     engine enqueue step t+1 before it has read step t's tokens back (``LLMEngine.async_decode``)."""
 
-    NF = 10  # per-row int32 fields before the block table
+    NF = 11  # per-row int32 fields before the block table
 
     def __init__(self, engine: "LLMEngine", Bc: int, cross: bool = False, greedy: bool = False,
                  splits: Optional[int] = None, full_vocab: bool = False):
@@ -202,12 +203,13 @@ class _DecodeGraph:
         f = lambda i: self.dbuf[i * Bc:(i + 1) * Bc]
         self.ids, self.pos, self.slots, self.lens, self.topk = f(0), f(1), f(2), f(3), f(4)
         self.temps, self.topp, self.u = f(5).view(torch.float32), f(6).view(torch.float32), f(7).view(torch.float32)
-        self.rowmap, self.prev = f(8), f(9)
+        self.rowmap, self.prev, self.state_slots = f(8), f(9), f(10)
         self.bt = self.dbuf[self.NF * Bc:].view(Bc, mb)
         self.slots.fill_(-1)
         self.lens.fill_(1)
         self.rowmap.fill_(-1)
         self.prev.fill_(-1)
+        self.state_slots.fill_(-1)
         self.toks = torch.zeros(Bc, dtype=torch.int32, device=dev)
         pin = dev.type == "cuda"
         self.host = [torch.zeros(self.words, dtype=torch.int32, pin_memory=pin) for _ in range(2)]
@@ -216,7 +218,7 @@ class _DecodeGraph:
         self.flip = 0
         self.splits = splits if splits is not None else engine.decode_splits(Bc, 0)
         self.batch = Batch(self.ids, self.pos, self.slots, self.bt, self.lens, None, Bc, 1, False, self.splits,
-                           prev_ids=self.prev)
+                           prev_ids=self.prev, states=engine.states, state_slots=self.state_slots)
         self.cross = cross
         self.greedy = greedy
         if cross:  # static image-K/V inputs of the cross-attention layers
@@ -277,6 +279,7 @@ class _DecodeGraph:
         v(7).view(np.float32)[:B] = uniforms
         v(8)[:B] = rowmap
         v(9)[:B] = -1 if prev is None else prev
+        v(10)[:B] = [s.state_slot for s in seqs]
         btv = h[self.NF * Bc:].reshape(Bc, -1)
         btv[:B] = bt
         if B < Bc:  # padding rows: no KV write, one-token context, greedy, no feedback
@@ -290,6 +293,7 @@ class _DecodeGraph:
             v(7).view(np.float32)[B:] = 0.0
             v(8)[B:] = -1
             v(9)[B:] = -1
+            v(10)[B:] = -1
             btv[B:] = 0
         self.dbuf.copy_(self.host[i], non_blocking=True)
         if self.cross:
@@ -338,7 +342,7 @@ class _Inflight:
 
 
 class LLMEngine:
-    """``cfg``: a config of :mod:`shai_amd.models.registry` (Llama family, mllama, Golulix)."""
+    """``cfg``: a config of :mod:`shai_amd.models.registry` (Llama family, mllama, Golulix, Faledra)."""
 
     def __init__(self, cfg, device="cuda", model_path: Optional[str] = None, seed: int = 0,
                  max_num_seqs: int = 64, max_model_len: int = 4096, num_kv_blocks: Optional[int] = None,
@@ -347,7 +351,7 @@ class LLMEngine:
                  quantization: Optional[str] = None, async_decode: Optional[bool] = None,
                  packed_prefill: bool = True, mixed_steps: bool = True, dtype: torch.dtype = torch.bfloat16):
         from ..models.mllama import MllamaConfig
-        from ..runtime import BlockManager
+        from ..runtime import BlockManager, SlotPool
         self.mcfg = cfg if isinstance(cfg, MllamaConfig) else None
         cls = model_class(cfg)
         if dtype not in cls.dtypes:
@@ -377,6 +381,9 @@ class LLMEngine:
         self.cross_tokens = self.model.tokens_per_image if self.mcfg is not None else 0
         self.max_cross_blocks = (self.cross_tokens + KV_BLOCK - 1) // KV_BLOCK
         per_seq = self.max_blocks + self.max_cross_blocks
+        # per-sequence state (recurrences, convolution inputs): one slot for every sequence that may run at a time
+        self.states = self.model.allocate_state(max_num_seqs, self.device) if self.model.has_state else None
+        self.state_slots = SlotPool(max_num_seqs)
         if num_kv_blocks is None:
             if self.device.type == "cuda":
                 free, total = torch.cuda.mem_get_info(self.device)
@@ -394,9 +401,10 @@ class LLMEngine:
         self._last_step = "decode"
         # packed varlen prefill (no [B, S_max] padding) with decode rows mixed into prefill steps (text models)
         self.packed_prefill = ((packed_prefill and os.environ.get("SHAI_PADDED_PREFILL", "0") != "1")
-                               or self.model.needs_prev_token)   # those models have the packed layout only
+                               or self.model.needs_prev_token or self.model.has_state)   # those have the packed layout only
         self.mixed_steps = mixed_steps
-        self.prefix_caching = enable_prefix_caching
+        # a shared prefix is cached blocks: it does not bring the state at its end
+        self.prefix_caching = enable_prefix_caching and not self.model.has_state
         self.use_graphs = use_graphs and self.device.type == "cuda"
         self.waiting: List[Sequence_] = []
         self.running: List[Sequence_] = []
@@ -489,7 +497,7 @@ class LLMEngine:
         self._inflight = None
         gone = self.waiting + self.running
         for s in gone:
-            if s.blocks or s.cross_blocks:
+            if s.blocks or s.cross_blocks or s.state_slot >= 0:
                 self._free(s)
             s.finished, s.finish_reason = True, "abort"
         self.waiting, self.running = [], []
@@ -507,8 +515,15 @@ class LLMEngine:
 
     def _free(self, s: Sequence_):
         self.bm.release(s.blocks + s.cross_blocks)
+        if s.state_slot >= 0:
+            self.state_slots.release(s.state_slot)
+            s.state_slot = -1
         s.blocks = []
         s.cross_blocks = []
+
+    def _ensure_slot(self, s: Sequence_):
+        if self.states is not None and s.state_slot < 0:
+            s.state_slot = self.state_slots.allocate()
 
     def _prefix_hashes(self, toks: Sequence[int], n_full: int) -> List[int]:
         hs, h = [], 0
@@ -523,8 +538,8 @@ class LLMEngine:
         if not self.waiting:
             return []
         watermark = max(1, len(self.running))
-        n = sched_admit([len(s.prompt) for s in self.waiting], self.bm.num_free, len(self.running),
-                        self.max_num_seqs, self.prefill_token_budget, watermark)
+        n = sched_admit([len(s.prompt) for s in self.waiting], self.bm.num_free,
+                        len(self.running) + len(self.driven), self.max_num_seqs, self.prefill_token_budget, watermark)
         if self.mcfg is not None:  # image K/V blocks are outside the native scheduler's block budget
             free, k = self.bm.num_free - watermark, 0
             for s in self.waiting[:n]:
@@ -566,6 +581,7 @@ class LLMEngine:
                 self.stats["prefix_hit_tokens"] += s.n_cached
             ok = self._ensure_blocks(s, len(s.prompt) + 1)
             assert ok, "scheduler admitted a prompt without blocks"
+            self._ensure_slot(s)
             if s.image is not None and not s.cross_blocks:
                 s.cross_blocks = self.bm.allocate(self.max_cross_blocks)
                 s._img_encoded = False
@@ -630,7 +646,15 @@ class LLMEngine:
                 prev[at] = toks[s.n_cached - 1]
         return Batch(t(ids), t(pos), t(slots), t(bt), t(lens), t(qlens), len(rows), max(news), True, 1,
                      t(last if want is None else want).long(), q_start=t(qstart),
-                     prev_ids=t(prev) if self.model.needs_prev_token else None)
+                     prev_ids=t(prev) if self.model.needs_prev_token else None, **self._packed_state(rows, news, t))
+
+    def _packed_state(self, rows, news, t) -> dict:
+        """What a packed step of a model with state needs besides."""
+        if self.states is None:
+            return {}
+        return {"states": self.states, "state_slots": t(np.asarray([s.state_slot for s in rows], dtype=np.int32)),
+                "row_seq": t(np.repeat(np.arange(len(rows), dtype=np.int32), news)), "q_lens_host": list(news),
+                "ctx_lens_host": [s.n_cached + n for s, n in zip(rows, news)]}
 
     # ------------------------------------------------------------------ externally driven requests
     def open_request(self) -> Sequence_:
@@ -639,6 +663,7 @@ class LLMEngine:
         if len(self.driven) + len(self.running) >= self.max_num_seqs:
             raise MemoryError(f"all {self.max_num_seqs} sequence slots are in use")
         s = Sequence_(next(self._ids), [], SamplingParams())
+        self._ensure_slot(s)
         self.driven.append(s)
         return s
 
@@ -1071,16 +1096,18 @@ class LLMService:
 
 def llama_config_for(model_id: str, model_path: Optional[str] = None, size: str = ""):
     """The config of a checkpoint folder (its config.json), else the one a model id names."""
+    from ..models.faledra import FaledraConfig
     from ..models.golulix import GolulixConfig
     from ..models.mllama import MllamaConfig
     cfg = config_from_path(model_path)
     if cfg is not None:
         return cfg
     m = (model_id or "").lower()
-    if "golulix" in m:
-        if size != "tiny":
-            raise ValueError("Golulix has no published size: give the folder of a checkpoint (config.json)")
-        return GolulixConfig.tiny()
+    for name, design in (("golulix", GolulixConfig), ("faledra", FaledraConfig)):
+        if name in m:
+            if size != "tiny":
+                raise ValueError(f"{name} has no published size: give the folder of a checkpoint (config.json)")
+            return design.tiny()
     vision = "vision" in m or "mllama" in m
     if size == "tiny":
         return MllamaConfig.tiny() if vision else LlamaConfig.tiny()

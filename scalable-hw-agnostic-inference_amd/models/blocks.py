@@ -1,6 +1,6 @@
 """Building blocks of decoders that are described layer by layer in their config (fp32 residual stream).
 
-Each block keeps its weights in the layout of :mod:`shai_amd.ops.lm` (width padded to 64, head sizes to 64 / 128 / 256,
+Each block keeps its weights in the layout of :mod:`shai_amd.ops.lm` (width padded to 64, head sizes to kernel sizes,
 gate / up rows interleaved, experts stacked) and packs them from checkpoint tensors in ``pack``: ``pack(get)`` maps the
 block's own tensor names (``get("q")``) to its parameters, so a model only supplies the prefix.
 """
@@ -32,6 +32,15 @@ def _padded(t: torch.Tensor, *shape) -> torch.Tensor:
 def _head_rows(t: torch.Tensor, heads: int, dim: int, pad: int, width: int) -> torch.Tensor:
     """[heads * dim, D] -> [heads * pad, width], every head's rows padded by zero rows."""
     return _padded(t.reshape(heads, dim, t.shape[1]), heads, pad, width).reshape(heads * pad, width)
+
+
+def check_checkpoint(sd: Dict[str, torch.Tensor], want: Dict[str, tuple]) -> None:
+    """A missing, unknown or misshapen tensor is an error."""
+    bad = ([k for k in want if k not in sd] + [k for k in sd if k not in want]
+           + [k for k in want if k in sd and tuple(sd[k].shape) != want[k]])
+    if bad:
+        raise ValueError(f"checkpoint does not fit config.json: {len(bad)} tensors missing, unknown or misshapen, "
+                         f"e.g. {bad[:5]}")
 
 
 class OffsetNorm(nn.Module):
@@ -216,9 +225,230 @@ class SoftcapHead(nn.Module):
         self.weight[:, :self.width].normal_(0, self.width ** -0.5, generator=gen)
 
 
+class GainNorm(nn.Module):
+    """RMSNorm gains as stored (applied by ``ops.lm.residual_norm``)."""
+
+    def __init__(self, width: int):
+        super().__init__()
+        self.width = width
+        self.weight = _param(lm.pad64(width), dtype=torch.float32)
+
+    def pack(self, t: torch.Tensor) -> torch.Tensor:
+        return _padded(t, lm.pad64(self.width))
+
+    def init_random_(self, gen):
+        self.weight[:self.width] = 1.0
+
+
+class InputConv(nn.Module):
+    """Causal convolution over time on each channel of a sublayer's normed input, added to it."""
+
+    def __init__(self, width: int, taps: int):
+        super().__init__()
+        if not 1 <= taps <= lm.MAX_TAPS:
+            raise ValueError(f"input convolutions of 1 to {lm.MAX_TAPS} taps are supported, got {taps}")
+        self.width, self.taps = width, taps
+        self.weight = _param(taps, lm.pad64(width), dtype=torch.float32)
+
+    def pack(self, t: torch.Tensor) -> torch.Tensor:
+        return _padded(t.T, self.taps, lm.pad64(self.width))
+
+    def init_random_(self, gen):
+        self.weight[:, :self.width].normal_(0, self.taps ** -0.5, generator=gen)
+
+
+@dataclass
+class LatentAttentionConfig:
+    heads: int
+    dim: int            # unrotated query / key size of a head
+    rot_dim: int        # rotated size
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    rot_base: float = 10000.0
+
+    def __post_init__(self):
+        if min(self.heads, self.dim, self.vdim, self.q_rank, self.kv_rank) < 1 or self.rot_dim < 2 or self.rot_dim % 2:
+            raise ValueError(f"bad attention sizes: {self}")
+        if self.kv_rank > lm.MAX_LATENT:
+            raise ValueError(f"latents of up to {lm.MAX_LATENT} values are supported, got {self.kv_rank}")
+
+
+class LatentAttention(nn.Module):
+    """Attention whose cache is one latent row and one rotated key part per token, shared by all heads; queries go through
+    a latent of their own; a learned sink per head in the denominator.
+
+    Decode steps and short portions attend in latent space: the queries go through W_uk, the attended latent through
+    W_uv (one small product per head each), and keys and values are never built.  Longer portions expand them per head
+    from the cached latents and run the flash kernel."""
+
+    def __init__(self, width: int, c: LatentAttentionConfig, eps: float, dtype=torch.bfloat16):
+        super().__init__()
+        self.c, self.width, self.eps, self.dtype = c, width, eps, dtype
+        pad8 = lambda n: (n + 7) // 8 * 8
+        self.np, self.kn = pad8(c.dim), lm.pad64(c.dim)          # unrotated part in a head's row; as a product's depth
+        self.qp, self.op = lm.pad64(c.q_rank), lm.pad64(c.rot_dim)
+        self.rp = next((r for r in (64, 128, 256, 512) if c.kv_rank <= r), lm.pad64(c.kv_rank))
+        fit = lm.latent_head_pad(self.np + pad8(c.rot_dim), c.vdim)
+        self.dk, self.dv = fit or (lm.pad64(self.np + pad8(c.rot_dim)), lm.pad64(c.vdim))
+        self.expands = fit is not None and dtype == torch.bfloat16
+        H, W = c.heads, lm.pad64(width)
+        self.down = _param(self.qp + self.rp + self.op, W, dtype=dtype)
+        self.q_norm = _param(self.qp, dtype=torch.float32)
+        self.kv_norm = _param(self.rp, dtype=torch.float32)
+        self.uq = _param(H * self.dk, self.qp, dtype=dtype)
+        self.uk = _param(H, self.rp, self.kn, dtype=dtype)       # queries into latent space
+        self.ukv = _param(H, self.np + self.dv, self.rp, dtype=dtype)
+        self.sink = _param(H, dtype=torch.float32)
+        self.o = _param(W, H * self.dv, dtype=dtype)
+        self.register_buffer("freq", lm.rope_freq(c.rot_base, c.rot_dim).to(self.o.device), persistent=False)
+
+    def shapes(self) -> Dict[str, tuple]:
+        c, D = self.c, self.width
+        return {"dq": (c.q_rank, D), "dq.norm": (c.q_rank,), "uq": (c.heads * (c.dim + c.rot_dim), c.q_rank),
+                "dkv": (c.kv_rank + c.rot_dim, D), "dkv.norm": (c.kv_rank,), "uk": (c.heads * c.dim, c.kv_rank),
+                "uv": (c.heads * c.vdim, c.kv_rank), "sink": (c.heads,), "o": (D, c.heads * c.vdim)}
+
+    def pack(self, get: Callable[[str], torch.Tensor]) -> Dict[str, torch.Tensor]:
+        c, W, H = self.c, self.down.shape[1], self.c.heads
+        dkv = get("dkv")
+        q = get("uq").reshape(H, c.dim + c.rot_dim, c.q_rank)
+        uk, uv = get("uk").reshape(H, c.dim, c.kv_rank), get("uv").reshape(H, c.vdim, c.kv_rank)
+        o = get("o").reshape(self.width, H, c.vdim)
+        return {"down": torch.cat([_padded(get("dq"), self.qp, W), _padded(dkv[:c.kv_rank], self.rp, W),
+                                   _padded(dkv[c.kv_rank:], self.op, W)]),
+                "q_norm": _padded(get("dq.norm"), self.qp), "kv_norm": _padded(get("dkv.norm"), self.rp),
+                "uq": torch.cat([_padded(q[:, :c.dim], H, self.np, self.qp),
+                                 _padded(q[:, c.dim:], H, self.dk - self.np, self.qp)], 1).reshape(H * self.dk, self.qp),
+                "uk": _padded(uk.transpose(1, 2), H, self.rp, self.kn),
+                "ukv": torch.cat([_padded(uk, H, self.np, self.rp), _padded(uv, H, self.dv, self.rp)], 1),
+                "sink": get("sink"), "o": _padded(o, W, H, self.dv).reshape(W, H * self.dv)}
+
+    def forward(self, h, batch, cache, step):
+        """``step``: the step's shared work (:class:`StepShared`)."""
+        c, H = self.c, self.c.heads
+        rope, plan = step.rope(self), step.plan(self.expands)
+        down = lm.matmul(h, self.down, torch.float32)
+        cq = lm.latent_prep(down, self.q_norm, self.kv_norm, rope, batch, cache, self.eps, c.q_rank, c.kv_rank)
+        q = lm.matmul(cq, self.uq, epi=lm.EPI_ROTARY, rope=rope, head=self.dk, rot0=self.np)
+        if not plan.groups:
+            return lm.matmul(self._in_latent_space(q, batch, cache, plan), self.o)
+        o = torch.empty(q.shape[0], H * self.dv, dtype=q.dtype, device=q.device)
+        for g in plan.groups:
+            lat = lm.latent_gather(cache, batch.block_table, g)
+            kv = lm.matmul(lat[:, :self.rp], self.ukv.view(-1, self.rp))
+            lm.latent_prefill(q, kv, lat, o, g, self.sink, H, self.np, c.rot_dim, self.rp, c.scale)
+        if plan.n:
+            rows = plan.rows
+            o.index_copy_(0, rows.long(), self._in_latent_space(q.index_select(0, rows), batch, cache, plan))
+        return lm.matmul(o, self.o)
+
+    def _in_latent_space(self, q, batch, cache, plan):
+        c, n = self.c, q.shape[0]
+        ql = lm.matmul_heads(q.view(n, c.heads, self.dk)[..., :self.kn], self.uk)
+        ol = lm.latent_rows(ql, q, cache, batch.block_table, plan, self.sink, self.np, c.rot_dim, c.scale)
+        return lm.matmul_heads(ol, self.ukv[:, self.np:]).view(n, c.heads * self.dv)
+
+    def cache_shape(self, blocks: int, block: int):
+        return blocks, block, self.rp + self.op
+
+    state_width = None
+
+    def init_random_(self, gen):
+        _init_packed(self, self.pack, self.shapes(), gen)
+
+
+class StepShared:
+    """What the layers of one step share: rotation angles per (base, dims) and the attention plan per kind."""
+
+    def __init__(self, batch):
+        self.batch, self._ropes, self._plans = batch, {}, {}
+
+    def rope(self, mix: LatentAttention):
+        key = (mix.c.rot_base, mix.c.rot_dim)
+        if key not in self._ropes:
+            self._ropes[key] = lm.rope_rows(self.batch.positions, mix.freq)
+        return self._ropes[key]
+
+    def plan(self, expands: bool):
+        if expands not in self._plans:
+            self._plans[expands] = lm.latent_plan(self.batch, expands)
+        return self._plans[expands]
+
+
+class MinGRU(nn.Module):
+    """Gated recurrence whose gates read the current token only; output gated by silu and projected.  One product gives
+    the output gate (weights' dtype) and the recurrence's inputs (fp32)."""
+
+    def __init__(self, width: int, size: int, dtype=torch.bfloat16):
+        super().__init__()
+        if size < 1:
+            raise ValueError(f"bad recurrence width {size}")
+        self.width, self.size = width, size
+        self.sp = lm.pad64(size)
+        self.gzx = _param(3 * self.sp, lm.pad64(width), dtype=dtype)
+        self.bias = _param(2 * self.sp, dtype=torch.float32)
+        self.o = _param(lm.pad64(width), self.sp, dtype=dtype)
+
+    @property
+    def state_width(self) -> int:
+        return self.sp
+
+    def shapes(self) -> Dict[str, tuple]:
+        n, D = self.size, self.width
+        return {"z": (n, D), "z.b": (n,), "x": (n, D), "x.b": (n,), "g": (n, D), "o": (D, n)}
+
+    def pack(self, get: Callable[[str], torch.Tensor]) -> Dict[str, torch.Tensor]:
+        W = self.gzx.shape[1]
+        return {"gzx": torch.cat([_padded(get(n), self.sp, W) for n in ("g", "z", "x")]),
+                "bias": torch.cat([_padded(get(n), self.sp) for n in ("z.b", "x.b")]),
+                "o": _padded(get("o"), W, self.sp)}
+
+    def forward(self, h, batch, state, step=None):
+        g, zx = lm.matmul_with_side(h, self.gzx, 2 * self.sp)
+        return lm.matmul(lm.mingru_scan(zx, g, self.bias, state, batch), self.o)
+
+    def cache_shape(self, blocks: int, block: int):
+        return None
+
+    def init_random_(self, gen):
+        _init_packed(self, self.pack, self.shapes(), gen)
+
+
+class XieluMLP(nn.Module):
+    """Dense feed-forward with the xIELU activation; its two learned numbers enter as softplus(p), 1/2 + softplus(q)."""
+
+    def __init__(self, width: int, ff: int, dtype=torch.bfloat16):
+        super().__init__()
+        self.width, self.ff = width, ff
+        self.up = _param(lm.pad64(ff), lm.pad64(width), dtype=dtype)
+        self.down = _param(lm.pad64(width), lm.pad64(ff), dtype=dtype)
+        self.act = _param(2, dtype=torch.float32)
+
+    def shapes(self) -> Dict[str, tuple]:
+        return {"up": (self.ff, self.width), "down": (self.width, self.ff), "act": (2,)}
+
+    def pack(self, get: Callable[[str], torch.Tensor]) -> Dict[str, torch.Tensor]:
+        act = torch.nn.functional.softplus(get("act").double())
+        return {"up": _padded(get("up"), *self.up.shape), "down": _padded(get("down"), *self.down.shape),
+                "act": (act + torch.tensor([0.0, 0.5], dtype=act.dtype, device=act.device)).float()}
+
+    def forward(self, h):
+        return lm.matmul(lm.matmul(h, self.up, epi=lm.EPI_XIELU, vec=self.act), self.down)
+
+    def init_random_(self, gen):
+        _init_packed(self, self.pack, self.shapes(), gen)
+
+
 def _init_packed(module: nn.Module, pack, shapes: Dict[str, tuple], gen) -> None:
-    """Fill a block from random full-size tensors of its checkpoint shapes (N(0, 1 / fan_in))."""
+    """Fill a block from random full-size tensors of its checkpoint shapes: matrices N(0, 1 / fan_in), norm gains 1, other
+    vectors 0."""
     dev, dtype = gen.device, next(module.parameters()).dtype
-    draw = lambda name: (torch.randn(shapes[name], generator=gen, device=dev) / math.sqrt(shapes[name][1])).to(dtype)
+
+    def draw(name):
+        if len(shapes[name]) == 1:
+            return torch.full(shapes[name], float(name.endswith("norm")), device=dev)
+        return (torch.randn(shapes[name], generator=gen, device=dev) / math.sqrt(shapes[name][1])).to(dtype)
     for k, v in pack(draw).items():
         getattr(module, k).copy_(v)

@@ -18,7 +18,7 @@ import torch
 import torch.nn as nn
 
 from .blocks import (BigramEmbedding, ChunkAttention, ChunkAttentionConfig, ClampedGLUConfig, MoE, MoEConfig,
-                     OffsetNorm, SoftcapHead)
+                     OffsetNorm, SoftcapHead, check_checkpoint)
 from .llama import KV_BLOCK, Batch
 from ..ops import lm
 from ..parallel.state import tp
@@ -118,6 +118,7 @@ class GolulixLayer(nn.Module):
 
 
 class GolulixForCausalLM(nn.Module):
+    has_state = False
     needs_prev_token = True   # Batch.prev_ids: the bigram embedding reads every row's preceding token
     dtypes = (torch.bfloat16, torch.float32)
 
@@ -197,12 +198,7 @@ class GolulixForCausalLM(nn.Module):
 
     def convert_hf_state_dict(self, sd: Dict[str, torch.Tensor]) -> Dict[str, torch.Tensor]:
         """Checkpoint tensors -> packed parameters; a missing, unknown or misshapen tensor is an error."""
-        want = self.checkpoint_shapes()
-        bad = ([k for k in want if k not in sd] + [k for k in sd if k not in want]
-               + [k for k in want if k in sd and tuple(sd[k].shape) != want[k]])
-        if bad:
-            raise ValueError(f"checkpoint does not fit config.json: {len(bad)} tensors missing, unknown or misshapen, "
-                             f"e.g. {bad[:5]}")
+        check_checkpoint(sd, self.checkpoint_shapes())
         W = lm.pad64(self.cfg.width)
         wide = lambda t: torch.nn.functional.pad(t, (0, W - t.shape[1]))
         out = {"embed.weight": wide(sd["embed"]), "head.weight": wide(sd["head"]),

@@ -160,6 +160,13 @@ class Batch:
     q_start: Optional[torch.Tensor] = None
     # each row's preceding token (-1: the row is its sequence's first), for models with ``needs_prev_token``
     prev_ids: Optional[torch.Tensor] = None
+    # models with ``has_state``: the engine's per-slot state, each sequence's slot (-1: none), and in a packed step the
+    # sequence of every row and the host's copies of q_lens / ctx_lens
+    states: Optional[tuple] = None
+    state_slots: Optional[torch.Tensor] = None      # [B] int32
+    row_seq: Optional[torch.Tensor] = None          # [T] int32
+    q_lens_host: Optional[List[int]] = None
+    ctx_lens_host: Optional[List[int]] = None
 
 
 class LlamaAttention(nn.Module):
@@ -235,6 +242,7 @@ class LlamaDecoderLayer(nn.Module):
 class LlamaForCausalLM(nn.Module):
     dtypes = (torch.bfloat16,)
     needs_prev_token = False
+    has_state = False
     attn_span: Optional[int] = None   # full causal attention
 
     def __init__(self, cfg: LlamaConfig):

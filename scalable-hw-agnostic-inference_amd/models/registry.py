@@ -2,7 +2,8 @@
 
 A model class offers the engine: ``forward(batch, kv_caches)`` -> logits, ``kv_heads_local``, ``fold_norms()``,
 ``allocate_cache(blocks, device)``, ``cache_bytes_per_block()``, and the attributes ``dtypes`` (weight formats it runs
-in), ``needs_prev_token`` (rows carry their preceding token) and ``attn_span`` (most keys a position sees, or None).
+in), ``needs_prev_token`` (rows carry their preceding token), ``attn_span`` (most keys a position sees, or None) and
+``has_state`` (sequences hold a slot of the state that ``allocate_state(slots, device)`` makes; ``Batch.states``).
 """
 from __future__ import annotations
 
@@ -10,15 +11,17 @@ import json
 import os
 from typing import Callable, Dict, Optional
 
+from .faledra import FaledraConfig, FaledraForCausalLM
 from .golulix import GolulixConfig, GolulixForCausalLM
 from .llama import LlamaConfig, LlamaForCausalLM
 from .mllama import MllamaConfig, MllamaForConditionalGeneration
 
 MODELS = {LlamaConfig: LlamaForCausalLM, MllamaConfig: MllamaForConditionalGeneration,
-          GolulixConfig: GolulixForCausalLM}
+          GolulixConfig: GolulixForCausalLM, FaledraConfig: FaledraForCausalLM}
 
 # config.json "architecture" -> config reader, for designs that name themselves that way
-ARCHITECTURES: Dict[str, Callable[[dict], object]] = {"Golulix": GolulixConfig.from_json}
+ARCHITECTURES: Dict[str, Callable[[dict], object]] = {"Golulix": GolulixConfig.from_json,
+                                                       "Faledra": FaledraConfig.from_json}
 
 
 def config_from_json(d: dict):

@@ -1,9 +1,11 @@
 """Decoder-block operators with an fp32 residual stream (``csrc/lm``, ``libshai_lm.so``).
 
-What a layer-list decoder needs beyond the Llama path of :mod:`shai_amd.ops`: an n-gram embedding, a residual-add +
-RMSNorm with the residual kept in fp32, one GEMM for dense and expert-grouped products, mixture-of-experts routing,
-and attention restricted to fixed-size chunks of the sequence with a per-head output gate.  Every op takes bf16 or fp32
-weights and activations; norms, routing, attention scores and the residual are fp32 in both.
+What a layer-list decoder needs beyond the Llama path of :mod:`shai_amd.ops`: an n-gram embedding, residual-add +
+RMSNorm with the residual kept in fp32 (optionally a norm on the added output and a short causal convolution on the
+normed one), one GEMM for dense, per-head and expert-grouped products, mixture-of-experts routing, attention restricted
+to fixed-size chunks of the sequence with a per-head output gate, attention over cached latents with a sink per head, and
+a gated linear recurrence.  Every op takes bf16 or fp32 weights and activations; norms, routing, attention scores,
+rotation angles, recurrent state and the residual are fp32 in both.
 
 Layout rules shared by all of them: the model width is padded to a multiple of 64 (``pad64``; the pad columns of
 activations and weights are zero), so a GEMM's K is always a multiple of 64.
@@ -14,15 +16,21 @@ GPU tensors run the native kernels (raising if the library is missing); CPU tens
 from __future__ import annotations
 
 from dataclasses import dataclass
-from typing import Optional
+from typing import List, NamedTuple, Optional
 
+import numpy as np
 import torch
 
 from .. import native
 from . import lm_reference as ref
 
-EPI_NONE, EPI_CLAMP_GLU, EPI_SOFTCAP = 0, 1, 2
+EPI_NONE, EPI_CLAMP_GLU, EPI_SOFTCAP, EPI_XIELU, EPI_ROTARY = 0, 1, 2, 3, 4
 MAX_EXPERTS, MAX_TOP = 1024, 64
+MAX_TAPS = 16                # convolution taps
+MAX_LATENT = 1024            # columns of a cached latent
+LATENT_SHORT = 16            # portions up to this many rows attend in latent space, longer ones expand keys and values
+LATENT_GROUP_ROWS = 1 << 18  # context rows that are expanded at a time
+SCAN_CHUNK, SCAN_MAX_CHUNKS = 64, 64
 
 
 def pad64(n: int) -> int:
@@ -91,36 +99,52 @@ def add_norm(x, delta, inject, w, eps: float, width: int, dtype, rows=None):
 
 
 def matmul(a, w, out_dtype=None, epi: int = EPI_NONE, param: float = 0.0, plan: Optional[Plan] = None,
-           gather: bool = False):
+           gather: bool = False, vec=None, rope=None, head: int = 0, rot0: int = 0):
     """c = epi(a w^T).  Dense: a [M, K], w [N, K].  Grouped (``plan``): w [E, N, K], row s of c belongs to the expert of
     slot s and reads a[token_of[s]] (``gather``) or a[s].
 
     EPI_CLAMP_GLU: w rows are (gate_i, up_i) pairs; with g = min(gate, param), u = clamp(up, +-param) the N / 2 outputs
-    are g sigmoid(1.702 g) (u + 1).  EPI_SOFTCAP: param * tanh(c / param)."""
+    are g sigmoid(1.702 g) (u + 1).  EPI_SOFTCAP: param * tanh(c / param).  EPI_XIELU: vec[0] c^2 + c / 2 above zero,
+    vec[1] (exp(c) - 1 - c) + c / 2 below.  EPI_ROTARY: columns rot0 .. rot0 + dims - 1 of every ``head`` columns are
+    interleaved pairs turned by the row's angles ``rope`` [M, dims] (:func:`rope_rows`)."""
     out_dtype = out_dtype or a.dtype
     if not a.is_cuda:
-        return ref.matmul(a, w, out_dtype, epi, param, plan, gather)
+        return ref.matmul(a, w, out_dtype, epi, param, plan, gather, vec, rope, head, rot0)
     N = w.shape[-2]
     M = plan.token_of.shape[0] if plan is not None else a.shape[0]
     c = torch.empty(M, N // 2 if epi == EPI_CLAMP_GLU else N, dtype=out_dtype, device=a.device)
     if plan is None:
-        _K().lm_gemm(a, w, c, None, None, None, 0, int(epi), float(param))
+        _K().lm_gemm(a, w, c, None, None, None, 0, int(epi), float(param), None, vec, rope, int(head), int(rot0))
     else:
         _K().lm_gemm(a, w, c, plan.tiles, plan.offsets, plan.token_of if gather else None, plan.bm, int(epi),
                      float(param))
     return c
 
 
-def glu_with_side(a, w, side: int, param: float):
-    """One product for two consumers of ``a``: the rows of w but the last ``side`` are (gate, up) pairs of a clamped GLU
-    (:func:`matmul` EPI_CLAMP_GLU), the last ``side`` rows a plain product in fp32.  Returns (glu, side product)."""
+def matmul_with_side(a, w, side: int, epi: int = EPI_NONE, param: float = 0.0):
+    """One product for two consumers of ``a``: the rows of w but the last ``side`` as in :func:`matmul` (EPI_NONE or
+    EPI_CLAMP_GLU), the last ``side`` rows a plain product in fp32.  Returns (product, side product)."""
     if not a.is_cuda:
-        return ref.matmul(a, w[:-side], a.dtype, EPI_CLAMP_GLU, param), ref.matmul(a, w[-side:], torch.float32, 0, 0.0)
+        return ref.matmul(a, w[:-side], a.dtype, epi, param), ref.matmul(a, w[-side:], torch.float32, 0, 0.0)
     M, N = a.shape[0], w.shape[0]
-    c = torch.empty(M, (N - side) // 2, dtype=a.dtype, device=a.device)
+    c = torch.empty(M, (N - side) // (2 if epi == EPI_CLAMP_GLU else 1), dtype=a.dtype, device=a.device)
     s = torch.empty(M, side, dtype=torch.float32, device=a.device)
-    _K().lm_gemm(a, w, c, None, None, None, 0, EPI_CLAMP_GLU, float(param), s)
+    _K().lm_gemm(a, w, c, None, None, None, 0, int(epi), float(param), s)
     return c, s
+
+
+def glu_with_side(a, w, side: int, param: float):
+    """:func:`matmul_with_side` with a clamped GLU."""
+    return matmul_with_side(a, w, side, EPI_CLAMP_GLU, param)
+
+
+def matmul_heads(a, w):
+    """c[t, h] = a[t, h] w[h]^T: a [T, H, K] and w [H, N, K] (any strides between rows and heads) -> [T, H, N]."""
+    if not a.is_cuda:
+        return torch.einsum("thk,hnk->thn", a.float(), w.float()).to(a.dtype).contiguous()
+    c = torch.empty(a.shape[0], a.shape[1], w.shape[1], dtype=a.dtype, device=a.device)
+    _K().lm_gemm_heads(a, w, c)
+    return c
 
 
 def grouped_bm(rows: int, experts: int) -> int:
@@ -189,3 +213,202 @@ def chunk_attention(qkvg, k_cache, v_cache, batch, heads: int, chunk: int, scale
     _K().chunk_attn_decode(qkvg, k_cache, v_cache, o, batch.block_table, batch.ctx_lens, batch.slots, ws, int(heads),
                            ns, int(chunk), float(scale))
     return o
+
+
+# ---------------------------------------------------------------------------------------------- normed residual, convolution
+class Embedding(NamedTuple):
+    """Residual source of a model's first norm: rows table[ids] * scale."""
+    ids: torch.Tensor
+    table: torch.Tensor
+    scale: float = 1.0
+
+
+@dataclass
+class Conv:
+    """Causal convolution over time on each channel of a norm's output, added to it: weight [taps, D] (fp32, oldest tap
+    first), state [slots, taps - 1, D] (fp32: the last inputs of every sequence).  ``tail`` [B, taps - 1, D] receives a
+    prefill step's last inputs (:func:`conv_commit` moves them into the state); None: a decode step, state updated here."""
+    weight: torch.Tensor
+    state: torch.Tensor
+    tail: Optional[torch.Tensor] = None
+
+
+def residual_norm(source, delta, wb, mult: float, step, w, eps: float, width: int, dtype, conv: Optional[Conv] = None,
+                  batch=None, rows=None, keep: bool = True):
+    """x = source (+ mult * RMSNorm(delta) wb) (+ step); h = RMSNorm(x) w, plus its convolution with ``conv``.
+
+    source: the fp32 residual [T, D] or an :class:`Embedding`.  Returns (x, h); the residual may be updated in place.
+    ``w`` None: no norm (h None).  ``rows`` (int32): h of these rows only, and with ``keep`` False x is None."""
+    emb = isinstance(source, Embedding)
+    if not (source.ids if emb else source).is_cuda:
+        return ref.residual_norm(source, delta, wb, mult, step, w, eps, width, dtype, conv, batch, rows, keep)
+    ids, table, scale = source if emb else (None, None, 1.0)
+    T, D = (ids.shape[0], table.shape[1]) if emb else source.shape
+    dev = ids.device if emb else source.device
+    x = None
+    if keep:
+        x = torch.empty(T, D, dtype=torch.float32, device=dev) if emb or conv is not None else source
+    h = torch.empty(T if rows is None else rows.shape[0], D, dtype=dtype, device=dev) if w is not None else None
+    args = (None if emb else source, ids, table, float(scale), delta, wb, float(mult), step, x, rows, w, float(eps),
+            int(width), h)
+    if conv is None:
+        _K().residual_norm(*args)
+    elif conv.tail is None:
+        _K().residual_norm(*args, conv.weight, conv.state, None, None, None, None, batch.positions, batch.state_slots)
+    else:
+        _K().residual_norm(*args, conv.weight, conv.state, conv.tail, batch.row_seq, batch.q_start, batch.q_lens,
+                           batch.positions, batch.state_slots)
+    return x, h
+
+
+def conv_commit(state, tail, batch) -> None:
+    """The last convolution inputs of a prefill step (tail [runs, B, taps - 1, D]) into state [runs, slots, taps - 1, D]."""
+    if not state.is_cuda:
+        ref.conv_commit(state, tail, batch)
+    else:
+        _K().conv_commit(state, tail, batch.q_lens, batch.state_slots)
+
+
+# ---------------------------------------------------------------------------------------------- rotary angles
+def rope_freq(base: float, dims: int) -> torch.Tensor:
+    """base^(-2 i / dims), i < dims / 2, as (float, remainder) pairs [dims / 2, 2]: angles of far positions keep their
+    32-bit accuracy."""
+    f = np.power(float(base), -2.0 * np.arange(dims // 2) / dims)
+    hi = f.astype(np.float32)
+    return torch.tensor(np.stack([hi, (f - hi).astype(np.float32)], 1))
+
+
+def rope_rows(positions, freq):
+    """(cos, sin) of every row's angles, [T, dims] fp32; computed once per step for all layers that rotate alike."""
+    if not positions.is_cuda:
+        return ref.rope_rows(positions, freq)
+    out = torch.empty(positions.shape[0], 2 * freq.shape[0], dtype=torch.float32, device=positions.device)
+    _K().rope_rows(positions, freq, out)
+    return out
+
+
+# ---------------------------------------------------------------------------------------------- latent attention
+def latent_head_pad(dk: int, dv: int) -> Optional[tuple]:
+    """Head sizes of the prefill kernel that hold (dk, dv), or None."""
+    for k, v in ((64, 64), (128, 64), (128, 128), (192, 128), (256, 256)):
+        if dk <= k and dv <= v:
+            return k, v
+    return None
+
+
+def latent_head_groups(heads: int) -> int:
+    """Workgroups that share a row's heads in a decode step: 16 heads each, 32 from 17 heads on."""
+    return 1 if heads <= 16 else -(-heads // 32)
+
+
+@dataclass
+class LatentGroup:
+    """Sequences of a prefill step whose keys and values are expanded together (device int32 tensors, [n] each)."""
+    seqs: torch.Tensor
+    ctx: torch.Tensor
+    q_lens: torch.Tensor
+    q_start: torch.Tensor
+    kv_start: torch.Tensor
+    rows: int
+    max_ctx: int
+    max_q: int
+
+
+@dataclass
+class LatentPlan:
+    """How a step's rows attend.  ``rows`` (None: all) attend one by one in latent space, as entries of block table row
+    ``seqs`` (None: entry i is sequence i) with ``ctx`` keys; the sequences of ``groups`` run as portions."""
+    n: int
+    rows: Optional[torch.Tensor]
+    seqs: Optional[torch.Tensor]
+    ctx: torch.Tensor
+    splits: int
+    groups: List[LatentGroup]
+
+
+def latent_plan(batch, expand: bool) -> LatentPlan:
+    """``expand``: portions longer than LATENT_SHORT rows run on expanded keys and values."""
+    if not batch.is_prefill:
+        return LatentPlan(batch.input_ids.shape[0], None, None, batch.ctx_lens, max(1, int(batch.num_splits or 1)), [])
+    dev = batch.input_ids.device
+    to = lambda a: torch.from_numpy(np.ascontiguousarray(a, dtype=np.int32)).to(dev, non_blocking=True)
+    q_lens, ctx = (np.asarray(a, dtype=np.int64) for a in (batch.q_lens_host, batch.ctx_lens_host))
+    start = np.concatenate([[0], np.cumsum(q_lens)])[:-1]
+    long = (q_lens > LATENT_SHORT) & expand
+    groups, at = [], 0
+    ids = np.nonzero(long)[0]
+    while at < len(ids):
+        n = max(1, int(np.searchsorted(np.cumsum(ctx[ids[at:]]), LATENT_GROUP_ROWS, side="right")))
+        g = ids[at:at + n]
+        at += n
+        pack = to(np.stack([g, ctx[g], q_lens[g], start[g], np.cumsum(ctx[g]) - ctx[g]]))
+        groups.append(LatentGroup(*pack.unbind(0), rows=int(ctx[g].sum()), max_ctx=int(ctx[g].max()),
+                                  max_q=int(q_lens[g].max())))
+    seq = np.repeat(np.arange(len(q_lens)), q_lens)
+    pos = np.arange(len(seq)) - start[seq] + (ctx - q_lens)[seq]
+    rows = np.nonzero(~long[seq])[0]
+    pack = to(np.stack([rows, seq[rows], pos[rows] + 1]))
+    splits = 1
+    if len(rows):
+        from . import decode_splits
+        splits = decode_splits(len(rows), 1, int(pos[rows].max()) + 1)
+    return LatentPlan(len(rows), pack[0] if groups else None, pack[1], pack[2], splits, groups)
+
+
+def latent_prep(d, wq, wkv, rope, batch, cache, eps: float, q_rank: int, kv_rank: int):
+    """The down projection's fp32 rows [q latent | kv latent | rotated key part] (each padded): norms both latents, turns
+    the key part, writes [kv latent | key part] to ``cache`` [blocks, 64, ..] at batch.slots.  Returns the normed q latent
+    in the cache's dtype."""
+    if not d.is_cuda:
+        return ref.latent_prep(d, wq, wkv, rope, batch, cache, eps, q_rank, kv_rank)
+    cq = torch.empty(d.shape[0], wq.shape[0], dtype=cache.dtype, device=d.device)
+    _K().latent_prep(d, wq, wkv, rope, batch.slots, cache, cq, float(eps), int(q_rank), int(kv_rank))
+    return cq
+
+
+def latent_rows(ql, q, cache, block_table, plan: LatentPlan, sink, np_: int, rot: int, scale: float):
+    """Softmax over the cached rows j < ctx of every entry, with exp(sink) in the denominator.  ql [n, H, rank]: queries
+    in latent space; the rotated part of head h is q[:, h, np_ : np_ + rot] (q [n, H * head]).  -> [n, H, rank]."""
+    if not q.is_cuda:
+        return ref.latent_rows(ql, q, cache, block_table, plan, sink, np_, rot, scale)
+    n, H, rp = ql.shape
+    o = torch.empty_like(ql)
+    ns = plan.splits
+    ws = torch.empty(n * H * ns * (rp + 4) if ns > 1 else 0, dtype=torch.float32, device=q.device)
+    _K().latent_attn_rows(ql, q, cache, o, block_table, plan.seqs, plan.ctx, sink, ws, ns, int(np_), int(rot), float(scale))
+    return o
+
+
+def latent_gather(cache, block_table, g: LatentGroup):
+    """The cached rows of a group's sequences back to back, [g.rows, ..]."""
+    if not cache.is_cuda:
+        return ref.latent_gather(cache, block_table, g)
+    out = torch.empty(g.rows, cache.shape[2], dtype=cache.dtype, device=cache.device)
+    _K().latent_gather(cache, block_table, g.seqs, g.ctx, g.kv_start, g.max_ctx, out)
+    return out
+
+
+def latent_prefill(q, kv, lat, o, g: LatentGroup, sink, heads: int, np_: int, rot: int, rank: int, scale: float) -> None:
+    """Causal attention of a group's portions: key j of head h is [kv[j, h, :np_] | lat[j, rank : rank + rot]], its value
+    kv[j, h, np_:]; writes the portions' rows of ``o`` [T, H dv]."""
+    if not q.is_cuda:
+        ref.latent_prefill(q, kv, lat, o, g, sink, heads, np_, rot, rank, scale)
+        return
+    _K().latent_attn_prefill(q, kv, lat, o, g.ctx, g.q_lens, g.q_start, g.kv_start, sink, g.max_q, int(heads), int(np_),
+                             int(rot), int(rank), float(scale))
+
+
+# ---------------------------------------------------------------------------------------------- gated recurrence
+def mingru_scan(zx, g, bias, state, batch):
+    """S_t = (1 - z) S_(t-1) + z c per channel and sequence, z = sigmoid(zx[:, :W] + bias), c = u + 1/2 (u >= 0) or
+    sigmoid(u), u = zx[:, W:] + bias; returns S silu(g).  ``state`` [slots, W] carries S (fp32); a sequence's first token
+    starts from zero."""
+    if not g.is_cuda:
+        return ref.mingru_scan(zx, g, bias, state, batch)
+    out = torch.empty_like(g)
+    max_q = int(batch.S) if batch.is_prefill else 1
+    n = -(-max_q // (SCAN_CHUNK * SCAN_MAX_CHUNKS)) * SCAN_CHUNK
+    chunks = -(-max_q // n)
+    ws = torch.empty(batch.B * chunks * 2 * g.shape[1] if chunks > 1 else 0, dtype=torch.float32, device=g.device)
+    _K().mingru_scan(zx, g, bias, state, out, batch.positions, batch.q_start, batch.q_lens, batch.state_slots, ws, max_q, n)
+    return out

@@ -35,20 +35,32 @@ def add_norm(x, delta, inject, w, eps, width, dtype, rows=None):
     return _norm(y, w, eps, width).to(dtype)
 
 
-def _epilogue(c, epi, param):
-    from .lm import EPI_CLAMP_GLU, EPI_SOFTCAP
+def _epilogue(c, epi, param, vec=None, rope=None, head=0, rot0=0):
+    from .lm import EPI_CLAMP_GLU, EPI_ROTARY, EPI_SOFTCAP, EPI_XIELU
     if epi == EPI_CLAMP_GLU:
         g = c[..., 0::2].clamp(max=param)
         u = c[..., 1::2].clamp(-param, param)
         return g * torch.sigmoid(1.702 * g) * (u + 1.0)
     if epi == EPI_SOFTCAP:
         return param * torch.tanh(c / param)
+    if epi == EPI_XIELU:
+        return torch.where(c > 0, vec[0] * c * c, vec[1] * (torch.expm1(c) - c)) + 0.5 * c
+    if epi == EPI_ROTARY:
+        c = c.view(c.shape[0], -1, head).clone()
+        rot = rope.shape[1]
+        c[..., rot0:rot0 + rot] = _turn(c[..., rot0:rot0 + rot], rope[:, None, :])
+        return c.view(c.shape[0], -1)
     return c
 
 
-def matmul(a, w, out_dtype, epi, param, plan=None, gather=False):
+def _turn(x, rope):
+    u, v, cs, sn = x[..., 0::2], x[..., 1::2], rope[..., 0::2], rope[..., 1::2]
+    return torch.stack([u * cs - v * sn, v * cs + u * sn], -1).flatten(-2)
+
+
+def matmul(a, w, out_dtype, epi, param, plan=None, gather=False, vec=None, rope=None, head=0, rot0=0):
     if plan is None:
-        return _epilogue(a.float() @ w.float().T, epi, param).to(out_dtype)
+        return _epilogue(a.float() @ w.float().T, epi, param, vec, rope, head, rot0).to(out_dtype)
     rows = a[plan.token_of.long()] if gather else a
     off = plan.offsets.tolist()
     parts = [_epilogue(rows[off[e]:off[e + 1]].float() @ w[e].float().T, epi, param)
@@ -99,3 +111,114 @@ def chunk_attention(qkvg, k_cache, v_cache, batch, heads, chunk, scale):
             s = torch.einsum("hd,nhd->hn", q[row0 + i].float().view(heads, dk), kk) * scale
             o[row0 + i] = torch.einsum("hn,nhd->hd", torch.softmax(s, -1), vv)
     return (o * torch.sigmoid(gate.float())[..., None]).reshape(T, heads * dv).to(qkvg.dtype)
+
+
+def _sequences(batch):
+    """(first row, rows, first position, state slot, sequence) of every sequence of a step."""
+    for b in range(batch.B):
+        row0 = int(batch.q_start[b]) if batch.is_prefill else b
+        n = int(batch.q_lens[b]) if batch.is_prefill else 1
+        yield row0, n, int(batch.positions[row0]), int(batch.state_slots[b]), b
+
+
+def residual_norm(source, delta, wb, mult, step, w, eps, width, dtype, conv, batch, rows, keep):
+    from .lm import Embedding
+    rms = lambda t, gain: t / torch.sqrt(t.pow(2).sum(-1, keepdim=True) / width + eps) * gain
+    x = source.table[source.ids.long()].float() * source.scale if isinstance(source, Embedding) else source.clone()
+    if delta is not None:
+        x = x + mult * rms(delta.float(), wb)
+    if step is not None:
+        x = x + step
+    if w is None:
+        return x, None
+    if rows is not None:
+        return (x if keep else None), rms(x[rows.long()], w).to(dtype)
+    h = rms(x, w)
+    if conv is not None:
+        y, k = h.clone(), conv.weight.shape[0] - 1
+        for row0, n, pos, slot, b in _sequences(batch):
+            past = conv.state[slot] if slot >= 0 else torch.zeros(k, h.shape[1])
+            past = past * (torch.arange(k) >= k - pos)[:, None] if pos < k else past
+            line = torch.cat([past, h[row0:row0 + n]])
+            for j in range(k + 1):
+                y[row0:row0 + n] += conv.weight[j] * line[j:j + n]
+            if conv.tail is not None:
+                conv.tail[b, k - min(n, k):] = line[n + k - min(n, k):]
+            elif slot >= 0:
+                conv.state[slot] = line[n:]
+        h = y
+    return x, h.to(dtype)
+
+
+def conv_commit(state, tail, batch):
+    k = state.shape[2]
+    for _, n, _, slot, b in _sequences(batch):
+        if slot >= 0:
+            state[:, slot] = torch.cat([state[:, slot], tail[:, b, k - min(n, k):]], 1)[:, -k:] if k else state[:, slot]
+
+
+def rope_rows(positions, freq):
+    a = positions.double()[:, None] * freq.double().sum(1)
+    return torch.stack([a.cos(), a.sin()], -1).flatten(1).float()
+
+
+def latent_prep(d, wq, wkv, rope, batch, cache, eps, q_rank, kv_rank):
+    qp, rp = wq.shape[0], wkv.shape[0]
+    rms = lambda t, n, gain: t / torch.sqrt(t.pow(2).sum(-1, keepdim=True) / n + eps) * gain
+    turn = d[:, qp + rp:].clone()
+    turn[:, :rope.shape[1]] = _turn(turn[:, :rope.shape[1]], rope)
+    row = torch.cat([rms(d[:, qp:qp + rp], kv_rank, wkv), turn], 1).to(cache.dtype)
+    for t, slot in enumerate(batch.slots[:d.shape[0]].tolist()):
+        if slot >= 0:
+            cache[slot // 64, slot % 64] = row[t]
+    return rms(d[:, :qp], q_rank, wq).to(cache.dtype)
+
+
+def _sink_softmax(s, sink):
+    return torch.softmax(torch.cat([s, sink[:, None]], 1), 1)[:, :-1]
+
+
+def latent_rows(ql, q, cache, block_table, plan, sink, np_, rot, scale):
+    n, H, rp = ql.shape
+    qr = q.view(n, H, -1)[..., np_:np_ + rot].float()
+    o = torch.zeros(n, H, rp)
+    for i, ctx in enumerate(plan.ctx[:n].tolist()):
+        key = torch.arange(ctx)
+        bt = block_table[int(plan.seqs[i]) if plan.seqs is not None else i].long()
+        row = cache[bt[key // 64], key % 64].float()
+        s = (ql[i].float() @ row[:, :rp].T + qr[i] @ row[:, rp:rp + rot].T) * scale
+        o[i] = _sink_softmax(s, sink) @ row[:, :rp]
+    return o.to(ql.dtype)
+
+
+def latent_gather(cache, block_table, g):
+    key = lambda n: torch.arange(n)
+    return torch.cat([cache[block_table[b].long()[key(n) // 64], key(n) % 64]
+                      for b, n in zip(g.seqs.tolist(), g.ctx.tolist())])
+
+
+def latent_prefill(q, kv, lat, o, g, sink, heads, np_, rot, rank, scale):
+    ov = o.view(o.shape[0], heads, -1)
+    for ctx, n, row0, k0 in zip(*(t.tolist() for t in (g.ctx, g.q_lens, g.q_start, g.kv_start))):
+        qs = q[row0:row0 + n].view(n, heads, -1).float()
+        kvs = kv[k0:k0 + ctx].view(ctx, heads, -1).float()
+        turn = lat[k0:k0 + ctx, rank:rank + rot].float()
+        hide = torch.arange(ctx)[None, :] > torch.arange(ctx - n, ctx)[:, None]
+        for h in range(heads):
+            s = qs[:, h, :np_] @ kvs[:, h, :np_].T + qs[:, h, np_:np_ + rot] @ turn.T
+            p = _sink_softmax((s * scale).masked_fill(hide, float("-inf")), sink[h].expand(n))
+            ov[row0:row0 + n, h] = (p @ kvs[:, h, np_:]).to(o.dtype)
+
+
+def mingru_scan(zx, g, bias, state, batch):
+    z, u = (zx + bias).chunk(2, 1)
+    keep, cand = torch.sigmoid(-z), torch.where(u >= 0, u + 0.5, torch.sigmoid(u))
+    add, S = torch.sigmoid(z) * cand, torch.zeros_like(z)
+    for row0, n, pos, slot, _ in _sequences(batch):
+        s = state[slot].clone() if slot >= 0 and pos > 0 else torch.zeros_like(z[0])
+        for t in range(row0, row0 + n):
+            s = keep[t] * s + add[t]
+            S[t] = s
+        if slot >= 0:
+            state[slot] = s
+    return (S * torch.nn.functional.silu(g.float())).to(g.dtype)

@@ -106,6 +106,25 @@ class BlockManager:
         return {"prefix_hits": int(a[0]), "prefix_queries": int(a[1]), "free": int(a[2]), "cached_free": int(a[3])}
 
 
+class SlotPool:
+    """Slots of per-sequence state; the one freed last is handed out first."""
+
+    def __init__(self, n: int):
+        self._free = list(range(n))[::-1]
+
+    @property
+    def num_free(self) -> int:
+        return len(self._free)
+
+    def allocate(self) -> int:
+        if not self._free:
+            raise MemoryError("out of sequence state slots")
+        return self._free.pop()
+
+    def release(self, slot: int) -> None:
+        self._free.append(slot)
+
+
 def sched_admit(prompt_tokens: Sequence[int], free_blocks: int, running: int, max_seqs: int, token_budget: int,
                 watermark_blocks: int) -> int:
     if not prompt_tokens:

@@ -49,7 +49,8 @@ def load_into(model: nn.Module, sd: Dict[str, torch.Tensor], convert: Optional[C
     if convert is not None:
         sd = convert(sd)
     dtype = next(model.parameters()).dtype
-    sd = {k: (v.to(dtype) if v.is_floating_point() else v) for k, v in sd.items()}
+    own = {k: p.dtype for k, p in model.named_parameters()}   # some blocks keep small fp32 tensors in a bf16 model
+    sd = {k: (v.to(own.get(k, dtype)) if v.is_floating_point() else v) for k, v in sd.items()}
     missing, unexpected = model.load_state_dict(sd, strict=False)
     if strict and (missing or unexpected):
         raise RuntimeError(f"checkpoint mismatch: missing={missing[:10]} unexpected={unexpected[:10]}")
