@@ -1,11 +1,12 @@
-"""Prefill and decode throughput of the Golulix design beside a Llama-family model of equal size.
+"""Prefill and decode throughput of a layer-list design (Golulix, Faledra) beside a Llama-family model of equal size.
 
 Both run through :class:`LLMEngine` (scheduler, paged cache, HIP-graph decode) with random weights.  A pair has the same
-width, layers, heads, head size and vocabulary, and the Llama MLP is as wide as the feed-forward work one Golulix token
-does (top x expert + shared expert), so the two do the same matrix work per token.
+width, layers, heads and vocabulary.  The Llama MLP is as wide as the feed-forward work one Golulix token does (top x
+expert + shared expert), or has as many weights as the Faledra feed-forward (3 D I = 2 D ff), so the two do the same
+matrix work per token there.
 
-    python bench.py --workload golulix [--golulix-size small|large|both]
-    python -m shai_amd.bench.decoder_design --model golulix --size small --phase decode --batch 64   # profiling
+    python bench.py --workload golulix|faledra [--design-size small|large|both]
+    python -m shai_amd.bench.decoder_design --design faledra --model faledra --size small --batch 64      # profiling
 """
 from __future__ import annotations
 
@@ -15,17 +16,27 @@ import time
 # width, layers, heads, kv heads, head size, chunk, experts, top, expert ff, shared ff, vocab, expert groups, kept
 SIZES = {"small": (2048, 8, 16, 4, 128, 2048, 64, 6, 1408, 2816, 32768, 8, 4),
          "large": (4096, 6, 32, 8, 128, 8192, 64, 4, 2048, 4096, 65536, 4, 2)}
+# width, attention layers, minGRU layers, heads, unrotated / rotated / value head size, query latent, key-value latent,
+# minGRU width, ff, vocab, kv heads of the Llama model (head size: the unrotated one)
+FALEDRA_SIZES = {"small": (2048, 6, 2, 16, 128, 64, 128, 768, 512, 2048, 8448, 32768, 4),
+                 "large": (4096, 4, 2, 32, 128, 64, 128, 1536, 512, 4096, 16896, 65536, 8)}
 
 
-def configs(size: str):
-    from ..models.golulix import GolulixConfig
+def configs(size: str, design: str = "golulix"):
     from ..models.llama import LlamaConfig
-    D, L, H, G, d, chunk, E, top, ff, sff, V, groups, keep = SIZES[size]
-    gol = GolulixConfig.uniform(layers=L, width=D, heads=H, kv_heads=G, dim=d, chunk=chunk, experts=E, top=top, ff=ff,
-                                shared_ff=sff, vocab=V, groups=groups, keep=keep)
-    ll = LlamaConfig(vocab_size=V, hidden_size=D, intermediate_size=top * ff + sff, num_hidden_layers=L,
-                     num_attention_heads=H, num_key_value_heads=G, head_dim=d, max_position_embeddings=32768)
-    return {"golulix": gol, "llama": ll}
+    if design == "faledra":
+        from ..models.faledra import FaledraConfig
+        D, A, R, H, d, rot, dv, q, kv, gru, ff, V, G = FALEDRA_SIZES[size]
+        cfg, L, inner = FaledraConfig.uniform(A, R, D, H, d, rot, dv, q, kv, gru, ff, V), A + R, 2 * ff // 3
+    else:
+        from ..models.golulix import GolulixConfig
+        D, L, H, G, d, chunk, E, top, ff, sff, V, groups, keep = SIZES[size]
+        cfg = GolulixConfig.uniform(layers=L, width=D, heads=H, kv_heads=G, dim=d, chunk=chunk, experts=E, top=top, ff=ff,
+                                    shared_ff=sff, vocab=V, groups=groups, keep=keep)
+        inner = top * ff + sff
+    ll = LlamaConfig(vocab_size=V, hidden_size=D, intermediate_size=inner, num_hidden_layers=L, num_attention_heads=H,
+                     num_key_value_heads=G, head_dim=d, max_position_embeddings=32768)
+    return {design: cfg, "llama": ll}
 
 
 def measure(cfg, batch: int, prompt: int, gen: int, repeats: int = 3, device: str = "cuda:0") -> dict:
@@ -62,42 +73,51 @@ def measure(cfg, batch: int, prompt: int, gen: int, repeats: int = 3, device: st
 
 
 def bench(args, rank: int, world: int) -> dict:
-    """The bench.py line: every (size, batch) pair of both models; ``value`` is Golulix decode at the largest batch."""
+    """The bench.py line: every (size, batch) pair of both models; ``value`` is the design's decode at the largest batch."""
     import torch
+    design = args.workload
     if world != 1:
-        raise SystemExit("--workload golulix runs on one GPU")
-    sizes = list(SIZES) if args.golulix_size == "both" else [args.golulix_size]
+        raise SystemExit(f"--workload {design} runs on one GPU")
+    sizes = list(SIZES) if args.design_size == "both" else [args.design_size]
     rows, P, G, t0 = [], 1024, 64, time.perf_counter()
     steps = max(1, args.steps)
     for size in sizes:
-        cfgs = configs(size)
+        cfgs = configs(size, design)
         for batch in (1, 8, args.batch):
             row = {"size": size, "batch": batch, "prompt_len": P, "gen_len": G}
             for name, cfg in cfgs.items():
                 row[name] = measure(cfg, batch, P, G, steps, f"cuda:{torch.cuda.current_device()}")
             rows.append(row)
     last = rows[-1]
-    return {"metric": "Golulix decode tokens/s (random weights, beside a Llama model of equal size)",
-            "value": last["golulix"]["decode_tok_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": 1,
+    model = {"golulix": lambda n: f"Golulix {n}: (width, layers, heads, kv heads, head size, chunk, experts, top, expert "
+                                  f"ff, shared ff, vocab, groups, kept) = {SIZES[n]}",
+             "faledra": lambda n: f"Faledra {n}: (width, attention layers, minGRU layers, heads, unrotated / rotated / value "
+                                  f"head size, query latent, key-value latent, minGRU width, ff, vocab) = "
+                                  f"{FALEDRA_SIZES[n][:-1]}"}[design](last["size"])
+    return {"metric": f"{design.capitalize()} decode tokens/s (random weights, beside a Llama model of equal size)",
+            "value": last[design]["decode_tok_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": 1,
             "ms_per_step": round(1000 * (time.perf_counter() - t0) / (len(rows) * 2 * (steps + 1)), 2),
             "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16",
             "data": "synthetic prompts, random-init weights",
-            "config": {"model": f"Golulix {last['size']}: (width, layers, heads, kv heads, head size, chunk, experts, "
-                                f"top, expert ff, shared ff, vocab, groups, kept) = {SIZES[last['size']]}",
-                       "global_batch": last["batch"], "seq_len": P + G, "parallelism": "dp1"},
+            "config": {"model": model, "global_batch": last["batch"], "seq_len": P + G, "parallelism": "dp1"},
             "pairs": rows}
 
 
 def main(argv=None):
     ap = argparse.ArgumentParser()
-    ap.add_argument("--model", choices=["golulix", "llama"], default="golulix")
+    ap.add_argument("--design", choices=["golulix", "faledra"], default="golulix")
+    ap.add_argument("--model", choices=["design", "golulix", "faledra", "llama"], default="design")
     ap.add_argument("--size", choices=sorted(SIZES), default="small")
     ap.add_argument("--batch", type=int, default=64)
     ap.add_argument("--prompt", type=int, default=1024)
     ap.add_argument("--gen", type=int, default=64)
     ap.add_argument("--repeats", type=int, default=2)
     a = ap.parse_args(argv)
-    print(measure(configs(a.size)[a.model], a.batch, a.prompt, a.gen, a.repeats), flush=True)
+    cfgs = configs(a.size, a.design)
+    name = a.design if a.model == "design" else a.model
+    if name not in cfgs:
+        ap.error(f"--model {a.model} is not part of --design {a.design}")
+    print(measure(cfgs[name], a.batch, a.prompt, a.gen, a.repeats), flush=True)
 
 
 if __name__ == "__main__":

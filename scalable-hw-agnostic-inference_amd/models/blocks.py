@@ -327,13 +327,18 @@ class LatentAttention(nn.Module):
 
     def forward(self, h, batch, cache, step):
         """``step``: the step's shared work (:class:`StepShared`)."""
-        c, H = self.c, self.c.heads
+        c = self.c
         rope, plan = step.rope(self), step.plan(self.expands)
         down = lm.matmul(h, self.down, torch.float32)
         cq = lm.latent_prep(down, self.q_norm, self.kv_norm, rope, batch, cache, self.eps, c.q_rank, c.kv_rank)
         q = lm.matmul(cq, self.uq, epi=lm.EPI_ROTARY, rope=rope, head=self.dk, rot0=self.np)
+        return lm.matmul(self.attend(q, batch, cache, plan), self.o)
+
+    def attend(self, q, batch, cache, plan):
+        """q [T, H dk], turned, over the cached latents (this step's included) -> [T, H dv]."""
+        c, H = self.c, self.c.heads
         if not plan.groups:
-            return lm.matmul(self._in_latent_space(q, batch, cache, plan), self.o)
+            return self._in_latent_space(q, batch, cache, plan)
         o = torch.empty(q.shape[0], H * self.dv, dtype=q.dtype, device=q.device)
         for g in plan.groups:
             lat = lm.latent_gather(cache, batch.block_table, g)
@@ -342,7 +347,7 @@ class LatentAttention(nn.Module):
         if plan.n:
             rows = plan.rows
             o.index_copy_(0, rows.long(), self._in_latent_space(q.index_select(0, rows), batch, cache, plan))
-        return lm.matmul(o, self.o)
+        return o
 
     def _in_latent_space(self, q, batch, cache, plan):
         c, n = self.c, q.shape[0]
