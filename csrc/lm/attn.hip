@@ -111,13 +111,13 @@ __device__ __forceinline__ int v_swz(int row, int ch) {
 }
 
 template <int DK, int DV, bool LAT>
-__global__ void __launch_bounds__(256, DK + DV > 256 ? 1 : 2) attn_prefill_kernel(const AttnArgs p) {
+__global__ void __launch_bounds__(256, DK + DV > (LAT ? 320 : 256) ? 1 : 2) attn_prefill_kernel(const AttnArgs p) {
   constexpr int KT = 64, CK = DK / 8, CV = DV / 8, NK = KT * CK / 256, NV = KT * CV / 256;
   constexpr int NS = DK / 16, ND = DV / 32;
   extern __shared__ __attribute__((aligned(16))) bf16_t smem[];
   bf16_t* sK = smem;
   bf16_t* sV = smem + 2 * KT * DK;
-  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+  const int tid = threadIdx.x, lane = tid & 63, wid = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int fr = lane & 31, fh = lane >> 5;
   const int b = blockIdx.z, h = blockIdx.y;
   const int hk = h / (p.H / p.G);
@@ -140,54 +140,59 @@ __global__ void __launch_bounds__(256, DK + DV > 256 ? 1 : 2) attn_prefill_kerne
   const int t0 = LAT ? 0 : (p_first - p_first % p.chunk) >> 6, t1 = (p_last >> 6) + 1;
   const int lo_last = LAT ? 0 : p_last - p_last % p.chunk;
 
-  uint4_ rk[NK], rv[NV];
-  auto load_tile = [&](int t) {
+  // LAT: keys and values go to LDS by DMA, the bank swizzle applied to the source.  Rows past the context repeat the last
+  // one (their scores are masked); columns past a key's parts hold other finite values (the queries are zero there).
+  auto stage_tile = [&](int t, int st) {
     if constexpr (LAT) {
-      const int left = ctx - t * KT, ld = p.np + DV;
-      const long key = p.kv_start[b] + t * KT;
-      const bf16_t* kv = static_cast<const bf16_t*>(p.kv) + (key * p.H + h) * ld;
-      const bf16_t* lat = static_cast<const bf16_t*>(p.lat) + key * p.lat_ld + p.rank;
+      const int ld = p.np + DV;
+      const bf16_t* kv = static_cast<const bf16_t*>(p.kv) + ((long)p.kv_start[b] * p.H + h) * ld;
+      const bf16_t* lat = static_cast<const bf16_t*>(p.lat) + (long)p.kv_start[b] * p.lat_ld + p.rank;
 #pragma unroll
       for (int i = 0; i < NK; ++i) {
-        const int id = tid + 256 * i, r = id / CK, col = (id % CK) * 8;
-        rk[i] = uint4_{0u, 0u, 0u, 0u};
-        if (r < left && col < p.np + p.rot)
-          rk[i] = *reinterpret_cast<const uint4_*>(col < p.np ? kv + (long)r * p.H * ld + col
-                                                              : lat + (long)r * p.lat_ld + col - p.np);
+        const int id = tid + 256 * i, r = id / CK, col = k_swz<DK>(r, id % CK) - r * DK;
+        const long row = min(t * KT + r, ctx - 1);
+        const bf16_t* src = col < p.np ? kv + row * p.H * ld + col : lat + row * p.lat_ld + min(col - p.np, p.lat_pad);
+        dma16(src, sK + st * KT * DK + (256 * i + 64 * wid) * 8);
       }
 #pragma unroll
       for (int i = 0; i < NV; ++i) {
-        const int id = tid + 256 * i, r = id / CV;
-        rv[i] = r < left ? *reinterpret_cast<const uint4_*>(kv + (long)r * p.H * ld + p.np + (id % CV) * 8)
-                         : uint4_{0u, 0u, 0u, 0u};
+        const int id = tid + 256 * i, r = id / CV, col = v_swz<DV>(r, id % CV) - r * DV;
+        const bf16_t* src = kv + (long)min(t * KT + r, ctx - 1) * p.H * ld + p.np + col;
+        dma16(src, sV + st * KT * DV + (256 * i + 64 * wid) * 8);
       }
-      return;
     }
-    const long cell = ((long)p.bt[(long)b * p.max_blocks + t] * p.G + hk) * 64;
-    const bf16_t* kb = static_cast<const bf16_t*>(p.kc) + cell * DK;
-    const bf16_t* vb = static_cast<const bf16_t*>(p.vc) + cell * DV;
-    const int left = ctx - t * KT;               // rows of this block that hold keys of the sequence
+  };
+  uint4_ rk[LAT ? 1 : NK], rv[LAT ? 1 : NV];
+  auto load_tile = [&](int t) {
+    if constexpr (!LAT) {
+      const long cell = ((long)p.bt[(long)b * p.max_blocks + t] * p.G + hk) * 64;
+      const bf16_t* kb = static_cast<const bf16_t*>(p.kc) + cell * DK;
+      const bf16_t* vb = static_cast<const bf16_t*>(p.vc) + cell * DV;
+      const int left = ctx - t * KT;               // rows of this block that hold keys of the sequence
 #pragma unroll
-    for (int i = 0; i < NK; ++i) {
-      const int id = tid + 256 * i;
-      rk[i] = id / CK < left ? *reinterpret_cast<const uint4_*>(kb + (long)id * 8) : uint4_{0u, 0u, 0u, 0u};
-    }
+      for (int i = 0; i < NK; ++i) {
+        const int id = tid + 256 * i;
+        rk[i] = id / CK < left ? *reinterpret_cast<const uint4_*>(kb + (long)id * 8) : uint4_{0u, 0u, 0u, 0u};
+      }
 #pragma unroll
-    for (int i = 0; i < NV; ++i) {
-      const int id = tid + 256 * i;
-      rv[i] = id / CV < left ? *reinterpret_cast<const uint4_*>(vb + (long)id * 8) : uint4_{0u, 0u, 0u, 0u};
+      for (int i = 0; i < NV; ++i) {
+        const int id = tid + 256 * i;
+        rv[i] = id / CV < left ? *reinterpret_cast<const uint4_*>(vb + (long)id * 8) : uint4_{0u, 0u, 0u, 0u};
+      }
     }
   };
   auto store_tile = [&](int st) {
+    if constexpr (!LAT) {
 #pragma unroll
-    for (int i = 0; i < NK; ++i) {
-      const int id = tid + 256 * i;
-      *reinterpret_cast<uint4_*>(sK + st * KT * DK + k_swz<DK>(id / CK, id % CK)) = rk[i];
-    }
+      for (int i = 0; i < NK; ++i) {
+        const int id = tid + 256 * i;
+        *reinterpret_cast<uint4_*>(sK + st * KT * DK + k_swz<DK>(id / CK, id % CK)) = rk[i];
+      }
 #pragma unroll
-    for (int i = 0; i < NV; ++i) {
-      const int id = tid + 256 * i;
-      *reinterpret_cast<uint4_*>(sV + st * KT * DV + v_swz<DV>(id / CV, id % CV)) = rv[i];
+      for (int i = 0; i < NV; ++i) {
+        const int id = tid + 256 * i;
+        *reinterpret_cast<uint4_*>(sV + st * KT * DV + v_swz<DV>(id / CV, id % CV)) = rv[i];
+      }
     }
   };
 
@@ -200,12 +205,20 @@ __global__ void __launch_bounds__(256, DK + DV > 256 ? 1 : 2) attn_prefill_kerne
   const float sl2 = p.scale * kLog2e;
   const int g16 = lane >> 4, i16 = lane & 15, tq = i16 >> 2, tp = i16 & 3;
 
-  load_tile(t0);
-  store_tile(0);
+  if constexpr (LAT) {
+    stage_tile(t0, 0);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  } else {
+    load_tile(t0);
+    store_tile(0);
+  }
   __syncthreads();
   for (int t = t0; t < t1; ++t) {
     const int cur = (t - t0) & 1;
-    if (t + 1 < t1) load_tile(t + 1);
+    if (t + 1 < t1) {
+      if constexpr (LAT) stage_tile(t + 1, cur ^ 1);
+      else load_tile(t + 1);
+    }
     const bf16_t* ks = sK + cur * KT * DK;
     const bf16_t* vs = sV + cur * KT * DV;
     float16_ sacc[2];
@@ -296,7 +309,8 @@ __global__ void __launch_bounds__(256, DK + DV > 256 ? 1 : 2) attn_prefill_kerne
         }
       }
     }
-    if (t + 1 < t1) store_tile(cur ^ 1);
+    if constexpr (LAT) asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    else if (t + 1 < t1) store_tile(cur ^ 1);
     __syncthreads();
   }
   const float l_tot = l_run + __shfl_xor(l_run, 32, 64);

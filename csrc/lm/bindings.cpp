@@ -204,11 +204,24 @@ void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<T
     SHAI_CHECK(W.dim() == 2 && g.a_rows == g.M, "dense lm_gemm: W [N, K], A [M, K]");
   }
   if (g.M == 0) return;
-  const long lim = 0x7fffffffL;
-  const bool tile = !f32 && (g.tiles ? bm >= 128 : g.M > 64) && (long)g.a_rows * g.lda * 2 < lim &&
-                    (long)g.N * g.K * 2 < lim;
-  if (tile) shai_lm::launch_gemm_tile(g, stream());
-  else shai_lm::launch_gemm(g, f32, stream());
+  const long lim = 0x7fffffffL, esize = f32 ? 4 : 2, osize = g.out_f32 ? 4 : 2;
+  const bool tile = !f32 && (g.tiles ? bm >= 128 && (long)g.a_rows * g.lda * 2 < lim : g.M > 64) && (long)g.N * g.K * 2 < lim;
+  if (!tile) return shai_lm::launch_gemm(g, f32, stream());
+  // the tiled kernel addresses A with 32-bit offsets: a longer A runs in parts
+  const int rows = g.tiles ? g.M : (int)std::min<long>(g.M, std::max<long>(256, (lim / (g.lda * 2)) / 256 * 256));
+  SHAI_CHECK(g.tiles || (long)rows * g.lda * 2 < lim, "lm_gemm: rows of A are too long");
+  const int total = g.M;
+  for (int at = 0; at < total; at += rows) {
+    shai_lm::GemmArgs part = g;
+    if (!g.tiles) {
+      part.M = part.a_rows = std::min(rows, total - at);
+      part.A = static_cast<const char*>(g.A) + at * g.lda * esize;
+      part.C = static_cast<char*>(g.C) + at * g.ldc * osize;
+      if (g.side) part.side = g.side + (long)at * (g.N - g.n_main);
+      if (g.rope) part.rope = g.rope + (long)at * g.rot;
+    }
+    shai_lm::launch_gemm_tile(part, stream());
+  }
 }
 
 // c[t, h] = a[t, h] w[h]^T for every head h: a [T, H, K], w [H, N, K], c [T, H, N], any strides between rows and heads
@@ -447,10 +460,11 @@ void latent_attn_prefill(const Tensor& q, const Tensor& kv, const Tensor& lat, c
   SHAI_CHECK((a.dk == 64 && a.dv == 64) || (a.dk == 128 && (a.dv == 64 || a.dv == 128)) || (a.dk == 192 && a.dv == 128) ||
                  (a.dk == 256 && a.dv == 256), "latent prefill head sizes: 64/64, 128/64, 128/128, 192/128 or 256/256");
   a.np = np;
-  a.rot = (rot + 7) / 8 * 8;
+  const int rp8 = (rot + 7) / 8 * 8;
   a.rank = rank;
   a.lat_ld = lat.size(1);
-  SHAI_CHECK(np >= 0 && np % 8 == 0 && np + a.rot <= a.dk && rank % 8 == 0 && rank + a.rot <= a.lat_ld && a.lat_ld % 8 == 0 &&
+  a.lat_pad = a.lat_ld - a.rank - 8;   // the queries are zero past the rotated part: any finite value will do there
+  SHAI_CHECK(np >= 0 && np % 8 == 0 && np + rp8 <= a.dk && rank % 8 == 0 && rank + rp8 <= a.lat_ld && a.lat_ld % 8 == 0 &&
                  kv.size(1) == heads * (np + a.dv) && kv.size(0) == lat.size(0), "latent prefill: kv [rows, H (np + dv)]");
   SHAI_CHECK(q_lens.numel() == a.B && q_start.numel() == a.B && kv_start.numel() == a.B && sink.numel() == heads && max_q >= 1 &&
                  a.B <= 65535 && a.H <= 65535, "per-sequence [B] tensors");

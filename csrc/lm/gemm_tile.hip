@@ -9,18 +9,9 @@
 
 namespace shai_lm {
 
-typedef __attribute__((address_space(3))) void lds_void;
 constexpr uint32_t kOob = 0x80000000u;
 
 __device__ __forceinline__ int swz(int row, int ch) { return row * 64 + ((ch ^ ((row >> 1) & 7)) << 3); }
-
-__device__ __forceinline__ __amdgpu_buffer_rsrc_t rsrc(const void* b, long bytes) {
-  return __builtin_amdgcn_make_buffer_rsrc(const_cast<void*>(b), (short)0, (int)bytes, 0x00020000);
-}
-
-__device__ __forceinline__ void dma16(__amdgpu_buffer_rsrc_t r, bf16_t* lds_wave_base, uint32_t voff) {
-  __builtin_amdgcn_raw_ptr_buffer_load_lds(r, (lds_void*)lds_wave_base, 16, voff, 0, 0, 0);
-}
 
 template <typename O, int BM, int BN, int WM, int WN>
 __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_kernel(const GemmArgs p) {
@@ -115,6 +106,37 @@ __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
   }
+  // bf16 results go through LDS, so that rows are stored 16 bytes a lane, whole lines at a time
+  const bool glu = p.epi == EPI_CLAMP_GLU;
+  if (sizeof(O) == 2 && p.ldc % 8 == 0 && (glu || p.N % 8 == 0) && (p.n_main == p.N || n0 + BN <= p.n_main)) {
+    constexpr int LD = BN + 8;
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < IM; ++i) {
+      const int r = wm * TM + i * 32 + fr;
+      const bool live = m0 + r < m_end;          // a row past the end has no angles to read
+#pragma unroll
+      for (int j = 0; j < JN; ++j)
+#pragma unroll
+        for (int g = 0; g < 4; ++g) {
+          const int n = wn * TN + j * 32 + 8 * g + 4 * fh;
+          float4_ c = float4_{acc[i][j][4 * g], acc[i][j][4 * g + 1], acc[i][j][4 * g + 2], acc[i][j][4 * g + 3]};
+          if (live) epilogue_cols<O>(p, m0 + r, n0 + n, c);
+          if (glu) *reinterpret_cast<uint32_t*>(smem + r * LD + (n >> 1)) = pack2(c[0], c[1]);
+          else store4(smem + r * LD + n, c);
+        }
+    }
+    __syncthreads();
+    const int cols = glu ? BN / 2 : BN, c0 = glu ? n0 >> 1 : n0, per = cols / 8;
+    bf16_t* out = static_cast<bf16_t*>(p.C);
+    for (int id = tid; id < BM * per; id += NW * 64) {
+      const int r = id / per, ch = (id % per) * 8;
+      if (m0 + r < m_end && c0 + ch < p.ldc)
+        *reinterpret_cast<uint4_*>(out + (long)(m0 + r) * p.ldc + c0 + ch) =
+            *reinterpret_cast<const uint4_*>(smem + r * LD + ch);
+    }
+    return;
+  }
 #pragma unroll
   for (int i = 0; i < IM; ++i) {
     const int m = m0 + wm * TM + i * 32 + fr;
@@ -132,7 +154,7 @@ template <int BM, int BN, int WM, int WN>
 static void tile(const GemmArgs& a, hipStream_t s) {
   const int tiles_m = a.tiles ? a.n_tiles : (a.M + BM - 1) / BM;
   const int grid = tiles_m * ((a.N + BN - 1) / BN);
-  constexpr int lds = 2 * (BM + BN) * 64 * 2;
+  constexpr int lds = 2 * (BM + BN) * 64 * 2 > BM * (BN + 8) * 2 ? 2 * (BM + BN) * 64 * 2 : BM * (BN + 8) * 2;
   auto go = [&](auto k) {
     (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
     k<<<grid, WM * WN * 64, lds, s>>>(a);

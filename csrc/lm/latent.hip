@@ -3,10 +3,11 @@
 //
 // latent_prep    after the down projection: norms of both latents, rotation of the key part, cache write.
 // latent_decode  bf16, single rows (decode steps, short portions): queries moved into latent space (q W_uk,h), so that a
-//                cached row serves as key and value of every head.  One workgroup per (row, 16 or 32 heads, split); a
-//                64-token page is staged in LDS once and feeds both products on the matrix cores: scores S^T = C Q^T
-//                (a wave per 16 keys), O^T = C^T P^T (a wave per quarter of the latent) with P as a bf16 value plus its
-//                bf16 remainder.
+//                cached row serves as key and value of every head.  One workgroup per (row, 16 or 32 heads, split); half
+//                pages of 32 tokens go to two LDS stages by DMA (buffer_load ... lds; its range check zero-fills rows
+//                past the context), the next one in flight behind the products of the one before: scores S^T = C Q^T (a
+//                wave per 16 keys and 16 heads, Q in registers), O^T = C^T P^T (a wave per quarter of the latent) with P
+//                as a bf16 value plus its bf16 remainder.
 // latent_rows    any size, fp32 or bf16: one wave per (row, head), plain online softmax.
 // latent_gather  cached rows of whole sequences back to back, for the prefill form: long portions expand keys and values
 //                per head and run the flash kernel (attn.hip).
@@ -147,25 +148,45 @@ void launch_latent_rows(const LatentArgs& a, bool f32, hipStream_t s) {
 
 // ------------------------------------------------------------------------------------------------ single rows, bf16
 template <int CR>
-__device__ __forceinline__ int lat_swz(int row, int ch) {      // element offset of 16-byte chunk `ch` of a staged row
+__device__ __forceinline__ int lat_swz(int row, int ch) {      // element offset of 16-byte chunk `ch` of a row
   return row * CR + ((ch ^ (CR % 128 == 0 ? row & 7 : (row >> 1) & 7)) << 3);
 }
 
 template <int RP, int OP, int NG>
-__global__ void __launch_bounds__(256, NG == 1 ? 2 : 1) latent_decode_kernel(const LatentArgs p) {
-  constexpr int CR = RP + OP, KS = CR / 32, CH = CR / 8, NL = CR / 32, ND = RP / 64;
+__global__ void __launch_bounds__(256, 2) latent_decode_kernel(const LatentArgs p) {
+  constexpr int CR = RP + OP, KS = CR / 32, CH = CR / 8, ND = RP / 64, NL = 32 * CH / 256;
+  static_assert(32 * CH % 256 == 0, "whole DMA instructions per wave");
   extern __shared__ __attribute__((aligned(16))) bf16_t smem[];
-  bf16_t* sC = smem;                             // [64][CR] the page
-  bf16_t* sP = sC + 64 * CR;                     // [value | remainder][2][16 NG][4][8]
-  float* sM = reinterpret_cast<float*>(sP + 2 * 2 * 16 * NG * 32);   // [4][16 NG]
-  bf16_t* sQ = reinterpret_cast<bf16_t*>(sM + 4 * 16 * NG);          // [16 NG][CR] (NG > 1)
-  constexpr int PL = 2 * 16 * NG * 32;           // elements of one half of sP
-  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, c = lane & 15, q4 = lane >> 4;
+  bf16_t* sP = smem + 2 * 32 * CR;               // [value | remainder][16 NG][4][8]
+  float* sM = reinterpret_cast<float*>(sP + 2 * 16 * NG * 32);       // [2][16 NG]
+  constexpr int PL = 16 * NG * 32;               // elements of one half of sP
+  const int tid = threadIdx.x, lane = tid & 63, c = lane & 15, q4 = lane >> 4;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int kt = w & 1, sg = w >> 1;             // this wave's scores: 16 keys, 16 heads
+  const bool scores = sg < NG;
   const int e = blockIdx.y, h0 = blockIdx.x * 16 * NG, split = blockIdx.z;
-  const int pos = p.ctx[e] - 1, nb = (pos >> 6) + 1, per = (nb + p.splits - 1) / p.splits;
-  const int s0 = split * per, s1 = min(nb, s0 + per);
+  const int pos = p.ctx[e] - 1, nb = (pos >> 5) + 1;                 // half pages
+  const int s0 = (int)((long)split * nb / p.splits), s1 = (int)((long)(split + 1) * nb / p.splits);
   const int* bt = p.bt + (long)(p.seqs ? p.seqs[e] : e) * p.max_blocks;
   const bf16_t* cache = static_cast<const bf16_t*>(p.cache);
+
+  // source offsets of this lane's 16-byte chunks of a half page; the bank swizzle is applied here
+  uint32_t off[NL];
+#pragma unroll
+  for (int i = 0; i < NL; ++i) {
+    const int id = (w * NL + i) * 64 + lane, r = id / CH;
+    off[i] = (uint32_t)(lat_swz<CR>(r, id % CH) * 2);
+  }
+  auto stage = [&](int t) {
+    const bf16_t* src = cache + ((long)bt[t >> 1] * 64 + (t & 1) * 32) * CR;
+    const int rows = min(32, pos + 1 - t * 32);
+    const __amdgpu_buffer_rsrc_t r = rsrc(src, rows * CR * 2);
+    bf16_t* dst = smem + ((t - s0) & 1) * 32 * CR + w * NL * 512;
+#pragma unroll
+    for (int i = 0; i < NL; ++i)
+      dma16(r, dst + i * 512, off[i]);
+  };
+  if (s0 < s1) stage(s0);
 
   // 8 values of head h's query at column k (zero past the rotated part and past the last head)
   auto query = [&](int h, int k) {
@@ -176,144 +197,116 @@ __global__ void __launch_bounds__(256, NG == 1 ? 2 : 1) latent_decode_kernel(con
                                               p.np + k - RP);
     return uint4_{0u, 0u, 0u, 0u};
   };
-  uint4_ qf[NG == 1 ? KS : 1];
-  if constexpr (NG == 1) {
+  uint4_ qf[KS];
 #pragma unroll
-    for (int s = 0; s < KS; ++s) qf[s] = query(h0 + c, 32 * s + 8 * q4);
-  } else {
-    for (int i = tid; i < 16 * NG * CH; i += 256)
-      *reinterpret_cast<uint4_*>(sQ + lat_swz<CR>(i / CH, i % CH)) = query(h0 + i / CH, (i % CH) * 8);
-  }
+  for (int k = 0; k < KS; ++k) qf[k] = query(scores ? h0 + 16 * sg + c : p.H, 32 * k + 8 * q4);
 
-  uint4_ rc[NL];
-  auto load = [&](int kb) {
-    const bf16_t* page = cache + (long)bt[kb] * 64 * CR;
-    const int left = pos + 1 - kb * 64;
-#pragma unroll
-    for (int i = 0; i < NL; ++i) {
-      const int id = tid + 256 * i;
-      rc[i] = id / CH < left ? *reinterpret_cast<const uint4_*>(page + (long)id * 8) : uint4_{0u, 0u, 0u, 0u};
-    }
-  };
   float4_ o[ND][NG];
-  float m[NG], l[NG];
+  float m[NG], l = 0.f;                          // l: this wave's keys and heads
 #pragma unroll
   for (int g = 0; g < NG; ++g) {
     m[g] = -INFINITY;
-    l[g] = 0.f;
 #pragma unroll
     for (int d = 0; d < ND; ++d) o[d][g] = float4_{0.f, 0.f, 0.f, 0.f};
   }
   const float sl2 = p.scale * kLog2e;
   const int tq = c >> 2, tp = c & 3;
 
-  if (s0 < s1) load(s0);
-  for (int kb = s0; kb < s1; ++kb) {
-    __syncthreads();                             // the page before is no longer read
+  for (int t = s0; t < s1; ++t) {
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();                             // this half page is complete, the one before is no longer read
+    if (t + 1 < s1) stage(t + 1);
+    const bf16_t* sC = smem + ((t - s0) & 1) * 32 * CR;
+    float4_ s = float4_{0.f, 0.f, 0.f, 0.f};
+    if (scores) {
+      float4_ s2 = s;
 #pragma unroll
-    for (int i = 0; i < NL; ++i) {
-      const int id = tid + 256 * i;
-      *reinterpret_cast<uint4_*>(sC + lat_swz<CR>(id / CH, id % CH)) = rc[i];
-    }
-    if (kb + 1 < s1) load(kb + 1);
-    __syncthreads();
-    float4_ s[NG];
-#pragma unroll
-    for (int g = 0; g < NG; ++g) s[g] = float4_{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int k = 0; k < KS; ++k) {
-      const bf16x8 kf = *reinterpret_cast<const bf16x8*>(sC + lat_swz<CR>(16 * w + c, 4 * k + q4));
-#pragma unroll
-      for (int g = 0; g < NG; ++g) {
-        bf16x8 qv;
-        if constexpr (NG == 1) qv = __builtin_bit_cast(bf16x8, qf[k]);
-        else qv = *reinterpret_cast<const bf16x8*>(sQ + lat_swz<CR>(16 * g + c, 4 * k + q4));
-        s[g] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qv, s[g], 0, 0, 0);
+      for (int k = 0; k < KS; k += 2) {
+        const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(sC + lat_swz<CR>(16 * kt + c, 4 * k + q4));
+        const bf16x8 k1 = *reinterpret_cast<const bf16x8*>(sC + lat_swz<CR>(16 * kt + c, 4 * k + 4 + q4));
+        s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k0, __builtin_bit_cast(bf16x8, qf[k]), s, 0, 0, 0);
+        s2 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k1, __builtin_bit_cast(bf16x8, qf[k + 1]), s2, 0, 0, 0);
       }
-    }
-    const int key0 = kb * 64 + 16 * w + 4 * q4;
-#pragma unroll
-    for (int g = 0; g < NG; ++g) {
+      s += s2;
+      const int key0 = t * 32 + 16 * kt + 4 * q4;
       float mx = -INFINITY;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        s[g][i] = key0 + i > pos ? -INFINITY : s[g][i] * sl2;
-        mx = fmaxf(mx, s[g][i]);
+        s[i] = key0 + i > pos ? -INFINITY : s[i] * sl2;
+        mx = fmaxf(mx, s[i]);
       }
       mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-      if (q4 == 0) sM[w * 16 * NG + 16 * g + c] = mx;
+      if (q4 == 0) sM[kt * 16 * NG + 16 * sg + c] = mx;
     }
     __syncthreads();
+    float alpha[NG];
 #pragma unroll
     for (int g = 0; g < NG; ++g) {
-      const float* q = sM + 16 * g + c;
-      const float mn = fmaxf(fmaxf(m[g], fmaxf(q[0], q[16 * NG])), fmaxf(q[32 * NG], q[48 * NG]));
-      const float alpha = __builtin_amdgcn_exp2f(m[g] - mn);   // mn is finite: every page holds a visible key
+      const float mn = fmaxf(m[g], fmaxf(sM[16 * g + c], sM[16 * NG + 16 * g + c]));
+      alpha[g] = __builtin_amdgcn_exp2f(m[g] - mn);             // mn is finite: every half page holds a visible key
       m[g] = mn;
+    }
+    if (scores) {
+      const float mn = NG > 1 && sg > 0 ? m[NG - 1] : m[0], al = NG > 1 && sg > 0 ? alpha[NG - 1] : alpha[0];
       float ls = 0.f;
-      __bf16 hi[4], lo[4];
+      typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
+      bf16x4 hi, lo;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const float x = __builtin_amdgcn_exp2f(s[g][i] - mn);
+        const float x = __builtin_amdgcn_exp2f(s[i] - mn);
         ls += x;
         hi[i] = (__bf16)x;
         lo[i] = (__bf16)(x - (float)hi[i]);
       }
-      l[g] = l[g] * alpha + ls;
-      typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
-      // keys 32 (w / 2) + 16 (w % 2) + 4 q4 + i: k-slot 8 q4 + 4 (w % 2) + i of the half w / 2
-      bf16_t* dst = sP + (((w >> 1) * 16 * NG + 16 * g + c) * 4 + q4) * 8 + 4 * (w & 1);
-      *reinterpret_cast<bf16x4*>(dst) = bf16x4{hi[0], hi[1], hi[2], hi[3]};
-      *reinterpret_cast<bf16x4*>(dst + PL) = bf16x4{lo[0], lo[1], lo[2], lo[3]};
-#pragma unroll
-      for (int d = 0; d < ND; ++d) o[d][g] *= alpha;
+      l = l * al + ls;
+      // key 16 kt + 4 q4 + i is k-slot 8 q4 + 4 kt + i of the product with C^T
+      bf16_t* dst = sP + ((16 * sg + c) * 4 + q4) * 8 + 4 * kt;
+      *reinterpret_cast<bf16x4*>(dst) = hi;
+      *reinterpret_cast<bf16x4*>(dst + PL) = lo;
     }
-    __syncthreads();
 #pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      bf16x8 ph[NG], pl[NG];
+    for (int g = 0; g < NG; ++g)
+#pragma unroll
+      for (int d = 0; d < ND; ++d) o[d][g] *= alpha[g];
+    __syncthreads();
+    bf16x8 ph[NG], pl[NG];
+#pragma unroll
+    for (int g = 0; g < NG; ++g) {
+      const bf16_t* src = sP + ((16 * g + c) * 4 + q4) * 8;
+      ph[g] = *reinterpret_cast<const bf16x8*>(src);
+      pl[g] = *reinterpret_cast<const bf16x8*>(src + PL);
+    }
+#pragma unroll
+    for (int d = 0; d < ND; ++d) {
+      const int col = w * (RP / 4) + 16 * d + 4 * tp, ch = col >> 3, half = (col >> 2) & 1;
+      const bf16_t* a0 = sC + lat_swz<CR>(4 * q4 + tq, ch) + 4 * half;
+      const bf16_t* a1 = sC + lat_swz<CR>(4 * q4 + tq + 16, ch) + 4 * half;
+      const s4v u0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s4v*)(a0));
+      const s4v u1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s4v*)(a1));
+      short8 v;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) { v[j] = u0[j]; v[4 + j] = u1[j]; }
 #pragma unroll
       for (int g = 0; g < NG; ++g) {
-        const bf16_t* src = sP + ((u * 16 * NG + 16 * g + c) * 4 + q4) * 8;
-        ph[g] = *reinterpret_cast<const bf16x8*>(src);
-        pl[g] = *reinterpret_cast<const bf16x8*>(src + PL);
-      }
-#pragma unroll
-      for (int d = 0; d < ND; ++d) {
-        const int col = w * (RP / 4) + 16 * d + 4 * tp, ch = col >> 3, half = (col >> 2) & 1;
-        const int r0 = 32 * u + 4 * q4 + tq;
-        const bf16_t* a0 = sC + lat_swz<CR>(r0, ch) + 4 * half;
-        const bf16_t* a1 = sC + lat_swz<CR>(r0 + 16, ch) + 4 * half;
-        const s4v u0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s4v*)(a0));
-        const s4v u1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s4v*)(a1));
-        short8 v;
-#pragma unroll
-        for (int j = 0; j < 4; ++j) { v[j] = u0[j]; v[4 + j] = u1[j]; }
-#pragma unroll
-        for (int g = 0; g < NG; ++g) {
-          o[d][g] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, v), ph[g], o[d][g], 0, 0, 0);
-          o[d][g] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, v), pl[g], o[d][g], 0, 0, 0);
-        }
+        o[d][g] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, v), ph[g], o[d][g], 0, 0, 0);
+        o[d][g] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, v), pl[g], o[d][g], 0, 0, 0);
       }
     }
   }
-  // the denominator: over the lanes that share a head, then over the waves
+  // the denominator: over the lanes that share a head, then over the two waves of a head
   __syncthreads();
-#pragma unroll
-  for (int g = 0; g < NG; ++g) {
-    float x = l[g];
-    x += __shfl_xor(x, 16, 64);
-    x += __shfl_xor(x, 32, 64);
-    if (q4 == 0) sM[w * 16 * NG + 16 * g + c] = x;
+  if (scores) {
+    l += __shfl_xor(l, 16, 64);
+    l += __shfl_xor(l, 32, 64);
+    if (q4 == 0) sM[kt * 16 * NG + 16 * sg + c] = l;
   }
   __syncthreads();
 #pragma unroll
   for (int g = 0; g < NG; ++g) {
     const int h = h0 + 16 * g + c;
     if (h >= p.H) continue;
-    const float* q = sM + 16 * g + c;
-    const float L = (q[0] + q[16 * NG]) + (q[32 * NG] + q[48 * NG]);
+    const float L = sM[16 * g + c] + sM[16 * NG + 16 * g + c];
     if (p.splits == 1) {
       const float sk = p.sink[h] * kLog2e, top = fmaxf(m[g], sk), a = __builtin_amdgcn_exp2f(m[g] - top);
       const float inv = a / (L * a + __builtin_amdgcn_exp2f(sk - top));
@@ -359,7 +352,7 @@ bool latent_decode_fits(int rp, int op) { return op == 64 && (rp == 64 || rp == 
 template <int RP, int NG>
 static void decode(const LatentArgs& a, hipStream_t s) {
   constexpr int CR = RP + 64;
-  constexpr int lds = (64 * CR + 2 * 2 * 16 * NG * 32) * 2 + 4 * 16 * NG * 4 + (NG > 1 ? 16 * NG * CR * 2 : 0);
+  constexpr int lds = (2 * 32 * CR + 2 * 16 * NG * 32) * 2 + 2 * 16 * NG * 4;
   (void)hipFuncSetAttribute(reinterpret_cast<const void*>(latent_decode_kernel<RP, 64, NG>),
                             hipFuncAttributeMaxDynamicSharedMemorySize, lds);
   latent_decode_kernel<RP, 64, NG><<<dim3((a.H + 16 * NG - 1) / (16 * NG), a.n, a.splits), 256, lds, s>>>(a);

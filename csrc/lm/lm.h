@@ -148,12 +148,12 @@ struct AttnArgs {
   int B, T, max_q, H, G, dk, dv, max_blocks, splits, chunk;
   float scale;
   // latent form of the prefill kernel: q rows at `qkvg`; keys of sequence b are rows kv_start[b] ..; a key is
-  // [kv[0 .. np) | lat[rank .. rank + rot)], its value kv[np .. np + dv)
+  // [kv[0 .. np) | lat[rank .. )], its value kv[np .. np + dv)
   const void* kv;          // [rows, H, np + dv]
   const void* lat;         // [rows, lat_ld]
   const int* kv_start;
   const float* sink;       // [H]
-  int np, rot, rank, lat_ld;
+  int np, rank, lat_ld, lat_pad;   // lat_pad: the last column after `rank` from which 8 values may be read
 };
 void launch_kv_store(const AttnArgs& a, bool f32, hipStream_t s);
 void launch_attn_prefill(const AttnArgs& a, bool f32, hipStream_t s);

@@ -23,6 +23,19 @@ __device__ __forceinline__ float load1(const bf16_t* p) { return bf2f(*p); }
 __device__ __forceinline__ void store1(float* p, float v) { *p = v; }
 __device__ __forceinline__ void store1(bf16_t* p, float v) { *p = f2bf(v); }
 
+// DMA to LDS: 16 bytes a lane, lane-linear from a wave-uniform LDS address; a buffer's range check zero-fills past its end
+typedef __attribute__((address_space(3))) void lds_void;
+typedef __attribute__((address_space(1))) void glb_void;
+__device__ __forceinline__ __amdgpu_buffer_rsrc_t rsrc(const void* b, long bytes) {
+  return __builtin_amdgcn_make_buffer_rsrc(const_cast<void*>(b), (short)0, (int)bytes, 0x00020000);
+}
+__device__ __forceinline__ void dma16(__amdgpu_buffer_rsrc_t r, bf16_t* lds_wave_base, uint32_t voff) {
+  __builtin_amdgcn_raw_ptr_buffer_load_lds(r, (lds_void*)lds_wave_base, 16, voff, 0, 0, 0);
+}
+__device__ __forceinline__ void dma16(const bf16_t* src, bf16_t* lds_wave_base) {
+  __builtin_amdgcn_global_load_lds((glb_void*)src, (lds_void*)lds_wave_base, 16, 0, 0);
+}
+
 __device__ __forceinline__ float sigmoid_f(float x) { return 1.f / (1.f + expf(-x)); }
 // clamped GLU: value (u + 1), gate g sigmoid(1.702 g), both limited
 __device__ __forceinline__ float clamp_glu(float g, float u, float lim) {
@@ -47,9 +60,46 @@ __device__ __forceinline__ float block_sum256(float v, float (*red)[4], int& tur
   return (r[0] + r[1]) + (r[2] + r[3]);
 }
 
-// xIELU: ap z^2 + z / 2 above zero, an (exp(z) - 1 - z) + z / 2 below
-__device__ __forceinline__ float xielu(float z, float ap, float an) {
-  return (z > 0.f ? ap * z * z : an * (expm1f(z) - z)) + 0.5f * z;
+// xIELU: ap z^2 + z / 2 above zero, an (exp(z) - 1 - z) + z / 2 below.  `fast` (results that are rounded to bf16): the
+// hardware exponential, a short series near zero.
+__device__ __forceinline__ float xielu(float z, float ap, float an, bool fast) {
+  float e;
+  if (fast) {
+    const float series = z * z * (0.5f + z * (1.f / 6.f + z * (1.f / 24.f + z * (1.f / 120.f))));
+    e = z > -0.3f ? series : __builtin_amdgcn_exp2f(z * 1.4426950408889634f) - 1.f - z;
+  } else {
+    e = expm1f(z) - z;
+  }
+  return (z > 0.f ? ap * z * z : an * e) + 0.5f * z;
+}
+
+// Epilogue of 4 consecutive columns n .. n + 3 of row m, in place (a GLU's two results: c[0], c[1]).
+template <typename O>
+__device__ __forceinline__ void epilogue_cols(const GemmArgs& p, long m, int n, float4_& c) {
+  if (p.epi == EPI_CLAMP_GLU) {
+    c[0] = clamp_glu(c[0], c[1], p.param);
+    c[1] = clamp_glu(c[2], c[3], p.param);
+  } else if (p.epi == EPI_SOFTCAP) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) c[i] = p.param * tanhf(c[i] / p.param);
+  } else if (p.epi == EPI_XIELU) {
+    const float ap = p.vec[0], an = p.vec[1];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) c[i] = xielu(c[i], ap, an, sizeof(O) == 2);
+  } else if (p.epi == EPI_ROTARY) {
+    const int d = n % p.head - p.rot0;
+    if (d >= 0 && d < p.rot && n < p.N) {
+      const float* t = p.rope + m * p.rot + d;
+      const float u = c[0], v = c[1];
+      c[0] = u * t[0] - v * t[1];
+      c[1] = v * t[0] + u * t[1];
+      if (d + 2 < p.rot) {
+        const float u2 = c[2], v2 = c[3];
+        c[2] = u2 * t[2] - v2 * t[3];
+        c[3] = v2 * t[2] + u2 * t[3];
+      }
+    }
+  }
 }
 
 // Store 4 consecutive columns n .. n + 3 of row m after the epilogue.  `out`: C of this product.
@@ -67,32 +117,12 @@ __device__ __forceinline__ void store_cols(const GemmArgs& p, O* out, long m, in
       if (n + i < p.N) o[i] = c[i];
     return;
   }
+  epilogue_cols<O>(p, m, n, c);
   if (p.epi == EPI_CLAMP_GLU) {
     const int j = n >> 1;
-    if (n < p.N) store1(out + m * p.ldc + j, clamp_glu(c[0], c[1], p.param));
-    if (n + 2 < p.N) store1(out + m * p.ldc + j + 1, clamp_glu(c[2], c[3], p.param));
+    if (n < p.N) store1(out + m * p.ldc + j, c[0]);
+    if (n + 2 < p.N) store1(out + m * p.ldc + j + 1, c[1]);
     return;
-  }
-  if (p.epi == EPI_SOFTCAP) {
-#pragma unroll
-    for (int i = 0; i < 4; ++i) c[i] = p.param * tanhf(c[i] / p.param);
-  } else if (p.epi == EPI_XIELU) {
-    const float ap = p.vec[0], an = p.vec[1];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) c[i] = xielu(c[i], ap, an);
-  } else if (p.epi == EPI_ROTARY) {
-    const int d = n % p.head - p.rot0;
-    if (d >= 0 && d < p.rot && n < p.N) {
-      const float* t = p.rope + m * p.rot + d;
-      const float u = c[0], v = c[1];
-      c[0] = u * t[0] - v * t[1];
-      c[1] = v * t[0] + u * t[1];
-      if (d + 2 < p.rot) {
-        const float u2 = c[2], v2 = c[3];
-        c[2] = u2 * t[2] - v2 * t[3];
-        c[3] = v2 * t[2] + u2 * t[3];
-      }
-    }
   }
   O* o = out + m * p.ldc + n;
   if (((p.N | p.ldc) & 3) == 0) {

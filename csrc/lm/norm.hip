@@ -87,45 +87,78 @@ __global__ void __launch_bounds__(256) add_norm_kernel(const AddNormArgs p) {
   }
 }
 
-// The row stays in registers through both norms.  With a convolution a workgroup walks `run` consecutive rows and keeps
-// the last taps - 1 inputs in registers; the ones before its first row are recomputed from their residual rows (which is
-// why x_out is not x then) or, before the step's first row of a sequence, come from the sequence's state.
-template <typename T, int NV, int TAPS>
-__global__ void __launch_bounds__(256) residual_norm_kernel(const ResidualNormArgs p) {
-  __shared__ float red[2][4];
+// sum over a workgroup of NT threads; `red` alternates between two buffers, one barrier per call
+template <int NT>
+__device__ __forceinline__ float block_sum(float v, float (*red)[NT / 64], int& turn) {
+  v = wave_sum(v);
+  float* r = red[turn];
+  turn ^= 1;
+  if ((threadIdx.x & 63) == 0) r[threadIdx.x >> 6] = v;
+  __syncthreads();
+  float x = r[0];
+#pragma unroll
+  for (int i = 1; i < NT / 64; ++i) x += r[i];
+  return x;
+}
+
+// The row stays in registers through both norms.  With a convolution a workgroup walks `run` consecutive rows, loads each
+// one ahead, and keeps the last taps - 1 inputs in registers; the ones before its first row are recomputed from their
+// residual rows (which is why x_out is not x then) or, before the step's first row of a sequence, come from the sequence's
+// state.
+template <typename T, int NT, int NV, int TAPS>
+__global__ void __launch_bounds__(NT) residual_norm_kernel(const ResidualNormArgs p) {
+  constexpr bool KEEP = TAPS > 0 && TAPS <= 4 && NV <= 2;   // gains and taps in registers for all rows
+  constexpr int KN = KEEP ? NV : 1, KT = KEEP ? TAPS : 1;
+  __shared__ float red[2][NT / 64];
   int turn = 0;
   const int c0 = threadIdx.x * 4;
   const float inv_w = 1.f / (float)p.width;
-  auto load = [&](long row, float4_(&v)[NV]) {
+  const float4_ zero = float4_{0.f, 0.f, 0.f, 0.f};
+  struct Row {
+    float4_ x[NV], d[NV];
+  };
+  auto fetch = [&](long row, Row& q) {
     const float* x = p.x ? p.x + row * p.Dp : nullptr;
     const T* e = x ? nullptr : static_cast<const T*>(p.table) + (long)min(max(p.ids[row], 0), p.V - 1) * p.Dp;
-    float4_ d[NV];
-    float ss = 0.f;
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int c = i * 1024 + c0;
-      v[i] = float4_{0.f, 0.f, 0.f, 0.f};
-      d[i] = v[i];
+      const int c = i * NT * 4 + c0;
+      q.x[i] = q.d[i] = zero;
       if (c < p.Dp) {
-        v[i] = x ? load4(x + c) : load4(e + c) * p.scale;
-        if (p.delta) d[i] = load4(static_cast<const T*>(p.delta) + row * p.Dp + c);
-        ss += d[i][0] * d[i][0] + d[i][1] * d[i][1] + d[i][2] * d[i][2] + d[i][3] * d[i][3];
+        q.x[i] = x ? load4(x + c) : load4(e + c) * p.scale;
+        if (p.delta) q.d[i] = load4(static_cast<const T*>(p.delta) + row * p.Dp + c);
       }
     }
+  };
+  float4_ kw[KN], kb[KN], kc[KT][KN];
+  if constexpr (KEEP) {
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = i * NT * 4 + c0;
+      const bool in = c < p.Dp;
+      kw[i] = in ? load4(p.w + c) : zero;
+      kb[i] = in && p.delta ? load4(p.wb + c) : zero;
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j)             // kc[j]: tap of the input j rows before
+        kc[j][i] = in && j < p.taps ? load4(p.cw + (long)(p.taps - 1 - j) * p.Dp + c) : zero;
+    }
+  }
+  auto add = [&](const Row& q, float4_(&v)[NV]) {
+    float r = 0.f;
     if (p.delta) {
-      ss = block_sum256(ss, red, turn);
-      const float r = p.mult / sqrtf(ss * inv_w + p.eps);
+      float ss = 0.f;
 #pragma unroll
-      for (int i = 0; i < NV; ++i) {
-        const int c = i * 1024 + c0;
-        if (c < p.Dp) v[i] += d[i] * r * load4(p.wb + c);
-      }
+      for (int i = 0; i < NV; ++i)
+        ss += q.d[i][0] * q.d[i][0] + q.d[i][1] * q.d[i][1] + q.d[i][2] * q.d[i][2] + q.d[i][3] * q.d[i][3];
+      r = p.mult / sqrtf(block_sum<NT>(ss, red, turn) * inv_w + p.eps);
     }
-    if (p.step) {
 #pragma unroll
-      for (int i = 0; i < NV; ++i) {
-        const int c = i * 1024 + c0;
-        if (c < p.Dp) v[i] += load4(p.step + c);
+    for (int i = 0; i < NV; ++i) {
+      const int c = i * NT * 4 + c0;
+      v[i] = q.x[i];
+      if (c < p.Dp) {
+        if (p.delta) v[i] += q.d[i] * r * (KEEP ? kb[KEEP ? i : 0] : load4(p.wb + c));
+        if (p.step) v[i] += load4(p.step + c);
       }
     }
   };
@@ -133,24 +166,25 @@ __global__ void __launch_bounds__(256) residual_norm_kernel(const ResidualNormAr
     float ss = 0.f;
 #pragma unroll
     for (int i = 0; i < NV; ++i) ss += v[i][0] * v[i][0] + v[i][1] * v[i][1] + v[i][2] * v[i][2] + v[i][3] * v[i][3];
-    ss = block_sum256(ss, red, turn);
-    const float r = 1.f / sqrtf(ss * inv_w + p.eps);
+    const float r = 1.f / sqrtf(block_sum<NT>(ss, red, turn) * inv_w + p.eps);
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int c = i * 1024 + c0;
-      if (c < p.Dp) v[i] = v[i] * r * load4(p.w + c);
+      const int c = i * NT * 4 + c0;
+      if (c < p.Dp) v[i] = v[i] * r * (KEEP ? kw[KEEP ? i : 0] : load4(p.w + c));
     }
   };
   auto put = [&](auto* dst, const float4_(&v)[NV]) {
 #pragma unroll
     for (int i = 0; i < NV; ++i)
-      if (i * 1024 + c0 < p.Dp) store4(dst + i * 1024 + c0, v[i]);
+      if (i * NT * 4 + c0 < p.Dp) store4(dst + i * NT * 4 + c0, v[i]);
   };
 
+  Row q;
   float4_ v[NV];
   if constexpr (TAPS == 0) {
     const long row = p.rows ? p.rows[blockIdx.x] : blockIdx.x;
-    load(row, v);
+    fetch(row, q);
+    add(q, v);
     if (p.x_out) put(p.x_out + row * p.Dp, v);
     if (!p.w) return;
     norm(v);
@@ -159,6 +193,7 @@ __global__ void __launch_bounds__(256) residual_norm_kernel(const ResidualNormAr
     float4_ hist[TAPS - 1][NV];                  // hist[j]: input of the row j + 1 before
     const int row0 = blockIdx.x * p.run, row1 = min(row0 + p.run, p.T);
     int seq = -1;
+    fetch(row0, q);
     for (int t = row0; t < row1; ++t) {
       const int b = p.row_seq ? p.row_seq[t] : t;
       const int at = p.row_seq ? t - p.q_start[b] : 0, pos = p.pos[t], slot = p.slots[b];
@@ -168,29 +203,37 @@ __global__ void __launch_bounds__(256) residual_norm_kernel(const ResidualNormAr
 #pragma unroll
         for (int j = 0; j < TAPS - 1; ++j) {
 #pragma unroll
-          for (int i = 0; i < NV; ++i) hist[j][i] = float4_{0.f, 0.f, 0.f, 0.f};
+          for (int i = 0; i < NV; ++i) hist[j][i] = zero;
           const int back = j + 1;
           if (back >= p.taps || back > pos) continue;
           if (back <= at) {                      // a row of this step
-            load(t - back, hist[j]);
+            Row o;
+            fetch(t - back, o);
+            add(o, hist[j]);
             norm(hist[j]);
           } else if (slot >= 0) {
             const float* s = st + (long)(p.taps - 1 - (back - at)) * p.Dp;
 #pragma unroll
             for (int i = 0; i < NV; ++i)
-              if (i * 1024 + c0 < p.Dp) hist[j][i] = load4(s + i * 1024 + c0);
+              if (i * NT * 4 + c0 < p.Dp) hist[j][i] = load4(s + i * NT * 4 + c0);
           }
         }
       }
-      load(t, v);
+      const Row cur = q;
+      if (t + 1 < row1) fetch(t + 1, q);
+      add(cur, v);
       put(p.x_out + (long)t * p.Dp, v);
       norm(v);
       float4_ y[NV];
 #pragma unroll
       for (int i = 0; i < NV; ++i) {
-        const int c = i * 1024 + c0;
+        const int c = i * NT * 4 + c0;
         y[i] = v[i];
-        if (c < p.Dp) {
+        if constexpr (KEEP) {
+          y[i] += kc[0][i] * v[i];
+#pragma unroll
+          for (int j = 0; j < TAPS - 1; ++j) y[i] += kc[j + 1][i] * hist[j][i];
+        } else if (c < p.Dp) {
           y[i] += load4(p.cw + (long)(p.taps - 1) * p.Dp + c) * v[i];
 #pragma unroll
           for (int j = 0; j < TAPS - 1; ++j)
@@ -271,26 +314,22 @@ void launch_rope_rows(const RopeRowsArgs& a, hipStream_t s) {
 void launch_embed_norm(const EmbedNormArgs& a, bool f32, hipStream_t s) { SHAI_LM_ROWS(embed_norm_kernel, a, f32, s); }
 void launch_add_norm(const AddNormArgs& a, bool f32, hipStream_t s) { SHAI_LM_ROWS(add_norm_kernel, a, f32, s); }
 
-template <typename T, int NV>
+template <typename T, int NT, int NV>
 static void residual_norm(const ResidualNormArgs& a, hipStream_t s) {
-  if (!a.cw) {
-    residual_norm_kernel<T, NV, 0><<<a.T, 256, 0, s>>>(a);
-    return;
-  }
-  const int grid = (a.T + a.run - 1) / a.run;
-  if (NV <= 8 && a.taps <= 4) residual_norm_kernel<T, NV, NV <= 8 ? 4 : 16><<<grid, 256, 0, s>>>(a);
-  else residual_norm_kernel<T, NV, 16><<<grid, 256, 0, s>>>(a);
+  const int grid = a.cw ? (a.T + a.run - 1) / a.run : a.T;
+  if (!a.cw) residual_norm_kernel<T, NT, NV, 0><<<grid, NT, 0, s>>>(a);
+  else if (a.taps <= 4) residual_norm_kernel<T, NT, NV, 4><<<grid, NT, 0, s>>>(a);
+  else residual_norm_kernel<T, NT, NV, 16><<<grid, NT, 0, s>>>(a);
 }
 
 void launch_residual_norm(const ResidualNormArgs& a, bool f32, hipStream_t s) {
-  const int nv = (a.Dp + 1023) / 1024;
   auto go = [&](auto tag) {
     using T = decltype(tag);
-    if (nv <= 1) residual_norm<T, 1>(a, s);
-    else if (nv <= 2) residual_norm<T, 2>(a, s);
-    else if (nv <= 4) residual_norm<T, 4>(a, s);
-    else if (nv <= 8) residual_norm<T, 8>(a, s);
-    else residual_norm<T, 16>(a, s);
+    if (a.Dp <= 1024) residual_norm<T, 256, 1>(a, s);
+    else if (a.Dp <= 2048) residual_norm<T, 256, 2>(a, s);
+    else if (a.Dp <= 4096) residual_norm<T, 512, 2>(a, s);
+    else if (a.Dp <= 8192) residual_norm<T, 1024, 2>(a, s);
+    else residual_norm<T, 1024, 4>(a, s);
   };
   if (f32) go(float{});
   else go(bf16_t{});
