@@ -252,6 +252,28 @@ void lm_gemm_heads(const Tensor& A, const Tensor& W, const Tensor& C) {
   if (g.M > 0) shai_lm::launch_gemm(g, f32, stream());
 }
 
+// partial sums of a w^T over equal parts of K: c [splits, M, N] fp32
+void lm_gemm_parts(const Tensor& A, const Tensor& W, const Tensor& C) {
+  const bool f32 = is_f32(A);
+  check(A, A.scalar_type(), "A");
+  check(W, A.scalar_type(), "W");
+  check(C, at::kFloat, "C");
+  shai_lm::GemmArgs g{};
+  SHAI_CHECK(A.dim() == 2 && W.dim() == 2 && C.dim() == 3, "lm_gemm_parts ranks");
+  g.M = g.a_rows = A.size(0);
+  g.N = g.n_main = g.ldc = W.size(0);
+  g.K = g.lda = A.size(1);
+  g.splits = C.size(0);
+  g.batch = 1;
+  g.out_f32 = true;
+  SHAI_CHECK(W.size(1) == g.K && g.K % 64 == 0 && C.size(1) == g.M && C.size(2) == g.N && g.splits >= 1 &&
+                 g.splits <= g.K / 64, "lm_gemm_parts shapes");
+  g.A = A.data_ptr();
+  g.W = W.data_ptr();
+  g.C = C.data_ptr();
+  if (g.M > 0) shai_lm::launch_gemm(g, f32, stream());
+}
+
 void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const optional<Tensor>& table, double scale,
                    const optional<Tensor>& delta, const optional<Tensor>& wb, double mult, const optional<Tensor>& step,
                    const optional<Tensor>& x_out, const optional<Tensor>& rows, const optional<Tensor>& w, double eps,
@@ -290,10 +312,13 @@ void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const
     return t->data_ptr<float>();
   };
   if (delta) {
-    check(*delta, dt, "delta");
-    SHAI_CHECK(delta->dim() == 2 && delta->size(0) == R && delta->size(1) == a.Dp && wb.has_value(),
-               "delta must be [rows, D], with its norm's gain");
+    const bool many = delta->dim() == 3;
+    check(*delta, many ? at::kFloat : dt, "delta");
+    SHAI_CHECK((many || delta->dim() == 2) && delta->size(-2) == R && delta->size(-1) == a.Dp && wb.has_value(),
+               "delta must be [rows, D] or [parts, rows, D], with its norm's gain");
     a.delta = delta->data_ptr();
+    a.parts = many ? delta->size(0) : 0;
+    a.part_stride = R * a.Dp;
   }
   a.wb = row_vec(wb, "wb");
   a.mult = mult;
@@ -346,7 +371,7 @@ void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const
       a.row_seq = row_seq->data_ptr<int>();
       a.q_start = q_start->data_ptr<int>();
       a.q_lens = q_lens->data_ptr<int>();
-      a.run = R >= 16384 ? 16 : R >= 4096 ? 8 : 4;
+      a.run = R >= 32768 ? 32 : R >= 8192 ? 16 : R >= 4096 ? 8 : 4;
     }
     SHAI_CHECK(slots->numel() >= a.B, "one state slot per sequence");
   }
@@ -397,8 +422,9 @@ void latent_prep(const Tensor& d, const Tensor& wq, const Tensor& wkv, const Ten
   check(cache, dt, "cache");
   check(cq, dt, "cq");
   shai_lm::LatentPrepArgs a{};
-  SHAI_CHECK(d.dim() == 2 && cq.dim() == 2 && cache.dim() == 3 && cache.size(1) == 64 && rope.dim() == 2, "latent_prep ranks");
-  a.T = d.size(0);
+  SHAI_CHECK((d.dim() == 2 || d.dim() == 3) && cq.dim() == 2 && cache.dim() == 3 && cache.size(1) == 64 && rope.dim() == 2, "latent_prep ranks");
+  a.T = d.size(-2);
+  a.parts = d.dim() == 3 ? d.size(0) : 1;
   a.qp = cq.size(1);
   a.rp = wkv.numel();
   a.op = cache.size(2) - a.rp;
@@ -407,7 +433,7 @@ void latent_prep(const Tensor& d, const Tensor& wq, const Tensor& wkv, const Ten
   a.kv_rank = kv_rank;
   a.eps = eps;
   SHAI_CHECK(a.qp % 64 == 0 && a.rp % 64 == 0 && a.op % 2 == 0 && a.op >= a.rot && a.rot % 2 == 0 && wq.numel() == a.qp &&
-                 d.size(1) == a.qp + a.rp + a.op && cq.size(0) == a.T && rope.size(0) == a.T && slots.numel() >= a.T &&
+                 d.size(-1) == a.qp + a.rp + a.op && (a.parts == 1 || (a.qp + a.rp + a.op) * 4 <= 65536 - 64) && cq.size(0) == a.T && rope.size(0) == a.T && slots.numel() >= a.T &&
                  q_rank >= 1 && q_rank <= a.qp && kv_rank >= 1 && kv_rank <= a.rp, "latent_prep shapes");
   a.d = d.data_ptr<float>();
   a.wq = wq.data_ptr<float>();
@@ -775,6 +801,7 @@ TORCH_LIBRARY_FRAGMENT(shai, m) {
   m.def("add_norm(Tensor(a!) x, Tensor? dense, Tensor? ye, Tensor? slot_of, Tensor? wts, Tensor? inject, Tensor? rows, Tensor? w, float eps, int width, Tensor(b!)? h) -> ()");
   m.def("lm_gemm(Tensor a, Tensor w, Tensor(a!) c, Tensor? tiles, Tensor? offsets, Tensor? gather, int bm, int epi, float param, Tensor(b!)? side=None, Tensor? vec=None, Tensor? rope=None, int head=0, int rot0=0) -> ()");
   m.def("lm_gemm_heads(Tensor a, Tensor w, Tensor(a!) c) -> ()");
+  m.def("lm_gemm_parts(Tensor a, Tensor w, Tensor(a!) c) -> ()");
   m.def("residual_norm(Tensor? x, Tensor? ids, Tensor? table, float scale, Tensor? delta, Tensor? wb, float mult, Tensor? step, Tensor(a!)? x_out, Tensor? rows, Tensor? w, float eps, int width, Tensor(b!)? h, Tensor? cw=None, Tensor(c!)? state=None, Tensor(d!)? tail=None, Tensor? row_seq=None, Tensor? q_start=None, Tensor? q_lens=None, Tensor? pos=None, Tensor? slots=None) -> ()");
   m.def("conv_commit(Tensor(a!) state, Tensor tail, Tensor q_lens, Tensor slots) -> ()");
   m.def("rope_rows(Tensor pos, Tensor freq, Tensor(a!) out) -> ()");
@@ -798,6 +825,7 @@ TORCH_LIBRARY_IMPL(shai, CUDA, m) {
   m.impl("add_norm", &add_norm);
   m.impl("lm_gemm", &lm_gemm);
   m.impl("lm_gemm_heads", &lm_gemm_heads);
+  m.impl("lm_gemm_parts", &lm_gemm_parts);
   m.impl("residual_norm", &residual_norm);
   m.impl("conv_commit", &conv_commit);
   m.impl("rope_rows", &rope_rows);

@@ -7,7 +7,8 @@
 // pair of W is folded in registers.  A k-step covers 64 values; lane group g = lane / 16 takes values 16 g .. 16 g + 15
 // of it in both operands (the order of k inside a dot product is free), i.e. every W row is read 128 bytes at a time.
 //
-// Dense: row tiles of A are blockIdx.y, products of a batch (one per attention head, say) blockIdx.z.  Grouped (experts): blockIdx.y is an entry of the tile list and blockIdx.z a
+// Dense: row tiles of A are blockIdx.y, products of a batch (one per attention head, say) or
+// parts of K (partial sums for the consumer to add) blockIdx.z.  Grouped (experts): blockIdx.y is an entry of the tile list and blockIdx.z a
 // 16 MT-row part of it; rows past the expert's last slot are computed on a clamped row and not stored.
 #include "lm_device.h"
 #include "lm.h"
@@ -86,8 +87,13 @@ __global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) 
   for (int i = 0; i < NT; ++i)
 #pragma unroll
     for (int j = 0; j < MT; ++j) acc[i][j] = float4_{0.f, 0.f, 0.f, 0.f};
-  // this wave's k-steps are wid, wid + NW, ...; D of them are in flight
-  const int steps = p.K / 64;
+  // this wave's k-steps are first + wid, first + wid + NW, ...; D of them are in flight
+  int steps = p.K / 64, first = 0;
+  if (p.splits > 1) {
+    first = (int)(blockIdx.z * (long)steps / p.splits);
+    steps = (int)((blockIdx.z + 1L) * steps / p.splits);
+    C += (long)blockIdx.z * p.M * p.N;
+  }
   Frag<T> w[D][NT], x[D][MT];
   auto fetch = [&](int u, int s) {
     if (s < steps) {
@@ -99,8 +105,8 @@ __global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) 
     }
   };
 #pragma unroll
-  for (int u = 0; u < D; ++u) fetch(u, wid + u * NW);
-  for (int s0 = wid; s0 < steps; s0 += NW * D) {
+  for (int u = 0; u < D; ++u) fetch(u, first + wid + u * NW);
+  for (int s0 = first + wid; s0 < steps; s0 += NW * D) {
 #pragma unroll
     for (int u = 0; u < D; ++u) {
       if (s0 + u * NW < steps) {
@@ -134,19 +140,25 @@ template <typename T, typename O>
 static void stream(const GemmArgs& a, hipStream_t s) {
   auto go = [&](auto kernel, int mt, int nt, int nw) {
     const dim3 grid((a.N + 16 * nt - 1) / (16 * nt), a.tiles ? a.n_tiles : (a.M + 16 * mt - 1) / (16 * mt),
-                    a.tiles ? (a.bm + 16 * mt - 1) / (16 * mt) : a.batch);
+                    a.tiles ? (a.bm + 16 * mt - 1) / (16 * mt) : a.splits > 1 ? a.splits : a.batch);
     kernel<<<grid, 64 * nw, 0, s>>>(a);
   };
   constexpr bool H = sizeof(T) == 2;              // fp32 fragments are twice the registers
 #define GO(MT_, NT_, NW_, D_) go(gemm_stream_kernel<T, O, MT_, NT_, NW_, H ? D_ : 1>, MT_, NT_, NW_)
   const int rows = a.tiles ? a.bm : a.M;
-  if (rows <= 16 || a.N < 512) GO(1, 1, 8, 4);
+  if (a.splits > 1) {
+    if (rows <= 16) GO(1, 1, 4, 4);
+    else if (rows <= 32) GO(2, 2, 4, 4);
+    else if (a.N < 2560 && a.K < 12288) GO(4, 2, 4, 3);
+    else GO(4, 4, 4, 2);
+  } else if (rows <= 16 || a.N < 512) GO(1, 1, 8, 4);
   else if (a.tiles) GO(4, 2, 4, 2);
   else if (a.N < 3072 || (rows <= 32 && a.N < 5120)) GO(2, 1, 8, 4);
   else if (a.N < 5120) GO(2, 2, 8, 2);
   else if (rows <= 32) GO(2, 4, 4, 3);
   else if (a.N < 8192) GO(4, 2, 4, 2);
-  else GO(4, 4, 4, 2);
+  else if (a.N < 16384) GO(4, 4, 4, 2);
+  else GO(4, 4, 2, 2);
 #undef GO
   SHAI_CHECK_LAUNCH();
 }

@@ -19,22 +19,28 @@ namespace shai_lm {
 typedef short s4v __attribute__((ext_vector_type(4)));
 constexpr float kLog2e = 1.4426950408889634f;
 
-template <typename T>
+// MANY: d is partial sums; they are added once, into LDS.
+template <typename T, bool MANY>
 __global__ void __launch_bounds__(256) latent_prep_kernel(const LatentPrepArgs p) {
   __shared__ float red[2][4];
+  extern __shared__ __attribute__((aligned(16))) float sum[];
   int turn = 0;
   const long t = blockIdx.x;
-  const float* d = p.d + t * (p.qp + p.rp + p.op);
-  const float* k = d + p.qp;
+  const int n = p.qp + p.rp + p.op;
+  const float* d = p.d + t * n;
   float sq = 0.f, sk = 0.f;
-  for (int c = threadIdx.x * 4; c < p.qp; c += 1024) {
-    const float4_ v = load4(d + c);
-    sq += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+  for (int c = threadIdx.x * 4; c < p.qp + p.rp + (MANY ? p.op : 0); c += 1024) {
+    float4_ v = load4(d + c);
+    if constexpr (MANY) {
+      for (int i = 1; i < p.parts; ++i) v += load4(d + (long)i * p.T * n + c);
+      store4(sum + c, v);
+    }
+    const float ss = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+    if (c < p.qp) sq += ss;
+    else if (c < p.qp + p.rp) sk += ss;
   }
-  for (int c = threadIdx.x * 4; c < p.rp; c += 1024) {
-    const float4_ v = load4(k + c);
-    sk += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
-  }
+  if constexpr (MANY) d = sum;                   // complete after the barriers of the sums below
+  const float* k = d + p.qp;
   sq = block_sum256(sq, red, turn);
   sk = block_sum256(sk, red, turn);
   const float rq = 1.f / sqrtf(sq / (float)p.q_rank + p.eps), rk = 1.f / sqrtf(sk / (float)p.kv_rank + p.eps);
@@ -58,8 +64,11 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(const LatentPrepArgs p
 }
 
 void launch_latent_prep(const LatentPrepArgs& a, bool f32, hipStream_t s) {
-  if (f32) latent_prep_kernel<float><<<a.T, 256, 0, s>>>(a);
-  else latent_prep_kernel<bf16_t><<<a.T, 256, 0, s>>>(a);
+  const int lds = (a.qp + a.rp + a.op) * 4;
+  if (f32 && a.parts > 1) latent_prep_kernel<float, true><<<a.T, 256, lds, s>>>(a);
+  else if (f32) latent_prep_kernel<float, false><<<a.T, 256, 0, s>>>(a);
+  else if (a.parts > 1) latent_prep_kernel<bf16_t, true><<<a.T, 256, lds, s>>>(a);
+  else latent_prep_kernel<bf16_t, false><<<a.T, 256, 0, s>>>(a);
   SHAI_CHECK_LAUNCH();
 }
 

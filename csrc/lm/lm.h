@@ -46,7 +46,9 @@ struct ResidualNormArgs {
   const void* table;       // [V, Dp]
   float scale;
   int V;
-  const void* delta;       // [*, Dp] sublayer output, or null
+  const void* delta;       // [*, Dp] sublayer output, or [parts, *, Dp] fp32 partial sums of it, or null
+  int parts;               // 0: delta is of the type of h
+  long part_stride;
   const float* wb;         // its norm's gain
   float mult;
   const float* step;       // [Dp] added to every row, or null
@@ -68,7 +70,7 @@ struct ResidualNormArgs {
   const int* slots;        // [B] state slot, -1: none
   int B, run;              // rows per workgroup
 };
-void launch_residual_norm(const ResidualNormArgs& a, bool f32, hipStream_t s);
+void launch_residual_norm(const ResidualNormArgs& a, bool f32, hipStream_t s);   // run <= 64
 
 struct ConvCommitArgs {    // the tails of a prefill step into the state of every layer run
   float* state;            // [runs, slots, taps - 1, Dp]
@@ -105,6 +107,7 @@ struct GemmArgs {
   float* side;
   bool out_f32;
   long lda, ldc;           // row strides of A and C
+  int splits;              // K cut into this many parts over blockIdx.z: C [splits, M, N] fp32 partial sums
   int batch;               // dense: products batched over blockIdx.z (streaming kernel only)
   long a_batch, w_batch, c_batch;
   const float* vec;        // EPI_XIELU: (alpha_p, alpha_n)
@@ -161,7 +164,7 @@ void launch_attn_decode(const AttnArgs& a, bool f32, hipStream_t s);
 void launch_latent_prefill(const AttnArgs& a, hipStream_t s);          // bf16
 
 struct LatentPrepArgs {
-  const float* d;          // [T, qp + rp + op]: query latent, key/value latent, rotated key part
+  const float* d;          // [parts, T, qp + rp + op], summed over parts: query latent, key/value latent, rotated key part
   const float* wq;         // [qp] gains (zero in the pads)
   const float* wkv;        // [rp]
   const float* rope;       // [T, rot]
@@ -169,7 +172,7 @@ struct LatentPrepArgs {
   void* cache;             // [blocks, 64, rp + op]
   void* cq;                // [T, qp]
   float eps;
-  int T, q_rank, kv_rank, rot, qp, rp, op;
+  int T, parts, q_rank, kv_rank, rot, qp, rp, op;
 };
 void launch_latent_prep(const LatentPrepArgs& a, bool f32, hipStream_t s);
 

@@ -101,55 +101,67 @@ __device__ __forceinline__ float block_sum(float v, float (*red)[NT / 64], int& 
   return x;
 }
 
-// The row stays in registers through both norms.  With a convolution a workgroup walks `run` consecutive rows, loads each
-// one ahead, and keeps the last taps - 1 inputs in registers; the ones before its first row are recomputed from their
+// 4 elements as they lie in memory: converted when they are used, so that a load issued ahead is not waited for early
+__device__ __forceinline__ float4_ raw4(const float* p) { return load4(p); }
+__device__ __forceinline__ uint2_ raw4(const bf16_t* p) { return *reinterpret_cast<const uint2_*>(p); }
+__device__ __forceinline__ float4_ wide4(float4_ v) { return v; }
+__device__ __forceinline__ float4_ wide4(uint2_ v) {
+  return float4_{__uint_as_float(v[0] << 16), __uint_as_float(v[0] & 0xffff0000u), __uint_as_float(v[1] << 16),
+                 __uint_as_float(v[1] & 0xffff0000u)};
+}
+
+// The row stays in registers through both norms.  With a convolution a workgroup walks `run` consecutive rows, two of them
+// loaded ahead, and keeps the last taps - 1 inputs in registers; the ones before its first row are recomputed from their
 // residual rows (which is why x_out is not x then) or, before the step's first row of a sequence, come from the sequence's
-// state.
-template <typename T, int NT, int NV, int TAPS>
-__global__ void __launch_bounds__(NT) residual_norm_kernel(const ResidualNormArgs p) {
-  constexpr bool KEEP = TAPS > 0 && TAPS <= 4 && NV <= 2;   // gains and taps in registers for all rows
+// state.  Whatever the rows share (gains, taps, the rows' places) is read before the first row: a load inside the loop
+// would wait for the rows ahead of it.  TD: the type of delta.
+constexpr int conv_waves(int taps, int nt, int nv) { return taps == 4 && nt <= 512 && nv <= 2 ? 4 : 1; }   // per SIMD
+template <typename T, typename TD, int NT, int NV, int TAPS>
+__global__ void __launch_bounds__(NT, conv_waves(TAPS, NT, NV)) residual_norm_kernel(const ResidualNormArgs p) {
+  constexpr bool CONV = TAPS > 0, KEEP = CONV && TAPS <= 4 && NV <= 2;   // KEEP: taps in registers
   constexpr int KN = KEEP ? NV : 1, KT = KEEP ? TAPS : 1;
+  using Raw = decltype(raw4(static_cast<const TD*>(nullptr)));
   __shared__ float red[2][NT / 64];
+  __shared__ __attribute__((aligned(16))) float sw[CONV ? 2 : 1][CONV ? NT * NV * 4 : 4];   // w, wb
   int turn = 0;
   const int c0 = threadIdx.x * 4;
   const float inv_w = 1.f / (float)p.width;
   const float4_ zero = float4_{0.f, 0.f, 0.f, 0.f};
   struct Row {
-    float4_ x[NV], d[NV];
+    float4_ x[NV];
+    Raw d[NV];
   };
   auto fetch = [&](long row, Row& q) {
     const float* x = p.x ? p.x + row * p.Dp : nullptr;
     const T* e = x ? nullptr : static_cast<const T*>(p.table) + (long)min(max(p.ids[row], 0), p.V - 1) * p.Dp;
+    const TD* d = static_cast<const TD*>(p.delta) + row * p.Dp;
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int c = i * NT * 4 + c0;
-      q.x[i] = q.d[i] = zero;
+      q.x[i] = zero;
+      q.d[i] = Raw{};
       if (c < p.Dp) {
         q.x[i] = x ? load4(x + c) : load4(e + c) * p.scale;
-        if (p.delta) q.d[i] = load4(static_cast<const T*>(p.delta) + row * p.Dp + c);
+        if (p.delta) q.d[i] = raw4(d + c);
+        if constexpr (sizeof(TD) == 4)
+          for (int k = 1; k < p.parts; ++k) q.d[i] += raw4(d + k * p.part_stride + c);
       }
     }
   };
-  float4_ kw[KN], kb[KN], kc[KT][KN];
-  if constexpr (KEEP) {
-#pragma unroll
-    for (int i = 0; i < NV; ++i) {
-      const int c = i * NT * 4 + c0;
-      const bool in = c < p.Dp;
-      kw[i] = in ? load4(p.w + c) : zero;
-      kb[i] = in && p.delta ? load4(p.wb + c) : zero;
-#pragma unroll
-      for (int j = 0; j < TAPS; ++j)             // kc[j]: tap of the input j rows before
-        kc[j][i] = in && j < p.taps ? load4(p.cw + (long)(p.taps - 1 - j) * p.Dp + c) : zero;
-    }
-  }
+  auto gain = [&](const float* g, int which, int i) {      // gains of this thread's columns
+    const int c = i * NT * 4 + c0;
+    if constexpr (CONV) return *reinterpret_cast<const float4_*>(&sw[which][c]);
+    else return load4(g + c);
+  };
   auto add = [&](const Row& q, float4_(&v)[NV]) {
     float r = 0.f;
     if (p.delta) {
       float ss = 0.f;
 #pragma unroll
-      for (int i = 0; i < NV; ++i)
-        ss += q.d[i][0] * q.d[i][0] + q.d[i][1] * q.d[i][1] + q.d[i][2] * q.d[i][2] + q.d[i][3] * q.d[i][3];
+      for (int i = 0; i < NV; ++i) {
+        const float4_ d = wide4(q.d[i]);
+        ss += d[0] * d[0] + d[1] * d[1] + d[2] * d[2] + d[3] * d[3];
+      }
       r = p.mult / sqrtf(block_sum<NT>(ss, red, turn) * inv_w + p.eps);
     }
 #pragma unroll
@@ -157,7 +169,7 @@ __global__ void __launch_bounds__(NT) residual_norm_kernel(const ResidualNormArg
       const int c = i * NT * 4 + c0;
       v[i] = q.x[i];
       if (c < p.Dp) {
-        if (p.delta) v[i] += q.d[i] * r * (KEEP ? kb[KEEP ? i : 0] : load4(p.wb + c));
+        if (p.delta) v[i] += wide4(q.d[i]) * r * gain(p.wb, 1, i);
         if (p.step) v[i] += load4(p.step + c);
       }
     }
@@ -168,10 +180,8 @@ __global__ void __launch_bounds__(NT) residual_norm_kernel(const ResidualNormArg
     for (int i = 0; i < NV; ++i) ss += v[i][0] * v[i][0] + v[i][1] * v[i][1] + v[i][2] * v[i][2] + v[i][3] * v[i][3];
     const float r = 1.f / sqrtf(block_sum<NT>(ss, red, turn) * inv_w + p.eps);
 #pragma unroll
-    for (int i = 0; i < NV; ++i) {
-      const int c = i * NT * 4 + c0;
-      if (c < p.Dp) v[i] = v[i] * r * (KEEP ? kw[KEEP ? i : 0] : load4(p.w + c));
-    }
+    for (int i = 0; i < NV; ++i)
+      if (i * NT * 4 + c0 < p.Dp) v[i] = v[i] * r * gain(p.w, 0, i);
   };
   auto put = [&](auto* dst, const float4_(&v)[NV]) {
 #pragma unroll
@@ -179,9 +189,9 @@ __global__ void __launch_bounds__(NT) residual_norm_kernel(const ResidualNormArg
       if (i * NT * 4 + c0 < p.Dp) store4(dst + i * NT * 4 + c0, v[i]);
   };
 
-  Row q;
   float4_ v[NV];
-  if constexpr (TAPS == 0) {
+  if constexpr (!CONV) {
+    Row q;
     const long row = p.rows ? p.rows[blockIdx.x] : blockIdx.x;
     fetch(row, q);
     add(q, v);
@@ -190,16 +200,36 @@ __global__ void __launch_bounds__(NT) residual_norm_kernel(const ResidualNormArg
     norm(v);
     put(static_cast<T*>(p.h) + (long)blockIdx.x * p.Dp, v);
   } else {
-    float4_ hist[TAPS - 1][NV];                  // hist[j]: input of the row j + 1 before
     const int row0 = blockIdx.x * p.run, row1 = min(row0 + p.run, p.T);
+    // lane i of every wave holds row i's place: its sequence, offset in the step, position, state slot, rows after it
+    const int mt = min(row0 + (int)(threadIdx.x & 63), row1 - 1);
+    const int m_b = p.row_seq ? p.row_seq[mt] : mt, m_pos = p.pos[mt], m_slot = p.slots[m_b];
+    const int m_at = p.row_seq ? mt - p.q_start[m_b] : 0, m_left = p.row_seq ? p.q_lens[m_b] - 1 - m_at : 0;
+    Row q0, q1;
+    fetch(row0, q0);
+    if (row0 + 1 < row1) fetch(row0 + 1, q1);
+    float4_ kc[KT][KN];                          // kc[j]: tap of the input j rows before
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = i * NT * 4 + c0;
+      const bool in = c < p.Dp;
+      store4(&sw[0][c], in ? load4(p.w + c) : zero);     // read back by this thread only
+      store4(&sw[1][c], in && p.delta ? load4(p.wb + c) : zero);
+      if constexpr (KEEP) {
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j)
+          kc[j][i] = in && j < p.taps ? load4(p.cw + (long)(p.taps - 1 - j) * p.Dp + c) : zero;
+      }
+    }
+    float4_ hist[TAPS - 1][NV];                  // hist[j]: input of the row j + 1 before
     int seq = -1;
-    fetch(row0, q);
     for (int t = row0; t < row1; ++t) {
-      const int b = p.row_seq ? p.row_seq[t] : t;
-      const int at = p.row_seq ? t - p.q_start[b] : 0, pos = p.pos[t], slot = p.slots[b];
+      const int b = __builtin_amdgcn_readlane(m_b, t - row0), at = __builtin_amdgcn_readlane(m_at, t - row0);
+      const int slot = __builtin_amdgcn_readlane(m_slot, t - row0);
       float* st = p.state + (long)max(slot, 0) * (p.taps - 1) * p.Dp;
       if (b != seq) {
         seq = b;
+        const int pos = __builtin_amdgcn_readlane(m_pos, t - row0);
 #pragma unroll
         for (int j = 0; j < TAPS - 1; ++j) {
 #pragma unroll
@@ -219,9 +249,9 @@ __global__ void __launch_bounds__(NT) residual_norm_kernel(const ResidualNormArg
           }
         }
       }
-      const Row cur = q;
-      if (t + 1 < row1) fetch(t + 1, q);
-      add(cur, v);
+      add(q0, v);
+      q0 = q1;
+      if (t + 2 < row1) fetch(t + 2, q1);
       put(p.x_out + (long)t * p.Dp, v);
       norm(v);
       float4_ y[NV];
@@ -242,7 +272,7 @@ __global__ void __launch_bounds__(NT) residual_norm_kernel(const ResidualNormArg
       }
       put(static_cast<T*>(p.h) + (long)t * p.Dp, y);
       if (p.row_seq) {
-        const int left = p.q_lens[b] - 1 - at;   // rows of the sequence after this one
+        const int left = __builtin_amdgcn_readlane(m_left, t - row0);
         if (left < p.taps - 1) put(p.tail + ((long)b * (p.taps - 1) + p.taps - 2 - left) * p.Dp, v);
       } else if (slot >= 0 && p.taps > 1) {      // the only workgroup that reads this state
         put(st + (long)(p.taps - 2) * p.Dp, v);
@@ -314,25 +344,27 @@ void launch_rope_rows(const RopeRowsArgs& a, hipStream_t s) {
 void launch_embed_norm(const EmbedNormArgs& a, bool f32, hipStream_t s) { SHAI_LM_ROWS(embed_norm_kernel, a, f32, s); }
 void launch_add_norm(const AddNormArgs& a, bool f32, hipStream_t s) { SHAI_LM_ROWS(add_norm_kernel, a, f32, s); }
 
-template <typename T, int NT, int NV>
+template <typename T, typename TD, int NT, int NV>
 static void residual_norm(const ResidualNormArgs& a, hipStream_t s) {
   const int grid = a.cw ? (a.T + a.run - 1) / a.run : a.T;
-  if (!a.cw) residual_norm_kernel<T, NT, NV, 0><<<grid, NT, 0, s>>>(a);
-  else if (a.taps <= 4) residual_norm_kernel<T, NT, NV, 4><<<grid, NT, 0, s>>>(a);
-  else residual_norm_kernel<T, NT, NV, 16><<<grid, NT, 0, s>>>(a);
+  if (!a.cw) residual_norm_kernel<T, TD, NT, NV, 0><<<grid, NT, 0, s>>>(a);
+  else if (a.taps <= 4) residual_norm_kernel<T, TD, NT, NV, 4><<<grid, NT, 0, s>>>(a);
+  else residual_norm_kernel<T, TD, NT, NV, 16><<<grid, NT, 0, s>>>(a);
+}
+
+template <typename T, typename TD>
+static void residual_norm(const ResidualNormArgs& a, hipStream_t s) {
+  if (a.Dp <= 1024) residual_norm<T, TD, 256, 1>(a, s);
+  else if (a.Dp <= 2048) residual_norm<T, TD, 256, 2>(a, s);
+  else if (a.Dp <= 4096) residual_norm<T, TD, 512, 2>(a, s);
+  else if (a.Dp <= 8192) residual_norm<T, TD, 1024, 2>(a, s);
+  else residual_norm<T, TD, 1024, 4>(a, s);
 }
 
 void launch_residual_norm(const ResidualNormArgs& a, bool f32, hipStream_t s) {
-  auto go = [&](auto tag) {
-    using T = decltype(tag);
-    if (a.Dp <= 1024) residual_norm<T, 256, 1>(a, s);
-    else if (a.Dp <= 2048) residual_norm<T, 256, 2>(a, s);
-    else if (a.Dp <= 4096) residual_norm<T, 512, 2>(a, s);
-    else if (a.Dp <= 8192) residual_norm<T, 1024, 2>(a, s);
-    else residual_norm<T, 1024, 4>(a, s);
-  };
-  if (f32) go(float{});
-  else go(bf16_t{});
+  if (f32) residual_norm<float, float>(a, s);
+  else if (a.parts) residual_norm<bf16_t, float>(a, s);
+  else residual_norm<bf16_t, bf16_t>(a, s);
   SHAI_CHECK_LAUNCH();
 }
 

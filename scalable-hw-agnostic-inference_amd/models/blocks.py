@@ -329,10 +329,10 @@ class LatentAttention(nn.Module):
         """``step``: the step's shared work (:class:`StepShared`)."""
         c = self.c
         rope, plan = step.rope(self), step.plan(self.expands)
-        down = lm.matmul(h, self.down, torch.float32)
+        down = lm.matmul_parts(h, self.down, torch.float32)
         cq = lm.latent_prep(down, self.q_norm, self.kv_norm, rope, batch, cache, self.eps, c.q_rank, c.kv_rank)
         q = lm.matmul(cq, self.uq, epi=lm.EPI_ROTARY, rope=rope, head=self.dk, rot0=self.np)
-        return lm.matmul(self.attend(q, batch, cache, plan), self.o)
+        return lm.matmul_parts(self.attend(q, batch, cache, plan), self.o)
 
     def attend(self, q, batch, cache, plan):
         """q [T, H dk], turned, over the cached latents (this step's included) -> [T, H dv]."""
@@ -412,7 +412,7 @@ class MinGRU(nn.Module):
 
     def forward(self, h, batch, state, step=None):
         g, zx = lm.matmul_with_side(h, self.gzx, 2 * self.sp)
-        return lm.matmul(lm.mingru_scan(zx, g, self.bias, state, batch), self.o)
+        return lm.matmul_parts(lm.mingru_scan(zx, g, self.bias, state, batch), self.o)
 
     def cache_shape(self, blocks: int, block: int):
         return None
@@ -440,7 +440,7 @@ class XieluMLP(nn.Module):
                 "act": (act + torch.tensor([0.0, 0.5], dtype=act.dtype, device=act.device)).float()}
 
     def forward(self, h):
-        return lm.matmul(lm.matmul(h, self.up, epi=lm.EPI_XIELU, vec=self.act), self.down)
+        return lm.matmul_parts(lm.matmul(h, self.up, epi=lm.EPI_XIELU, vec=self.act), self.down)
 
     def init_random_(self, gen):
         _init_packed(self, self.pack, self.shapes(), gen)

@@ -30,6 +30,7 @@ MAX_TAPS = 16                # convolution taps
 MAX_LATENT = 1024            # columns of a cached latent
 LATENT_SHORT = 16            # portions up to this many rows attend in latent space, longer ones expand keys and values
 LATENT_GROUP_ROWS = 1 << 18  # context rows that are expanded at a time
+PARTS, PARTS_ROWS, PARTS_COLUMNS = 4, 64, 8192   # partial sums of decode products
 SCAN_CHUNK, SCAN_MAX_CHUNKS = 64, 64
 
 
@@ -131,6 +132,17 @@ def matmul_with_side(a, w, side: int, epi: int = EPI_NONE, param: float = 0.0):
     s = torch.empty(M, side, dtype=torch.float32, device=a.device)
     _K().lm_gemm(a, w, c, None, None, None, 0, int(epi), float(param), s)
     return c, s
+
+
+def matmul_parts(a, w, out_dtype=None):
+    """a w^T for a consumer that adds partial sums (:func:`residual_norm`, :func:`latent_prep`): [parts, M, N] fp32 for a
+    few rows of a narrow product, which needs K cut up to fill the chip; else :func:`matmul`."""
+    M, K, N = a.shape[0], a.shape[1], w.shape[0]
+    if not a.is_cuda or a.dtype != torch.bfloat16 or M > PARTS_ROWS or N > PARTS_COLUMNS or K < PARTS * 128:
+        return matmul(a, w, out_dtype)
+    c = torch.empty(PARTS, M, N, dtype=torch.float32, device=a.device)
+    _K().lm_gemm_parts(a, w, c)
+    return c
 
 
 def glu_with_side(a, w, side: int, param: float):
@@ -237,7 +249,7 @@ def residual_norm(source, delta, wb, mult: float, step, w, eps: float, width: in
                   batch=None, rows=None, keep: bool = True):
     """x = source (+ mult * RMSNorm(delta) wb) (+ step); h = RMSNorm(x) w, plus its convolution with ``conv``.
 
-    source: the fp32 residual [T, D] or an :class:`Embedding`.  Returns (x, h); the residual may be updated in place.
+    source: the fp32 residual [T, D] or an :class:`Embedding`.  delta: [T, D], or partial sums [parts, T, D] fp32.  Returns (x, h); the residual may be updated in place.
     ``w`` None: no norm (h None).  ``rows`` (int32): h of these rows only, and with ``keep`` False x is None."""
     emb = isinstance(source, Embedding)
     if not (source.ids if emb else source).is_cuda:
@@ -356,12 +368,12 @@ def latent_plan(batch, expand: bool) -> LatentPlan:
 
 
 def latent_prep(d, wq, wkv, rope, batch, cache, eps: float, q_rank: int, kv_rank: int):
-    """The down projection's fp32 rows [q latent | kv latent | rotated key part] (each padded): norms both latents, turns
+    """The down projection's fp32 rows [q latent | kv latent | rotated key part] (each padded; or partial sums): norms both latents, turns
     the key part, writes [kv latent | key part] to ``cache`` [blocks, 64, ..] at batch.slots.  Returns the normed q latent
     in the cache's dtype."""
     if not d.is_cuda:
         return ref.latent_prep(d, wq, wkv, rope, batch, cache, eps, q_rank, kv_rank)
-    cq = torch.empty(d.shape[0], wq.shape[0], dtype=cache.dtype, device=d.device)
+    cq = torch.empty(d.shape[-2], wq.shape[0], dtype=cache.dtype, device=d.device)
     _K().latent_prep(d, wq, wkv, rope, batch.slots, cache, cq, float(eps), int(q_rank), int(kv_rank))
     return cq
 

@@ -31,6 +31,11 @@ def close(got, want, tol, what=""):
     assert err < tol, f"{what}: {err:.2e}"
 
 
+def whole(y):
+    """A block's output, its partial sums added."""
+    return y.sum(0) if y.dim() == 3 else y
+
+
 class Stepper:
     """Sequences in a paged pool with shuffled pages and state slots: ``step`` makes the batch of their next rows."""
 
@@ -112,6 +117,12 @@ def check_matmul(device, dtype):
             y, side = lm.matmul_with_side(ad, wd[:rows].contiguous(), rows - main)
             close(y, ref[:, :main], tol, "main")
             close(side, ref[:, main:rows], 3e-4, "side")
+    for m, n, k in ((1, 64, 512), (16, 70, 576), (30, 640, 1024), (64, 3000, 640), (50, 130, 832)):
+        a = torch.randn(m, k, generator=g).to(dtype)
+        w = (torch.randn(n, k, generator=g) / k ** 0.5).to(dtype)
+        y = lm.matmul_parts(a.to(device), w.to(device))
+        assert y.dim() == (3 if device != "cpu" and dtype == torch.bfloat16 else 2)
+        close(whole(y), a.double() @ w.double().T, 3e-4, "parts")
     for T, H, K, N, head in ((1, 3, 64, 64, 128), (19, 8, 128, 192, 192), (70, 20, 64, 512, 64)):
         a = torch.randn(T, H * head, generator=g).to(dtype)
         w = (torch.randn(H, N + 8, K, generator=g) / K ** 0.5).to(dtype)
@@ -153,6 +164,12 @@ def check_residual_norm(device, dtype):
                 close(xs[:, :width], want, 2e-5, "x")
                 assert not xs[:, width:].any() and not h[:, width:].any()
                 close(h[:, :width], R.rms_norm(want, w.double(), 1e-3), tol, "h")
+                if delta is not None and device != "cpu":   # the same output as partial sums
+                    parts = torch.stack([up(d).float() * 0.5, up(d).float() * 0.25, up(d).float() * 0.25])
+                    src = source.clone() if isinstance(source, torch.Tensor) else source
+                    xp, hp = lm.residual_norm(src, parts, *args[1:], up(w), 1e-3, width, dtype)
+                    close(xp[:, :width], want, 2e-5, "x of parts")
+                    close(hp, h.double().cpu(), tol, "h of parts")
                 src = source.clone() if isinstance(source, torch.Tensor) else source
                 rows = torch.tensor([T - 1, 0, T - 1], dtype=torch.int32, device=device)
                 none, h = lm.residual_norm(src, *args, up(w), 1e-3, width, torch.float32 if delta is None and src is not source
@@ -170,7 +187,8 @@ def check_conv(device, dtype):
     come from the state, the ones before a sequence's start are zero whatever the slot holds."""
     tol = 3e-5 if dtype == torch.float32 else 0.06
     for width, taps, lengths in ((50, 4, (70, 3, 21, 1)), (130, 1, (9, 4)), (64, 2, (40, 12)), (70, 9, (45, 17, 5)),
-                                 (2050, 3, (11, 6)), (48, 16, (40, 30))):
+                                 (2050, 3, (11, 6)), (48, 16, (40, 30)), (5000, 4, (7, 2)),
+                                 (9000, 2, (5, 3))):
         g = torch.Generator().manual_seed(width)
         r = lambda *s: torch.randn(*s, generator=g)
         xs, ds = [r(n, width) for n in lengths], [r(n, width).to(dtype) for n in lengths]
@@ -231,7 +249,7 @@ def check_latent_attention(device, dtype):
 
             def fn(batch, rows):
                 h = pad(torch.stack([hs[b][p] for b, p in rows])).to(device, dtype)
-                return m(h, batch, cache, StepShared(batch))[:, :72]
+                return whole(m(h, batch, cache, StepShared(batch)))[:, :72]
 
             got = drive(lengths, cuts, device, fn, splits)
             for a, b in zip(got, want):
@@ -352,7 +370,7 @@ def check_blocks(device, dtype):
             getattr(m, k).copy_(v)
         m.to(device)
         state = torch.full((3, m.sp), JUNK, device=device)
-        fn = lambda batch, rows: m(pad(h[[p for _, p in rows]]).to(device, dtype), batch, state)[:, :width]
+        fn = lambda batch, rows: whole(m(pad(h[[p for _, p in rows]]).to(device, dtype), batch, state))[:, :width]
         want = R.mingru(h.double(), lambda name: w["l0.mix." + name].double())
         for cuts in ((n,), (13, 1, 1)):
             close(drive((n,), cuts, device, fn)[0] / want.std(), want / want.std(), tol, "mingru")
@@ -360,7 +378,7 @@ def check_blocks(device, dtype):
         for k, v in f.pack(lambda name: w["l0.mlp." + name]).items():
             getattr(f, k).copy_(v)
         want = R.feed_forward(h.double(), lambda name: w["l0.mlp." + name].double())
-        close(f.to(device)(pad(h).to(device, dtype))[:, :width] / want.std(), want / want.std(), tol, "xielu")
+        close(whole(f.to(device)(pad(h).to(device, dtype)))[:, :width] / want.std(), want / want.std(), tol, "xielu")
 
 
 MECHANISMS = [check_matmul, check_rope_rows, check_residual_norm, check_conv, check_latent_attention, check_needle,
