@@ -32,7 +32,14 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(const LatentPrepArgs p
   for (int c = threadIdx.x * 4; c < p.qp + p.rp + (MANY ? p.op : 0); c += 1024) {
     float4_ v = load4(d + c);
     if constexpr (MANY) {
-      for (int i = 1; i < p.parts; ++i) v += load4(d + (long)i * p.T * n + c);
+      for (int i = 1; i < p.parts; i += 3) {
+        float4_ e[3];
+#pragma unroll
+        for (int j = 0; j < 3; ++j) e[j] = load4(d + (long)min(i + j, p.parts - 1) * p.T * n + c);
+        v += e[0];
+        if (i + 1 < p.parts) v += e[1];
+        if (i + 2 < p.parts) v += e[2];
+      }
       store4(sum + c, v);
     }
     const float ss = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];

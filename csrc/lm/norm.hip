@@ -144,7 +144,12 @@ __global__ void __launch_bounds__(NT, conv_waves(TAPS, NT, NV)) residual_norm_ke
         q.x[i] = x ? load4(x + c) : load4(e + c) * p.scale;
         if (p.delta) q.d[i] = raw4(d + c);
         if constexpr (sizeof(TD) == 4)
-          for (int k = 1; k < p.parts; ++k) q.d[i] += raw4(d + k * p.part_stride + c);
+          for (int k = 1; k < p.parts; k += 3) {           // three loads at a time, none of them waited for alone
+            float4_ e[3];
+#pragma unroll
+            for (int j = 0; j < 3; ++j) e[j] = raw4(d + min(k + j, p.parts - 1) * p.part_stride + c);
+            q.d[i] += e[0] + (k + 1 < p.parts ? e[1] : zero) + (k + 2 < p.parts ? e[2] : zero);
+          }
       }
     }
   };
@@ -208,6 +213,23 @@ __global__ void __launch_bounds__(NT, conv_waves(TAPS, NT, NV)) residual_norm_ke
     Row q0, q1;
     fetch(row0, q0);
     if (row0 + 1 < row1) fetch(row0 + 1, q1);
+    float4_ hist[TAPS - 1][NV];                  // hist[j]: input of the row j + 1 before
+    // the inputs before the step's first row of a sequence, `at` rows before this one
+    auto past = [&](int slot, int at, int pos) {
+      const float* st = p.state + (long)slot * (p.taps - 1) * p.Dp;
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) {
+        const bool in = j + 1 < p.taps && j + 1 > at && j + 1 <= pos && slot >= 0;
+#pragma unroll
+        for (int i = 0; i < NV; ++i)
+          hist[j][i] = in && i * NT * 4 + c0 < p.Dp ? load4(st + (long)(p.taps - 2 - j + at) * p.Dp + i * NT * 4 + c0) : zero;
+      }
+    };
+    int seq = -1;
+    if (!p.row_seq) {                            // decode: this row's state in flight with the rest
+      seq = row0;
+      past(__builtin_amdgcn_readlane(m_slot, 0), 0, __builtin_amdgcn_readlane(m_pos, 0));
+    }
     float4_ kc[KT][KN];                          // kc[j]: tap of the input j rows before
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
@@ -221,33 +243,21 @@ __global__ void __launch_bounds__(NT, conv_waves(TAPS, NT, NV)) residual_norm_ke
           kc[j][i] = in && j < p.taps ? load4(p.cw + (long)(p.taps - 1 - j) * p.Dp + c) : zero;
       }
     }
-    float4_ hist[TAPS - 1][NV];                  // hist[j]: input of the row j + 1 before
-    int seq = -1;
     for (int t = row0; t < row1; ++t) {
       const int b = __builtin_amdgcn_readlane(m_b, t - row0), at = __builtin_amdgcn_readlane(m_at, t - row0);
       const int slot = __builtin_amdgcn_readlane(m_slot, t - row0);
       float* st = p.state + (long)max(slot, 0) * (p.taps - 1) * p.Dp;
       if (b != seq) {
         seq = b;
-        const int pos = __builtin_amdgcn_readlane(m_pos, t - row0);
+        past(slot, at, __builtin_amdgcn_readlane(m_pos, t - row0));
 #pragma unroll
-        for (int j = 0; j < TAPS - 1; ++j) {
-#pragma unroll
-          for (int i = 0; i < NV; ++i) hist[j][i] = zero;
-          const int back = j + 1;
-          if (back >= p.taps || back > pos) continue;
-          if (back <= at) {                      // a row of this step
+        for (int j = 0; j < TAPS - 1; ++j)
+          if (j + 1 < p.taps && j + 1 <= at) {   // a row of this step
             Row o;
-            fetch(t - back, o);
+            fetch(t - j - 1, o);
             add(o, hist[j]);
             norm(hist[j]);
-          } else if (slot >= 0) {
-            const float* s = st + (long)(p.taps - 1 - (back - at)) * p.Dp;
-#pragma unroll
-            for (int i = 0; i < NV; ++i)
-              if (i * NT * 4 + c0 < p.Dp) hist[j][i] = load4(s + i * NT * 4 + c0);
           }
-        }
       }
       add(q0, v);
       q0 = q1;
