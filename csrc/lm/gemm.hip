@@ -151,6 +151,10 @@ static void stream(const GemmArgs& a, hipStream_t s) {
     else if (rows <= 32) GO(2, 2, 4, 4);
     else if (a.N < 2560 && a.K < 12288) GO(4, 2, 4, 3);
     else GO(4, 4, 4, 2);
+  } else if (!a.tiles && a.K <= 256) {            // too few k-steps to split over many waves
+    if (rows <= 16) GO(1, 2, 2, 2);
+    else if (rows <= 32) GO(2, 2, 2, 2);
+    else GO(4, 2, 2, 2);
   } else if (rows <= 16 || a.N < 512) GO(1, 1, 8, 4);
   else if (a.tiles) GO(4, 2, 4, 2);
   else if (a.N < 3072 || (rows <= 32 && a.N < 5120)) GO(2, 1, 8, 4);
