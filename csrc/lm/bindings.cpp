@@ -271,7 +271,11 @@ void lm_gemm_parts(const Tensor& A, const Tensor& W, const Tensor& C) {
   g.A = A.data_ptr();
   g.W = W.data_ptr();
   g.C = C.data_ptr();
-  if (g.M > 0) shai_lm::launch_gemm(g, f32, stream());
+  if (g.M == 0) return;
+  const long lim = 0x7fffffffL;
+  const bool tile = !f32 && g.M > 64 && (long)g.M * g.K * 2 < lim && (long)g.N * g.K * 2 < lim;
+  if (tile) shai_lm::launch_gemm_tile(g, stream());
+  else shai_lm::launch_gemm(g, f32, stream());
 }
 
 void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const optional<Tensor>& table, double scale,
@@ -371,7 +375,7 @@ void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const
       a.row_seq = row_seq->data_ptr<int>();
       a.q_start = q_start->data_ptr<int>();
       a.q_lens = q_lens->data_ptr<int>();
-      a.run = R >= 32768 ? 32 : R >= 8192 ? 16 : R >= 4096 ? 8 : 4;
+      a.run = R >= 32768 ? 32 : R >= 8192 ? 16 : R >= 4096 ? 8 : R >= 2048 ? 4 : 2;
     }
     SHAI_CHECK(slots->numel() >= a.B, "one state slot per sequence");
   }

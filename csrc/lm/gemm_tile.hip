@@ -1,4 +1,5 @@
-// C = epi(A W^T), LDS-tiled bf16 form for many rows (prefill): 128 x 128 tiles of 4 waves or 256 x 256 tiles of 8, 64-wide
+// C = epi(A W^T), LDS-tiled bf16 form for many rows (prefill): 64 x 64 or 128 x 128 tiles of 4 waves or 256 x 256 tiles of
+// 8, 64-wide
 // k-tiles moved global -> LDS by DMA (buffer_load ... lds, 16 bytes per lane) into two stages; the load of k-tile t + 1 is
 // issued before the MFMAs of t.  The bank swizzle is applied to the per-lane source chunk.  Buffer range checks zero-fill
 // rows past the ends.  Dense or grouped by expert: the row tiles of a grouped product come from the tile list, each with
@@ -78,14 +79,20 @@ __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_
 #pragma unroll
       for (int r = 0; r < 16; ++r) acc[i][j][r] = 0.f;
 
-  const int nk = p.K / 64;
+  int nk = p.K / 64, k0 = 0;
+  O* C = static_cast<O*>(p.C);
+  if (p.splits > 1) {                            // this workgroup's part of K, its own partial sums
+    k0 = (int)(blockIdx.y * (long)nk / p.splits);
+    nk = (int)((blockIdx.y + 1L) * nk / p.splits) - k0;
+    C += (long)blockIdx.y * p.M * p.N;
+  }
   const int fr = lane & 31, fh = lane >> 5;
-  stage(0, 0);
+  stage(0, k0);
   asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
   __syncthreads();
   for (int kt = 0; kt < nk; ++kt) {
     const int cur = kt & 1;
-    if (kt + 1 < nk) stage(cur ^ 1, kt + 1);
+    if (kt + 1 < nk) stage(cur ^ 1, k0 + kt + 1);
     const bf16_t* sa = smem + cur * STAGE;
     const bf16_t* sw = sa + BM * 64;
 #pragma unroll
@@ -128,7 +135,7 @@ __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_
     }
     __syncthreads();
     const int cols = glu ? BN / 2 : BN, c0 = glu ? n0 >> 1 : n0, per = cols / 8;
-    bf16_t* out = static_cast<bf16_t*>(p.C);
+    bf16_t* out = reinterpret_cast<bf16_t*>(C);
     for (int id = tid; id < BM * per; id += NW * 64) {
       const int r = id / per, ch = (id % per) * 8;
       if (m0 + r < m_end && c0 + ch < p.ldc)
@@ -145,7 +152,7 @@ __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_
     for (int j = 0; j < JN; ++j)
 #pragma unroll
       for (int g = 0; g < 4; ++g)
-        store_cols<O>(p, static_cast<O*>(p.C), m, n0 + wn * TN + j * 32 + 8 * g + 4 * fh,
+        store_cols<O>(p, C, m, n0 + wn * TN + j * 32 + 8 * g + 4 * fh,
                       float4_{acc[i][j][4 * g], acc[i][j][4 * g + 1], acc[i][j][4 * g + 2], acc[i][j][4 * g + 3]});
   }
 }
@@ -157,7 +164,7 @@ static void tile(const GemmArgs& a, hipStream_t s) {
   constexpr int lds = 2 * (BM + BN) * 64 * 2 > BM * (BN + 8) * 2 ? 2 * (BM + BN) * 64 * 2 : BM * (BN + 8) * 2;
   auto go = [&](auto k) {
     (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-    k<<<grid, WM * WN * 64, lds, s>>>(a);
+    k<<<dim3(grid, a.splits > 1 ? a.splits : 1), WM * WN * 64, lds, s>>>(a);
   };
   if (a.out_f32) go(gemm_tile_kernel<float, BM, BN, WM, WN>);
   else go(gemm_tile_kernel<bf16_t, BM, BN, WM, WN>);
@@ -165,9 +172,12 @@ static void tile(const GemmArgs& a, hipStream_t s) {
 }
 
 void launch_gemm_tile(const GemmArgs& a, hipStream_t s) {
-  // 256 x 256 tiles (8 waves) once they fill the chip, 128 x 128 (4 waves, two workgroups per CU) below
-  const bool big = a.tiles ? a.bm == 256 : (long)((a.M + 255) / 256) * ((a.N + 255) / 256) >= 192;
+  // 256 x 256 tiles (8 waves) once they fill the chip, 128 x 128 (4 waves, two workgroups per CU) below, 64 x 64 where
+  // those would leave most of it idle
+  const long m128 = (a.M + 127) / 128, n128 = (a.N + 127) / 128;
+  const bool big = a.tiles ? a.bm == 256 : a.splits <= 1 && (long)((a.M + 255) / 256) * ((a.N + 255) / 256) >= 192;
   if (big) tile<256, 256, 2, 4>(a, s);
+  else if (!a.tiles && a.splits <= 1 && m128 * n128 < 256 && a.K <= 2048) tile<64, 64, 2, 2>(a, s);
   else tile<128, 128, 2, 2>(a, s);
 }
 

@@ -30,7 +30,7 @@ MAX_TAPS = 16                # convolution taps
 MAX_LATENT = 1024            # columns of a cached latent
 LATENT_SHORT = 16            # portions up to this many rows attend in latent space, longer ones expand keys and values
 LATENT_GROUP_ROWS = 1 << 18  # context rows that are expanded at a time
-PARTS, PARTS_ROWS, PARTS_COLUMNS = 4, 64, 8192   # partial sums of decode products
+PARTS, PARTS_COLUMNS = 4, 8192   # partial sums: at most so many, of products up to so wide in a decode step
 SCAN_CHUNK, SCAN_MAX_CHUNKS = 64, 64
 
 
@@ -135,12 +135,17 @@ def matmul_with_side(a, w, side: int, epi: int = EPI_NONE, param: float = 0.0):
 
 
 def matmul_parts(a, w, out_dtype=None):
-    """a w^T for a consumer that adds partial sums (:func:`residual_norm`, :func:`latent_prep`): [parts, M, N] fp32 for a
-    few rows of a narrow product, which needs K cut up to fill the chip; else :func:`matmul`."""
+    """a w^T for a consumer that adds partial sums (:func:`residual_norm`, :func:`latent_prep`): [parts, M, N] fp32
+    where the product needs K cut up to fill the chip (few rows, few columns); else :func:`matmul`."""
     M, K, N = a.shape[0], a.shape[1], w.shape[0]
-    if not a.is_cuda or a.dtype != torch.bfloat16 or M > PARTS_ROWS or N > PARTS_COLUMNS or K < PARTS * 128:
+    if M <= 64:
+        parts = PARTS if N <= PARTS_COLUMNS and K >= PARTS * 128 else 1
+    else:   # tiles of 128 x 128: two for each of the 256 CUs
+        tiles = -(-M // 128) * (-(-N // 128))
+        parts = min(PARTS, 512 // tiles, K // 512) if tiles < 256 else 1
+    if not a.is_cuda or a.dtype != torch.bfloat16 or parts <= 1:
         return matmul(a, w, out_dtype)
-    c = torch.empty(PARTS, M, N, dtype=torch.float32, device=a.device)
+    c = torch.empty(parts, M, N, dtype=torch.float32, device=a.device)
     _K().lm_gemm_parts(a, w, c)
     return c
 
@@ -419,7 +424,8 @@ def mingru_scan(zx, g, bias, state, batch):
         return ref.mingru_scan(zx, g, bias, state, batch)
     out = torch.empty_like(g)
     max_q = int(batch.S) if batch.is_prefill else 1
-    n = -(-max_q // (SCAN_CHUNK * SCAN_MAX_CHUNKS)) * SCAN_CHUNK
+    least = SCAN_CHUNK if g.shape[0] > 4096 else SCAN_CHUNK // 2
+    n = -(-max_q // (least * SCAN_MAX_CHUNKS)) * least
     chunks = -(-max_q // n)
     ws = torch.empty(batch.B * chunks * 2 * g.shape[1] if chunks > 1 else 0, dtype=torch.float32, device=g.device)
     _K().mingru_scan(zx, g, bias, state, out, batch.positions, batch.q_start, batch.q_lens, batch.state_slots, ws, max_q, n)

@@ -117,7 +117,8 @@ def check_matmul(device, dtype):
             y, side = lm.matmul_with_side(ad, wd[:rows].contiguous(), rows - main)
             close(y, ref[:, :main], tol, "main")
             close(side, ref[:, main:rows], 3e-4, "side")
-    for m, n, k in ((1, 64, 512), (16, 70, 576), (30, 640, 1024), (64, 3000, 640), (50, 130, 832)):
+    for m, n, k in ((1, 64, 512), (16, 70, 576), (30, 640, 1024), (64, 3000, 640), (50, 130, 832), (65, 200, 1024),
+                    (300, 520, 1088), (1000, 128, 2112)):
         a = torch.randn(m, k, generator=g).to(dtype)
         w = (torch.randn(n, k, generator=g) / k ** 0.5).to(dtype)
         y = lm.matmul_parts(a.to(device), w.to(device))
