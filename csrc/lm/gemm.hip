@@ -7,9 +7,9 @@
 // pair of W is folded in registers.  A k-step covers 64 values; lane group g = lane / 16 takes values 16 g .. 16 g + 15
 // of it in both operands (the order of k inside a dot product is free), i.e. every W row is read 128 bytes at a time.
 //
-// Dense: row tiles of A are blockIdx.y, products of a batch (one per attention head, say) or
-// parts of K (partial sums for the consumer to add) blockIdx.z.  Grouped (experts): blockIdx.y is an entry of the tile list and blockIdx.z a
-// 16 MT-row part of it; rows past the expert's last slot are computed on a clamped row and not stored.
+// Dense: row tiles of A are blockIdx.y, products of a batch (one per attention head, say) or parts of K (partial sums for
+// the consumer to add) blockIdx.z.  Grouped (experts): blockIdx.y is an entry of the tile list and blockIdx.z a 16 MT-row
+// part of it; rows past the expert's last slot are computed on a clamped row and not stored.
 #include "lm_device.h"
 #include "lm.h"
 
@@ -134,8 +134,8 @@ __global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) 
   }
 }
 
-// Workgroup shapes (16 MT rows of A x 16 NT rows of W, NW waves along K, D k-steps in flight), from a sweep at decode sizes: enough
-// workgroups to fill the chip come first, then fewer passes over W (MT), then fewer re-reads of A (NT).
+// Workgroup shapes (16 MT rows of A x 16 NT rows of W, NW waves along K, D k-steps in flight), from a sweep at decode
+// sizes: enough workgroups to fill the chip come first, then fewer passes over W (MT), then fewer re-reads of A (NT).
 template <typename T, typename O>
 static void stream(const GemmArgs& a, hipStream_t s) {
   auto go = [&](auto kernel, int mt, int nt, int nw) {

@@ -1,6 +1,6 @@
 // Launchers of the decoder-block kernels (libshai_lm.so): decoders with an fp32 residual stream, mixture-of-experts
-// layers, chunked and latent attention, and gated recurrences.  Every kernel takes bf16 or fp32 weights / activations (`f32`); norms, routing, scores
-// and the residual are fp32 in both.  The model width is padded to a multiple of 64 by the caller.
+// layers, chunked and latent attention, and gated recurrences.  Every kernel takes bf16 or fp32 weights / activations
+// (`f32`); norms, routing, scores, recurrent state and the residual are fp32 in both.  The model width is padded to a multiple of 64 by the caller.
 #pragma once
 #include <hip/hip_runtime.h>
 #include <stdint.h>

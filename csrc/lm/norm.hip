@@ -221,8 +221,10 @@ __global__ void __launch_bounds__(NT, conv_waves(TAPS, NT, NV)) residual_norm_ke
       for (int j = 0; j < TAPS - 1; ++j) {
         const bool in = j + 1 < p.taps && j + 1 > at && j + 1 <= pos && slot >= 0;
 #pragma unroll
-        for (int i = 0; i < NV; ++i)
-          hist[j][i] = in && i * NT * 4 + c0 < p.Dp ? load4(st + (long)(p.taps - 2 - j + at) * p.Dp + i * NT * 4 + c0) : zero;
+        for (int i = 0; i < NV; ++i) {
+          const int c = i * NT * 4 + c0;
+          hist[j][i] = in && c < p.Dp ? load4(st + (long)(p.taps - 2 - j + at) * p.Dp + c) : zero;
+        }
       }
     };
     int seq = -1;

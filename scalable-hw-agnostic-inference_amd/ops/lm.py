@@ -232,7 +232,7 @@ def chunk_attention(qkvg, k_cache, v_cache, batch, heads: int, chunk: int, scale
     return o
 
 
-# ---------------------------------------------------------------------------------------------- normed residual, convolution
+# ------------------------------------------------------------------------------------------- normed residual, convolution
 class Embedding(NamedTuple):
     """Residual source of a model's first norm: rows table[ids] * scale."""
     ids: torch.Tensor
@@ -254,7 +254,8 @@ def residual_norm(source, delta, wb, mult: float, step, w, eps: float, width: in
                   batch=None, rows=None, keep: bool = True):
     """x = source (+ mult * RMSNorm(delta) wb) (+ step); h = RMSNorm(x) w, plus its convolution with ``conv``.
 
-    source: the fp32 residual [T, D] or an :class:`Embedding`.  delta: [T, D], or partial sums [parts, T, D] fp32.  Returns (x, h); the residual may be updated in place.
+    source: the fp32 residual [T, D] or an :class:`Embedding`.  delta: [T, D], or partial sums
+    [parts, T, D] fp32.  Returns (x, h); the residual may be updated in place.
     ``w`` None: no norm (h None).  ``rows`` (int32): h of these rows only, and with ``keep`` False x is None."""
     emb = isinstance(source, Embedding)
     if not (source.ids if emb else source).is_cuda:
@@ -373,8 +374,8 @@ def latent_plan(batch, expand: bool) -> LatentPlan:
 
 
 def latent_prep(d, wq, wkv, rope, batch, cache, eps: float, q_rank: int, kv_rank: int):
-    """The down projection's fp32 rows [q latent | kv latent | rotated key part] (each padded; or partial sums): norms both latents, turns
-    the key part, writes [kv latent | key part] to ``cache`` [blocks, 64, ..] at batch.slots.  Returns the normed q latent
+    """The down projection's fp32 rows [q latent | kv latent | rotated key part] (each padded; or partial sums):
+    norms both latents, turns the key part, writes [kv latent | key part] to ``cache`` [blocks, 64, ..] at batch.slots.  Returns the normed q latent
     in the cache's dtype."""
     if not d.is_cuda:
         return ref.latent_prep(d, wq, wkv, rope, batch, cache, eps, q_rank, kv_rank)

@@ -5,7 +5,7 @@ import copy
 import decoder_cases
 import faledra_reference as R
 import torch
-from decoder_cases import (F32_TOL, assert_logits, check_replay_files, greedy_oracle, name,  # noqa: F401
+from decoder_cases import (F32_TOL, check_replay_files, greedy_oracle, name,  # noqa: F401
                            position_errors, replay_lines, run, run_batches)
 
 from shai_amd.engines.llm import LLMEngine, SamplingParams
@@ -15,6 +15,12 @@ from shai_amd.models.registry import config_from_json
 from shai_amd.ops import lm
 
 JUNK = 37.0                      # what caches and state slots hold before anything is written
+
+
+def assert_logits(got, want, dtype, what=""):
+    """Every position (nothing in this design turns a rounding error into a jump)."""
+    e = position_errors(got, want)
+    assert e.max() < (F32_TOL if dtype == torch.float32 else 0.03), f"{what}: {e.max():.2e} at {int(e.argmax())}"
 
 
 class Case(decoder_cases.Case):
@@ -453,7 +459,7 @@ def check_long_decode(tmp, device, dtype):
 def check_batches(tmp, device, dtype):
     c = Case(tmp, device, dtype, seed=6)
     eng = c.engine(512)
-    run_batches(c, eng, {f"q{i}": c.tokens(n) for i, n in enumerate((130, 1, 75, 64, 2, 190, 33, 128))})
+    run_batches(c, eng, {f"q{i}": c.tokens(n) for i, n in enumerate((130, 1, 75, 64, 2, 190, 33, 128))}, assert_logits)
     assert eng.state_slots.num_free == eng.max_num_seqs
 
 
