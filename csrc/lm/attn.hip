@@ -1,9 +1,12 @@
-// Attention inside fixed-size chunks of the sequence, over a paged cache ([blocks, G, 64, dk | dv]).
+// Attention inside fixed-size chunks of the sequence or inside a sliding window, over a paged cache
+// ([blocks, G, 64, dk | dv]).
 //
-// Position i sees the keys lo .. i with lo = i - i % chunk; scores are (q . k) * scale, softmaxed in fp32, and every
-// head's output is multiplied by sigmoid(its gate logit).  The rows of a step are [q | k | v | gate] (one GEMM).
+// Position i sees the keys lo .. i with lo = i - i % chunk or, with a window, i - chunk + 1; scores are (q . k) * scale,
+// softmaxed in fp32, and the output is multiplied by sigmoid of a gate logit per head or per element.  The rows of a step
+// are [q | k | v | gate] (one GEMM), or [q | gate] where another layer has written the cache.
 //
 // kv_store      the step's k / v rows into the cache.
+// head_prep     the same with q and k rotated by position and divided by their root mean square (q in place).
 // prefill       bf16: flash attention, 4 waves x 32 queries, scores swapped (S^T = K Q^T) so that a lane holds one
 //               query's scores; P feeds O^T = V^T P^T from registers as a bf16 pair (value + remainder, 16 significant
 //               bits).  Only the 64-key blocks of the chunks that the workgroup's queries lie in are visited.
@@ -11,7 +14,8 @@
 //               cached latents: plain causal, no gate, a sink per head in the denominator.
 // decode        bf16: one workgroup per (sequence, kv head, split); each wave takes whole 64-key blocks, K straight from
 //               memory into the matrix cores (the group's query heads are the 16 columns), fp32 P against V on the
-//               VALU; the new token's k / v are written to the cache by the workgroup that reads them.
+//               VALU; the new token's k / v are written to the cache by the workgroup that reads them.  With rotation
+//               and norm of q and k (PREP) every workgroup prepares its query heads in LDS first.
 // attn_rows     fp32 (any sizes): one wave per (row, head), plain online softmax.
 #include "lm_device.h"
 
@@ -19,6 +23,11 @@ namespace shai_lm {
 
 typedef short s4v __attribute__((ext_vector_type(4)));
 constexpr float kLog2e = 1.4426950408889634f;
+
+// the first key that position pos sees
+__device__ __forceinline__ int first_key(const AttnArgs& p, int pos) {
+  return p.window ? max(0, pos - p.chunk + 1) : pos - pos % p.chunk;
+}
 
 template <typename T>
 __global__ void __launch_bounds__(256) kv_store_kernel(const AttnArgs p) {
@@ -43,6 +52,93 @@ void launch_kv_store(const AttnArgs& a, bool f32, hipStream_t s) {
   SHAI_CHECK_LAUNCH();
 }
 
+// 8 consecutive elements
+__device__ __forceinline__ void load8(const bf16_t* p, float* x) { unpack8(*reinterpret_cast<const uint4_*>(p), x); }
+__device__ __forceinline__ void load8(const float* p, float* x) {
+  *reinterpret_cast<float4_*>(x) = load4(p);
+  *reinterpret_cast<float4_*>(x + 4) = load4(p + 4);
+}
+__device__ __forceinline__ void store8(bf16_t* p, const float* x) { *reinterpret_cast<uint4_*>(p) = pack8(x); }
+__device__ __forceinline__ void store8(float* p, const float* x) {
+  store4(p, *reinterpret_cast<const float4_*>(x));
+  store4(p + 4, *reinterpret_cast<const float4_*>(x + 4));
+}
+
+// One head by n / 8 lanes of a wave, lane j holding elements 8 j .. 8 j + 7: dimension i < rot / 2 turned with i + rot / 2 by
+// the row's angles, then the head divided by its root mean square over `dim` (the pads behind are zero).  `stage`: n
+// floats of LDS.  Every lane of the wave calls it.
+__device__ __forceinline__ void turn_and_norm(float (&x)[8], float* stage, const float* rope, int rot, int dim, float eps,
+                                              int j, int lanes) {
+  const int half = rot >> 1;
+  store8(stage + 8 * j, x);
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int e = 8 * j + i;
+    if (e < rot) {
+      const bool low = e < half;
+      const float other = stage[low ? e + half : e - half];
+      const float* t = rope + 2 * (low ? e : e - half);
+      x[i] = x[i] * t[0] + (low ? -other : other) * t[1];
+    }
+    ss += x[i] * x[i];
+  }
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  for (int o = lanes >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+  const float r = 1.f / sqrtf(ss / (float)dim + eps);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) x[i] *= r;
+}
+
+template <typename T, int DK>
+__global__ void __launch_bounds__(256) head_prep_kernel(const AttnArgs p) {
+  constexpr int LPH = DK / 8, HP = 256 / LPH;    // lanes per head, heads at a time
+  __shared__ __attribute__((aligned(16))) float stage[HP][DK];
+  __shared__ __attribute__((aligned(16))) float angle[DK];
+  const long t = blockIdx.x;
+  const int tid = threadIdx.x, slot = p.slots[t];
+  T* row = const_cast<T*>(static_cast<const T*>(p.qkvg)) + t * p.ld;
+  for (int i = tid; i < p.rot; i += 256) angle[i] = p.rope[t * p.rot + i];
+  __syncthreads();
+  const int n = p.H + (p.own_kv && slot >= 0 ? p.G : 0), j = tid % LPH, blk = slot >> 6, in = slot & 63;
+  for (int h0 = 0; h0 < n; h0 += HP) {
+    const int h = h0 + tid / LPH;
+    float x[8];
+    load8(row + (long)min(h, n - 1) * DK + 8 * j, x);
+    turn_and_norm(x, stage[tid / LPH], angle, p.rot, p.dim, p.eps, j, LPH);
+    if (h < p.H) store8(row + (long)h * DK + 8 * j, x);
+    else if (h < n) store8(static_cast<T*>(p.kc) + (((long)blk * p.G + h - p.H) * 64 + in) * DK + 8 * j, x);
+  }
+  if (n == p.H) return;
+  const T* v = row + (long)(p.H + p.G) * DK;
+  for (int i = tid; i < p.G * p.dv / 8; i += 256) {
+    const int e = 8 * i, g = e / p.dv;
+    float x[8];
+    load8(v + e, x);
+    store8(static_cast<T*>(p.vc) + (((long)blk * p.G + g) * 64 + in) * p.dv + (e - g * p.dv), x);
+  }
+}
+
+template <typename T>
+static void head_prep(const AttnArgs& a, hipStream_t s) {
+  if (a.dk == 64) head_prep_kernel<T, 64><<<a.T, 256, 0, s>>>(a);
+  else if (a.dk == 128) head_prep_kernel<T, 128><<<a.T, 256, 0, s>>>(a);
+  else head_prep_kernel<T, 256><<<a.T, 256, 0, s>>>(a);
+}
+
+void launch_head_prep(const AttnArgs& a, bool f32, hipStream_t s) {
+  if (f32) head_prep<float>(a, s);
+  else head_prep<bf16_t>(a, s);
+  SHAI_CHECK_LAUNCH();
+}
+
+// the step's keys and values into the cache (and, with rotation and norm, the queries prepared in place)
+static void store_step(const AttnArgs& a, bool f32, hipStream_t s) {
+  if (a.rope) launch_head_prep(a, f32, s);
+  else if (a.own_kv) launch_kv_store(a, f32, s);
+}
+
 // ------------------------------------------------------------------------------------------------ any-size rows
 template <typename T>
 __global__ void __launch_bounds__(256) attn_rows_kernel(const AttnArgs p) {
@@ -53,7 +149,7 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(const AttnArgs p) {
   const int q_len = p.q_lens ? p.q_lens[b] : 1;
   if (i >= q_len || h >= p.H) return;            // whole waves: no barrier below, only wave-local LDS
   const long t = (p.q_lens ? p.q_start[b] : b) + i;
-  const int pos = p.ctx[b] - q_len + i, lo = pos - pos % p.chunk;
+  const int pos = p.ctx[b] - q_len + i, lo = first_key(p, pos);
   const int g = h / (p.H / p.G);
   const T* row = static_cast<const T*>(p.qkvg) + t * p.ld;
   for (int d = lane; d < p.dk; d += 64) sq[w][d] = load1(row + (long)h * p.dk + d);
@@ -91,11 +187,13 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(const AttnArgs p) {
     }
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
   }
-  const float gate = sigmoid_f(load1(row + (long)p.H * p.dk + (long)p.G * (p.dk + p.dv) + h)) / l;
+  const T* gate = row + p.gate_off + (long)h * p.gate_w;
   T* out = static_cast<T*>(p.o) + t * (long)p.H * p.dv + (long)h * p.dv;
 #pragma unroll
-  for (int c = 0; c < 4; ++c)
-    if (lane + 64 * c < p.dv) store1(out + lane + 64 * c, o[c] * gate);
+  for (int c = 0; c < 4; ++c) {
+    const int col = lane + 64 * c;
+    if (col < p.dv) store1(out + col, o[c] * (sigmoid_f(load1(gate + (p.gate_w > 1 ? col : 0))) / l));
+  }
 }
 
 // ------------------------------------------------------------------------------------------------ prefill (bf16)
@@ -124,7 +222,7 @@ __global__ void __launch_bounds__(256, DK + DV > (LAT ? 320 : 256) ? 1 : 2) attn
   const int q_len = p.q_lens[b], q0 = blockIdx.x * 128;
   if (q0 >= q_len) return;
   const int ctx = p.ctx[b], c_off = ctx - q_len;
-  const int qi = q0 + wid * 32 + fr, pos = qi + c_off, lo = LAT ? 0 : pos - pos % p.chunk;
+  const int qi = q0 + wid * 32 + fr, pos = qi + c_off, lo = LAT ? 0 : first_key(p, pos);
   const long row0 = p.q_start[b];
   const bf16_t* rows = static_cast<const bf16_t*>(p.qkvg) + row0 * p.ld;
 
@@ -135,10 +233,10 @@ __global__ void __launch_bounds__(256, DK + DV > (LAT ? 320 : 256) ? 1 : 2) attn
     for (int s = 0; s < NS; ++s)
       qf[s] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4_*>(qp + 16 * s + 8 * fh));
   }
-  // blocks from the first query's chunk to the last query's position
+  // blocks from the first query's first key to the last query's position
   const int p_first = q0 + c_off, p_last = min(q0 + 127, q_len - 1) + c_off;
-  const int t0 = LAT ? 0 : (p_first - p_first % p.chunk) >> 6, t1 = (p_last >> 6) + 1;
-  const int lo_last = LAT ? 0 : p_last - p_last % p.chunk;
+  const int t0 = LAT ? 0 : first_key(p, p_first) >> 6, t1 = (p_last >> 6) + 1;
+  const int lo_last = LAT ? 0 : first_key(p, p_last);
 
   // LAT: keys and values go to LDS by DMA, the bank swizzle applied to the source.  Rows past the context repeat the last
   // one (their scores are masked); columns past a key's parts hold other finite values (the queries are zero there).
@@ -320,14 +418,24 @@ __global__ void __launch_bounds__(256, DK + DV > (LAT ? 320 : 256) ? 1 : 2) attn
       const float sk = p.sink[h] * kLog2e, top = fmaxf(m_run, sk), a = __builtin_amdgcn_exp2f(m_run - top);
       inv = a / (l_tot * a + __builtin_amdgcn_exp2f(sk - top));
     } else {
-      inv = sigmoid_f(bf2f(rows[(long)qi * p.ld + (long)p.H * DK + (long)p.G * (DK + DV) + h])) / l_tot;
+      inv = (p.gate_w > 1 ? 1.f : sigmoid_f(bf2f(rows[(long)qi * p.ld + p.gate_off + h]))) / l_tot;
     }
     bf16_t* op = static_cast<bf16_t*>(p.o) + (row0 + qi) * (long)p.H * DV + (long)h * DV;
 #pragma unroll
     for (int d = 0; d < ND; ++d)
 #pragma unroll
-      for (int g = 0; g < 4; ++g)
-        store4(op + d * 32 + 8 * g + 4 * fh, float4_{o[d][4 * g], o[d][4 * g + 1], o[d][4 * g + 2], o[d][4 * g + 3]} * inv);
+      for (int g = 0; g < 4; ++g) {
+        const int col = d * 32 + 8 * g + 4 * fh;
+        float4_ y = float4_{o[d][4 * g], o[d][4 * g + 1], o[d][4 * g + 2], o[d][4 * g + 3]} * inv;
+        if constexpr (!LAT) {
+          if (p.gate_w > 1) {
+            const float4_ z = load4(rows + (long)qi * p.ld + p.gate_off + (long)h * DV + col);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) y[i] *= sigmoid_f(z[i]);
+          }
+        }
+        store4(op + col, y);
+      }
   }
 }
 
@@ -366,12 +474,14 @@ void launch_attn_prefill(const AttnArgs& a, bool f32, hipStream_t s) {
 // ------------------------------------------------------------------------------------------------ decode (bf16)
 // One workgroup: kv head g's query heads h0 .. h0 + R - 1 (R <= 16, RH = R rounded up) of sequence b, one split of the
 // visible 64-key blocks.  Wave w takes blocks w, w + 4, ... of the split.
-template <int DK, int DV, int RH>
+template <int DK, int DV, int RH, bool PREP>
 __global__ void __launch_bounds__(256) attn_decode_kernel(const AttnArgs p, int per_group, int store) {
   constexpr int LPK = DV / 8, KP = 64 / LPK, IT = 64 / KP;   // V: LPK lanes per key, KP keys at a time
   constexpr int VB = IT > 16 ? 16 : IT;                      // V loads in flight
   __shared__ float sp[4][64][RH];
-  __shared__ float so[4][RH][DV];
+  __shared__ __attribute__((aligned(16))) float so[4][RH][DV];
+  __shared__ __attribute__((aligned(16))) bf16_t sq[PREP ? RH : 1][PREP ? DK : 8];
+  static_assert(!PREP || 4 * RH * DV >= (RH + 1) * DK, "prepared heads are staged in so");
   __shared__ float sm[4][16], sl[4][16];
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
   const int c = lane & 15, q4 = lane >> 4;
@@ -379,7 +489,7 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(const AttnArgs p, int 
   const int g = blockIdx.x / parts, part = blockIdx.x % parts;
   const int b = blockIdx.y, split = blockIdx.z;
   const int h0 = g * group + part * per_group, R = min(per_group, group - part * per_group);
-  const int pos = p.ctx[b] - 1, lo = pos - pos % p.chunk;
+  const int pos = p.ctx[b] - 1, lo = first_key(p, pos);
   const int b0 = lo >> 6, b1 = (pos >> 6) + 1;
   const int per = (b1 - b0 + p.splits - 1) / p.splits;
   const int s0 = b0 + split * per, s1 = min(b1, s0 + per);
@@ -393,9 +503,24 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(const AttnArgs p, int 
     const long cell = ((long)(slot >> 6) * p.G + g) * 64 + (slot & 63);
     const bf16_t* kn = row + (long)p.H * DK + (long)g * DK;
     const bf16_t* vn = row + (long)p.H * DK + (long)p.G * DK + (long)g * DV;
-    if (tid < DK / 8) reinterpret_cast<uint4_*>(kc + cell * DK)[tid] = reinterpret_cast<const uint4_*>(kn)[tid];
-    else if (tid >= 64 && tid - 64 < DV / 8)
+    if (tid < DK / 8) {
+      if constexpr (!PREP) reinterpret_cast<uint4_*>(kc + cell * DK)[tid] = reinterpret_cast<const uint4_*>(kn)[tid];
+    } else if (tid >= 64 && tid - 64 < DV / 8)
       reinterpret_cast<uint4_*>(vc + cell * DV)[tid - 64] = reinterpret_cast<const uint4_*>(vn)[tid - 64];
+  }
+  if constexpr (PREP) {                          // the heads of this workgroup, and k where it is stored
+    constexpr int LPH = DK / 8, HP = 256 / LPH;
+    const bool key = store && slot >= 0 && s1 == b1 && s0 < s1;
+    const int n = R + key, j = tid % LPH;
+    for (int i0 = 0; i0 < n; i0 += HP) {
+      const int i = i0 + tid / LPH, ii = min(i, n - 1);
+      float x[8];
+      load8(row + (long)(ii < R ? h0 + ii : p.H + g) * DK + 8 * j, x);
+      // the spare lanes repeat the last head with the same values
+      turn_and_norm(x, &so[0][0][0] + ii * DK, p.rope + (long)b * p.rot, p.rot, p.dim, p.eps, j, LPH);
+      if (i < R) store8(&sq[i][8 * j], x);
+      else if (i < n) store8(kc + (((long)(slot >> 6) * p.G + g) * 64 + (slot & 63)) * DK + 8 * j, x);
+    }
   }
   __syncthreads();
 
@@ -404,7 +529,8 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(const AttnArgs p, int 
   for (int s = 0; s < DK / 64; ++s)
 #pragma unroll
     for (int u = 0; u < 2; ++u)
-      qf[s][u] = c < R ? *reinterpret_cast<const uint4_*>(row + (long)(h0 + c) * DK + 64 * s + 16 * q4 + 8 * u)
+      qf[s][u] = c < R ? *reinterpret_cast<const uint4_*>((PREP ? &sq[min(c, RH - 1)][0] : row + (long)(h0 + c) * DK) +
+                                                          64 * s + 16 * q4 + 8 * u)
                        : uint4_{0u, 0u, 0u, 0u};
   float o[RH][8];
 #pragma unroll
@@ -517,7 +643,7 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(const AttnArgs p, int 
       }
     }
     if (p.splits == 1) {
-      const float gate = bf2f(row[(long)p.H * DK + (long)p.G * (DK + DV) + h]);
+      const float gate = bf2f(row[p.gate_off + (long)h * p.gate_w + (p.gate_w > 1 ? d : 0)]);
       static_cast<bf16_t*>(p.o)[((long)b * p.H + h) * DV + d] = f2bf(x / L * sigmoid_f(gate));
     } else {
       float* ws = p.ws + (((long)b * p.H + h) * p.splits + split) * (DV + 2);
@@ -550,31 +676,41 @@ __global__ void __launch_bounds__(256) attn_decode_fold_kernel(const AttnArgs p)
 #pragma unroll 8
   for (int s = 0; s < p.splits; ++s) x += ws[(long)s * (p.dv + 2) + d] * se[s];
   const float L = total;
-  const float gate = bf2f(static_cast<const bf16_t*>(p.qkvg)[(long)b * p.ld + (long)p.H * p.dk +
-                                                             (long)p.G * (p.dk + p.dv) + h]);
+  const float gate = bf2f(static_cast<const bf16_t*>(p.qkvg)[(long)b * p.ld + p.gate_off + (long)h * p.gate_w +
+                                                             (p.gate_w > 1 ? d : 0)]);
   static_cast<bf16_t*>(p.o)[((long)b * p.H + h) * p.dv + d] = f2bf(x / L * sigmoid_f(gate));
+}
+
+template <int DK, int DV, bool PREP>
+static void decode_heads(const AttnArgs& a, hipStream_t s) {
+  const int group = a.H / a.G;
+  // heads per workgroup: 16 columns, 8 at the largest head size (LDS); more heads take several workgroups
+  constexpr int MAXR = DV > 128 ? 8 : 16;
+  const int per = group < MAXR ? group : MAXR, parts = (group + per - 1) / per;
+  const dim3 grid(a.G * parts, a.B, a.splits);
+  const int store = parts == 1 && a.own_kv;
+  if (per == 1) attn_decode_kernel<DK, DV, 1, PREP><<<grid, 256, 0, s>>>(a, per, store);
+  else if (per <= 4) attn_decode_kernel<DK, DV, 4, PREP><<<grid, 256, 0, s>>>(a, per, store);
+  else if (per <= 8) attn_decode_kernel<DK, DV, 8, PREP><<<grid, 256, 0, s>>>(a, per, store);
+  else if constexpr (DV <= 128) attn_decode_kernel<DK, DV, 16, PREP><<<grid, 256, 0, s>>>(a, per, store);
+  if (a.splits > 1) attn_decode_fold_kernel<<<dim3(a.H, a.B), 256, 0, s>>>(a);
 }
 
 template <int DK, int DV>
 static void decode(const AttnArgs& a, hipStream_t s) {
-  const int group = a.H / a.G;
-  // heads per workgroup: 16 columns, 8 at the largest head size (LDS); more heads take several workgroups, and the
-  // cache write is then a launch of its own (no single workgroup reads the new row)
-  constexpr int MAXR = DV > 128 ? 8 : 16;
-  const int per = group < MAXR ? group : MAXR, parts = (group + per - 1) / per;
-  if (parts > 1) launch_kv_store(a, false, s);
-  const dim3 grid(a.G * parts, a.B, a.splits);
-  const int store = parts == 1;
-  if (per == 1) attn_decode_kernel<DK, DV, 1><<<grid, 256, 0, s>>>(a, per, store);
-  else if (per <= 4) attn_decode_kernel<DK, DV, 4><<<grid, 256, 0, s>>>(a, per, store);
-  else if (per <= 8) attn_decode_kernel<DK, DV, 8><<<grid, 256, 0, s>>>(a, per, store);
-  else if constexpr (DV <= 128) attn_decode_kernel<DK, DV, 16><<<grid, 256, 0, s>>>(a, per, store);
-  if (a.splits > 1) attn_decode_fold_kernel<<<dim3(a.H, a.B), 256, 0, s>>>(a);
+  if (a.H / a.G > (DV > 128 ? 8 : 16)) {         // no single workgroup reads the new row: its own launch
+    store_step(a, false, s);
+    decode_heads<DK, DV, false>(a, s);
+  } else if (a.rope) {
+    decode_heads<DK, DV, true>(a, s);
+  } else {
+    decode_heads<DK, DV, false>(a, s);
+  }
 }
 
 void launch_attn_decode(const AttnArgs& a, bool f32, hipStream_t s) {
   if (f32) {
-    launch_kv_store(a, true, s);
+    store_step(a, true, s);
     attn_rows_kernel<float><<<dim3(1, (a.H + 3) / 4, a.B), 256, 0, s>>>(a);
   } else {
     SHAI_LM_HEADS(decode, a, s);

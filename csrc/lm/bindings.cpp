@@ -134,7 +134,7 @@ void add_norm(const Tensor& x, const optional<Tensor>& dense, const optional<Ten
 void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<Tensor>& tiles,
              const optional<Tensor>& offsets, const optional<Tensor>& gather, int64_t bm, int64_t epi, double param,
              const optional<Tensor>& side, const optional<Tensor>& vec, const optional<Tensor>& rope, int64_t head,
-             int64_t rot0) {
+             int64_t rot0, const optional<Tensor>& ids, const optional<Tensor>& table) {
   const bool f32 = is_f32(A);
   SHAI_CHECK(A.is_cuda() && A.dim() == 2 && A.stride(1) == 1 && A.stride(0) % 8 == 0 && A.stride(0) >= A.size(1) &&
                  reinterpret_cast<uintptr_t>(A.data_ptr()) % 16 == 0, "A rows must be contiguous and 16-byte aligned");
@@ -150,21 +150,22 @@ void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<T
   g.param = param;
   g.out_f32 = C.scalar_type() == at::kFloat;
   SHAI_CHECK(A.size(1) == g.K && g.K % 64 == 0 && g.N >= 1, "lm_gemm: K must match and be a multiple of 64");
-  SHAI_CHECK(epi >= 0 && epi <= 4, "lm_gemm epilogue");
+  SHAI_CHECK(epi >= 0 && epi <= 7, "lm_gemm epilogue");
+  const bool glu = shai_lm::glu_epi(epi);
   g.n_main = g.N;
   g.lda = A.stride(0);
   g.batch = 1;
   if (side) {  // the last rows of W are a plain product, stored in fp32
     check(*side, at::kFloat, "side");
-    SHAI_CHECK(!tiles && (epi == shai_lm::EPI_CLAMP_GLU || epi == shai_lm::EPI_NONE) && side->dim() == 2 &&
+    SHAI_CHECK(!tiles && (glu || epi == shai_lm::EPI_NONE) && side->dim() == 2 &&
                    side->size(0) == g.M && side->size(1) >= 1 && side->size(1) < g.N,
                "side output: dense plain or GLU products, [M, last rows of W]");
     g.n_main = g.N - side->size(1);
     SHAI_CHECK(g.n_main % 4 == 0, "side output: the other rows of W must be a multiple of 4");
     g.side = side->data_ptr<float>();
   }
-  SHAI_CHECK(epi != shai_lm::EPI_CLAMP_GLU || g.n_main % 2 == 0, "GLU products need (gate, up) row pairs");
-  g.ldc = epi == shai_lm::EPI_CLAMP_GLU ? g.n_main / 2 : g.n_main;
+  SHAI_CHECK(!glu || g.n_main % 2 == 0, "GLU products need (gate, up) row pairs");
+  g.ldc = glu ? g.n_main / 2 : g.n_main;
   SHAI_CHECK(C.size(1) == g.ldc, "lm_gemm output columns");
   if (epi == shai_lm::EPI_XIELU) {
     SHAI_CHECK(vec.has_value() && vec->numel() == 2, "the xIELU epilogue needs its two coefficients");
@@ -180,6 +181,19 @@ void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<T
     g.rot0 = rot0;
     SHAI_CHECK(g.rot % 2 == 0 && rot0 % 4 == 0 && rot0 >= 0 && head % 4 == 0 && rot0 + g.rot <= head && g.N % head == 0,
                "rotary epilogue: heads of ", head, " columns, the rotated ones from a multiple of 4");
+  }
+  if (epi == shai_lm::EPI_GELU_ROWS) {
+    SHAI_CHECK(ids.has_value() && table.has_value() && !tiles && ids->numel() >= g.M && table->is_cuda() &&
+                   table->scalar_type() == A.scalar_type() && table->dim() == 2 && table->size(0) >= 1 && table->size(1) == g.N &&
+                   table->stride(1) == 1 && table->stride(0) % 4 == 0 && g.N % 4 == 0 &&
+                   reinterpret_cast<uintptr_t>(table->data_ptr()) % 16 == 0,
+               "table rows: ids [M] and a table [rows, N] of the type of A, rows 4-element aligned");
+    check_i32(*ids, "ids");
+    g.ids = ids->data_ptr<int>();
+    g.table = table->data_ptr();
+    g.table_ld = table->stride(0);
+    g.table_rows = table->size(0);
+    g.table_f32 = f32;
   }
   g.A = A.data_ptr();
   g.W = W.data_ptr();
@@ -219,6 +233,7 @@ void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<T
       part.C = static_cast<char*>(g.C) + at * g.ldc * osize;
       if (g.side) part.side = g.side + (long)at * (g.N - g.n_main);
       if (g.rope) part.rope = g.rope + (long)at * g.rot;
+      if (g.ids) part.ids = g.ids + at;
     }
     shai_lm::launch_gemm_tile(part, stream());
   }
@@ -283,12 +298,14 @@ void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const
                    const optional<Tensor>& x_out, const optional<Tensor>& rows, const optional<Tensor>& w, double eps,
                    int64_t width, const optional<Tensor>& h, const optional<Tensor>& cw, const optional<Tensor>& state,
                    const optional<Tensor>& tail, const optional<Tensor>& row_seq, const optional<Tensor>& q_start,
-                   const optional<Tensor>& q_lens, const optional<Tensor>& pos, const optional<Tensor>& slots) {
+                   const optional<Tensor>& q_lens, const optional<Tensor>& pos, const optional<Tensor>& slots,
+                   const optional<Tensor>& bb, const optional<Tensor>& b, const optional<Tensor>& ye,
+                   const optional<Tensor>& slot_of, const optional<Tensor>& wts) {
   shai_lm::ResidualNormArgs a{};
   a.width = width;
   a.eps = eps;
   long R;
-  at::ScalarType dt = h ? h->scalar_type() : delta ? delta->scalar_type() : table ? table->scalar_type() : at::kFloat;
+  at::ScalarType dt = h ? h->scalar_type() : ye ? ye->scalar_type() : delta ? delta->scalar_type() : table ? table->scalar_type() : at::kFloat;
   SHAI_CHECK(dt == at::kFloat || dt == at::kBFloat16, "bf16 or fp32");
   SHAI_CHECK(x.has_value() != ids.has_value(), "residual_norm: a residual or token ids");
   if (x) {
@@ -324,10 +341,25 @@ void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const
     a.parts = many ? delta->size(0) : 0;
     a.part_stride = R * a.Dp;
   }
+  if (ye) {  // the weighted outputs of a token's experts
+    check(*ye, dt, "ye");
+    SHAI_CHECK(!delta && wb.has_value() && slot_of.has_value() && wts.has_value(), "expert outputs: the only delta, with slot_of, weights and gain");
+    check_i32(*slot_of, "slot_of");
+    check(*wts, at::kFloat, "wts");
+    a.top = slot_of->size(1);
+    SHAI_CHECK(slot_of->size(0) == R && wts->sizes() == slot_of->sizes() && ye->size(0) == R * a.top && ye->size(1) == a.Dp,
+               "expert outputs must be [rows * top, D]");
+    a.ye = ye->data_ptr();
+    a.slot_of = slot_of->data_ptr<int>();
+    a.wts = wts->data_ptr<float>();
+  }
   a.wb = row_vec(wb, "wb");
+  a.bb = row_vec(bb, "bb");
   a.mult = mult;
   a.step = row_vec(step, "step");
   a.w = row_vec(w, "w");
+  a.b = row_vec(b, "b");
+  SHAI_CHECK(!b || w.has_value(), "a norm's bias comes with its gain");
   if (x_out) {
     check(*x_out, at::kFloat, "x_out");
     SHAI_CHECK(x_out->size(0) == R && x_out->size(1) == a.Dp, "x_out must be [rows, D]");
@@ -335,12 +367,12 @@ void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const
   }
   if (rows) {
     check_i32(*rows, "rows");
-    SHAI_CHECK(!cw && w.has_value(), "rows selects rows to normalise");
+    SHAI_CHECK(!cw && h.has_value(), "rows selects rows of h");
     a.rows = rows->data_ptr<int>();
     a.T = rows->numel();
   }
-  if (w) {
-    SHAI_CHECK(h.has_value(), "a norm needs an output h");
+  SHAI_CHECK(!w || h.has_value(), "a norm needs an output h");
+  if (h) {
     check(*h, dt, "h");
     SHAI_CHECK(h->numel() == (long)a.T * a.Dp, "h must be [rows, D]");
     a.h = h->data_ptr();
@@ -349,8 +381,8 @@ void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const
     check(*cw, at::kFloat, "cw");
     SHAI_CHECK(cw->dim() == 2 && cw->size(1) == a.Dp && cw->size(0) >= 1 && cw->size(0) <= 16, "convolution: 1 to 16 taps");
     a.taps = cw->size(0);
-    SHAI_CHECK(w.has_value() && x_out.has_value() && (!x || x->data_ptr() != x_out->data_ptr()),
-               "convolution: needs the norm, and x_out apart from x");
+    SHAI_CHECK(h.has_value() && x_out.has_value() && (!x || x->data_ptr() != x_out->data_ptr()),
+               "convolution: needs an output h, and x_out apart from x");
     SHAI_CHECK(state.has_value() && pos.has_value() && slots.has_value() && pos->numel() >= R, "convolution: state, pos, slots");
     check(*state, at::kFloat, "state");
     check_i32(*pos, "pos");
@@ -614,7 +646,71 @@ void mingru_scan(const Tensor& zx, const Tensor& g, const Tensor& bias, const Te
   if (a.T > 0) shai_lm::launch_mingru_scan(a, f32, stream());
 }
 
-void moe_route(const Tensor& logits, int64_t groups, int64_t keep, const Tensor& ids, const Tensor& wts) {
+void hgrn2(const Tensor& qv, const Tensor& z, const Tensor& bias, const Tensor& lower, const Tensor& gain,
+           const Tensor& state, const Tensor& out, const Tensor& pos, const optional<Tensor>& q_start,
+           const optional<Tensor>& q_lens, const Tensor& slots, const Tensor& ws, int64_t max_q, int64_t len, int64_t vdim,
+           double eps) {
+  const bool f32 = is_f32(qv);
+  check(qv, qv.scalar_type(), "qv");
+  check(out, qv.scalar_type(), "out");
+  for (auto* t : {&z, &bias, &lower, &gain, &state}) check(*t, at::kFloat, "hgrn2 fp32 tensor");
+  check_i32(pos, "pos");
+  check_i32(slots, "slots");
+  shai_lm::Hgrn2Args a{};
+  SHAI_CHECK(qv.dim() == 2 && z.dim() == 2 && out.dim() == 2 && state.dim() == 4 && max_q >= 1 && len >= 32 && len % 32 == 0,
+             "hgrn2 ranks");
+  a.T = qv.size(0);
+  a.H = state.size(1);
+  a.dk = state.size(2);
+  a.dv = state.size(3);
+  SHAI_CHECK((a.dk == 64 && a.dv == 64) || (a.dk == 64 && a.dv == 128) || (a.dk == 128 && a.dv == 64) ||
+                 (a.dk == 128 && a.dv == 128) || (a.dk == 256 && a.dv == 256), "stored head sizes: 64 / 128 each, or 256 / 256");
+  SHAI_CHECK(a.H >= 1 && a.H <= 65535 && qv.size(1) == (long)a.H * (a.dk + a.dv) && z.size(0) == a.T && z.size(1) == (long)a.H * a.dk &&
+                 bias.numel() == (long)a.H * a.dk && lower.numel() == bias.numel() && gain.numel() == a.dv &&
+                 out.size(0) == a.T && out.size(1) == (long)a.H * a.dv && pos.numel() >= a.T && vdim >= 1 && vdim <= a.dv,
+             "hgrn2 shapes");
+  a.B = a.T;
+  a.vdim = vdim;
+  a.eps = eps;
+  a.len = len;
+  a.segments = 1;
+  if (q_lens) {
+    SHAI_CHECK(q_start.has_value(), "prefill: q_start");
+    check_i32(*q_lens, "q_lens");
+    check_i32(*q_start, "q_start");
+    a.B = q_lens->numel();
+    SHAI_CHECK(q_start->numel() == a.B, "one start per sequence");
+    a.q_lens = q_lens->data_ptr<int>();
+    a.q_start = q_start->data_ptr<int>();
+    if (!f32) a.segments = (max_q + len - 1) / len;
+  }
+  SHAI_CHECK(slots.numel() >= a.B && a.B <= 65535 && a.segments <= 65535, "one state slot per sequence");
+  SHAI_CHECK(a.segments == 1 || (ws.scalar_type() == at::kFloat && ws.is_contiguous() &&
+                                 ws.numel() >= (long)a.B * a.segments * a.H * a.dk * (a.dv + 1)), "hgrn2 workspace");
+  a.qv = qv.data_ptr();
+  a.z = z.data_ptr<float>();
+  a.bias = bias.data_ptr<float>();
+  a.lower = lower.data_ptr<float>();
+  a.gain = gain.data_ptr<float>();
+  a.state = state.data_ptr<float>();
+  a.out = out.data_ptr();
+  a.pos = pos.data_ptr<int>();
+  a.slots = slots.data_ptr<int>();
+  a.ws = a.segments > 1 ? ws.data_ptr<float>() : nullptr;
+  if (a.T == 0) return;
+  if (f32 || !a.q_lens) shai_lm::launch_hgrn2_rows(a, f32, stream());
+  else shai_lm::launch_hgrn2_chunks(a, stream());
+}
+
+const float* route_bias(const optional<Tensor>& bias, int E) {
+  if (!bias) return nullptr;
+  check(*bias, at::kFloat, "bias");
+  SHAI_CHECK(bias->numel() == E, "router bias must be [E]");
+  return bias->data_ptr<float>();
+}
+
+void moe_route(const Tensor& logits, int64_t groups, int64_t keep, const Tensor& ids, const Tensor& wts,
+               const optional<Tensor>& bias, bool renorm) {
   check(logits, at::kFloat, "logits");
   check_i32(ids, "ids");
   check(wts, at::kFloat, "wts");
@@ -627,6 +723,9 @@ void moe_route(const Tensor& logits, int64_t groups, int64_t keep, const Tensor&
   SHAI_CHECK(ids.size(0) == a.T && wts.sizes() == ids.sizes(), "route outputs must be [T, top]");
   SHAI_CHECK(a.E <= 1024 && groups >= 1 && a.E % groups == 0 && keep >= 1 && keep <= groups && a.top >= 1 &&
                  a.top <= keep * (a.E / groups), "route: up to 1024 experts in equal groups, top within the kept ones");
+  SHAI_CHECK(!renorm || a.top <= 64, "route: up to 64 renormalised picks");
+  a.bias = route_bias(bias, a.E);
+  a.renorm = renorm;
   a.logits = logits.data_ptr<float>();
   a.ids = ids.data_ptr<int>();
   a.wts = wts.data_ptr<float>();
@@ -635,7 +734,8 @@ void moe_route(const Tensor& logits, int64_t groups, int64_t keep, const Tensor&
 
 // logits -> picks -> slots for up to 16 tokens in one launch (moe_route + moe_plan with 16-row tiles)
 void moe_route_plan(const Tensor& logits, int64_t groups, int64_t keep, const Tensor& ids, const Tensor& wts,
-                    const Tensor& offsets, const Tensor& token_of, const Tensor& slot_of, const Tensor& tiles) {
+                    const Tensor& offsets, const Tensor& token_of, const Tensor& slot_of, const Tensor& tiles,
+                    const optional<Tensor>& bias, bool renorm) {
   check(logits, at::kFloat, "logits");
   check(wts, at::kFloat, "wts");
   for (auto* t : {&ids, &offsets, &token_of, &slot_of, &tiles}) check_i32(*t, "moe_route_plan tensor");
@@ -650,6 +750,9 @@ void moe_route_plan(const Tensor& logits, int64_t groups, int64_t keep, const Te
   SHAI_CHECK(reinterpret_cast<uintptr_t>(ids.data_ptr()) % 16 == 0, "moe_route_plan: ids must be 16-byte aligned");
   SHAI_CHECK(groups >= 1 && r.E % groups == 0 && keep >= 1 && keep <= groups && r.top >= 1 &&
                  r.top <= keep * (r.E / groups), "route: experts in equal groups, top within the kept ones");
+  SHAI_CHECK(!renorm || r.top <= 64, "route: up to 64 renormalised picks");
+  r.bias = route_bias(bias, r.E);
+  r.renorm = renorm;
   r.logits = logits.data_ptr<float>();
   r.ids = ids.data_ptr<int>();
   r.wts = wts.data_ptr<float>();
@@ -691,7 +794,9 @@ void moe_plan(const Tensor& ids, int64_t bm, const Tensor& offsets, const Tensor
   if (a.P > 0) shai_lm::launch_plan(a, stream());
 }
 
-shai_lm::AttnArgs attn_args(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor* o, int64_t heads) {
+// gate_w: gate logits per head (1 or dv).  own_kv false: rows are [q | gate], the cache holds another layer's keys and values
+shai_lm::AttnArgs attn_args(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor* o, int64_t heads,
+                            bool per_element = false, bool own_kv = true) {
   const auto dt = qkvg.scalar_type();
   is_f32(qkvg);
   check(qkvg, dt, "qkvg");
@@ -709,7 +814,10 @@ shai_lm::AttnArgs attn_args(const Tensor& qkvg, const Tensor& kc, const Tensor& 
   SHAI_CHECK(a.dk % 64 == 0 && a.dv % 64 == 0 && ((a.dk <= 128 && a.dv <= 128) || (a.dk == 256 && a.dv == 256)),
              "stored head sizes: 64 / 128 each, or 256 / 256");
   SHAI_CHECK(a.H >= 1 && a.G >= 1 && a.H % a.G == 0, "query heads must be a multiple of kv heads");
-  SHAI_CHECK(a.ld % 8 == 0 && a.ld >= (long)a.H * a.dk + (long)a.G * (a.dk + a.dv) + a.H, "qkvg row too short");
+  a.own_kv = own_kv;
+  a.gate_w = per_element ? a.dv : 1;
+  a.gate_off = a.H * a.dk + (own_kv ? a.G * (a.dk + a.dv) : 0);
+  SHAI_CHECK(a.ld % 8 == 0 && a.ld >= (long)a.gate_off + (long)a.H * a.gate_w, "qkvg row too short");
   a.qkvg = qkvg.data_ptr();
   a.kc = kc.data_ptr();
   a.vc = vc.data_ptr();
@@ -721,6 +829,29 @@ shai_lm::AttnArgs attn_args(const Tensor& qkvg, const Tensor& kc, const Tensor& 
   return a;
 }
 
+// rotation and norm of q and k: angles of every row, the head size before padding
+void set_turn(shai_lm::AttnArgs& a, const optional<Tensor>& rope, int64_t dim, double eps) {
+  if (!rope) return;
+  check(*rope, at::kFloat, "rope");
+  SHAI_CHECK(rope->dim() == 2 && rope->size(0) >= a.T && rope->size(1) % 2 == 0 && dim >= 1 && dim <= a.dk &&
+                 rope->size(1) <= dim, "rope must be [T, rotated dimensions of a head]");
+  a.rope = rope->data_ptr<float>();
+  a.rot = rope->size(1);
+  a.dim = dim;
+  a.eps = eps;
+}
+
+// q of the step in place and, with own keys, k and v into the cache
+void head_prep(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor& slots, int64_t heads, const Tensor& rope,
+               int64_t dim, double eps, bool own_kv) {
+  shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, nullptr, heads, false, own_kv);
+  set_turn(a, rope, dim, eps);
+  check_i32(slots, "slots");
+  SHAI_CHECK(slots.numel() >= a.T, "one slot per row");
+  a.slots = slots.data_ptr<int>();
+  if (a.T > 0) shai_lm::launch_head_prep(a, is_f32(qkvg), stream());
+}
+
 void kv_store(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor& slots, int64_t heads) {
   shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, nullptr, heads);
   check_i32(slots, "slots");
@@ -729,10 +860,11 @@ void kv_store(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tens
   if (a.T > 0) shai_lm::launch_kv_store(a, is_f32(qkvg), stream());
 }
 
-void chunk_attn_prefill(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor& o, const Tensor& bt,
+// `chunk`: the size of the chunks or, with `window`, of the sliding window
+void gated_attn_prefill(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor& o, const Tensor& bt,
                         const Tensor& ctx, const Tensor& q_lens, const Tensor& q_start, int64_t max_q, int64_t heads,
-                        int64_t chunk, double scale) {
-  shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, &o, heads);
+                        int64_t chunk, double scale, bool window, bool per_element, bool own_kv) {
+  shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, &o, heads, per_element, own_kv);
   for (auto* t : {&bt, &ctx, &q_lens, &q_start}) check_i32(*t, "batch tensor");
   a.B = bt.size(0);
   a.max_blocks = bt.size(1);
@@ -743,15 +875,18 @@ void chunk_attn_prefill(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, 
   a.q_lens = q_lens.data_ptr<int>();
   a.q_start = q_start.data_ptr<int>();
   a.max_q = max_q;
-  a.chunk = chunk;
+  a.chunk = std::min<int64_t>(chunk, 1 << 30);
+  a.window = window;
   a.scale = scale;
   shai_lm::launch_attn_prefill(a, is_f32(qkvg), stream());
 }
 
-void chunk_attn_decode(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor& o, const Tensor& bt,
+void gated_attn_decode(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor& o, const Tensor& bt,
                        const Tensor& ctx, const Tensor& slots, const Tensor& ws, int64_t heads, int64_t splits,
-                       int64_t chunk, double scale) {
-  shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, &o, heads);
+                       int64_t chunk, double scale, bool window, bool per_element, bool own_kv,
+                       const optional<Tensor>& rope, int64_t dim, double eps) {
+  shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, &o, heads, per_element, own_kv);
+  set_turn(a, rope, dim, eps);
   for (auto* t : {&bt, &ctx, &slots}) check_i32(*t, "batch tensor");
   a.B = bt.size(0);
   a.max_blocks = bt.size(1);
@@ -766,7 +901,8 @@ void chunk_attn_decode(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, c
   a.ws = splits > 1 ? ws.data_ptr<float>() : nullptr;
   a.splits = splits;
   a.max_q = 1;
-  a.chunk = chunk;
+  a.chunk = std::min<int64_t>(chunk, 1 << 30);
+  a.window = window;
   a.scale = scale;
   shai_lm::launch_attn_decode(a, is_f32(qkvg), stream());
 }
@@ -803,10 +939,10 @@ void token_feedback(const Tensor& ids, const Tensor& rowmap, const Tensor& prev)
 TORCH_LIBRARY_FRAGMENT(shai, m) {
   m.def("embed_norm(Tensor ids, Tensor? prev, Tensor table, Tensor? bigram, int mul_prev, int mul_cur, Tensor w, float eps, int width, Tensor(a!) x, Tensor(b!) h) -> ()");
   m.def("add_norm(Tensor(a!) x, Tensor? dense, Tensor? ye, Tensor? slot_of, Tensor? wts, Tensor? inject, Tensor? rows, Tensor? w, float eps, int width, Tensor(b!)? h) -> ()");
-  m.def("lm_gemm(Tensor a, Tensor w, Tensor(a!) c, Tensor? tiles, Tensor? offsets, Tensor? gather, int bm, int epi, float param, Tensor(b!)? side=None, Tensor? vec=None, Tensor? rope=None, int head=0, int rot0=0) -> ()");
+  m.def("lm_gemm(Tensor a, Tensor w, Tensor(a!) c, Tensor? tiles, Tensor? offsets, Tensor? gather, int bm, int epi, float param, Tensor(b!)? side=None, Tensor? vec=None, Tensor? rope=None, int head=0, int rot0=0, Tensor? ids=None, Tensor? table=None) -> ()");
   m.def("lm_gemm_heads(Tensor a, Tensor w, Tensor(a!) c) -> ()");
   m.def("lm_gemm_parts(Tensor a, Tensor w, Tensor(a!) c) -> ()");
-  m.def("residual_norm(Tensor? x, Tensor? ids, Tensor? table, float scale, Tensor? delta, Tensor? wb, float mult, Tensor? step, Tensor(a!)? x_out, Tensor? rows, Tensor? w, float eps, int width, Tensor(b!)? h, Tensor? cw=None, Tensor(c!)? state=None, Tensor(d!)? tail=None, Tensor? row_seq=None, Tensor? q_start=None, Tensor? q_lens=None, Tensor? pos=None, Tensor? slots=None) -> ()");
+  m.def("residual_norm(Tensor? x, Tensor? ids, Tensor? table, float scale, Tensor? delta, Tensor? wb, float mult, Tensor? step, Tensor(a!)? x_out, Tensor? rows, Tensor? w, float eps, int width, Tensor(b!)? h, Tensor? cw=None, Tensor(c!)? state=None, Tensor(d!)? tail=None, Tensor? row_seq=None, Tensor? q_start=None, Tensor? q_lens=None, Tensor? pos=None, Tensor? slots=None, Tensor? bb=None, Tensor? b=None, Tensor? ye=None, Tensor? slot_of=None, Tensor? wts=None) -> ()");
   m.def("conv_commit(Tensor(a!) state, Tensor tail, Tensor q_lens, Tensor slots) -> ()");
   m.def("rope_rows(Tensor pos, Tensor freq, Tensor(a!) out) -> ()");
   m.def("latent_prep(Tensor d, Tensor wq, Tensor wkv, Tensor rope, Tensor slots, Tensor(a!) cache, Tensor(b!) cq, float eps, int q_rank, int kv_rank) -> ()");
@@ -814,12 +950,14 @@ TORCH_LIBRARY_FRAGMENT(shai, m) {
   m.def("latent_attn_prefill(Tensor q, Tensor kv, Tensor lat, Tensor(a!) o, Tensor ctx, Tensor q_lens, Tensor q_start, Tensor kv_start, Tensor sink, int max_q, int heads, int np, int rot, int rank, float scale) -> ()");
   m.def("latent_attn_rows(Tensor ql, Tensor q, Tensor cache, Tensor(a!) o, Tensor block_table, Tensor? seqs, Tensor ctx, Tensor sink, Tensor(b!) ws, int splits, int np, int rot, float scale) -> ()");
   m.def("mingru_scan(Tensor zx, Tensor g, Tensor bias, Tensor(a!) state, Tensor(b!) out, Tensor pos, Tensor? q_start, Tensor? q_lens, Tensor slots, Tensor(c!) ws, int max_q, int len) -> ()");
-  m.def("moe_route(Tensor logits, int groups, int keep, Tensor(a!) ids, Tensor(b!) wts) -> ()");
-  m.def("moe_route_plan(Tensor logits, int groups, int keep, Tensor(a!) ids, Tensor(b!) wts, Tensor(c!) offsets, Tensor(d!) token_of, Tensor(e!) slot_of, Tensor(f!) tiles) -> ()");
+  m.def("moe_route(Tensor logits, int groups, int keep, Tensor(a!) ids, Tensor(b!) wts, Tensor? bias=None, bool renorm=False) -> ()");
+  m.def("moe_route_plan(Tensor logits, int groups, int keep, Tensor(a!) ids, Tensor(b!) wts, Tensor(c!) offsets, Tensor(d!) token_of, Tensor(e!) slot_of, Tensor(f!) tiles, Tensor? bias=None, bool renorm=False) -> ()");
   m.def("moe_plan(Tensor ids, int bm, Tensor(a!) offsets, Tensor(b!) token_of, Tensor(c!) slot_of, Tensor(d!) tiles) -> ()");
   m.def("kv_store(Tensor qkvg, Tensor(a!) k_cache, Tensor(b!) v_cache, Tensor slots, int heads) -> ()");
-  m.def("chunk_attn_prefill(Tensor qkvg, Tensor k_cache, Tensor v_cache, Tensor(a!) o, Tensor block_table, Tensor ctx_lens, Tensor q_lens, Tensor q_start, int max_q, int heads, int chunk, float scale) -> ()");
-  m.def("chunk_attn_decode(Tensor qkvg, Tensor(a!) k_cache, Tensor(b!) v_cache, Tensor(c!) o, Tensor block_table, Tensor ctx_lens, Tensor slots, Tensor(d!) ws, int heads, int splits, int chunk, float scale) -> ()");
+  m.def("head_prep(Tensor(a!) qkvg, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slots, int heads, Tensor rope, int dim, float eps, bool own_kv) -> ()");
+  m.def("hgrn2(Tensor qv, Tensor z, Tensor bias, Tensor lower, Tensor gain, Tensor(a!) state, Tensor(b!) out, Tensor pos, Tensor? q_start, Tensor? q_lens, Tensor slots, Tensor(c!) ws, int max_q, int len, int vdim, float eps) -> ()");
+  m.def("gated_attn_prefill(Tensor qkvg, Tensor k_cache, Tensor v_cache, Tensor(a!) o, Tensor block_table, Tensor ctx_lens, Tensor q_lens, Tensor q_start, int max_q, int heads, int chunk, float scale, bool window=False, bool per_element=False, bool own_kv=True) -> ()");
+  m.def("gated_attn_decode(Tensor qkvg, Tensor(a!) k_cache, Tensor(b!) v_cache, Tensor(c!) o, Tensor block_table, Tensor ctx_lens, Tensor slots, Tensor(d!) ws, int heads, int splits, int chunk, float scale, bool window=False, bool per_element=False, bool own_kv=True, Tensor? rope=None, int dim=0, float eps=0.) -> ()");
   m.def("sample(Tensor logits, Tensor temps, Tensor top_k, Tensor top_p, Tensor uniforms, Tensor(a!) out) -> ()");
   m.def("token_feedback(Tensor(a!) ids, Tensor rowmap, Tensor prev) -> ()");
 }
@@ -842,8 +980,10 @@ TORCH_LIBRARY_IMPL(shai, CUDA, m) {
   m.impl("moe_route_plan", &moe_route_plan);
   m.impl("moe_plan", &moe_plan);
   m.impl("kv_store", &kv_store);
-  m.impl("chunk_attn_prefill", &chunk_attn_prefill);
-  m.impl("chunk_attn_decode", &chunk_attn_decode);
+  m.impl("head_prep", &head_prep);
+  m.impl("hgrn2", &hgrn2);
+  m.impl("gated_attn_prefill", &gated_attn_prefill);
+  m.impl("gated_attn_decode", &gated_attn_decode);
   m.impl("sample", &sample);
   m.impl("token_feedback", &token_feedback);
 }

@@ -114,7 +114,7 @@ __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_
     __syncthreads();
   }
   // bf16 results go through LDS, so that rows are stored 16 bytes a lane, whole lines at a time
-  const bool glu = p.epi == EPI_CLAMP_GLU;
+  const bool glu = glu_epi(p.epi);
   if (sizeof(O) == 2 && p.ldc % 8 == 0 && (glu || p.N % 8 == 0) && (p.n_main == p.N || n0 + BN <= p.n_main)) {
     constexpr int LD = BN + 8;
     __syncthreads();

@@ -38,8 +38,9 @@ struct AddNormArgs {
 void launch_add_norm(const AddNormArgs& a, bool f32, hipStream_t s);
 
 // Residual add with a norm of its own, the next sublayer's norm, and its input convolution:
-//   x' = x + mult * RMSNorm(delta) wb (+ step),   h = RMSNorm(x') w,   h += causal convolution of h over time
-// Every part but the source of x may be absent.
+//   x' = x + mult * norm(delta) wb (+ bb) (+ step),   h = norm(x') w (+ b),   h += causal convolution of h over time
+// Every part but the source of x may be absent.  A norm with a bias is a layer norm (mean taken off), one without is an
+// RMS norm; h without w is x' itself.
 struct ResidualNormArgs {
   const float* x;          // [*, Dp], or null: x = table[ids] * scale
   const int* ids;
@@ -49,15 +50,21 @@ struct ResidualNormArgs {
   const void* delta;       // [*, Dp] sublayer output, or [parts, *, Dp] fp32 partial sums of it, or null
   int parts;               // 0: delta is of the type of h
   long part_stride;
+  const void* ye;          // [slots, Dp] expert outputs, their weighted sum added to delta, or null
+  const int* slot_of;      // [*, top]
+  const float* wts;        // [*, top]
+  int top;
   const float* wb;         // its norm's gain
+  const float* bb;         // its norm's bias, or null
   float mult;
   const float* step;       // [Dp] added to every row, or null
   float* x_out;            // [*, Dp], or null
   const int* rows;         // optional: only these rows (no convolution)
-  const float* w;          // gain, or null: no norm output
+  const float* w;          // gain, or null: no norm
+  const float* b;          // bias, or null
   float eps;
   int T, Dp, width;
-  void* h;                 // [T, Dp]
+  void* h;                 // [T, Dp], or null
   // convolution (cw null: none)
   const float* cw;         // [taps, Dp], oldest tap first
   int taps;
@@ -89,7 +96,9 @@ struct RopeRowsArgs {      // cos / sin of pos * freq, every row of a step
 };
 void launch_rope_rows(const RopeRowsArgs& a, hipStream_t s);
 
-enum Epi : int { EPI_NONE = 0, EPI_CLAMP_GLU = 1, EPI_SOFTCAP = 2, EPI_XIELU = 3, EPI_ROTARY = 4 };
+enum Epi : int { EPI_NONE = 0, EPI_CLAMP_GLU = 1, EPI_SOFTCAP = 2, EPI_XIELU = 3, EPI_ROTARY = 4, EPI_GELU_GLU = 5,
+                 EPI_RELU2 = 6, EPI_GELU_ROWS = 7 };
+constexpr __host__ __device__ bool glu_epi(int epi) { return epi == EPI_CLAMP_GLU || epi == EPI_GELU_GLU; }
 struct GemmArgs {
   const void* A;           // [rows, K]
   const void* W;           // [N, K] or [E, N, K]
@@ -113,6 +122,11 @@ struct GemmArgs {
   const float* vec;        // EPI_XIELU: (alpha_p, alpha_n)
   const float* rope;       // EPI_ROTARY: [M, rot] cos / sin pairs; columns rot0 .. rot0 + rot - 1 of every `head` columns
   int head, rot0, rot;
+  const int* ids;          // EPI_GELU_ROWS: [M] row of `table` (the type of A) that multiplies row m
+  const void* table;       // [table_rows, N] with rows table_ld apart
+  long table_ld;
+  int table_rows;
+  bool table_f32;
 };
 void launch_gemm(const GemmArgs& a, bool f32, hipStream_t s);          // streaming kernel, any M
 void launch_gemm_tile(const GemmArgs& a, hipStream_t s);               // LDS-tiled bf16 kernel (gemm_tile.hip)
@@ -122,6 +136,8 @@ struct RouteArgs {
   int T, E, top, groups, keep;
   int* ids;                // [T, top]
   float* wts;              // [T, top]
+  const float* bias;       // [E] added to the logits, or null
+  bool renorm;             // weights: softmax over the chosen logits only (else their share of all experts' softmax)
 };
 void launch_route(const RouteArgs& a, hipStream_t s);
 
@@ -137,8 +153,14 @@ void launch_plan(const PlanArgs& a, hipStream_t s);
 void launch_route_plan(const RouteArgs& r, const PlanArgs& a, hipStream_t s);   // T <= 16, E <= 256
 
 struct AttnArgs {
-  const void* qkvg;        // [T, ld]: q (H dk), k (G dk), v (G dv), gate logits (H)
+  const void* qkvg;        // [T, ld]: q (H dk), k (G dk), v (G dv), gate logits (H gate_w)
   long ld;
+  int gate_off, gate_w;    // column of the gate logits; 1 per head or dv of them
+  bool own_kv;             // rows hold k and v (else another layer's are in the cache, and the gate follows q)
+  bool window;             // a position sees itself and the chunk - 1 before it (else its own chunk)
+  const float* rope;       // [T, rot] cos / sin of every row, or null: q and k are used as they are.  Otherwise dimension
+  int rot, dim;            // i < rot / 2 of a head is turned with i + rot / 2, and the head divided by its rms over `dim`
+  float eps;
   void* kc;                // [blocks, G, 64, dk]
   void* vc;                // [blocks, G, 64, dv]
   void* o;                 // [T, H dv]
@@ -159,6 +181,7 @@ struct AttnArgs {
   int np, rank, lat_ld, lat_pad;   // lat_pad: the last column after `rank` from which 8 values may be read
 };
 void launch_kv_store(const AttnArgs& a, bool f32, hipStream_t s);
+void launch_head_prep(const AttnArgs& a, bool f32, hipStream_t s);     // q in place, k (turned, normed) and v to the cache
 void launch_attn_prefill(const AttnArgs& a, bool f32, hipStream_t s);
 void launch_attn_decode(const AttnArgs& a, bool f32, hipStream_t s);
 void launch_latent_prefill(const AttnArgs& a, hipStream_t s);          // bf16
@@ -219,5 +242,24 @@ struct ScanArgs {          // minGRU: S = (1 - z) S + z c, out = S silu(g)
   int T, B, W, max_q, len, chunks;
 };
 void launch_mingru_scan(const ScanArgs& a, bool f32, hipStream_t s);
+
+struct Hgrn2Args {         // S = diag(f) S + (1 - f) v^T, o = S^T silu(q), out = o / rms(o) gain, head by head
+  const void* qv;          // [T, H dk + H dv]
+  const float* z;          // [T, H dk] forget logits before their bias
+  const float* bias;       // [H dk]
+  const float* lower;      // [H dk] lower bound of f (1 in the pads)
+  const float* gain;       // [dv] (0 in the pads)
+  float* state;            // [slots, H, dk, dv]
+  void* out;               // [T, H dv]
+  const int* pos;          // [T]
+  const int* q_start;      // [B], null: one row per sequence (decode)
+  const int* q_lens;
+  const int* slots;        // [B], -1: none
+  float* ws;               // [B, segments, H, dk dv + dk] when a sequence has several segments
+  int T, B, H, dk, dv, vdim, len, segments;   // len: rows of a segment, a multiple of 32
+  float eps;
+};
+void launch_hgrn2_rows(const Hgrn2Args& a, bool f32, hipStream_t s);   // row by row
+void launch_hgrn2_chunks(const Hgrn2Args& a, hipStream_t s);           // bf16, 32 rows at a time
 
 }  // namespace shai_lm

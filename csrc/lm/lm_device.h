@@ -73,6 +73,12 @@ __device__ __forceinline__ float xielu(float z, float ap, float an, bool fast) {
   return (z > 0.f ? ap * z * z : an * e) + 0.5f * z;
 }
 
+// the tanh form of gelu: z / (1 + exp(-2 u)) = z (1 + tanh u) / 2
+__device__ __forceinline__ float gelu_tanh(float z) {
+  const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
+  return z / (1.f + expf(-2.f * u));
+}
+
 // Epilogue of 4 consecutive columns n .. n + 3 of row m, in place (a GLU's two results: c[0], c[1]).
 template <typename O>
 __device__ __forceinline__ void epilogue_cols(const GemmArgs& p, long m, int n, float4_& c) {
@@ -86,6 +92,20 @@ __device__ __forceinline__ void epilogue_cols(const GemmArgs& p, long m, int n, 
     const float ap = p.vec[0], an = p.vec[1];
 #pragma unroll
     for (int i = 0; i < 4; ++i) c[i] = xielu(c[i], ap, an, sizeof(O) == 2);
+  } else if (p.epi == EPI_GELU_GLU) {
+    c[0] = gelu_tanh(c[0]) * c[1];
+    c[1] = gelu_tanh(c[2]) * c[3];
+  } else if (p.epi == EPI_RELU2) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) c[i] = c[i] > 0.f ? c[i] * c[i] : 0.f;
+  } else if (p.epi == EPI_GELU_ROWS) {
+    if (n < p.N) {
+      const long at = (long)min(max(p.ids[m], 0), p.table_rows - 1) * p.table_ld + n;
+      const float4_ e = p.table_f32 ? load4(static_cast<const float*>(p.table) + at)
+                                    : load4(static_cast<const bf16_t*>(p.table) + at);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) c[i] = gelu_tanh(c[i]) * e[i];
+    }
   } else if (p.epi == EPI_ROTARY) {
     const int d = n % p.head - p.rot0;
     if (d >= 0 && d < p.rot && n < p.N) {
@@ -118,7 +138,7 @@ __device__ __forceinline__ void store_cols(const GemmArgs& p, O* out, long m, in
     return;
   }
   epilogue_cols<O>(p, m, n, c);
-  if (p.epi == EPI_CLAMP_GLU) {
+  if (glu_epi(p.epi)) {
     const int j = n >> 1;
     if (n < p.N) store1(out + m * p.ldc + j, c[0]);
     if (n + 2 < p.N) store1(out + m * p.ldc + j + 1, c[1]);

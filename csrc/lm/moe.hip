@@ -1,4 +1,5 @@
-// Mixture-of-experts routing: group-limited top-k of softmax scores, and the sort of (token, k) pairs by expert.
+// Mixture-of-experts routing: group-limited top-k of softmax scores (weights: those scores, or a softmax over the chosen
+// logits only), and the sort of (token, k) pairs by expert.
 #include "lm_device.h"
 #include "lm.h"
 
@@ -34,30 +35,32 @@ __device__ __forceinline__ void route_token(const RouteArgs& p, int t, float* sc
 #pragma unroll
   for (int i = 0; i < NE; ++i) {
     const int e = lane + 64 * i;
-    z[i] = live && e < p.E ? p.logits[(long)t * p.E + e] : -INFINITY;
+    z[i] = live && e < p.E ? p.logits[(long)t * p.E + e] + (p.bias ? p.bias[e] : 0.f) : -INFINITY;
     if (!(z[i] == z[i])) z[i] = -INFINITY;      // a padding row may carry NaN: it still needs valid picks
+    if (p.renorm && e < p.E) z[i] = fmaxf(z[i], -3e38f);
     m = fmaxf(m, z[i]);
   }
   m = wave_max_dpp(m);
   if (m == -INFINITY) m = 0.f;
-  float sum = 0.f;
+  if (!p.renorm) {                               // scores: softmax over all experts (else the logits themselves)
+    float sum = 0.f;
 #pragma unroll
-  for (int i = 0; i < NE; ++i) {
-    z[i] = expf(z[i] - m);
-    sum += lane + 64 * i < p.E ? z[i] : 0.f;
-  }
-  sum = wave_sum(sum);
-  const float inv = sum > 0.f ? 1.f / sum : 0.f;
+    for (int i = 0; i < NE; ++i) {
+      z[i] = expf(z[i] - m);
+      sum += lane + 64 * i < p.E ? z[i] : 0.f;
+    }
+    sum = wave_sum(sum);
+    const float inv = sum > 0.f ? 1.f / sum : 0.f;
 #pragma unroll
-  for (int i = 0; i < NE; ++i) {
-    const int e = lane + 64 * i;
-    z[i] *= inv;
-    if (e < p.E) sc[e] = z[i];
+    for (int i = 0; i < NE; ++i) z[i] *= inv;
   }
+#pragma unroll
+  for (int i = 0; i < NE; ++i)
+    if (lane + 64 * i < p.E) sc[lane + 64 * i] = z[i];
   __syncthreads();
   const int per = p.E / p.groups;
   for (int g = lane; g < p.groups; g += 64) {
-    float b = -1.f;
+    float b = -INFINITY;
     for (int j = 0; j < per; ++j) b = fmaxf(b, sc[g * per + j]);
     gs[g] = b;
   }
@@ -71,12 +74,13 @@ __device__ __forceinline__ void route_token(const RouteArgs& p, int t, float* sc
       const float mine = gs[g];
       int better = 0;
       for (int j = 0; j < p.groups; ++j) better += gs[j] > mine || (gs[j] == mine && j < g);
-      if (better >= p.keep) z[i] = -1.f;
+      if (better >= p.keep) z[i] = -INFINITY;
     }
-    if (e >= p.E) z[i] = -2.f;
+    if (e >= p.E) z[i] = -INFINITY;
   }
+  float mine = -INFINITY;                        // renorm: lane k's pick
   for (int k = 0; k < p.top; ++k) {
-    float best = -3.f;
+    float best = -INFINITY;
     int bi = 0x7fffffff;
 #pragma unroll
     for (int i = 0; i < NE; ++i) {
@@ -94,11 +98,16 @@ __device__ __forceinline__ void route_token(const RouteArgs& p, int t, float* sc
     }
 #pragma unroll
     for (int i = 0; i < NE; ++i)
-      if (lane + 64 * i == bi) z[i] = -4.f;
+      if (lane + 64 * i == bi) z[i] = -INFINITY;
+    if (lane == k) mine = bv;
     if (live && lane == 0) {
       p.ids[(long)t * p.top + k] = bi;
-      p.wts[(long)t * p.top + k] = bv;
+      if (!p.renorm) p.wts[(long)t * p.top + k] = bv;
     }
+  }
+  if (p.renorm) {
+    const float e = lane < p.top ? expf(mine - m) : 0.f, sum = wave_sum(e);
+    if (live && lane < p.top) p.wts[(long)t * p.top + lane] = e / sum;
   }
 }
 

@@ -110,23 +110,24 @@ __device__ __forceinline__ float4_ wide4(uint2_ v) {
                  __uint_as_float(v[1] & 0xffff0000u)};
 }
 
-// The row stays in registers through both norms.  With a convolution a workgroup walks `run` consecutive rows, two of them
+// The row stays in registers through both norms (RMS norms, or layer norms where there is a bias).  With a convolution a workgroup walks `run` consecutive rows, two of them
 // loaded ahead, and keeps the last taps - 1 inputs in registers; the ones before its first row are recomputed from their
 // residual rows (which is why x_out is not x then) or, before the step's first row of a sequence, come from the sequence's
 // state.  Whatever the rows share (gains, taps, the rows' places) is read before the first row: a load inside the loop
 // would wait for the rows ahead of it.  TD: the type of delta.
-constexpr int conv_waves(int taps, int nt, int nv) { return taps == 4 && nt <= 512 && nv <= 2 ? 4 : 1; }   // per SIMD
+constexpr int conv_waves(int taps, int nt, int nv) { return taps > 0 && taps <= 4 && nt <= 512 && nv <= 2 ? 4 : 1; }   // per SIMD
 template <typename T, typename TD, int NT, int NV, int TAPS>
 __global__ void __launch_bounds__(NT, conv_waves(TAPS, NT, NV)) residual_norm_kernel(const ResidualNormArgs p) {
   constexpr bool CONV = TAPS > 0, KEEP = CONV && TAPS <= 4 && NV <= 2;   // KEEP: taps in registers
   constexpr int KN = KEEP ? NV : 1, KT = KEEP ? TAPS : 1;
   using Raw = decltype(raw4(static_cast<const TD*>(nullptr)));
   __shared__ float red[2][NT / 64];
-  __shared__ __attribute__((aligned(16))) float sw[CONV ? 2 : 1][CONV ? NT * NV * 4 : 4];   // w, wb
+  __shared__ __attribute__((aligned(16))) float sw[CONV ? 2 : 1][CONV ? NT * NV * 4 : 4];   // w (without it: bb), wb
   int turn = 0;
   const int c0 = threadIdx.x * 4;
   const float inv_w = 1.f / (float)p.width;
   const float4_ zero = float4_{0.f, 0.f, 0.f, 0.f};
+  const bool has_delta = p.delta || p.ye;
   struct Row {
     float4_ x[NV];
     Raw d[NV];
@@ -143,13 +144,21 @@ __global__ void __launch_bounds__(NT, conv_waves(TAPS, NT, NV)) residual_norm_ke
       if (c < p.Dp) {
         q.x[i] = x ? load4(x + c) : load4(e + c) * p.scale;
         if (p.delta) q.d[i] = raw4(d + c);
-        if constexpr (sizeof(TD) == 4)
+        if constexpr (sizeof(TD) == 4) {
+          if (p.ye) {                                      // (the only part then: no other delta)
+            float4_ s = zero;
+#pragma unroll 4
+            for (int k = 0; k < p.top; ++k)
+              s += p.wts[row * p.top + k] * load4(static_cast<const T*>(p.ye) + (long)p.slot_of[row * p.top + k] * p.Dp + c);
+            q.d[i] = s;
+          }
           for (int k = 1; k < p.parts; k += 3) {           // three loads at a time, none of them waited for alone
             float4_ e[3];
 #pragma unroll
             for (int j = 0; j < 3; ++j) e[j] = raw4(d + min(k + j, p.parts - 1) * p.part_stride + c);
             q.d[i] += e[0] + (k + 1 < p.parts ? e[1] : zero) + (k + 2 < p.parts ? e[2] : zero);
           }
+        }
       }
     }
   };
@@ -158,35 +167,53 @@ __global__ void __launch_bounds__(NT, conv_waves(TAPS, NT, NV)) residual_norm_ke
     if constexpr (CONV) return *reinterpret_cast<const float4_*>(&sw[which][c]);
     else return load4(g + c);
   };
+  // 1 / root of the mean square of d; with `centre` its mean is taken off first (pad columns stay out of both)
+  auto scale_of = [&](float4_(&d)[NV], bool centre) {
+    float ss = 0.f;
+    if (centre) {
+      float s = 0.f;
+#pragma unroll
+      for (int i = 0; i < NV; ++i) s += (d[i][0] + d[i][1]) + (d[i][2] + d[i][3]);
+      const float mean = block_sum<NT>(s, red, turn) * inv_w;
+#pragma unroll
+      for (int i = 0; i < NV; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) d[i][j] = i * NT * 4 + c0 + j < p.width ? d[i][j] - mean : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i) ss += d[i][0] * d[i][0] + d[i][1] * d[i][1] + d[i][2] * d[i][2] + d[i][3] * d[i][3];
+    return 1.f / sqrtf(block_sum<NT>(ss, red, turn) * inv_w + p.eps);
+  };
   auto add = [&](const Row& q, float4_(&v)[NV]) {
     float r = 0.f;
-    if (p.delta) {
-      float ss = 0.f;
+    float4_ d[NV];
+    if (has_delta) {
 #pragma unroll
-      for (int i = 0; i < NV; ++i) {
-        const float4_ d = wide4(q.d[i]);
-        ss += d[0] * d[0] + d[1] * d[1] + d[2] * d[2] + d[3] * d[3];
-      }
-      r = p.mult / sqrtf(block_sum<NT>(ss, red, turn) * inv_w + p.eps);
+      for (int i = 0; i < NV; ++i) d[i] = wide4(q.d[i]);
+      r = p.mult * scale_of(d, p.bb != nullptr);
     }
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int c = i * NT * 4 + c0;
       v[i] = q.x[i];
       if (c < p.Dp) {
-        if (p.delta) v[i] += wide4(q.d[i]) * r * gain(p.wb, 1, i);
+        if (has_delta) {
+          v[i] += d[i] * r * gain(p.wb, 1, i);
+          if (p.bb) v[i] += p.mult * (CONV && !p.w ? gain(p.bb, 0, i) : load4(p.bb + c));
+        }
         if (p.step) v[i] += load4(p.step + c);
       }
     }
   };
   auto norm = [&](float4_(&v)[NV]) {
-    float ss = 0.f;
-#pragma unroll
-    for (int i = 0; i < NV; ++i) ss += v[i][0] * v[i][0] + v[i][1] * v[i][1] + v[i][2] * v[i][2] + v[i][3] * v[i][3];
-    const float r = 1.f / sqrtf(block_sum<NT>(ss, red, turn) * inv_w + p.eps);
+    if (!p.w) return;
+    const float r = scale_of(v, p.b != nullptr);
 #pragma unroll
     for (int i = 0; i < NV; ++i)
-      if (i * NT * 4 + c0 < p.Dp) v[i] = v[i] * r * gain(p.w, 0, i);
+      if (i * NT * 4 + c0 < p.Dp) {
+        v[i] = v[i] * r * gain(p.w, 0, i);
+        if (p.b) v[i] += load4(p.b + i * NT * 4 + c0);
+      }
   };
   auto put = [&](auto* dst, const float4_(&v)[NV]) {
 #pragma unroll
@@ -201,7 +228,7 @@ __global__ void __launch_bounds__(NT, conv_waves(TAPS, NT, NV)) residual_norm_ke
     fetch(row, q);
     add(q, v);
     if (p.x_out) put(p.x_out + row * p.Dp, v);
-    if (!p.w) return;
+    if (!p.h) return;
     norm(v);
     put(static_cast<T*>(p.h) + (long)blockIdx.x * p.Dp, v);
   } else {
@@ -237,8 +264,9 @@ __global__ void __launch_bounds__(NT, conv_waves(TAPS, NT, NV)) residual_norm_ke
     for (int i = 0; i < NV; ++i) {
       const int c = i * NT * 4 + c0;
       const bool in = c < p.Dp;
-      store4(&sw[0][c], in ? load4(p.w + c) : zero);     // read back by this thread only
-      store4(&sw[1][c], in && p.delta ? load4(p.wb + c) : zero);
+      const float* first = p.w ? p.w : p.bb;
+      store4(&sw[0][c], in && first ? load4(first + c) : zero);     // read back by this thread only
+      store4(&sw[1][c], in && has_delta ? load4(p.wb + c) : zero);
       if constexpr (KEEP) {
 #pragma unroll
         for (int j = 0; j < TAPS; ++j)
@@ -360,6 +388,7 @@ template <typename T, typename TD, int NT, int NV>
 static void residual_norm(const ResidualNormArgs& a, hipStream_t s) {
   const int grid = a.cw ? (a.T + a.run - 1) / a.run : a.T;
   if (!a.cw) residual_norm_kernel<T, TD, NT, NV, 0><<<grid, NT, 0, s>>>(a);
+  else if (a.taps <= 2) residual_norm_kernel<T, TD, NT, NV, 2><<<grid, NT, 0, s>>>(a);
   else if (a.taps <= 4) residual_norm_kernel<T, TD, NT, NV, 4><<<grid, NT, 0, s>>>(a);
   else residual_norm_kernel<T, TD, NT, NV, 16><<<grid, NT, 0, s>>>(a);
 }
@@ -375,7 +404,7 @@ static void residual_norm(const ResidualNormArgs& a, hipStream_t s) {
 
 void launch_residual_norm(const ResidualNormArgs& a, bool f32, hipStream_t s) {
   if (f32) residual_norm<float, float>(a, s);
-  else if (a.parts) residual_norm<bf16_t, float>(a, s);
+  else if (a.parts || a.ye) residual_norm<bf16_t, float>(a, s);
   else residual_norm<bf16_t, bf16_t>(a, s);
   SHAI_CHECK_LAUNCH();
 }

@@ -8,7 +8,7 @@ from __future__ import annotations
 
 import math
 from dataclasses import dataclass
-from typing import Callable, Dict, Optional
+from typing import Callable, Dict, Optional, Union
 
 import torch
 import torch.nn as nn
@@ -32,6 +32,11 @@ def _padded(t: torch.Tensor, *shape) -> torch.Tensor:
 def _head_rows(t: torch.Tensor, heads: int, dim: int, pad: int, width: int) -> torch.Tensor:
     """[heads * dim, D] -> [heads * pad, width], every head's rows padded by zero rows."""
     return _padded(t.reshape(heads, dim, t.shape[1]), heads, pad, width).reshape(heads * pad, width)
+
+
+def _head_columns(t: torch.Tensor, heads: int, dim: int, pad: int, width: int) -> torch.Tensor:
+    """[D, heads * dim] -> [width, heads * pad], every head's columns padded by zero columns."""
+    return _padded(t.reshape(t.shape[0], heads, dim), width, heads, pad).reshape(width, heads * pad)
 
 
 def check_checkpoint(sd: Dict[str, torch.Tensor], want: Dict[str, tuple]) -> None:
@@ -138,13 +143,21 @@ class ClampedGLUConfig:
 
 
 @dataclass
+class ReLU2Config:
+    """Feed-forward without a gate: down max(up h, 0)^2."""
+    ff: int
+
+
+@dataclass
 class MoEConfig:
     experts: int
     top: int
-    expert: ClampedGLUConfig
+    expert: Union[ClampedGLUConfig, ReLU2Config]
     groups: int = 1
     keep: int = 1
     shared: Optional[ClampedGLUConfig] = None
+    bias: bool = False       # the router's logits have one
+    renorm: bool = False     # weights are a softmax over the chosen logits only
 
     def __post_init__(self):
         if (self.experts % self.groups or not 1 <= self.keep <= self.groups
@@ -159,8 +172,8 @@ def _interleave(gate: torch.Tensor, up: torch.Tensor, ff: int, width: int) -> to
 
 
 class MoE(nn.Module):
-    """Softmax-scored experts chosen inside the best expert groups (scores not renormalised), clamped-GLU experts, and
-    an optional shared expert.  Returns :class:`ops.lm.Experts` for the next residual add to combine."""
+    """Softmax-scored experts chosen inside the best expert groups, clamped-GLU or squared-ReLU experts, and an optional
+    shared expert.  Returns :class:`ops.lm.Experts` for the next residual add to combine."""
 
     def __init__(self, width: int, c: MoEConfig, dtype=torch.bfloat16):
         super().__init__()
@@ -169,25 +182,37 @@ class MoE(nn.Module):
         # the shared expert's gate / up rows and the router's rows: one product
         S = lm.pad64(c.shared.ff) if c.shared is not None else 0
         self.front = _param(2 * S + c.experts, W, dtype=dtype)
-        self.gate_up = _param(c.experts, 2 * F, W, dtype=dtype)
+        self.gated = isinstance(c.expert, ClampedGLUConfig)
+        if self.gated:
+            self.gate_up = _param(c.experts, 2 * F, W, dtype=dtype)
+        else:
+            self.up = _param(c.experts, F, W, dtype=dtype)
         self.down = _param(c.experts, W, F, dtype=dtype)
+        self.bias = _param(c.experts, dtype=torch.float32) if c.bias else None
         if c.shared is not None:
             self.shared_down = _param(W, S, dtype=dtype)
 
     def shapes(self) -> Dict[str, tuple]:
         c, D = self.c, self.width
         s = {"router": (c.experts, D)}
+        if c.bias:
+            s["router.b"] = (c.experts,)
         named = [(f"e{i}", c.expert) for i in range(c.experts)] + ([("shared", c.shared)] if c.shared else [])
         for name, e in named:
-            s.update({f"{name}.gate": (e.ff, D), f"{name}.up": (e.ff, D), f"{name}.down": (D, e.ff)})
+            s.update({f"{name}.up": (e.ff, D), f"{name}.down": (D, e.ff)})
+            if isinstance(e, ClampedGLUConfig):
+                s[f"{name}.gate"] = (e.ff, D)
         return s
 
     def pack(self, get: Callable[[str], torch.Tensor]) -> Dict[str, torch.Tensor]:
         c, W, F = self.c, self.front.shape[1], self.down.shape[2]
+        each = lambda fn: torch.stack([fn(f"e{i}.") for i in range(c.experts)])
         out = {"front": _padded(get("router"), c.experts, W),
-               "gate_up": torch.stack([_interleave(get(f"e{i}.gate"), get(f"e{i}.up"), F, W)
-                                       for i in range(c.experts)]),
+               **({"gate_up": each(lambda e: _interleave(get(e + "gate"), get(e + "up"), F, W))} if self.gated
+                  else {"up": each(lambda e: _padded(get(e + "up"), F, W))}),
                "down": torch.stack([_padded(get(f"e{i}.down"), W, F) for i in range(c.experts)])}
+        if c.bias:
+            out["bias"] = get("router.b")
         if c.shared is not None:
             S = self.shared_down.shape[1]
             out["front"] = torch.cat([_interleave(get("shared.gate"), get("shared.up"), S, W), out["front"]])
@@ -200,8 +225,11 @@ class MoE(nn.Module):
             s, z = lm.glu_with_side(h, self.front, c.experts, c.shared.limit)
         else:
             z = lm.matmul(h, self.front, torch.float32)
-        wts, plan = lm.route_experts(z, c.top, c.groups, c.keep)
-        a = lm.matmul(h, self.gate_up, epi=lm.EPI_CLAMP_GLU, param=c.expert.limit, plan=plan, gather=True)
+        wts, plan = lm.route_experts(z, c.top, c.groups, c.keep, self.bias, c.renorm)
+        if self.gated:
+            a = lm.matmul(h, self.gate_up, epi=lm.EPI_CLAMP_GLU, param=c.expert.limit, plan=plan, gather=True)
+        else:
+            a = lm.matmul(h, self.up, epi=lm.EPI_RELU2, plan=plan, gather=True)
         y = lm.matmul(a, self.down, plan=plan)
         dense = lm.matmul(s, self.shared_down) if c.shared is not None else None
         return lm.Experts(y, plan.slot_of, wts, dense)
@@ -358,6 +386,10 @@ class LatentAttention(nn.Module):
     def cache_shape(self, blocks: int, block: int):
         return blocks, block, self.rp + self.op
 
+    @property
+    def rope_key(self):
+        return self.c.rot_base, self.c.rot_dim, None
+
     state_width = None
 
     def init_random_(self, gen):
@@ -370,8 +402,9 @@ class StepShared:
     def __init__(self, batch):
         self.batch, self._ropes, self._plans = batch, {}, {}
 
-    def rope(self, mix: LatentAttention):
-        key = (mix.c.rot_base, mix.c.rot_dim)
+    def rope(self, mix):
+        """Angles for a mixer with ``rope_key`` (what its frequencies follow from) and ``freq``."""
+        key = mix.rope_key
         if key not in self._ropes:
             self._ropes[key] = lm.rope_rows(self.batch.positions, mix.freq)
         return self._ropes[key]
@@ -441,6 +474,222 @@ class XieluMLP(nn.Module):
 
     def forward(self, h):
         return lm.matmul_parts(lm.matmul(h, self.up, epi=lm.EPI_XIELU, vec=self.act), self.down)
+
+    def init_random_(self, gen):
+        _init_packed(self, self.pack, self.shapes(), gen)
+
+
+class AffineNorm(nn.Module):
+    """Layer norm with gain and bias (applied by ``ops.lm.residual_norm``)."""
+
+    def __init__(self, width: int):
+        super().__init__()
+        self.width = width
+        self.weight = _param(lm.pad64(width), dtype=torch.float32)
+        self.bias = _param(lm.pad64(width), dtype=torch.float32)
+
+    @property
+    def affine(self) -> lm.Affine:
+        return lm.Affine(self.weight, self.bias)
+
+    def shapes(self) -> Dict[str, tuple]:
+        return {"": (self.width,), ".b": (self.width,)}
+
+    def pack(self, get: Callable[[str], torch.Tensor]) -> Dict[str, torch.Tensor]:
+        return {"weight": _padded(get(""), lm.pad64(self.width)), "bias": _padded(get(".b"), lm.pad64(self.width))}
+
+    def init_random_(self, gen):
+        self.weight[:self.width] = 1.0
+
+
+class TokenShift(InputConv):
+    """A mixer's input moved towards the previous token's, channel by channel: h + (h' - h) s, i.e. a convolution of two
+    taps (s, -s) added to h."""
+
+    def __init__(self, width: int):
+        super().__init__(width, 2)
+
+    def pack(self, t: torch.Tensor) -> torch.Tensor:
+        return super().pack(torch.stack([t.float(), -t.float()], 1))
+
+    def init_random_(self, gen):
+        s = torch.rand(self.width, generator=gen, device=gen.device)
+        self.weight[0, :self.width], self.weight[1, :self.width] = s, -s
+
+
+@dataclass
+class WindowAttentionConfig:
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: int                                  # a position sees itself and the window - 1 before it
+    rot_dims: int                                # rotated dimensions of a head
+    rot_base: float = 10000.0
+    rot_scaling: Optional[lm.RopeScaling] = None
+    kv_from: Optional[int] = None                # layer whose keys and values are used
+
+    def __post_init__(self):
+        if (self.heads % self.kv_heads or self.window < 1 or self.rot_dims % 2 or not 0 < self.rot_dims <= self.dim
+                or min(self.dim, self.vdim) < 1):
+            raise ValueError(f"bad attention sizes: {self}")
+
+
+class WindowAttention(nn.Module):
+    """Sliding-window attention with rotated (half against half) and rms-normed queries and keys and a sigmoid gate per
+    output element.  q, k, v and the gate logits come from one GEMM; with ``kv_from`` only q and the gate, and the keys and
+    values are those in another layer's cache."""
+
+    state_shape = None
+
+    def __init__(self, width: int, c: WindowAttentionConfig, eps: float, dtype=torch.bfloat16):
+        super().__init__()
+        self.c, self.width, self.eps = c, width, eps
+        self.dk, self.dv = lm.head_pad(c.dim, c.vdim)
+        kv = c.kv_heads * (self.dk + self.dv) if c.kv_from is None else 0
+        self.qkvg = _param(c.heads * (self.dk + self.dv) + kv, lm.pad64(width), dtype=dtype)
+        self.o = _param(lm.pad64(width), c.heads * self.dv, dtype=dtype)
+        self.register_buffer("freq", lm.rope_freq(c.rot_base, c.rot_dims, c.rot_scaling).to(self.o.device),
+                             persistent=False)
+
+    @property
+    def rope_key(self):
+        return self.c.rot_base, self.c.rot_dims, self.c.rot_scaling
+
+    def shapes(self) -> Dict[str, tuple]:
+        c, D = self.c, self.width
+        s = {"q": (c.heads * c.dim, D), "g": (c.heads * c.vdim, D), "o": (D, c.heads * c.vdim)}
+        if c.kv_from is None:
+            s.update({"k": (c.kv_heads * c.dim, D), "v": (c.kv_heads * c.vdim, D)})
+        return s
+
+    def pack(self, get: Callable[[str], torch.Tensor]) -> Dict[str, torch.Tensor]:
+        c, W = self.c, self.qkvg.shape[1]
+        rows = [_head_rows(get("q"), c.heads, c.dim, self.dk, W)]
+        if c.kv_from is None:
+            rows += [_head_rows(get("k"), c.kv_heads, c.dim, self.dk, W),
+                     _head_rows(get("v"), c.kv_heads, c.vdim, self.dv, W)]
+        rows.append(_head_rows(get("g"), c.heads, c.vdim, self.dv, W))
+        return {"qkvg": torch.cat(rows), "o": _head_columns(get("o"), c.heads, c.vdim, self.dv, W)}
+
+    def forward(self, h, batch, cache, step):
+        c = self.c
+        o = lm.gated_attention(lm.matmul(h, self.qkvg), *cache, batch, c.heads, c.window, c.scale, window=True,
+                               per_element=True, own_kv=c.kv_from is None,
+                               turn=lm.HeadTurn(step.rope(self), c.dim, self.eps))
+        return lm.matmul_parts(o, self.o)
+
+    def cache_shapes(self, blocks: int, block: int):
+        if self.c.kv_from is not None:
+            return None
+        g = self.c.kv_heads
+        return (blocks, g, block, self.dk), (blocks, g, block, self.dv)
+
+    def init_random_(self, gen):
+        _init_packed(self, self.pack, self.shapes(), gen)
+
+
+@dataclass
+class Hgrn2Config:
+    heads: int
+    dim: int
+    vdim: int
+
+    def __post_init__(self):
+        if min(self.heads, self.dim, self.vdim) < 1:
+            raise ValueError(f"bad recurrence sizes: {self}")
+
+
+class Hgrn2(nn.Module):
+    """Linear attention with a matrix state per head whose forget gate (bounded below) also decides what is written; every
+    head's output is rms-normed.  One product gives queries and values (weights' dtype) and forget logits (fp32)."""
+
+    def __init__(self, width: int, c: Hgrn2Config, eps: float, dtype=torch.bfloat16):
+        super().__init__()
+        self.c, self.width, self.eps = c, width, eps
+        self.dk, self.dv = lm.head_pad(c.dim, c.vdim)
+        H, W = c.heads, lm.pad64(width)
+        self.qvf = _param(H * (2 * self.dk + self.dv), W, dtype=dtype)
+        self.bias = _param(H * self.dk, dtype=torch.float32)
+        self.lower = _param(H * self.dk, dtype=torch.float32)
+        self.gain = _param(self.dv, dtype=torch.float32)
+        self.o = _param(W, H * self.dv, dtype=dtype)
+
+    @property
+    def state_shape(self) -> tuple:
+        return self.c.heads, self.dk, self.dv
+
+    def shapes(self) -> Dict[str, tuple]:
+        c, D = self.c, self.width
+        n, m = c.heads * c.dim, c.heads * c.vdim
+        return {"q": (n, D), "f": (n, D), "f.b": (n,), "lower": (n,), "v": (m, D), "norm": (c.vdim,), "o": (D, m)}
+
+    def pack(self, get: Callable[[str], torch.Tensor]) -> Dict[str, torch.Tensor]:
+        c, H, W = self.c, self.c.heads, self.qvf.shape[1]
+        rows = lambda name, dim, pad: _head_rows(get(name), H, dim, pad, W)
+        lower = get("lower").reshape(H, c.dim)
+        pads = torch.cat([lower, lower.new_ones(H, self.dk - c.dim)], 1)      # a pad channel keeps its (zero) state
+        return {"qvf": torch.cat([rows("q", c.dim, self.dk), rows("v", c.vdim, self.dv), rows("f", c.dim, self.dk)]),
+                "bias": _padded(get("f.b").reshape(H, c.dim), H, self.dk).reshape(-1), "lower": pads.reshape(-1),
+                "gain": _padded(get("norm"), self.dv), "o": _head_columns(get("o"), H, c.vdim, self.dv, W)}
+
+    def forward(self, h, batch, state, step=None):
+        qv, z = lm.matmul_with_side(h, self.qvf, self.c.heads * self.dk)
+        o = lm.hgrn2(qv, z, self.bias, self.lower, self.gain, state, batch, self.c.vdim, self.eps)
+        return lm.matmul_parts(o, self.o)
+
+    def cache_shapes(self, blocks: int, block: int):
+        return None
+
+    def init_random_(self, gen):
+        _init_packed(self, self.pack, self.shapes(), gen)
+
+
+class GeluGLU(nn.Module):
+    """Dense feed-forward down (gelu_tanh(gate h) up h)."""
+
+    def __init__(self, width: int, ff: int, dtype=torch.bfloat16):
+        super().__init__()
+        self.width, self.ff = width, ff
+        self.gate_up = _param(2 * lm.pad64(ff), lm.pad64(width), dtype=dtype)
+        self.down = _param(lm.pad64(width), lm.pad64(ff), dtype=dtype)
+
+    def shapes(self) -> Dict[str, tuple]:
+        return {"gate": (self.ff, self.width), "up": (self.ff, self.width), "down": (self.width, self.ff)}
+
+    def pack(self, get: Callable[[str], torch.Tensor]) -> Dict[str, torch.Tensor]:
+        W, F = self.down.shape
+        return {"gate_up": _interleave(get("gate"), get("up"), F, W), "down": _padded(get("down"), W, F)}
+
+    def forward(self, h):
+        return lm.matmul_parts(lm.matmul(h, self.gate_up, epi=lm.EPI_GELU_GLU), self.down)
+
+    def init_random_(self, gen):
+        _init_packed(self, self.pack, self.shapes(), gen)
+
+
+class TokenSide(nn.Module):
+    """Per-layer token input: proj (gelu_tanh(gate x) * the token's row of a table), rms-normed by the residual add."""
+
+    def __init__(self, width: int, dim: int, dtype=torch.bfloat16):
+        super().__init__()
+        self.width, self.dim = width, dim
+        n, W = lm.pad64(dim), lm.pad64(width)
+        self.gate = _param(n, W, dtype=dtype)
+        self.proj = _param(W, n, dtype=dtype)
+        self.norm = _param(W, dtype=torch.float32)
+
+    def shapes(self) -> Dict[str, tuple]:
+        return {"gate": (self.dim, self.width), "proj": (self.width, self.dim), "norm": (self.width,)}
+
+    def pack(self, get: Callable[[str], torch.Tensor]) -> Dict[str, torch.Tensor]:
+        return {"gate": _padded(get("gate"), *self.gate.shape), "proj": _padded(get("proj"), *self.proj.shape),
+                "norm": _padded(get("norm"), *self.norm.shape)}
+
+    def forward(self, h, ids, table):
+        g = lm.matmul(h, self.gate, epi=lm.EPI_GELU_ROWS, ids=ids, table=table)
+        return lm.matmul_parts(g, self.proj)
 
     def init_random_(self, gen):
         _init_packed(self, self.pack, self.shapes(), gen)

@@ -15,13 +15,16 @@ from .faledra import FaledraConfig, FaledraForCausalLM
 from .golulix import GolulixConfig, GolulixForCausalLM
 from .llama import LlamaConfig, LlamaForCausalLM
 from .mllama import MllamaConfig, MllamaForConditionalGeneration
+from .nalizen import NalizenConfig, NalizenForCausalLM
 
 MODELS = {LlamaConfig: LlamaForCausalLM, MllamaConfig: MllamaForConditionalGeneration,
-          GolulixConfig: GolulixForCausalLM, FaledraConfig: FaledraForCausalLM}
+          GolulixConfig: GolulixForCausalLM, FaledraConfig: FaledraForCausalLM,
+          NalizenConfig: NalizenForCausalLM}
 
 # config.json "architecture" -> config reader, for designs that name themselves that way
 ARCHITECTURES: Dict[str, Callable[[dict], object]] = {"Golulix": GolulixConfig.from_json,
-                                                       "Faledra": FaledraConfig.from_json}
+                                                       "Faledra": FaledraConfig.from_json,
+                                                       "Nalizen": NalizenConfig.from_json}
 
 
 def config_from_json(d: dict):

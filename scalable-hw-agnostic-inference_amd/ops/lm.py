@@ -1,10 +1,10 @@
 """Decoder-block operators with an fp32 residual stream (``csrc/lm``, ``libshai_lm.so``).
 
-What a layer-list decoder needs beyond the Llama path of :mod:`shai_amd.ops`: an n-gram embedding, residual-add +
-RMSNorm with the residual kept in fp32 (optionally a norm on the added output and a short causal convolution on the
-normed one), one GEMM for dense, per-head and expert-grouped products, mixture-of-experts routing, attention restricted
-to fixed-size chunks of the sequence with a per-head output gate, attention over cached latents with a sink per head, and
-a gated linear recurrence.  Every op takes bf16 or fp32 weights and activations; norms, routing, attention scores,
+What a layer-list decoder needs beyond the Llama path of :mod:`shai_amd.ops`: an n-gram embedding, residual-add + norm
+(RMS or layer norm) with the residual kept in fp32 (optionally a norm on the added output and a short causal convolution
+on the sum or its norm), one GEMM for dense, per-head and expert-grouped products, mixture-of-experts routing, attention
+restricted to fixed-size chunks of the sequence or a sliding window with an output gate, attention over cached latents
+with a sink per head, a gated linear recurrence, and linear attention with a gated matrix state.  Every op takes bf16 or fp32 weights and activations; norms, routing, attention scores,
 rotation angles, recurrent state and the residual are fp32 in both.
 
 Layout rules shared by all of them: the model width is padded to a multiple of 64 (``pad64``; the pad columns of
@@ -24,7 +24,8 @@ import torch
 from .. import native
 from . import lm_reference as ref
 
-EPI_NONE, EPI_CLAMP_GLU, EPI_SOFTCAP, EPI_XIELU, EPI_ROTARY = 0, 1, 2, 3, 4
+EPI_NONE, EPI_CLAMP_GLU, EPI_SOFTCAP, EPI_XIELU, EPI_ROTARY, EPI_GELU_GLU, EPI_RELU2, EPI_GELU_ROWS = range(8)
+GLU_EPIS = (EPI_CLAMP_GLU, EPI_GELU_GLU)
 MAX_EXPERTS, MAX_TOP = 1024, 64
 MAX_TAPS = 16                # convolution taps
 MAX_LATENT = 1024            # columns of a cached latent
@@ -32,6 +33,7 @@ LATENT_SHORT = 16            # portions up to this many rows attend in latent sp
 LATENT_GROUP_ROWS = 1 << 18  # context rows that are expanded at a time
 PARTS, PARTS_COLUMNS = 4, 8192   # partial sums: at most so many, of products up to so wide in a decode step
 SCAN_CHUNK, SCAN_MAX_CHUNKS = 64, 64
+STATE_SEGMENT, STATE_MAX_SEGMENTS = 128, 32      # rows of a matrix-state segment at least; segments at most
 
 
 def pad64(n: int) -> int:
@@ -100,22 +102,25 @@ def add_norm(x, delta, inject, w, eps: float, width: int, dtype, rows=None):
 
 
 def matmul(a, w, out_dtype=None, epi: int = EPI_NONE, param: float = 0.0, plan: Optional[Plan] = None,
-           gather: bool = False, vec=None, rope=None, head: int = 0, rot0: int = 0):
+           gather: bool = False, vec=None, rope=None, head: int = 0, rot0: int = 0, ids=None, table=None):
     """c = epi(a w^T).  Dense: a [M, K], w [N, K].  Grouped (``plan``): w [E, N, K], row s of c belongs to the expert of
     slot s and reads a[token_of[s]] (``gather``) or a[s].
 
     EPI_CLAMP_GLU: w rows are (gate_i, up_i) pairs; with g = min(gate, param), u = clamp(up, +-param) the N / 2 outputs
     are g sigmoid(1.702 g) (u + 1).  EPI_SOFTCAP: param * tanh(c / param).  EPI_XIELU: vec[0] c^2 + c / 2 above zero,
     vec[1] (exp(c) - 1 - c) + c / 2 below.  EPI_ROTARY: columns rot0 .. rot0 + dims - 1 of every ``head`` columns are
-    interleaved pairs turned by the row's angles ``rope`` [M, dims] (:func:`rope_rows`)."""
+    interleaved pairs turned by the row's angles ``rope`` [M, dims] (:func:`rope_rows`).  EPI_GELU_GLU: w rows in pairs,
+    gelu_tanh(gate) up.  EPI_RELU2: max(c, 0)^2.  EPI_GELU_ROWS: gelu_tanh(c) times row ids[m] of ``table`` [rows, N] (a
+    view with any row stride)."""
     out_dtype = out_dtype or a.dtype
     if not a.is_cuda:
-        return ref.matmul(a, w, out_dtype, epi, param, plan, gather, vec, rope, head, rot0)
+        return ref.matmul(a, w, out_dtype, epi, param, plan, gather, vec, rope, head, rot0, ids, table)
     N = w.shape[-2]
     M = plan.token_of.shape[0] if plan is not None else a.shape[0]
-    c = torch.empty(M, N // 2 if epi == EPI_CLAMP_GLU else N, dtype=out_dtype, device=a.device)
+    c = torch.empty(M, N // 2 if epi in GLU_EPIS else N, dtype=out_dtype, device=a.device)
     if plan is None:
-        _K().lm_gemm(a, w, c, None, None, None, 0, int(epi), float(param), None, vec, rope, int(head), int(rot0))
+        _K().lm_gemm(a, w, c, None, None, None, 0, int(epi), float(param), None, vec, rope, int(head), int(rot0),
+                     ids, table)
     else:
         _K().lm_gemm(a, w, c, plan.tiles, plan.offsets, plan.token_of if gather else None, plan.bm, int(epi),
                      float(param))
@@ -128,7 +133,7 @@ def matmul_with_side(a, w, side: int, epi: int = EPI_NONE, param: float = 0.0):
     if not a.is_cuda:
         return ref.matmul(a, w[:-side], a.dtype, epi, param), ref.matmul(a, w[-side:], torch.float32, 0, 0.0)
     M, N = a.shape[0], w.shape[0]
-    c = torch.empty(M, (N - side) // (2 if epi == EPI_CLAMP_GLU else 1), dtype=a.dtype, device=a.device)
+    c = torch.empty(M, (N - side) // (2 if epi in GLU_EPIS else 1), dtype=a.dtype, device=a.device)
     s = torch.empty(M, side, dtype=torch.float32, device=a.device)
     _K().lm_gemm(a, w, c, None, None, None, 0, int(epi), float(param), s)
     return c, s
@@ -170,15 +175,16 @@ def grouped_bm(rows: int, experts: int) -> int:
     return 16 if rows < 48 * experts else 128 if rows < 512 * experts else 256
 
 
-def route(logits, top: int, groups: int, keep: int):
+def route(logits, top: int, groups: int, keep: int, bias=None, renorm: bool = False):
     """Group-limited top-k routing from fp32 logits [T, E]: (expert ids int32 [T, top], softmax scores fp32 [T, top]).
-    The E experts form ``groups`` equal runs; only the ``keep`` runs with the largest best score are eligible."""
+    The E experts form ``groups`` equal runs; only the ``keep`` runs with the largest best score are eligible.  ``bias``
+    [E] (fp32) is added to the logits; ``renorm``: the scores are a softmax over the chosen logits only."""
     if not logits.is_cuda:
-        return ref.route(logits, top, groups, keep)
+        return ref.route(logits, top, groups, keep, bias, renorm)
     T = logits.shape[0]
     ids = torch.empty(T, top, dtype=torch.int32, device=logits.device)
     wts = torch.empty(T, top, dtype=torch.float32, device=logits.device)
-    _K().moe_route(logits, int(groups), int(keep), ids, wts)
+    _K().moe_route(logits, int(groups), int(keep), ids, wts, bias, bool(renorm))
     return ids, wts
 
 
@@ -195,41 +201,63 @@ def plan_experts(ids, experts: int) -> Plan:
     return plan
 
 
-def route_experts(logits, top: int, groups: int, keep: int):
+def route_experts(logits, top: int, groups: int = 1, keep: int = 1, bias=None, renorm: bool = False):
     """:func:`route` and :func:`plan_experts` -> (combine weights [T, top], plan); one launch for a few tokens."""
     T, E = logits.shape
     if not logits.is_cuda or T > 16 or E > 256 or grouped_bm(T * top, E) != 16:
-        ids, wts = route(logits, top, groups, keep)
+        ids, wts = route(logits, top, groups, keep, bias, renorm)
         return wts, plan_experts(ids, E)
     P = T * top
     i32 = lambda *s: torch.empty(*s, dtype=torch.int32, device=logits.device)
     ids, wts = i32(T, top), torch.empty(T, top, dtype=torch.float32, device=logits.device)
     plan = Plan(i32(E + 1), i32(P), i32(T, top), i32(min(P, E + P // 16), 2), 16)
-    _K().moe_route_plan(logits, int(groups), int(keep), ids, wts, plan.offsets, plan.token_of, plan.slot_of, plan.tiles)
+    _K().moe_route_plan(logits, int(groups), int(keep), ids, wts, plan.offsets, plan.token_of, plan.slot_of, plan.tiles,
+                        bias, bool(renorm))
     return wts, plan
 
 
-def chunk_attention(qkvg, k_cache, v_cache, batch, heads: int, chunk: int, scale: float):
-    """Attention of one step over a paged cache: softmax over the keys j <= i of position i's own chunk (positions
-    chunk * n .. chunk * (n + 1) - 1), each head's output times sigmoid(its gate).
+class HeadTurn(NamedTuple):
+    """Rotation and norm of queries and keys before they meet: dimension i < rot / 2 of a head is turned with i + rot / 2 by
+    the row's angles ``rope`` [T, rot] (:func:`rope_rows`), then the head is divided by its rms over ``dim``."""
+    rope: torch.Tensor
+    dim: int
+    eps: float
 
-    ``qkvg`` [T, >= H dk + G (dk + dv) + H] holds q, k, v and the gate logits of the step's rows; k / v are written to
-    the caches [blocks, G, 64, dk | dv] at ``batch.slots`` (-1: padding row).  Returns [T, H dv]."""
+
+def gated_attention(qkvg, k_cache, v_cache, batch, heads: int, size: int, scale: float, window: bool = False,
+                    per_element: bool = False, own_kv: bool = True, turn: Optional[HeadTurn] = None):
+    """Attention of one step over a paged cache: softmax over the keys j <= i of position i's own chunk (positions
+    size * n .. size * (n + 1) - 1) or, with ``window``, of the size positions that end with i; the output times
+    sigmoid(gate logits), one per head or (``per_element``) per output element.
+
+    ``qkvg`` [T, >= H dk + G (dk + dv) + gates] holds q, k, v and the gate logits of the step's rows; k / v are written to
+    the caches [blocks, G, 64, dk | dv] at ``batch.slots`` (-1: padding row), with ``turn`` as the turned keys (and q may
+    be prepared in place).  ``own_kv`` False: rows are [q | gates], and the cache is another layer's, which has written
+    this step's rows.  Returns [T, H dv]."""
     if not qkvg.is_cuda:
-        return ref.chunk_attention(qkvg, k_cache, v_cache, batch, heads, chunk, scale)
+        return ref.gated_attention(qkvg, k_cache, v_cache, batch, heads, size, scale, window, per_element, own_kv, turn)
     dv = v_cache.shape[3]
     T = qkvg.shape[0]
     o = torch.empty(T, heads * dv, dtype=qkvg.dtype, device=qkvg.device)
     if batch.is_prefill:
-        _K().kv_store(qkvg, k_cache, v_cache, batch.slots, int(heads))
-        _K().chunk_attn_prefill(qkvg, k_cache, v_cache, o, batch.block_table, batch.ctx_lens, batch.q_lens,
-                                batch.q_start, int(batch.S), int(heads), int(chunk), float(scale))
+        if turn is not None:
+            _K().head_prep(qkvg, k_cache, v_cache, batch.slots, int(heads), turn.rope, int(turn.dim), float(turn.eps), own_kv)
+        elif own_kv:
+            _K().kv_store(qkvg, k_cache, v_cache, batch.slots, int(heads))
+        _K().gated_attn_prefill(qkvg, k_cache, v_cache, o, batch.block_table, batch.ctx_lens, batch.q_lens,
+                                batch.q_start, int(batch.S), int(heads), int(size), float(scale), window, per_element, own_kv)
         return o
-    ns = max(1, min(int(batch.num_splits or 1), (chunk + 63) // 64, 64))
+    ns = max(1, min(int(batch.num_splits or 1), (size + 63) // 64, 64))
     ws = torch.empty(T * heads * ns * (dv + 2) if ns > 1 else 0, dtype=torch.float32, device=qkvg.device)
-    _K().chunk_attn_decode(qkvg, k_cache, v_cache, o, batch.block_table, batch.ctx_lens, batch.slots, ws, int(heads),
-                           ns, int(chunk), float(scale))
+    _K().gated_attn_decode(qkvg, k_cache, v_cache, o, batch.block_table, batch.ctx_lens, batch.slots, ws, int(heads),
+                           ns, int(size), float(scale), window, per_element, own_kv,
+                           *(turn and (turn.rope, int(turn.dim), float(turn.eps)) or ()))
     return o
+
+
+def chunk_attention(qkvg, k_cache, v_cache, batch, heads: int, chunk: int, scale: float):
+    """:func:`gated_attention` inside chunks, a gate per head."""
+    return gated_attention(qkvg, k_cache, v_cache, batch, heads, chunk, scale)
 
 
 # ------------------------------------------------------------------------------------------- normed residual, convolution
@@ -240,9 +268,22 @@ class Embedding(NamedTuple):
     scale: float = 1.0
 
 
+class Affine(NamedTuple):
+    """Gain and bias of a layer norm ((x - mean) / sqrt(variance + eps) gain + bias), where a gain alone means an RMS norm."""
+    gain: Optional[torch.Tensor]
+    bias: Optional[torch.Tensor]
+
+
+PLAIN = Affine(None, None)   # no norm: the residual itself
+
+
+def _gain_bias(w):
+    return w if isinstance(w, Affine) else (w, None)
+
+
 @dataclass
 class Conv:
-    """Causal convolution over time on each channel of a norm's output, added to it: weight [taps, D] (fp32, oldest tap
+    """Causal convolution over time on each channel of a norm's output (or of the plain residual), added to it: weight [taps, D] (fp32, oldest tap
     first), state [slots, taps - 1, D] (fp32: the last inputs of every sequence).  ``tail`` [B, taps - 1, D] receives a
     prefill step's last inputs (:func:`conv_commit` moves them into the state); None: a decode step, state updated here."""
     weight: torch.Tensor
@@ -252,30 +293,38 @@ class Conv:
 
 def residual_norm(source, delta, wb, mult: float, step, w, eps: float, width: int, dtype, conv: Optional[Conv] = None,
                   batch=None, rows=None, keep: bool = True):
-    """x = source (+ mult * RMSNorm(delta) wb) (+ step); h = RMSNorm(x) w, plus its convolution with ``conv``.
+    """x = source (+ mult * norm(delta)) (+ step); h = norm(x), plus its convolution with ``conv``.
 
-    source: the fp32 residual [T, D] or an :class:`Embedding`.  delta: [T, D], or partial sums
-    [parts, T, D] fp32.  Returns (x, h); the residual may be updated in place.
-    ``w`` None: no norm (h None).  ``rows`` (int32): h of these rows only, and with ``keep`` False x is None."""
+    source: the fp32 residual [T, D] or an :class:`Embedding`.  delta: [T, D], partial sums [parts, T, D] fp32, or
+    :class:`Experts` without a dense part.  wb, w: the norms' gains (RMS norm) or :class:`Affine` (layer norm); w PLAIN:
+    h = x.  Returns (x, h); the residual may be updated in place.  ``w`` None: no h.  ``rows`` (int32): h of these rows only, and with ``keep`` False x is None."""
     emb = isinstance(source, Embedding)
     if not (source.ids if emb else source).is_cuda:
         return ref.residual_norm(source, delta, wb, mult, step, w, eps, width, dtype, conv, batch, rows, keep)
     ids, table, scale = source if emb else (None, None, 1.0)
     T, D = (ids.shape[0], table.shape[1]) if emb else source.shape
     dev = ids.device if emb else source.device
+    (wb, bb), no_h, (w, b) = _gain_bias(wb), w is None, _gain_bias(w)
+    ye = {}
+    if isinstance(delta, Experts):
+        assert delta.dense is None
+        ye = dict(ye=delta.y, slot_of=delta.slot_of, wts=delta.weights)
+        delta = None
     x = None
     if keep:
         x = torch.empty(T, D, dtype=torch.float32, device=dev) if emb or conv is not None else source
-    h = torch.empty(T if rows is None else rows.shape[0], D, dtype=dtype, device=dev) if w is not None else None
+    h = torch.empty(T if rows is None else rows.shape[0], D, dtype=dtype, device=dev) if not no_h else None
+    ye.update(bb=bb, b=b)
     args = (None if emb else source, ids, table, float(scale), delta, wb, float(mult), step, x, rows, w, float(eps),
             int(width), h)
     if conv is None:
-        _K().residual_norm(*args)
+        _K().residual_norm(*args, **ye)
     elif conv.tail is None:
-        _K().residual_norm(*args, conv.weight, conv.state, None, None, None, None, batch.positions, batch.state_slots)
+        _K().residual_norm(*args, conv.weight, conv.state, None, None, None, None, batch.positions, batch.state_slots,
+                           **ye)
     else:
         _K().residual_norm(*args, conv.weight, conv.state, conv.tail, batch.row_seq, batch.q_start, batch.q_lens,
-                           batch.positions, batch.state_slots)
+                           batch.positions, batch.state_slots, **ye)
     return x, h
 
 
@@ -288,10 +337,24 @@ def conv_commit(state, tail, batch) -> None:
 
 
 # ---------------------------------------------------------------------------------------------- rotary angles
-def rope_freq(base: float, dims: int) -> torch.Tensor:
-    """base^(-2 i / dims), i < dims / 2, as (float, remainder) pairs [dims / 2, 2]: angles of far positions keep their
-    32-bit accuracy."""
+class RopeScaling(NamedTuple):
+    """Frequency scaling by wavelength: those up to original / high stay, those from original / low on are divided by
+    ``factor``, and between the two the scaled and the unscaled frequency are blended."""
+    factor: float
+    low: float
+    high: float
+    original: float
+
+
+def rope_freq(base: float, dims: int, scaling: Optional[RopeScaling] = None) -> torch.Tensor:
+    """base^(-2 i / dims), i < dims / 2, scaled, as (float, remainder) pairs [dims / 2, 2]: angles of far positions keep
+    their 32-bit accuracy."""
     f = np.power(float(base), -2.0 * np.arange(dims // 2) / dims)
+    if scaling is not None:
+        turns = scaling.original * f / (2.0 * np.pi)         # full turns within the original length
+        s = np.clip((turns - scaling.low) / max(scaling.high - scaling.low, 1e-30), 0.0, 1.0)
+        f = np.where(turns > scaling.high, f, np.where(turns < scaling.low, f / scaling.factor,
+                                                       (1.0 - s) * f / scaling.factor + s * f))
     hi = f.astype(np.float32)
     return torch.tensor(np.stack([hi, (f - hi).astype(np.float32)], 1))
 
@@ -430,4 +493,30 @@ def mingru_scan(zx, g, bias, state, batch):
     chunks = -(-max_q // n)
     ws = torch.empty(batch.B * chunks * 2 * g.shape[1] if chunks > 1 else 0, dtype=torch.float32, device=g.device)
     _K().mingru_scan(zx, g, bias, state, out, batch.positions, batch.q_start, batch.q_lens, batch.state_slots, ws, max_q, n)
+    return out
+
+
+# ---------------------------------------------------------------------------------------------- matrix state
+def hgrn2(qv, z, bias, lower, gain, state, batch, vdim: int, eps: float):
+    """Linear attention whose forget gate also decides what is written: per head, with f = lower + (1 - lower)
+    sigmoid(z + bias), S = diag(f) S + (1 - f) v^T and o = S^T silu(q); returns o / rms(o over vdim) gain, [T, H dv].
+
+    qv [T, H dk + H dv]: queries and values; z [T, H dk] fp32 forget logits; bias, lower [H dk] (pads: lower 1); gain [dv].
+    ``state`` [slots, H, dk, dv] carries S (fp32); a sequence's first token starts from zero."""
+    if not qv.is_cuda:
+        return ref.hgrn2(qv, z, bias, lower, gain, state, batch, vdim, eps)
+    T, (_, H, dk, dv) = qv.shape[0], state.shape
+    out = torch.empty(T, H * dv, dtype=qv.dtype, device=qv.device)
+    max_q, n, unit = (int(batch.S) if batch.is_prefill else 1), STATE_SEGMENT, H * dk * (dv + 1)
+    segments = 1
+    if max_q > n and qv.dtype == torch.bfloat16:
+        # enough workgroups for the chip where few long sequences would not give them, in at most 256 MB of totals
+        want = min(-(-512 // (H * max(1, T // max_q))), STATE_MAX_SEGMENTS, max(1, (1 << 26) // (batch.B * unit)))
+        n = max(n, -(-max_q // (32 * want)) * 32)
+        segments = -(-max_q // n)
+    else:
+        n = -(-max_q // 32) * 32
+    ws = torch.empty(batch.B * segments * unit if segments > 1 else 0, dtype=torch.float32, device=qv.device)
+    _K().hgrn2(qv, z, bias, lower, gain, state, out, batch.positions, batch.q_start, batch.q_lens, batch.state_slots, ws,
+               max_q, n, int(vdim), float(eps))
     return out

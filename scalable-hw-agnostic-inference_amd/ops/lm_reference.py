@@ -35,8 +35,18 @@ def add_norm(x, delta, inject, w, eps, width, dtype, rows=None):
     return _norm(y, w, eps, width).to(dtype)
 
 
-def _epilogue(c, epi, param, vec=None, rope=None, head=0, rot0=0):
-    from .lm import EPI_CLAMP_GLU, EPI_ROTARY, EPI_SOFTCAP, EPI_XIELU
+def _gelu_tanh(z):
+    return torch.nn.functional.gelu(z, approximate="tanh")
+
+
+def _epilogue(c, epi, param, vec=None, rope=None, head=0, rot0=0, ids=None, table=None):
+    from .lm import EPI_CLAMP_GLU, EPI_GELU_GLU, EPI_GELU_ROWS, EPI_RELU2, EPI_ROTARY, EPI_SOFTCAP, EPI_XIELU
+    if epi == EPI_GELU_GLU:
+        return _gelu_tanh(c[..., 0::2]) * c[..., 1::2]
+    if epi == EPI_RELU2:
+        return torch.relu(c) ** 2
+    if epi == EPI_GELU_ROWS:
+        return _gelu_tanh(c) * table[ids.long()].float()
     if epi == EPI_CLAMP_GLU:
         g = c[..., 0::2].clamp(max=param)
         u = c[..., 1::2].clamp(-param, param)
@@ -58,9 +68,9 @@ def _turn(x, rope):
     return torch.stack([u * cs - v * sn, v * cs + u * sn], -1).flatten(-2)
 
 
-def matmul(a, w, out_dtype, epi, param, plan=None, gather=False, vec=None, rope=None, head=0, rot0=0):
+def matmul(a, w, out_dtype, epi, param, plan=None, gather=False, vec=None, rope=None, head=0, rot0=0, ids=None, table=None):
     if plan is None:
-        return _epilogue(a.float() @ w.float().T, epi, param, vec, rope, head, rot0).to(out_dtype)
+        return _epilogue(a.float() @ w.float().T, epi, param, vec, rope, head, rot0, ids, table).to(out_dtype)
     rows = a[plan.token_of.long()] if gather else a
     off = plan.offsets.tolist()
     parts = [_epilogue(rows[off[e]:off[e + 1]].float() @ w[e].float().T, epi, param)
@@ -68,12 +78,15 @@ def matmul(a, w, out_dtype, epi, param, plan=None, gather=False, vec=None, rope=
     return torch.cat(parts, 0).to(out_dtype)
 
 
-def route(logits, top, groups, keep):
-    s = torch.softmax(logits.float(), -1)
+def route(logits, top, groups, keep, bias=None, renorm=False):
+    logits = logits.float() if bias is None else logits.float() + bias
+    s = torch.softmax(logits, -1)
     T, E = s.shape
     best = s.view(T, groups, E // groups).amax(-1)
     ok = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, best.topk(keep, -1).indices, True)
     w, ids = s.masked_fill(~ok.repeat_interleave(E // groups, 1), -1.0).topk(top, -1)
+    if renorm:
+        w = torch.softmax(logits.gather(1, ids), -1)
     return ids.int(), w
 
 
@@ -89,12 +102,26 @@ def plan_experts(ids, experts, bm):
     return Plan(off, (order // top).int(), slot_of.view(T, top), torch.empty(0, 2, dtype=torch.int32), bm)
 
 
-def chunk_attention(qkvg, k_cache, v_cache, batch, heads, chunk, scale):
+def _turn_heads(x, dim_pad, turn):
+    """Rotation (dimension i with i + rot / 2) and rms norm of every head of x [T, heads * dim_pad]."""
+    x = x.float().view(x.shape[0], -1, dim_pad).clone()
+    half = turn.rope.shape[1] // 2
+    cs, sn = turn.rope[:, None, 0::2], turn.rope[:, None, 1::2]
+    u, v = x[..., :half].clone(), x[..., half:2 * half].clone()
+    x[..., :half], x[..., half:2 * half] = u * cs - v * sn, v * cs + u * sn
+    return x / torch.sqrt(x.pow(2).sum(-1, keepdim=True) / turn.dim + turn.eps)
+
+
+def gated_attention(qkvg, k_cache, v_cache, batch, heads, size, scale, window, per_element, own_kv, turn):
     G, dk, dv = k_cache.shape[1], k_cache.shape[3], v_cache.shape[3]
     T = qkvg.shape[0]
-    q, k, v, gate = qkvg[:, :heads * dk + G * (dk + dv) + heads].split([heads * dk, G * dk, G * dv, heads], -1)
+    n_gate, kv = heads * (dv if per_element else 1), (G * dk, G * dv) if own_kv else (0, 0)
+    q, k, v, gate = qkvg[:, :heads * dk + sum(kv) + n_gate].split([heads * dk, *kv, n_gate], -1)
+    if turn is not None:
+        q = _turn_heads(q, dk, turn).to(qkvg.dtype).view(T, -1)
+        k = _turn_heads(k, dk, turn).to(qkvg.dtype).view(T, -1) if own_kv else k
     for t, slot in enumerate(batch.slots[:T].tolist()):
-        if slot >= 0:
+        if slot >= 0 and own_kv:
             k_cache[slot // 64, :, slot % 64] = k[t].view(G, dk)
             v_cache[slot // 64, :, slot % 64] = v[t].view(G, dv)
     o = torch.zeros(T, heads, dv)
@@ -105,12 +132,12 @@ def chunk_attention(qkvg, k_cache, v_cache, batch, heads, chunk, scale):
         bt = batch.block_table[b].long()
         for i in range(n_q):
             pos = ctx - n_q + i
-            key = torch.arange(pos // chunk * chunk, pos + 1)
+            key = torch.arange(max(0, pos - size + 1) if window else pos // size * size, pos + 1)
             kk = k_cache[bt[key // 64], :, key % 64].float().repeat_interleave(heads // G, 1)   # [n, H, dk]
             vv = v_cache[bt[key // 64], :, key % 64].float().repeat_interleave(heads // G, 1)
             s = torch.einsum("hd,nhd->hn", q[row0 + i].float().view(heads, dk), kk) * scale
             o[row0 + i] = torch.einsum("hn,nhd->hd", torch.softmax(s, -1), vv)
-    return (o * torch.sigmoid(gate.float())[..., None]).reshape(T, heads * dv).to(qkvg.dtype)
+    return (o * torch.sigmoid(gate.float()).view(T, heads, -1)).reshape(T, heads * dv).to(qkvg.dtype)
 
 
 def _sequences(batch):
@@ -122,8 +149,19 @@ def _sequences(batch):
 
 
 def residual_norm(source, delta, wb, mult, step, w, eps, width, dtype, conv, batch, rows, keep):
-    from .lm import Embedding
-    rms = lambda t, gain: t / torch.sqrt(t.pow(2).sum(-1, keepdim=True) / width + eps) * gain
+    from .lm import PLAIN, Affine, Embedding, Experts
+
+    def rms(t, w):
+        gain, bias = w if isinstance(w, Affine) else (w, None)
+        if w is PLAIN:
+            return t
+        if bias is not None:
+            mean = t.sum(-1, keepdim=True) / width
+            t = torch.where(torch.arange(t.shape[-1]) < width, t - mean, torch.zeros(()))
+        y = t / torch.sqrt(t.pow(2).sum(-1, keepdim=True) / width + eps) * gain
+        return y if bias is None else y + bias
+    if isinstance(delta, Experts):
+        delta = (delta.y.float()[delta.slot_of.long()] * delta.weights[..., None]).sum(1)
     x = source.table[source.ids.long()].float() * source.scale if isinstance(source, Embedding) else source.clone()
     if delta is not None:
         x = x + mult * rms(delta.float(), wb)
@@ -222,3 +260,21 @@ def mingru_scan(zx, g, bias, state, batch):
         if slot >= 0:
             state[slot] = s
     return (S * torch.nn.functional.silu(g.float())).to(g.dtype)
+
+
+def hgrn2(qv, z, bias, lower, gain, state, batch, vdim, eps):
+    _, H, dk, dv = state.shape
+    T = qv.shape[0]
+    q = torch.nn.functional.silu(qv[:, :H * dk].float()).view(T, H, dk)
+    v = qv[:, H * dk:].float().view(T, H, dv)
+    f = (lower + (1 - lower) * torch.sigmoid(z + bias)).view(T, H, dk)
+    k = ((1 - lower) * torch.sigmoid(-(z + bias))).view(T, H, dk)
+    o = torch.zeros(T, H, dv)
+    for row0, n, pos, slot, _ in _sequences(batch):
+        S = state[slot].clone() if slot >= 0 and pos > 0 else torch.zeros(H, dk, dv)
+        for t in range(row0, row0 + n):
+            S = f[t][..., None] * S + k[t][..., None] * v[t][:, None]
+            o[t] = (S * q[t][..., None]).sum(1)
+        if slot >= 0:
+            state[slot] = S
+    return (o / torch.sqrt(o.pow(2).sum(-1, keepdim=True) / vdim + eps) * gain).reshape(T, H * dv).to(qv.dtype)
