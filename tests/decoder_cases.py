@@ -1,4 +1,4 @@
-"""What the tests of the layer-list decoders (Golulix, Faledra) share: cases on the framework's engine, driven by portions,
+"""What the tests of the layer-list decoders (Golulix, Faledra, Nalizen) share: cases on the framework's engine, driven by portions,
 batches, generation and trace replay, and their comparison with a design's oracle."""
 import json
 
@@ -6,9 +6,12 @@ import numpy as np
 import torch
 
 from shai_amd.engines import trace
+from shai_amd.models.llama import Batch
+from shai_amd.ops import lm
 
 # error of a position: rms over the vocabulary of the logit difference (mean taken off), in units of the logits' rms
 F32_TOL, BF16_TOL = 1e-4, 0.06
+JUNK = 37.0                      # what caches and state slots hold before anything is written
 
 
 def position_errors(got, want):
@@ -61,7 +64,7 @@ class Case:
         eng = trace.build_engine(self.path, name(self.dtype), max_tokens, self.device)
         if dirty:   # whatever an unwritten cache row or state slot holds must not matter
             for t in tensors((eng.kv, eng.states)):
-                t.fill_(37.0)
+                t.fill_(JUNK)
         return eng
 
 
@@ -128,3 +131,73 @@ def check_replay_files(c, toks, out, said, dtype):
     assert_logits(read(7), want[[1, 31]], dtype)
     assert_logits(read(8), want[[0]], dtype)
     assert not (out / "1.f32").exists()
+
+
+# ---------------------------------------------------------------------------------------------- blocks without an engine
+def pad(t, n=None):
+    """The last axis with zeros up to ``n`` (default: the next multiple of 64)."""
+    return torch.nn.functional.pad(t, (0, (n or lm.pad64(t.shape[-1])) - t.shape[-1]))
+
+
+def close(got, want, tol, what=""):
+    err = (got.double().cpu() - want.double()).abs().max()
+    assert err < tol, f"{what}: {err:.2e}"
+
+
+def whole(y):
+    """A block's output, its partial sums added."""
+    return y.sum(0) if y.dim() == 3 else y
+
+
+class Stepper:
+    """Sequences in a paged pool with shuffled pages and state slots: ``step`` makes the batch of their next rows."""
+
+    def __init__(self, lengths, device, blocks=None, slots=None):
+        self.device, self.at = device, [0] * len(lengths)
+        g = torch.Generator().manual_seed(sum(lengths))
+        need = [(n + 63) // 64 for n in lengths]
+        perm = torch.randperm(sum(need) + 3, generator=g).tolist()
+        self.blocks = sum(need) + 3
+        self.table = torch.zeros(len(lengths), max(need), dtype=torch.int32)
+        for b, n in enumerate(need):
+            self.table[b, :n] = torch.tensor([perm.pop() for _ in range(n)])
+        self.slots = torch.randperm(len(lengths) + 2, generator=g)[:len(lengths)].int()
+
+    def step(self, news, splits=1):
+        """``news``: rows of every sequence (0: left out).  Returns (batch, [(sequence, first position, rows)])."""
+        d = self.device
+        i32 = lambda x: torch.as_tensor(x, dtype=torch.int32).to(d).contiguous()
+        who = [(b, self.at[b], n) for b, n in enumerate(news) if n]
+        pos = torch.cat([torch.arange(p, p + n) for _, p, n in who])
+        seq = torch.cat([torch.full((n,), b) for b, _, n in who])
+        cell = self.table[seq, pos // 64] * 64 + pos % 64
+        for b, _, n in who:
+            self.at[b] += n
+        bt, ctx = i32(self.table[[b for b, _, _ in who]]), [p + n for _, p, n in who]
+        slots = i32(self.slots[[b for b, _, _ in who]])
+        if max(news) == 1:
+            return Batch(i32(pos), i32(pos), i32(cell), bt, i32(ctx), None, len(who), 1, False, splits,
+                         state_slots=slots), who
+        ql = [n for _, _, n in who]
+        start = [sum(ql[:i]) for i in range(len(ql))]
+        return Batch(i32(pos), i32(pos), i32(cell), bt, i32(ctx), i32(ql), len(who), max(ql), True, 1, q_start=i32(start),
+                     state_slots=slots, row_seq=i32([i for i, n in enumerate(ql) for _ in range(n)]), q_lens_host=ql,
+                     ctx_lens_host=ctx), who
+
+
+def drive(lengths, cuts, device, fn, splits=1):
+    """Feed every sequence in portions (``cuts``: cycled, another phase per sequence, 0 leaves it out), all in one batch;
+    ``fn(batch, rows)`` gets the (sequence, position) rows and returns their outputs.  -> [output of every sequence]."""
+    st, i, out = Stepper(lengths, device), 0, [[] for _ in lengths]
+    while any(a < n for a, n in zip(st.at, lengths)):
+        news = [min(cuts[(i + b) % len(cuts)], n - st.at[b]) for b, n in enumerate(lengths)]
+        i += 1
+        if not any(news):
+            continue
+        batch, who = st.step(news, splits)
+        y = fn(batch, [(b, p + j) for b, p, n in who for j in range(n)])
+        at = 0
+        for b, _, n in who:
+            out[b].append(y[at:at + n].cpu())
+            at += n
+    return [torch.cat(o) for o in out]

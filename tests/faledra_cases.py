@@ -5,16 +5,13 @@ import copy
 import decoder_cases
 import faledra_reference as R
 import torch
-from decoder_cases import (F32_TOL, check_replay_files, greedy_oracle, name,  # noqa: F401
-                           position_errors, replay_lines, run, run_batches)
+from decoder_cases import (F32_TOL, JUNK, Stepper, check_replay_files, close, drive, greedy_oracle, name,  # noqa: F401
+                           pad, position_errors, replay_lines, run, run_batches, whole)
 
 from shai_amd.engines.llm import LLMEngine, SamplingParams
 from shai_amd.models.blocks import LatentAttention, LatentAttentionConfig, MinGRU, StepShared, XieluMLP
-from shai_amd.models.llama import Batch
 from shai_amd.models.registry import config_from_json
 from shai_amd.ops import lm
-
-JUNK = 37.0                      # what caches and state slots hold before anything is written
 
 
 def assert_logits(got, want, dtype, what=""):
@@ -25,75 +22,6 @@ def assert_logits(got, want, dtype, what=""):
 
 class Case(decoder_cases.Case):
     ref = R
-
-
-def pad(t, n=None):
-    """The last axis with zeros up to ``n`` (default: the next multiple of 64)."""
-    return torch.nn.functional.pad(t, (0, (n or lm.pad64(t.shape[-1])) - t.shape[-1]))
-
-
-def close(got, want, tol, what=""):
-    err = (got.double().cpu() - want.double()).abs().max()
-    assert err < tol, f"{what}: {err:.2e}"
-
-
-def whole(y):
-    """A block's output, its partial sums added."""
-    return y.sum(0) if y.dim() == 3 else y
-
-
-class Stepper:
-    """Sequences in a paged pool with shuffled pages and state slots: ``step`` makes the batch of their next rows."""
-
-    def __init__(self, lengths, device, blocks=None, slots=None):
-        self.device, self.at = device, [0] * len(lengths)
-        g = torch.Generator().manual_seed(sum(lengths))
-        need = [(n + 63) // 64 for n in lengths]
-        perm = torch.randperm(sum(need) + 3, generator=g).tolist()
-        self.blocks = sum(need) + 3
-        self.table = torch.zeros(len(lengths), max(need), dtype=torch.int32)
-        for b, n in enumerate(need):
-            self.table[b, :n] = torch.tensor([perm.pop() for _ in range(n)])
-        self.slots = torch.randperm(len(lengths) + 2, generator=g)[:len(lengths)].int()
-
-    def step(self, news, splits=1):
-        """``news``: rows of every sequence (0: left out).  Returns (batch, [(sequence, first position, rows)])."""
-        d = self.device
-        i32 = lambda x: torch.as_tensor(x, dtype=torch.int32).to(d).contiguous()
-        who = [(b, self.at[b], n) for b, n in enumerate(news) if n]
-        pos = torch.cat([torch.arange(p, p + n) for _, p, n in who])
-        seq = torch.cat([torch.full((n,), b) for b, _, n in who])
-        cell = self.table[seq, pos // 64] * 64 + pos % 64
-        for b, _, n in who:
-            self.at[b] += n
-        bt, ctx = i32(self.table[[b for b, _, _ in who]]), [p + n for _, p, n in who]
-        slots = i32(self.slots[[b for b, _, _ in who]])
-        if max(news) == 1:
-            return Batch(i32(pos), i32(pos), i32(cell), bt, i32(ctx), None, len(who), 1, False, splits,
-                         state_slots=slots), who
-        ql = [n for _, _, n in who]
-        start = [sum(ql[:i]) for i in range(len(ql))]
-        return Batch(i32(pos), i32(pos), i32(cell), bt, i32(ctx), i32(ql), len(who), max(ql), True, 1, q_start=i32(start),
-                     state_slots=slots, row_seq=i32([i for i, n in enumerate(ql) for _ in range(n)]), q_lens_host=ql,
-                     ctx_lens_host=ctx), who
-
-
-def drive(lengths, cuts, device, fn, splits=1):
-    """Feed every sequence in portions (``cuts``: cycled, another phase per sequence, 0 leaves it out), all in one batch;
-    ``fn(batch, rows)`` gets the (sequence, position) rows and returns their outputs.  -> [output of every sequence]."""
-    st, i, out = Stepper(lengths, device), 0, [[] for _ in lengths]
-    while any(a < n for a, n in zip(st.at, lengths)):
-        news = [min(cuts[(i + b) % len(cuts)], n - st.at[b]) for b, n in enumerate(lengths)]
-        i += 1
-        if not any(news):
-            continue
-        batch, who = st.step(news, splits)
-        y = fn(batch, [(b, p + j) for b, p, n in who for j in range(n)])
-        at = 0
-        for b, _, n in who:
-            out[b].append(y[at:at + n].cpu())
-            at += n
-    return [torch.cat(o) for o in out]
 
 
 # ---------------------------------------------------------------------------------------------- mechanisms alone

@@ -152,3 +152,83 @@ def forward(tokens, cfg, w, dtype=torch.float64):
         x = x + side_input(x, e, eps, w[p + "side.gate"], w[p + "side.proj"], w[p + "side.norm"])
         trail.append(x)
     return layer_norm(x, w["final.norm"], w["final.norm.b"], eps) @ w["embed"].T, trail
+
+
+# ---------------------------------------------------------------------------------------------- random models
+def dense(ff=40):
+    return {"kind": "dense", "ff": ff}
+
+
+def experts(n=5, top=2, ff=24):
+    return {"kind": "moe", "router": {"experts": n, "top": top}, "expert": {"ff": ff}}
+
+
+def scaling(factor=6.0, low=0.7, high=3.0, original=90):
+    return {"factor": factor, "low": low, "high": high, "original": original}
+
+
+def attention_layer(heads=6, kv_heads=2, dim=20, vdim=28, window=37, base=60.0, dims=12, scale=0.4, stretch=scaling(),
+                    kv_from=None, mlp=dense()):
+    rot = {"base": base, "dims": dims}
+    if stretch:
+        rot["scaling"] = dict(stretch)
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "mask": {"size": window}, "rot": rot, "scale": scale}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "attention", "mixer": m, "mlp": mlp and dict(mlp)}
+
+
+def hgrn2_layer(heads=3, dim=20, vdim=36, mlp=experts()):
+    return {"type": "hgrn2", "mixer": {"heads": heads, "dim": dim, "vdim": vdim}, "mlp": mlp and dict(mlp)}
+
+
+def random_config(layers=None, vocab=97, width=56, side=10, embed_scale=2.5, eps=1e-4):
+    layers = layers or [attention_layer(), hgrn2_layer(), attention_layer(kv_from=0, window=51, scale=0.3, mlp=experts()),
+                        hgrn2_layer(2, 70, 24, dense(50))]
+    return {"architecture": "Nalizen", "vocab": vocab, "width": width, "norm": {"eps": eps}, "token_side": {"dim": side},
+            "embedding": {"scale": embed_scale}, "layers": layers}
+
+
+def random_weights(cfg, seed=0):
+    """bfloat16-exact random weights under their checkpoint names (fp32 tensors)."""
+    g = torch.Generator().manual_seed(seed)
+    b = lambda t: t.bfloat16().float()
+    r = lambda *s, std=None: b(torch.randn(*s, generator=g) * (s[-1] ** -0.5 if std is None else std))
+    gain = lambda n: b(1.0 + 0.3 * torch.randn(n, generator=g))
+    D, L, S = cfg["width"], len(cfg["layers"]), cfg["token_side"]["dim"]
+    w = {"embed": r(cfg["vocab"], D, std=0.5), "side.embed": r(cfg["vocab"], L * S, std=1.0),
+         "final.norm": gain(D), "final.norm.b": r(D, std=0.3)}
+    for i, lc in enumerate(cfg["layers"]):
+        m, p, ff = lc["mixer"], f"l{i}.", lc.get("mlp")
+        w[p + "norm1"], w[p + "norm1.b"], w[p + "shift"] = gain(D), r(D, std=0.3), b(torch.rand(D, generator=g) * 1.2 - 0.1)
+        w[p + "side.gate"], w[p + "side.proj"], w[p + "side.norm"] = r(S, D), r(D, S), b(0.5 * gain(D))
+        H, d, vd = m["heads"], m["dim"], m["vdim"]
+        w[p + "mix.q"], w[p + "mix.o"] = r(H * d, D), r(D, H * vd)
+        if lc["type"] == "attention":
+            w[p + "mix.g"] = r(H * vd, D)
+            if m.get("kv_from") is None:
+                w[p + "mix.k"], w[p + "mix.v"] = r(m["kv_heads"] * d, D), r(m["kv_heads"] * vd, D)
+        else:
+            w[p + "mix.f"], w[p + "mix.f.b"], w[p + "mix.v"] = r(H * d, D), r(H * d, std=1.0), r(H * vd, D)
+            w[p + "mix.lower"] = b(torch.rand(H * d, generator=g) ** 0.3 * 0.98)       # many channels reach far back
+            w[p + "mix.norm"] = gain(vd)
+        if ff:
+            w[p + "norm2"], w[p + "norm2.b"] = gain(D), r(D, std=0.3)
+        if ff and ff["kind"] == "dense":
+            w[p + "mlp.gate"], w[p + "mlp.up"], w[p + "mlp.down"] = r(ff["ff"], D), r(ff["ff"], D), r(D, ff["ff"])
+        elif ff:
+            E, F = ff["router"]["experts"], ff["expert"]["ff"]
+            w[p + "mlp.router"], w[p + "mlp.router.b"] = r(E, D, std=2 * D ** -0.5), r(E, std=1.0)
+            for e in range(E):
+                w[p + f"mlp.e{e}.up"], w[p + f"mlp.e{e}.down"] = r(F, D), r(D, F)
+    return w
+
+
+def save_checkpoint(path, cfg, w):
+    """config.json + model.safetensors (bfloat16) in ``path``."""
+    from safetensors.torch import save_file
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    save_file({k: v.bfloat16().contiguous() for k, v in w.items()}, os.path.join(path, "model.safetensors"))
+    return str(path)

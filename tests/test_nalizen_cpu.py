@@ -1,0 +1,139 @@
+"""Nalizen on the CPU references: the engine integration (registry, loader, cache, state slots, scheduler, sampling, trace
+replay) against the plain oracle, and that the comparison notices a planted mistake."""
+import copy
+
+import nalizen_cases as C
+import nalizen_reference as R
+import pytest
+import torch
+
+CPU, F32, BF16 = "cpu", torch.float32, torch.bfloat16
+
+
+@pytest.mark.parametrize("check", C.MECHANISMS, ids=lambda f: f.__name__)
+def test_mechanism(check):
+    check(CPU, F32)
+
+
+@pytest.mark.parametrize("key", sorted(C.SHAPES))
+def test_shapes(tmp_path, key):
+    C.check_shape(tmp_path, CPU, F32, key)
+
+
+@pytest.mark.parametrize("check", C.MODELS, ids=lambda f: f.__name__)
+def test_model(tmp_path, check):
+    check(tmp_path, CPU, F32)
+
+
+def test_model_bf16(tmp_path):
+    C.check_batches(tmp_path, CPU, BF16)
+
+
+@pytest.mark.parametrize("kw", [{}, {"async_decode": False}, {"mixed_steps": False}, {"num_kv_blocks": 7}],
+                         ids=["default", "sync", "unmixed", "preempt"])
+def test_greedy_generation(tmp_path, kw):
+    C.check_greedy(tmp_path, CPU, F32, **kw)
+
+
+def test_planted_mistakes_show(tmp_path):
+    c = C.Case(tmp_path, CPU, F32, seed=11)
+    toks = c.tokens(64)
+    eng = c.engine()
+    got = C.run(eng, eng.open_request(), toks, (40, 1, 2))
+    assert C.position_errors(got, c.oracle(toks)).max() < C.F32_TOL
+    for what, cfg, w in C.planted(c.cfg, c.w):
+        e = C.position_errors(got, R.forward(toks, cfg, w)[0])
+        assert e.max() > 50 * C.F32_TOL, what
+
+
+def test_checkpoint_must_fit(tmp_path):
+    from shai_amd.engines import trace
+    c = C.Case(tmp_path, CPU, F32, seed=12)
+    for change in (lambda w: w.pop("l1.shift"), lambda w: w.update({"l2.mix.k": w["l0.mix.k"]}),
+                   lambda w: w.update({"side.embed": w["side.embed"][:, 1:]})):
+        w = dict(c.w)
+        change(w)
+        path = R.save_checkpoint(tmp_path / "bad", c.cfg, w)
+        with pytest.raises(ValueError, match="does not fit"):
+            trace.build_engine(path, "float32", 128, CPU)
+
+
+def test_registry_and_config(tmp_path):
+    from shai_amd.engines.llm import LLMEngine, llama_config_for
+    from shai_amd.models.nalizen import NalizenConfig, NalizenForCausalLM
+    from shai_amd.models.registry import config_from_json, model_class
+    c = C.Case(tmp_path, CPU, F32, seed=13)
+    cfg = llama_config_for("anything", c.path)
+    assert isinstance(cfg, NalizenConfig) and model_class(cfg) is NalizenForCausalLM
+    assert isinstance(llama_config_for("nalizen", None, "tiny"), NalizenConfig)
+
+    def changed(i, fn):
+        layers = copy.deepcopy(c.cfg["layers"])
+        fn(layers[i])
+        return dict(c.cfg, layers=layers)
+    for bad in (changed(2, lambda x: x["mixer"].update(kv_from=1)), changed(2, lambda x: x["mixer"].update(kv_from=2)),
+                changed(2, lambda x: x["mixer"].update(kv_heads=3)), changed(2, lambda x: x["mixer"]["rot"].update(base=9.0)),
+                changed(0, lambda x: x["mixer"]["rot"].update(dims=7)), changed(0, lambda x: x["mixer"]["mask"].update(size=0)),
+                changed(0, lambda x: x.update(type="recurrent")), changed(1, lambda x: x["mlp"].update(kind="other")),
+                changed(1, lambda x: x["mlp"]["router"].update(top=9)), dict(c.cfg, layers=[])):
+        with pytest.raises(ValueError):
+            cfg = config_from_json(bad)
+            model_class(cfg)(cfg, F32)
+    with pytest.raises(ValueError):
+        LLMEngine(NalizenConfig.tiny(), device=CPU, quantization="fp8")
+
+
+def test_shared_keys_take_no_cache():
+    """A layer that uses another one's keys and values has no pool of its own."""
+    from shai_amd.models.nalizen import NalizenConfig, NalizenForCausalLM
+    sizes = (64, 4, 2, 32, 40, 2, 24, 40, 64, 4, 2, 32, 8, 50)
+    one, two = (NalizenForCausalLM(NalizenConfig.uniform(k, *sizes)) for k in ("ar", "arS"))
+    assert one.cache_bytes_per_block() == two.cache_bytes_per_block() > 0
+    kv, by_layer = two.allocate_cache(3, CPU)
+    assert by_layer[2][0] is by_layer[0][0] and by_layer[1] is None
+
+
+def test_random_init_generates():
+    """No checkpoint: deterministic random weights, zero padding, tokens through the scheduler and the sampler."""
+    from shai_amd.engines.llm import LLMEngine, SamplingParams
+    from shai_amd.models.nalizen import NalizenConfig
+    mk = lambda: LLMEngine(NalizenConfig.tiny(), device=CPU, max_num_seqs=2, max_model_len=128)
+    a, b = mk(), mk()
+    assert all(torch.equal(x, y) for x, y in zip(a.model.parameters(), b.model.parameters()))
+    p = SamplingParams(max_tokens=6, seed=1)
+    out = [s.output for s in a.generate([[1, 2, 3], [7] * 70], p)]
+    assert out == [s.output for s in b.generate([[1, 2, 3], [7] * 70], p)] and all(len(o) == 6 for o in out)
+
+
+def test_aborted_requests_give_slots_back():
+    from shai_amd.engines.llm import LLMEngine
+    from shai_amd.models.nalizen import NalizenConfig
+    eng = LLMEngine(NalizenConfig.tiny(), device=CPU, max_num_seqs=2, max_model_len=128)
+    for _ in range(3):
+        eng.add_request([1, 2, 3])
+    eng.step()
+    assert eng.state_slots.num_free == 0
+    eng.abort_all()
+    assert eng.state_slots.num_free == 2 and eng.bm.num_free == eng.num_kv_blocks
+
+
+def test_trace_replay(tmp_path):
+    from shai_amd.engines import trace
+    c = C.Case(tmp_path, CPU, F32, seed=14)
+    toks, said = c.tokens(32), []
+    out = tmp_path / "out"
+    out.mkdir()
+    eng = trace.build_engine(c.path, "float32", 128, CPU)
+    assert eng.num_kv_blocks == 2 and eng.max_num_seqs == 4 and eng.state_slots.num_free == 4
+    trace.replay(eng, C.replay_lines(c, toks), str(out), said.append)
+    C.check_replay_files(c, toks, out, said, F32)
+
+
+def test_serving_api_with_nalizen():
+    from fastapi.testclient import TestClient
+    from shai_amd.serving.common import ServerEnv
+    from shai_amd.serving.llm_api import create_app
+    env = ServerEnv(app="llm", model_id="nalizen", device="cpu", config="tiny", pod_name="p")
+    with TestClient(create_app(env=env)) as client:
+        r = client.post("/generate", json={"prompt": "hello there", "max_new_tokens": 4})
+        assert r.status_code == 200 and r.json()["text"]
