@@ -52,8 +52,8 @@ EXTRA_KFLAGS = {"kernels/attention3.hip": "-mllvm -amdgpu-mfma-vgpr-form -fno-sl
 BINDING_SRCS = ["bindings.cpp"]
 # the decoder-block kernels and the token-level ops of every language model's step (their own library: a model that
 # runs on them alone needs nothing else compiled)
-LM_SRCS = ["lm/norm.hip", "lm/gemm.hip", "lm/gemm_tile.hip", "lm/moe.hip", "lm/attn.hip", "lm/latent.hip", "lm/scan.hip", "lm/hgrn2.hip",
-           "kernels/sampling.hip"]
+LM_SRCS = ["lm/norm.hip", "lm/gemm.hip", "lm/gemm_tile.hip", "lm/moe.hip", "lm/attn.hip", "lm/latent.hip", "lm/scan.hip",
+           "lm/hgrn2.hip", "kernels/sampling.hip"]
 LM_BINDING_SRCS = ["lm/bindings.cpp"]
 RUNTIME_SRCS = ["runtime/block_manager.cpp", "runtime/scheduler.cpp"]
 COMM_SRCS = ["comm/p2p_allreduce.hip"]

@@ -305,7 +305,9 @@ void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const
   a.width = width;
   a.eps = eps;
   long R;
-  at::ScalarType dt = h ? h->scalar_type() : ye ? ye->scalar_type() : delta ? delta->scalar_type() : table ? table->scalar_type() : at::kFloat;
+  at::ScalarType dt = at::kFloat;               // of every tensor but the residual and partial sums
+  for (auto* t : {&delta, &table, &ye, &h})
+    if (*t) dt = (*t)->scalar_type();
   SHAI_CHECK(dt == at::kFloat || dt == at::kBFloat16, "bf16 or fp32");
   SHAI_CHECK(x.has_value() != ids.has_value(), "residual_norm: a residual or token ids");
   if (x) {
@@ -343,7 +345,8 @@ void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const
   }
   if (ye) {  // the weighted outputs of a token's experts
     check(*ye, dt, "ye");
-    SHAI_CHECK(!delta && wb.has_value() && slot_of.has_value() && wts.has_value(), "expert outputs: the only delta, with slot_of, weights and gain");
+    SHAI_CHECK(!delta && wb.has_value() && slot_of.has_value() && wts.has_value(),
+               "expert outputs: the only delta, with slot_of, weights and gain");
     check_i32(*slot_of, "slot_of");
     check(*wts, at::kFloat, "wts");
     a.top = slot_of->size(1);
@@ -665,8 +668,8 @@ void hgrn2(const Tensor& qv, const Tensor& z, const Tensor& bias, const Tensor& 
   a.dv = state.size(3);
   SHAI_CHECK((a.dk == 64 && a.dv == 64) || (a.dk == 64 && a.dv == 128) || (a.dk == 128 && a.dv == 64) ||
                  (a.dk == 128 && a.dv == 128) || (a.dk == 256 && a.dv == 256), "stored head sizes: 64 / 128 each, or 256 / 256");
-  SHAI_CHECK(a.H >= 1 && a.H <= 65535 && qv.size(1) == (long)a.H * (a.dk + a.dv) && z.size(0) == a.T && z.size(1) == (long)a.H * a.dk &&
-                 bias.numel() == (long)a.H * a.dk && lower.numel() == bias.numel() && gain.numel() == a.dv &&
+  SHAI_CHECK(a.H >= 1 && a.H <= 65535 && qv.size(1) == (long)a.H * (a.dk + a.dv) && z.size(0) == a.T &&
+                 z.size(1) == (long)a.H * a.dk && bias.numel() == (long)a.H * a.dk && lower.numel() == bias.numel() && gain.numel() == a.dv &&
                  out.size(0) == a.T && out.size(1) == (long)a.H * a.dv && pos.numel() >= a.T && vdim >= 1 && vdim <= a.dv,
              "hgrn2 shapes");
   a.B = a.T;

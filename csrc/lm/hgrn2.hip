@@ -4,7 +4,8 @@
 //
 // rows     row by row, S in registers: decode steps of both formats (bound by the state's traffic) and fp32 prompts.
 // chunks   bf16 prompts, 32 rows at a time on the matrix cores.  With b the running sum of log2 f inside a chunk,
-//            o_t = sum_{s <= t} v_s sum_d q_t k_s 2^(b_t - b_s) + S^T (q_t 2^b_t),   S' = 2^(b_end) S + sum_s (k_s 2^(b_end - b_s)) v_s^T.
+//            o_t = sum_{s <= t} v_s sum_d q_t k_s 2^(b_t - b_s) + S^T (q_t 2^b_t),
+//            S'  = 2^(b_end) S + sum_s (k_s 2^(b_end - b_s)) v_s^T.
 //          Differences of b are never split around a far reference: pairs (s, t) in different 16-row halves meet at the
 //          half's border, those in different 8-row blocks of a half at the block's border (both factors at most 1), and
 //          those inside a block at its fourth row, where the logarithms, limited to -28 a row, keep the factors below

@@ -110,8 +110,8 @@ __device__ __forceinline__ float4_ wide4(uint2_ v) {
                  __uint_as_float(v[1] & 0xffff0000u)};
 }
 
-// The row stays in registers through both norms (RMS norms, or layer norms where there is a bias).  With a convolution a workgroup walks `run` consecutive rows, two of them
-// loaded ahead, and keeps the last taps - 1 inputs in registers; the ones before its first row are recomputed from their
+// The row stays in registers through both norms (RMS norms, or layer norms where there is a bias).  With a convolution a
+// workgroup walks `run` consecutive rows, two of them loaded ahead, and keeps the last taps - 1 inputs in registers; the ones before its first row are recomputed from their
 // residual rows (which is why x_out is not x then) or, before the step's first row of a sequence, come from the sequence's
 // state.  Whatever the rows share (gains, taps, the rows' places) is read before the first row: a load inside the loop
 // would wait for the rows ahead of it.  TD: the type of delta.

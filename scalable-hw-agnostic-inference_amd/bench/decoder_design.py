@@ -1,11 +1,12 @@
-"""Prefill and decode throughput of a layer-list design (Golulix, Faledra) beside a Llama-family model of equal size.
+"""Prefill and decode throughput of a layer-list design (Golulix, Faledra, Nalizen) beside models of equal size.
 
 Both run through :class:`LLMEngine` (scheduler, paged cache, HIP-graph decode) with random weights.  A pair has the same
 width, layers, heads and vocabulary.  The Llama MLP is as wide as the feed-forward work one Golulix token does (top x
 expert + shared expert), or has as many weights as the Faledra feed-forward (3 D I = 2 D ff), so the two do the same
-matrix work per token there.
+matrix work per token there.  Nalizen runs beside Golulix too (both are mixtures of experts): equal routing, and gated
+experts of the same number of weights as its ungated ones.
 
-    python bench.py --workload golulix|faledra [--design-size small|large|both]
+    python bench.py --workload golulix|faledra|nalizen [--design-size small|large|both]
     python -m shai_amd.bench.decoder_design --design faledra --model faledra --size small --batch 64      # profiling
 """
 from __future__ import annotations
@@ -22,12 +23,26 @@ FALEDRA_SIZES = {"small": (2048, 6, 2, 16, 128, 64, 128, 768, 512, 2048, 8448, 3
                  "large": (4096, 4, 2, 32, 128, 64, 128, 1536, 512, 4096, 16896, 65536, 8)}
 
 
+# layers (NalizenConfig.uniform), width, heads, kv heads, head size, window, recurrence heads, their key and value size, dense
+# ff, experts, top, expert ff, token input size, vocab
+NALIZEN_SIZES = {"small": ("aRRSARRS", 2048, 16, 4, 128, 1024, 16, 128, 128, 8448, 64, 6, 2112, 256, 32768),
+                 "large": ("aRSARS", 4096, 32, 8, 128, 4096, 32, 128, 128, 8192, 64, 4, 3072, 256, 65536)}
+
+
 def configs(size: str, design: str = "golulix"):
     from ..models.llama import LlamaConfig
+    out = {}
     if design == "faledra":
         from ..models.faledra import FaledraConfig
         D, A, R, H, d, rot, dv, q, kv, gru, ff, V, G = FALEDRA_SIZES[size]
         cfg, L, inner = FaledraConfig.uniform(A, R, D, H, d, rot, dv, q, kv, gru, ff, V), A + R, 2 * ff // 3
+    elif design == "nalizen":
+        from ..models.golulix import GolulixConfig
+        from ..models.nalizen import NalizenConfig
+        kinds, D, H, G, d, window, _, _, _, ff, E, top, eff, _, V = NALIZEN_SIZES[size]
+        cfg, L, inner = NalizenConfig.uniform(*NALIZEN_SIZES[size]), len(kinds), 2 * top * eff // 3
+        out["golulix"] = GolulixConfig.uniform(layers=L, width=D, heads=H, kv_heads=G, dim=d, chunk=window, experts=E, top=top,
+                                               ff=2 * eff // 3, shared_ff=64, vocab=V)
     else:
         from ..models.golulix import GolulixConfig
         D, L, H, G, d, chunk, E, top, ff, sff, V, groups, keep = SIZES[size]
@@ -36,7 +51,7 @@ def configs(size: str, design: str = "golulix"):
         inner = top * ff + sff
     ll = LlamaConfig(vocab_size=V, hidden_size=D, intermediate_size=inner, num_hidden_layers=L, num_attention_heads=H,
                      num_key_value_heads=G, head_dim=d, max_position_embeddings=32768)
-    return {design: cfg, "llama": ll}
+    return {design: cfg, **out, "llama": ll}
 
 
 def measure(cfg, batch: int, prompt: int, gen: int, repeats: int = 3, device: str = "cuda:0") -> dict:
@@ -93,10 +108,13 @@ def bench(args, rank: int, world: int) -> dict:
                                   f"ff, shared ff, vocab, groups, kept) = {SIZES[n]}",
              "faledra": lambda n: f"Faledra {n}: (width, attention layers, minGRU layers, heads, unrotated / rotated / value "
                                   f"head size, query latent, key-value latent, minGRU width, ff, vocab) = "
-                                  f"{FALEDRA_SIZES[n][:-1]}"}[design](last["size"])
+                                  f"{FALEDRA_SIZES[n][:-1]}",
+             "nalizen": lambda n: f"Nalizen {n}: (layers, width, heads, kv heads, head size, window, recurrence heads, key and "
+                                  f"value size, dense ff, experts, top, expert ff, token input, vocab) = "
+                                  f"{NALIZEN_SIZES[n]}"}[design](last["size"])
     return {"metric": f"{design.capitalize()} decode tokens/s (random weights, beside a Llama model of equal size)",
             "value": last[design]["decode_tok_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": 1,
-            "ms_per_step": round(1000 * (time.perf_counter() - t0) / (len(rows) * 2 * (steps + 1)), 2),
+            "ms_per_step": round(1000 * (time.perf_counter() - t0) / (sum(len(configs(r['size'], design)) for r in rows) * (steps + 1)), 2),
             "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16",
             "data": "synthetic prompts, random-init weights",
             "config": {"model": model, "global_batch": last["batch"], "seq_len": P + G, "parallelism": "dp1"},
@@ -105,8 +123,8 @@ def bench(args, rank: int, world: int) -> dict:
 
 def main(argv=None):
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=["golulix", "faledra"], default="golulix")
-    ap.add_argument("--model", choices=["design", "golulix", "faledra", "llama"], default="design")
+    ap.add_argument("--design", choices=["golulix", "faledra", "nalizen"], default="golulix")
+    ap.add_argument("--model", choices=["design", "golulix", "faledra", "nalizen", "llama"], default="design")
     ap.add_argument("--size", choices=sorted(SIZES), default="small")
     ap.add_argument("--batch", type=int, default=64)
     ap.add_argument("--prompt", type=int, default=1024)

@@ -4,8 +4,8 @@ What a layer-list decoder needs beyond the Llama path of :mod:`shai_amd.ops`: an
 (RMS or layer norm) with the residual kept in fp32 (optionally a norm on the added output and a short causal convolution
 on the sum or its norm), one GEMM for dense, per-head and expert-grouped products, mixture-of-experts routing, attention
 restricted to fixed-size chunks of the sequence or a sliding window with an output gate, attention over cached latents
-with a sink per head, a gated linear recurrence, and linear attention with a gated matrix state.  Every op takes bf16 or fp32 weights and activations; norms, routing, attention scores,
-rotation angles, recurrent state and the residual are fp32 in both.
+with a sink per head, a gated linear recurrence, and linear attention with a gated matrix state.  Every op takes bf16 or fp32 weights and activations; norms,
+routing, attention scores, rotation angles, recurrent state and the residual are fp32 in both.
 
 Layout rules shared by all of them: the model width is padded to a multiple of 64 (``pad64``; the pad columns of
 activations and weights are zero), so a GEMM's K is always a multiple of 64.
@@ -283,9 +283,10 @@ def _gain_bias(w):
 
 @dataclass
 class Conv:
-    """Causal convolution over time on each channel of a norm's output (or of the plain residual), added to it: weight [taps, D] (fp32, oldest tap
-    first), state [slots, taps - 1, D] (fp32: the last inputs of every sequence).  ``tail`` [B, taps - 1, D] receives a
-    prefill step's last inputs (:func:`conv_commit` moves them into the state); None: a decode step, state updated here."""
+    """Causal convolution over time on each channel of a norm's output (or of the plain residual), added to it: weight
+    [taps, D] (fp32, oldest tap first), state [slots, taps - 1, D] (fp32: the last inputs of every sequence).  ``tail``
+    [B, taps - 1, D] receives a prefill step's last inputs (:func:`conv_commit` moves them into the state); None: a decode
+    step, state updated here."""
     weight: torch.Tensor
     state: torch.Tensor
     tail: Optional[torch.Tensor] = None
@@ -297,7 +298,8 @@ def residual_norm(source, delta, wb, mult: float, step, w, eps: float, width: in
 
     source: the fp32 residual [T, D] or an :class:`Embedding`.  delta: [T, D], partial sums [parts, T, D] fp32, or
     :class:`Experts` without a dense part.  wb, w: the norms' gains (RMS norm) or :class:`Affine` (layer norm); w PLAIN:
-    h = x.  Returns (x, h); the residual may be updated in place.  ``w`` None: no h.  ``rows`` (int32): h of these rows only, and with ``keep`` False x is None."""
+    h = x.  Returns (x, h); the residual may be updated in place.  ``w`` None: no h.  ``rows`` (int32): h of these rows
+    only, and with ``keep`` False x is None."""
     emb = isinstance(source, Embedding)
     if not (source.ids if emb else source).is_cuda:
         return ref.residual_norm(source, delta, wb, mult, step, w, eps, width, dtype, conv, batch, rows, keep)

@@ -39,6 +39,8 @@ def check_matmul(device, dtype):
         ref, ad, wd = a.double() @ w.double().T, a.to(device), w.to(device)
         close(lm.matmul(ad, wd, epi=lm.EPI_GELU_GLU), R.gelu_tanh(ref[:, 0::2]) * ref[:, 1::2], 3 * tol, "gelu glu")
         close(lm.matmul(ad, wd, epi=lm.EPI_RELU2), torch.relu(ref) ** 2, 5 * tol, "relu2")
+        if n % 8:
+            continue
         table = torch.randn(23, 3 * n, generator=g).to(dtype)
         ids = torch.randint(0, 23, (m,), generator=g).int()
         y = lm.matmul(ad, wd, epi=lm.EPI_GELU_ROWS, ids=ids.to(device), table=table.to(device)[:, n:2 * n])
@@ -115,7 +117,7 @@ def check_norms(device, dtype):
 def check_token_shift(device, dtype):
     """The shifted residual over portions of every size, in batches, with reused state slots: what comes before a portion is
     the state's, before a sequence's start it is zero whatever the slot holds."""
-    tol = 3e-5 if dtype == torch.float32 else 0.06
+    tol = 3e-5 if dtype == torch.float32 else 0.1
     for width, lengths in ((50, (70, 3, 21, 1)), (130, (9, 4)), (2050, (11, 6)), (5000, (7, 2)), (9000, (5, 3))):
         g = torch.Generator().manual_seed(width)
         r = lambda *s: torch.randn(*s, generator=g)
@@ -174,8 +176,8 @@ def check_feed_forward(device, dtype):
         hp = pad(h).to(device, dtype)
         m = fill(MoE(D, MoEConfig(E, top, ReLU2Config(ff), bias=True, renorm=True), dtype), lambda n: w["l0.mlp." + n], device)
         gain, bias = w["l0.norm2"], w["l0.norm2.b"]
-        x, _ = lm.residual_norm(torch.zeros(T, lm.pad64(D), device=device), m(hp), lm.Affine(pad(gain).to(device), pad(bias).to(device)),
-                                1.0, None, None, 1e-4, D, dtype)
+        zero, affine = torch.zeros(T, lm.pad64(D), device=device), lm.Affine(pad(gain).to(device), pad(bias).to(device))
+        x, _ = lm.residual_norm(zero.clone(), m(hp), affine, 1.0, None, None, 1e-4, D, dtype)
         want = R.layer_norm(R.moe_ff(h.double(), top, lambda n: w["l0.mlp." + n].double()), gain.double(), bias.double(), 1e-4)
         err = (x[:, :D].cpu().double() - want).abs().amax(-1) / want.std()
         assert err.quantile(0.95) < tol, (T, err.max())             # (a near tie may choose another expert)
@@ -186,8 +188,8 @@ def check_feed_forward(device, dtype):
         m = fill(TokenSide(D, sd, dtype), lambda n: w["l1.side." + n], device)
         ids = torch.arange(T).int() % cfg["vocab"]
         e = w["side.embed"][ids.long(), sd:]
-        y, _ = lm.residual_norm(torch.zeros(T, lm.pad64(D), device=device), m(hp, torch.arange(T).int().to(device), pad(e).to(device, dtype)),
-                                m.norm, 1.0, None, None, 1e-4, D, dtype)
+        y = m(hp, torch.arange(T).int().to(device), pad(e).to(device, dtype))
+        y, _ = lm.residual_norm(zero, y, m.norm, 1.0, None, None, 1e-4, D, dtype)
         want = R.side_input(h.double(), e.double(), 1e-4, *(w["l1.side." + n].double() for n in ("gate", "proj", "norm")))
         close(y[:, :D] / want.std(), want / want.std(), tol, "side")
 
@@ -231,7 +233,8 @@ def check_attention(device, dtype):
         for cuts, splits in (((200,), 1), ((1,), 3), ((70, 1, 16, 17, 2), 1), ((64, 1, 1, 0), 2)):
             if cuts == (1,) and i > 3:
                 continue
-            cache = [torch.full(s, JUNK, dtype=dtype, device=device) for s in blocks[0][2].cache_shapes(Stepper(lengths, "cpu").blocks, 64)]
+            shapes = blocks[0][2].cache_shapes(Stepper(lengths, "cpu").blocks, 64)
+            cache = [torch.full(s, JUNK, dtype=dtype, device=device) for s in shapes]
 
             def fn(batch, rows):
                 h = pad(torch.stack([hs[b][p] for b, p in rows])).to(device, dtype)
@@ -336,8 +339,9 @@ def check_state(device, dtype):
             q = q.double()
             o = R.hgrn2_rows(q * torch.sigmoid(q), z.double() + bias.double(), lower.double(), v.double())
             want.append((R.rms(o, 1e-5) * gain.double()))
-        zero = R.hgrn2_rows(qs[0].double(), zs[0].double() + bias.double(), lower.double(), vs[0].double() * (torch.arange(lengths[0]) > 0)[:, None, None])
-        assert lengths[0] < 60 or not torch.allclose(R.rms(zero, 1e-5)[-1] * gain, want[0][-1], atol=0.05)
+        q, later = qs[0].double(), vs[0].double() * (torch.arange(lengths[0]) > 0)[:, None, None]
+        without = R.hgrn2_rows(q * torch.sigmoid(q), zs[0].double() + bias.double(), lower.double(), later)
+        assert not torch.allclose(R.rms(without, 1e-5)[-1] * gain, want[0][-1], atol=0.05)
         hp = lambda t, m: pad(t, m).reshape(len(t), -1)
         qv = [torch.cat([hp(q, dk), hp(v, dv)], 1).to(device) for q, v in zip(qs, vs)]
         zp = [hp(z, dk).to(device) for z in zs]
@@ -379,7 +383,8 @@ MECHANISMS = [check_matmul, check_rope, check_norms, check_token_shift, check_ro
 # ---------------------------------------------------------------------------------------------- whole models
 SHAPES = {
     "base": {},
-    "attention_only": dict(layers=[A(heads=1, kv_heads=1, dim=64, vdim=64, dims=64), A(heads=5, kv_heads=1, mlp=R.experts(3, 3, 70))]),
+    "attention_only": dict(layers=[A(heads=1, kv_heads=1, dim=64, vdim=64, dims=64),
+                                   A(heads=5, kv_heads=1, mlp=R.experts(3, 3, 70))]),
     "hgrn2_only": dict(layers=[G(), G(1, 64, 64, R.dense(64)), G(5, 9, 100)], width=64, side=64),
     "one_layer": dict(layers=[A(window=1, mlp=R.experts(1, 1, 30))], side=1),
     "no_mlp": dict(layers=[A(mlp=None), G(mlp=None), A(kv_from=0, mlp=None), G()], width=100, vocab=33),

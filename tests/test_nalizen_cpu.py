@@ -137,3 +137,13 @@ def test_serving_api_with_nalizen():
     with TestClient(create_app(env=env)) as client:
         r = client.post("/generate", json={"prompt": "hello there", "max_new_tokens": 4})
         assert r.status_code == 200 and r.json()["text"]
+
+
+def test_bench_option_measures_every_model(monkeypatch):
+    from shai_amd.bench import decoder_design as dd
+    monkeypatch.setitem(dd.NALIZEN_SIZES, "small", ("aRS", 64, 2, 1, 32, 40, 2, 32, 32, 96, 4, 2, 48, 16, 128))
+    cfgs = dd.configs("small", "nalizen")
+    assert list(cfgs) == ["nalizen", "golulix", "llama"]
+    for cfg in cfgs.values():
+        r = dd.measure(cfg, 2, 40, 3, repeats=1, device="cpu")
+        assert r["prefill_tok_s"] > 0 and r["decode_tok_s"] > 0
