@@ -3,8 +3,8 @@
 Both run through :class:`LLMEngine` (scheduler, paged cache, HIP-graph decode) with random weights.  A pair has the same
 width, layers, heads and vocabulary.  The Llama MLP is as wide as the feed-forward work one Golulix token does (top x
 expert + shared expert), or has as many weights as the Faledra feed-forward (3 D I = 2 D ff), so the two do the same
-matrix work per token there.  Nalizen runs beside Golulix too (both are mixtures of experts): equal routing, and gated
-experts of the same number of weights as its ungated ones.
+matrix work per token there.  Nalizen runs beside Golulix too (both are mixtures of experts): equal routing, gated experts
+of the same number of weights as its ungated ones, and a chunk that holds the whole sequence.
 
     python bench.py --workload golulix|faledra|nalizen [--design-size small|large|both]
     python -m shai_amd.bench.decoder_design --design faledra --model faledra --size small --batch 64      # profiling
@@ -41,8 +41,8 @@ def configs(size: str, design: str = "golulix"):
         from ..models.nalizen import NalizenConfig
         kinds, D, H, G, d, window, _, _, _, ff, E, top, eff, _, V = NALIZEN_SIZES[size]
         cfg, L, inner = NalizenConfig.uniform(*NALIZEN_SIZES[size]), len(kinds), 2 * top * eff // 3
-        out["golulix"] = GolulixConfig.uniform(layers=L, width=D, heads=H, kv_heads=G, dim=d, chunk=window, experts=E, top=top,
-                                               ff=2 * eff // 3, shared_ff=64, vocab=V)
+        out["golulix"] = GolulixConfig.uniform(layers=L, width=D, heads=H, kv_heads=G, dim=d, chunk=2 * window, experts=E,
+                                               top=top, ff=2 * eff // 3, shared_ff=64, vocab=V)
     else:
         from ..models.golulix import GolulixConfig
         D, L, H, G, d, chunk, E, top, ff, sff, V, groups, keep = SIZES[size]
