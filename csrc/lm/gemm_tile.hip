@@ -1,6 +1,5 @@
 // C = epi(A W^T), LDS-tiled bf16 form for many rows (prefill): 64 x 64 or 128 x 128 tiles of 4 waves or 256 x 256 tiles of
-// 8, 64-wide
-// k-tiles moved global -> LDS by DMA (buffer_load ... lds, 16 bytes per lane) into two stages; the load of k-tile t + 1 is
+// 8, 64-wide k-tiles moved global -> LDS by DMA (buffer_load ... lds, 16 bytes per lane) into two stages; the load of k-tile t + 1 is
 // issued before the MFMAs of t.  The bank swizzle is applied to the per-lane source chunk.  Buffer range checks zero-fill
 // rows past the ends.  Dense or grouped by expert: the row tiles of a grouped product come from the tile list, each with
 // its own W and with A rows gathered per lane.  Tiles are walked XCD by XCD in groups of 8 row tiles that share their W
@@ -172,10 +171,12 @@ static void tile(const GemmArgs& a, hipStream_t s) {
 }
 
 void launch_gemm_tile(const GemmArgs& a, hipStream_t s) {
-  // 256 x 256 tiles (8 waves) once they fill the chip, 128 x 128 (4 waves, two workgroups per CU) below, 64 x 64 where
-  // those would leave most of it idle
+  // 256 x 256 tiles (8 waves) once they fill the chip, 128 x 128 (4 waves, two workgroups per CU) below and for narrow
+  // outputs and short K (a second workgroup computes while the first one stores), 64 x 64 where those would leave most of
+  // the chip idle
   const long m128 = (a.M + 127) / 128, n128 = (a.N + 127) / 128;
-  const bool big = a.tiles ? a.bm == 256 : a.splits <= 1 && (long)((a.M + 255) / 256) * ((a.N + 255) / 256) >= 192;
+  const bool fills = a.N > 128 && a.K > 1536 && (long)((a.M + 255) / 256) * ((a.N + 255) / 256) >= 192;
+  const bool big = a.tiles ? a.bm == 256 : a.splits <= 1 && fills;
   if (big) tile<256, 256, 2, 4>(a, s);
   else if (!a.tiles && a.splits <= 1 && m128 * n128 < 256 && a.K <= 2048) tile<64, 64, 2, 2>(a, s);
   else tile<128, 128, 2, 2>(a, s);
