@@ -48,7 +48,7 @@ struct Frag<float> {
   }
 };
 
-template <typename T, typename O, int MT, int NT, int NW, int D>
+template <typename T, typename O, int EC, int MT, int NT, int NW, int D>
 __global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) {
   __shared__ float4_ red[NW][MT][64];
   const int lane = threadIdx.x & 63;
@@ -129,14 +129,14 @@ __global__ void __launch_bounds__(NW * 64) gemm_stream_kernel(const GemmArgs p) 
 #pragma unroll
       for (int w = 1; w < NW; ++w) c += red[w][t][lane];
       const int m = row0 + 16 * t + r;
-      if (m < rows_end) store_cols<O>(p, C, m, n0 + 16 * i + 4 * g, c);
+      if (m < rows_end) store_cols<O, EC>(p, C, m, n0 + 16 * i + 4 * g, c);
     }
   }
 }
 
 // Workgroup shapes (16 MT rows of A x 16 NT rows of W, NW waves along K, D k-steps in flight), from a sweep at decode
 // sizes: enough workgroups to fill the chip come first, then fewer passes over W (MT), then fewer re-reads of A (NT).
-template <typename T, typename O>
+template <typename T, typename O, int EC>
 static void stream(const GemmArgs& a, hipStream_t s) {
   auto go = [&](auto kernel, int mt, int nt, int nw) {
     const dim3 grid((a.N + 16 * nt - 1) / (16 * nt), a.tiles ? a.n_tiles : (a.M + 16 * mt - 1) / (16 * mt),
@@ -144,13 +144,15 @@ static void stream(const GemmArgs& a, hipStream_t s) {
     kernel<<<grid, 64 * nw, 0, s>>>(a);
   };
   constexpr bool H = sizeof(T) == 2;              // fp32 fragments are twice the registers
-#define GO(MT_, NT_, NW_, D_) go(gemm_stream_kernel<T, O, MT_, NT_, NW_, H ? D_ : 1>, MT_, NT_, NW_)
+#define GO(MT_, NT_, NW_, D_) go(gemm_stream_kernel<T, O, EC, MT_, NT_, NW_, H ? D_ : 1>, MT_, NT_, NW_)
   const int rows = a.tiles ? a.bm : a.M;
   if (a.splits > 1) {
-    if (rows <= 16) GO(1, 1, 4, 4);
-    else if (rows <= 32) GO(2, 2, 4, 4);
-    else if (a.N < 2560 && a.K < 12288) GO(4, 2, 4, 3);
-    else GO(4, 4, 4, 2);
+    if constexpr (epi_in(EC, EPI_NONE)) {         // partial sums
+      if (rows <= 16) GO(1, 1, 4, 4);
+      else if (rows <= 32) GO(2, 2, 4, 4);
+      else if (a.N < 2560 && a.K < 12288) GO(4, 2, 4, 3);
+      else GO(4, 4, 4, 2);
+    }
   } else if (!a.tiles && a.K <= 256) {            // too few k-steps to split over many waves
     if (rows <= 16) GO(1, 2, 2, 2);
     else if (rows <= 32) GO(2, 2, 2, 2);
@@ -168,9 +170,14 @@ static void stream(const GemmArgs& a, hipStream_t s) {
 }
 
 void launch_gemm(const GemmArgs& a, bool f32, hipStream_t s) {
-  if (f32) stream<float, float>(a, s);
-  else if (a.out_f32) stream<bf16_t, float>(a, s);
-  else stream<bf16_t, bf16_t>(a, s);
+  const int ec = epi_class(a.epi);
+  if (f32) stream<float, float, EC_ANY>(a, s);
+  else if (a.out_f32 && ec == EC_PLAIN) stream<bf16_t, float, EC_PLAIN>(a, s);
+  else if (a.out_f32) stream<bf16_t, float, EC_ANY>(a, s);
+  else if (ec == EC_PLAIN) stream<bf16_t, bf16_t, EC_PLAIN>(a, s);
+  else if (ec == EC_CLAMP) stream<bf16_t, bf16_t, EC_CLAMP>(a, s);
+  else if (ec == EC_GELU) stream<bf16_t, bf16_t, EC_GELU>(a, s);
+  else stream<bf16_t, bf16_t, EC_OTHER>(a, s);
 }
 
 }  // namespace shai_lm

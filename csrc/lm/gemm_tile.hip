@@ -1,6 +1,6 @@
 // C = epi(A W^T), LDS-tiled bf16 form for many rows (prefill): 64 x 64 or 128 x 128 tiles of 4 waves or 256 x 256 tiles of
-// 8, 64-wide k-tiles moved global -> LDS by DMA (buffer_load ... lds, 16 bytes per lane) into two stages; the load of k-tile t + 1 is
-// issued before the MFMAs of t.  The bank swizzle is applied to the per-lane source chunk.  Buffer range checks zero-fill
+// 8, 64-wide k-tiles moved global -> LDS by DMA (buffer_load ... lds, 16 bytes per lane) into two stages; the load of
+// k-tile t + 1 is issued before the MFMAs of t.  The bank swizzle is applied to the per-lane source chunk.  Buffer range checks zero-fill
 // rows past the ends.  Dense or grouped by expert: the row tiles of a grouped product come from the tile list, each with
 // its own W and with A rows gathered per lane.  Tiles are walked XCD by XCD in groups of 8 row tiles that share their W
 // columns.
@@ -13,7 +13,7 @@ constexpr uint32_t kOob = 0x80000000u;
 
 __device__ __forceinline__ int swz(int row, int ch) { return row * 64 + ((ch ^ ((row >> 1) & 7)) << 3); }
 
-template <typename O, int BM, int BN, int WM, int WN>
+template <typename O, int EC, int BM, int BN, int WM, int WN>
 __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_kernel(const GemmArgs p) {
   constexpr int NW = WM * WN, TM = BM / WM, TN = BN / WN, IM = TM / 32, JN = TN / 32;
   constexpr int JA = BM / 8 / NW, JB = BN / 8 / NW, STAGE = (BM + BN) * 64;
@@ -113,7 +113,7 @@ __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_
     __syncthreads();
   }
   // bf16 results go through LDS, so that rows are stored 16 bytes a lane, whole lines at a time
-  const bool glu = glu_epi(p.epi);
+  const bool glu = glu_class(EC) && glu_epi(p.epi);
   if (sizeof(O) == 2 && p.ldc % 8 == 0 && (glu || p.N % 8 == 0) && (p.n_main == p.N || n0 + BN <= p.n_main)) {
     constexpr int LD = BN + 8;
     __syncthreads();
@@ -127,7 +127,7 @@ __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_
         for (int g = 0; g < 4; ++g) {
           const int n = wn * TN + j * 32 + 8 * g + 4 * fh;
           float4_ c = float4_{acc[i][j][4 * g], acc[i][j][4 * g + 1], acc[i][j][4 * g + 2], acc[i][j][4 * g + 3]};
-          if (live) epilogue_cols<O>(p, m0 + r, n0 + n, c);
+          if (live) epilogue_cols<O, EC>(p, m0 + r, n0 + n, c);
           if (glu) *reinterpret_cast<uint32_t*>(smem + r * LD + (n >> 1)) = pack2(c[0], c[1]);
           else store4(smem + r * LD + n, c);
         }
@@ -151,7 +151,7 @@ __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_
     for (int j = 0; j < JN; ++j)
 #pragma unroll
       for (int g = 0; g < 4; ++g)
-        store_cols<O>(p, C, m, n0 + wn * TN + j * 32 + 8 * g + 4 * fh,
+        store_cols<O, EC>(p, C, m, n0 + wn * TN + j * 32 + 8 * g + 4 * fh,
                       float4_{acc[i][j][4 * g], acc[i][j][4 * g + 1], acc[i][j][4 * g + 2], acc[i][j][4 * g + 3]});
   }
 }
@@ -165,8 +165,13 @@ static void tile(const GemmArgs& a, hipStream_t s) {
     (void)hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, lds);
     k<<<dim3(grid, a.splits > 1 ? a.splits : 1), WM * WN * 64, lds, s>>>(a);
   };
-  if (a.out_f32) go(gemm_tile_kernel<float, BM, BN, WM, WN>);
-  else go(gemm_tile_kernel<bf16_t, BM, BN, WM, WN>);
+  const int ec = epi_class(a.epi);
+  if (a.out_f32 && ec == EC_PLAIN) go(gemm_tile_kernel<float, EC_PLAIN, BM, BN, WM, WN>);
+  else if (a.out_f32) go(gemm_tile_kernel<float, EC_ANY, BM, BN, WM, WN>);
+  else if (ec == EC_PLAIN) go(gemm_tile_kernel<bf16_t, EC_PLAIN, BM, BN, WM, WN>);
+  else if (ec == EC_CLAMP) go(gemm_tile_kernel<bf16_t, EC_CLAMP, BM, BN, WM, WN>);
+  else if (ec == EC_GELU) go(gemm_tile_kernel<bf16_t, EC_GELU, BM, BN, WM, WN>);
+  else go(gemm_tile_kernel<bf16_t, EC_OTHER, BM, BN, WM, WN>);
   SHAI_CHECK_LAUNCH();
 }
 

@@ -99,6 +99,14 @@ void launch_rope_rows(const RopeRowsArgs& a, hipStream_t s);
 enum Epi : int { EPI_NONE = 0, EPI_CLAMP_GLU = 1, EPI_SOFTCAP = 2, EPI_XIELU = 3, EPI_ROTARY = 4, EPI_GELU_GLU = 5,
                  EPI_RELU2 = 6, EPI_GELU_ROWS = 7 };
 constexpr __host__ __device__ bool glu_epi(int epi) { return epi == EPI_CLAMP_GLU || epi == EPI_GELU_GLU; }
+// The bf16 kernels are compiled per class of epilogues: code of the others costs a kernel registers and instruction cache.
+enum EpiClass : int { EC_PLAIN = 0, EC_CLAMP = 1, EC_GELU = 2, EC_OTHER = 3, EC_ANY = 4 };
+constexpr __host__ __device__ int epi_class(int epi) {
+  return epi == EPI_NONE || epi == EPI_RELU2 ? EC_PLAIN : epi == EPI_CLAMP_GLU ? EC_CLAMP
+         : epi == EPI_GELU_GLU || epi == EPI_GELU_ROWS ? EC_GELU : EC_OTHER;
+}
+constexpr __host__ __device__ bool epi_in(int ec, int epi) { return ec == EC_ANY || ec == epi_class(epi); }
+constexpr __host__ __device__ bool glu_class(int ec) { return ec == EC_ANY || ec == EC_CLAMP || ec == EC_GELU; }
 struct GemmArgs {
   const void* A;           // [rows, K]
   const void* W;           // [N, K] or [E, N, K]

@@ -73,40 +73,43 @@ __device__ __forceinline__ float xielu(float z, float ap, float an, bool fast) {
   return (z > 0.f ? ap * z * z : an * e) + 0.5f * z;
 }
 
-// the tanh form of gelu: z / (1 + exp(-2 u)) = z (1 + tanh u) / 2
-__device__ __forceinline__ float gelu_tanh(float z) {
+// the tanh form of gelu: z / (1 + exp(-2 u)) = z (1 + tanh u) / 2.  `fast`: the hardware exponential and reciprocal.
+__device__ __forceinline__ float gelu_tanh(float z, bool fast) {
   const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
+  if (fast) return z * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-2.f * 1.4426950408889634f * u));
   return z / (1.f + expf(-2.f * u));
 }
 
 // Epilogue of 4 consecutive columns n .. n + 3 of row m, in place (a GLU's two results: c[0], c[1]).
-template <typename O>
+template <typename O, int EC>
 __device__ __forceinline__ void epilogue_cols(const GemmArgs& p, long m, int n, float4_& c) {
-  if (p.epi == EPI_CLAMP_GLU) {
+  constexpr bool fast = sizeof(O) == 2;
+  const auto is = [&](int epi) { return epi_in(EC, epi) && p.epi == epi; };
+  if (is(EPI_CLAMP_GLU)) {
     c[0] = clamp_glu(c[0], c[1], p.param);
     c[1] = clamp_glu(c[2], c[3], p.param);
-  } else if (p.epi == EPI_SOFTCAP) {
+  } else if (is(EPI_SOFTCAP)) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) c[i] = p.param * tanhf(c[i] / p.param);
-  } else if (p.epi == EPI_XIELU) {
+  } else if (is(EPI_XIELU)) {
     const float ap = p.vec[0], an = p.vec[1];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) c[i] = xielu(c[i], ap, an, sizeof(O) == 2);
-  } else if (p.epi == EPI_GELU_GLU) {
-    c[0] = gelu_tanh(c[0]) * c[1];
-    c[1] = gelu_tanh(c[2]) * c[3];
-  } else if (p.epi == EPI_RELU2) {
+    for (int i = 0; i < 4; ++i) c[i] = xielu(c[i], ap, an, fast);
+  } else if (is(EPI_GELU_GLU)) {
+    c[0] = gelu_tanh(c[0], fast) * c[1];
+    c[1] = gelu_tanh(c[2], fast) * c[3];
+  } else if (is(EPI_RELU2)) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) c[i] = c[i] > 0.f ? c[i] * c[i] : 0.f;
-  } else if (p.epi == EPI_GELU_ROWS) {
+  } else if (is(EPI_GELU_ROWS)) {
     if (n < p.N) {
       const long at = (long)min(max(p.ids[m], 0), p.table_rows - 1) * p.table_ld + n;
       const float4_ e = p.table_f32 ? load4(static_cast<const float*>(p.table) + at)
                                     : load4(static_cast<const bf16_t*>(p.table) + at);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) c[i] = gelu_tanh(c[i]) * e[i];
+      for (int i = 0; i < 4; ++i) c[i] = gelu_tanh(c[i], fast) * e[i];
     }
-  } else if (p.epi == EPI_ROTARY) {
+  } else if (is(EPI_ROTARY)) {
     const int d = n % p.head - p.rot0;
     if (d >= 0 && d < p.rot && n < p.N) {
       const float* t = p.rope + m * p.rot + d;
@@ -123,7 +126,7 @@ __device__ __forceinline__ void epilogue_cols(const GemmArgs& p, long m, int n, 
 }
 
 // Store 4 consecutive columns n .. n + 3 of row m after the epilogue.  `out`: C of this product.
-template <typename O>
+template <typename O, int EC>
 __device__ __forceinline__ void store_cols(const GemmArgs& p, O* out, long m, int n, float4_ c) {
   if (n >= p.n_main) {
     const int ld = p.N - p.n_main, j = n - p.n_main;
@@ -137,8 +140,8 @@ __device__ __forceinline__ void store_cols(const GemmArgs& p, O* out, long m, in
       if (n + i < p.N) o[i] = c[i];
     return;
   }
-  epilogue_cols<O>(p, m, n, c);
-  if (glu_epi(p.epi)) {
+  epilogue_cols<O, EC>(p, m, n, c);
+  if (glu_class(EC) && glu_epi(p.epi)) {
     const int j = n >> 1;
     if (n < p.N) store1(out + m * p.ldc + j, c[0]);
     if (n + 2 < p.N) store1(out + m * p.ldc + j + 1, c[1]);
