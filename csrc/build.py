@@ -53,7 +53,7 @@ BINDING_SRCS = ["bindings.cpp"]
 # the decoder-block kernels and the token-level ops of every language model's step (their own library: a model that
 # runs on them alone needs nothing else compiled)
 LM_SRCS = ["lm/norm.hip", "lm/gemm.hip", "lm/gemm_tile.hip", "lm/moe.hip", "lm/attn.hip", "lm/latent.hip", "lm/scan.hip",
-           "lm/hgrn2.hip", "kernels/sampling.hip"]
+           "lm/hgrn2.hip", "lm/rule.hip", "kernels/sampling.hip"]
 LM_BINDING_SRCS = ["lm/bindings.cpp"]
 RUNTIME_SRCS = ["runtime/block_manager.cpp", "runtime/scheduler.cpp"]
 COMM_SRCS = ["comm/p2p_allreduce.hip"]

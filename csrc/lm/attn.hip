@@ -3,10 +3,13 @@
 //
 // Position i sees the keys lo .. i with lo = i - i % chunk or, with a window, i - chunk + 1; scores are (q . k) * scale,
 // softmaxed in fp32, and the output is multiplied by sigmoid of a gate logit per head or per element.  The rows of a step
-// are [q | k | v | gate] (one GEMM), or [q | gate] where another layer has written the cache.
+// are [q | k | v | gate] (one GEMM), or [q | gate] where another layer has written the cache.  Without a gate they are
+// [q | k], the values are the keys before their norm and rotation, a head's scores have a factor of their own and its
+// denominator a sink.
 //
 // kv_store      the step's k / v rows into the cache.
-// head_prep     the same with q and k rotated by position and divided by their root mean square (q in place).
+// head_prep     the same with q and k rotated by position and divided by their root mean square, or normed with a gain and
+//               then rotated (q in place).
 // prefill       bf16: flash attention, 4 waves x 32 queries, scores swapped (S^T = K Q^T) so that a lane holds one
 //               query's scores; P feeds O^T = V^T P^T from registers as a bf16 pair (value + remainder, 16 significant
 //               bits).  Only the 64-key blocks of the chunks that the workgroup's queries lie in are visited.
@@ -35,14 +38,14 @@ __global__ void __launch_bounds__(256) kv_store_kernel(const AttnArgs p) {
   const long t = blockIdx.x;
   const int slot = p.slots[t];
   if (slot < 0) return;
-  const T* row = static_cast<const T*>(p.qkvg) + t * p.ld + (long)p.H * p.dk;
+  const T* row = static_cast<const T*>(p.qkvg) + t * p.ld;
   const int blk = slot >> 6, in = slot & 63;
   const int nk = p.G * p.dk / V, nv = p.G * p.dv / V;
   for (int i = threadIdx.x; i < nk + nv; i += 256) {
     const bool isv = i >= nk;
     const int e = (isv ? i - nk : i) * V, d = isv ? p.dv : p.dk, g = e / d;
     T* dst = static_cast<T*>(isv ? p.vc : p.kc) + (((long)blk * p.G + g) * 64 + in) * d + (e - g * d);
-    *reinterpret_cast<uint4_*>(dst) = *reinterpret_cast<const uint4_*>(row + (isv ? (long)p.G * p.dk : 0L) + e);
+    *reinterpret_cast<uint4_*>(dst) = *reinterpret_cast<const uint4_*>(row + (isv ? p.v_off : p.H * p.dk) + e);
   }
 }
 
@@ -65,11 +68,20 @@ __device__ __forceinline__ void store8(float* p, const float* x) {
 }
 
 // One head by n / 8 lanes of a wave, lane j holding elements 8 j .. 8 j + 7: dimension i < rot / 2 turned with i + rot / 2 by
-// the row's angles, then the head divided by its root mean square over `dim` (the pads behind are zero).  `stage`: n
-// floats of LDS.  Every lane of the wave calls it.
+// the row's angles, then the head divided by its root mean square over `dim` (the pads behind are zero); with `gain` the norm
+// comes first.  `stage`: n floats of LDS.  Every lane of the wave calls it.
 __device__ __forceinline__ void turn_and_norm(float (&x)[8], float* stage, const float* rope, int rot, int dim, float eps,
-                                              int j, int lanes) {
+                                              int j, int lanes, const float* gain) {
   const int half = rot >> 1;
+  if (gain) {
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
+    for (int o = lanes >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+    const float r = 1.f / sqrtf(ss / (float)dim + eps);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) x[i] *= r * gain[8 * j + i];
+  }
   store8(stage + 8 * j, x);
   __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
   float ss = 0.f;
@@ -85,6 +97,7 @@ __device__ __forceinline__ void turn_and_norm(float (&x)[8], float* stage, const
     ss += x[i] * x[i];
   }
   __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  if (gain) return;
   for (int o = lanes >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
   const float r = 1.f / sqrtf(ss / (float)dim + eps);
 #pragma unroll
@@ -106,12 +119,12 @@ __global__ void __launch_bounds__(256) head_prep_kernel(const AttnArgs p) {
     const int h = h0 + tid / LPH;
     float x[8];
     load8(row + (long)min(h, n - 1) * DK + 8 * j, x);
-    turn_and_norm(x, stage[tid / LPH], angle, p.rot, p.dim, p.eps, j, LPH);
+    turn_and_norm(x, stage[tid / LPH], angle, p.rot, p.dim, p.eps, j, LPH, h < p.H ? p.q_gain : p.k_gain);
     if (h < p.H) store8(row + (long)h * DK + 8 * j, x);
     else if (h < n) store8(static_cast<T*>(p.kc) + (((long)blk * p.G + h - p.H) * 64 + in) * DK + 8 * j, x);
   }
   if (n == p.H) return;
-  const T* v = row + (long)(p.H + p.G) * DK;
+  const T* v = row + p.v_off;
   for (int i = tid; i < p.G * p.dv / 8; i += 256) {
     const int e = 8 * i, g = e / p.dv;
     float x[8];
@@ -154,6 +167,7 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(const AttnArgs p) {
   const T* row = static_cast<const T*>(p.qkvg) + t * p.ld;
   for (int d = lane; d < p.dk; d += 64) sq[w][d] = load1(row + (long)h * p.dk + d);
   __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  const float scale = p.scale * (p.temp ? p.temp[h] : 1.f);
   float o[4] = {0.f, 0.f, 0.f, 0.f}, m = -INFINITY, l = 0.f;
   for (int kb = lo >> 6; kb <= pos >> 6; ++kb) {
     const long cell = ((long)p.bt[(long)b * p.max_blocks + kb] * p.G + g) * 64;
@@ -166,7 +180,7 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(const AttnArgs p) {
         const float4_ k4 = load4(kr + d), q4 = load4(&sq[w][d]);
         acc += k4[0] * q4[0] + k4[1] * q4[1] + k4[2] * q4[2] + k4[3] * q4[3];
       }
-      s = acc * p.scale;
+      s = acc * scale;
     }
     const float mn = fmaxf(m, wave_max(s));      // finite: the first block holds lo, every later one a visible key
     const float alpha = expf(m - mn), e = expf(s - mn);
@@ -187,12 +201,18 @@ __global__ void __launch_bounds__(256) attn_rows_kernel(const AttnArgs p) {
     }
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
   }
+  float up = p.out_scale;
+  if (p.sink) {
+    const float sk = p.sink[h], top = fmaxf(m, sk), a = expf(m - top);
+    l = l * a + expf(sk - top);
+    up *= a;
+  }
   const T* gate = row + p.gate_off + (long)h * p.gate_w;
-  T* out = static_cast<T*>(p.o) + t * (long)p.H * p.dv + (long)h * p.dv;
+  T* out = static_cast<T*>(p.o) + t * p.ldo + (long)h * p.dv;
 #pragma unroll
   for (int c = 0; c < 4; ++c) {
     const int col = lane + 64 * c;
-    if (col < p.dv) store1(out + col, o[c] * (sigmoid_f(load1(gate + (p.gate_w > 1 ? col : 0))) / l));
+    if (col < p.dv) store1(out + col, o[c] * ((p.gate_w ? sigmoid_f(load1(gate + (p.gate_w > 1 ? col : 0))) : up) / l));
   }
 }
 
@@ -300,7 +320,7 @@ __global__ void __launch_bounds__(256, DK + DV > (LAT ? 320 : 256) ? 1 : 2) attn
 #pragma unroll
     for (int r = 0; r < 16; ++r) o[d][r] = 0.f;
   float m_run = -INFINITY, l_run = 0.f;
-  const float sl2 = p.scale * kLog2e;
+  const float sl2 = p.scale * kLog2e * (!LAT && p.temp ? p.temp[h] : 1.f);
   const int g16 = lane >> 4, i16 = lane & 15, tq = i16 >> 2, tp = i16 & 3;
 
   if constexpr (LAT) {
@@ -414,13 +434,13 @@ __global__ void __launch_bounds__(256, DK + DV > (LAT ? 320 : 256) ? 1 : 2) attn
   const float l_tot = l_run + __shfl_xor(l_run, 32, 64);
   if (qi < q_len) {
     float inv;
-    if constexpr (LAT) {
+    if (LAT || p.sink) {
       const float sk = p.sink[h] * kLog2e, top = fmaxf(m_run, sk), a = __builtin_amdgcn_exp2f(m_run - top);
-      inv = a / (l_tot * a + __builtin_amdgcn_exp2f(sk - top));
+      inv = (LAT ? a : a * p.out_scale) / (l_tot * a + __builtin_amdgcn_exp2f(sk - top));
     } else {
-      inv = (p.gate_w > 1 ? 1.f : sigmoid_f(bf2f(rows[(long)qi * p.ld + p.gate_off + h]))) / l_tot;
+      inv = (p.gate_w > 1 ? 1.f : p.gate_w ? sigmoid_f(bf2f(rows[(long)qi * p.ld + p.gate_off + h])) : p.out_scale) / l_tot;
     }
-    bf16_t* op = static_cast<bf16_t*>(p.o) + (row0 + qi) * (long)p.H * DV + (long)h * DV;
+    bf16_t* op = static_cast<bf16_t*>(p.o) + (row0 + qi) * p.ldo + (long)h * DV;
 #pragma unroll
     for (int d = 0; d < ND; ++d)
 #pragma unroll
@@ -472,6 +492,17 @@ void launch_attn_prefill(const AttnArgs& a, bool f32, hipStream_t s) {
 }
 
 // ------------------------------------------------------------------------------------------------ decode (bf16)
+// what a head's summed output is multiplied by: the denominator L (of exponents to the base 2 above M) with its sink, the gate
+__device__ __forceinline__ float out_factor(const AttnArgs& p, const bf16_t* row, int h, int d, float M, float L) {
+  float up = p.gate_w ? sigmoid_f(bf2f(row[p.gate_off + (long)h * p.gate_w + (p.gate_w > 1 ? d : 0)])) : p.out_scale;
+  if (p.sink) {
+    const float sk = p.sink[h] * kLog2e, top = fmaxf(M, sk), a = __builtin_amdgcn_exp2f(M - top);
+    L = L * a + __builtin_amdgcn_exp2f(sk - top);
+    up *= a;
+  }
+  return up / L;
+}
+
 // One workgroup: kv head g's query heads h0 .. h0 + R - 1 (R <= 16, RH = R rounded up) of sequence b, one split of the
 // visible 64-key blocks.  Wave w takes blocks w, w + 4, ... of the split.
 template <int DK, int DV, int RH, bool PREP>
@@ -502,7 +533,7 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(const AttnArgs p, int 
   if (store && slot >= 0 && s1 == b1 && s0 < s1) {
     const long cell = ((long)(slot >> 6) * p.G + g) * 64 + (slot & 63);
     const bf16_t* kn = row + (long)p.H * DK + (long)g * DK;
-    const bf16_t* vn = row + (long)p.H * DK + (long)p.G * DK + (long)g * DV;
+    const bf16_t* vn = row + p.v_off + (long)g * DV;
     if (tid < DK / 8) {
       if constexpr (!PREP) reinterpret_cast<uint4_*>(kc + cell * DK)[tid] = reinterpret_cast<const uint4_*>(kn)[tid];
     } else if (tid >= 64 && tid - 64 < DV / 8)
@@ -517,7 +548,8 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(const AttnArgs p, int 
       float x[8];
       load8(row + (long)(ii < R ? h0 + ii : p.H + g) * DK + 8 * j, x);
       // the spare lanes repeat the last head with the same values
-      turn_and_norm(x, &so[0][0][0] + ii * DK, p.rope + (long)b * p.rot, p.rot, p.dim, p.eps, j, LPH);
+      turn_and_norm(x, &so[0][0][0] + ii * DK, p.rope + (long)b * p.rot, p.rot, p.dim, p.eps, j, LPH,
+                    ii < R ? p.q_gain : p.k_gain);
       if (i < R) store8(&sq[i][8 * j], x);
       else if (i < n) store8(kc + (((long)(slot >> 6) * p.G + g) * 64 + (slot & 63)) * DK + 8 * j, x);
     }
@@ -538,7 +570,7 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(const AttnArgs p, int 
 #pragma unroll
     for (int j = 0; j < 8; ++j) o[r][j] = 0.f;
   float m = -INFINITY, l = 0.f;                  // of head c (replicated over q4)
-  const float sl2 = p.scale * kLog2e;
+  const float sl2 = p.scale * kLog2e * (p.temp ? p.temp[h0 + min(c, R - 1)] : 1.f);
   const int vk = lane / LPK, vcol = (lane % LPK) * 8;
 
   for (int kb = s0 + w; kb < s1; kb += 4) {
@@ -643,8 +675,7 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(const AttnArgs p, int 
       }
     }
     if (p.splits == 1) {
-      const float gate = bf2f(row[p.gate_off + (long)h * p.gate_w + (p.gate_w > 1 ? d : 0)]);
-      static_cast<bf16_t*>(p.o)[((long)b * p.H + h) * DV + d] = f2bf(x / L * sigmoid_f(gate));
+      static_cast<bf16_t*>(p.o)[(long)b * p.ldo + h * DV + d] = f2bf(x * out_factor(p, row, h, d, M, L));
     } else {
       float* ws = p.ws + (((long)b * p.H + h) * p.splits + split) * (DV + 2);
       ws[d] = x;
@@ -658,7 +689,7 @@ __global__ void __launch_bounds__(256) attn_decode_kernel(const AttnArgs p, int 
 
 __global__ void __launch_bounds__(256) attn_decode_fold_kernel(const AttnArgs p) {
   __shared__ float se[64];
-  __shared__ float total;
+  __shared__ float total, top;
   const int h = blockIdx.x, b = blockIdx.y, d = threadIdx.x;
   const float* ws = p.ws + ((long)b * p.H + h) * p.splits * (p.dv + 2);
   if (d < 64) {                                  // one lane per split (at most 64)
@@ -668,17 +699,18 @@ __global__ void __launch_bounds__(256) attn_decode_fold_kernel(const AttnArgs p)
     const float e = d < p.splits ? __builtin_amdgcn_exp2f(m - M) : 0.f;
     se[d] = e;
     const float L = wave_sum(l * e);
-    if (d == 0) total = L;
+    if (d == 0) {
+      total = L;
+      top = M;
+    }
   }
   __syncthreads();
   if (d >= p.dv) return;
   float x = 0.f;
 #pragma unroll 8
   for (int s = 0; s < p.splits; ++s) x += ws[(long)s * (p.dv + 2) + d] * se[s];
-  const float L = total;
-  const float gate = bf2f(static_cast<const bf16_t*>(p.qkvg)[(long)b * p.ld + p.gate_off + (long)h * p.gate_w +
-                                                             (p.gate_w > 1 ? d : 0)]);
-  static_cast<bf16_t*>(p.o)[((long)b * p.H + h) * p.dv + d] = f2bf(x / L * sigmoid_f(gate));
+  static_cast<bf16_t*>(p.o)[(long)b * p.ldo + h * p.dv + d] =
+      f2bf(x * out_factor(p, static_cast<const bf16_t*>(p.qkvg) + (long)b * p.ld, h, d, top, total));
 }
 
 template <int DK, int DV, bool PREP>

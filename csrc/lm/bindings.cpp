@@ -33,6 +33,17 @@ bool is_f32(const Tensor& t) {
   SHAI_CHECK(t.scalar_type() == at::kFloat || t.scalar_type() == at::kBFloat16, "bf16 or fp32, got ", t.scalar_type());
   return t.scalar_type() == at::kFloat;
 }
+// a matrix of contiguous rows that may lie apart
+void check_rows(const Tensor& t, at::ScalarType dt, const char* name) {
+  SHAI_CHECK(t.is_cuda() && t.dim() == 2 && t.scalar_type() == dt && (t.size(1) <= 1 || t.stride(1) == 1) &&
+                 (t.size(0) <= 1 || t.stride(0) >= t.size(1)), name, " must be a GPU ", dt, " matrix of contiguous rows");
+}
+// the same, read or written 16 bytes at a time
+void check_rows16(const Tensor& t, at::ScalarType dt, const char* name) {
+  check_rows(t, dt, name);
+  SHAI_CHECK(t.stride(0) * t.element_size() % 16 == 0 && reinterpret_cast<uintptr_t>(t.data_ptr()) % 16 == 0, name,
+             " rows must be 16-byte aligned");
+}
 void check_width(int64_t Dp, int64_t width) {
   SHAI_CHECK(Dp % 64 == 0 && Dp <= 16384 && width >= 1 && width <= Dp, "width ", width, " in rows of ", Dp,
              ": rows must be a multiple of 64 and at most 16384");
@@ -134,12 +145,13 @@ void add_norm(const Tensor& x, const optional<Tensor>& dense, const optional<Ten
 void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<Tensor>& tiles,
              const optional<Tensor>& offsets, const optional<Tensor>& gather, int64_t bm, int64_t epi, double param,
              const optional<Tensor>& side, const optional<Tensor>& vec, const optional<Tensor>& rope, int64_t head,
-             int64_t rot0, const optional<Tensor>& ids, const optional<Tensor>& table) {
+             int64_t rot0, const optional<Tensor>& ids, const optional<Tensor>& table, int64_t act) {
   const bool f32 = is_f32(A);
   SHAI_CHECK(A.is_cuda() && A.dim() == 2 && A.stride(1) == 1 && A.stride(0) % 8 == 0 && A.stride(0) >= A.size(1) &&
                  reinterpret_cast<uintptr_t>(A.data_ptr()) % 16 == 0, "A rows must be contiguous and 16-byte aligned");
   check(W, A.scalar_type(), "W");
-  check(C, f32 || C.scalar_type() == at::kFloat ? at::kFloat : at::kBFloat16, "C");
+  SHAI_CHECK(C.scalar_type() == at::kFloat || (!f32 && C.scalar_type() == at::kBFloat16), "C: fp32, or bf16 as A");
+  check_rows(C, C.scalar_type(), "C");
   shai_lm::GemmArgs g{};
   SHAI_CHECK(A.dim() == 2 && C.dim() == 2 && (W.dim() == 2 || W.dim() == 3), "lm_gemm ranks");
   g.a_rows = A.size(0);
@@ -157,16 +169,19 @@ void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<T
   g.batch = 1;
   if (side) {  // the last rows of W are a plain product, stored in fp32
     check(*side, at::kFloat, "side");
-    SHAI_CHECK(!tiles && (glu || epi == shai_lm::EPI_NONE) && side->dim() == 2 &&
+    SHAI_CHECK(!tiles && (glu || epi == shai_lm::EPI_NONE || epi == shai_lm::EPI_RELU2) && side->dim() == 2 &&
                    side->size(0) == g.M && side->size(1) >= 1 && side->size(1) < g.N,
-               "side output: dense plain or GLU products, [M, last rows of W]");
+               "side output: dense plain, squared ReLU or GLU products, [M, last rows of W]");
     g.n_main = g.N - side->size(1);
     SHAI_CHECK(g.n_main % 4 == 0, "side output: the other rows of W must be a multiple of 4");
     g.side = side->data_ptr<float>();
   }
   SHAI_CHECK(!glu || g.n_main % 2 == 0, "GLU products need (gate, up) row pairs");
-  g.ldc = glu ? g.n_main / 2 : g.n_main;
-  SHAI_CHECK(C.size(1) == g.ldc, "lm_gemm output columns");
+  SHAI_CHECK(reinterpret_cast<uintptr_t>(C.data_ptr()) % 16 == 0, "C must be 16-byte aligned");
+  SHAI_CHECK(C.size(1) == (glu ? g.n_main / 2 : g.n_main), "lm_gemm output columns");
+  g.ldc = g.M > 1 ? C.stride(0) : std::max<int64_t>(C.stride(0), C.size(1));
+  g.n_act = act > 0 ? act : g.n_main;
+  SHAI_CHECK(act == 0 || (epi == shai_lm::EPI_RELU2 && act % 4 == 0 && act <= g.n_main), "act: leading columns, a multiple of 4");
   if (epi == shai_lm::EPI_XIELU) {
     SHAI_CHECK(vec.has_value() && vec->numel() == 2, "the xIELU epilogue needs its two coefficients");
     check_f32(*vec, "vec");
@@ -252,7 +267,7 @@ void lm_gemm_heads(const Tensor& A, const Tensor& W, const Tensor& C) {
   g.M = g.a_rows = A.size(0);
   g.batch = A.size(1);
   g.K = A.size(2);
-  g.N = g.n_main = W.size(1);
+  g.N = g.n_main = g.n_act = W.size(1);
   SHAI_CHECK(W.size(0) == g.batch && W.size(2) == g.K && W.stride(1) == g.K && g.K % 64 == 0 && g.N % 4 == 0 &&
                  C.size(0) == g.M && C.size(1) == g.batch && C.size(2) == g.N && g.batch <= 65535, "lm_gemm_heads shapes");
   g.A = A.data_ptr();
@@ -270,14 +285,15 @@ void lm_gemm_heads(const Tensor& A, const Tensor& W, const Tensor& C) {
 // partial sums of a w^T over equal parts of K: c [splits, M, N] fp32
 void lm_gemm_parts(const Tensor& A, const Tensor& W, const Tensor& C) {
   const bool f32 = is_f32(A);
-  check(A, A.scalar_type(), "A");
+  check_rows16(A, A.scalar_type(), "A");
   check(W, A.scalar_type(), "W");
   check(C, at::kFloat, "C");
   shai_lm::GemmArgs g{};
   SHAI_CHECK(A.dim() == 2 && W.dim() == 2 && C.dim() == 3, "lm_gemm_parts ranks");
   g.M = g.a_rows = A.size(0);
-  g.N = g.n_main = g.ldc = W.size(0);
-  g.K = g.lda = A.size(1);
+  g.N = g.n_main = g.n_act = g.ldc = W.size(0);
+  g.K = A.size(1);
+  g.lda = A.stride(0);
   g.splits = C.size(0);
   g.batch = 1;
   g.out_f32 = true;
@@ -288,7 +304,7 @@ void lm_gemm_parts(const Tensor& A, const Tensor& W, const Tensor& C) {
   g.C = C.data_ptr();
   if (g.M == 0) return;
   const long lim = 0x7fffffffL;
-  const bool tile = !f32 && g.M > 64 && (long)g.M * g.K * 2 < lim && (long)g.N * g.K * 2 < lim;
+  const bool tile = !f32 && g.M > 64 && (long)g.M * g.lda * 2 < lim && (long)g.N * g.K * 2 < lim;
   if (tile) shai_lm::launch_gemm_tile(g, stream());
   else shai_lm::launch_gemm(g, f32, stream());
 }
@@ -337,8 +353,8 @@ void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const
   if (delta) {
     const bool many = delta->dim() == 3;
     check(*delta, many ? at::kFloat : dt, "delta");
-    SHAI_CHECK((many || delta->dim() == 2) && delta->size(-2) == R && delta->size(-1) == a.Dp && wb.has_value(),
-               "delta must be [rows, D] or [parts, rows, D], with its norm's gain");
+    SHAI_CHECK((many || delta->dim() == 2) && delta->size(-2) == R && delta->size(-1) == a.Dp && (wb.has_value() || !bb),
+               "delta must be [rows, D] or [parts, rows, D]; a norm's bias comes with its gain");
     a.delta = delta->data_ptr();
     a.parts = many ? delta->size(0) : 0;
     a.part_stride = R * a.Dp;
@@ -382,6 +398,7 @@ void residual_norm(const optional<Tensor>& x, const optional<Tensor>& ids, const
   }
   if (cw) {
     check(*cw, at::kFloat, "cw");
+    SHAI_CHECK(!(delta || ye) || wb, "convolution: a delta has a norm");
     SHAI_CHECK(cw->dim() == 2 && cw->size(1) == a.Dp && cw->size(0) >= 1 && cw->size(0) <= 16, "convolution: 1 to 16 taps");
     a.taps = cw->size(0);
     SHAI_CHECK(h.has_value() && x_out.has_value() && (!x || x->data_ptr() != x_out->data_ptr()),
@@ -520,6 +537,7 @@ void latent_attn_prefill(const Tensor& q, const Tensor& kv, const Tensor& lat, c
                  o.size(1) % heads == 0 && q.size(0) == o.size(0), "latent prefill: q [T, H dk], o [T, H dv]");
   a.T = q.size(0);
   a.ld = q.size(1);
+  a.ldo = o.size(1);
   a.dk = q.size(1) / heads;
   a.dv = o.size(1) / heads;
   SHAI_CHECK((a.dk == 64 && a.dv == 64) || (a.dk == 128 && (a.dv == 64 || a.dv == 128)) || (a.dk == 192 && a.dv == 128) ||
@@ -705,6 +723,149 @@ void hgrn2(const Tensor& qv, const Tensor& z, const Tensor& bias, const Tensor& 
   else shai_lm::launch_hgrn2_chunks(a, stream());
 }
 
+// Delta rule (conv, beta, ring given) or retention (rope given): sizes checked, everything but the workspace filled in
+shai_lm::RuleArgs rule_args(const Tensor& x, const Tensor& gate, const Tensor& state, const Tensor& out, const Tensor& pos,
+                            const Tensor& slots, int64_t kv_heads, int64_t dim, int64_t vdim, int64_t gate_kind, double eps,
+                            const Tensor& rate, const optional<Tensor>& decay, const optional<Tensor>& beta,
+                            const optional<Tensor>& conv, const optional<Tensor>& bias, const optional<Tensor>& gain,
+                            const optional<Tensor>& ring, const optional<Tensor>& rope, const optional<Tensor>& q_start,
+                            const optional<Tensor>& q_lens) {
+  const auto dt = x.scalar_type();
+  is_f32(x);
+  check_rows16(x, dt, "x");
+  check_rows(gate, dt, "gate");
+  check_rows(out, dt, "out");
+  check(state, at::kFloat, "state");
+  check(rate, at::kFloat, "rate");
+  check_i32(pos, "pos");
+  check_i32(slots, "slots");
+  shai_lm::RuleArgs a{};
+  SHAI_CHECK(state.dim() == 4, "state must be [slots, H, dk, dv]");
+  a.T = x.size(0);
+  a.H = state.size(1);
+  a.dk = state.size(2);
+  a.dv = state.size(3);
+  a.G = kv_heads;
+  SHAI_CHECK((a.dk == 64 && a.dv == 64) || (a.dk == 64 && a.dv == 128) || (a.dk == 128 && a.dv == 64) ||
+                 (a.dk == 128 && a.dv == 128) || (a.dk == 256 && a.dv == 256), "stored head sizes: 64 / 128 each, or 256 / 256");
+  const long channels = 2L * a.G * a.dk + (long)a.H * a.dv;
+  SHAI_CHECK(a.H >= 1 && a.H <= 65535 && a.G >= 1 && a.H % a.G == 0 && x.size(1) == channels && gate.size(0) == a.T &&
+                 gate.size(1) == (long)a.H * a.dv && out.size(0) == a.T && out.size(1) == gate.size(1) && pos.numel() >= a.T &&
+                 dim >= 1 && dim <= a.dk && vdim >= 1 && vdim <= a.dv && (gate_kind == 0 || gate_kind == 1), "rule shapes");
+  a.dim = dim;
+  a.vdim = vdim;
+  a.gate_kind = gate_kind;
+  a.eps = eps;
+  a.x = x.data_ptr();
+  a.gate = gate.data_ptr();
+  a.state = state.data_ptr<float>();
+  a.out = out.data_ptr();
+  a.rate = rate.data_ptr<float>();
+  a.pos = pos.data_ptr<int>();
+  a.slots = slots.data_ptr<int>();
+  a.ldx = x.stride(0);
+  a.ldg = gate.stride(0);
+  a.ldo = out.stride(0);
+  a.taps = 1;
+  if (conv) {
+    SHAI_CHECK(decay.has_value() && beta.has_value() && bias.has_value() && gain.has_value() && ring.has_value(),
+               "delta rule: decay, beta, bias, gain and ring");
+    check(*conv, at::kFloat, "conv");
+    check_rows(*decay, at::kFloat, "decay");
+    check_rows(*beta, at::kFloat, "beta");
+    check(*bias, at::kFloat, "bias");
+    check(*gain, at::kFloat, "gain");
+    check(*ring, dt, "ring");
+    a.taps = conv->size(0);
+    a.mode = decay->size(1) == a.H && bias->numel() == a.H ? 1 : 2;
+    SHAI_CHECK(conv->dim() == 2 && a.taps >= 1 && a.taps <= 16 && conv->size(1) == channels && ring->dim() == 3 &&
+                   ring->size(0) == state.size(0) && ring->size(1) == a.taps && ring->size(2) == channels && rate.numel() == a.H &&
+                   gain->numel() == a.dv && beta->size(0) == a.T && beta->size(1) == a.H && decay->size(0) == a.T &&
+                   (a.mode == 1 || decay->size(1) == (long)a.H * a.dk) && bias->numel() == decay->size(1), "delta rule shapes");
+    a.conv = conv->data_ptr<float>();
+    a.decay = decay->data_ptr<float>();
+    a.beta = beta->data_ptr<float>();
+    a.bias = bias->data_ptr<float>();
+    a.gain = gain->data_ptr<float>();
+    a.ring = ring->data_ptr();
+    a.ldd = decay->stride(0);
+    a.ldb = beta->stride(0);
+  } else {
+    SHAI_CHECK(rope.has_value(), "retention: rope");
+    check(*rope, at::kFloat, "rope");
+    SHAI_CHECK(a.G == a.H && rope->dim() == 2 && rope->size(0) >= a.T && rope->size(1) % 2 == 0 && rope->size(1) <= dim &&
+                   rate.numel() == 2L * a.H, "retention shapes");
+    a.rope = rope->data_ptr<float>();
+    a.rot = rope->size(1);
+  }
+  a.B = a.T;
+  if (q_lens) {
+    SHAI_CHECK(q_start.has_value(), "prefill: q_start");
+    check_i32(*q_lens, "q_lens");
+    check_i32(*q_start, "q_start");
+    a.B = q_lens->numel();
+    SHAI_CHECK(q_start->numel() == a.B, "one start per sequence");
+    a.q_lens = q_lens->data_ptr<int>();
+    a.q_start = q_start->data_ptr<int>();
+  }
+  SHAI_CHECK(slots.numel() >= a.B && a.B <= 65535, "one state slot per sequence");
+  return a;
+}
+
+void rule_rows(const Tensor& x, const Tensor& gate, const Tensor& state, const Tensor& out, const Tensor& pos,
+               const Tensor& slots, int64_t kv_heads, int64_t dim, int64_t vdim, int64_t gate_kind, double eps,
+               const Tensor& rate, const optional<Tensor>& decay, const optional<Tensor>& beta, const optional<Tensor>& conv,
+               const optional<Tensor>& bias, const optional<Tensor>& gain, const optional<Tensor>& ring,
+               const optional<Tensor>& rope, const optional<Tensor>& q_start, const optional<Tensor>& q_lens) {
+  const shai_lm::RuleArgs a = rule_args(x, gate, state, out, pos, slots, kv_heads, dim, vdim, gate_kind, eps, rate, decay,
+                                        beta, conv, bias, gain, ring, rope, q_start, q_lens);
+  if (a.T > 0) shai_lm::launch_rule_rows(a, is_f32(x), stream());
+}
+
+// q_start / q_lens describe the packed rows of x (their sum is T); max_q: the largest of q_lens
+void rule_chunks(const Tensor& x, const Tensor& gate, const Tensor& state, const Tensor& out, const Tensor& pos,
+                 const Tensor& slots, int64_t kv_heads, int64_t dim, int64_t vdim, int64_t gate_kind, double eps,
+                 const Tensor& rate, const optional<Tensor>& decay, const optional<Tensor>& beta, const optional<Tensor>& conv,
+                 const optional<Tensor>& bias, const optional<Tensor>& gain, const optional<Tensor>& ring,
+                 const optional<Tensor>& rope, const Tensor& q_start, const Tensor& q_lens, const Tensor& ws, int64_t max_q,
+                 int64_t head0, int64_t heads) {
+  shai_lm::RuleArgs a = rule_args(x, gate, state, out, pos, slots, kv_heads, dim, vdim, gate_kind, eps, rate, decay, beta,
+                                  conv, bias, gain, ring, rope, q_start, q_lens);
+  SHAI_CHECK(x.scalar_type() == at::kBFloat16, "chunks: bf16 rows");
+  check(ws, at::kByte, "ws");
+  SHAI_CHECK(head0 >= 0 && heads >= 1 && head0 + heads <= a.H && max_q >= 1 && (max_q + 31) / 32 <= 0x7fffffff &&
+                 ws.numel() >= ((long)a.T / 32 + a.B) * heads * shai_lm::rule_chunk_bytes(a.dk, a.dv), "rule_chunks workspace");
+  a.ws = ws.data_ptr();
+  a.head0 = head0;
+  a.heads = heads;
+  a.max_q = std::min<int64_t>(max_q, a.T);
+  if (a.T > 0) shai_lm::launch_rule_chunks(a, stream());
+}
+
+int64_t rule_chunk_bytes(int64_t dk, int64_t dv) { return shai_lm::rule_chunk_bytes(dk, dv); }
+
+void ring_commit(const Tensor& x, const Tensor& ring, const Tensor& pos, const Tensor& q_start, const Tensor& q_lens,
+                 const Tensor& slots) {
+  check_rows(x, ring.scalar_type(), "x");
+  check(ring, ring.scalar_type(), "ring");
+  for (auto* t : {&pos, &q_start, &q_lens, &slots}) check_i32(*t, "ring_commit tensor");
+  shai_lm::RingArgs a{};
+  SHAI_CHECK(ring.dim() == 3 && x.size(1) == ring.size(2), "ring must be [slots, taps, columns of x]");
+  a.B = q_lens.numel();
+  a.n_slots = ring.size(0);
+  a.taps = ring.size(1);
+  a.channels = ring.size(2);
+  a.ldx = x.stride(0);
+  SHAI_CHECK(a.taps >= 1 && q_start.numel() == a.B && slots.numel() >= a.B && pos.numel() >= x.size(0) && a.B <= 65535, "ring_commit shapes");
+  a.x = x.data_ptr();
+  a.ring = ring.data_ptr();
+  a.pos = pos.data_ptr<int>();
+  a.q_start = q_start.data_ptr<int>();
+  a.q_lens = q_lens.data_ptr<int>();
+  a.slots = slots.data_ptr<int>();
+  if (a.B > 0) shai_lm::launch_ring_commit(a, is_f32(ring), stream());
+}
+
 const float* route_bias(const optional<Tensor>& bias, int E) {
   if (!bias) return nullptr;
   check(*bias, at::kFloat, "bias");
@@ -799,17 +960,17 @@ void moe_plan(const Tensor& ids, int64_t bm, const Tensor& offsets, const Tensor
 
 // gate_w: gate logits per head (1 or dv).  own_kv false: rows are [q | gate], the cache holds another layer's keys and values
 shai_lm::AttnArgs attn_args(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor* o, int64_t heads,
-                            bool per_element = false, bool own_kv = true) {
+                            bool per_element = false, bool own_kv = true, bool tied = false) {
   const auto dt = qkvg.scalar_type();
   is_f32(qkvg);
-  check(qkvg, dt, "qkvg");
+  check_rows16(qkvg, dt, "qkvg");
   check(kc, dt, "k_cache");
   check(vc, dt, "v_cache");
-  SHAI_CHECK(qkvg.dim() == 2 && kc.dim() == 4 && vc.dim() == 4 && kc.size(0) == vc.size(0) && kc.size(1) == vc.size(1) &&
+  SHAI_CHECK(kc.dim() == 4 && vc.dim() == 4 && kc.size(0) == vc.size(0) && kc.size(1) == vc.size(1) &&
                  kc.size(2) == 64 && vc.size(2) == 64, "caches must be [blocks, G, 64, dk | dv]");
   shai_lm::AttnArgs a{};
   a.T = qkvg.size(0);
-  a.ld = qkvg.size(1);
+  a.ld = qkvg.stride(0);
   a.H = heads;
   a.G = kc.size(1);
   a.dk = kc.size(3);
@@ -818,23 +979,41 @@ shai_lm::AttnArgs attn_args(const Tensor& qkvg, const Tensor& kc, const Tensor& 
              "stored head sizes: 64 / 128 each, or 256 / 256");
   SHAI_CHECK(a.H >= 1 && a.G >= 1 && a.H % a.G == 0, "query heads must be a multiple of kv heads");
   a.own_kv = own_kv;
-  a.gate_w = per_element ? a.dv : 1;
-  a.gate_off = a.H * a.dk + (own_kv ? a.G * (a.dk + a.dv) : 0);
-  SHAI_CHECK(a.ld % 8 == 0 && a.ld >= (long)a.gate_off + (long)a.H * a.gate_w, "qkvg row too short");
+  a.out_scale = 1.f;
+  if (tied) {  // [q | k]: the values are the keys, no gate
+    SHAI_CHECK(own_kv && !per_element && a.dk == a.dv, "keys as values: one head size");
+    a.v_off = a.H * a.dk;
+    SHAI_CHECK(qkvg.size(1) >= (long)(a.H + a.G) * a.dk, "qk row too short");
+  } else {
+    a.v_off = (a.H + a.G) * a.dk;
+    a.gate_w = per_element ? a.dv : 1;
+    a.gate_off = a.H * a.dk + (own_kv ? a.G * (a.dk + a.dv) : 0);
+    SHAI_CHECK(qkvg.size(1) % 8 == 0 && qkvg.size(1) >= (long)a.gate_off + (long)a.H * a.gate_w, "qkvg row too short");
+  }
   a.qkvg = qkvg.data_ptr();
   a.kc = kc.data_ptr();
   a.vc = vc.data_ptr();
   if (o) {
-    check(*o, dt, "o");
-    SHAI_CHECK(o->dim() == 2 && o->size(0) == a.T && o->size(1) == (long)a.H * a.dv, "o must be [T, H dv]");
+    check_rows16(*o, dt, "o");
+    SHAI_CHECK(o->size(0) == a.T && o->size(1) == (long)a.H * a.dv, "o must be [T, H dv]");
     a.o = o->data_ptr();
+    a.ldo = o->stride(0);
   }
   return a;
 }
 
 // rotation and norm of q and k: angles of every row, the head size before padding
-void set_turn(shai_lm::AttnArgs& a, const optional<Tensor>& rope, int64_t dim, double eps) {
+void set_turn(shai_lm::AttnArgs& a, const optional<Tensor>& rope, int64_t dim, double eps, const optional<Tensor>& q_gain,
+              const optional<Tensor>& k_gain) {
   if (!rope) return;
+  SHAI_CHECK(q_gain.has_value() == k_gain.has_value(), "gains of both queries and keys, or none");
+  if (q_gain) {
+    check(*q_gain, at::kFloat, "q_gain");
+    check(*k_gain, at::kFloat, "k_gain");
+    SHAI_CHECK(q_gain->numel() == a.dk && k_gain->numel() == a.dk, "gains must be [dk]");
+    a.q_gain = q_gain->data_ptr<float>();
+    a.k_gain = k_gain->data_ptr<float>();
+  }
   check(*rope, at::kFloat, "rope");
   SHAI_CHECK(rope->dim() == 2 && rope->size(0) >= a.T && rope->size(1) % 2 == 0 && dim >= 1 && dim <= a.dk &&
                  rope->size(1) <= dim, "rope must be [T, rotated dimensions of a head]");
@@ -844,19 +1023,31 @@ void set_turn(shai_lm::AttnArgs& a, const optional<Tensor>& rope, int64_t dim, d
   a.eps = eps;
 }
 
+// attention without gates: factors on the scores, sinks, factor on the output
+void set_ungated(shai_lm::AttnArgs& a, const optional<Tensor>& temp, const optional<Tensor>& sink, double out_scale) {
+  if (!sink) return;
+  SHAI_CHECK(temp.has_value(), "attention without gates: temp and sink");
+  check_f32(*temp, "temp");
+  check_f32(*sink, "sink");
+  SHAI_CHECK(temp->numel() == a.H && sink->numel() == a.H, "temp and sink must be [H]");
+  a.temp = temp->data_ptr<float>();
+  a.sink = sink->data_ptr<float>();
+  a.out_scale = out_scale;
+}
+
 // q of the step in place and, with own keys, k and v into the cache
 void head_prep(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor& slots, int64_t heads, const Tensor& rope,
-               int64_t dim, double eps, bool own_kv) {
-  shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, nullptr, heads, false, own_kv);
-  set_turn(a, rope, dim, eps);
+               int64_t dim, double eps, bool own_kv, bool tied, const optional<Tensor>& q_gain, const optional<Tensor>& k_gain) {
+  shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, nullptr, heads, false, own_kv, tied);
+  set_turn(a, rope, dim, eps, q_gain, k_gain);
   check_i32(slots, "slots");
   SHAI_CHECK(slots.numel() >= a.T, "one slot per row");
   a.slots = slots.data_ptr<int>();
   if (a.T > 0) shai_lm::launch_head_prep(a, is_f32(qkvg), stream());
 }
 
-void kv_store(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor& slots, int64_t heads) {
-  shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, nullptr, heads);
+void kv_store(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor& slots, int64_t heads, bool tied) {
+  shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, nullptr, heads, false, true, tied);
   check_i32(slots, "slots");
   SHAI_CHECK(slots.numel() >= a.T, "one slot per row");
   a.slots = slots.data_ptr<int>();
@@ -866,8 +1057,10 @@ void kv_store(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tens
 // `chunk`: the size of the chunks or, with `window`, of the sliding window
 void gated_attn_prefill(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor& o, const Tensor& bt,
                         const Tensor& ctx, const Tensor& q_lens, const Tensor& q_start, int64_t max_q, int64_t heads,
-                        int64_t chunk, double scale, bool window, bool per_element, bool own_kv) {
-  shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, &o, heads, per_element, own_kv);
+                        int64_t chunk, double scale, bool window, bool per_element, bool own_kv, const optional<Tensor>& temp,
+                        const optional<Tensor>& sink, double out_scale) {
+  shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, &o, heads, per_element, own_kv, sink.has_value());
+  set_ungated(a, temp, sink, out_scale);
   for (auto* t : {&bt, &ctx, &q_lens, &q_start}) check_i32(*t, "batch tensor");
   a.B = bt.size(0);
   a.max_blocks = bt.size(1);
@@ -887,9 +1080,12 @@ void gated_attn_prefill(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, 
 void gated_attn_decode(const Tensor& qkvg, const Tensor& kc, const Tensor& vc, const Tensor& o, const Tensor& bt,
                        const Tensor& ctx, const Tensor& slots, const Tensor& ws, int64_t heads, int64_t splits,
                        int64_t chunk, double scale, bool window, bool per_element, bool own_kv,
-                       const optional<Tensor>& rope, int64_t dim, double eps) {
-  shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, &o, heads, per_element, own_kv);
-  set_turn(a, rope, dim, eps);
+                       const optional<Tensor>& rope, int64_t dim, double eps, const optional<Tensor>& q_gain,
+                       const optional<Tensor>& k_gain, const optional<Tensor>& temp, const optional<Tensor>& sink,
+                       double out_scale) {
+  shai_lm::AttnArgs a = attn_args(qkvg, kc, vc, &o, heads, per_element, own_kv, sink.has_value());
+  set_turn(a, rope, dim, eps, q_gain, k_gain);
+  set_ungated(a, temp, sink, out_scale);
   for (auto* t : {&bt, &ctx, &slots}) check_i32(*t, "batch tensor");
   a.B = bt.size(0);
   a.max_blocks = bt.size(1);
@@ -942,7 +1138,7 @@ void token_feedback(const Tensor& ids, const Tensor& rowmap, const Tensor& prev)
 TORCH_LIBRARY_FRAGMENT(shai, m) {
   m.def("embed_norm(Tensor ids, Tensor? prev, Tensor table, Tensor? bigram, int mul_prev, int mul_cur, Tensor w, float eps, int width, Tensor(a!) x, Tensor(b!) h) -> ()");
   m.def("add_norm(Tensor(a!) x, Tensor? dense, Tensor? ye, Tensor? slot_of, Tensor? wts, Tensor? inject, Tensor? rows, Tensor? w, float eps, int width, Tensor(b!)? h) -> ()");
-  m.def("lm_gemm(Tensor a, Tensor w, Tensor(a!) c, Tensor? tiles, Tensor? offsets, Tensor? gather, int bm, int epi, float param, Tensor(b!)? side=None, Tensor? vec=None, Tensor? rope=None, int head=0, int rot0=0, Tensor? ids=None, Tensor? table=None) -> ()");
+  m.def("lm_gemm(Tensor a, Tensor w, Tensor(a!) c, Tensor? tiles, Tensor? offsets, Tensor? gather, int bm, int epi, float param, Tensor(b!)? side=None, Tensor? vec=None, Tensor? rope=None, int head=0, int rot0=0, Tensor? ids=None, Tensor? table=None, int act=0) -> ()");
   m.def("lm_gemm_heads(Tensor a, Tensor w, Tensor(a!) c) -> ()");
   m.def("lm_gemm_parts(Tensor a, Tensor w, Tensor(a!) c) -> ()");
   m.def("residual_norm(Tensor? x, Tensor? ids, Tensor? table, float scale, Tensor? delta, Tensor? wb, float mult, Tensor? step, Tensor(a!)? x_out, Tensor? rows, Tensor? w, float eps, int width, Tensor(b!)? h, Tensor? cw=None, Tensor(c!)? state=None, Tensor(d!)? tail=None, Tensor? row_seq=None, Tensor? q_start=None, Tensor? q_lens=None, Tensor? pos=None, Tensor? slots=None, Tensor? bb=None, Tensor? b=None, Tensor? ye=None, Tensor? slot_of=None, Tensor? wts=None) -> ()");
@@ -956,11 +1152,15 @@ TORCH_LIBRARY_FRAGMENT(shai, m) {
   m.def("moe_route(Tensor logits, int groups, int keep, Tensor(a!) ids, Tensor(b!) wts, Tensor? bias=None, bool renorm=False) -> ()");
   m.def("moe_route_plan(Tensor logits, int groups, int keep, Tensor(a!) ids, Tensor(b!) wts, Tensor(c!) offsets, Tensor(d!) token_of, Tensor(e!) slot_of, Tensor(f!) tiles, Tensor? bias=None, bool renorm=False) -> ()");
   m.def("moe_plan(Tensor ids, int bm, Tensor(a!) offsets, Tensor(b!) token_of, Tensor(c!) slot_of, Tensor(d!) tiles) -> ()");
-  m.def("kv_store(Tensor qkvg, Tensor(a!) k_cache, Tensor(b!) v_cache, Tensor slots, int heads) -> ()");
-  m.def("head_prep(Tensor(a!) qkvg, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slots, int heads, Tensor rope, int dim, float eps, bool own_kv) -> ()");
+  m.def("kv_store(Tensor qkvg, Tensor(a!) k_cache, Tensor(b!) v_cache, Tensor slots, int heads, bool tied=False) -> ()");
+  m.def("head_prep(Tensor(a!) qkvg, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slots, int heads, Tensor rope, int dim, float eps, bool own_kv, bool tied=False, Tensor? q_gain=None, Tensor? k_gain=None) -> ()");
   m.def("hgrn2(Tensor qv, Tensor z, Tensor bias, Tensor lower, Tensor gain, Tensor(a!) state, Tensor(b!) out, Tensor pos, Tensor? q_start, Tensor? q_lens, Tensor slots, Tensor(c!) ws, int max_q, int len, int vdim, float eps) -> ()");
-  m.def("gated_attn_prefill(Tensor qkvg, Tensor k_cache, Tensor v_cache, Tensor(a!) o, Tensor block_table, Tensor ctx_lens, Tensor q_lens, Tensor q_start, int max_q, int heads, int chunk, float scale, bool window=False, bool per_element=False, bool own_kv=True) -> ()");
-  m.def("gated_attn_decode(Tensor qkvg, Tensor(a!) k_cache, Tensor(b!) v_cache, Tensor(c!) o, Tensor block_table, Tensor ctx_lens, Tensor slots, Tensor(d!) ws, int heads, int splits, int chunk, float scale, bool window=False, bool per_element=False, bool own_kv=True, Tensor? rope=None, int dim=0, float eps=0.) -> ()");
+  m.def("rule_rows(Tensor x, Tensor gate, Tensor(a!) state, Tensor(b!) out, Tensor pos, Tensor slots, int kv_heads, int dim, int vdim, int gate_kind, float eps, Tensor rate, Tensor? decay=None, Tensor? beta=None, Tensor? conv=None, Tensor? bias=None, Tensor? gain=None, Tensor(c!)? ring=None, Tensor? rope=None, Tensor? q_start=None, Tensor? q_lens=None) -> ()");
+  m.def("rule_chunks(Tensor x, Tensor gate, Tensor(a!) state, Tensor(b!) out, Tensor pos, Tensor slots, int kv_heads, int dim, int vdim, int gate_kind, float eps, Tensor rate, Tensor? decay=None, Tensor? beta=None, Tensor? conv=None, Tensor? bias=None, Tensor? gain=None, Tensor? ring=None, Tensor? rope=None, *, Tensor q_start, Tensor q_lens, Tensor(c!) ws, int max_q, int head0, int heads) -> ()");
+  m.def("rule_chunk_bytes(int dk, int dv) -> int", &rule_chunk_bytes);
+  m.def("ring_commit(Tensor x, Tensor(a!) ring, Tensor pos, Tensor q_start, Tensor q_lens, Tensor slots) -> ()");
+  m.def("gated_attn_prefill(Tensor qkvg, Tensor k_cache, Tensor v_cache, Tensor(a!) o, Tensor block_table, Tensor ctx_lens, Tensor q_lens, Tensor q_start, int max_q, int heads, int chunk, float scale, bool window=False, bool per_element=False, bool own_kv=True, Tensor? temp=None, Tensor? sink=None, float out_scale=1.) -> ()");
+  m.def("gated_attn_decode(Tensor qkvg, Tensor(a!) k_cache, Tensor(b!) v_cache, Tensor(c!) o, Tensor block_table, Tensor ctx_lens, Tensor slots, Tensor(d!) ws, int heads, int splits, int chunk, float scale, bool window=False, bool per_element=False, bool own_kv=True, Tensor? rope=None, int dim=0, float eps=0., Tensor? q_gain=None, Tensor? k_gain=None, Tensor? temp=None, Tensor? sink=None, float out_scale=1.) -> ()");
   m.def("sample(Tensor logits, Tensor temps, Tensor top_k, Tensor top_p, Tensor uniforms, Tensor(a!) out) -> ()");
   m.def("token_feedback(Tensor(a!) ids, Tensor rowmap, Tensor prev) -> ()");
 }
@@ -985,6 +1185,9 @@ TORCH_LIBRARY_IMPL(shai, CUDA, m) {
   m.impl("kv_store", &kv_store);
   m.impl("head_prep", &head_prep);
   m.impl("hgrn2", &hgrn2);
+  m.impl("rule_rows", &rule_rows);
+  m.impl("rule_chunks", &rule_chunks);
+  m.impl("ring_commit", &ring_commit);
   m.impl("gated_attn_prefill", &gated_attn_prefill);
   m.impl("gated_attn_decode", &gated_attn_decode);
   m.impl("sample", &sample);

@@ -114,7 +114,7 @@ __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_
   }
   // bf16 results go through LDS, so that rows are stored 16 bytes a lane, whole lines at a time
   const bool glu = glu_class(EC) && glu_epi(p.epi);
-  if (sizeof(O) == 2 && p.ldc % 8 == 0 && (glu || p.N % 8 == 0) && (p.n_main == p.N || n0 + BN <= p.n_main)) {
+  if (sizeof(O) == 2 && p.ldc % 8 == 0 && (glu || p.n_main % 8 == 0) && (p.n_main == p.N || n0 + BN <= p.n_main)) {
     constexpr int LD = BN + 8;
     __syncthreads();
 #pragma unroll
@@ -133,11 +133,11 @@ __global__ void __launch_bounds__(WM * WN * 64, WM * WN == 4 ? 2 : 1) gemm_tile_
         }
     }
     __syncthreads();
-    const int cols = glu ? BN / 2 : BN, c0 = glu ? n0 >> 1 : n0, per = cols / 8;
+    const int cols = glu ? BN / 2 : BN, c0 = glu ? n0 >> 1 : n0, per = cols / 8, end = glu ? p.n_main >> 1 : p.n_main;
     bf16_t* out = reinterpret_cast<bf16_t*>(C);
     for (int id = tid; id < BM * per; id += NW * 64) {
       const int r = id / per, ch = (id % per) * 8;
-      if (m0 + r < m_end && c0 + ch < p.ldc)
+      if (m0 + r < m_end && c0 + ch < end)
         *reinterpret_cast<uint4_*>(out + (long)(m0 + r) * p.ldc + c0 + ch) =
             *reinterpret_cast<const uint4_*>(smem + r * LD + ch);
     }

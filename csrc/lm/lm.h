@@ -54,7 +54,7 @@ struct ResidualNormArgs {
   const int* slot_of;      // [*, top]
   const float* wts;        // [*, top]
   int top;
-  const float* wb;         // its norm's gain
+  const float* wb;         // its norm's gain, or null: added without a norm
   const float* bb;         // its norm's bias, or null
   float mult;
   const float* step;       // [Dp] added to every row, or null
@@ -122,6 +122,7 @@ struct GemmArgs {
   float param;
   int n_main;              // columns n_main .. N - 1 are a plain fp32 product, stored in side [M, N - n_main]
   float* side;
+  int n_act;               // columns from n_act on are plain (EPI_RELU2 only; n_main: none)
   bool out_f32;
   long lda, ldc;           // row strides of A and C
   int splits;              // K cut into this many parts over blockIdx.z: C [splits, M, N] fp32 partial sums
@@ -162,13 +163,18 @@ void launch_route_plan(const RouteArgs& r, const PlanArgs& a, hipStream_t s);   
 
 struct AttnArgs {
   const void* qkvg;        // [T, ld]: q (H dk), k (G dk), v (G dv), gate logits (H gate_w)
-  long ld;
-  int gate_off, gate_w;    // column of the gate logits; 1 per head or dv of them
+  long ld, ldo;            // row strides of qkvg and o
+  int v_off;               // column of the values (that of the keys where those are the values)
+  int gate_off, gate_w;    // column of the gate logits; 1 per head or dv of them, 0: no gate
   bool own_kv;             // rows hold k and v (else another layer's are in the cache, and the gate follows q)
   bool window;             // a position sees itself and the chunk - 1 before it (else its own chunk)
   const float* rope;       // [T, rot] cos / sin of every row, or null: q and k are used as they are.  Otherwise dimension
   int rot, dim;            // i < rot / 2 of a head is turned with i + rot / 2, and the head divided by its rms over `dim`
   float eps;
+  const float* q_gain;     // [dk], or null: with gains the norm comes first, then the rotation
+  const float* k_gain;
+  const float* temp;       // [H] factor on a head's scores, or null
+  float out_scale;         // factor on the output where there is no gate
   void* kc;                // [blocks, G, 64, dk]
   void* vc;                // [blocks, G, 64, dv]
   void* o;                 // [T, H dv]
@@ -185,7 +191,7 @@ struct AttnArgs {
   const void* kv;          // [rows, H, np + dv]
   const void* lat;         // [rows, lat_ld]
   const int* kv_start;
-  const float* sink;       // [H]
+  const float* sink;       // [H] exp(sink) is added to a head's denominator; or null (not in the latent form)
   int np, rank, lat_ld, lat_pad;   // lat_pad: the last column after `rank` from which 8 values may be read
 };
 void launch_kv_store(const AttnArgs& a, bool f32, hipStream_t s);
@@ -269,5 +275,44 @@ struct Hgrn2Args {         // S = diag(f) S + (1 - f) v^T, o = S^T silu(q), out 
 };
 void launch_hgrn2_rows(const Hgrn2Args& a, bool f32, hipStream_t s);   // row by row
 void launch_hgrn2_chunks(const Hgrn2Args& a, hipStream_t s);           // bf16, 32 rows at a time
+
+struct RuleArgs {          // delta rule (mode 1: a decay per head, 2: per key channel) or retention (mode 0), see rule.hip
+  int mode;
+  const void* x;           // [T, 2 G dk + H dv]: projected q, k, v
+  const void* gate;        // [T, H dv]
+  const float* decay;      // [T, H] or [T, H dk] logits before their bias
+  const float* beta;       // [T, H] logits
+  long ldx, ldg, ldd, ldb, ldo;    // row strides
+  const float* conv;       // [taps, channels of x], oldest tap first
+  const float* rate;       // [H]; retention: [2, H] decays and their base-2 logarithms
+  const float* bias;       // [H] or [H dk]
+  const float* gain;       // [dv] (0 in the pads); retention: none
+  const float* rope;       // retention: [T, rot] cos / sin
+  void* ring;              // [slots, taps, channels] of the type of x
+  float* state;            // [slots, H, dk, dv]
+  void* out;               // [T, H dv]
+  const int* pos;          // [T]
+  const int* q_start;      // [B], null: one row per sequence (decode)
+  const int* q_lens;
+  const int* slots;        // [B], -1: none
+  void* ws;                // chunks: [T / 32 + B, heads] prepared chunks
+  int T, B, H, G, dk, dv, dim, vdim, taps, rot, gate_kind, max_q, head0, heads;
+  float eps;
+};
+void launch_rule_rows(const RuleArgs& a, bool f32, hipStream_t s);     // row by row
+void launch_rule_chunks(const RuleArgs& a, hipStream_t s);             // bf16, 32 rows at a time; heads head0 .. of a prefill step
+long rule_chunk_bytes(int dk, int dv);                                 // workspace of one chunk of one head
+
+struct RingArgs {          // the last inputs of a prefill step into the rings
+  const void* x;
+  void* ring;
+  const int* pos;
+  const int* q_start;
+  const int* q_lens;
+  const int* slots;
+  long ldx;
+  int B, n_slots, taps, channels;
+};
+void launch_ring_commit(const RingArgs& a, bool f32, hipStream_t s);
 
 }  // namespace shai_lm

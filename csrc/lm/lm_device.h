@@ -100,7 +100,7 @@ __device__ __forceinline__ void epilogue_cols(const GemmArgs& p, long m, int n, 
     c[1] = gelu_tanh(c[2], fast) * c[3];
   } else if (is(EPI_RELU2)) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) c[i] = c[i] > 0.f ? c[i] * c[i] : 0.f;
+    for (int i = 0; i < 4; ++i) c[i] = n >= p.n_act ? c[i] : c[i] > 0.f ? c[i] * c[i] : 0.f;
   } else if (is(EPI_GELU_ROWS)) {
     if (n < p.N) {
       const long at = (long)min(max(p.ids[m], 0), p.table_rows - 1) * p.table_ld + n;
@@ -148,7 +148,7 @@ __device__ __forceinline__ void store_cols(const GemmArgs& p, O* out, long m, in
     return;
   }
   O* o = out + m * p.ldc + n;
-  if (((p.N | p.ldc) & 3) == 0) {
+  if (((p.n_main | (int)p.ldc) & 3) == 0) {
     if (n < p.N) store4(o, c);
   } else {
 #pragma unroll

@@ -190,7 +190,7 @@ __global__ void __launch_bounds__(NT, conv_waves(TAPS, NT, NV)) residual_norm_ke
     if (has_delta) {
 #pragma unroll
       for (int i = 0; i < NV; ++i) d[i] = wide4(q.d[i]);
-      r = p.mult * scale_of(d, p.bb != nullptr);
+      r = p.wb ? p.mult * scale_of(d, p.bb != nullptr) : p.mult;
     }
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
@@ -198,7 +198,7 @@ __global__ void __launch_bounds__(NT, conv_waves(TAPS, NT, NV)) residual_norm_ke
       v[i] = q.x[i];
       if (c < p.Dp) {
         if (has_delta) {
-          v[i] += d[i] * r * gain(p.wb, 1, i);
+          v[i] += p.wb ? d[i] * r * gain(p.wb, 1, i) : d[i] * r;
           if (p.bb) v[i] += p.mult * (CONV && !p.w ? gain(p.bb, 0, i) : load4(p.bb + c));
         }
         if (p.step) v[i] += load4(p.step + c);

@@ -342,7 +342,7 @@ class _Inflight:
 
 
 class LLMEngine:
-    """``cfg``: a config of :mod:`shai_amd.models.registry` (Llama family, mllama, Golulix, Faledra, Nalizen)."""
+    """``cfg``: a config of :mod:`shai_amd.models.registry` (Llama family, mllama, Golulix, Faledra, Nalizen, Pugozen)."""
 
     def __init__(self, cfg, device="cuda", model_path: Optional[str] = None, seed: int = 0,
                  max_num_seqs: int = 64, max_model_len: int = 4096, num_kv_blocks: Optional[int] = None,
@@ -1100,11 +1100,13 @@ def llama_config_for(model_id: str, model_path: Optional[str] = None, size: str 
     from ..models.golulix import GolulixConfig
     from ..models.mllama import MllamaConfig
     from ..models.nalizen import NalizenConfig
+    from ..models.pugozen import PugozenConfig
     cfg = config_from_path(model_path)
     if cfg is not None:
         return cfg
     m = (model_id or "").lower()
-    for name, design in (("golulix", GolulixConfig), ("faledra", FaledraConfig), ("nalizen", NalizenConfig)):
+    for name, design in (("golulix", GolulixConfig), ("faledra", FaledraConfig), ("nalizen", NalizenConfig),
+                         ("pugozen", PugozenConfig)):
         if name in m:
             if size != "tiny":
                 raise ValueError(f"{name} has no published size: give the folder of a checkpoint (config.json)")

@@ -695,14 +695,308 @@ class TokenSide(nn.Module):
         _init_packed(self, self.pack, self.shapes(), gen)
 
 
+# ---------------------------------------------------------------------------------------------- joint layers
+class JointLayer(nn.Module):
+    """Sublayers that read one norm's output and whose sum is added to the residual: one or more mixers and an ungated
+    squared-ReLU feed-forward (``ff`` 0: none).  One product gives every mixer's inputs and the activated feed-forward, one
+    product over the mixers' outputs and the feed-forward sums them all in fp32.
+
+    A mixer supplies the rows of its input projections (``in_rows``, with an fp32 part of ``side_rows``) and the columns of its
+    output projection (``out_cols``), reads its inputs from the step's rows and writes its output beside the others'."""
+
+    def __init__(self, width: int, mixers, ff: int, dtype=torch.bfloat16):
+        super().__init__()
+        self.width, self.ff, self.fp = width, ff, lm.pad64(ff)
+        self.mixers = nn.ModuleDict(mixers)              # name in the checkpoint ("only": none) -> mixer
+        self.out_cols = sum(m.out_cols for m in self.mixers.values())
+        self.in_rows = sum(m.in_rows for m in self.mixers.values())
+        self.side_rows = sum(m.side_rows for m in self.mixers.values())
+        W = lm.pad64(width)
+        self.w_in = _param(self.fp + self.in_rows + self.side_rows, W, dtype=dtype)
+        self.w_out = _param(W, self.out_cols + self.fp, dtype=dtype)
+
+    def shapes(self) -> Dict[str, tuple]:
+        s = {f"mix.{self._dot(n)}{k}": v for n, m in self.mixers.items() for k, v in m.shapes().items()}
+        if self.ff:
+            s.update({"mlp.up": (self.ff, self.width), "mlp.down": (self.width, self.ff)})
+        return s
+
+    @staticmethod
+    def _dot(name: str) -> str:
+        return "" if name == "only" else name + "."
+
+    def _gets(self, get):
+        return [(m, lambda k, p=f"mix.{self._dot(n)}": get(p + k)) for n, m in self.mixers.items()]
+
+    def pack(self, get: Callable[[str], torch.Tensor]) -> Dict[str, torch.Tensor]:
+        """This layer's own parameters (a mixer packs the rest of its tensors)."""
+        W, gets = self.w_in.shape[1], self._gets(get)
+        rows = ([_padded(get("mlp.up"), self.fp, W)] if self.ff else []) + [m.pack_in(g) for m, g in gets]
+        rows += [m.pack_side(g) for m, g in gets if m.side_rows]
+        cols = [m.pack_out(g) for m, g in gets] + ([_padded(get("mlp.down"), W, self.fp)] if self.ff else [])
+        return {"w_in": torch.cat(rows), "w_out": torch.cat(cols, 1)}
+
+    def pack_all(self, get) -> Dict[str, torch.Tensor]:
+        out = self.pack(get)
+        for (n, m), (_, g) in zip(self.mixers.items(), self._gets(get)):
+            out.update({f"mixers.{n}.{k}": v for k, v in m.pack(g).items()})
+        return out
+
+    def forward(self, h, batch, cache, state, step):
+        """``cache`` / ``state``: what the mixers that have a key-value cache / a recurrent state keep of this layer run."""
+        n = self.out_cols + self.fp
+        rows = torch.empty(h.shape[0], n + self.in_rows, dtype=h.dtype, device=h.device)
+        side = lm.matmul_joint(h, self.w_in, rows[:, self.out_cols:], self.fp, self.side_rows)
+        i, s, o = n, 0, 0
+        for m in self.mixers.values():
+            m(rows[:, i:i + m.in_rows], side[:, s:s + m.side_rows] if m.side_rows else None, rows[:, o:o + m.out_cols], batch,
+              cache if m.cached else state, step)
+            i, s, o = i + m.in_rows, s + m.side_rows, o + m.out_cols
+        return lm.matmul_parts(rows[:, :n], self.w_out)
+
+    def cache_shapes(self, blocks: int, block: int):
+        return next((m.cache_shapes(blocks, block) for m in self.mixers.values() if m.cached), None)
+
+    def state_shapes(self):
+        """[(shape per slot, whether it is fp32 in a bf16 model too)] of the recurrent mixer, or None."""
+        return next((m.state_shapes() for m in self.mixers.values() if not m.cached), None)
+
+    def init_random_(self, gen):
+        _init_packed(self, self.pack, self.shapes(), gen)
+
+
+@dataclass
+class TiedAttentionConfig:
+    heads: int
+    kv_heads: int
+    dim: int                                     # of queries, keys and values
+    scale: float
+    rot_dims: int
+    rot_base: float = 10000.0
+    out_scale: float = 1.0                       # factor on the mixer's output
+
+    def __post_init__(self):
+        if (min(self.heads, self.kv_heads, self.dim) < 1 or self.heads % self.kv_heads or self.rot_dims % 2
+                or not 0 < self.rot_dims <= self.dim):
+            raise ValueError(f"bad attention sizes: {self}")
+
+
+class TiedAttention(nn.Module):
+    """Causal attention whose values are the projected keys: queries and keys rms-normed per head with a gain and then rotated
+    (half against half), a factor per head on the scores, a learned sink per head in the denominator."""
+
+    cached, side_rows = True, 0
+
+    def __init__(self, width: int, c: TiedAttentionConfig, eps: float):
+        super().__init__()
+        self.c, self.width, self.eps = c, width, eps
+        self.dk, _ = lm.head_pad(c.dim, c.dim)
+        self.in_rows, self.out_cols = (c.heads + c.kv_heads) * self.dk, c.heads * self.dk
+        f32 = lambda n: _param(n, dtype=torch.float32)
+        self.q_gain, self.k_gain, self.temp, self.sink = f32(self.dk), f32(self.dk), f32(c.heads), f32(c.heads)
+        self.register_buffer("freq", lm.rope_freq(c.rot_base, c.rot_dims).to(self.sink.device), persistent=False)
+
+    @property
+    def rope_key(self):
+        return self.c.rot_base, self.c.rot_dims, None
+
+    def shapes(self) -> Dict[str, tuple]:
+        c, D = self.c, self.width
+        return {"q": (c.heads * c.dim, D), "k": (c.kv_heads * c.dim, D), "q.norm": (c.dim,), "k.norm": (c.dim,),
+                "temp": (c.heads,), "sink": (c.heads,), "o": (D, c.heads * c.dim)}
+
+    def pack(self, get: Callable[[str], torch.Tensor]) -> Dict[str, torch.Tensor]:
+        return {"q_gain": _padded(get("q.norm"), self.dk), "k_gain": _padded(get("k.norm"), self.dk), "temp": get("temp"),
+                "sink": get("sink")}
+
+    def pack_in(self, get):
+        c, W = self.c, lm.pad64(self.width)
+        return torch.cat([_head_rows(get("q"), c.heads, c.dim, self.dk, W), _head_rows(get("k"), c.kv_heads, c.dim, self.dk, W)])
+
+    def pack_out(self, get):
+        return _head_columns(get("o"), self.c.heads, self.c.dim, self.dk, lm.pad64(self.width))
+
+    def forward(self, x, side, out, batch, cache, step):
+        c = self.c
+        lm.gated_attention(x, *cache, batch, c.heads, lm.WHOLE, c.scale, window=True,
+                           turn=lm.HeadTurn(step.rope(self), c.dim, self.eps, self.q_gain, self.k_gain),
+                           plain=lm.Ungated(self.temp, self.sink, out, c.out_scale))
+
+    def cache_shapes(self, blocks: int, block: int):
+        return ((blocks, self.c.kv_heads, block, self.dk),) * 2
+
+    def init_random_(self, gen):
+        _init_packed(self, self.pack, self.shapes(), gen)
+
+
+@dataclass
+class DeltaRuleConfig:
+    heads: int
+    kv_heads: int                                # heads of queries and keys
+    dim: int
+    vdim: int
+    taps: int
+    ranks: Optional[tuple] = None                # of the thin products for (decay, output gate); None: whole products,
+                                                 # and one decay per head instead of one per key channel
+    gate: int = lm.GATE_SILU
+    out_scale: float = 1.0
+
+    def __post_init__(self):
+        if min(self.heads, self.kv_heads, self.dim, self.vdim, *(self.ranks or ())) < 1 or self.heads % self.kv_heads:
+            raise ValueError(f"bad delta rule sizes: {self}")
+        if not 1 <= self.taps <= lm.MAX_TAPS:
+            raise ValueError(f"short convolutions of 1 to {lm.MAX_TAPS} taps are supported, got {self.taps}")
+
+
+class DeltaRule(nn.Module):
+    """Linear attention whose matrix state per head is decayed (per head, or per key channel) and written by the delta rule;
+    queries, keys and values pass a short convolution and silu, queries and keys are unit vectors, every head's output is
+    rms-normed and gated.  Decay and write strength logits leave their products in fp32."""
+
+    cached = False
+
+    def __init__(self, width: int, c: DeltaRuleConfig, eps: float, dtype=torch.bfloat16):
+        super().__init__()
+        self.c, self.width, self.eps, self.dtype = c, width, eps, dtype
+        H, G = c.heads, c.kv_heads
+        self.dk, self.dv = lm.head_pad(c.dim, c.vdim)
+        self.channels = 2 * G * self.dk + H * self.dv
+        self.low = [lm.pad64(r) for r in c.ranks] if c.ranks else None
+        self.in_rows = self.channels + (sum(self.low) if self.low else H * self.dv)
+        self.side_rows = H if self.low else 2 * H
+        self.out_cols = H * self.dv
+        f32 = lambda *n: _param(*n, dtype=torch.float32)
+        self.conv = f32(c.taps, self.channels)
+        self.rate, self.bias, self.gain = f32(H), f32(H * (self.dk if self.low else 1)), f32(self.dv)
+        if self.low:   # both thin products' second halves as one: [gate | decay] from [decay part | gate part]
+            self.up = _param(H * (self.dv + self.dk), sum(self.low), dtype=dtype)
+        self.shape = lm.RuleShape(G, c.dim, c.vdim, c.gate)
+
+    def shapes(self) -> Dict[str, tuple]:
+        c, D, H = self.c, self.width, self.c.heads
+        kv, n, m = c.kv_heads * c.dim, H * c.dim, H * c.vdim
+        s = {"b": (H, D), "A_log": (H,), "norm": (c.vdim,), "o": (D, m), "dt_bias": (n if c.ranks else H,)}
+        for name, rows in (("q", kv), ("k", kv), ("v", m)):
+            s.update({name: (rows, D), name + ".conv": (rows, c.taps)})
+        if c.ranks:
+            a, g = c.ranks
+            s.update({"a1": (a, D), "a2": (n, a), "g1": (g, D), "g2": (m, g)})
+        else:
+            s.update({"a": (H, D), "g": (m, D)})
+        return s
+
+    def _spread(self, get, suffix: str, width: int) -> torch.Tensor:
+        """Rows of queries, keys and values, every head padded."""
+        c = self.c
+        return torch.cat([_head_rows(get(n + suffix), heads, d, pad, width)
+                          for n, heads, d, pad in (("q", c.kv_heads, c.dim, self.dk), ("k", c.kv_heads, c.dim, self.dk),
+                                                   ("v", c.heads, c.vdim, self.dv))])
+
+    def pack(self, get: Callable[[str], torch.Tensor]) -> Dict[str, torch.Tensor]:
+        c, H = self.c, self.c.heads
+        out = {"conv": self._spread(get, ".conv", c.taps).T, "rate": get("A_log").double().exp().float(),
+               "gain": _padded(get("norm").float() * c.out_scale, self.dv), "bias": get("dt_bias")}
+        if self.low:
+            a, g = self.low
+            out["bias"] = _padded(get("dt_bias").reshape(H, c.dim), H, self.dk).reshape(-1)
+            gate = _head_rows(get("g2"), H, c.vdim, self.dv, g)
+            decay = _head_rows(get("a2"), H, c.dim, self.dk, a)
+            out["up"] = torch.cat([torch.cat([gate.new_zeros(len(gate), a), gate], 1),
+                                   torch.cat([decay, decay.new_zeros(len(decay), g)], 1)])
+        return out
+
+    def pack_in(self, get):
+        W = lm.pad64(self.width)
+        last = ([_padded(get(n), r, W) for n, r in zip(("a1", "g1"), self.low)] if self.low
+                else [_head_rows(get("g"), self.c.heads, self.c.vdim, self.dv, W)])
+        return torch.cat([self._spread(get, "", W)] + last)
+
+    def pack_side(self, get):
+        return _padded(torch.cat([get(n) for n in (("b",) if self.low else ("b", "a"))]), self.side_rows, lm.pad64(self.width))
+
+    def pack_out(self, get):
+        return _head_columns(get("o"), self.c.heads, self.c.vdim, self.dv, lm.pad64(self.width))
+
+    def forward(self, x, side, out, batch, state, step):
+        H, n = self.c.heads, self.channels
+        gate, decay = x[:, n:], side[:, H:]
+        if self.low:
+            gate, decay = lm.matmul_with_side(gate, self.up, H * self.dk)
+        lm.delta_rule(x[:, :n], gate, decay, side[:, :H], self.conv, self.rate, self.bias, self.gain, *state, batch, out,
+                      self.shape, self.eps)
+
+    def state_shapes(self):
+        return [((self.c.heads, self.dk, self.dv), True), ((self.c.taps, self.channels), False)]
+
+    def init_random_(self, gen):
+        _init_packed(self, self.pack, self.shapes(), gen)
+
+
+@dataclass
+class RetentionConfig:
+    decay: tuple                                 # of every head
+    dim: int
+    vdim: int
+    rot_dims: int
+    rot_base: float = 10000.0
+
+    def __post_init__(self):
+        if (not self.decay or min(self.dim, self.vdim) < 1 or self.rot_dims % 2 or not 0 < self.rot_dims <= self.dim
+                or not all(0.0 <= d <= 1.0 for d in self.decay)):
+            raise ValueError(f"bad retention sizes: {self}")
+
+
+class Retention(nn.Module):
+    """Linear attention with a matrix state and a fixed decay per head, rotated queries and keys, every head's output
+    rms-normed and gated by silu."""
+
+    cached, side_rows = False, 0
+
+    def __init__(self, width: int, c: RetentionConfig, eps: float):
+        super().__init__()
+        self.c, self.width, self.eps = c, width, eps
+        self.H = H = len(c.decay)
+        self.dk, self.dv = lm.head_pad(c.dim, c.vdim)
+        self.in_rows, self.out_cols = H * (2 * self.dk + 2 * self.dv), H * self.dv
+        self.shape = lm.RuleShape(H, c.dim, c.vdim, lm.GATE_SILU)
+        self.register_buffer("freq", lm.rope_freq(c.rot_base, c.rot_dims), persistent=False)
+        self.register_buffer("decay", lm.decay_rates(c.decay), persistent=False)
+
+    @property
+    def rope_key(self):
+        return self.c.rot_base, self.c.rot_dims, None
+
+    def shapes(self) -> Dict[str, tuple]:
+        c, D, n, m = self.c, self.width, self.H * self.c.dim, self.H * self.c.vdim
+        return {"q": (n, D), "k": (n, D), "v": (m, D), "g": (m, D), "o": (D, m)}
+
+    def pack(self, get) -> Dict[str, torch.Tensor]:
+        return {}
+
+    def pack_in(self, get):
+        c, W = self.c, lm.pad64(self.width)
+        return torch.cat([_head_rows(get(n), self.H, d, pad, W) for n, d, pad in (
+            ("q", c.dim, self.dk), ("k", c.dim, self.dk), ("v", c.vdim, self.dv), ("g", c.vdim, self.dv))])
+
+    def pack_out(self, get):
+        return _head_columns(get("o"), self.H, self.c.vdim, self.dv, lm.pad64(self.width))
+
+    def forward(self, x, side, out, batch, state, step):
+        n = self.H * (2 * self.dk + self.dv)
+        lm.retention(x[:, :n], x[:, n:], self.decay, step.rope(self), state[0], batch, out, self.shape, self.eps)
+
+    def state_shapes(self):
+        return [((self.H, self.dk, self.dv), True)]
+
+
 def _init_packed(module: nn.Module, pack, shapes: Dict[str, tuple], gen) -> None:
-    """Fill a block from random full-size tensors of its checkpoint shapes: matrices N(0, 1 / fan_in), norm gains 1, other
+    """Fill a block from random full-size tensors of its checkpoint shapes: matrices N(0, 1 / fan_in), gains 1, other
     vectors 0."""
     dev, dtype = gen.device, next(module.parameters()).dtype
 
     def draw(name):
         if len(shapes[name]) == 1:
-            return torch.full(shapes[name], float(name.endswith("norm")), device=dev)
+            return torch.full(shapes[name], float(name.endswith(("norm", "temp"))), device=dev)
         return (torch.randn(shapes[name], generator=gen, device=dev) / math.sqrt(shapes[name][1])).to(dtype)
     for k, v in pack(draw).items():
-        getattr(module, k).copy_(v)
+        module.get_parameter(k).copy_(v)

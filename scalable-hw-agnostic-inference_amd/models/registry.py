@@ -16,24 +16,29 @@ from .golulix import GolulixConfig, GolulixForCausalLM
 from .llama import LlamaConfig, LlamaForCausalLM
 from .mllama import MllamaConfig, MllamaForConditionalGeneration
 from .nalizen import NalizenConfig, NalizenForCausalLM
+from .pugozen import PugozenConfig, PugozenForCausalLM
 
 MODELS = {LlamaConfig: LlamaForCausalLM, MllamaConfig: MllamaForConditionalGeneration,
           GolulixConfig: GolulixForCausalLM, FaledraConfig: FaledraForCausalLM,
-          NalizenConfig: NalizenForCausalLM}
+          NalizenConfig: NalizenForCausalLM, PugozenConfig: PugozenForCausalLM}
 
 # config.json "architecture" -> config reader, for designs that name themselves that way
 ARCHITECTURES: Dict[str, Callable[[dict], object]] = {"Golulix": GolulixConfig.from_json,
                                                        "Faledra": FaledraConfig.from_json,
-                                                       "Nalizen": NalizenConfig.from_json}
+                                                       "Nalizen": NalizenConfig.from_json,
+                                                       "Pugozen": PugozenConfig.from_json}
+# those with sizes that only the shapes of the checkpoint's tensors tell
+SIZED_BY_TENSORS = ("Pugozen",)
 
 
-def config_from_json(d: dict):
-    """The config object of a parsed config.json (HF-style files: Llama family, or mllama with a vision tower)."""
+def config_from_json(d: dict, shapes: Optional[Dict[str, tuple]] = None):
+    """The config object of a parsed config.json (HF-style files: Llama family, or mllama with a vision tower).  ``shapes``:
+    those of the checkpoint's tensors, for the designs that need them."""
     name = d.get("architecture")
     if name is not None:
         if name not in ARCHITECTURES:
             raise ValueError(f"unknown architecture {name!r}: known are {sorted(ARCHITECTURES)}")
-        return ARCHITECTURES[name](d)
+        return ARCHITECTURES[name](d, shapes) if name in SIZED_BY_TENSORS else ARCHITECTURES[name](d)
     if "vision_config" in d and "text_config" in d:
         return MllamaConfig.from_hf(d)
     return LlamaConfig.from_hf(d.get("text_config", d))
@@ -45,7 +50,11 @@ def config_from_path(path: Optional[str]):
     if not f or not os.path.exists(f):
         return None
     with open(f) as h:
-        return config_from_json(json.load(h))
+        d = json.load(h)
+    if d.get("architecture") not in SIZED_BY_TENSORS:
+        return config_from_json(d)
+    from ..weights import find_safetensors, safetensors_shapes
+    return config_from_json(d, safetensors_shapes(find_safetensors(path)))
 
 
 def model_class(cfg):

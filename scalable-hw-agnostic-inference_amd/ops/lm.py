@@ -3,9 +3,10 @@
 What a layer-list decoder needs beyond the Llama path of :mod:`shai_amd.ops`: an n-gram embedding, residual-add + norm
 (RMS or layer norm) with the residual kept in fp32 (optionally a norm on the added output and a short causal convolution
 on the sum or its norm), one GEMM for dense, per-head and expert-grouped products, mixture-of-experts routing, attention
-restricted to fixed-size chunks of the sequence or a sliding window with an output gate, attention over cached latents
-with a sink per head, a gated linear recurrence, and linear attention with a gated matrix state.  Every op takes bf16 or fp32 weights and activations; norms,
-routing, attention scores, rotation angles, recurrent state and the residual are fp32 in both.
+restricted to fixed-size chunks of the sequence or a sliding window with an output gate or causal with a sink per head,
+attention over cached latents with a sink per head, a gated linear recurrence, and linear attention with a matrix state (gated,
+written by the delta rule, or with a fixed decay).  Every op takes bf16 or fp32 weights and activations; norms, routing,
+attention scores, rotation angles, recurrent state and the residual are fp32 in both.
 
 Layout rules shared by all of them: the model width is padded to a multiple of 64 (``pad64``; the pad columns of
 activations and weights are zero), so a GEMM's K is always a multiple of 64.
@@ -34,6 +35,9 @@ LATENT_GROUP_ROWS = 1 << 18  # context rows that are expanded at a time
 PARTS, PARTS_COLUMNS = 4, 8192   # partial sums: at most so many, of products up to so wide in a decode step
 SCAN_CHUNK, SCAN_MAX_CHUNKS = 64, 64
 STATE_SEGMENT, STATE_MAX_SEGMENTS = 128, 32      # rows of a matrix-state segment at least; segments at most
+WHOLE = 1 << 30              # window that holds any sequence
+RULE_CHUNK = 32              # rows of a chunk of the delta rule and of retention
+RULE_WORKSPACE = 1 << 30     # bytes of prepared chunks at a time (more heads take several rounds)
 
 
 def pad64(n: int) -> int:
@@ -139,6 +143,21 @@ def matmul_with_side(a, w, side: int, epi: int = EPI_NONE, param: float = 0.0):
     return c, s
 
 
+def matmul_joint(a, w, out, act: int, side: int):
+    """One product for several consumers of ``a``, into ``out`` [M, n] (a view with any row stride): its first ``act``
+    columns are max(c, 0)^2, the others plain.  The last ``side`` rows of w ([n + side, K]) are a plain product in fp32,
+    which is returned (None without any)."""
+    n = out.shape[1]
+    if not a.is_cuda:
+        c = a.float() @ w.float().T
+        out[:, :act] = (torch.relu(c[:, :act]) ** 2).to(out.dtype)
+        out[:, act:] = c[:, act:n].to(out.dtype)
+        return c[:, n:].contiguous() if side else None
+    s = torch.empty(a.shape[0], side, dtype=torch.float32, device=a.device) if side else None
+    _K().lm_gemm(a, w, out, None, None, None, 0, EPI_RELU2 if act else EPI_NONE, 0.0, s, act=int(act))
+    return s
+
+
 def matmul_parts(a, w, out_dtype=None):
     """a w^T for a consumer that adds partial sums (:func:`residual_norm`, :func:`latent_prep`): [parts, M, N] fp32
     where the product needs K cut up to fill the chip (few rows, few columns); else :func:`matmul`."""
@@ -218,14 +237,29 @@ def route_experts(logits, top: int, groups: int = 1, keep: int = 1, bias=None, r
 
 class HeadTurn(NamedTuple):
     """Rotation and norm of queries and keys before they meet: dimension i < rot / 2 of a head is turned with i + rot / 2 by
-    the row's angles ``rope`` [T, rot] (:func:`rope_rows`), then the head is divided by its rms over ``dim``."""
+    the row's angles ``rope`` [T, rot] (:func:`rope_rows`), then the head is divided by its rms over ``dim``.  With gains
+    (fp32, stored head size, zero in the pads) the norm comes first, with them, and the rotation after it."""
     rope: torch.Tensor
     dim: int
     eps: float
+    q_gain: Optional[torch.Tensor] = None
+    k_gain: Optional[torch.Tensor] = None
+
+
+@dataclass
+class Ungated:
+    """Attention without an output gate: the values are the projected keys (rows are [q | k]), each head's scores times
+    ``temp`` [H], exp(``sink`` [H]) in its denominator, its output times ``out_scale`` (into ``out`` [T, H dv], a view with
+    any row stride)."""
+    temp: torch.Tensor
+    sink: torch.Tensor
+    out: torch.Tensor
+    out_scale: float = 1.0
 
 
 def gated_attention(qkvg, k_cache, v_cache, batch, heads: int, size: int, scale: float, window: bool = False,
-                    per_element: bool = False, own_kv: bool = True, turn: Optional[HeadTurn] = None):
+                    per_element: bool = False, own_kv: bool = True, turn: Optional[HeadTurn] = None,
+                    plain: Optional[Ungated] = None):
     """Attention of one step over a paged cache: softmax over the keys j <= i of position i's own chunk (positions
     size * n .. size * (n + 1) - 1) or, with ``window``, of the size positions that end with i; the output times
     sigmoid(gate logits), one per head or (``per_element``) per output element.
@@ -233,25 +267,33 @@ def gated_attention(qkvg, k_cache, v_cache, batch, heads: int, size: int, scale:
     ``qkvg`` [T, >= H dk + G (dk + dv) + gates] holds q, k, v and the gate logits of the step's rows; k / v are written to
     the caches [blocks, G, 64, dk | dv] at ``batch.slots`` (-1: padding row), with ``turn`` as the turned keys (and q may
     be prepared in place).  ``own_kv`` False: rows are [q | gates], and the cache is another layer's, which has written
-    this step's rows.  Returns [T, H dv]."""
+    this step's rows.  ``plain``: no gates, another form of keys, values and scores (:class:`Ungated`).  Returns [T, H dv]."""
     if not qkvg.is_cuda:
-        return ref.gated_attention(qkvg, k_cache, v_cache, batch, heads, size, scale, window, per_element, own_kv, turn)
+        return ref.gated_attention(qkvg, k_cache, v_cache, batch, heads, size, scale, window, per_element, own_kv, turn, plain)
     dv = v_cache.shape[3]
     T = qkvg.shape[0]
-    o = torch.empty(T, heads * dv, dtype=qkvg.dtype, device=qkvg.device)
+    more, gains = {}, {}
+    if plain is not None:
+        o, more = plain.out, dict(temp=plain.temp, sink=plain.sink, out_scale=float(plain.out_scale))
+    else:
+        o = torch.empty(T, heads * dv, dtype=qkvg.dtype, device=qkvg.device)
+    if turn is not None and turn.q_gain is not None:
+        gains = dict(q_gain=turn.q_gain, k_gain=turn.k_gain)
     if batch.is_prefill:
         if turn is not None:
-            _K().head_prep(qkvg, k_cache, v_cache, batch.slots, int(heads), turn.rope, int(turn.dim), float(turn.eps), own_kv)
+            _K().head_prep(qkvg, k_cache, v_cache, batch.slots, int(heads), turn.rope, int(turn.dim), float(turn.eps), own_kv,
+                           tied=plain is not None, **gains)
         elif own_kv:
-            _K().kv_store(qkvg, k_cache, v_cache, batch.slots, int(heads))
+            _K().kv_store(qkvg, k_cache, v_cache, batch.slots, int(heads), tied=plain is not None)
         _K().gated_attn_prefill(qkvg, k_cache, v_cache, o, batch.block_table, batch.ctx_lens, batch.q_lens,
-                                batch.q_start, int(batch.S), int(heads), int(size), float(scale), window, per_element, own_kv)
+                                batch.q_start, int(batch.S), int(heads), int(size), float(scale), window, per_element, own_kv,
+                                **more)
         return o
     ns = max(1, min(int(batch.num_splits or 1), (size + 63) // 64, 64))
     ws = torch.empty(T * heads * ns * (dv + 2) if ns > 1 else 0, dtype=torch.float32, device=qkvg.device)
     _K().gated_attn_decode(qkvg, k_cache, v_cache, o, batch.block_table, batch.ctx_lens, batch.slots, ws, int(heads),
                            ns, int(size), float(scale), window, per_element, own_kv,
-                           *(turn and (turn.rope, int(turn.dim), float(turn.eps)) or ()))
+                           *(turn and (turn.rope, int(turn.dim), float(turn.eps)) or ()), **gains, **more)
     return o
 
 
@@ -297,8 +339,8 @@ def residual_norm(source, delta, wb, mult: float, step, w, eps: float, width: in
     """x = source (+ mult * norm(delta)) (+ step); h = norm(x), plus its convolution with ``conv``.
 
     source: the fp32 residual [T, D] or an :class:`Embedding`.  delta: [T, D], partial sums [parts, T, D] fp32, or
-    :class:`Experts` without a dense part.  wb, w: the norms' gains (RMS norm) or :class:`Affine` (layer norm); w PLAIN:
-    h = x.  Returns (x, h); the residual may be updated in place.  ``w`` None: no h.  ``rows`` (int32): h of these rows
+    :class:`Experts` without a dense part.  wb, w: the norms' gains (RMS norm) or :class:`Affine` (layer norm); wb PLAIN:
+    delta is added as it is; w PLAIN: h = x.  Returns (x, h); the residual may be updated in place.  ``w`` None: no h.  ``rows`` (int32): h of these rows
     only, and with ``keep`` False x is None."""
     emb = isinstance(source, Embedding)
     if not (source.ids if emb else source).is_cuda:
@@ -522,3 +564,75 @@ def hgrn2(qv, z, bias, lower, gain, state, batch, vdim: int, eps: float):
     _K().hgrn2(qv, z, bias, lower, gain, state, out, batch.positions, batch.q_start, batch.q_lens, batch.state_slots, ws,
                max_q, n, int(vdim), float(eps))
     return out
+
+
+# ---------------------------------------------------------------------------------------------- delta rule, retention
+GATE_SILU, GATE_SIGMOID = 0, 1
+
+
+@dataclass
+class RuleShape:
+    """Sizes of a matrix-state mixer: ``dim`` / ``vdim`` before padding, ``kv_heads`` heads of queries and keys for the
+    state's heads, and what its output gate is passed through."""
+    kv_heads: int
+    dim: int
+    vdim: int
+    gate: int = GATE_SILU
+
+
+def _rule_run(x, gate, state, out, batch, shape: RuleShape, eps: float, commit, **args):
+    """The launches of one step: decode and fp32 rows one by one; bf16 portions in chunks, as many heads at a time as the
+    workspace holds."""
+    T, (_, H, dk, dv) = x.shape[0], state.shape
+    args = dict(pos=batch.positions, slots=batch.state_slots, kv_heads=int(shape.kv_heads), dim=int(shape.dim),
+                vdim=int(shape.vdim), gate_kind=int(shape.gate), eps=float(eps), **args)
+    if not batch.is_prefill:
+        _K().rule_rows(x, gate, state, out, **args)
+        return
+    args.update(q_start=batch.q_start, q_lens=batch.q_lens)
+    if x.dtype == torch.float32:
+        _K().rule_rows(x, gate, state, out, **args)
+    else:
+        unit, chunks = _K().rule_chunk_bytes(dk, dv), T // RULE_CHUNK + batch.B
+        at_a_time = max(1, min(H, RULE_WORKSPACE // (chunks * unit)))
+        ws = torch.empty(chunks * at_a_time * unit, dtype=torch.uint8, device=x.device)
+        for h in range(0, H, at_a_time):
+            _K().rule_chunks(x, gate, state, out, ws=ws, max_q=int(batch.S), head0=h, heads=min(at_a_time, H - h), **args)
+    if commit is not None:
+        _K().ring_commit(x, commit, batch.positions, batch.q_start, batch.q_lens, batch.state_slots)
+
+
+def delta_rule(x, gate, decay, beta, conv, rate, bias, gain, state, ring, batch, out, shape: RuleShape, eps: float) -> None:
+    """Linear attention whose matrix state S [dk, dv] per head is written by the delta rule: S = diag(g) S,
+    u = sigmoid(beta) (v - S^T k), S = S + k u^T, o = S^T q; out = o / rms(o over vdim) gain act(gate).
+
+    x [T, G dk + G dk + H dv] holds the projected queries, keys and values.  Each of their channels passes a causal
+    convolution over time (``conv`` [taps, channels], oldest tap first) and silu; queries and keys are then made unit vectors
+    (queries also times dim^-1/2), head h using those of head h / (H / G).  g = exp(-rate softplus(decay + bias)) with
+    ``decay`` fp32 [T, H] (bias [H]: one decay per head) or [T, H dk] (bias [H dk]: one per key channel); rate [H]; beta
+    logits fp32 [T, H]; gate [T, H dv]; gain [dv] (zero in the pads).  ``state`` [slots, H, dk, dv] (fp32) and ``ring``
+    [slots, taps, channels] (the last inputs, each at its position modulo taps) carry a sequence; its first token starts from
+    zero.  x, gate, decay, beta and out may be views with any row stride."""
+    if not x.is_cuda:
+        ref.delta_rule(x, gate, decay, beta, conv, rate, bias, gain, state, ring, batch, out, shape, eps)
+        return
+    _rule_run(x, gate, state, out, batch, shape, eps, ring, decay=decay, beta=beta, conv=conv, rate=rate, bias=bias, gain=gain,
+              ring=ring)
+
+
+def decay_rates(decay) -> torch.Tensor:
+    """Decays in [0, 1] and their base-2 logarithms, [2, H] fp32 (2^-40 leaves nothing of a state)."""
+    d = np.asarray(decay, dtype=np.float64)
+    return torch.tensor(np.stack([d, np.log2(np.maximum(d, 2.0 ** -40))]), dtype=torch.float32)
+
+
+def retention(x, gate, decay, rope, state, batch, out, shape: RuleShape, eps: float) -> None:
+    """Linear attention with a fixed decay per head: S = decay S + k v^T, o = S^T q; out = o / rms(o over vdim) act(gate).
+
+    x [T, H (2 dk + dv)]: projected queries, keys and values; dimension i < rot / 2 of queries and keys is turned with
+    i + rot / 2 by the row's angles ``rope`` [T, rot], keys are then multiplied by dim^-1/2.  ``decay`` [2, H] fp32: the decays
+    and their base-2 logarithms.  ``state`` [slots, H, dk, dv] as in :func:`delta_rule`."""
+    if not x.is_cuda:
+        ref.retention(x, gate, decay, rope, state, batch, out, shape, eps)
+        return
+    _rule_run(x, gate, state, out, batch, shape, eps, None, rate=decay, rope=rope)

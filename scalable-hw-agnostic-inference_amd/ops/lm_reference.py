@@ -102,28 +102,42 @@ def plan_experts(ids, experts, bm):
     return Plan(off, (order // top).int(), slot_of.view(T, top), torch.empty(0, 2, dtype=torch.int32), bm)
 
 
-def _turn_heads(x, dim_pad, turn):
-    """Rotation (dimension i with i + rot / 2) and rms norm of every head of x [T, heads * dim_pad]."""
-    x = x.float().view(x.shape[0], -1, dim_pad).clone()
-    half = turn.rope.shape[1] // 2
-    cs, sn = turn.rope[:, None, 0::2], turn.rope[:, None, 1::2]
+def _turn_heads(x, dim_pad, turn, gain=None):
+    """Rotation (dimension i with i + rot / 2) and rms norm of every head of x [T, heads * dim_pad]; with a gain the norm
+    comes first."""
+    x = x.float().reshape(x.shape[0], -1, dim_pad).clone()
+    rms = lambda x: x / torch.sqrt(x.pow(2).sum(-1, keepdim=True) / turn.dim + turn.eps)
+    if gain is not None:
+        x = rms(x) * gain
+    x = _rotate_half(x, turn.rope)
+    return rms(x) if gain is None else x
+
+
+def _rotate_half(x, rope):
+    x, half = x.clone(), rope.shape[1] // 2
+    cs, sn = rope[:, None, 0::2], rope[:, None, 1::2]
     u, v = x[..., :half].clone(), x[..., half:2 * half].clone()
     x[..., :half], x[..., half:2 * half] = u * cs - v * sn, v * cs + u * sn
-    return x / torch.sqrt(x.pow(2).sum(-1, keepdim=True) / turn.dim + turn.eps)
+    return x
 
 
-def gated_attention(qkvg, k_cache, v_cache, batch, heads, size, scale, window, per_element, own_kv, turn):
+def gated_attention(qkvg, k_cache, v_cache, batch, heads, size, scale, window, per_element, own_kv, turn, plain=None):
     G, dk, dv = k_cache.shape[1], k_cache.shape[3], v_cache.shape[3]
     T = qkvg.shape[0]
-    n_gate, kv = heads * (dv if per_element else 1), (G * dk, G * dv) if own_kv else (0, 0)
-    q, k, v, gate = qkvg[:, :heads * dk + sum(kv) + n_gate].split([heads * dk, *kv, n_gate], -1)
+    if plain is not None:
+        q, k = qkvg[:, :(heads + G) * dk].split([heads * dk, G * dk], -1)
+        v = k
+    else:
+        n_gate, kv = heads * (dv if per_element else 1), (G * dk, G * dv) if own_kv else (0, 0)
+        q, k, v, gate = qkvg[:, :heads * dk + sum(kv) + n_gate].split([heads * dk, *kv, n_gate], -1)
     if turn is not None:
-        q = _turn_heads(q, dk, turn).to(qkvg.dtype).view(T, -1)
-        k = _turn_heads(k, dk, turn).to(qkvg.dtype).view(T, -1) if own_kv else k
+        q = _turn_heads(q, dk, turn, turn.q_gain).to(qkvg.dtype).view(T, -1)
+        k = _turn_heads(k, dk, turn, turn.k_gain).to(qkvg.dtype).view(T, -1) if own_kv else k
+    scale = torch.full((heads,), scale) if plain is None else scale * plain.temp
     for t, slot in enumerate(batch.slots[:T].tolist()):
         if slot >= 0 and own_kv:
-            k_cache[slot // 64, :, slot % 64] = k[t].view(G, dk)
-            v_cache[slot // 64, :, slot % 64] = v[t].view(G, dv)
+            k_cache[slot // 64, :, slot % 64] = k[t].reshape(G, dk)
+            v_cache[slot // 64, :, slot % 64] = v[t].reshape(G, dv)
     o = torch.zeros(T, heads, dv)
     for b in range(batch.B):
         n_q = int(batch.q_lens[b]) if batch.is_prefill else 1
@@ -135,8 +149,12 @@ def gated_attention(qkvg, k_cache, v_cache, batch, heads, size, scale, window, p
             key = torch.arange(max(0, pos - size + 1) if window else pos // size * size, pos + 1)
             kk = k_cache[bt[key // 64], :, key % 64].float().repeat_interleave(heads // G, 1)   # [n, H, dk]
             vv = v_cache[bt[key // 64], :, key % 64].float().repeat_interleave(heads // G, 1)
-            s = torch.einsum("hd,nhd->hn", q[row0 + i].float().view(heads, dk), kk) * scale
-            o[row0 + i] = torch.einsum("hn,nhd->hd", torch.softmax(s, -1), vv)
+            s = torch.einsum("hd,nhd->hn", q[row0 + i].float().reshape(heads, dk), kk) * scale[:, None]
+            p = torch.softmax(s, -1) if plain is None else _sink_softmax(s, plain.sink)
+            o[row0 + i] = torch.einsum("hn,nhd->hd", p, vv)
+    if plain is not None:
+        plain.out.copy_((o * plain.out_scale).view(T, heads * dv))
+        return plain.out
     return (o * torch.sigmoid(gate.float()).view(T, heads, -1)).reshape(T, heads * dv).to(qkvg.dtype)
 
 
@@ -153,7 +171,7 @@ def residual_norm(source, delta, wb, mult, step, w, eps, width, dtype, conv, bat
 
     def rms(t, w):
         gain, bias = w if isinstance(w, Affine) else (w, None)
-        if w is PLAIN:
+        if w is None or w is PLAIN:
             return t
         if bias is not None:
             mean = t.sum(-1, keepdim=True) / width
@@ -278,3 +296,67 @@ def hgrn2(qv, z, bias, lower, gain, state, batch, vdim, eps):
         if slot >= 0:
             state[slot] = S
     return (o / torch.sqrt(o.pow(2).sum(-1, keepdim=True) / vdim + eps) * gain).reshape(T, H * dv).to(qv.dtype)
+
+
+def _gate(z, kind):
+    return torch.nn.functional.silu(z) if kind == 0 else torch.sigmoid(z)
+
+
+def _rule_out(o, gain, gate, out, shape, eps):
+    T, H, dv = o.shape
+    o = o / torch.sqrt(o.pow(2).sum(-1, keepdim=True) / shape.vdim + eps)
+    if gain is not None:
+        o = o * gain
+    out.copy_(o.reshape(T, H * dv) * _gate(gate.float(), shape.gate))
+
+
+def delta_rule(x, gate, decay, beta, conv, rate, bias, gain, state, ring, batch, out, shape, eps):
+    _, H, dk, dv = state.shape
+    T, G, taps, C = x.shape[0], shape.kv_heads, conv.shape[0], conv.shape[1]
+    x = x.float()
+    y = torch.zeros(T, C)
+    for row0, n, pos, slot, _ in _sequences(batch):
+        past = torch.zeros(taps - 1, C)
+        for j in range(1, taps):
+            if pos - j >= 0 and slot >= 0:
+                past[-j] = ring[slot, (pos - j) % taps].float()
+        line = torch.cat([past, x[row0:row0 + n]])
+        for j in range(taps):
+            y[row0:row0 + n] += conv[j] * line[j:j + n]
+        if slot >= 0:
+            for t in range(max(0, n - taps), n):
+                ring[slot, (pos + t) % taps] = x[row0 + t].to(ring.dtype)
+    y = torch.nn.functional.silu(y)
+    unit = lambda t: t / torch.sqrt(t.pow(2).sum(-1, keepdim=True) + 1e-6)
+    q, k, v = y.split([G * dk, G * dk, H * dv], 1)
+    q = (unit(q.reshape(T, G, dk)) * shape.dim ** -0.5).repeat_interleave(H // G, 1)
+    k, v = unit(k.reshape(T, G, dk)).repeat_interleave(H // G, 1), v.reshape(T, H, dv)
+    g = torch.exp(-rate[:, None] * torch.nn.functional.softplus(decay.float() + bias).reshape(T, H, -1))
+    b, o = torch.sigmoid(beta.float()), torch.zeros(T, H, dv)
+    for row0, n, pos, slot, _ in _sequences(batch):
+        S = state[slot].clone() if slot >= 0 and pos > 0 else torch.zeros(H, dk, dv)
+        for t in range(row0, row0 + n):
+            S = g[t][..., None] * S
+            u = b[t][:, None] * (v[t] - (S * k[t][..., None]).sum(1))
+            S = S + k[t][..., None] * u[:, None]
+            o[t] = (S * q[t][..., None]).sum(1)
+        if slot >= 0:
+            state[slot] = S
+    _rule_out(o, gain, gate, out, shape, eps)
+
+
+def retention(x, gate, decay, rope, state, batch, out, shape, eps):
+    _, H, dk, dv = state.shape
+    T = x.shape[0]
+    q, k, v = x.float().split([H * dk, H * dk, H * dv], 1)
+    q = _rotate_half(q.reshape(T, H, dk), rope)
+    k, v = _rotate_half(k.reshape(T, H, dk), rope) * shape.dim ** -0.5, v.reshape(T, H, dv)
+    o = torch.zeros(T, H, dv)
+    for row0, n, pos, slot, _ in _sequences(batch):
+        S = state[slot].clone() if slot >= 0 and pos > 0 else torch.zeros(H, dk, dv)
+        for t in range(row0, row0 + n):
+            S = decay[0][:, None, None] * S + k[t][..., None] * v[t][:, None]
+            o[t] = (S * q[t][..., None]).sum(1)
+        if slot >= 0:
+            state[slot] = S
+    _rule_out(o, None, gate, out, shape, eps)

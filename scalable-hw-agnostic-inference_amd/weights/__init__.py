@@ -44,6 +44,16 @@ def load_safetensors(files) -> Dict[str, torch.Tensor]:
     return sd
 
 
+def safetensors_shapes(files) -> Dict[str, tuple]:
+    """Shape of every tensor (headers only)."""
+    from safetensors import safe_open
+    out = {}
+    for f in files:
+        with safe_open(f, framework="pt", device="cpu") as h:
+            out.update({k: tuple(h.get_slice(k).get_shape()) for k in h.keys()})
+    return out
+
+
 def load_into(model: nn.Module, sd: Dict[str, torch.Tensor], convert: Optional[Callable] = None,
               strict: bool = False) -> nn.Module:
     if convert is not None:
