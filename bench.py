@@ -16,8 +16,8 @@ native LLM engine at TP = N (see shai_amd.engines.llm).
 
 ``--workload vit``: ViT-base/16 224x224 classification images/s at batch 32 per GPU.
 
-``--workload golulix`` / ``faledra`` / ``nalizen``: prefill and decode tokens/s of the design beside a Llama model of equal
-size, nalizen beside Golulix too (shai_amd.bench.decoder_design).
+``--workload golulix`` / ``faledra`` / ``nalizen`` / ``pugozen``: prefill and decode tokens/s of the design beside a Llama model
+of equal size, nalizen beside Golulix and pugozen beside Nalizen too (shai_amd.bench.decoder_design).
 
 ``--tp T`` (mistral / flux): tensor-parallel degree of one replica; the N GPUs run N / T replicas
 (data parallel x tensor parallel).  Defaults: mistral T = N (one engine over all GPUs, strong scaling),
@@ -401,7 +401,7 @@ def main():
     ap.add_argument("--steps", type=int, default=3)
     ap.add_argument("--warmup", type=int, default=1)
     ap.add_argument("--workload", default="sd21", choices=["sd21", "mistral", "flux", "mllama", "vit", "t5", "golulix",
-                                                               "faledra", "nalizen"])
+                                                               "faledra", "nalizen", "pugozen"])
     ap.add_argument("--batch", type=int, default=None,
                     help="per-GPU batch: images per step (sd21: 32, flux: 1) / concurrent sequences (mistral: 64, "
                          "mllama: 8)")
@@ -417,7 +417,7 @@ def main():
     ap.add_argument("--llm-model", default="mistral_7b", choices=["mistral_7b", "llama3_8b", "deepseek_r1_distill_70b"],
                     help="--workload mistral: which Llama-architecture model (BASELINE config 4 is mistral_7b)")
     ap.add_argument("--design-size", "--golulix-size", default="both", choices=["small", "large", "both"],
-                    help="--workload golulix / faledra / nalizen: which layer sizes to measure")
+                    help="--workload golulix / faledra / nalizen / pugozen: which layer sizes to measure")
     ap.add_argument("--cpu-dry-run", action="store_true",
                     help="tests only: tiny SD2.1 config on the CPU over gloo (launcher / rendezvous / JSON plumbing)")
     ap.add_argument("--tp", type=int, default=None,
@@ -433,13 +433,14 @@ def main():
         args.tp = args.gpus if args.workload in ("mistral", "mllama") else 1
     if args.batch is None:  # dynamic-batching caps a serving replica would use for each workload
         args.batch = {"sd21": 32, "mistral": 64, "flux": 1, "mllama": 8, "vit": 32, "t5": 32,
-                      "golulix": 64, "faledra": 64, "nalizen": 64}[args.workload]
+                      "golulix": 64, "faledra": 64, "nalizen": 64, "pugozen": 64}[args.workload]
     import torch
     rank, world, local = _dist_init(args.gpus)
     with torch.inference_mode():
         fn = {"sd21": bench_sd21, "mistral": bench_mistral, "flux": bench_flux,
               "mllama": bench_mllama, "vit": bench_vit, "t5": bench_t5,
-              "golulix": bench_design, "faledra": bench_design, "nalizen": bench_design}[args.workload]
+              "golulix": bench_design, "faledra": bench_design, "nalizen": bench_design,
+              "pugozen": bench_design}[args.workload]
         res = fn(args, rank, world)
     if DEVICE == "cpu":
         res["data"] = "CPU DRY RUN (tiny config, gloo): plumbing check, not a measurement"

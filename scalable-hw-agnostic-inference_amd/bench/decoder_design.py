@@ -1,12 +1,14 @@
-"""Prefill and decode throughput of a layer-list design (Golulix, Faledra, Nalizen) beside models of equal size.
+"""Prefill and decode throughput of a layer-list design (Golulix, Faledra, Nalizen, Pugozen) beside models of equal size.
 
 Both run through :class:`LLMEngine` (scheduler, paged cache, HIP-graph decode) with random weights.  A pair has the same
 width, layers, heads and vocabulary.  The Llama MLP is as wide as the feed-forward work one Golulix token does (top x
 expert + shared expert), or has as many weights as the Faledra feed-forward (3 D I = 2 D ff), so the two do the same
 matrix work per token there.  Nalizen runs beside Golulix too (both are mixtures of experts): equal routing, gated experts
-of the same number of weights as its ungated ones, and a chunk that holds the whole sequence.
+of the same number of weights as its ungated ones, and a chunk that holds the whole sequence.  Pugozen runs beside a Nalizen
+model with dense feed-forwards of as many weights: window attention (a window that holds the sequence) where Pugozen has
+attention beside a delta rule, HGRN2 of equal heads where it has a recurrence alone.
 
-    python bench.py --workload golulix|faledra|nalizen [--design-size small|large|both]
+    python bench.py --workload golulix|faledra|nalizen|pugozen [--design-size small|large|both]
     python -m shai_amd.bench.decoder_design --design faledra --model faledra --size small --batch 64      # profiling
 """
 from __future__ import annotations
@@ -28,6 +30,11 @@ FALEDRA_SIZES = {"small": (2048, 6, 2, 16, 128, 64, 128, 768, 512, 2048, 8448, 3
 NALIZEN_SIZES = {"small": ("aRRSARRS", 2048, 16, 4, 128, 1024, 16, 128, 128, 8448, 64, 6, 2112, 256, 32768),
                  "large": ("aRSARS", 4096, 32, 8, 128, 4096, 32, 128, 128, 8192, 64, 4, 3072, 256, 65536)}
 
+# layers (PugozenConfig.uniform), width, heads, kv heads, head size, recurrence heads, query / key heads of the delta rule, key and
+# value size, rank of thin products, ff, vocab
+PUGOZEN_SIZES = {"small": ("DPRPDPRP", 2048, 16, 4, 128, 16, 8, 128, 128, 128, 8448, 32768),
+                 "large": ("DPRDPR", 4096, 32, 8, 128, 32, 16, 128, 128, 128, 12288, 65536)}
+
 
 def configs(size: str, design: str = "golulix"):
     from ..models.llama import LlamaConfig
@@ -36,6 +43,13 @@ def configs(size: str, design: str = "golulix"):
         from ..models.faledra import FaledraConfig
         D, A, R, H, d, rot, dv, q, kv, gru, ff, V, G = FALEDRA_SIZES[size]
         cfg, L, inner = FaledraConfig.uniform(A, R, D, H, d, rot, dv, q, kv, gru, ff, V), A + R, 2 * ff // 3
+    elif design == "pugozen":
+        from ..models.nalizen import NalizenConfig
+        from ..models.pugozen import PugozenConfig
+        kinds, D, H, G, d, sh, _, sd, sv, _, ff, V = PUGOZEN_SIZES[size]
+        cfg, L, inner = PugozenConfig.uniform(*PUGOZEN_SIZES[size]), len(kinds), 2 * ff // 3
+        out["nalizen"] = NalizenConfig.uniform("".join("a" if k.upper() == "P" else "r" for k in kinds), D, H, G, d, 1 << 20, sh,
+                                               sd, sv, inner, 1, 1, 64, 64, V)
     elif design == "nalizen":
         from ..models.golulix import GolulixConfig
         from ..models.nalizen import NalizenConfig
@@ -111,7 +125,9 @@ def bench(args, rank: int, world: int) -> dict:
                                   f"{FALEDRA_SIZES[n][:-1]}",
              "nalizen": lambda n: f"Nalizen {n}: (layers, width, heads, kv heads, head size, window, recurrence heads, key and "
                                   f"value size, dense ff, experts, top, expert ff, token input, vocab) = "
-                                  f"{NALIZEN_SIZES[n]}"}[design](last["size"])
+                                  f"{NALIZEN_SIZES[n]}",
+             "pugozen": lambda n: f"Pugozen {n}: (layers, width, heads, kv heads, head size, recurrence heads, query / key heads "
+                                  f"of the delta rule, key and value size, rank, ff, vocab) = {PUGOZEN_SIZES[n]}"}[design](last["size"])
     return {"metric": f"{design.capitalize()} decode tokens/s (random weights, beside a Llama model of equal size)",
             "value": last[design]["decode_tok_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps, "warmup": 1,
             "ms_per_step": round(1000 * (time.perf_counter() - t0) / (sum(len(configs(r['size'], design)) for r in rows) * (steps + 1)), 2),
@@ -123,8 +139,8 @@ def bench(args, rank: int, world: int) -> dict:
 
 def main(argv=None):
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=["golulix", "faledra", "nalizen"], default="golulix")
-    ap.add_argument("--model", choices=["design", "golulix", "faledra", "nalizen", "llama"], default="design")
+    ap.add_argument("--design", choices=["golulix", "faledra", "nalizen", "pugozen"], default="golulix")
+    ap.add_argument("--model", choices=["design", "golulix", "faledra", "nalizen", "pugozen", "llama"], default="design")
     ap.add_argument("--size", choices=sorted(SIZES), default="small")
     ap.add_argument("--batch", type=int, default=64)
     ap.add_argument("--prompt", type=int, default=1024)

@@ -65,6 +65,15 @@ class PugozenConfig:
         size)."""
         entries = d["layers"]
 
+        def own(i, x):
+            """The layer whose tensors layer i uses, if not its own."""
+            j = x.get("weights_of")
+            for _ in entries:
+                if j is None or not 0 <= int(j) < len(entries) or entries[int(j)].get("weights_of") is None:
+                    return None if j is None else int(j)
+                j = entries[int(j)]["weights_of"]
+            raise ValueError(f"layer {i}: no layer has its weights")
+
         def rule(m, **kw):
             return DeltaRuleConfig(int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"]), int(m["conv"]), **kw)
 
@@ -79,10 +88,10 @@ class PugozenConfig:
                 return rule(m)
             if kind != "parallel":
                 raise ValueError(f"unknown mixer type {kind!r}")
-            a, r, own = m["left"], m["right"], x.get("weights_of")
+            a, r, j = m["left"], m["right"], own(i, x)
             if int(a["vdim"]) != int(a["dim"]):
                 raise ValueError(f"layer {i}: values are the projected keys, so vdim must be dim")
-            at = f"l{i if own is None else int(own)}.mix.right."
+            at = f"l{i if j is None else j}.mix.right."
             ranks = tuple(int(shapes[at + n][0]) if shapes and at + n in shapes else int(r["dim"]) for n in ("a1", "g1"))
             return (TiedAttentionConfig(int(a["heads"]), int(a["kv_heads"]), int(a["dim"]), float(a["scale"]),
                                         int(a["rot"]["dims"]), float(a["rot"]["base"]), float(m["left_scale"])),
@@ -96,10 +105,9 @@ class PugozenConfig:
             return int(m["ff"])
 
         eos = d.get("eos_token_id")
-        own = lambda x: None if x.get("weights_of") is None else int(x["weights_of"])
         return PugozenConfig(
             vocab_size=int(d["vocab"]), width=int(d["width"]),
-            layers=[PugozenLayerConfig(mixer(i, x), ff(x.get("mlp")), own(x)) for i, x in enumerate(entries)],
+            layers=[PugozenLayerConfig(mixer(i, x), ff(x.get("mlp")), own(i, x)) for i, x in enumerate(entries)],
             eps=float(d["norm"]["eps"]), embed_scale=float(d["embedding"]["scale"]),
             bos_token_id=int(d.get("bos_token_id") or 0), eos_token_id=int(eos) if eos is not None else None)
 

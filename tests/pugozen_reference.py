@@ -3,6 +3,7 @@ Shares no code with ``shai_amd``: tests compare the framework with it.
 
 ``cfg`` is the parsed config.json, ``w`` a dict of full tensors under their checkpoint names.  A whole sequence is
 recomputed from its first token, so there is no cache, no batch and no state to get wrong."""
+import copy
 import json
 import os
 
@@ -192,15 +193,15 @@ def parallel_layer(heads=6, kv_heads=2, dim=20, base=60.0, dims=12, scale=0.3, r
     return {"type": "parallel", "mixer": m, "mlp": mlp and dict(mlp)}
 
 
-def again(layers, j):
-    """A layer with layer j's weights."""
-    return dict(layers[j], weights_of=j)
+def again(layer, j):
+    """A layer like ``layer``, layer j, with its weights."""
+    return dict(copy.deepcopy(layer), weights_of=j)
 
 
 def random_config(layers=None, vocab=97, width=56, embed_scale=2.5, eps=1e-4):
     if layers is None:
         layers = [parallel_layer(), delta_layer(), retention_layer()]
-        layers += [again(layers, 0), again(layers, 1)]
+        layers += [again(layers[0], 0), again(layers[1], 1)]
     return {"architecture": "Pugozen", "vocab": vocab, "width": width, "norm": {"eps": eps},
             "embedding": {"scale": embed_scale}, "layers": layers}
 
