@@ -295,13 +295,15 @@ struct RuleArgs {          // delta rule (mode 1: a decay per head, 2: per key c
   const int* q_start;      // [B], null: one row per sequence (decode)
   const int* q_lens;
   const int* slots;        // [B], -1: none
-  void* ws;                // chunks: [T / 32 + B, heads] prepared chunks
+  void* ws;                // chunks: ws_chunks = T / 32 + B prepared chunks (rule_chunk_bytes each)
+  long ws_chunks;
   int T, B, H, G, dk, dv, dim, vdim, taps, rot, gate_kind, max_q, head0, heads;
   float eps;
 };
 void launch_rule_rows(const RuleArgs& a, bool f32, hipStream_t s);     // row by row
 void launch_rule_chunks(const RuleArgs& a, hipStream_t s);             // bf16, 32 rows at a time; heads head0 .. of a prefill step
-long rule_chunk_bytes(int dk, int dv);                                 // workspace of one chunk of one head
+// workspace of one chunk of `heads` heads and `keys` heads of queries and keys (those of every head with a decay per channel)
+long rule_chunk_bytes(int dk, int dv, int heads, int keys);
 
 struct RingArgs {          // the last inputs of a prefill step into the rings
   const void* x;

@@ -8,17 +8,17 @@
 //
 // rows     row by row, S in registers, convolution to gate in one launch: decode steps of both formats (bound by the state's
 //          traffic) and fp32 prompts.
-// chunks   bf16 prompts in chunks of 32 rows, two launches.  With B_t the product of the decays up to row t of a chunk,
+// chunks   bf16 prompts in chunks of 32 rows, three launches.  With B_t the product of the decays up to row t of a chunk,
 //            A[t, s] = b_t sum_d k_t k_s B_t / B_s (s < t),   P[t, s] = sum_d q_t k_s B_t / B_s (s <= t),
 //            U = (I + A)^-1 diag(b) (V - (B K) S),   O = (B Q) S + P U,   S' = B_end S + (K B_end / B)^T U.
-//          prep (a workgroup per chunk and head, all at once): convolution, norms, decays, the two score matrices, the inverse,
-//          and every operand of the second launch in the order its lanes load it.
-//          scan (a workgroup per sequence and head): chunk after chunk, each wave its columns of S (registers); operands are
-//          loaded one chunk ahead, straight into registers.
+//          prep (a workgroup per chunk and head of queries and keys, all at once): convolution, norms, decays per channel, the
+//          two score matrices, and the operands of the scan in the order its lanes load them.
+//          solve (a wave per chunk and head): the inverse, and decays per head.
+//          scan (a workgroup per sequence and head): chunk after chunk, each wave 16 columns of S (registers); prepared
+//          chunks are loaded to LDS one ahead.
 //          Quotients of decays come from differences of running logarithms.  A decay per channel enters the matrix products
-//          through a reference row that lies between the two rows (the end of a 16-row half or of an 8-row block), so both
-//          factors are at most 1; rows of one 8-row block are multiplied out one by one in fp32.  Operands of matrix products
-//          are a bf16 value plus its bf16 remainder; sums are fp32.
+//          through a reference between the two rows: the border of the 16-row halves, that of a half's 8-row blocks, or a
+//          block's fourth row.  Operands of matrix products are a bf16 value plus its bf16 remainder; sums are fp32.
 #include "matrix_state.h"
 
 namespace shai_lm {
@@ -27,12 +27,12 @@ constexpr int kRetention = 0, kHead = 1, kChannel = 2;     // decay: fixed; per 
 constexpr float kLeast = -40.f;                            // base-2 logarithm of a decay that leaves nothing in fp32
 
 __device__ __forceinline__ float softplus_exact(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
-// base-2 logarithm of exp(-rate softplus(x))
-__device__ __forceinline__ float log_decay(float x, float rate) {
+// base-2 logarithm of exp(-rate softplus(x)), limited
+__device__ __forceinline__ float log_decay(float x, float rate, float least) {
   const float e = __builtin_amdgcn_exp2f(-fabsf(x) * kInvLn2);
   const float series = e * (1.f - e * (0.5f - e * (1.f / 3.f - e * (0.25f - e * 0.2f)))) * kInvLn2;
   const float sp = fmaxf(x, 0.f) * kInvLn2 + (e < 0.03f ? series : __builtin_amdgcn_logf(1.f + e));
-  return fmaxf(-rate * sp, kLeast);
+  return fmaxf(-rate * sp, least);
 }
 template <bool FAST>
 __device__ __forceinline__ float gate_act(float z, int kind) {
@@ -235,40 +235,280 @@ void launch_ring_commit(const RingArgs& a, bool f32, hipStream_t s) {
 
 // ------------------------------------------------------------------------------------------------ 32 rows at a time
 constexpr int kC = 32;
-// A prepared chunk of one head, in 16-byte units: fragments are [64 lanes] of 16 bytes, values and remainders one after the
-// other.  Row operands (time x channels, u: rows 16 u ..): a lane holds channels 32 i + 4 g .. and 32 i + 16 + 4 g .. of its row;
-// column operands (channels x time) and score operands (time x time): times 4 g .. and 16 + 4 g ...
-template <int DK, int DV>
-struct Unit {
-  static constexpr int NI = DK / 32, NK = DK / 16, ND = DV / 16;
+// Prepared chunks, in 16-byte units: fragments are [64 lanes] of 16 bytes, values and remainders one after the other.  Row
+// operands (time x channels, u: rows 16 u ..): a lane holds channels 32 i + 4 g .. and 32 i + 16 + 4 g .. of its row; column
+// operands (channels x time) and score operands (time x time): times 4 g .. and 16 + 4 g ...
+// Rows: one per head with a decay per channel (decays applied), else one per key head (the scan applies the decays).
+template <int DK>
+struct RowUnit {
+  static constexpr int NI = DK / 32, NK = DK / 16;
   static constexpr int kd = 0;                               // B K     [u 2][i NI][2][64]
-  static constexpr int qd = kd + 2 * NI * 128;               // B Q     the same
+  static constexpr int qd = kd + 2 * NI * 128;               // B Q     the same (retention starts here)
   static constexpr int ke = qd + 2 * NI * 128;               // K B_end / B  [i NK][2][64]
-  static constexpr int tf = ke + NK * 128;                   // (I + A)^-1 diag(b)  [u 2][2][64]
-  static constexpr int pf = tf + 256;                        // P
-  static constexpr int vf = pf + 256;                        // V: [u 2][d ND][64 lanes] of 4 rows x 1 column, 8 bytes
-  static constexpr int dec = vf + ND * 64;                   // B_end [DK]
-  static constexpr int size = dec + DK / 4;
+  static constexpr int size = ke + NK * 128;
 };
+template <int DV>
+struct HeadUnit {
+  static constexpr int ND = DV / 16;
+  static constexpr int tf = 0;                               // (I + A)^-1 diag(b)  [u 2][2][64]
+  static constexpr int pf = tf + 256;                        // P (retention starts here)
+  static constexpr int vf = pf + 256;                        // V: [u 2][d ND][64 lanes] of 4 rows x 1 column, 8 bytes
+  static constexpr int dec = vf + ND * 64;                   // floats: B_end [DK], or B [32], B_end / B [32], B_end
+  static constexpr int size = dec + 64;
+};
+// Scores before the solve, fp32 [2][32][32]: A and P (a decay per channel), or k k^T and q k^T.
+constexpr int kScores = 512;
 // chunks of earlier sequences never reach the next one's first
 __device__ __forceinline__ long first_chunk(const RuleArgs& p, int b) { return p.q_start[b] / kC + b; }
 
-long rule_chunk_bytes(int dk, int dv) { return 16L * (dk * 24 + 512 + dv * 4 + dk / 4); }
+__device__ __forceinline__ uint4_* head_unit(const RuleArgs& p, long chunk, int head, int size) {
+  return static_cast<uint4_*>(p.ws) + (chunk * p.heads + head) * size;
+}
+// behind all head units; then the scores
+__device__ __forceinline__ uint4_* row_unit(const RuleArgs& p, long chunk, int key, int keys, int size, int head_size) {
+  return static_cast<uint4_*>(p.ws) + p.ws_chunks * p.heads * head_size + (chunk * keys + key) * size;
+}
+__device__ __forceinline__ float* score_unit(const RuleArgs& p, long chunk, int key, int keys, int size, int head_size) {
+  return reinterpret_cast<float*>(static_cast<uint4_*>(p.ws) + p.ws_chunks * (p.heads * (long)head_size + keys * (long)size) +
+                                  (chunk * keys + key) * kScores);
+}
 
-template <int MODE, int DK, int DV, int KT>
-__global__ void __launch_bounds__(256) rule_prep_kernel(const RuleArgs p) {
-  using U = Unit<DK, DV>;
-  constexpr bool DELTA = MODE != kRetention;
-  constexpr int LD = DK + 4, LS = 36, VQ = DK / 8, VV = DV / 8;
-  static_assert(U::size * 16 == 16 * (DK * 24 + 512 + DV * 4 + DK / 4), "chunk size");
+long rule_chunk_bytes(int dk, int dv, int heads, int keys) {
+  return 16L * ((long)keys * (dk * 24 + kScores) + (long)heads * (512 + dv * 4 + 64));
+}
+
+// ---- inputs of 4 rows x 8 channels
+// Channels ch .. of rows r0 .. r0 + 3 of a chunk after their convolution and silu; rows behind the last live one are zero.
+// `x`: the chunk's first row, row `at` of the step; before the step's first row the ring's inputs count.
+__device__ __forceinline__ void conv_rows(const RuleArgs& p, const bf16_t* x, int ch, int channels, int r0, int at, int live,
+                                          int pos0, int slot, float (&y)[4][8]) {
+  const bf16_t* ring = static_cast<const bf16_t*>(p.ring) + (long)max(slot, 0) * p.taps * channels + ch;
+  const int ring0 = pos0 % p.taps;
+  auto input = [&](int r) {                       // (rows behind the last one repeat it: their results are dropped)
+    if (at + r >= 0) return *reinterpret_cast<const uint4_*>(x + (long)min(r, live - 1) * p.ldx + ch);
+    const int m = ring0 + at + r;
+    if (at + r > -p.taps && pos0 + at + r >= 0 && slot >= 0)
+      return *reinterpret_cast<const uint4_*>(ring + (long)(m < 0 ? m + p.taps : m) * channels);
+    return uint4_{0u, 0u, 0u, 0u};
+  };
+  auto tap = [&](int j, float (&wt)[8]) {         // of the input j rows before
+    const float* cw = p.conv + (long)(p.taps - 1 - min(j, p.taps - 1)) * channels + ch;
+    const float on = j < p.taps ? 1.f : 0.f;
+    *reinterpret_cast<float4_*>(wt) = load4(cw) * on;
+    *reinterpret_cast<float4_*>(wt + 4) = load4(cw + 4) * on;
+  };
+#pragma unroll
+  for (int r = 0; r < 4; ++r)
+#pragma unroll
+    for (int i = 0; i < 8; ++i) y[r][i] = 0.f;
+  if (p.taps <= 4) {
+    uint4_ in[7];
+    float wt[4][8];
+#pragma unroll
+    for (int i = 0; i < 7; ++i) in[i] = input(r0 + i - 3);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) tap(j, wt[j]);
+#pragma unroll
+    for (int i = 0; i < 7; ++i) {
+      float f[8];
+      unpack8(in[i], f);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int j = r - i + 3;
+        if (j >= 0 && j < 4) {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) y[r][e] += wt[j < 0 || j > 3 ? 0 : j][e] * f[e];
+        }
+      }
+    }
+  } else {
+    for (int j = 0; j < p.taps; ++j) {
+      float wt[8];
+      tap(j, wt);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        float f[8];
+        unpack8(input(r0 + r - j), f);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) y[r][i] += wt[i] * f[i];
+      }
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < 4; ++r)
+#pragma unroll
+    for (int i = 0; i < 8; ++i) y[r][i] = r0 + r < live ? silu_fast(y[r][i]) : 0.f;
+}
+
+// the same without a convolution: channels d0 .. of the head at x, turned where `rope` is given
+__device__ __forceinline__ void turn_rows(const RuleArgs& p, const bf16_t* x, int d0, int r0, int live, const float* rope,
+                                          float (&y)[4][8]) {
+  const int half = p.rot >> 1;
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int t = r0 + r;
+    const bf16_t* row = x + (long)min(t, live - 1) * p.ldx;
+    unpack8(t < live ? *reinterpret_cast<const uint4_*>(row + d0) : uint4_{0u, 0u, 0u, 0u}, y[r]);
+    if (rope && d0 < p.rot && t < live) {
+      const float* a = rope + (long)t * p.rot;
+      if ((half & 7) == 0) {                      // the partners are 8 consecutive channels too
+        const bool low = d0 < half;
+        const float* cs = a + 2 * (low ? d0 : d0 - half);
+        float o[8];
+        unpack8(*reinterpret_cast<const uint4_*>(row + (low ? d0 + half : d0 - half)), o);
+#pragma unroll
+        for (int i = 0; i < 8; i += 2) {
+          const float4_ c = load4(cs + 2 * i);
+          y[r][i] = y[r][i] * c[0] + (low ? -o[i] : o[i]) * c[1];
+          y[r][i + 1] = y[r][i + 1] * c[2] + (low ? -o[i + 1] : o[i + 1]) * c[3];
+        }
+      } else {
+        for (int i = 0; i < 8; ++i) {
+          const int d = d0 + i;
+          if (d < p.rot) {
+            const bool low = d < half;
+            const float o = bf2f(row[low ? d + half : d - half]);
+            const float* cs = a + 2 * (low ? d : d - half);
+            y[r][i] = y[r][i] * cs[0] + (low ? -o : o) * cs[1];
+          }
+        }
+      }
+    }
+  }
+}
+
+// factor that makes a row of y (VQ lanes of 8 channels each) a unit vector, times dim^-1/2 for queries
+template <int VQ>
+__device__ __forceinline__ float unit_factor(const float (&y)[8], bool query, int dim) {
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) ss += y[i] * y[i];
+#pragma unroll
+  for (int d = 1; d < VQ; d <<= 1) ss += __shfl_xor(ss, d, 64);
+  return __builtin_amdgcn_rsqf(query ? (ss + 1e-6f) * (float)dim : ss + 1e-6f);
+}
+
+// values of rows 4 rg .., columns 8 vec ..
+template <int DV>
+__device__ __forceinline__ void put_values(uint4_* unit, int rg, int vec, const float (&y)[4][8]) {
+  uint2_* dst = reinterpret_cast<uint2_*>(unit + HeadUnit<DV>::vf) + ((rg >> 2) * HeadUnit<DV>::ND + (vec >> 1)) * 64 +
+                (rg & 3) * 16 + (vec & 1) * 8;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) dst[i] = uint2_{pack2(y[0][i], y[1][i]), pack2(y[2][i], y[3][i])};
+}
+
+// ---- decay per channel: a row's logarithm is kept relative to the fourth row of its 8-row block (c), so that
+// 2^c and 2^-c stay in range (rows forget 2^-24 at most); what lies between two blocks, or a block and a border, is one factor
+// per channel.  `fac`: [0 + j] start of the chunk to block j, [4 + j] block j to the chunk's end, [8 + j] block j to or from the
+// border of the halves, [12 + j] to or from the border of the half's two blocks.
+constexpr float kLeastChannel = -24.f;
+
+// One decay per head, or a fixed one: a workgroup prepares a chunk's queries and keys, their products, and the values of the
+// heads that share them.  Queries and keys lie in LDS as values and remainders, as the matrix products read them.
+template <bool DELTA, int DK, int DV>
+__global__ void __launch_bounds__(512, 4) rule_prep_head_kernel(const RuleArgs p) {
+  using U = RowUnit<DK>;
+  using HU = HeadUnit<DV>;
+  constexpr int NT = 512, LD = DK + 8, VQ = DK / 8, VV = DV / 8;
+  extern __shared__ __attribute__((aligned(16))) bf16_t planes[];
+  bf16_t* sq = planes;                            // [2][32][LD] values, remainders
+  bf16_t* sk = sq + 2 * kC * LD;
+  const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int group = p.H / p.G, keys = p.heads / group;
+  const int b = blockIdx.z, key = p.head0 / group + blockIdx.y, at = blockIdx.x * kC;
+  const int total = p.q_lens[b];
+  if (at >= total) return;
+  const int live = min(kC, total - at);
+  const long row0 = p.q_start[b] + at;
+  const int slot = p.slots[b], pos0 = p.pos[p.q_start[b]];
+  const int channels = 2 * p.G * DK + p.H * DV;
+  const bf16_t* x = static_cast<const bf16_t*>(p.x) + row0 * p.ldx;
+  const long chunk = first_chunk(p, b) + blockIdx.x;
+  uint4_* rows = row_unit(p, chunk, blockIdx.y, keys, U::size, HU::size);
+  float* scores = score_unit(p, chunk, blockIdx.y, keys, U::size, HU::size);
+  auto head = [&](int j) { return head_unit(p, chunk, blockIdx.y * group + j, HU::size); };
+
+  // ---- inputs: a task is 4 rows x 8 channels of q, k or a head's v
+  for (int id = tid; id < 2 * DK + group * DV; id += NT) {
+    const int what = id < DK ? 0 : id < 2 * DK ? 1 : 2, e = id - what * DK;
+    const int vec = what < 2 ? e % VQ : e % VV, rg = what < 2 ? e / VQ : e / VV % 8, j = what < 2 ? 0 : e / DV;
+    const int first = what < 2 ? (what * p.G + key) * DK : 2 * p.G * DK + (key * group + j) * DV;
+    float y[4][8];
+    if constexpr (DELTA) conv_rows(p, x, first + 8 * vec, channels, 4 * rg, at, live, pos0, slot, y);
+    else turn_rows(p, x + first, 8 * vec, 4 * rg, live, what < 2 ? p.rope + row0 * p.rot : nullptr, y);
+    if (what < 2) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float scale = DELTA ? unit_factor<VQ>(y[r], what == 0, p.dim) : what ? __builtin_amdgcn_rsqf((float)p.dim) : 1.f;
+        const Split f = split8(float4_{y[r][0], y[r][1], y[r][2], y[r][3]} * scale,
+                               float4_{y[r][4], y[r][5], y[r][6], y[r][7]} * scale);
+        bf16_t* dst = (what ? sk : sq) + (4 * rg + r) * LD + 8 * vec;
+        *reinterpret_cast<bf16x8*>(dst) = f.hi;
+        *reinterpret_cast<bf16x8*>(dst + kC * LD) = f.lo;
+      }
+    } else {
+      put_values<DV>(head(j), rg, vec, y);
+    }
+  }
+  __syncthreads();
+
+  // ---- k k^T and q k^T: tiles (rows 16 .., keys 0 ..), (0, 0), (16, 16) by a wave each
+  const int g = lane >> 4, c16 = lane & 15;
+  if (w < 6 && (DELTA || (w & 1))) {
+    const int tile = w >> 1, tr = tile == 1 ? 0 : 16, tc = tile == 2 ? 16 : 0;
+    const bf16_t* left = ((w & 1) ? sq : sk) + (tr + c16) * LD + 8 * g;
+    const bf16_t* right = sk + (tc + c16) * LD + 8 * g;
+    auto frag = [&](const bf16_t* m) {
+      return Split{*reinterpret_cast<const bf16x8*>(m), *reinterpret_cast<const bf16x8*>(m + kC * LD)};
+    };
+    float4_ acc = float4_{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < U::NI; ++i) acc = mac(frag(left + 32 * i), frag(right + 32 * i), acc);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) scores[(w & 1) * 1024 + (tr + 4 * g + j) * 32 + tc + c16] = acc[j];
+  }
+  {                                               // queries and keys as operands
+    constexpr int NR = 2 * U::NI;
+    for (int f = (DELTA ? 0 : NR) + 7 - w; f < 2 * NR + U::NK; f += 8) {     // (the last waves have no scores)
+      uint4_ plane[2];
+      if (f < 2 * NR) {
+        const int i = f % NR;
+        const bf16_t* src = (f < NR ? sk : sq) + (16 * (i / U::NI) + c16) * LD + 32 * (i % U::NI) + 4 * g;
+#pragma unroll
+        for (int v = 0; v < 2; ++v) {
+          const uint2_ lo = *reinterpret_cast<const uint2_*>(src + v * kC * LD);
+          const uint2_ hi = *reinterpret_cast<const uint2_*>(src + v * kC * LD + 16);
+          plane[v] = uint4_{lo[0], lo[1], hi[0], hi[1]};
+        }
+      } else {
+        const bf16_t* src = sk + 4 * g * LD + 16 * (f - 2 * NR) + c16;
+#pragma unroll
+        for (int v = 0; v < 2; ++v)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            const bf16_t* y = src + v * kC * LD + (16 * (j >> 1) + 2 * (j & 1)) * LD;
+            plane[v][j] = (uint32_t)y[0] | (uint32_t)y[LD] << 16;
+          }
+      }
+      uint4_* dst = rows + (f < NR ? U::kd + f * 128 : f < 2 * NR ? U::qd + (f - NR) * 128 : U::ke + (f - 2 * NR) * 128);
+      dst[lane] = plane[0];
+      dst[64 + lane] = plane[1];
+    }
+  }
+}
+
+template <int DK, int DV>
+__global__ void __launch_bounds__(512, 4) rule_prep_channel_kernel(const RuleArgs p) {
+  using U = RowUnit<DK>;
+  using HU = HeadUnit<DV>;
+  constexpr int NT = 512, LD = DK + 4, VQ = DK / 8, VV = DV / 8;
   extern __shared__ __attribute__((aligned(16))) float lds[];
-  float* sq = lds;                                // [32][LD]
-  float* sk = sq + kC * LD;
-  float* sA = sk + kC * LD;                       // [32][LS]
-  float* sP = sA + kC * LS;
-  float* sT = sP + kC * LS;
-  float* sbeta = sT + kC * LS;                    // [32]
-  float* sb = sbeta + kC;                         // running logarithms: [32], or [32][LD] per channel
+  float* sq = lds;                                // [32][LD] q, then q 2^c
+  float* sk = sq + kC * LD;                       // [32][LD] k, then k 2^c
+  float* sbeta = sk + kC * LD;                    // [32]
+  float* sb = sbeta + kC;                         // [32][LD] c, then k 2^-c
+  float* sref = sb + kC * LD;                     // logarithms at the blocks' fourth rows [4][DK] and ends [4][DK]
+  float* fac = sref + 8 * DK;                     // [16][DK]
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int b = blockIdx.z, h = p.head0 + blockIdx.y, at = blockIdx.x * kC;
   const int total = p.q_lens[b];
@@ -278,487 +518,490 @@ __global__ void __launch_bounds__(256) rule_prep_kernel(const RuleArgs p) {
   const int slot = p.slots[b], pos0 = p.pos[p.q_start[b]];
   const int grp = h / (p.H / p.G), channels = 2 * p.G * DK + p.H * DV;
   const bf16_t* x = static_cast<const bf16_t*>(p.x) + row0 * p.ldx;
-  const bf16_t* ring = DELTA ? static_cast<const bf16_t*>(p.ring) + (long)max(slot, 0) * p.taps * channels : nullptr;
-  uint4_* unit = static_cast<uint4_*>(p.ws) + ((first_chunk(p, b) + blockIdx.x) * p.heads + blockIdx.y) * U::size;
+  const long chunk = first_chunk(p, b) + blockIdx.x;
+  uint4_* head = head_unit(p, chunk, blockIdx.y, HU::size);
+  uint4_* rows = row_unit(p, chunk, blockIdx.y, p.heads, U::size, HU::size);
+  float* scores = score_unit(p, chunk, blockIdx.y, p.heads, U::size, HU::size);
 
   // ---- inputs: a task is 4 rows x 8 channels of q, k or v
-  for (int id = tid; id < 2 * DK + DV; id += 256) {
+  for (int id = tid; id < 2 * DK + DV; id += NT) {
     const int what = id < DK ? 0 : id < 2 * DK ? 1 : 2, e = id - what * DK;
     const int vec = what < 2 ? e % VQ : e % VV, rg = what < 2 ? e / VQ : e / VV;
-    const int ch = 8 * vec + (what == 2 ? 2 * p.G * DK + h * DV : (DELTA ? what * p.G + grp : what * p.H + h) * DK);
+    const int ch = 8 * vec + (what == 2 ? 2 * p.G * DK + h * DV : (what * p.G + grp) * DK);
     float y[4][8];
-    if constexpr (DELTA) {
-      float wt[KT][8];
-#pragma unroll
-      for (int j = 0; j < KT; ++j) {
-        const float* cw = p.conv + (long)(p.taps - 1 - min(j, p.taps - 1)) * channels + ch;
-        const float4_ lo = load4(cw), hi = load4(cw + 4);
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          wt[j][i] = j < p.taps ? lo[i] : 0.f;
-          wt[j][4 + i] = j < p.taps ? hi[i] : 0.f;
-        }
-      }
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-#pragma unroll
-        for (int i = 0; i < 8; ++i) y[r][i] = 0.f;
-#pragma unroll
-      for (int i = 1 - KT; i < 4; ++i) {
-        const int r = 4 * rg + i, step = at + r, pos = pos0 + step;          // row of the chunk, of the step, position
-        const bf16_t* src = nullptr;
-        if (r < live && i > -p.taps) {
-          if (step >= 0) src = x + (long)r * p.ldx + ch;
-          else if (pos >= 0 && slot >= 0) src = ring + (long)(pos % p.taps) * channels + ch;
-        }
-        float f[8];
-        unpack8(src ? *reinterpret_cast<const uint4_*>(src) : uint4_{0u, 0u, 0u, 0u}, f);
-#pragma unroll
-        for (int rr = 0; rr < 4; ++rr)
-          if (rr - i >= 0 && rr - i < KT) {
-#pragma unroll
-            for (int j = 0; j < 8; ++j) y[rr][j] += wt[rr - i][j] * f[j];
-          }
-      }
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-#pragma unroll
-        for (int i = 0; i < 8; ++i) y[r][i] = 4 * rg + r < live ? silu_fast(y[r][i]) : 0.f;
-    } else {
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = 4 * rg + r;
-        unpack8(t < live ? *reinterpret_cast<const uint4_*>(x + (long)t * p.ldx + ch) : uint4_{0u, 0u, 0u, 0u}, y[r]);
-        if (what < 2 && 8 * vec < p.rot && t < live) {
-          const int half = p.rot >> 1;
-          const bf16_t* head = x + (long)t * p.ldx + ch - 8 * vec;
-          const float* a = p.rope + (row0 + t) * p.rot;
-#pragma unroll
-          for (int i = 0; i < 8; ++i) {
-            const int d = 8 * vec + i;
-            if (d < p.rot) {
-              const bool low = d < half;
-              const float other = bf2f(head[low ? d + half : d - half]);
-              const float* cs = a + 2 * (low ? d : d - half);
-              y[r][i] = y[r][i] * cs[0] + (low ? -other : other) * cs[1];
-            }
-          }
-        }
-      }
-    }
+    conv_rows(p, x, ch, channels, 4 * rg, at, live, pos0, slot, y);
     if (what < 2) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        float scale = what ? 1.f / sqrtf((float)p.dim) : 1.f;
-        if constexpr (DELTA) {
-          float ss = 0.f;
-#pragma unroll
-          for (int i = 0; i < 8; ++i) ss += y[r][i] * y[r][i];
-#pragma unroll
-          for (int d = 1; d < VQ; d <<= 1) ss += __shfl_xor(ss, d, 64);
-          scale = 1.f / sqrtf(ss + 1e-6f) * (what ? 1.f : 1.f / sqrtf((float)p.dim));
-        }
+        const float scale = unit_factor<VQ>(y[r], what == 0, p.dim);
         float* dst = (what ? sk : sq) + (4 * rg + r) * LD + 8 * vec;
         store4(dst, float4_{y[r][0], y[r][1], y[r][2], y[r][3]} * scale);
         store4(dst + 4, float4_{y[r][4], y[r][5], y[r][6], y[r][7]} * scale);
       }
     } else {
-      uint2_* dst = reinterpret_cast<uint2_*>(unit + U::vf);
-#pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        const int col = 8 * vec + i;
-        dst[((rg >> 2) * U::ND + (col >> 4)) * 64 + (rg & 3) * 16 + (col & 15)] =
-            uint2_{pack2(y[0][i], y[1][i]), pack2(y[2][i], y[3][i])};
-      }
+      put_values<DV>(head, rg, vec, y);
     }
   }
 
-  // ---- write strengths and running logarithms of the decays
-  if constexpr (DELTA) {
-    if (tid >= 64 && tid < 96) {
-      const int t = tid - 64;
-      sbeta[t] = t < live ? sigmoid_f(p.beta[(row0 + t) * p.ldb + h]) : 0.f;
-    }
-  }
-  if constexpr (MODE == kRetention) {
-    if (tid < kC) sb[tid] = (float)min(tid + 1, live) * fmaxf(p.rate[p.H + h], kLeast);
-  } else if constexpr (MODE == kHead) {
-    if (tid < 64) {                               // whole wave: lanes 32 .. take part in the shuffles
-      const int t = tid & 31;
-      float lg = t < live ? log_decay(p.decay[(row0 + min(t, live - 1)) * p.ldd + h] + p.bias[h], p.rate[h]) : 0.f;
+  // ---- write strengths and running logarithms of the decays (by the waves with the fewest tasks)
+  if (tid < kC) sbeta[tid] = tid < live ? sigmoid_f(p.beta[(row0 + tid) * p.ldb + h]) : 0.f;
+  {
+    const int d = tid - (NT - DK);
+    if (d >= 0) {
+      const float bias = p.bias[h * DK + d], rate = p.rate[h];
+      const float* z = p.decay + row0 * p.ldd + h * DK + d;
+      float run = 0.f;
+#pragma unroll 1
+      for (int j = 0; j < 4; ++j) {
+        float lg[8];
 #pragma unroll
-      for (int d = 1; d < kC; d <<= 1) {
-        const float other = __shfl_up(lg, d, 32);
-        if (t >= d) lg += other;
+        for (int i = 0; i < 8; ++i) lg[i] = z[(long)min(8 * j + i, live - 1) * p.ldd];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          run += 8 * j + i < live ? log_decay(lg[i] + bias, rate, kLeastChannel) : 0.f;
+          lg[i] = run;
+        }
+        sref[j * DK + d] = lg[3];
+        sref[(4 + j) * DK + d] = run;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) sb[(8 * j + i) * LD + d] = lg[i] - lg[3];
       }
-      if (tid < kC) sb[tid] = lg;
     }
-  } else {
-    constexpr int RG = 256 / DK, RR = kC / RG;    // groups of rows, rows of a group
-    const int d = tid % DK, first = (tid / DK) * RR;
-    const float bias = p.bias[h * DK + d], rate = p.rate[h];
-    const float* z = p.decay + row0 * p.ldd + h * DK + d;
-    float lg[RR], run = 0.f;
-#pragma unroll
-    for (int i = 0; i < RR; ++i) lg[i] = z[(long)min(first + i, live - 1) * p.ldd];
-#pragma unroll
-    for (int i = 0; i < RR; ++i) {
-      run += first + i < live ? log_decay(lg[i] + bias, rate) : 0.f;
-      lg[i] = run;
-    }
-    if constexpr (RG > 1) {
-      sb[(tid / DK) * LD + d] = run;              // group totals, before the rows are stored
-      __syncthreads();
-      run = 0.f;
-      for (int i = 0; i < tid / DK; ++i) run += sb[i * LD + d];
-      __syncthreads();
-    } else {
-      run = 0.f;
-    }
-#pragma unroll
-    for (int i = 0; i < RR; ++i) sb[(first + i) * LD + d] = lg[i] + run;
   }
   __syncthreads();
 
-  // ---- scores: tiles (rows 16 .., keys 0 ..), (0, 0), (16, 16) by a wave each
+  // ---- q 2^c, k 2^c, k 2^-c, and the factors between blocks
+  {
+#pragma unroll 2
+    for (int id = tid; id < kC * DK / 4; id += NT) {
+      const int o = id / (DK / 4) * LD + id % (DK / 4) * 4;
+      const float4_ c = load4(sb + o), q = load4(sq + o), k = load4(sk + o);
+      float4_ up, dn;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        up[j] = __builtin_amdgcn_exp2f(c[j]);
+        dn[j] = __builtin_amdgcn_exp2f(-c[j]);
+      }
+      store4(sq + o, q * up);
+      store4(sk + o, k * up);
+      store4(sb + o, k * dn);
+    }
+    for (int id = tid; id < 16 * DK; id += NT) {
+      const int kind = id / (4 * DK), j = id / DK & 3, d = id % DK;
+      const float r = sref[j * DK + d];
+      const float m = sref[(kind == 1 ? 7 : kind == 2 ? 5 : j < 2 ? 4 : 6) * DK + d];
+      const bool to = kind == 1 || (kind == 2 ? j < 2 : !(j & 1));           // from the block to the border
+      fac[id] = __builtin_amdgcn_exp2f(kind == 0 ? r : to ? m - r : r - m);
+    }
+    __syncthreads();
+  }
+
+  // ---- scores: tiles (rows 16 .., keys 0 ..), (0, 0), (16, 16), of k and of q by a wave each
   const int g = lane >> 4, c16 = lane & 15;
   const float4_ zero = float4_{0.f, 0.f, 0.f, 0.f};
-  if (w < 3) {
-    const int tr = w == 1 ? 0 : 16, tc = w == 2 ? 16 : 0;
-    const int ref = w == 2 ? 23 : w == 1 ? 7 : 15;               // reference row of the decays per channel
-    float4_ acc_a = zero, acc_p = zero;
-    auto frag = [&](const float* m, int row, int d0, int sign) {  // sign: of the row's logarithm above the reference's; 0: drop
-      float4_ lo = load4(m + row * LD + d0), hi = load4(m + row * LD + d0 + 4);
-      if constexpr (MODE == kChannel) {
-        const float4_ r0 = load4(sb + ref * LD + d0), r1 = load4(sb + ref * LD + d0 + 4);
-        const float4_ b0 = load4(sb + row * LD + d0), b1 = load4(sb + row * LD + d0 + 4);
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          lo[j] = sign ? lo[j] * __builtin_amdgcn_exp2f(sign > 0 ? b0[j] - r0[j] : r0[j] - b0[j]) : 0.f;
-          hi[j] = sign ? hi[j] * __builtin_amdgcn_exp2f(sign > 0 ? b1[j] - r1[j] : r1[j] - b1[j]) : 0.f;
-        }
-      }
-      return split8(lo, hi);
+  if (w < 6) {
+    const int tile = w >> 1, tr = tile == 1 ? 0 : 16, tc = tile == 2 ? 16 : 0;
+    const bool of_q = w & 1, late = c16 >= 8;
+    const float* left = (of_q ? sq : sk) + (tr + c16) * LD;
+    float4_ acc = zero, in = zero;
+    auto frag = [&](const float* row, int d0) { return split8(load4(row + d0), load4(row + d0 + 4)); };
+    auto scaled = [&](const float* row, const float* f, int d0) {
+      return split8(load4(row + d0) * load4(f + d0), load4(row + d0 + 4) * load4(f + d0 + 4));
     };
-    const int late = c16 >= 8;
 #pragma unroll 2
     for (int i = 0; i < U::NI; ++i) {
       const int d0 = 32 * i + 8 * g;
-      const Split kc = frag(sk, tc + c16, d0, w == 0 || !late ? -1 : 1);      // keys (a half's later rows as rows)
-      const Split qr = frag(sq, tr + c16, d0, w == 0 || late ? 1 : 0);
-      acc_p = mac(qr, kc, acc_p);
-      if constexpr (DELTA) {
-        if (w == 0) acc_a = mac(frag(sk, tr + c16, d0, 1), kc, acc_a);
-        else acc_a = mac(kc, kc, acc_a);
+      const float* dn = sb + (tc + c16) * LD;     // k 2^-c
+      if (tile == 0) {
+        acc = mac(scaled(left, fac + (10 + late) * DK, d0), scaled(dn, fac + (8 + late) * DK, d0), acc);
+      } else {
+        const float* f = fac + (12 + (tr >> 3) + late) * DK;
+        const Split keys = scaled(late ? sk + (tr + c16) * LD : dn, f, d0);
+        in = mac(frag(left, d0), frag(dn, d0), in);
+        if (of_q) {
+          Split rows = scaled(left, f, d0);
+          const bf16x8 none = __builtin_bit_cast(bf16x8, uint4_{0u, 0u, 0u, 0u});
+          rows.hi = late ? rows.hi : none;
+          rows.lo = late ? rows.lo : none;
+          acc = mac(rows, keys, acc);
+        } else {
+          acc = mac(keys, keys, acc);
+        }
       }
     }
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int t = tr + 4 * g + j, s = tc + c16;
-      if constexpr (MODE == kChannel) {
-        if (w == 0 || (4 * g + j >= 8 && !late)) {
-          sA[t * LS + s] = sbeta[t] * acc_a[j];
-          sP[t * LS + s] = acc_p[j];
-        }
-      } else if (s <= t) {
-        const float dec = __builtin_amdgcn_exp2f(sb[t] - sb[s]);
-        if constexpr (DELTA) sA[t * LS + s] = s < t ? sbeta[t] * dec * acc_a[j] : 0.f;
-        sP[t * LS + s] = dec * acc_p[j];
-      }
+      float y = tile && (t >> 3) == (s >> 3) ? in[j] : acc[j];
+      y = of_q ? y : s < t ? y * sbeta[t] : 0.f;
+      scores[of_q * 1024 + t * 32 + s] = y;
     }
-  }
-  if constexpr (MODE == kChannel) {               // pairs inside an 8-row block: a wave per block, a lane per pair
-    const int t = 8 * w + (lane >> 3), s = 8 * w + (lane & 7);
-    if (s <= t) {
-      float a = 0.f, q = 0.f;
-#pragma unroll 2
-      for (int d = 0; d < DK; d += 4) {
-        const float4_ bt = load4(sb + t * LD + d), bs = load4(sb + s * LD + d), ks = load4(sk + s * LD + d);
-        const float4_ kt = load4(sk + t * LD + d), qt = load4(sq + t * LD + d);
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const float e = ks[j] * __builtin_amdgcn_exp2f(bt[j] - bs[j]);
-          a += kt[j] * e;
-          q += qt[j] * e;
-        }
-      }
-      sA[t * LS + s] = s < t ? sbeta[t] * a : 0.f;
-      sP[t * LS + s] = q;
-    }
-  }
-  __syncthreads();
-
-  // ---- (I + A)^-1: both 16 x 16 blocks on the diagonal by columns, then the one below them
-  if constexpr (DELTA) {
-    if (w == 0) {
-      const int o = (lane >> 5) * 16, j = lane & 15;
-      float col[16];
-#pragma unroll
-      for (int t = 0; t < 16; ++t) {
-        float y = t == j ? 1.f : 0.f;
-#pragma unroll
-        for (int s = 0; s < t; ++s) y -= sA[(o + t) * LS + o + s] * col[s];
-        col[t] = y;
-      }
-      if (!(lane & 16)) {
-#pragma unroll
-        for (int t = 0; t < 16; ++t) sT[(o + t) * LS + o + j] = col[t];
-      }
-    }
-    __syncthreads();
-    const int r = tid >> 4, c = tid & 15;
-    float y = 0.f;
-#pragma unroll
-    for (int s = 0; s < 16; ++s) y += sA[(16 + r) * LS + s] * sT[s * LS + c];
-    sT[r * LS + 16 + c] = y;                      // (above the diagonal: free)
-    __syncthreads();
-    y = 0.f;
-#pragma unroll
-    for (int s = 0; s < 16; ++s) y -= sT[(16 + r) * LS + 16 + s] * sT[s * LS + 16 + c];
-    sT[(16 + r) * LS + c] = y;
-    __syncthreads();
   }
 
   // ---- operands of the scan
   auto put = [&](int place, const Split& f) {
+    rows[place + lane] = __builtin_bit_cast(uint4_, f.hi);
+    rows[place + 64 + lane] = __builtin_bit_cast(uint4_, f.lo);
+  };
+  {
+    constexpr int NR = 2 * U::NI;
+    for (int f = 7 - w; f < 2 * NR + U::NK; f += 8) {             // (the last waves have no scores)
+      if (f < 2 * NR) {                           // rows decayed from the chunk's start
+        const int i = f % NR, row = 16 * (i / U::NI) + c16, d0 = 32 * (i % U::NI) + 4 * g;
+        const float* src = (f < NR ? sk : sq) + row * LD + d0;
+        const float* e = fac + (row >> 3) * DK + d0;
+        put((f < NR ? U::kd : U::qd) + i * 128, split8(load4(src) * load4(e), load4(src + 16) * load4(e + 16)));
+      } else {                                    // keys decayed to its end, by channel
+        const int i = f - 2 * NR, ch = 16 * i + c16;
+        const float* src = sb + 4 * g * LD + ch;
+        float4_ y[2];
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) y[u][j] = src[(16 * u + j) * LD] * fac[(4 + 2 * u + (g >> 1)) * DK + ch];
+        put(U::ke + i * 128, split8(y[0], y[1]));
+      }
+    }
+  }
+  if (tid < DK) reinterpret_cast<float*>(head + HU::dec)[tid] = fac[3 * DK + tid] * fac[7 * DK + tid];
+}
+
+// The rest of a head's chunk by one wave: (I + A)^-1 diag(b), P, and the decays of its rows.  LDS: A below the diagonal, the
+// inverse's transpose above it (its diagonal is 1).
+template <int MODE, int DK, int DV>
+__global__ void __launch_bounds__(256, 4) rule_solve_kernel(const RuleArgs p) {
+  using HU = HeadUnit<DV>;
+  constexpr bool DELTA = MODE != kRetention, CHANNEL = MODE == kChannel;
+  constexpr int LS = 36;
+  __shared__ __attribute__((aligned(16))) float sm[4][DELTA ? kC * LS : 4], sb[4][kC], sbeta[4][kC];
+  const int lane = threadIdx.x & 63, w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int g = lane >> 4, c16 = lane & 15, tl = lane & 31;
+  const int b = blockIdx.z, h = p.head0 + blockIdx.y, at = (blockIdx.x * 4 + w) * kC;
+  const int total = p.q_lens[b];
+  if (at >= total) return;                        // whole waves: no barrier below
+  const int live = min(kC, total - at), group = CHANNEL ? 1 : p.H / p.G;
+  const long row = p.q_start[b] + at + min(tl, live - 1), chunk = first_chunk(p, b) + blockIdx.x * 4 + w;
+  uint4_* unit = head_unit(p, chunk, blockIdx.y, HU::size);
+  const float* scores = score_unit(p, chunk, blockIdx.y / group, p.heads / group, RowUnit<DK>::size, HU::size);
+  float* m = sm[w];
+  float* lb = sb[w];
+  float* beta = sbeta[w];
+  float a[DELTA ? 16 : 1];
+  if constexpr (DELTA) {
+#pragma unroll
+    for (int i = 0; i < 16; ++i) a[i] = scores[64 * i + lane];               // rows 2 i, 2 i + 1
+  }
+  float4_ pr[2][2];
+#pragma unroll
+  for (int u = 0; u < 2; ++u)
+#pragma unroll
+    for (int v = 0; v < 2; ++v) pr[u][v] = load4(scores + 1024 + (16 * u + c16) * 32 + 16 * v + 4 * g);
+  float lg = 0.f, bt = 0.f;
+  if constexpr (DELTA) bt = tl < live ? sigmoid_f(p.beta[row * p.ldb + h]) : 0.f;
+  if constexpr (MODE == kHead) {
+    lg = tl < live ? log_decay(p.decay[row * p.ldd + h] + p.bias[h], p.rate[h], kLeast) : 0.f;
+#pragma unroll
+    for (int d = 1; d < kC; d <<= 1) {
+      const float other = __shfl_up(lg, d, 32);
+      if (tl >= d) lg += other;
+    }
+  } else if constexpr (!CHANNEL) {
+    lg = (float)min(tl + 1, live) * fmaxf(p.rate[p.H + h], kLeast);
+  }
+  if (lane < kC) {
+    lb[tl] = lg;
+    beta[tl] = bt;
+  }
+  if constexpr (!CHANNEL) {
+    const float end = __shfl(lg, 31, 64);
+    float* dec = reinterpret_cast<float*>(unit + HU::dec);
+    dec[lane] = __builtin_amdgcn_exp2f(lane < kC ? lg : end - lg);
+    if (lane == 0) dec[64] = __builtin_amdgcn_exp2f(end);
+  }
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  auto put = [&](int place, const Split& f) {
     unit[place + lane] = __builtin_bit_cast(uint4_, f.hi);
     unit[place + 64 + lane] = __builtin_bit_cast(uint4_, f.lo);
   };
-  constexpr int NR = 2 * U::NI;
-  for (int f = w; f < 2 * NR + U::NK + 4; f += 4) {
-    if (f < 2 * NR) {                             // rows decayed from the chunk's start
-      if (!DELTA && f < NR) continue;
-      const int i = f % NR, row = 16 * (i / U::NI) + c16, d0 = 32 * (i % U::NI) + 4 * g;
-      const float* src = (f < NR ? sk : sq) + row * LD + d0;
-      float4_ lo = load4(src), hi = load4(src + 16);
-      if constexpr (MODE == kChannel) {
-        const float4_ b0 = load4(sb + row * LD + d0), b1 = load4(sb + row * LD + d0 + 16);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          lo[j] *= __builtin_amdgcn_exp2f(b0[j]);
-          hi[j] *= __builtin_amdgcn_exp2f(b1[j]);
-        }
-      } else {
-        const float e = __builtin_amdgcn_exp2f(sb[row]);
-        lo *= e;
-        hi *= e;
+  for (int u = 0; u < 2; ++u) {
+    const int t = 16 * u + c16;
+    const float l = lb[t];
+#pragma unroll
+    for (int v = 0; v < 2; ++v)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int s = 16 * v + 4 * g + i;
+        const float y = CHANNEL ? pr[u][v][i] : pr[u][v][i] * __builtin_amdgcn_exp2f(fminf(l - lb[s], 0.f));
+        pr[u][v][i] = s > t ? 0.f : y;            // (scores above the diagonal are not all written)
       }
-      put((f < NR ? U::kd : U::qd) + i * 128, split8(lo, hi));
-    } else if (f < 2 * NR + U::NK) {              // keys decayed to its end, by channel
-      const int i = f - 2 * NR, ch = 16 * i + c16;
-      float4_ y[2];
+    put(HU::pf + u * 128, split8(pr[u][0], pr[u][1]));
+  }
+  if constexpr (DELTA) {
 #pragma unroll
-      for (int u = 0; u < 2; ++u)
+    for (int i = 0; i < 16; ++i) {
+      const int t = 2 * i + (lane >> 5);
+      if (tl < t) m[t * LS + tl] = CHANNEL ? a[i] : a[i] * beta[t] * __builtin_amdgcn_exp2f(lb[t] - lg);
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    float col[16];
+    {                                             // both 16 x 16 blocks on the diagonal by columns
+      const float* blk = m + ((lane >> 5) * 16) * LS + (lane >> 5) * 16;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int t = 16 * u + 4 * g + j;
-          const float d = MODE == kChannel ? sb[31 * LD + ch] - sb[t * LD + ch] : sb[31] - sb[t];
-          y[u][j] = sk[t * LD + ch] * __builtin_amdgcn_exp2f(d);
+      for (int t = 0; t < 16; ++t) {
+        if (t % 4 == 0) __builtin_amdgcn_sched_barrier(0);                  // four rows in registers at a time
+        float y = t == c16 ? 1.f : 0.f, y2 = 0.f;
+#pragma unroll
+        for (int s = 0; s < t; ++s) {
+          const float e = blk[t * LS + s] * col[s];
+          if (s & 1) y2 -= e;
+          else y -= e;
         }
-      put(U::ke + i * 128, split8(y[0], y[1]));
-    } else {                                      // the inverse (times the write strengths) and the scores of q
-      const int i = f - 2 * NR - U::NK, u = i & 1, t = 16 * u + c16;
-      const bool inv = i < 2;
-      if (!DELTA && inv) continue;
-      float4_ y[2];
+        col[t] = y + y2;
+      }
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      float* up = m + ((lane >> 5) * 16 + c16) * LS + (lane >> 5) * 16;
+#pragma unroll
+      for (int t = 1; t < 16; ++t)
+        if (t > c16 && !(lane & 16)) up[t] = col[t];
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    {                                             // A21 T11, kept above the diagonal
+      float y[4];
+#pragma unroll
+      for (int s = 0; s < 16; ++s) col[s] = s == c16 ? 1.f : s > c16 ? m[c16 * LS + s] : 0.f;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        y[i] = 0.f;
+#pragma unroll
+        for (int s = 0; s < 16; ++s) y[i] += m[(16 + 4 * g + i) * LS + s] * col[s];
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) m[(4 * g + i) * LS + 16 + c16] = y[i];
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    {                                             // -T22 of it, transposed
+      float4_ y = float4_{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int s = 0; s < 16; ++s) {
+        const float e = s == c16 ? 1.f : s < c16 ? m[(16 + s) * LS + 16 + c16] : 0.f;
+        y -= e * load4(m + s * LS + 16 + 4 * g);
+      }
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+#pragma unroll
+      for (int i = 0; i < 4; ++i) m[(4 * g + i) * LS + 16 + c16] = y[i];
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      float4_ inv[2];
+      const int t = 16 * u + c16;
 #pragma unroll
       for (int v = 0; v < 2; ++v)
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int s = 16 * v + 4 * g + j;
-          y[v][j] = s > t ? 0.f : inv ? sT[t * LS + s] * sbeta[s] : sP[t * LS + s];
+        for (int i = 0; i < 4; ++i) {
+          const int s = 16 * v + 4 * g + i;
+          inv[v][i] = (s < t ? m[s * LS + t] : s == t ? 1.f : 0.f) * beta[s];
         }
-      put((inv ? U::tf : U::pf) + u * 128, split8(y[0], y[1]));
+      put(HU::tf + u * 128, split8(inv[0], inv[1]));
     }
   }
-  float* dec = reinterpret_cast<float*>(unit + U::dec);
-  if (tid < DK) dec[tid] = __builtin_amdgcn_exp2f(MODE == kChannel ? sb[31 * LD + tid] : sb[31]);
 }
 
-// NW waves of ND x 16 columns each; AHEAD: the next chunk's operands are loaded as soon as this one's are used up
-template <bool DELTA, int DK, int DV, int ND, bool AHEAD>
-__global__ void __launch_bounds__(DV / ND * 4, 1) rule_scan_kernel(const RuleArgs p) {
-  using U = Unit<DK, DV>;
-  constexpr int NW = DV / (16 * ND), NI = U::NI, NK = U::NK;
-  __shared__ float red[2][NW][kC];
+// x + its neighbours, inside 8 or 16 lanes
+template <int CTRL>
+__device__ __forceinline__ float add_dpp(float x) {
+  return x + __uint_as_float(__builtin_amdgcn_update_dpp(0u, __float_as_uint(x), CTRL, 0xf, 0xf, true));
+}
+template <int N>
+__device__ __forceinline__ float lanes_sum(float x) {
+  x = add_dpp<0xB1>(x);                           // quad_perm 1 0 3 2
+  x = add_dpp<0x4E>(x);                           // quad_perm 2 3 0 1
+  x = add_dpp<0x141>(x);                          // mirror of 8 lanes
+  if constexpr (N >= 16) x = add_dpp<0x140>(x);   // mirror of 16 lanes
+  if constexpr (N >= 32) x += __shfl_xor(x, 16, 64);
+  return x;
+}
+
+// Waves of 16 columns of S each.  A prepared chunk goes to LDS by DMA, one chunk ahead (AHEAD: one workgroup per CU) or while
+// another workgroup of the CU computes.
+template <int MODE, int DK, int DV, bool AHEAD>
+__global__ void __launch_bounds__(DV * 4) rule_scan_kernel(const RuleArgs p) {
+  using U = RowUnit<DK>;
+  using HU = HeadUnit<DV>;
+  constexpr bool DELTA = MODE != kRetention, CHANNEL = MODE == kChannel;
+  constexpr int NW = DV / 16, NI = U::NI, NK = U::NK, LO = DV + 4, TPR = DV / 8;
+  constexpr int FU = DELTA ? 0 : U::qd, FH = DELTA ? 0 : HU::pf;             // what retention does not use is not loaded
+  constexpr int SIZE = U::size + HU::size;
+  extern __shared__ __attribute__((aligned(16))) uint4_ staged[];
+  // [32][LO] outputs: behind the chunks or, with one, in place of its row operands (used up by then)
+  float* so = reinterpret_cast<float*>(AHEAD ? staged + 2 * SIZE : staged);
+  static_assert(kC * LO * 4 <= U::size * 16, "outputs in place of row operands");
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int g = lane >> 4, c16 = lane & 15;
-  const int b = blockIdx.y, h = p.head0 + blockIdx.x;
+  const int b = blockIdx.y, h = p.head0 + blockIdx.x, group = CHANNEL ? 1 : p.H / p.G;
   const int total = p.q_lens[b];
   if (total < 1) return;
   const int chunks = (total + kC - 1) / kC;
   const long row0 = p.q_start[b];
-  const int slot = p.slots[b], col0 = w * ND * 16 + c16;
+  const int slot = p.slots[b];
   const bool old = slot >= 0 && p.pos[row0] > 0;
-  float* st = p.state + ((long)max(slot, 0) * p.H + h) * DK * DV + col0;
+  float* st = p.state + ((long)max(slot, 0) * p.H + h) * DK * DV + 16 * w + c16;
 
-  float4_ S[NK][ND];                              // rows 16 i + 4 g .., column 16 d of the wave's
+  const int keys = p.heads / group;
+  const uint4_* head = head_unit(p, first_chunk(p, b), blockIdx.x, HU::size) + lane;
+  const uint4_* rows = row_unit(p, first_chunk(p, b), blockIdx.x / group, keys, U::size, HU::size) + lane;
+  auto stage = [&](int c) {
+    uint4_* dst = staged + (AHEAD ? (c & 1) * SIZE : 0);
+    const uint4_* su = rows + (long)c * keys * U::size;
+    for (int i = FU / 64 + w; i < U::size / 64; i += NW)
+      dma16(reinterpret_cast<const bf16_t*>(su + 64 * i), reinterpret_cast<bf16_t*>(dst + 64 * i));
+    const uint4_* sh = head + (long)c * p.heads * HU::size;
+    for (int i = FH / 64 + w; i < HU::size / 64; i += NW)
+      dma16(reinterpret_cast<const bf16_t*>(sh + 64 * i), reinterpret_cast<bf16_t*>(dst + U::size + 64 * i));
+  };
+  stage(0);
+  float4_ S[NK];                                  // rows 16 i + 4 g .., the wave's columns
 #pragma unroll
   for (int i = 0; i < NK; ++i)
 #pragma unroll
-    for (int d = 0; d < ND; ++d)
+    for (int j = 0; j < 4; ++j) S[i][j] = old ? st[(long)(16 * i + 4 * g + j) * DV] : 0.f;
+  // epilogue: a thread's row of the chunk and 8 columns
+  const int er = tid / TPR, ec = tid % TPR * 8;
+  float gain[8];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) S[i][d][j] = old ? st[(long)(16 * i + 4 * g + j) * DV + 16 * d] : 0.f;
-  float gain[ND];
-#pragma unroll
-  for (int d = 0; d < ND; ++d) gain[d] = DELTA ? p.gain[col0 + 16 * d] : 1.f;
-
-  const uint4_* unit = static_cast<const uint4_*>(p.ws) + (first_chunk(p, b) * p.heads + blockIdx.x) * U::size;
-  const long stride = (long)p.heads * U::size;
-  auto frag = [&](const uint4_* u, int place) {
-    return Split{__builtin_bit_cast(bf16x8, u[place + lane]), __builtin_bit_cast(bf16x8, u[place + 64 + lane])};
-  };
-  constexpr int A = AHEAD ? 1 : 0;
-  Split kd[A && DELTA ? 2 : 1][A && DELTA ? NI : 1], qd[A ? 2 : 1][A ? NI : 1], ke[A ? NK : 1], tf[2], pf[2];
-  uint2_ vf[2][ND];
-  auto load_rows = [&](const uint4_* u) {
-    if constexpr (AHEAD) {
-#pragma unroll
-      for (int i = 0; i < 2; ++i)
-#pragma unroll
-        for (int j = 0; j < NI; ++j) {
-          if constexpr (DELTA) kd[i][j] = frag(u, U::kd + (i * NI + j) * 128);
-          qd[i][j] = frag(u, U::qd + (i * NI + j) * 128);
-        }
-    }
-  };
-  auto load_keys = [&](const uint4_* u) {
-    if constexpr (AHEAD) {
-#pragma unroll
-      for (int i = 0; i < NK; ++i) ke[i] = frag(u, U::ke + i * 128);
-    }
-  };
-  auto load_rest = [&](const uint4_* u) {
-#pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      if constexpr (DELTA) tf[i] = frag(u, U::tf + i * 128);
-      pf[i] = frag(u, U::pf + i * 128);
-#pragma unroll
-      for (int d = 0; d < ND; ++d) vf[i][d] = reinterpret_cast<const uint2_*>(u + U::vf)[(i * U::ND + w * ND + d) * 64 + lane];
-    }
-  };
-  load_rows(unit);
-  load_rest(unit);
-  load_keys(unit);
+  for (int i = 0; i < 8; ++i) gain[i] = DELTA ? p.gain[ec + i] : 1.f;
+  const float inv_vdim = 1.f / (float)p.vdim;
+  const bf16_t* gate = static_cast<const bf16_t*>(p.gate) + row0 * p.ldg + h * DV + ec;
+  bf16_t* out = static_cast<bf16_t*>(p.out) + row0 * p.ldo + h * DV + ec;
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  __syncthreads();
   for (int c = 0; c < chunks; ++c) {
-    const uint4_* cur = unit;
-    if (c + 1 < chunks) unit += stride;           // (the last chunk loads itself again)
-    const int at = c * kC;
-    float4_ dec[NK];
-#pragma unroll
-    for (int i = 0; i < NK; ++i) dec[i] = reinterpret_cast<const float4_*>(cur + U::dec)[4 * i + g];
-    bf16_t z[2][4][ND];                           // gates of the rows and columns this lane will store
-#pragma unroll
-    for (int u = 0; u < 2; ++u)
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const bf16_t* gate = static_cast<const bf16_t*>(p.gate) + (row0 + min(at + 16 * u + 4 * g + j, total - 1)) * p.ldg + h * DV + col0;
-#pragma unroll
-        for (int d = 0; d < ND; ++d) z[u][j][d] = gate[16 * d];
-      }
-
-    float4_ R[2][ND] = {}, O[2][ND] = {};
+    const uint4_* cur = staged + (AHEAD ? (c & 1) * SIZE : 0);
+    const uint4_* curh = cur + U::size;
+    const int t = c * kC + er;
+    if (AHEAD && c + 1 < chunks) stage(c + 1);
+    const uint4_ z = *reinterpret_cast<const uint4_*>(gate + (long)min(t, total - 1) * p.ldg);
+    auto frag = [&](const uint4_* u, int place) {
+      return Split{__builtin_bit_cast(bf16x8, u[place + lane]), __builtin_bit_cast(bf16x8, u[place + 64 + lane])};
+    };
+    float4_ R[2] = {}, O[2] = {};
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
-      Split sf[ND];
-#pragma unroll
-      for (int d = 0; d < ND; ++d) sf[d] = split8(S[2 * i][d], S[2 * i + 1][d]);
+      const Split sf = split8(S[2 * i], S[2 * i + 1]);
 #pragma unroll
       for (int u = 0; u < 2; ++u) {
-        if constexpr (DELTA) {
-          const Split k = AHEAD ? kd[u][AHEAD ? i : 0] : frag(cur, U::kd + (u * NI + i) * 128);
-#pragma unroll
-          for (int d = 0; d < ND; ++d) R[u][d] = mac(k, sf[d], R[u][d]);
-        }
-        const Split q = AHEAD ? qd[AHEAD ? u : 0][AHEAD ? i : 0] : frag(cur, U::qd + (u * NI + i) * 128);
-#pragma unroll
-        for (int d = 0; d < ND; ++d) O[u][d] = mac(q, sf[d], O[u][d]);
+        if constexpr (DELTA) R[u] = mac(frag(cur, U::kd + (u * NI + i) * 128), sf, R[u]);
+        O[u] = mac(frag(cur, U::qd + (u * NI + i) * 128), sf, O[u]);
       }
     }
-    load_rows(unit);
-    Split uf[ND];
+    const float* dec = reinterpret_cast<const float*>(curh + HU::dec);
+    uint2_ vr[2];
+    float4_ v[2];
 #pragma unroll
-    for (int d = 0; d < ND; ++d) {
-      float4_ v[2];
-#pragma unroll
-      for (int u = 0; u < 2; ++u)
-        v[u] = float4_{__uint_as_float(vf[u][d][0] << 16), __uint_as_float(vf[u][d][0] & 0xffff0000u),
-                       __uint_as_float(vf[u][d][1] << 16), __uint_as_float(vf[u][d][1] & 0xffff0000u)};
-      if constexpr (DELTA) {
-        const Split rf = split8(v[0] - R[0][d], v[1] - R[1][d]);
-        const float4_ zero = float4_{0.f, 0.f, 0.f, 0.f};
-        uf[d] = split8(mac(tf[0], rf, zero), mac(tf[1], rf, zero));
-      } else {
-        uf[d] = split8(v[0], v[1]);
+    for (int u = 0; u < 2; ++u) {
+      vr[u] = reinterpret_cast<const uint2_*>(curh + HU::vf)[(u * HU::ND + w) * 64 + lane];
+      v[u] = float4_{__uint_as_float(vr[u][0] << 16), __uint_as_float(vr[u][0] & 0xffff0000u), __uint_as_float(vr[u][1] << 16),
+                     __uint_as_float(vr[u][1] & 0xffff0000u)};
+      if constexpr (!CHANNEL) {                   // decays from the chunk's start
+        const float4_ from = load4(dec + 16 * u + 4 * g);
+        R[u] *= from;
+        O[u] *= from;
       }
-#pragma unroll
-      for (int u = 0; u < 2; ++u) O[u][d] = mac(pf[u], uf[d], O[u][d]);
     }
-    load_rest(unit);
+    Split uf;                                     // U, its rows decayed to the chunk's end for the state
+    if constexpr (DELTA) {
+      const Split rf = split8(v[0] - R[0], v[1] - R[1]);
+      const float4_ zero = float4_{0.f, 0.f, 0.f, 0.f};
+      v[0] = mac(frag(curh, HU::tf), rf, zero);
+      v[1] = mac(frag(curh, HU::tf + 128), rf, zero);
+      uf = split8(v[0], v[1]);
 #pragma unroll
-    for (int i = 0; i < NK; ++i) {
-      const Split k = AHEAD ? ke[AHEAD ? i : 0] : frag(cur, U::ke + i * 128);
+      for (int u = 0; u < 2; ++u) O[u] = mac(frag(curh, HU::pf + u * 128), uf, O[u]);
+    } else {
+      const bf16x8 vf = __builtin_bit_cast(bf16x8, uint4_{vr[0][0], vr[0][1], vr[1][0], vr[1][1]});
 #pragma unroll
-      for (int d = 0; d < ND; ++d) S[i][d] = mac(k, uf[d], S[i][d] * dec[i]);
+      for (int u = 0; u < 2; ++u) {
+        const Split f = frag(curh, HU::pf + u * 128);
+        O[u] = mac(f.lo, vf, mac(f.hi, vf, O[u]));
+      }
     }
-    load_keys(unit);
+    if constexpr (CHANNEL) {
+#pragma unroll
+      for (int i = 0; i < NK; ++i) S[i] = mac(frag(cur, U::ke + i * 128), uf, S[i] * load4(dec + 16 * i + 4 * g));
+    } else {
+      uf = split8(v[0] * load4(dec + 32 + 4 * g), v[1] * load4(dec + 48 + 4 * g));
+      const float all = dec[64];
+#pragma unroll
+      for (int i = 0; i < NK; ++i) S[i] = mac(frag(cur, U::ke + i * 128), uf, S[i] * all);
+    }
 
-    // the heads' norm over all waves' columns, gain and gate
-    float* mine = red[c & 1][w];
+    __syncthreads();                              // every wave is done with the row operands and the last chunk's outputs
 #pragma unroll
     for (int u = 0; u < 2; ++u)
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        float ss = 0.f;
-#pragma unroll
-        for (int d = 0; d < ND; ++d) ss += O[u][d][j] * O[u][d][j];
-#pragma unroll
-        for (int d = 1; d < 16; d <<= 1) ss += __shfl_xor(ss, d, 64);
-        if (c16 == 0) mine[16 * u + 4 * g + j] = ss;
-      }
+      for (int j = 0; j < 4; ++j) so[(16 * u + 4 * g + j) * LO + 16 * w + c16] = O[u][j];
+    if constexpr (AHEAD) asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
+    // every head's norm, gain and gate
+    float y[8], zf[8], ss = 0.f;
+    *reinterpret_cast<float4_*>(y) = load4(so + er * LO + ec);
+    *reinterpret_cast<float4_*>(y + 4) = load4(so + er * LO + ec + 4);
+    if constexpr (!AHEAD) {
+      __syncthreads();
+      if (c + 1 < chunks) stage(c + 1);
+    }
 #pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      float4_ sum = float4_{0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < 8; ++i) ss += y[i] * y[i];
+    const float r = __builtin_amdgcn_rsqf(lanes_sum<TPR>(ss) * inv_vdim + p.eps);
+    unpack8(z, zf);
 #pragma unroll
-      for (int v = 0; v < NW; ++v) sum += load4(&red[c & 1][v][16 * u + 4 * g]);
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int t = at + 16 * u + 4 * g + j;
-        const float r = 1.f / sqrtf(sum[j] / (float)p.vdim + p.eps);
-        bf16_t* out = static_cast<bf16_t*>(p.out) + (row0 + t) * p.ldo + h * DV + col0;
-        if (t < total) {
-#pragma unroll
-          for (int d = 0; d < ND; ++d)
-            out[16 * d] = f2bf(O[u][d][j] * r * gain[d] * gate_act<true>(bf2f(z[u][j][d]), p.gate_kind));
-        }
-      }
+    for (int i = 0; i < 8; ++i) y[i] *= r * gain[i] * gate_act<true>(zf[i], p.gate_kind);
+    if (t < total) *reinterpret_cast<uint4_*>(out + (long)t * p.ldo) = pack8(y);
+    if constexpr (!AHEAD) {
+      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+      __syncthreads();
     }
   }
   if (slot >= 0) {
 #pragma unroll
     for (int i = 0; i < NK; ++i)
 #pragma unroll
-      for (int d = 0; d < ND; ++d)
-#pragma unroll
-        for (int j = 0; j < 4; ++j) st[(long)(16 * i + 4 * g + j) * DV + 16 * d] = S[i][d][j];
+      for (int j = 0; j < 4; ++j) st[(long)(16 * i + 4 * g + j) * DV] = S[i][j];
   }
 }
 
-template <int MODE, int DK, int DV, int KT>
-static void prep(const RuleArgs& a, hipStream_t s) {
-  constexpr int lds = 4 * (2 * kC * (DK + 4) + 3 * kC * 36 + kC + (MODE == kChannel ? kC * (DK + 4) : kC));
-  (void)hipFuncSetAttribute(reinterpret_cast<const void*>(rule_prep_kernel<MODE, DK, DV, KT>),
+template <int MODE, int DK, int DV, bool AHEAD>
+static void scan(const RuleArgs& a, hipStream_t s) {
+  constexpr int unit = (RowUnit<DK>::size + HeadUnit<DV>::size) * 16;
+  constexpr int lds = AHEAD ? 2 * unit + kC * (DV + 4) * 4 : unit;
+  static_assert(lds <= 160 * 1024, "prepared chunks in LDS");
+  (void)hipFuncSetAttribute(reinterpret_cast<const void*>(rule_scan_kernel<MODE, DK, DV, AHEAD>),
                             hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-  rule_prep_kernel<MODE, DK, DV, KT><<<dim3((a.max_q + kC - 1) / kC, a.heads, a.B), 256, lds, s>>>(a);
+  rule_scan_kernel<MODE, DK, DV, AHEAD><<<dim3(a.heads, a.B), DV * 4, lds, s>>>(a);
 }
 
 template <int MODE, int DK, int DV>
 static void chunks(const RuleArgs& a, hipStream_t s) {
-  if (MODE == kRetention || a.taps <= 4) prep<MODE, DK, DV, 4>(a, s);
-  else prep<MODE, DK, DV, 16>(a, s);
-  constexpr int ND = DV == 64 ? 1 : 2;
-  rule_scan_kernel<MODE != kRetention, DK, DV, ND, (DK <= 128)><<<dim3(a.heads, a.B), DV / ND * 4, 0, s>>>(a);
+  const int n = (a.max_q + kC - 1) / kC;
+  if constexpr (MODE == kChannel) {
+    constexpr int lds = 4 * (3 * kC * (DK + 4) + kC + 24 * DK);
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(rule_prep_channel_kernel<DK, DV>),
+                              hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    rule_prep_channel_kernel<DK, DV><<<dim3(n, a.heads, a.B), 512, lds, s>>>(a);
+  } else {
+    constexpr bool DELTA = MODE == kHead;
+    constexpr int lds = 2 * 4 * kC * (DK + 8);
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(rule_prep_head_kernel<DELTA, DK, DV>),
+                              hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    rule_prep_head_kernel<DELTA, DK, DV><<<dim3(n, a.heads / (a.H / a.G), a.B), 512, lds, s>>>(a);
+  }
+  rule_solve_kernel<MODE, DK, DV><<<dim3((n + 3) / 4, a.heads, a.B), 256, 0, s>>>(a);
+  // one chunk ahead where no second workgroup of the CU would fill the wait
+  if constexpr (DK <= 128) {
+    if ((long)a.heads * a.B <= 384) return scan<MODE, DK, DV, true>(a, s);
+  }
+  scan<MODE, DK, DV, false>(a, s);
 }
 
 void launch_rule_chunks(const RuleArgs& a, hipStream_t s) {

@@ -37,7 +37,7 @@ SCAN_CHUNK, SCAN_MAX_CHUNKS = 64, 64
 STATE_SEGMENT, STATE_MAX_SEGMENTS = 128, 32      # rows of a matrix-state segment at least; segments at most
 WHOLE = 1 << 30              # window that holds any sequence
 RULE_CHUNK = 32              # rows of a chunk of the delta rule and of retention
-RULE_WORKSPACE = 1 << 30     # bytes of prepared chunks at a time (more heads take several rounds)
+RULE_WORKSPACE = 1 << 32     # bytes of prepared chunks at a time (more heads take several rounds)
 
 
 def pad64(n: int) -> int:
@@ -593,11 +593,16 @@ def _rule_run(x, gate, state, out, batch, shape: RuleShape, eps: float, commit, 
     if x.dtype == torch.float32:
         _K().rule_rows(x, gate, state, out, **args)
     else:
-        unit, chunks = _K().rule_chunk_bytes(dk, dv), T // RULE_CHUNK + batch.B
-        at_a_time = max(1, min(H, RULE_WORKSPACE // (chunks * unit)))
-        ws = torch.empty(chunks * at_a_time * unit, dtype=torch.uint8, device=x.device)
-        for h in range(0, H, at_a_time):
-            _K().rule_chunks(x, gate, state, out, ws=ws, max_q=int(batch.S), head0=h, heads=min(at_a_time, H - h), **args)
+        # whole groups of heads with common queries and keys; rounds of equal size
+        groups, per_channel = int(shape.kv_heads), "decay" in args and args["decay"].shape[1] != H
+        size = H // groups
+        need = lambda n: (T // RULE_CHUNK + batch.B) * _K().rule_chunk_bytes(dk, dv, n * size, n * (size if per_channel else 1))
+        rounds = -(-groups // max(1, min(groups, RULE_WORKSPACE // need(1))))
+        n = -(-groups // rounds)
+        ws = torch.empty(need(n), dtype=torch.uint8, device=x.device)
+        for g in range(0, groups, n):
+            _K().rule_chunks(x, gate, state, out, ws=ws, max_q=int(batch.S), head0=g * size, heads=min(n, groups - g) * size,
+                             **args)
     if commit is not None:
         _K().ring_commit(x, commit, batch.positions, batch.q_start, batch.q_lens, batch.state_slots)
 
