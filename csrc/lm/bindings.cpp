@@ -838,7 +838,7 @@ void rule_chunks(const Tensor& x, const Tensor& gate, const Tensor& state, const
   const int group = a.H / a.G;
   a.ws_chunks = (long)a.T / 32 + a.B;
   SHAI_CHECK(head0 >= 0 && heads >= 1 && head0 + heads <= a.H && head0 % group == 0 && heads % group == 0 && max_q >= 1 &&
-                 ws.numel() >= a.ws_chunks * shai_lm::rule_chunk_bytes(a.dk, a.dv, heads, a.mode == 2 ? heads : heads / group),
+                 ws.numel() >= a.ws_chunks * shai_lm::rule_chunk_bytes(a.dk, a.dv, heads, a.mode == 2 ? heads : heads / group, a.mode == 2),
              "rule_chunks: whole groups of heads, workspace");
   a.ws = ws.data_ptr();
   a.head0 = head0;
@@ -847,8 +847,8 @@ void rule_chunks(const Tensor& x, const Tensor& gate, const Tensor& state, const
   if (a.T > 0) shai_lm::launch_rule_chunks(a, stream());
 }
 
-int64_t rule_chunk_bytes(int64_t dk, int64_t dv, int64_t heads, int64_t keys) {
-  return shai_lm::rule_chunk_bytes(dk, dv, heads, keys);
+int64_t rule_chunk_bytes(int64_t dk, int64_t dv, int64_t heads, int64_t keys, bool channel) {
+  return shai_lm::rule_chunk_bytes(dk, dv, heads, keys, channel);
 }
 
 void ring_commit(const Tensor& x, const Tensor& ring, const Tensor& pos, const Tensor& q_start, const Tensor& q_lens,
@@ -1164,7 +1164,7 @@ TORCH_LIBRARY_FRAGMENT(shai, m) {
   m.def("hgrn2(Tensor qv, Tensor z, Tensor bias, Tensor lower, Tensor gain, Tensor(a!) state, Tensor(b!) out, Tensor pos, Tensor? q_start, Tensor? q_lens, Tensor slots, Tensor(c!) ws, int max_q, int len, int vdim, float eps) -> ()");
   m.def("rule_rows(Tensor x, Tensor gate, Tensor(a!) state, Tensor(b!) out, Tensor pos, Tensor slots, int kv_heads, int dim, int vdim, int gate_kind, float eps, Tensor rate, Tensor? decay=None, Tensor? beta=None, Tensor? conv=None, Tensor? bias=None, Tensor? gain=None, Tensor(c!)? ring=None, Tensor? rope=None, Tensor? q_start=None, Tensor? q_lens=None) -> ()");
   m.def("rule_chunks(Tensor x, Tensor gate, Tensor(a!) state, Tensor(b!) out, Tensor pos, Tensor slots, int kv_heads, int dim, int vdim, int gate_kind, float eps, Tensor rate, Tensor? decay=None, Tensor? beta=None, Tensor? conv=None, Tensor? bias=None, Tensor? gain=None, Tensor? ring=None, Tensor? rope=None, *, Tensor q_start, Tensor q_lens, Tensor(c!) ws, int max_q, int head0, int heads) -> ()");
-  m.def("rule_chunk_bytes(int dk, int dv, int heads, int keys) -> int", &rule_chunk_bytes);
+  m.def("rule_chunk_bytes(int dk, int dv, int heads, int keys, bool channel) -> int", &rule_chunk_bytes);
   m.def("ring_commit(Tensor x, Tensor(a!) ring, Tensor pos, Tensor q_start, Tensor q_lens, Tensor slots) -> ()");
   m.def("gated_attn_prefill(Tensor qkvg, Tensor k_cache, Tensor v_cache, Tensor(a!) o, Tensor block_table, Tensor ctx_lens, Tensor q_lens, Tensor q_start, int max_q, int heads, int chunk, float scale, bool window=False, bool per_element=False, bool own_kv=True, Tensor? temp=None, Tensor? sink=None, float out_scale=1.) -> ()");
   m.def("gated_attn_decode(Tensor qkvg, Tensor(a!) k_cache, Tensor(b!) v_cache, Tensor(c!) o, Tensor block_table, Tensor ctx_lens, Tensor slots, Tensor(d!) ws, int heads, int splits, int chunk, float scale, bool window=False, bool per_element=False, bool own_kv=True, Tensor? rope=None, int dim=0, float eps=0., Tensor? q_gain=None, Tensor? k_gain=None, Tensor? temp=None, Tensor? sink=None, float out_scale=1.) -> ()");

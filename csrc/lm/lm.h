@@ -303,7 +303,7 @@ struct RuleArgs {          // delta rule (mode 1: a decay per head, 2: per key c
 void launch_rule_rows(const RuleArgs& a, bool f32, hipStream_t s);     // row by row
 void launch_rule_chunks(const RuleArgs& a, hipStream_t s);             // bf16, 32 rows at a time; heads head0 .. of a prefill step
 // workspace of one chunk of `heads` heads and `keys` heads of queries and keys (those of every head with a decay per channel)
-long rule_chunk_bytes(int dk, int dv, int heads, int keys);
+long rule_chunk_bytes(int dk, int dv, int heads, int keys, bool channel);
 
 struct RingArgs {          // the last inputs of a prefill step into the rings
   const void* x;

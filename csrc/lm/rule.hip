@@ -235,27 +235,50 @@ void launch_ring_commit(const RingArgs& a, bool f32, hipStream_t s) {
 
 // ------------------------------------------------------------------------------------------------ 32 rows at a time
 constexpr int kC = 32;
-// Prepared chunks, in 16-byte units: fragments are [64 lanes] of 16 bytes, values and remainders one after the other.  Row
-// operands (time x channels, u: rows 16 u ..): a lane holds channels 32 i + 4 g .. and 32 i + 16 + 4 g .. of its row; column
-// operands (channels x time) and score operands (time x time): times 4 g .. and 16 + 4 g ...
-// Rows: one per head with a decay per channel (decays applied), else one per key head (the scan applies the decays).
-template <int DK>
+// Prepared chunks, in 16-byte units.  Rows of a chunk (time x channels) are kept in the order in which the scan reads them from LDS,
+// as rows and, transposed, as columns.  Keys and queries: bf16 values and then their remainders; of every 32 channels, 4 g .. and
+// 16 + 4 g .. share a 16-byte piece, and the pieces of a row are permuted by its number modulo 8.  Values: 8-byte pieces
+// permuted by `turned`.  Score operands (time x time) are fragments of [64 lanes] of 16 bytes, values and remainders one after
+// the other, u: rows 16 u ..; a lane holds times 4 g .. and 16 + 4 g ..
+// Row units: one per head with a decay per channel (decays applied), else one per key head (the scan applies the decays).
+template <int DK, bool CHANNEL>
 struct RowUnit {
-  static constexpr int NI = DK / 32, NK = DK / 16;
-  static constexpr int kd = 0;                               // B K     [u 2][i NI][2][64]
-  static constexpr int qd = kd + 2 * NI * 128;               // B Q     the same (retention starts here)
-  static constexpr int ke = qd + 2 * NI * 128;               // K B_end / B  [i NK][2][64]
-  static constexpr int size = ke + NK * 128;
+  static constexpr int part = DK * 8;                        // [2][32][DK]
+  static constexpr int kd = 0;                               // K, or B K
+  static constexpr int qd = part;                            // Q, or B Q
+  static constexpr int ke = CHANNEL ? 2 * part : 0;          // K B_end / B
+  static constexpr int size = CHANNEL ? 3 * part : 2 * part;
 };
 template <int DV>
 struct HeadUnit {
-  static constexpr int ND = DV / 16;
   static constexpr int tf = 0;                               // (I + A)^-1 diag(b)  [u 2][2][64]
   static constexpr int pf = tf + 256;                        // P (retention starts here)
-  static constexpr int vf = pf + 256;                        // V: [u 2][d ND][64 lanes] of 4 rows x 1 column, 8 bytes
-  static constexpr int dec = vf + ND * 64;                   // floats: B_end [DK], or B [32], B_end / B [32], B_end
+  static constexpr int vf = pf + 256;                        // V [32][DV], values only
+  static constexpr int dec = vf + DV * 4;                    // floats: B_end [DK], or B [32], B_end / B [32], B_end
   static constexpr int size = dec + 64;
 };
+__device__ __forceinline__ int turned(int t) { return (t & 3) << 2 | (t >> 2 & 3); }
+// 8 columns 8 vec .. of row t of the values
+template <int DV>
+__device__ __forceinline__ void put_values(uint4_* part, int t, int vec, uint4_ y) {
+  const int x = turned(t);
+  part[t * (DV / 8) + (vec ^ (x >> 1))] = x & 1 ? uint4_{y[2], y[3], y[0], y[1]} : y;
+}
+__device__ __forceinline__ uint32_t dpp_swap2(uint32_t x) {       // lanes 0 1 2 3 of every four <- 2 3 0 1
+  return __builtin_amdgcn_update_dpp(0u, x, 0x4E, 0xf, 0xf, true);
+}
+// 8 channels 8 vec .. of row t; lanes of consecutive `vec` call it together
+template <int DK>
+__device__ __forceinline__ void put_row(uint4_* part, int t, int vec, const Split& f) {
+  const bool second = vec & 2;                    // of the 16 channels that share pieces with 16 others
+  const int piece = 4 * (vec >> 2) + 2 * (vec & 1) + second;
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const uint4_ y = __builtin_bit_cast(uint4_, i ? f.lo : f.hi);
+    const uint32_t a = dpp_swap2(second ? y[0] : y[2]), b = dpp_swap2(second ? y[1] : y[3]);
+    part[i * 4 * DK + t * (DK / 8) + (piece ^ (t & 7))] = second ? uint4_{a, b, y[2], y[3]} : uint4_{y[0], y[1], a, b};
+  }
+}
 // Scores before the solve, fp32 [2][32][32]: A and P (a decay per channel), or k k^T and q k^T.
 constexpr int kScores = 512;
 // chunks of earlier sequences never reach the next one's first
@@ -273,8 +296,8 @@ __device__ __forceinline__ float* score_unit(const RuleArgs& p, long chunk, int 
                                   (chunk * keys + key) * kScores);
 }
 
-long rule_chunk_bytes(int dk, int dv, int heads, int keys) {
-  return 16L * ((long)keys * (dk * 24 + kScores) + (long)heads * (512 + dv * 4 + 64));
+long rule_chunk_bytes(int dk, int dv, int heads, int keys, bool channel) {
+  return 16L * ((long)keys * (dk * (channel ? 24 : 16) + kScores) + (long)heads * (512 + dv * 4 + 64));
 }
 
 // ---- inputs of 4 rows x 8 channels
@@ -282,15 +305,6 @@ long rule_chunk_bytes(int dk, int dv, int heads, int keys) {
 // `x`: the chunk's first row, row `at` of the step; before the step's first row the ring's inputs count.
 __device__ __forceinline__ void conv_rows(const RuleArgs& p, const bf16_t* x, int ch, int channels, int r0, int at, int live,
                                           int pos0, int slot, float (&y)[4][8]) {
-  const bf16_t* ring = static_cast<const bf16_t*>(p.ring) + (long)max(slot, 0) * p.taps * channels + ch;
-  const int ring0 = pos0 % p.taps;
-  auto input = [&](int r) {                       // (rows behind the last one repeat it: their results are dropped)
-    if (at + r >= 0) return *reinterpret_cast<const uint4_*>(x + (long)min(r, live - 1) * p.ldx + ch);
-    const int m = ring0 + at + r;
-    if (at + r > -p.taps && pos0 + at + r >= 0 && slot >= 0)
-      return *reinterpret_cast<const uint4_*>(ring + (long)(m < 0 ? m + p.taps : m) * channels);
-    return uint4_{0u, 0u, 0u, 0u};
-  };
   auto tap = [&](int j, float (&wt)[8]) {         // of the input j rows before
     const float* cw = p.conv + (long)(p.taps - 1 - min(j, p.taps - 1)) * channels + ch;
     const float on = j < p.taps ? 1.f : 0.f;
@@ -301,11 +315,12 @@ __device__ __forceinline__ void conv_rows(const RuleArgs& p, const bf16_t* x, in
   for (int r = 0; r < 4; ++r)
 #pragma unroll
     for (int i = 0; i < 8; ++i) y[r][i] = 0.f;
-  if (p.taps <= 4) {
+  if (at > 0 && p.taps <= 4) {                    // every input is a row of the step
     uint4_ in[7];
     float wt[4][8];
 #pragma unroll
-    for (int i = 0; i < 7; ++i) in[i] = input(r0 + i - 3);
+    for (int i = 0; i < 7; ++i)                   // (rows behind the last one repeat it: their results are dropped)
+      in[i] = *reinterpret_cast<const uint4_*>(x + (long)min(r0 + i - 3, live - 1) * p.ldx + ch);
 #pragma unroll
     for (int j = 0; j < 4; ++j) tap(j, wt[j]);
 #pragma unroll
@@ -322,15 +337,21 @@ __device__ __forceinline__ void conv_rows(const RuleArgs& p, const bf16_t* x, in
       }
     }
   } else {
+    const bf16_t* ring = static_cast<const bf16_t*>(p.ring) + (long)max(slot, 0) * p.taps * channels + ch;
+    const int ring0 = pos0 % p.taps;
+#pragma unroll 1
     for (int j = 0; j < p.taps; ++j) {
       float wt[8];
       tap(j, wt);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
+        const int i = min(r0 + r, live - 1) - j, m = ring0 + at + i;
+        const bool here = at + i >= 0, past = pos0 + at + i >= 0 && slot >= 0;
+        const bf16_t* src = here ? x + (long)i * p.ldx + ch : ring + (long)(m < 0 ? m + p.taps : m) * channels;
         float f[8];
-        unpack8(input(r0 + r - j), f);
+        unpack8(here || past ? *reinterpret_cast<const uint4_*>(src) : uint4_{0u, 0u, 0u, 0u}, f);
 #pragma unroll
-        for (int i = 0; i < 8; ++i) y[r][i] += wt[i] * f[i];
+        for (int e = 0; e < 8; ++e) y[r][e] += wt[e] * f[e];
       }
     }
   }
@@ -388,26 +409,11 @@ __device__ __forceinline__ float unit_factor(const float (&y)[8], bool query, in
   return __builtin_amdgcn_rsqf(query ? (ss + 1e-6f) * (float)dim : ss + 1e-6f);
 }
 
-// values of rows 4 rg .., columns 8 vec ..
-template <int DV>
-__device__ __forceinline__ void put_values(uint4_* unit, int rg, int vec, const float (&y)[4][8]) {
-  uint2_* dst = reinterpret_cast<uint2_*>(unit + HeadUnit<DV>::vf) + ((rg >> 2) * HeadUnit<DV>::ND + (vec >> 1)) * 64 +
-                (rg & 3) * 16 + (vec & 1) * 8;
-#pragma unroll
-  for (int i = 0; i < 8; ++i) dst[i] = uint2_{pack2(y[0][i], y[1][i]), pack2(y[2][i], y[3][i])};
-}
-
-// ---- decay per channel: a row's logarithm is kept relative to the fourth row of its 8-row block (c), so that
-// 2^c and 2^-c stay in range (rows forget 2^-24 at most); what lies between two blocks, or a block and a border, is one factor
-// per channel.  `fac`: [0 + j] start of the chunk to block j, [4 + j] block j to the chunk's end, [8 + j] block j to or from the
-// border of the halves, [12 + j] to or from the border of the half's two blocks.
-constexpr float kLeastChannel = -24.f;
-
 // One decay per head, or a fixed one: a workgroup prepares a chunk's queries and keys, their products, and the values of the
 // heads that share them.  Queries and keys lie in LDS as values and remainders, as the matrix products read them.
 template <bool DELTA, int DK, int DV>
 __global__ void __launch_bounds__(512, 4) rule_prep_head_kernel(const RuleArgs p) {
-  using U = RowUnit<DK>;
+  using U = RowUnit<DK, false>;
   using HU = HeadUnit<DV>;
   constexpr int NT = 512, LD = DK + 8, VQ = DK / 8, VV = DV / 8;
   extern __shared__ __attribute__((aligned(16))) bf16_t planes[];
@@ -445,9 +451,11 @@ __global__ void __launch_bounds__(512, 4) rule_prep_head_kernel(const RuleArgs p
         bf16_t* dst = (what ? sk : sq) + (4 * rg + r) * LD + 8 * vec;
         *reinterpret_cast<bf16x8*>(dst) = f.hi;
         *reinterpret_cast<bf16x8*>(dst + kC * LD) = f.lo;
+        put_row<DK>(rows + (what ? U::kd : U::qd), 4 * rg + r, vec, f);
       }
     } else {
-      put_values<DV>(head(j), rg, vec, y);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) put_values<DV>(head(j) + HU::vf, 4 * rg + r, vec, pack8(y[r]));
     }
   }
   __syncthreads();
@@ -463,43 +471,21 @@ __global__ void __launch_bounds__(512, 4) rule_prep_head_kernel(const RuleArgs p
     };
     float4_ acc = float4_{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int i = 0; i < U::NI; ++i) acc = mac(frag(left + 32 * i), frag(right + 32 * i), acc);
+    for (int i = 0; i < DK / 32; ++i) acc = mac(frag(left + 32 * i), frag(right + 32 * i), acc);
 #pragma unroll
     for (int j = 0; j < 4; ++j) scores[(w & 1) * 1024 + (tr + 4 * g + j) * 32 + tc + c16] = acc[j];
   }
-  {                                               // queries and keys as operands
-    constexpr int NR = 2 * U::NI;
-    for (int f = (DELTA ? 0 : NR) + 7 - w; f < 2 * NR + U::NK; f += 8) {     // (the last waves have no scores)
-      uint4_ plane[2];
-      if (f < 2 * NR) {
-        const int i = f % NR;
-        const bf16_t* src = (f < NR ? sk : sq) + (16 * (i / U::NI) + c16) * LD + 32 * (i % U::NI) + 4 * g;
-#pragma unroll
-        for (int v = 0; v < 2; ++v) {
-          const uint2_ lo = *reinterpret_cast<const uint2_*>(src + v * kC * LD);
-          const uint2_ hi = *reinterpret_cast<const uint2_*>(src + v * kC * LD + 16);
-          plane[v] = uint4_{lo[0], lo[1], hi[0], hi[1]};
-        }
-      } else {
-        const bf16_t* src = sk + 4 * g * LD + 16 * (f - 2 * NR) + c16;
-#pragma unroll
-        for (int v = 0; v < 2; ++v)
-#pragma unroll
-          for (int j = 0; j < 4; ++j) {
-            const bf16_t* y = src + v * kC * LD + (16 * (j >> 1) + 2 * (j & 1)) * LD;
-            plane[v][j] = (uint32_t)y[0] | (uint32_t)y[LD] << 16;
-          }
-      }
-      uint4_* dst = rows + (f < NR ? U::kd + f * 128 : f < 2 * NR ? U::qd + (f - NR) * 128 : U::ke + (f - 2 * NR) * 128);
-      dst[lane] = plane[0];
-      dst[64 + lane] = plane[1];
-    }
-  }
 }
+
+// Decays per channel: a row's logarithm is kept relative to the fourth row of its 8-row block (c), so that 2^c and 2^-c stay in
+// range (rows forget 2^-24 at most); what lies between two blocks, or a block and a border, is one factor per channel.  `fac`:
+// [0 + j] start of the chunk to block j, [4 + j] block j to the chunk's end, [8 + j] block j to or from the border of the halves,
+// [12 + j] to or from the border of the half's two blocks.
+constexpr float kLeastChannel = -24.f;
 
 template <int DK, int DV>
 __global__ void __launch_bounds__(512, 4) rule_prep_channel_kernel(const RuleArgs p) {
-  using U = RowUnit<DK>;
+  using U = RowUnit<DK, true>;
   using HU = HeadUnit<DV>;
   constexpr int NT = 512, LD = DK + 4, VQ = DK / 8, VV = DV / 8;
   extern __shared__ __attribute__((aligned(16))) float lds[];
@@ -539,7 +525,8 @@ __global__ void __launch_bounds__(512, 4) rule_prep_channel_kernel(const RuleArg
         store4(dst + 4, float4_{y[r][4], y[r][5], y[r][6], y[r][7]} * scale);
       }
     } else {
-      put_values<DV>(head, rg, vec, y);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) put_values<DV>(head + HU::vf, 4 * rg + r, vec, pack8(y[r]));
     }
   }
 
@@ -609,7 +596,7 @@ __global__ void __launch_bounds__(512, 4) rule_prep_channel_kernel(const RuleArg
       return split8(load4(row + d0) * load4(f + d0), load4(row + d0 + 4) * load4(f + d0 + 4));
     };
 #pragma unroll 2
-    for (int i = 0; i < U::NI; ++i) {
+    for (int i = 0; i < DK / 32; ++i) {
       const int d0 = 32 * i + 8 * g;
       const float* dn = sb + (tc + c16) * LD;     // k 2^-c
       if (tile == 0) {
@@ -639,29 +626,14 @@ __global__ void __launch_bounds__(512, 4) rule_prep_channel_kernel(const RuleArg
   }
 
   // ---- operands of the scan
-  auto put = [&](int place, const Split& f) {
-    rows[place + lane] = __builtin_bit_cast(uint4_, f.hi);
-    rows[place + 64 + lane] = __builtin_bit_cast(uint4_, f.lo);
-  };
-  {
-    constexpr int NR = 2 * U::NI;
-    for (int f = 7 - w; f < 2 * NR + U::NK; f += 8) {             // (the last waves have no scores)
-      if (f < 2 * NR) {                           // rows decayed from the chunk's start
-        const int i = f % NR, row = 16 * (i / U::NI) + c16, d0 = 32 * (i % U::NI) + 4 * g;
-        const float* src = (f < NR ? sk : sq) + row * LD + d0;
-        const float* e = fac + (row >> 3) * DK + d0;
-        put((f < NR ? U::kd : U::qd) + i * 128, split8(load4(src) * load4(e), load4(src + 16) * load4(e + 16)));
-      } else {                                    // keys decayed to its end, by channel
-        const int i = f - 2 * NR, ch = 16 * i + c16;
-        const float* src = sb + 4 * g * LD + ch;
-        float4_ y[2];
-#pragma unroll
-        for (int u = 0; u < 2; ++u)
-#pragma unroll
-          for (int j = 0; j < 4; ++j) y[u][j] = src[(16 * u + j) * LD] * fac[(4 + 2 * u + (g >> 1)) * DK + ch];
-        put(U::ke + i * 128, split8(y[0], y[1]));
-      }
-    }
+  for (int id = tid; id < kC * VQ; id += NT) {
+    const int t = id / VQ, vec = id % VQ, o = t * LD + 8 * vec;
+    const float* from = fac + (t >> 3) * DK + 8 * vec;
+    const float* to = from + 4 * DK;
+    const float4_ f0 = load4(from), f1 = load4(from + 4);
+    put_row<DK>(rows + U::kd, t, vec, split8(load4(sk + o) * f0, load4(sk + o + 4) * f1));
+    put_row<DK>(rows + U::qd, t, vec, split8(load4(sq + o) * f0, load4(sq + o + 4) * f1));
+    put_row<DK>(rows + U::ke, t, vec, split8(load4(sb + o) * load4(to), load4(sb + o + 4) * load4(to + 4)));
   }
   if (tid < DK) reinterpret_cast<float*>(head + HU::dec)[tid] = fac[3 * DK + tid] * fac[7 * DK + tid];
 }
@@ -682,7 +654,7 @@ __global__ void __launch_bounds__(256, 4) rule_solve_kernel(const RuleArgs p) {
   const int live = min(kC, total - at), group = CHANNEL ? 1 : p.H / p.G;
   const long row = p.q_start[b] + at + min(tl, live - 1), chunk = first_chunk(p, b) + blockIdx.x * 4 + w;
   uint4_* unit = head_unit(p, chunk, blockIdx.y, HU::size);
-  const float* scores = score_unit(p, chunk, blockIdx.y / group, p.heads / group, RowUnit<DK>::size, HU::size);
+  const float* scores = score_unit(p, chunk, blockIdx.y / group, p.heads / group, RowUnit<DK, CHANNEL>::size, HU::size);
   float* m = sm[w];
   float* lb = sb[w];
   float* beta = sbeta[w];
@@ -823,23 +795,41 @@ __device__ __forceinline__ float lanes_sum(float x) {
   return x;
 }
 
-// Waves of 16 columns of S each.  A prepared chunk goes to LDS by DMA, one chunk ahead (AHEAD: one workgroup per CU) or while
-// another workgroup of the CU computes.
+typedef short s4v __attribute__((ext_vector_type(4)));
+
+// 16 bytes a lane to LDS at the wave-uniform byte address `lds`, lane after lane.  Written out, so that the compiler does not wait
+// for it before every read of LDS: the caller waits (vmcnt) before the barrier after which the data are read.
+__device__ __forceinline__ void dma16_unwaited(const uint4_* src, uint32_t lds) {
+  asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off" ::"s"(lds), "v"(src) : "memory", "m0");
+}
+__device__ __forceinline__ void wait_vm() {
+  __builtin_amdgcn_s_waitcnt(0x0f70);             // vmcnt(0)
+  asm volatile("" ::: "memory");
+}
+__device__ __forceinline__ uint32_t lds_address(const void* p) {
+  return (uint32_t)(uintptr_t)(__attribute__((address_space(3))) const void*)p;
+}
+
+// Waves of 16 columns of S each.  A prepared chunk goes to LDS by DMA, one chunk ahead where two fit (AHEAD).
 template <int MODE, int DK, int DV, bool AHEAD>
-__global__ void __launch_bounds__(DV * 4) rule_scan_kernel(const RuleArgs p) {
-  using U = RowUnit<DK>;
-  using HU = HeadUnit<DV>;
+__global__ void __launch_bounds__(DV * 4) __attribute__((amdgpu_waves_per_eu(DV / 64, DV / 64)))
+rule_scan_kernel(const RuleArgs p) {
   constexpr bool DELTA = MODE != kRetention, CHANNEL = MODE == kChannel;
-  constexpr int NW = DV / 16, NI = U::NI, NK = U::NK, LO = DV + 4, TPR = DV / 8;
-  constexpr int FU = DELTA ? 0 : U::qd, FH = DELTA ? 0 : HU::pf;             // what retention does not use is not loaded
+  using U = RowUnit<DK, CHANNEL>;
+  using HU = HeadUnit<DV>;
+  constexpr int NW = DV / 16, NI = DK / 32, NK = DK / 16, LO = DV + 4, TPR = DV / 8;
+  constexpr int FH = DELTA ? 0 : HU::pf;          // what retention does not use is not loaded
   constexpr int SIZE = U::size + HU::size;
   extern __shared__ __attribute__((aligned(16))) uint4_ staged[];
-  // [32][LO] outputs: behind the chunks or, with one, in place of its row operands (used up by then)
+  // [32][LO] outputs: behind the chunks or, with one, in its place (used up by then)
   float* so = reinterpret_cast<float*>(AHEAD ? staged + 2 * SIZE : staged);
-  static_assert(kC * LO * 4 <= U::size * 16, "outputs in place of row operands");
+  static_assert(kC * LO * 4 <= SIZE * 16, "outputs in place of the chunk");
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int g = lane >> 4, c16 = lane & 15;
-  const int b = blockIdx.y, h = p.head0 + blockIdx.x, group = CHANNEL ? 1 : p.H / p.G;
+  // heads that share rows follow each other on one XCD (workgroups go round them)
+  const int jobs = p.heads * p.B, q8 = jobs >> 3, r8 = jobs & 7, xcd = blockIdx.x & 7;
+  const int job = (xcd < r8 ? xcd * (q8 + 1) : r8 * (q8 + 1) + (xcd - r8) * q8) + (blockIdx.x >> 3);
+  const int b = job / p.heads, hi = job % p.heads, h = p.head0 + hi, group = CHANNEL ? 1 : p.H / p.G;
   const int total = p.q_lens[b];
   if (total < 1) return;
   const int chunks = (total + kC - 1) / kC;
@@ -849,16 +839,23 @@ __global__ void __launch_bounds__(DV * 4) rule_scan_kernel(const RuleArgs p) {
   float* st = p.state + ((long)max(slot, 0) * p.H + h) * DK * DV + 16 * w + c16;
 
   const int keys = p.heads / group;
-  const uint4_* head = head_unit(p, first_chunk(p, b), blockIdx.x, HU::size) + lane;
-  const uint4_* rows = row_unit(p, first_chunk(p, b), blockIdx.x / group, keys, U::size, HU::size) + lane;
+  const uint4_* head = head_unit(p, first_chunk(p, b), hi, HU::size) + lane;
+  const uint4_* rows = row_unit(p, first_chunk(p, b), hi / group, keys, U::size, HU::size) + lane;
+  const uint32_t at0 = __builtin_amdgcn_readfirstlane(lds_address(staged));
   auto stage = [&](int c) {
-    uint4_* dst = staged + (AHEAD ? (c & 1) * SIZE : 0);
+    const uint32_t dst = at0 + (AHEAD && (c & 1) ? SIZE * 16 : 0);
     const uint4_* su = rows + (long)c * keys * U::size;
-    for (int i = FU / 64 + w; i < U::size / 64; i += NW)
-      dma16(reinterpret_cast<const bf16_t*>(su + 64 * i), reinterpret_cast<bf16_t*>(dst + 64 * i));
     const uint4_* sh = head + (long)c * p.heads * HU::size;
-    for (int i = FH / 64 + w; i < HU::size / 64; i += NW)
-      dma16(reinterpret_cast<const bf16_t*>(sh + 64 * i), reinterpret_cast<bf16_t*>(dst + U::size + 64 * i));
+#pragma unroll
+    for (int j = 0; j < (U::size / 64 + NW - 1) / NW; ++j) {
+      const int i = j * NW + w;
+      if (i < U::size / 64) dma16_unwaited(su + 64 * i, dst + 1024 * i);
+    }
+#pragma unroll
+    for (int j = 0; j < ((HU::size - FH) / 64 + NW - 1) / NW; ++j) {
+      const int i = FH / 64 + j * NW + w;
+      if (i < HU::size / 64) dma16_unwaited(sh + 64 * i, dst + U::size * 16 + 1024 * i);
+    }
   };
   stage(0);
   float4_ S[NK];                                  // rows 16 i + 4 g .., the wave's columns
@@ -866,6 +863,15 @@ __global__ void __launch_bounds__(DV * 4) rule_scan_kernel(const RuleArgs p) {
   for (int i = 0; i < NK; ++i)
 #pragma unroll
     for (int j = 0; j < 4; ++j) S[i][j] = old ? st[(long)(16 * i + 4 * g + j) * DV] : 0.f;
+  // pieces of this lane: 16 bytes of row c16, 8 bytes of row 4 g + tq (channels 32 i ..: i even, odd), and of its values
+  const int tq = c16 >> 2, tp = c16 & 3;
+  int row_at[2], col_at[2];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    row_at[i] = c16 * (DK / 8) + ((4 * i + g) ^ (c16 & 7));
+    col_at[i] = (4 * g + tq) * (DK / 4) + 2 * ((4 * i + tp) ^ (4 * (g & 1) + tq));
+  }
+  const int value_at = (4 * g + tq) * (DV / 4) + 4 * ((w & 3) ^ tq) + 16 * (w >> 2) + (tp ^ g);
   // epilogue: a thread's row of the chunk and 8 columns
   const int er = tid / TPR, ec = tid % TPR * 8;
   float gain[8];
@@ -874,74 +880,146 @@ __global__ void __launch_bounds__(DV * 4) rule_scan_kernel(const RuleArgs p) {
   const float inv_vdim = 1.f / (float)p.vdim;
   const bf16_t* gate = static_cast<const bf16_t*>(p.gate) + row0 * p.ldg + h * DV + ec;
   bf16_t* out = static_cast<bf16_t*>(p.out) + row0 * p.ldo + h * DV + ec;
-  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  wait_vm();
   __syncthreads();
   for (int c = 0; c < chunks; ++c) {
     const uint4_* cur = staged + (AHEAD ? (c & 1) * SIZE : 0);
     const uint4_* curh = cur + U::size;
     const int t = c * kC + er;
-    if (AHEAD && c + 1 < chunks) stage(c + 1);
     const uint4_ z = *reinterpret_cast<const uint4_*>(gate + (long)min(t, total - 1) * p.ldg);
-    auto frag = [&](const uint4_* u, int place) {
-      return Split{__builtin_bit_cast(bf16x8, u[place + lane]), __builtin_bit_cast(bf16x8, u[place + 64 + lane])};
+    if (AHEAD && c + 1 < chunks) stage(c + 1);
+    auto frag = [&](int place) {
+      return Split{__builtin_bit_cast(bf16x8, curh[place + lane]), __builtin_bit_cast(bf16x8, curh[place + 64 + lane])};
     };
-    float4_ R[2] = {}, O[2] = {};
+    // row 16 u + c16: channels 32 i + 4 g .. and 32 i + 16 + 4 g ..
+    auto row = [&](int place, int u, int i) {
+      const uint4_* m = cur + place + u * 2 * DK + 8 * (i >> 1) + row_at[i & 1];
+      return Split{__builtin_bit_cast(bf16x8, m[0]), __builtin_bit_cast(bf16x8, m[4 * DK])};
+    };
+    // a column, 8-byte piece `at` in rows of n: times 4 g .. and 16 + 4 g ..
+    auto column = [&](const uint4_* part, int n, int at) {
+      const uint2_* m = reinterpret_cast<const uint2_*>(part) + at;
+      const s4v lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s4v*)(m));
+      const s4v hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s4v*)(m + 16 * n));
+      const uint2_ a = __builtin_bit_cast(uint2_, lo), b2 = __builtin_bit_cast(uint2_, hi);
+      return uint4_{a[0], a[1], b2[0], b2[1]};
+    };
+    auto key_column = [&](int i) {                // channel 16 i + c16
+      uint4_ y[2];
+#pragma unroll
+      for (int v = 0; v < 2; ++v) y[v] = column(cur + U::ke + v * 4 * DK, DK / 4, col_at[i >> 1 & 1] + 16 * (i >> 2) + (i & 1));
+      return Split{__builtin_bit_cast(bf16x8, y[0]), __builtin_bit_cast(bf16x8, y[1])};
+    };
+    // Operands are read from LDS a step ahead of the products that use them; independent sums take turns.
+    auto hold = [] {
+      if constexpr (AHEAD) __builtin_amdgcn_sched_barrier(0);
+    };
+    constexpr int NR = DELTA ? 4 : 2;             // sums of a step: K S (rows 0 .., 16 ..), then Q S
+    float4_ acc[NR] = {};
+    Split f[NI][NR];
+    auto load_rows = [&](int i) {
+#pragma unroll
+      for (int j = 0; j < NR; ++j) f[i][j] = row(DELTA && j < 2 ? U::kd : U::qd, j & 1, i);
+    };
+    load_rows(0);
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
+      if (i + 1 < NI) load_rows(i + 1);
+      hold();
       const Split sf = split8(S[2 * i], S[2 * i + 1]);
 #pragma unroll
-      for (int u = 0; u < 2; ++u) {
-        if constexpr (DELTA) R[u] = mac(frag(cur, U::kd + (u * NI + i) * 128), sf, R[u]);
-        O[u] = mac(frag(cur, U::qd + (u * NI + i) * 128), sf, O[u]);
-      }
+      for (int j = 0; j < NR; ++j) acc[j] = mac(f[i][j].hi, sf.hi, acc[j]);
+#pragma unroll
+      for (int j = 0; j < NR; ++j) acc[j] = mac(f[i][j].lo, sf.hi, acc[j]);
+#pragma unroll
+      for (int j = 0; j < NR; ++j) acc[j] = mac(f[i][j].hi, sf.lo, acc[j]);
     }
+    float4_* O = acc + NR - 2;
     const float* dec = reinterpret_cast<const float*>(curh + HU::dec);
-    uint2_ vr[2];
+    const uint4_ vr = column(curh + HU::vf, DV / 4, value_at);
+    Split pf[2] = {frag(HU::pf), frag(HU::pf + 128)}, tf[2];
+    if constexpr (DELTA) {
+      tf[0] = frag(HU::tf);
+      tf[1] = frag(HU::tf + 128);
+    }
+    float4_ from[2], to[2];
+    float all = 0.f;
+    if constexpr (!CHANNEL) {
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        from[u] = load4(dec + 16 * u + 4 * g);
+        to[u] = load4(dec + 32 + 16 * u + 4 * g);
+      }
+      all = dec[64];
+    }
+    Split kc[NK];
+    float4_ kdec[CHANNEL ? NK : 1];
+    auto load_keys = [&](int i) {
+#pragma unroll
+      for (int j = i; j < i + 2 && j < NK; ++j) {
+        kc[j] = key_column(j);
+        if constexpr (CHANNEL) kdec[j] = load4(dec + 16 * j + 4 * g);
+      }
+    };
+    load_keys(0);
+    hold();
     float4_ v[2];
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
-      vr[u] = reinterpret_cast<const uint2_*>(curh + HU::vf)[(u * HU::ND + w) * 64 + lane];
-      v[u] = float4_{__uint_as_float(vr[u][0] << 16), __uint_as_float(vr[u][0] & 0xffff0000u), __uint_as_float(vr[u][1] << 16),
-                     __uint_as_float(vr[u][1] & 0xffff0000u)};
+      v[u] = float4_{__uint_as_float(vr[2 * u] << 16), __uint_as_float(vr[2 * u] & 0xffff0000u),
+                     __uint_as_float(vr[2 * u + 1] << 16), __uint_as_float(vr[2 * u + 1] & 0xffff0000u)};
       if constexpr (!CHANNEL) {                   // decays from the chunk's start
-        const float4_ from = load4(dec + 16 * u + 4 * g);
-        R[u] *= from;
-        O[u] *= from;
+        if constexpr (DELTA) acc[u] *= from[u];
+        O[u] *= from[u];
       }
     }
     Split uf;                                     // U, its rows decayed to the chunk's end for the state
     if constexpr (DELTA) {
-      const Split rf = split8(v[0] - R[0], v[1] - R[1]);
-      const float4_ zero = float4_{0.f, 0.f, 0.f, 0.f};
-      v[0] = mac(frag(curh, HU::tf), rf, zero);
-      v[1] = mac(frag(curh, HU::tf + 128), rf, zero);
+      const Split rf = split8(v[0] - acc[0], v[1] - acc[1]);
+#pragma unroll
+      for (int u = 0; u < 2; ++u) v[u] = mac(tf[u].hi, rf.hi, float4_{0.f, 0.f, 0.f, 0.f});
+#pragma unroll
+      for (int u = 0; u < 2; ++u) v[u] = mac(tf[u].lo, rf.hi, v[u]);
+#pragma unroll
+      for (int u = 0; u < 2; ++u) v[u] = mac(tf[u].hi, rf.lo, v[u]);
       uf = split8(v[0], v[1]);
 #pragma unroll
-      for (int u = 0; u < 2; ++u) O[u] = mac(frag(curh, HU::pf + u * 128), uf, O[u]);
-    } else {
-      const bf16x8 vf = __builtin_bit_cast(bf16x8, uint4_{vr[0][0], vr[0][1], vr[1][0], vr[1][1]});
+      for (int u = 0; u < 2; ++u) O[u] = mac(pf[u].hi, uf.hi, O[u]);
 #pragma unroll
-      for (int u = 0; u < 2; ++u) {
-        const Split f = frag(curh, HU::pf + u * 128);
-        O[u] = mac(f.lo, vf, mac(f.hi, vf, O[u]));
-      }
+      for (int u = 0; u < 2; ++u) O[u] = mac(pf[u].lo, uf.hi, O[u]);
+#pragma unroll
+      for (int u = 0; u < 2; ++u) O[u] = mac(pf[u].hi, uf.lo, O[u]);
+    } else {
+      const bf16x8 vf = __builtin_bit_cast(bf16x8, vr);
+#pragma unroll
+      for (int u = 0; u < 2; ++u) O[u] = mac(pf[u].hi, vf, O[u]);
+#pragma unroll
+      for (int u = 0; u < 2; ++u) O[u] = mac(pf[u].lo, vf, O[u]);
     }
-    if constexpr (CHANNEL) {
+    if constexpr (!CHANNEL) uf = split8(v[0] * to[0], v[1] * to[1]);
 #pragma unroll
-      for (int i = 0; i < NK; ++i) S[i] = mac(frag(cur, U::ke + i * 128), uf, S[i] * load4(dec + 16 * i + 4 * g));
-    } else {
-      uf = split8(v[0] * load4(dec + 32 + 4 * g), v[1] * load4(dec + 48 + 4 * g));
-      const float all = dec[64];
+    for (int i = 0; i < NK; i += 2) {             // two tiles of the state at a time
+      load_keys(i + 2);
+      hold();
 #pragma unroll
-      for (int i = 0; i < NK; ++i) S[i] = mac(frag(cur, U::ke + i * 128), uf, S[i] * all);
+      for (int j = i; j < i + 2; ++j) {
+        if constexpr (CHANNEL) S[j] *= kdec[j];
+        else S[j] *= all;
+      }
+#pragma unroll
+      for (int j = i; j < i + 2; ++j) S[j] = mac(kc[j].hi, uf.hi, S[j]);
+#pragma unroll
+      for (int j = i; j < i + 2; ++j) S[j] = mac(kc[j].lo, uf.hi, S[j]);
+#pragma unroll
+      for (int j = i; j < i + 2; ++j) S[j] = mac(kc[j].hi, uf.lo, S[j]);
     }
 
-    __syncthreads();                              // every wave is done with the row operands and the last chunk's outputs
+    __syncthreads();                              // every wave is done with the chunk and the last one's outputs
 #pragma unroll
     for (int u = 0; u < 2; ++u)
 #pragma unroll
       for (int j = 0; j < 4; ++j) so[(16 * u + 4 * g + j) * LO + 16 * w + c16] = O[u][j];
-    if constexpr (AHEAD) asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    if constexpr (AHEAD) wait_vm();
     __syncthreads();
     // every head's norm, gain and gate
     float y[8], zf[8], ss = 0.f;
@@ -959,7 +1037,7 @@ __global__ void __launch_bounds__(DV * 4) rule_scan_kernel(const RuleArgs p) {
     for (int i = 0; i < 8; ++i) y[i] *= r * gain[i] * gate_act<true>(zf[i], p.gate_kind);
     if (t < total) *reinterpret_cast<uint4_*>(out + (long)t * p.ldo) = pack8(y);
     if constexpr (!AHEAD) {
-      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+      wait_vm();
       __syncthreads();
     }
   }
@@ -973,12 +1051,12 @@ __global__ void __launch_bounds__(DV * 4) rule_scan_kernel(const RuleArgs p) {
 
 template <int MODE, int DK, int DV, bool AHEAD>
 static void scan(const RuleArgs& a, hipStream_t s) {
-  constexpr int unit = (RowUnit<DK>::size + HeadUnit<DV>::size) * 16;
+  constexpr int unit = (RowUnit<DK, MODE == kChannel>::size + HeadUnit<DV>::size) * 16;
   constexpr int lds = AHEAD ? 2 * unit + kC * (DV + 4) * 4 : unit;
   static_assert(lds <= 160 * 1024, "prepared chunks in LDS");
   (void)hipFuncSetAttribute(reinterpret_cast<const void*>(rule_scan_kernel<MODE, DK, DV, AHEAD>),
                             hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-  rule_scan_kernel<MODE, DK, DV, AHEAD><<<dim3(a.heads, a.B), DV * 4, lds, s>>>(a);
+  rule_scan_kernel<MODE, DK, DV, AHEAD><<<a.heads * a.B, DV * 4, lds, s>>>(a);
 }
 
 template <int MODE, int DK, int DV>
@@ -997,11 +1075,7 @@ static void chunks(const RuleArgs& a, hipStream_t s) {
     rule_prep_head_kernel<DELTA, DK, DV><<<dim3(n, a.heads / (a.H / a.G), a.B), 512, lds, s>>>(a);
   }
   rule_solve_kernel<MODE, DK, DV><<<dim3((n + 3) / 4, a.heads, a.B), 256, 0, s>>>(a);
-  // one chunk ahead where no second workgroup of the CU would fill the wait
-  if constexpr (DK <= 128) {
-    if ((long)a.heads * a.B <= 384) return scan<MODE, DK, DV, true>(a, s);
-  }
-  scan<MODE, DK, DV, false>(a, s);
+  scan<MODE, DK, DV, (DK <= 128)>(a, s);
 }
 
 void launch_rule_chunks(const RuleArgs& a, hipStream_t s) {

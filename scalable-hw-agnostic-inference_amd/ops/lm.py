@@ -596,7 +596,7 @@ def _rule_run(x, gate, state, out, batch, shape: RuleShape, eps: float, commit, 
         # whole groups of heads with common queries and keys; rounds of equal size
         groups, per_channel = int(shape.kv_heads), "decay" in args and args["decay"].shape[1] != H
         size = H // groups
-        need = lambda n: (T // RULE_CHUNK + batch.B) * _K().rule_chunk_bytes(dk, dv, n * size, n * (size if per_channel else 1))
+        need = lambda n: (T // RULE_CHUNK + batch.B) * _K().rule_chunk_bytes(dk, dv, n * size, n * (size if per_channel else 1), per_channel)
         rounds = -(-groups // max(1, min(groups, RULE_WORKSPACE // need(1))))
         n = -(-groups // rounds)
         ws = torch.empty(need(n), dtype=torch.uint8, device=x.device)
