@@ -44,7 +44,7 @@ __device__ __forceinline__ float gate_act(float z, int kind) {
 // Thread: 4 columns x DK / RG rows of S.  S^T k and S^T q are taken from the decayed state in one pass: with kq = k . q,
 // o = S^T q + kq u.
 template <typename T, int MODE, int DK, int DV, int NT>
-__global__ void __launch_bounds__(NT) rule_rows_kernel(const RuleArgs p) {
+__global__ void __launch_bounds__(NT, NT > 256 ? 4 : 3) rule_rows_kernel(const RuleArgs p) {
   constexpr bool DELTA = MODE != kRetention;
   constexpr int NC = DV / 4, RG = NT / NC, R = DK / RG, NW = NT / 64, KW = DK / 64;
   static_assert(R % 4 == 0 && NC <= 64 && NT >= DV && NT >= 2 * DK, "shape");
@@ -65,15 +65,17 @@ __global__ void __launch_bounds__(NT) rule_rows_kernel(const RuleArgs p) {
   for (int i = 0; i < R; ++i) S[i] = old ? load4(st + (long)i * DV) : float4_{0.f, 0.f, 0.f, 0.f};
   const T* x = static_cast<const T*>(p.x);
   T* ring = DELTA ? static_cast<T*>(p.ring) + (long)max(slot, 0) * p.taps * channels : nullptr;
+  const int ring0 = DELTA ? pos0 % p.taps : 0;
   // channel ch of row t after its convolution and silu
   auto conv = [&](long t, int ch) {
-    float y = p.conv[(long)(p.taps - 1) * channels + ch] * load1(x + t * p.ldx + ch);
-#pragma unroll 4
+    const int row = (int)(t - t0);
+    float y = p.conv[(p.taps - 1) * channels + ch] * load1(x + t * p.ldx + ch);
+#pragma unroll 3
     for (int j = 1; j < p.taps; ++j) {
-      const int at = pos0 + (int)(t - t0) - j;               // its position
-      const bool here = t - j >= t0;
-      const T* src = here ? x + (t - j) * p.ldx + ch : ring + (long)(max(at, 0) % p.taps) * channels + ch;
-      if (here || (at >= 0 && slot >= 0)) y += p.conv[(long)(p.taps - 1 - j) * channels + ch] * load1(src);
+      const int m = ring0 + row - j;                         // before the step's first row: its place in the ring
+      const bool here = row >= j;
+      const T* src = here ? x + (t - j) * p.ldx + ch : ring + (m < 0 ? m + p.taps : m) * channels + ch;
+      if (here || (pos0 + row >= j && slot >= 0)) y += p.conv[(p.taps - 1 - j) * channels + ch] * load1(src);
     }
     return silu_exact(y);
   };
@@ -110,7 +112,7 @@ __global__ void __launch_bounds__(NT) rule_rows_kernel(const RuleArgs p) {
       }
     }
     __syncthreads();
-    float rq = 1.f, rk = rsqrtf((float)p.dim), gh = MODE == kRetention ? p.rate[h] : 1.f, beta = 1.f;
+    float rq = 1.f, rk = 1.f, gh = MODE == kRetention ? p.rate[h] : 1.f, beta = 1.f;
     if constexpr (DELTA) {
       float s0 = 0.f, s1 = 0.f;
 #pragma unroll
@@ -130,6 +132,7 @@ __global__ void __launch_bounds__(NT) rule_rows_kernel(const RuleArgs p) {
     float kq = 0.f;
 #pragma unroll
     for (int i = 0; i < R; i += 4) {
+      __builtin_amdgcn_sched_barrier(0);          // four rows of k and q in registers at a time
       const float4_ k = load4(sk + r0 + i) * rk, q = load4(sq + r0 + i) * rq;
       const float4_ f = MODE == kChannel ? load4(sg + r0 + i) : float4_{gh, gh, gh, gh};
 #pragma unroll
@@ -171,6 +174,7 @@ __global__ void __launch_bounds__(NT) rule_rows_kernel(const RuleArgs p) {
       const float4_ u = beta * (v - sum);
 #pragma unroll
       for (int i = 0; i < R; i += 4) {
+        __builtin_amdgcn_sched_barrier(0);
         const float4_ k = load4(sk + r0 + i) * rk;
 #pragma unroll
         for (int j = 0; j < 4; ++j) S[i + j] += k[j] * u;

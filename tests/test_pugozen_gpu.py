@@ -68,3 +68,12 @@ def test_trace_run_program(cuda, tmp_path):
         assert r.returncode == 0, r.stderr[-2000:]
         said = [ln for ln in r.stdout.splitlines() if ln.startswith("done")]
         C.check_replay_files(c, toks, out, said, dtype)
+
+
+def test_prompts_in_rounds(cuda, monkeypatch):
+    """Heads whose prepared chunks do not fit the workspace together run in several rounds."""
+    monkeypatch.setattr(C.lm, "RULE_WORKSPACE", 1)
+    C.check_mixers(cuda, torch.bfloat16)
+    monkeypatch.setattr(C.lm, "RULE_WORKSPACE", 1 << 20)
+    C.check_delta(cuda, torch.bfloat16)
+    C.check_retention(cuda, torch.bfloat16)
