@@ -150,7 +150,7 @@ static void stream(const GemmArgs& a, hipStream_t s) {
     if constexpr (epi_in(EC, EPI_NONE)) {         // partial sums
       if (rows <= 16) GO(1, 1, 4, 4);
       else if (rows <= 32) GO(2, 2, 4, 4);
-      else if (a.N < 2560 && a.K < 12288) GO(4, 2, 4, 3);
+      else if (a.N < 2560 && a.K < 16384) GO(4, 2, 4, 3);
       else GO(4, 4, 4, 2);
     }
   } else if (!a.tiles && a.K <= 256) {            // too few k-steps to split over many waves
@@ -163,8 +163,10 @@ static void stream(const GemmArgs& a, hipStream_t s) {
   else if (a.N < 5120) GO(2, 2, 8, 2);
   else if (rows <= 32) GO(2, 4, 4, 3);
   else if (a.N < 8192) GO(4, 2, 4, 2);
-  else if (a.N < 16384) GO(4, 4, 4, 2);
-  else GO(4, 4, 2, 2);
+  else if (H && a.N <= 12288) GO(4, 3, 4, 2);    // up to 20480 columns: as few as give every CU one workgroup
+  else if (a.N <= 16384) GO(4, 4, 4, 3);
+  else if (H && a.N <= 20480) GO(4, 5, 4, 2);
+  else GO(4, 4, 2, 3);
 #undef GO
   SHAI_CHECK_LAUNCH();
 }
