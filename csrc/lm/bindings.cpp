@@ -236,10 +236,11 @@ void lm_gemm(const Tensor& A, const Tensor& W, const Tensor& C, const optional<T
   const long lim = 0x7fffffffL, esize = f32 ? 4 : 2, osize = g.out_f32 ? 4 : 2;
   const bool tile = !f32 && (g.tiles ? bm >= 128 && (long)g.a_rows * g.lda * 2 < lim : g.M > 64) && (long)g.N * g.K * 2 < lim;
   if (!tile) return shai_lm::launch_gemm(g, f32, stream());
-  // the tiled kernel addresses A with 32-bit offsets: a longer A runs in parts
-  const int rows = g.tiles ? g.M : (int)std::min<long>(g.M, std::max<long>(256, (lim / (g.lda * 2)) / 256 * 256));
-  SHAI_CHECK(g.tiles || (long)rows * g.lda * 2 < lim, "lm_gemm: rows of A are too long");
+  // the tiled kernel addresses A with 32-bit offsets: a longer A runs in equal parts
   const int total = g.M;
+  const long most = std::max<long>(256, (lim / (g.lda * 2)) / 256 * 256), parts = (total + most - 1) / most;
+  const int rows = g.tiles ? total : (int)std::min<long>(total, ((total + parts - 1) / parts + 255) / 256 * 256);
+  SHAI_CHECK(g.tiles || (long)rows * g.lda * 2 < lim, "lm_gemm: rows of A are too long");
   for (int at = 0; at < total; at += rows) {
     shai_lm::GemmArgs part = g;
     if (!g.tiles) {
