@@ -829,7 +829,7 @@ void rule_chunks(const Tensor& x, const Tensor& gate, const Tensor& state, const
                  const Tensor& rate, const optional<Tensor>& decay, const optional<Tensor>& beta, const optional<Tensor>& conv,
                  const optional<Tensor>& bias, const optional<Tensor>& gain, const optional<Tensor>& ring,
                  const optional<Tensor>& rope, const Tensor& q_start, const Tensor& q_lens, const Tensor& ws, int64_t max_q,
-                 int64_t head0, int64_t heads) {
+                 int64_t head0, int64_t heads, int64_t seg, const optional<Tensor>& seg_ws) {
   shai_lm::RuleArgs a = rule_args(x, gate, state, out, pos, slots, kv_heads, dim, vdim, gate_kind, eps, rate, decay, beta,
                                   conv, bias, gain, ring, rope, q_start, q_lens);
   SHAI_CHECK(x.scalar_type() == at::kBFloat16, "chunks: bf16 rows");
@@ -845,7 +845,22 @@ void rule_chunks(const Tensor& x, const Tensor& gate, const Tensor& state, const
   a.head0 = head0;
   a.heads = heads;
   a.max_q = std::min<int64_t>(max_q, a.T);
+  a.seg = (a.max_q + 31) / 32 * 32;
+  a.cuts = 1;
+  if (seg > 0 && seg < a.max_q) {
+    SHAI_CHECK(seg % 32 == 0 && seg_ws, "rule_chunks: segments are whole chunks and have a workspace");
+    check(*seg_ws, at::kByte, "seg_ws");
+    a.seg = seg;
+    a.cuts = (a.max_q + a.seg - 1) / a.seg;
+    SHAI_CHECK(seg_ws->numel() >= ((long)a.T / seg + a.B) * shai_lm::rule_segment_bytes(a.dk, a.dv, heads, a.mode == 0) &&
+                   (long)heads * a.B * a.cuts * 8 < 0x7fffffffL, "rule_chunks: workspace of segments");
+    a.seg_ws = static_cast<float*>(seg_ws->data_ptr());
+  }
   if (a.T > 0) shai_lm::launch_rule_chunks(a, stream());
+}
+
+int64_t rule_segment_bytes(int64_t dk, int64_t dv, int64_t heads, bool retention) {
+  return shai_lm::rule_segment_bytes(dk, dv, heads, retention);
 }
 
 int64_t rule_chunk_bytes(int64_t dk, int64_t dv, int64_t heads, int64_t keys, bool channel) {
@@ -1164,7 +1179,8 @@ TORCH_LIBRARY_FRAGMENT(shai, m) {
   m.def("head_prep(Tensor(a!) qkvg, Tensor(b!) k_cache, Tensor(c!) v_cache, Tensor slots, int heads, Tensor rope, int dim, float eps, bool own_kv, bool tied=False, Tensor? q_gain=None, Tensor? k_gain=None) -> ()");
   m.def("hgrn2(Tensor qv, Tensor z, Tensor bias, Tensor lower, Tensor gain, Tensor(a!) state, Tensor(b!) out, Tensor pos, Tensor? q_start, Tensor? q_lens, Tensor slots, Tensor(c!) ws, int max_q, int len, int vdim, float eps) -> ()");
   m.def("rule_rows(Tensor x, Tensor gate, Tensor(a!) state, Tensor(b!) out, Tensor pos, Tensor slots, int kv_heads, int dim, int vdim, int gate_kind, float eps, Tensor rate, Tensor? decay=None, Tensor? beta=None, Tensor? conv=None, Tensor? bias=None, Tensor? gain=None, Tensor(c!)? ring=None, Tensor? rope=None, Tensor? q_start=None, Tensor? q_lens=None) -> ()");
-  m.def("rule_chunks(Tensor x, Tensor gate, Tensor(a!) state, Tensor(b!) out, Tensor pos, Tensor slots, int kv_heads, int dim, int vdim, int gate_kind, float eps, Tensor rate, Tensor? decay=None, Tensor? beta=None, Tensor? conv=None, Tensor? bias=None, Tensor? gain=None, Tensor? ring=None, Tensor? rope=None, *, Tensor q_start, Tensor q_lens, Tensor(c!) ws, int max_q, int head0, int heads) -> ()");
+  m.def("rule_chunks(Tensor x, Tensor gate, Tensor(a!) state, Tensor(b!) out, Tensor pos, Tensor slots, int kv_heads, int dim, int vdim, int gate_kind, float eps, Tensor rate, Tensor? decay=None, Tensor? beta=None, Tensor? conv=None, Tensor? bias=None, Tensor? gain=None, Tensor? ring=None, Tensor? rope=None, *, Tensor q_start, Tensor q_lens, Tensor(c!) ws, int max_q, int head0, int heads, int seg=0, Tensor(d!)? seg_ws=None) -> ()");
+  m.def("rule_segment_bytes(int dk, int dv, int heads, bool retention) -> int", &rule_segment_bytes);
   m.def("rule_chunk_bytes(int dk, int dv, int heads, int keys, bool channel) -> int", &rule_chunk_bytes);
   m.def("ring_commit(Tensor x, Tensor(a!) ring, Tensor pos, Tensor q_start, Tensor q_lens, Tensor slots) -> ()");
   m.def("gated_attn_prefill(Tensor qkvg, Tensor k_cache, Tensor v_cache, Tensor(a!) o, Tensor block_table, Tensor ctx_lens, Tensor q_lens, Tensor q_start, int max_q, int heads, int chunk, float scale, bool window=False, bool per_element=False, bool own_kv=True, Tensor? temp=None, Tensor? sink=None, float out_scale=1.) -> ()");

@@ -297,6 +297,8 @@ struct RuleArgs {          // delta rule (mode 1: a decay per head, 2: per key c
   const int* slots;        // [B], -1: none
   void* ws;                // chunks: ws_chunks = T / 32 + B prepared chunks (rule_chunk_bytes each)
   long ws_chunks;
+  float* seg_ws;           // T / seg + B units (rule_segment_bytes each), if sequences are cut
+  int seg, cuts;           // rows of a segment (a multiple of 32), segments of the longest sequence
   int T, B, H, G, dk, dv, dim, vdim, taps, rot, gate_kind, max_q, head0, heads;
   float eps;
 };
@@ -304,6 +306,8 @@ void launch_rule_rows(const RuleArgs& a, bool f32, hipStream_t s);     // row by
 void launch_rule_chunks(const RuleArgs& a, hipStream_t s);             // bf16, 32 rows at a time; heads head0 .. of a prefill step
 // workspace of one chunk of `heads` heads and `keys` heads of queries and keys (those of every head with a decay per channel)
 long rule_chunk_bytes(int dk, int dv, int heads, int keys, bool channel);
+// workspace of a segment of `heads` heads
+long rule_segment_bytes(int dk, int dv, int heads, bool retention);
 
 struct RingArgs {          // the last inputs of a prefill step into the rings
   const void* x;

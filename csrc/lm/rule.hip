@@ -16,6 +16,9 @@
 //          solve (a wave per chunk and head): the inverse, and decays per head.
 //          scan (a workgroup per sequence and head): chunk after chunk, each wave 16 columns of S (registers); prepared
 //          chunks are loaded to LDS one ahead.
+//          Few long sequences are cut into segments.  A segment is affine in the state, S' = M S + L: a first scan starts
+//          from zero for L and, without values, from the identity for M; `link` chains the segments' states; then every
+//          segment is scanned from its own.
 //          Quotients of decays come from differences of running logarithms.  A decay per channel enters the matrix products
 //          through a reference between the two rows: the border of the 16-row halves, that of a half's 8-row blocks, or a
 //          block's fourth row.  Operands of matrix products are a bf16 value plus its bf16 remainder; sums are fp32.
@@ -814,8 +817,14 @@ __device__ __forceinline__ uint32_t lds_address(const void* p) {
   return (uint32_t)(uintptr_t)(__attribute__((address_space(3))) const void*)p;
 }
 
+// Segment j of sequence b: its last state L [DK][DV], after `link` the next segment's first; of the delta rule then M [DK][DK].
+__device__ __forceinline__ float* segment_unit(const RuleArgs& p, int b, int j, int head, long size) {
+  return p.seg_ws + (((long)p.q_start[b] / p.seg + b + j) * p.heads + head) * size;
+}
+
 // Waves of 16 columns of S each.  A prepared chunk goes to LDS by DMA, one chunk ahead where two fit (AHEAD).
-template <int MODE, int DK, int DV, bool AHEAD>
+// TOTALS: L and M of every segment but a sequence's last.
+template <int MODE, int DK, int DV, bool AHEAD, bool TOTALS>
 __global__ void __launch_bounds__(DV * 4) __attribute__((amdgpu_waves_per_eu(DV / 64, DV / 64)))
 rule_scan_kernel(const RuleArgs p) {
   constexpr bool DELTA = MODE != kRetention, CHANNEL = MODE == kChannel;
@@ -831,20 +840,26 @@ rule_scan_kernel(const RuleArgs p) {
   const int tid = threadIdx.x, lane = tid & 63, w = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int g = lane >> 4, c16 = lane & 15;
   // heads that share rows follow each other on one XCD (workgroups go round them)
-  const int jobs = p.heads * p.B, q8 = jobs >> 3, r8 = jobs & 7, xcd = blockIdx.x & 7;
+  constexpr int KINDS = TOTALS && DELTA ? 1 + (DK + DV - 1) / DV : 1;     // L, then DV columns of M each
+  constexpr long SEGMENT = DK * (DELTA ? DV + DK : DV);
+  const int cuts = TOTALS ? p.cuts - 1 : p.cuts;
+  const int jobs = p.heads * p.B * cuts * KINDS, q8 = jobs >> 3, r8 = jobs & 7, xcd = blockIdx.x & 7;
   const int job = (xcd < r8 ? xcd * (q8 + 1) : r8 * (q8 + 1) + (xcd - r8) * q8) + (blockIdx.x >> 3);
-  const int b = job / p.heads, hi = job % p.heads, h = p.head0 + hi, group = CHANNEL ? 1 : p.H / p.G;
-  const int total = p.q_lens[b];
-  if (total < 1) return;
+  const int unit = job / p.heads, hi = job % p.heads, h = p.head0 + hi, group = CHANNEL ? 1 : p.H / p.G;
+  const int kind = unit % KINDS, j0 = unit / KINDS % cuts, b = unit / KINDS / cuts;
+  const long begin = (long)j0 * p.seg, left = p.q_lens[b] - begin;
+  if (left < 1 || (TOTALS && (left <= p.seg || (kind && j0 == 0)))) return;
+  const int total = (int)min(left, (long)p.seg);
   const int chunks = (total + kC - 1) / kC;
-  const long row0 = p.q_start[b];
+  const long row0 = p.q_start[b] + begin;
   const int slot = p.slots[b];
-  const bool old = slot >= 0 && p.pos[row0] > 0;
+  const bool old = slot >= 0 && p.pos[p.q_start[b]] > 0;
   float* st = p.state + ((long)max(slot, 0) * p.H + h) * DK * DV + 16 * w + c16;
 
   const int keys = p.heads / group;
-  const uint4_* head = head_unit(p, first_chunk(p, b), hi, HU::size) + lane;
-  const uint4_* rows = row_unit(p, first_chunk(p, b), hi / group, keys, U::size, HU::size) + lane;
+  const long chunk0 = first_chunk(p, b) + begin / kC;
+  const uint4_* head = head_unit(p, chunk0, hi, HU::size) + lane;
+  const uint4_* rows = row_unit(p, chunk0, hi / group, keys, U::size, HU::size) + lane;
   const uint32_t at0 = __builtin_amdgcn_readfirstlane(lds_address(staged));
   auto stage = [&](int c) {
     const uint32_t dst = at0 + (AHEAD && (c & 1) ? SIZE * 16 : 0);
@@ -853,7 +868,7 @@ rule_scan_kernel(const RuleArgs p) {
 #pragma unroll
     for (int j = 0; j < (U::size / 64 + NW - 1) / NW; ++j) {
       const int i = j * NW + w;
-      if (i < U::size / 64) dma16_unwaited(su + 64 * i, dst + 1024 * i);
+      if (i < U::size / 64 && !(TOTALS && 64 * i >= U::qd && 64 * i < U::qd + U::part)) dma16_unwaited(su + 64 * i, dst + 1024 * i);
     }
 #pragma unroll
     for (int j = 0; j < ((HU::size - FH) / 64 + NW - 1) / NW; ++j) {
@@ -863,10 +878,20 @@ rule_scan_kernel(const RuleArgs p) {
   };
   stage(0);
   float4_ S[NK];                                  // rows 16 i + 4 g .., the wave's columns
+  if (TOTALS && kind) {
 #pragma unroll
-  for (int i = 0; i < NK; ++i)
+    for (int i = 0; i < NK; ++i)
 #pragma unroll
-    for (int j = 0; j < 4; ++j) S[i][j] = old ? st[(long)(16 * i + 4 * g + j) * DV] : 0.f;
+      for (int j = 0; j < 4; ++j) S[i][j] = 16 * i + 4 * g + j == (kind - 1) * DV + 16 * w + c16 ? 1.f : 0.f;
+  } else {
+    const bool linked = !TOTALS && j0 > 0;
+    const float* from = linked ? segment_unit(p, b, j0 - 1, hi, SEGMENT) + 16 * w + c16 : st;
+    const bool some = linked || (old && j0 == 0);
+#pragma unroll
+    for (int i = 0; i < NK; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) S[i][j] = some ? from[(long)(16 * i + 4 * g + j) * DV] : 0.f;
+  }
   // pieces of this lane: 16 bytes of row c16, 8 bytes of row 4 g + tq (channels 32 i ..: i even, odd), and of its values
   const int tq = c16 >> 2, tp = c16 & 3;
   int row_at[2], col_at[2];
@@ -880,7 +905,7 @@ rule_scan_kernel(const RuleArgs p) {
   const int er = tid / TPR, ec = tid % TPR * 8;
   float gain[8];
 #pragma unroll
-  for (int i = 0; i < 8; ++i) gain[i] = DELTA ? p.gain[ec + i] : 1.f;
+  for (int i = 0; i < 8; ++i) gain[i] = DELTA && !TOTALS ? p.gain[ec + i] : 1.f;
   const float inv_vdim = 1.f / (float)p.vdim;
   const bf16_t* gate = static_cast<const bf16_t*>(p.gate) + row0 * p.ldg + h * DV + ec;
   bf16_t* out = static_cast<bf16_t*>(p.out) + row0 * p.ldo + h * DV + ec;
@@ -890,7 +915,8 @@ rule_scan_kernel(const RuleArgs p) {
     const uint4_* cur = staged + (AHEAD ? (c & 1) * SIZE : 0);
     const uint4_* curh = cur + U::size;
     const int t = c * kC + er;
-    const uint4_ z = *reinterpret_cast<const uint4_*>(gate + (long)min(t, total - 1) * p.ldg);
+    uint4_ z = {};
+    if constexpr (!TOTALS) z = *reinterpret_cast<const uint4_*>(gate + (long)min(t, total - 1) * p.ldg);
     if (AHEAD && c + 1 < chunks) stage(c + 1);
     auto frag = [&](int place) {
       return Split{__builtin_bit_cast(bf16x8, curh[place + lane]), __builtin_bit_cast(bf16x8, curh[place + 64 + lane])};
@@ -918,16 +944,16 @@ rule_scan_kernel(const RuleArgs p) {
     auto hold = [] {
       if constexpr (AHEAD) __builtin_amdgcn_sched_barrier(0);
     };
-    constexpr int NR = DELTA ? 4 : 2;             // sums of a step: K S (rows 0 .., 16 ..), then Q S
-    float4_ acc[NR] = {};
-    Split f[NI][NR];
+    constexpr int NR = (DELTA ? 2 : 0) + (TOTALS ? 0 : 2);     // sums of a step: K S (rows 0 .., 16 ..), then Q S
+    float4_ acc[NR + 1] = {};
+    Split f[NI][NR + 1];
     auto load_rows = [&](int i) {
 #pragma unroll
       for (int j = 0; j < NR; ++j) f[i][j] = row(DELTA && j < 2 ? U::kd : U::qd, j & 1, i);
     };
-    load_rows(0);
+    if constexpr (NR > 0) load_rows(0);
 #pragma unroll
-    for (int i = 0; i < NI; ++i) {
+    for (int i = 0; i < (NR > 0 ? NI : 0); ++i) {
       if (i + 1 < NI) load_rows(i + 1);
       hold();
       const Split sf = split8(S[2 * i], S[2 * i + 1]);
@@ -938,10 +964,14 @@ rule_scan_kernel(const RuleArgs p) {
 #pragma unroll
       for (int j = 0; j < NR; ++j) acc[j] = mac(f[i][j].hi, sf.lo, acc[j]);
     }
-    float4_* O = acc + NR - 2;
+    float4_* O = acc + (DELTA ? 2 : 0);           // not with TOTALS
     const float* dec = reinterpret_cast<const float*>(curh + HU::dec);
     const uint4_ vr = column(curh + HU::vf, DV / 4, value_at);
-    Split pf[2] = {frag(HU::pf), frag(HU::pf + 128)}, tf[2];
+    Split pf[2], tf[2];
+    if constexpr (!TOTALS) {
+      pf[0] = frag(HU::pf);
+      pf[1] = frag(HU::pf + 128);
+    }
     if constexpr (DELTA) {
       tf[0] = frag(HU::tf);
       tf[1] = frag(HU::tf + 128);
@@ -972,9 +1002,10 @@ rule_scan_kernel(const RuleArgs p) {
     for (int u = 0; u < 2; ++u) {
       v[u] = float4_{__uint_as_float(vr[2 * u] << 16), __uint_as_float(vr[2 * u] & 0xffff0000u),
                      __uint_as_float(vr[2 * u + 1] << 16), __uint_as_float(vr[2 * u + 1] & 0xffff0000u)};
+      if (TOTALS && kind) v[u] = float4_{0.f, 0.f, 0.f, 0.f};
       if constexpr (!CHANNEL) {                   // decays from the chunk's start
         if constexpr (DELTA) acc[u] *= from[u];
-        O[u] *= from[u];
+        if constexpr (!TOTALS) O[u] *= from[u];
       }
     }
     Split uf;                                     // U, its rows decayed to the chunk's end for the state
@@ -987,13 +1018,15 @@ rule_scan_kernel(const RuleArgs p) {
 #pragma unroll
       for (int u = 0; u < 2; ++u) v[u] = mac(tf[u].hi, rf.lo, v[u]);
       uf = split8(v[0], v[1]);
+      if constexpr (!TOTALS) {
 #pragma unroll
-      for (int u = 0; u < 2; ++u) O[u] = mac(pf[u].hi, uf.hi, O[u]);
+        for (int u = 0; u < 2; ++u) O[u] = mac(pf[u].hi, uf.hi, O[u]);
 #pragma unroll
-      for (int u = 0; u < 2; ++u) O[u] = mac(pf[u].lo, uf.hi, O[u]);
+        for (int u = 0; u < 2; ++u) O[u] = mac(pf[u].lo, uf.hi, O[u]);
 #pragma unroll
-      for (int u = 0; u < 2; ++u) O[u] = mac(pf[u].hi, uf.lo, O[u]);
-    } else {
+        for (int u = 0; u < 2; ++u) O[u] = mac(pf[u].hi, uf.lo, O[u]);
+      }
+    } else if constexpr (!TOTALS) {
       const bf16x8 vf = __builtin_bit_cast(bf16x8, vr);
 #pragma unroll
       for (int u = 0; u < 2; ++u) O[u] = mac(pf[u].hi, vf, O[u]);
@@ -1018,6 +1051,15 @@ rule_scan_kernel(const RuleArgs p) {
       for (int j = i; j < i + 2; ++j) S[j] = mac(kc[j].hi, uf.lo, S[j]);
     }
 
+    if constexpr (TOTALS) {
+      if constexpr (!AHEAD) {
+        __syncthreads();
+        if (c + 1 < chunks) stage(c + 1);
+      }
+      wait_vm();
+      __syncthreads();
+      continue;
+    }
     __syncthreads();                              // every wave is done with the chunk and the last one's outputs
 #pragma unroll
     for (int u = 0; u < 2; ++u)
@@ -1045,7 +1087,16 @@ rule_scan_kernel(const RuleArgs p) {
       __syncthreads();
     }
   }
-  if (slot >= 0) {
+  if constexpr (TOTALS) {
+    const int col = (kind ? (kind - 1) * DV : 0) + 16 * w + c16, width = kind ? DK : DV;
+    float* to = segment_unit(p, b, j0, hi, SEGMENT) + (kind ? DK * DV : 0) + col;
+    if (col < width) {
+#pragma unroll
+      for (int i = 0; i < NK; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) to[(long)(16 * i + 4 * g + j) * width] = S[i][j];
+    }
+  } else if (slot >= 0 && left <= p.seg) {
 #pragma unroll
     for (int i = 0; i < NK; ++i)
 #pragma unroll
@@ -1053,15 +1104,69 @@ rule_scan_kernel(const RuleArgs p) {
   }
 }
 
+// The first state of every segment but a sequence's first: S = M S + L, fp32.  A workgroup per sequence, head and 16 columns, a
+// wave per 16 rows.
+template <bool DELTA, int DK, int DV>
+__global__ void __launch_bounds__(DK * 4) rule_link_kernel(const RuleArgs p) {
+  constexpr long SEGMENT = DK * (DELTA ? DV + DK : DV);
+  constexpr int NQ = DELTA ? DK / 16 : 1;
+  __shared__ __attribute__((aligned(16))) float x[DELTA ? 16 * (DK + 4) : 1];      // the state, a column after the other
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, g = lane >> 4, c16 = lane & 15;
+  const int b = blockIdx.z, hi = blockIdx.y, col = blockIdx.x * 16 + c16;
+  const int total = p.q_lens[b], links = (total - 1) / p.seg;                      // segments with one behind them
+  if (links < 2) return;
+  auto unit = [&](int j) { return segment_unit(p, b, j, hi, SEGMENT); };
+  auto last = [&](int j) {
+    float4_ y;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) y[i] = unit(j)[(long)(16 * w + 4 * g + i) * DV + col];
+    return y;
+  };
+  float4_ S = last(0);
+  const float fixed = DELTA ? 0.f : __builtin_amdgcn_exp2f((float)p.seg * fmaxf(p.rate[p.H + p.head0 + hi], kLeast));
+  for (int j = 1; j < links; ++j) {
+    float4_ next = last(j);
+    if constexpr (DELTA) {
+      float4_ m[NQ];
+#pragma unroll
+      for (int q = 0; q < NQ; ++q) m[q] = load4(unit(j) + DK * DV + (16 * w + c16) * DK + 16 * q + 4 * g);
+      __syncthreads();                            // the last state is read
+      *reinterpret_cast<float4_*>(x + c16 * (DK + 4) + 16 * w + 4 * g) = S;
+      __syncthreads();
+#pragma unroll
+      for (int q = 0; q < NQ; ++q) {
+        const float4_ y = load4(x + c16 * (DK + 4) + 16 * q + 4 * g);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) next = __builtin_amdgcn_mfma_f32_16x16x4f32(m[q][i], y[i], next, 0, 0, 0);
+      }
+    } else {
+      next += fixed * S;
+    }
+    S = next;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) unit(j)[(long)(16 * w + 4 * g + i) * DV + col] = S[i];
+  }
+}
+
 template <int MODE, int DK, int DV, bool AHEAD>
 static void scan(const RuleArgs& a, hipStream_t s) {
+  constexpr bool DELTA = MODE != kRetention;
   constexpr int unit = (RowUnit<DK, MODE == kChannel>::size + HeadUnit<DV>::size) * 16;
   constexpr int lds = AHEAD ? 2 * unit + kC * (DV + 4) * 4 : unit;
   static_assert(lds <= 160 * 1024, "prepared chunks in LDS");
-  (void)hipFuncSetAttribute(reinterpret_cast<const void*>(rule_scan_kernel<MODE, DK, DV, AHEAD>),
+  if (a.cuts > 1) {
+    constexpr int kinds = DELTA ? 1 + (DK + DV - 1) / DV : 1;
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(rule_scan_kernel<MODE, DK, DV, AHEAD, true>),
+                              hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    rule_scan_kernel<MODE, DK, DV, AHEAD, true><<<a.heads * a.B * (a.cuts - 1) * kinds, DV * 4, lds, s>>>(a);
+    rule_link_kernel<DELTA, DK, DV><<<dim3(DV / 16, a.heads, a.B), DK * 4, 0, s>>>(a);
+  }
+  (void)hipFuncSetAttribute(reinterpret_cast<const void*>(rule_scan_kernel<MODE, DK, DV, AHEAD, false>),
                             hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-  rule_scan_kernel<MODE, DK, DV, AHEAD><<<a.heads * a.B, DV * 4, lds, s>>>(a);
+  rule_scan_kernel<MODE, DK, DV, AHEAD, false><<<a.heads * a.B * a.cuts, DV * 4, lds, s>>>(a);
 }
+
+long rule_segment_bytes(int dk, int dv, int heads, bool retention) { return 4L * heads * dk * (retention ? dv : dv + dk); }
 
 template <int MODE, int DK, int DV>
 static void chunks(const RuleArgs& a, hipStream_t s) {

@@ -580,6 +580,15 @@ class RuleShape:
     gate: int = GATE_SILU
 
 
+def rule_segment(rows: int, scans: int, retention: bool) -> int:
+    """Rows of the segments that sequences of up to ``rows`` rows are cut into, 0: not cut.  ``scans``: sequences times heads,
+    a workgroup each when uncut.  A first scan over the segments takes one workgroup each for retention and two for the delta
+    rule; both scans together must be shorter than one over the whole sequence."""
+    chunks, per = -(-rows // RULE_CHUNK), 1 if retention else 2
+    n = min((256 // scans + 2 * per - 1) // per, chunks // 4)
+    return -(-chunks // n) * RULE_CHUNK if n >= 3 else 0
+
+
 def _rule_run(x, gate, state, out, batch, shape: RuleShape, eps: float, commit, **args):
     """The launches of one step: decode and fp32 rows one by one; bf16 portions in chunks, as many heads at a time as the
     workspace holds."""
@@ -600,9 +609,12 @@ def _rule_run(x, gate, state, out, batch, shape: RuleShape, eps: float, commit, 
         rounds = -(-groups // max(1, min(groups, RULE_WORKSPACE // need(1))))
         n = -(-groups // rounds)
         ws = torch.empty(need(n), dtype=torch.uint8, device=x.device)
+        seg = rule_segment(int(batch.S), -(-T // int(batch.S)) * n * size, "decay" not in args)
+        seg_ws = torch.empty((T // seg + batch.B) * _K().rule_segment_bytes(dk, dv, n * size, "decay" not in args),
+                             dtype=torch.uint8, device=x.device) if seg else None
         for g in range(0, groups, n):
             _K().rule_chunks(x, gate, state, out, ws=ws, max_q=int(batch.S), head0=g * size, heads=min(n, groups - g) * size,
-                             **args)
+                             seg=seg, seg_ws=seg_ws, **args)
     if commit is not None:
         _K().ring_commit(x, commit, batch.positions, batch.q_start, batch.q_lens, batch.state_slots)
 

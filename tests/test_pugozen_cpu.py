@@ -158,3 +158,19 @@ def test_bench_option_measures_every_model(monkeypatch):
     for cfg in cfgs.values():
         r = dd.measure(cfg, 2, 40, 3, repeats=1, device="cpu")
         assert r["prefill_tok_s"] > 0 and r["decode_tok_s"] > 0
+
+
+def test_segments_of_prompts():
+    """Whole chunks, at least four to a segment; both scans of a cut prompt are shorter than one over all of it, and the first
+    one's workgroups run at once."""
+    for retention in (False, True):
+        for scans in (1, 3, 16, 32, 64, 100, 256, 5000):
+            for rows in (1, 31, 384, 385, 1000, 1024, 8192, 100000):
+                seg = C.lm.rule_segment(rows, scans, retention)
+                if not seg:
+                    continue
+                cuts = -(-rows // seg)
+                assert seg % C.lm.RULE_CHUNK == 0 and seg >= 4 * C.lm.RULE_CHUNK and cuts >= 3 and 2 * seg < rows
+                assert scans * ((cuts - 1) if retention else 2 * cuts - 3) <= 256
+    assert C.lm.rule_segment(8192, 16, False) == 928 and C.lm.rule_segment(8192, 16, True) == 512
+    assert not C.lm.rule_segment(1024, 128, False) and not C.lm.rule_segment(100, 1, True)

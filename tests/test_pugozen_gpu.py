@@ -77,3 +77,11 @@ def test_prompts_in_rounds(cuda, monkeypatch):
     monkeypatch.setattr(C.lm, "RULE_WORKSPACE", 1 << 20)
     C.check_delta(cuda, torch.bfloat16)
     C.check_retention(cuda, torch.bfloat16)
+
+
+@pytest.mark.parametrize("rows", [32, 96])
+def test_prompts_in_segments(cuda, monkeypatch, rows):
+    """Prompts cut into segments that are scanned side by side: at every head size, in batches of unequal lengths."""
+    monkeypatch.setattr(C.lm, "rule_segment", lambda *_: rows)
+    for check in (C.check_delta, C.check_delta_memory, C.check_retention, C.check_mixers):
+        check(cuda, torch.bfloat16)
