@@ -43,7 +43,7 @@ import torch
 
 from ..utils import profiling as prof
 from .. import ops
-from . import new_graph
+from . import capture, new_graph
 from ..models.llama import KV_BLOCK, Batch, LlamaConfig
 from ..models.registry import config_from_path, model_class
 from ..parallel.state import tp
@@ -240,7 +240,7 @@ class _DecodeGraph:
                     self._program()
             torch.cuda.current_stream().wait_stream(s)
             self.graph = new_graph(dev)
-            with torch.cuda.graph(self.graph):
+            with capture(self.graph):
                 self._program()
             engine.last_tokens.copy_(saved)
 

@@ -268,3 +268,37 @@ def test_decode_attention_rope_qkv_cpu_fallback_matches_two_step():
     want = ops.decode_attention_rope(qkv, kc2, vc2, bt, lens, pos, cos, sin, slots, H, Hk)
     assert torch.equal(kc, kc2) and torch.equal(vc, vc2)
     assert torch.allclose(o.float(), want.float(), atol=1e-2, rtol=1e-2)
+
+
+def test_no_garbage_collection_during_a_capture(monkeypatch):
+    """What other engines left in reference cycles is destroyed before or after a graph's capture, not in it; the collector is
+    on again afterwards, also after an error."""
+    import contextlib
+    import gc
+    from shai_amd.engines import capture
+    freed = []
+
+    class Left:
+        def __init__(self):
+            self.me = self
+
+        def __del__(self):
+            freed.append(1)
+
+    monkeypatch.setattr(torch.cuda, "graph", lambda g, **kw: contextlib.nullcontext())
+    old = gc.get_threshold()
+    gc.collect()
+    gc.set_threshold(1, 1, 1)
+    try:
+        with capture(None):
+            Left()
+            keep = [[i] for i in range(1000)]
+            assert not freed and not gc.isenabled()
+        keep += [[i] for i in range(1000)]
+        assert gc.isenabled() and freed
+        with pytest.raises(RuntimeError):
+            with capture(None):
+                raise RuntimeError
+        assert gc.isenabled()
+    finally:
+        gc.set_threshold(*old)

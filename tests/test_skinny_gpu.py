@@ -3,6 +3,7 @@ import pytest
 import torch
 
 from shai_amd import ops
+from shai_amd.engines import capture
 
 pytestmark = pytest.mark.gpu
 SKINNY = 1000
@@ -93,7 +94,7 @@ def test_skinny_graph_replay_rearms_tickets(cuda):
     with torch.cuda.stream(s):
         ops.gemm_into(x, w, out, force_cfg=SKINNY_FIX + 8)
     torch.cuda.current_stream().wait_stream(s)
-    with torch.cuda.graph(g):
+    with capture(g):
         for _ in range(3):  # back-to-back launches reuse the same tickets
             ops.gemm_into(x, w, out, force_cfg=SKINNY_FIX + 8)
     for i in range(5):
@@ -337,7 +338,7 @@ def test_skinny_fixup_concurrent_streams_and_many_tiles(cuda):
         ops.gemm_into(x, w, gout, force_cfg=SKINNY_FIX + kg)
     torch.cuda.current_stream().wait_stream(side)
     g = torch.cuda.CUDAGraph()
-    with torch.cuda.graph(g):
+    with capture(g):
         for _ in range(4):
             ops.gemm_into(x, w, gout, force_cfg=SKINNY_FIX + kg)
     eout = torch.empty_like(ref)
@@ -415,7 +416,7 @@ def test_skinny2_glu_residual_and_graph(cuda, cfg):
         ops.gemm_into(x, w, o2, force_cfg=cfg)
     torch.cuda.current_stream().wait_stream(s)
     g = torch.cuda.CUDAGraph()
-    with torch.cuda.graph(g):
+    with capture(g):
         for _ in range(3):
             ops.gemm_into(x, w, o2, force_cfg=cfg)
     for _ in range(3):
