@@ -1,4 +1,4 @@
-"""What the tests of the layer-list decoders (Golulix, Faledra, Nalizen) share: cases on the framework's engine, driven by
+"""What the tests of the layer-list decoders (Golulix, Faledra, Nalizen, Pugozen) share: cases on the framework's engine, driven by
 portions, batches, generation and trace replay, and their comparison with a design's oracle."""
 import json
 
